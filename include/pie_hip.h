@@ -32,7 +32,7 @@ extern "C" {
 
 enum { PIE_OK = 0, PIE_E_ARG = -1, PIE_E_SHAPE = -2, PIE_E_ALIGN = -3, PIE_E_HIP = -4, PIE_E_STATE = -5, PIE_E_ARCH = -6, PIE_E_RANGE = -7,
        PIE_EXHAUSTED = 1 /* pie_page_alloc: no free page (the reference's std::nullopt); not an error */ };
-enum { PIE_BF16 = 1, PIE_F16 = 2, PIE_I8 = 3 /* KV page storage only: int8 rows + per-head fp16 scales (page pool, pie_paged_*_i8) */ };
+enum { PIE_BF16 = 1, PIE_F16 = 2, PIE_I8 = 3 /* KV page storage only: int8 rows + per-head fp16 scales (page pool, pie_paged_*_i8) */, PIE_F32 = 4 /* layer-stack models only */ };
 
 /* pie_core.hello()  (src/pie_core/src/bindings.cpp:8; asserted by tests/python/test_basic.py:16). */
 const char *pie_hello(void);
@@ -543,6 +543,83 @@ size_t pie_w4m_bytes(int N, int K);
 int pie_repack_w4s_to_w4m(const void *w4s, int N, int K, void *w4m, void *stream);
 int pie_qgemm_w4m(const void *x, const void *w4m, int M, int N, int K, int dtype, void *y, void *stream);
 
+
+/* ---------------------------------------------------------------- layer-stack models (no reference counterpart: models whose layers are listed one by one
+ * in config.json, each with its own mixer, feed-forward and sizes).  pie_stack_* runs a whole pass -- prompts, portions of prompts and single decoded
+ * tokens side by side, each row with its own position and sequence -- over a paged cache.  dtype PIE_BF16: bf16 products with fp32 accumulation; the
+ * residual stream, norms, attention scores and weights, gates are fp32.  dtype PIE_F32: everything fp32. */
+typedef struct pie_stack pie_stack;
+
+/* packed weight of a Linear [N, K] in the stack's dtype: W16M tiles, or fp32 rows of 64 ceil(K / 64).  w: row-major bf16 [N][K] on the device. */
+size_t pie_stack_weight_bytes(int dtype, int N, int K);
+int pie_stack_pack_weight(const void *w, int N, int K, int dtype, void *packed, void *stream);
+
+/* Dynamic Tanh: w * tanh(alpha x) + b, element by element.  w, b: fp32 [width] on the device. */
+typedef struct {
+    const float *w, *b;
+    float alpha;
+} pie_point_norm;
+
+typedef struct {
+    int dtype, width, vocab, n_layers;
+    float logit_scale;
+    const void *embed;         /* bf16 [vocab][width] */
+    const void *head;          /* packed [vocab, width] */
+    pie_point_norm final_norm;
+} pie_stack_config;
+
+enum { PIE_MIXER_LATENT = 1 };
+enum { PIE_FF_NONE = 0, PIE_FF_RELU2 = 1, PIE_FF_TABLE_MOE = 2 };
+
+/* One layer: x += post1(mixer(pre1(x))); x += post2(ff(pre2(x))).
+ * Latent mixer, with dim8 / vdim8 = dim / vdim rounded up to 8:  w_in packed [heads * dim8 + rank, width] (rows past dim of a head zero, the latent's
+ * down-projection last); w_uk heads x packed [rank, dim] (each head's up-projection of keys, transposed); w_uv heads x packed [vdim, rank];
+ * w_o packed [width, heads * vdim8]; w_kv packed [heads * (dim8 + vdim8), rank] (all keys, then all values: long prompts spell K and V out; may be
+ * NULL); c_norm fp32 [rank].  window <= 0: no limit.
+ * Experts: w_gate_up experts x packed [2 * size, width] with rows (2 i, 2 i + 1) = (gate_i, up_i); w_down experts x packed [width, size];
+ * table int32 [vocab][top].  Shared expert likewise when shared_size > 0, times sigmoid(shared_gate . input), shared_gate fp32 [width]. */
+typedef struct {
+    pie_point_norm pre1, post1, pre2, post2;
+    int mixer, heads, dim, vdim, rank, window;
+    float scale, eps;
+    const void *w_in, *w_uk, *w_uv, *w_o, *w_kv;
+    const float *c_norm;
+    int ff, ff_size;           /* ff_size: the dense width, or one expert's */
+    const void *w_up, *w_down; /* dense */
+    int experts, top, shared_size;
+    const int32_t *table;
+    const void *w_gate_up, *w_expert_down, *s_gate_up, *s_down;
+    const float *shared_gate;
+} pie_stack_layer;
+
+int pie_stack_create(const pie_stack_config *cfg, pie_stack **out);
+int pie_stack_destroy(pie_stack *s);
+int pie_stack_set_layer(pie_stack *s, int i, const pie_stack_layer *layer);
+/* elements per cached token of layer i (its page is [64][that many] in the stack's dtype), and bytes of one page */
+int pie_stack_page_row(const pie_stack *s, int i);
+size_t pie_stack_page_bytes(const pie_stack *s, int i);
+
+/* One pass.  Device arrays unless noted.  Rows are grouped in runs: run r = rows [row0, row0 + n_rows) at consecutive positions of sequence `seq` (a row of
+ * `table`), runs in row order, covering all rows.  Every row's latent is appended to its page, then the row attends to its sequence's cached tokens and
+ * itself.  want: the rows whose logits are asked for (NULL: all n_rows in order; n_want = n_rows).  logits fp32 [n_want][vocab]; logprobs (nullable)
+ * likewise; next (nullable) the greedy tokens.  advance: afterwards ids[i] = next[i] and pos[i] += 1 (all rows wanted, one per run), and with a
+ * history, history[pos of row 0] = next[0] at the new position.  tap (nullable): fp32 [n_layers][n_rows][width], the residual stream after each layer.
+ * flags: PIE_STEP_GRAPH replays a captured graph once a pass of the same shape and addresses has run before. */
+typedef struct {
+    int n_rows, n_seqs, table_width, n_runs, n_want, advance, history_len, reserved;
+    int32_t *ids, *pos;
+    const int32_t *row_seq, *table, *runs;
+    const int32_t *runs_host;  /* the same [n_runs][4] {row0, n_rows, seq, 0} in host memory */
+    const int32_t *want;
+    float *logits, *logprobs;
+    int32_t *next, *history;
+    void *const *slabs;        /* host array [n_layers] of device addresses */
+    size_t n_pages;
+    float *tap;
+} pie_stack_batch;
+int pie_stack_forward(pie_stack *s, const pie_stack_batch *b, int flags, void *stream);
+/* kernel launches of the last pass that was not replayed */
+int pie_stack_launches(const pie_stack *s);
 
 #ifdef __cplusplus
 }

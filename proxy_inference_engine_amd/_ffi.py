@@ -12,7 +12,7 @@ from pathlib import Path
 import torch
 
 _PKG = Path(__file__).resolve().parent
-PIE_BF16, PIE_F16 = 1, 2
+PIE_BF16, PIE_F16, PIE_F32 = 1, 2, 4
 PIE_STEP_LOGITS, PIE_STEP_GRAPH = 1, 2
 PIE_OPT_KV_I8 = 2
 # test / tuning switches (include/pie_hip.h: pie_set_knob); -1 restores a default
@@ -21,8 +21,17 @@ KNOBS = {"prefill_min": 0, "prefill_chunk": 1, "prefill_resident": 2, "small_m":
 PIE_I8 = 3  # KV page storage: int8 rows + per-head fp16 scales
 KERNELS = {"embed": 0, "qkv": 1, "attn": 2, "o_proj": 3, "gate_up": 4, "down": 5, "lm_head": 6, "tail": 7}
 
-EXPORTS = [
+# libpie_base.so: what the layer-stack models need; libpie_hip.so links it and adds the rest
+BASE_EXPORTS = [
     "pie_hello", "pie_version", "pie_last_error", "pie_device_info", "pie_set_knob", "pie_get_knob",
+    "pie_page_pool_slab_bytes", "pie_page_pool_create", "pie_page_pool_destroy", "pie_page_pool_size", "pie_page_pool_num_free",
+    "pie_page_alloc", "pie_page_free", "pie_page_add_ref", "pie_page_ref_count", "pie_page_num_tokens", "pie_page_set_num_tokens",
+    "pie_page_ptrs", "pie_page_i8_bytes", "pie_page_scale_ptrs",
+    "pie_w16m_bytes", "pie_repack_w16m", "pie_linear_w16m_workspace", "pie_linear_w16m",
+    "pie_stack_weight_bytes", "pie_stack_pack_weight", "pie_stack_create", "pie_stack_destroy", "pie_stack_set_layer", "pie_stack_page_row",
+    "pie_stack_page_bytes", "pie_stack_forward", "pie_stack_launches",
+]
+EXPORTS = BASE_EXPORTS + [
     "pie_quantize_w4g64", "pie_dequantize_w4g64", "pie_w4s_bytes", "pie_repack_w4g64", "pie_w8s_bytes", "pie_repack_w8g64", "pie_qgemv_w8g64", "pie_quantize_g64", "pie_dequantize_g64", "pie_embedding_g64", "pie_w4s32_bytes", "pie_repack_w4g32", "pie_qgemv_w4g32", "pie_w8s32_bytes", "pie_repack_w8g32", "pie_qgemv_w8g32", "pie_embedding_g32",
     "pie_w2s_bytes", "pie_repack_w2g64", "pie_qgemv_w2g64", "pie_w6s_bytes", "pie_repack_w6g64", "pie_qgemv_w6g64",
     "pie_w16s_bytes", "pie_repack_dense", "pie_gemv_dense", "pie_embedding_dense", "pie_qgemv_w4g64", "pie_qgemv_w4g64_f32",
@@ -32,11 +41,9 @@ EXPORTS = [
     "pie_decoder_set_kv", "pie_decoder_set_paged_kv", "pie_decoder_step_batch", "pie_decoder_prefill_batch", "pie_decoder_step_mixed", "pie_decoder_set_state", "pie_decoder_step", "pie_decoder_prefill", "pie_decoder_prefill_embeds",
     "pie_decoder_bind_outputs", "pie_decoder_set_token_from", "pie_decoder_step_bytes",
     "pie_decoder_launch_kernel", "pie_decoder_kernel_bytes", "pie_decoder_configure", "pie_decoder_status",
-    "pie_page_pool_slab_bytes", "pie_page_pool_create", "pie_page_pool_destroy", "pie_page_pool_size", "pie_page_pool_num_free",
-    "pie_page_alloc", "pie_page_free", "pie_page_add_ref", "pie_page_ref_count", "pie_page_num_tokens", "pie_page_set_num_tokens",
-    "pie_page_ptrs", "pie_paged_attn_workspace_bytes", "pie_paged_attn_decode", "pie_paged_kv_append",
-    "pie_page_i8_bytes", "pie_page_scale_ptrs", "pie_page_i8_set_scales", "pie_paged_kv_append_i8", "pie_paged_attn_decode_i8",
-    "pie_w16m_bytes", "pie_repack_w16m", "pie_linear_w16m_workspace", "pie_linear_w16m", "pie_gelu", "pie_vision_qkv_rope", "pie_sdpa_segments", "pie_bias_silu_mul", "pie_add_bias", "pie_add_bias_rms_norm",
+    "pie_paged_attn_workspace_bytes", "pie_paged_attn_decode", "pie_paged_kv_append",
+    "pie_page_i8_set_scales", "pie_paged_kv_append_i8", "pie_paged_attn_decode_i8",
+    "pie_gelu", "pie_vision_qkv_rope", "pie_sdpa_segments", "pie_bias_silu_mul", "pie_add_bias", "pie_add_bias_rms_norm",
     "pie_w4m_bytes", "pie_repack_w4s_to_w4m", "pie_qgemm_w4m",
     "pie_comm_create", "pie_comm_rccl_unique_id", "pie_comm_create_rccl", "pie_comm_export", "pie_comm_connect", "pie_allreduce_f32", "pie_comm_status", "pie_comm_destroy", "pie_decoder_set_comm", "pie_sample", "pie_sample_workspace_bytes",
 ]
@@ -62,6 +69,35 @@ class pie_global_weights(C.Structure):
                 ("fmt_embed", C.c_int), ("fmt_lm_head", C.c_int)]
 
 
+class pie_point_norm(C.Structure):
+    _fields_ = [("w", C.c_void_p), ("b", C.c_void_p), ("alpha", C.c_float)]
+
+
+class pie_stack_config(C.Structure):
+    _fields_ = [("dtype", C.c_int), ("width", C.c_int), ("vocab", C.c_int), ("n_layers", C.c_int), ("logit_scale", C.c_float),
+                ("embed", C.c_void_p), ("head", C.c_void_p), ("final_norm", pie_point_norm)]
+
+
+class pie_stack_layer(C.Structure):
+    _fields_ = [("pre1", pie_point_norm), ("post1", pie_point_norm), ("pre2", pie_point_norm), ("post2", pie_point_norm),
+                ("mixer", C.c_int), ("heads", C.c_int), ("dim", C.c_int), ("vdim", C.c_int), ("rank", C.c_int), ("window", C.c_int),
+                ("scale", C.c_float), ("eps", C.c_float),
+                ("w_in", C.c_void_p), ("w_uk", C.c_void_p), ("w_uv", C.c_void_p), ("w_o", C.c_void_p), ("w_kv", C.c_void_p), ("c_norm", C.c_void_p),
+                ("ff", C.c_int), ("ff_size", C.c_int), ("w_up", C.c_void_p), ("w_down", C.c_void_p),
+                ("experts", C.c_int), ("top", C.c_int), ("shared_size", C.c_int), ("table", C.c_void_p),
+                ("w_gate_up", C.c_void_p), ("w_expert_down", C.c_void_p), ("s_gate_up", C.c_void_p), ("s_down", C.c_void_p), ("shared_gate", C.c_void_p)]
+
+
+class pie_stack_batch(C.Structure):
+    _fields_ = [(n, C.c_int) for n in ("n_rows", "n_seqs", "table_width", "n_runs", "n_want", "advance", "history_len", "reserved")] + \
+               [(n, C.c_void_p) for n in ("ids", "pos", "row_seq", "table", "runs", "runs_host", "want", "logits", "logprobs", "next", "history", "slabs")] + \
+               [("n_pages", C.c_size_t), ("tap", C.c_void_p)]
+
+
+PIE_MIXER_LATENT = 1
+PIE_FF_NONE, PIE_FF_RELU2, PIE_FF_TABLE_MOE = 0, 1, 2
+
+
 def set_knob(name: str, value: int | None) -> None:
     """One of the library's test / tuning switches (KNOBS); None restores its default."""
     check(load().pie_set_knob(KNOBS[name], -1 if value is None else int(value)))
@@ -72,7 +108,48 @@ def lib_path() -> Path:
     return Path(env) if env else _PKG / "lib" / "libpie_hip.so"
 
 
-_lib = None
+_base = _lib = None
+
+
+def _open(path: Path, exports: list[str]) -> C.CDLL:
+    if not path.exists():
+        raise RuntimeError(
+            f"{path} not found: build it with `python -m proxy_inference_engine_amd.build` "
+            "(the MI355X path has no CPU or PyTorch fallback)")
+    lib = C.CDLL(str(path))
+    for name in exports:
+        if not hasattr(lib, name):
+            raise RuntimeError(f"{path} does not export {name}")
+    return lib
+
+
+def base() -> C.CDLL:
+    """Loads libpie_base.so alone: error plumbing, page pool, 16-bit GEMM, layer-stack models."""
+    global _base
+    if _base is not None:
+        return _base
+    lib = _open(_PKG / "lib" / "libpie_base.so", BASE_EXPORTS)
+    for name in ("pie_hello", "pie_version", "pie_last_error"):
+        getattr(lib, name).restype = C.c_char_p
+    for name in ("pie_page_pool_slab_bytes", "pie_page_pool_size", "pie_page_pool_num_free", "pie_stack_weight_bytes", "pie_stack_page_bytes"):
+        getattr(lib, name).restype = C.c_size_t
+    lib.pie_page_pool_slab_bytes.argtypes = [C.c_size_t, C.c_int, C.c_int, C.c_int]
+    lib.pie_page_pool_create.argtypes = [C.c_size_t, C.c_int, C.c_int, C.c_int, C.c_void_p, C.POINTER(C.c_void_p)]
+    lib.pie_page_pool_destroy.argtypes = lib.pie_page_pool_size.argtypes = lib.pie_page_pool_num_free.argtypes = [C.c_void_p]
+    lib.pie_page_alloc.argtypes = [C.c_void_p, C.POINTER(C.c_uint32)]
+    lib.pie_page_free.argtypes = lib.pie_page_add_ref.argtypes = [C.c_void_p, C.c_uint32]
+    lib.pie_page_ref_count.argtypes = [C.c_void_p, C.c_uint32, C.POINTER(C.c_uint32)]
+    lib.pie_page_num_tokens.argtypes = [C.c_void_p, C.c_uint32, C.POINTER(C.c_size_t)]
+    lib.pie_page_set_num_tokens.argtypes = [C.c_void_p, C.c_uint32, C.c_size_t]
+    lib.pie_stack_weight_bytes.argtypes = [C.c_int, C.c_int, C.c_int]
+    lib.pie_stack_pack_weight.argtypes = [C.c_void_p, C.c_int, C.c_int, C.c_int, C.c_void_p, C.c_void_p]
+    lib.pie_stack_create.argtypes = [C.POINTER(pie_stack_config), C.POINTER(C.c_void_p)]
+    lib.pie_stack_destroy.argtypes = lib.pie_stack_launches.argtypes = [C.c_void_p]
+    lib.pie_stack_set_layer.argtypes = [C.c_void_p, C.c_int, C.POINTER(pie_stack_layer)]
+    lib.pie_stack_page_row.argtypes = lib.pie_stack_page_bytes.argtypes = [C.c_void_p, C.c_int]
+    lib.pie_stack_forward.argtypes = [C.c_void_p, C.POINTER(pie_stack_batch), C.c_int, C.c_void_p]
+    _base = lib
+    return lib
 
 
 def load() -> C.CDLL:
@@ -80,15 +157,8 @@ def load() -> C.CDLL:
     global _lib
     if _lib is not None:
         return _lib
-    path = lib_path()
-    if not path.exists():
-        raise RuntimeError(
-            f"{path} not found: build it with `python -m proxy_inference_engine_amd.build` "
-            "(the MI355X path has no CPU or PyTorch fallback)")
-    lib = C.CDLL(str(path))
-    for name in EXPORTS:
-        if not hasattr(lib, name):
-            raise RuntimeError(f"{path} does not export {name}")
+    base()  # its soname satisfies libpie_hip.so's dependency, also for a variant build elsewhere (PIE_HIP_LIB)
+    lib = _open(lib_path(), EXPORTS)
     for name in ("pie_hello", "pie_version", "pie_last_error"):
         getattr(lib, name).restype = C.c_char_p
     for name in ("pie_w4s_bytes", "pie_w16s_bytes", "pie_w8s_bytes", "pie_w4s32_bytes", "pie_w8s32_bytes", "pie_w2s_bytes", "pie_w6s_bytes", "pie_sdpa_decode_workspace_bytes", "pie_decoder_step_bytes", "pie_decoder_kernel_bytes"):
@@ -164,7 +234,7 @@ def load() -> C.CDLL:
 def check(rc: int) -> None:
     if rc == 0:
         return
-    msg = load().pie_last_error().decode("utf-8", "replace")
+    msg = base().pie_last_error().decode("utf-8", "replace")
     if rc in (-1, -2, -3):  # PIE_E_ARG / SHAPE / ALIGN: the caller's fault
         raise ValueError(f"pie_hip: {msg} (code {rc})")
     if rc == -7:  # PIE_E_RANGE: std::out_of_range in the reference
@@ -184,6 +254,15 @@ def dtype_code(dt: torch.dtype) -> int:
     if dt == torch.float16:
         return PIE_F16
     raise ValueError(f"activation dtype must be bfloat16 or float16, got {dt}")
+
+
+def stack_dtype_code(dt: torch.dtype) -> int:
+    """Compute type of a layer-stack model."""
+    if dt == torch.bfloat16:
+        return PIE_BF16
+    if dt == torch.float32:
+        return PIE_F32
+    raise ValueError(f"a layer-stack model computes in bfloat16 or float32, got {dt}")
 
 
 def p(t: torch.Tensor | None) -> C.c_void_p:

@@ -1,9 +1,11 @@
-"""Builds libpie_hip.so (hand-written HIP for gfx950) in-tree with hipcc.
+"""Builds the native libraries (hand-written HIP for gfx950) in-tree with hipcc.
 
     python -m proxy_inference_engine_amd.build [--force]
 
-hipcc cross-compiles without a GPU, so this runs in the build container; the resulting .so is
-git-ignored and travels to the GPU box with the repo snapshot.
+libpie_base.so: error plumbing, page pool, the 16-bit GEMM, the layer-stack models -- everything a layer-stack model needs, and all that
+build_base() compiles (the trace runner in a fresh checkout).  libpie_hip.so: the Llama decoder, the quantised formats, the vision tower,
+sampling; it links the base library.  hipcc cross-compiles without a GPU, so this runs in the build container; the libraries are git-ignored
+and travel to the GPU box with the repo snapshot.
 """
 from __future__ import annotations
 
@@ -17,9 +19,13 @@ PKG = Path(__file__).resolve().parent
 CSRC = PKG / "csrc"
 LIB_DIR = PKG / "lib"
 LIB = LIB_DIR / "libpie_hip.so"
-SOURCES = ["w4_gemv.hip", "ops.hip", "decoder.hip", "prefill.hip", "vision.hip", "w4m_gemm.hip", "tp_comm.hip", "sampler.hip", "paged_i8.hip", "page_pool.cpp"]
+BASE_LIB = LIB_DIR / "libpie_base.so"
+BASE_SOURCES = ["base.hip", "w16_gemm.hip", "rows_gemm.hip", "latent_attn.hip", "layer_stack.hip", "page_pool.cpp"]
+SOURCES = ["w4_gemv.hip", "ops.hip", "decoder.hip", "prefill.hip", "vision.hip", "w4m_gemm.hip", "tp_comm.hip", "sampler.hip", "paged_i8.hip"]
+# packed-fp32-ops off: hipcc otherwise forms v_pk_{add,mul,fma}_f32 from ordinary float code, and some of their forms are not reliable here
 FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-ffp-contract=off", "-fno-fast-math",
          "-Wall", "-Wno-unused-function", "-D__HIP_PLATFORM_AMD__"]
+HIP_FLAGS = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
 def _hipcc() -> str:
@@ -29,12 +35,8 @@ def _hipcc() -> str:
     raise RuntimeError("hipcc not found")
 
 
-def _stale() -> bool:
-    if not LIB.exists():
-        return True
-    t = LIB.stat().st_mtime
-    deps = list(CSRC.glob("*.hip")) + list(CSRC.glob("*.hpp")) + list(CSRC.glob("*.cpp")) + [PKG.parent / "include" / "pie_hip.h"]
-    return any(d.stat().st_mtime > t for d in deps)
+def _headers() -> list[Path]:
+    return list(CSRC.glob("*.hpp")) + [PKG.parent / "include" / "pie_hip.h"]
 
 
 def source_hash() -> str:
@@ -48,32 +50,51 @@ def source_hash() -> str:
     return h.hexdigest()[:12]
 
 
-def build(force: bool = False, verbose: bool = False) -> Path:
-    if not force and not _stale():
-        return LIB
+def _make(lib: Path, sources: list[str], extra_link: list[str], deps: list[Path], force: bool, verbose: bool) -> Path:
+    """Compiles what changed of `sources` and links `lib` when anything did."""
+    stamps = [f.stat().st_mtime for f in [CSRC / src for src in sources] + _headers() + deps]
+    if not force and lib.exists() and lib.stat().st_mtime >= max(stamps):
+        return lib
     LIB_DIR.mkdir(exist_ok=True)
     obj_dir = LIB_DIR / "obj"
     obj_dir.mkdir(exist_ok=True)
     hipcc = _hipcc()
+    newest_header = max(h.stat().st_mtime for h in _headers())
 
-    def compile_one(src: str) -> Path:
+    def compile_one(src: str) -> bool:
         obj = obj_dir / (src + ".o")
-        extra = [f'-DPIE_BUILD_HASH="{source_hash()}"'] if src == "decoder.hip" else []
-        cmd = [hipcc, *FLAGS, *extra, "-c", str(CSRC / src), "-o", str(obj)]
+        stamp = max(newest_header, (CSRC / src).stat().st_mtime)
+        if src == "base.hip":  # carries the hash of all sources
+            stamp = max([stamp] + [f.stat().st_mtime for f in list(CSRC.glob("*.hip")) + list(CSRC.glob("*.cpp"))])
+        if not force and obj.exists() and obj.stat().st_mtime > stamp:
+            return False
+        extra = [f'-DPIE_BUILD_HASH="{source_hash()}"'] if src == "base.hip" else []
+        cmd = [hipcc, *FLAGS, *(HIP_FLAGS if src.endswith(".hip") else []), *extra, "-c", str(CSRC / src), "-o", str(obj)]
         r = subprocess.run(cmd, capture_output=True, text=True)
         if r.returncode != 0:
             raise RuntimeError(f"hipcc failed for {src}:\n{r.stderr[-6000:]}")
         if verbose and r.stderr.strip():
-            print(r.stderr, file=sys.stderr)
-        return obj
+            print("\n".join(ln for ln in r.stderr.splitlines() if "packed-fp32-ops" not in ln), file=sys.stderr)
+        return True
 
-    with ThreadPoolExecutor(max_workers=min(8, len(SOURCES))) as ex:
-        objs = list(ex.map(compile_one, SOURCES))
-    cmd = [hipcc, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", str(LIB), *map(str, objs), "-ldl"]
-    r = subprocess.run(cmd, capture_output=True, text=True)
-    if r.returncode != 0:
-        raise RuntimeError(f"link failed:\n{r.stderr[-4000:]}")
-    return LIB
+    with ThreadPoolExecutor(max_workers=min(8, len(sources))) as ex:
+        changed = any(list(ex.map(compile_one, sources)))
+    objs = [obj_dir / (s + ".o") for s in sources]
+    if changed or not lib.exists() or any(o.stat().st_mtime > lib.stat().st_mtime for o in objs + deps):
+        cmd = [hipcc, "--offload-arch=gfx950", "-shared", "-fPIC", f"-Wl,-soname,{lib.name}", "-o", str(lib), *map(str, objs), *extra_link]
+        r = subprocess.run(cmd, capture_output=True, text=True)
+        if r.returncode != 0:
+            raise RuntimeError(f"link failed:\n{r.stderr[-4000:]}")
+    return lib
+
+
+def build_base(force: bool = False, verbose: bool = False) -> Path:
+    return _make(BASE_LIB, BASE_SOURCES, [], [], force, verbose)
+
+
+def build(force: bool = False, verbose: bool = False) -> Path:
+    base = build_base(force, verbose)
+    return _make(LIB, SOURCES, [f"-L{LIB_DIR}", "-lpie_base", "-Wl,-rpath,$ORIGIN", "-ldl"], [base], force, verbose)
 
 
 if __name__ == "__main__":

@@ -35,7 +35,7 @@ class BaseCache(ABC):
                     arrays[f"{i}.{j}"] = t.detach().to("cpu").contiguous()
             meta[f"0.{i}"] = str(c.meta_state)
             # a paged cache is stored as its gathered rows, the layout a ReusableKVCache restores from
-            meta[f"2.{i}"] = "ReusableKVCache" if type(c).__name__ == "PagedKVCache" else type(c).__name__
+            meta[f"2.{i}"] = {"PagedKVCache": "ReusableKVCache", "PagedLatentCache": "SavedLatentCache"}.get(type(c).__name__, type(c).__name__)
         for k, v in (metadata or {}).items():
             meta[f"1.{k}"] = str(v)
         save_file(arrays, file_name, metadata=meta)
@@ -45,7 +45,7 @@ class BaseCache(ABC):
         from safetensors import safe_open
         if device is None:
             device = "cuda" if torch.cuda.is_available() else "cpu"
-        classes = {"ReusableKVCache": ReusableKVCache}
+        classes = {"ReusableKVCache": ReusableKVCache, "SavedLatentCache": SavedLatentCache}
         with safe_open(file_name, framework="pt", device="cpu") as f:
             meta = f.metadata() or {}
             n = sum(1 for k in meta if k.startswith("2."))
@@ -94,5 +94,6 @@ class BaseCache(ABC):
 
 from .reusable import ReusableKVCache  # noqa: E402
 from .paged import PageAllocator, PagedKVCache, PagedSequence  # noqa: E402
+from .latent import LatentPageAllocator, PagedLatentCache, SavedLatentCache  # noqa: E402
 
-__all__ = ["BaseCache", "ReusableKVCache", "PagedKVCache", "PagedSequence", "PageAllocator"]
+__all__ = ["BaseCache", "ReusableKVCache", "PagedKVCache", "PagedSequence", "PageAllocator", "LatentPageAllocator", "PagedLatentCache", "SavedLatentCache"]

@@ -34,16 +34,16 @@ class KVPage:
 
     def get_ref_count(self) -> int:
         n = C.c_uint32()
-        _f.check(_f.load().pie_page_ref_count(self._pool._h, self._id, C.byref(n)))
+        _f.check(_f.base().pie_page_ref_count(self._pool._h, self._id, C.byref(n)))
         return n.value
 
     def num_tokens(self) -> int:
         n = C.c_size_t()
-        _f.check(_f.load().pie_page_num_tokens(self._pool._h, self._id, C.byref(n)))
+        _f.check(_f.base().pie_page_num_tokens(self._pool._h, self._id, C.byref(n)))
         return n.value
 
     def set_num_tokens(self, n: int) -> None:
-        _f.check(_f.load().pie_page_set_num_tokens(self._pool._h, self._id, n))
+        _f.check(_f.base().pie_page_set_num_tokens(self._pool._h, self._id, n))
 
     def _block(self, which: int, layer: int) -> torch.Tensor:
         p = self._pool
@@ -86,7 +86,7 @@ class PageAllocator:
         """num_layers > 1: one slab plane per decoder layer ([num_layers, slab bytes]); a page id names the same slice
         of every plane, so one block table serves all layers."""
         self._h = C.c_void_p()
-        lib = self._lib = _f.load()
+        lib = self._lib = _f.base()
         code = _f.PIE_I8 if dtype == torch.int8 else _f.dtype_code(dtype)  # int8: the reference page's own storage (page.hpp:25-32)
         if num_pages < 0 or num_heads < 0 or head_dim < 0:
             raise ValueError("PageAllocator: negative argument")
@@ -100,7 +100,7 @@ class PageAllocator:
         self.page_bytes = nbytes // num_pages
         if dtype == torch.int8 and self.slab is not None:  # key_cache_scale_ / value_cache_scale_ = mx::ones (page.hpp:31-32)
             for layer in range(num_layers):
-                _f.check(lib.pie_page_i8_set_scales(C.c_void_p(self.slab[layer].data_ptr()), num_pages, num_heads, head_dim, None, num_pages, None, None,
+                _f.check(_f.load().pie_page_i8_set_scales(C.c_void_p(self.slab[layer].data_ptr()), num_pages, num_heads, head_dim, None, num_pages, None, None,
                                                     _f.stream()))
 
     def __del__(self):
@@ -112,10 +112,19 @@ class PageAllocator:
             except Exception:  # noqa: BLE001
                 pass
 
+    @property
+    def device(self) -> torch.device | None:
+        """Where the pages live; None: bookkeeping only."""
+        return None if self.slab is None else self.slab.device
+
+    def copy_page(self, src: int, dst: int) -> None:
+        pb = self.page_bytes
+        self.slab[:, dst * pb:(dst + 1) * pb] = self.slab[:, src * pb:(src + 1) * pb]
+
     def allocate_page(self) -> int | None:
         """A free page id with ref count 1 and no tokens, or None when the pool is exhausted (page_allocator.cpp:68-79)."""
         out = C.c_uint32()
-        rc = _f.load().pie_page_alloc(self._h, C.byref(out))
+        rc = _f.base().pie_page_alloc(self._h, C.byref(out))
         if rc == 1:  # PIE_EXHAUSTED
             return None
         _f.check(rc)
@@ -123,10 +132,10 @@ class PageAllocator:
 
     def free_page(self, page_id: int) -> None:
         """Drops one reference; the page returns to the free list at zero (page_allocator.cpp:81-87)."""
-        _f.check(_f.load().pie_page_free(self._h, _id(page_id)))
+        _f.check(_f.base().pie_page_free(self._h, _id(page_id)))
 
     def add_ref(self, page_id: int) -> None:
-        _f.check(_f.load().pie_page_add_ref(self._h, _id(page_id)))
+        _f.check(_f.base().pie_page_add_ref(self._h, _id(page_id)))
 
     def get_page(self, page_id: int) -> KVPage:
         pid = _id(page_id)
@@ -135,10 +144,10 @@ class PageAllocator:
         return KVPage(self, pid)
 
     def size(self) -> int:
-        return _f.load().pie_page_pool_size(self._h)
+        return _f.base().pie_page_pool_size(self._h)
 
     def get_num_free_pages(self) -> int:
-        return _f.load().pie_page_pool_num_free(self._h)
+        return _f.base().pie_page_pool_num_free(self._h)
 
 
 def _id(page_id: int) -> int:
@@ -154,12 +163,12 @@ class PagedSequence:
     slab plane.  Growing takes pages from the allocator -- nothing is copied, unlike ReusableKVCache's reallocation."""
 
     def __init__(self, allocator: PageAllocator, max_blocks: int = 16):
-        if allocator.slab is None:
+        if allocator.device is None:
             raise ValueError("PagedSequence needs a PageAllocator with device storage")
         self.allocator = allocator
         self.pages: list[int] = []
         self.offset = 0
-        self.table = torch.zeros(max(1, max_blocks), dtype=torch.int32, device=allocator.slab.device)
+        self.table = torch.zeros(max(1, max_blocks), dtype=torch.int32, device=allocator.device)
 
     @property
     def max_blocks(self) -> int:
@@ -223,8 +232,7 @@ class PagedSequence:
             if pid is None:
                 other.release()
                 raise RuntimeError("KV page pool exhausted")
-            pb, src = self.allocator.page_bytes, self.pages[full]
-            self.allocator.slab[:, pid * pb:(pid + 1) * pb] = self.allocator.slab[:, src * pb:(src + 1) * pb]
+            self.allocator.copy_page(self.pages[full], pid)
             other.pages.append(pid)
         other.offset = self.offset
         if other.pages:

@@ -20,7 +20,7 @@ import torch
 
 logger = logging.getLogger(__name__)
 
-from .kv_cache import BaseCache, PagedKVCache, ReusableKVCache
+from .kv_cache import BaseCache, PagedKVCache, ReusableKVCache, SavedLatentCache
 
 
 def _as_list(ids) -> list[int]:
@@ -51,6 +51,11 @@ class PromptCache:
     def __call__(self, prompt_ids):
         return self.reuse_cache(prompt_ids)
 
+    def adopt(self, model) -> None:
+        """Caches restored from a file into the form the model runs on (a paged model copies the saved rows into pages of its pool)."""
+        if self.cache and hasattr(model, "adopt_cache"):
+            self.cache = model.adopt_cache(self.cache)
+
     def create_kv_cache(self, model) -> None:
         if hasattr(model, "make_cache") and callable(model.make_cache):
             self.cache = model.make_cache()
@@ -80,7 +85,7 @@ class PromptCache:
         if common == 0:
             return prompt_ids
         for layer_cache in self.cache:
-            assert isinstance(layer_cache, (ReusableKVCache, PagedKVCache))
+            assert isinstance(layer_cache, (ReusableKVCache, PagedKVCache, SavedLatentCache))
             layer_cache.reuse(len(ids), common)
         # DEVIATION from prompt_cache.py:52-76, which leaves computed_ids untouched here: after a diverging request B the
         # reference's history reads A + B[k:] while the KV rows beyond k belong to B, so a later request that matches A beyond k

@@ -1,0 +1,530 @@
+// layer_stack.hip -- native runtime of the layer-stack models: one pass over a list of layers that may all differ (pie_stack_*, include/pie_hip.h).
+//
+// A pass is a batch of rows, each with its own sequence and position: whole prompts, portions and single decoded tokens are the same thing here.
+// Launches per layer (every norm is element-wise and rides in the epilogue of the kernel that produces its input):
+//   [q | latent down]     Linear                                      (rows_gemm.hip)
+//   latent RMS norm + page append                                     (latent_attn.hip)
+//   q -> latent space     Linear per head
+//   attention over the latents [+ merge of the key splits]            (latent_attn.hip)
+//   latents -> values     Linear per head
+//   output projection     Linear; epilogue: x += post1(y), h = pre2(x)
+//   dense: up (relu^2), down; epilogue: x += post2(y), h = next layer's pre1(x)
+//   experts: gate|up (silu * up) and down over the active experts and the shared one, then the weighted sum with the same epilogue
+// The experts of a token are a table lookup, so all layers' row lists are made by one launch in front of the pass.
+#include <cstring>
+#include <algorithm>
+#include <new>
+#include <vector>
+
+#include "stack_types.hpp"
+
+namespace {
+
+struct RouteLayer {      // one mixture layer's row lists (device pointers)
+    const int *table;
+    int top, experts, max_active;
+    int *active, *offset, *list, *place;  // [max_active], [experts + 1], [M * top] rows by expert, [M * top] position of (row, slot)
+};
+
+__global__ void __launch_bounds__(1024) k_route(const RouteLayer *layers, const int *ids, int M, int vocab) {
+    extern __shared__ int s_cnt[];  // [experts] counts, then [experts] cursors
+    const RouteLayer L = layers[blockIdx.x];
+    int *s_cur = s_cnt + L.experts;
+    const int n = M * L.top;
+    auto expert = [&](int i) {
+        const int t = min(max(ids[i / L.top], 0), vocab - 1);
+        return min(max(L.table[(size_t)t * L.top + i % L.top], 0), L.experts - 1);
+    };
+    for (int e = threadIdx.x; e < L.experts; e += blockDim.x) s_cnt[e] = 0;
+    __syncthreads();
+    for (int i = threadIdx.x; i < n; i += blockDim.x) atomicAdd(&s_cnt[expert(i)], 1);
+    __syncthreads();
+    if (threadIdx.x < 64) {
+        int base = 0, n_active = 0;
+        for (int e0 = 0; e0 < L.experts; e0 += 64) {
+            const int e = e0 + (int)threadIdx.x, c = e < L.experts ? s_cnt[e] : 0;
+            int incl = c;
+#pragma unroll
+            for (int o = 1; o < 64; o <<= 1) {
+                const int v = __shfl_up(incl, o, 64);
+                if ((int)threadIdx.x >= o) incl += v;
+            }
+            if (e < L.experts) s_cur[e] = L.offset[e] = base + incl - c;
+            const unsigned long long has = __ballot(c > 0);
+            const int slot = n_active + __popcll(has & ((1ull << threadIdx.x) - 1ull));
+            if (c > 0 && slot < L.max_active) L.active[slot] = e;
+            base += __shfl(incl, 63, 64), n_active += __popcll(has);
+        }
+        if (threadIdx.x == 0) L.offset[L.experts] = base;
+        for (int i = n_active + (int)threadIdx.x; i < L.max_active; i += 64) L.active[i] = -1;
+    }
+    __syncthreads();
+    for (int i = threadIdx.x; i < n; i += blockDim.x) {
+        const int p = atomicAdd(&s_cur[expert(i)], 1);
+        L.list[p] = i / L.top;
+        L.place[i] = p;
+    }
+}
+
+template <class E>
+__global__ void __launch_bounds__(256) k_stack_embed(const int *ids, const u16 *table, int vocab, int W, PointNorm next, float *x, int ldx, typename E::type *h, int ldh) {
+    const size_t m = blockIdx.y;
+    const int n = blockIdx.x * 256 + threadIdx.x;
+    if (n >= W) return;
+    const int t = min(max(ids[m], 0), vocab - 1);
+    const float v = BF16::to_f32(table[(size_t)t * W + n]);
+    x[m * ldx + n] = v;
+    h[m * ldh + n] = E::pack(point_norm(next, n, v));
+}
+
+// y = sum over the token's slots of its experts' outputs / top (+ sigmoid(gate . input) * shared output); x += post(y); h = next(x)
+struct CombineArgs {
+    const float *part, *part_s;  // [M * top][ldp] by position, [M][ldp]
+    int ldp;
+    const int *place;
+    int top, W;
+    const float *gate;           // [W] or nullptr
+    PointNorm pre, post, next;   // pre: the sublayer's input norm (the gate's dot product is taken in fp32 on it)
+    float *x;
+    int ldx;
+    void *h;
+    int ldh;
+};
+template <class E>
+__global__ void __launch_bounds__(256) k_moe_combine(const CombineArgs a) {
+    __shared__ float red[4];
+    const size_t m = blockIdx.x;
+    float *x = a.x + m * a.ldx;
+    float g = 0.0f;
+    if (a.gate) {
+        float d = 0.0f;
+        for (int n = threadIdx.x; n < a.W; n += 256) d = fmaf(point_norm(a.pre, n, x[n]), a.gate[n], d);
+        d = wave_sum(d);
+        if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = d;
+        __syncthreads();
+        g = 1.0f / (1.0f + expf(-((red[0] + red[1]) + (red[2] + red[3]))));
+    }
+    const float share = 1.0f / (float)a.top;
+    for (int n = threadIdx.x; n < a.W; n += 256) {
+        float y = 0.0f;
+        for (int s = 0; s < a.top; ++s) y = fmaf(share, a.part[(size_t)a.place[m * a.top + s] * a.ldp + n], y);
+        if (a.gate) y = fmaf(g, a.part_s[m * a.ldp + n], y);
+        const float v = x[n] + point_norm(a.post, n, y);
+        x[n] = v;
+        ((typename E::type *)a.h)[m * a.ldh + n] = E::pack(point_norm(a.next, n, v));
+    }
+}
+
+// log-softmax and greedy token over fp32 logits: per-tile (max, sum, first argmax), then every workgroup of a row merges the row's tiles
+constexpr int ST_TILES = 64;
+struct RowStat {
+    float max, sum;
+    int arg, pad;
+};
+__global__ void __launch_bounds__(256) k_f32_stats(const float *logits, int V, RowStat *stats) {
+    __shared__ float s_max[4], s_sum[4];
+    __shared__ int s_arg[4];
+    logits += (size_t)blockIdx.y * V;
+    const int len = (V + ST_TILES - 1) / ST_TILES, begin = blockIdx.x * len, end = min(V, begin + len), wave = threadIdx.x >> 6;
+    float mx = -INFINITY;
+    int arg = 0x7fffffff;
+    for (int i = begin + threadIdx.x; i < end; i += 256)
+        if (logits[i] > mx) mx = logits[i], arg = i;
+    const float wm = wave_max(mx);
+    int cand = mx == wm ? arg : 0x7fffffff;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) cand = min(cand, __shfl_xor(cand, o, 64));
+    if ((threadIdx.x & 63) == 0) s_max[wave] = wm, s_arg[wave] = cand;
+    __syncthreads();
+    float tm = s_max[0];
+    int ta = s_arg[0];
+    for (int w = 1; w < 4; ++w)
+        if (s_max[w] > tm || (s_max[w] == tm && s_arg[w] < ta)) tm = s_max[w], ta = s_arg[w];
+    float se = 0.0f;
+    for (int i = begin + threadIdx.x; i < end; i += 256) se += expf(logits[i] - tm);
+    se = wave_sum(se);
+    if ((threadIdx.x & 63) == 0) s_sum[wave] = se;
+    __syncthreads();
+    if (threadIdx.x == 0) stats[blockIdx.y * ST_TILES + blockIdx.x] = {tm, (s_sum[0] + s_sum[1]) + (s_sum[2] + s_sum[3]), ta, 0};
+}
+__global__ void __launch_bounds__(256) k_f32_finish(const float *logits, int V, const RowStat *stats, float *logprobs, int *next, int advance, int *ids, int *pos,
+                                                    int *history, int history_len) {
+    const size_t r = blockIdx.y;
+    const int lane = threadIdx.x & 63;
+    const RowStat st = stats[r * ST_TILES + lane];  // (every wave merges the same 64 tiles)
+    const float mx = wave_max(st.max);
+    int cand = st.max == mx ? st.arg : 0x7fffffff;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) cand = min(cand, __shfl_xor(cand, o, 64));
+    const float lse = mx + logf(wave_sum(st.sum > 0.0f ? st.sum * expf(st.max - mx) : 0.0f));
+    if (logprobs)
+        for (int i = blockIdx.x * 256 + threadIdx.x; i < V; i += gridDim.x * 256) logprobs[r * V + i] = logits[r * V + i] - lse;
+    if (blockIdx.x == 0 && threadIdx.x == 0) {
+        next[r] = cand;
+        if (advance) {
+            const int p = pos[r] + 1;
+            ids[r] = cand, pos[r] = p;
+            if (history && r == 0 && p < history_len) history[p] = cand;
+        }
+    }
+}
+
+template <class T>
+struct Buf {  // a device buffer that only grows; new memory is zero (row paddings stay finite), 64 elements of slack behind it
+    T *p = nullptr;
+    size_t cap = 0;
+    int need(size_t n, bool *moved) {
+        if (n <= cap) return PIE_OK;
+        if (p) PIE_HIP_TRY(hipFree(p));
+        p = nullptr, cap = 0;
+        PIE_HIP_TRY(hipMalloc((void **)&p, (n + 64) * sizeof(T)));
+        PIE_HIP_TRY(hipMemset(p, 0, (n + 64) * sizeof(T)));
+        cap = n, *moved = true;
+        return PIE_OK;
+    }
+    ~Buf() {
+        if (p) (void)hipFree(p);
+    }
+};
+
+int up8(int n) { return (n + 7) & ~7; }
+
+struct GraphKey {
+    pie_stack_batch b;
+    std::vector<void *> slabs;
+    std::vector<int32_t> runs;
+    bool same(const GraphKey &o) const { return memcmp(&b, &o.b, sizeof b) == 0 && slabs == o.slabs && runs == o.runs; }
+};
+struct GraphSlot {
+    GraphKey key;
+    hipGraphExec_t exec = nullptr;
+    unsigned long long used = 0;
+};
+
+}  // namespace
+
+struct pie_stack {
+    pie_stack_config cfg;
+    std::vector<pie_stack_layer> layers;
+    std::vector<char> have;
+    // workspace, by rows of a pass
+    Buf<float> x, c_raw, part, part_s, attn_ws;
+    Buf<char> h, q, ql, oc, o, act, act_e, act_s, hsel;
+    Buf<RowStat> stats;
+    Buf<int> route_ints;
+    Buf<RouteLayer> route_dev;
+    std::vector<RouteLayer> route;  // per layer; experts == 0: not a mixture
+    int route_rows = 0, n_route = 0, route_lds = 0;
+    std::vector<GraphSlot> graphs;
+    unsigned long long tick = 0;
+    int launches = 0;
+    void drop_graphs() {
+        for (GraphSlot &g : graphs)
+            if (g.exec) (void)hipGraphExecDestroy(g.exec);
+        graphs.clear();
+    }
+    ~pie_stack() { drop_graphs(); }
+};
+
+namespace {
+
+size_t esize(const pie_stack *s) { return s->cfg.dtype == PIE_F32 ? 4 : 2; }
+PointNorm norm_of(const pie_point_norm &n) { return {n.w, n.b, n.alpha}; }
+
+int stack_reserve(pie_stack *s, const pie_stack_batch &b, hipStream_t st) {
+    const size_t M = (size_t)b.n_rows, E = esize(s), W8 = up8(s->cfg.width);
+    size_t q = 0, c = 0, ql = 0, o = 0, act = 0, act_e = 0, act_s = 0, part = 0, part_s = 0, ints = 0;
+    for (const pie_stack_layer &L : s->layers) {
+        q = std::max(q, (size_t)L.heads * up8(L.dim)), c = std::max(c, (size_t)up8(L.rank)), ql = std::max(ql, (size_t)L.heads * up8(L.rank));
+        o = std::max(o, (size_t)L.heads * up8(L.vdim));
+        if (L.ff == PIE_FF_RELU2) act = std::max(act, (size_t)up8(L.ff_size));
+        if (L.ff == PIE_FF_TABLE_MOE) {
+            act_e = std::max(act_e, (size_t)L.top * up8(L.ff_size)), part = std::max(part, (size_t)L.top * W8);
+            if (L.shared_size) act_s = std::max(act_s, (size_t)up8(L.shared_size)), part_s = W8;
+        }
+    }
+    bool moved = false;
+    int rc = 0;
+    if (M > (size_t)1 << 20) return pie::fail(PIE_E_SHAPE, "pie_stack_forward: too many rows in one pass");
+    if ((rc = s->x.need(M * W8, &moved)) || (rc = s->c_raw.need(M * c, &moved)) || (rc = s->part.need(M * part, &moved)) || (rc = s->part_s.need(M * part_s, &moved)) ||
+        (rc = s->h.need(M * W8 * E, &moved)) || (rc = s->q.need(M * q * E, &moved)) || (rc = s->ql.need(M * ql * E, &moved)) || (rc = s->oc.need(M * ql * E, &moved)) ||
+        (rc = s->o.need(M * o * E, &moved)) || (rc = s->act.need(M * act * E, &moved)) || (rc = s->act_e.need(M * act_e * E, &moved)) ||
+        (rc = s->act_s.need(M * act_s * E, &moved)) || (rc = s->stats.need((size_t)b.n_want * ST_TILES, &moved)))
+        return rc;
+    if (s->n_route && (int)M > s->route_rows) {
+        s->route_rows = (int)M;
+        for (const RouteLayer &r : s->route)
+            if (r.experts) ints += r.experts + (size_t)r.experts + 1 + 2 * M * r.top;
+        if ((rc = s->route_ints.need(ints, &moved)) || (rc = s->route_dev.need(s->n_route, &moved))) return rc;
+        int *p = s->route_ints.p;
+        std::vector<RouteLayer> dev;
+        s->route_lds = 0;
+        for (RouteLayer &r : s->route) {
+            if (!r.experts) continue;
+            r.active = p, p += r.experts, r.offset = p, p += r.experts + 1, r.list = p, p += M * r.top, r.place = p, p += M * r.top;
+            r.max_active = r.experts;
+            s->route_lds = std::max(s->route_lds, 2 * r.experts * 4);
+            dev.push_back(r);
+        }
+        PIE_HIP_TRY(hipStreamSynchronize(st));
+        PIE_HIP_TRY(hipMemcpy(s->route_dev.p, dev.data(), dev.size() * sizeof(RouteLayer), hipMemcpyHostToDevice));
+        moved = true;
+    }
+    if (moved) {
+        PIE_HIP_TRY(hipDeviceSynchronize());
+        s->drop_graphs();
+    }
+    return PIE_OK;
+}
+
+// key splits of a layer's attention: enough workgroups for the chip, at least 64 keys each; from capacities only, so that a captured step keeps its plan
+int plan_splits(const pie_stack_batch &b, const pie_stack_layer &L, int n_tiles) {
+    long ctx = (long)b.table_width * PAGE_TOKENS;
+    if (L.window > 0 && L.window + 64 < ctx) ctx = L.window + 64;
+    long s = 512 / n_tiles;
+    s = std::min(s, ctx / 64);
+    s = std::min(s, 64L);
+    return (int)std::max(s, 1L);
+}
+
+int stack_tiles(const int32_t *runs, int n_runs, int H) {
+    int n = 0;
+    for (int i = 0; i < n_runs; ++i) n += (runs[4 * i + 1] * H + 63) / 64;
+    return n;
+}
+
+struct Pass {
+    pie_stack *s;
+    const pie_stack_batch &b;
+    hipStream_t st;
+    int rc = PIE_OK, launches = 0;
+    void linear(const RowsArgs &a, int batches = 1) {
+        if (!rc) rc = rows_gemm_launch(s->cfg.dtype, a, batches, st), ++launches;
+    }
+};
+
+void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const PointNorm &next) {
+    pie_stack *s = p.s;
+    const pie_stack_batch &b = p.b;
+    const int M = b.n_rows, W = s->cfg.width, W8 = up8(W), D8 = up8(L.dim), V8 = up8(L.vdim), R8 = up8(L.rank), H = L.heads, dt = s->cfg.dtype;
+    RowsArgs a = {};
+    a.m = {(const char *)L.w_in, H * D8 + L.rank, W, s->h.p, W8, s->q.p, H * D8};
+    a.M = M, a.epi = ROWS_SPLIT, a.split = H * D8, a.y2 = s->c_raw.p, a.ldy2 = R8;
+    p.linear(a);
+    if (!p.rc)
+        p.rc = latent_append_launch(dt, s->c_raw.p, R8, L.c_norm, L.eps, M, L.rank, R8, b.pos, b.row_seq, b.table, b.table_width, (int)b.n_pages, b.n_seqs,
+                                    b.slabs[li], p.st),
+        ++p.launches;
+    RowsArgs k = {};
+    k.m = {(const char *)L.w_uk, L.rank, L.dim, s->q.p, H * D8, s->ql.p, H * R8};
+    k.M = M, k.epi = ROWS_STORE, k.w_batch = rows_weight_bytes(dt, L.rank, L.dim), k.x_batch = D8, k.y_batch = R8;
+    p.linear(k, H);
+    LatentAttnArgs t = {};
+    t.q = s->ql.p, t.slab = b.slabs[li], t.table = b.table, t.table_width = b.table_width, t.n_pages = (int)b.n_pages, t.n_seqs = b.n_seqs, t.pos = b.pos;
+    t.runs = (const RowRun *)b.runs, t.n_runs = b.n_runs, t.n_tiles = stack_tiles(b.runs_host, b.n_runs, H), t.single = b.n_runs == M, t.row_seq = b.row_seq;
+    t.H = H, t.R = L.rank, t.ldr = R8, t.M = M, t.window = L.window, t.scale = L.scale, t.splits = plan_splits(b, L, t.n_tiles), t.ws = s->attn_ws.p, t.out = s->oc.p;
+    if (!p.rc) p.rc = latent_attn_launch(dt, t, p.st), p.launches += t.splits > 1 ? 2 : 1;
+    RowsArgs v = {};
+    v.m = {(const char *)L.w_uv, L.vdim, L.rank, s->oc.p, H * R8, s->o.p, H * V8};
+    v.M = M, v.epi = ROWS_STORE, v.w_batch = rows_weight_bytes(dt, L.vdim, L.rank), v.x_batch = R8, v.y_batch = V8;
+    p.linear(v, H);
+    RowsArgs o = {};
+    o.m = {(const char *)L.w_o, W, H * V8, s->o.p, H * V8, nullptr, 0};
+    o.M = M, o.epi = ROWS_RESIDUAL, o.res = s->x.p, o.ld_res = W8, o.post = norm_of(L.post1), o.next = next, o.h = s->h.p, o.ldh = W8;
+    p.linear(o);
+}
+
+void feed_forward(Pass &p, int li, const pie_stack_layer &L, const PointNorm &next) {
+    pie_stack *s = p.s;
+    const int M = p.b.n_rows, W = s->cfg.width, W8 = up8(W), F = L.ff_size, F8 = up8(F), dt = s->cfg.dtype;
+    if (L.ff == PIE_FF_RELU2) {
+        RowsArgs u = {};
+        u.m = {(const char *)L.w_up, F, W, s->h.p, W8, s->act.p, F8};
+        u.M = M, u.epi = ROWS_RELU2;
+        p.linear(u);
+        RowsArgs d = {};
+        d.m = {(const char *)L.w_down, W, F, s->act.p, F8, nullptr, 0};
+        d.M = M, d.epi = ROWS_RESIDUAL, d.res = s->x.p, d.ld_res = W8, d.post = norm_of(L.post2), d.next = next, d.h = s->h.p, d.ldh = W8;
+        p.linear(d);
+        return;
+    }
+    const RouteLayer &r = s->route[li];
+    const int S = L.shared_size, S8 = up8(S), groups = (int)std::min((long)L.experts, (long)M * L.top) + (S ? 1 : 0);
+    RowsArgs u = {};
+    u.m = {(const char *)L.w_gate_up, 2 * F, W, s->h.p, W8, s->act_e.p, F8};
+    u.M = M, u.epi = ROWS_SILU_MUL, u.w_batch = rows_weight_bytes(dt, 2 * F, W), u.active = r.active, u.offset = r.offset, u.list = r.list, u.gather = true;
+    if (S) u.shared = {(const char *)L.s_gate_up, 2 * S, W, s->h.p, W8, s->act_s.p, S8};
+    p.linear(u, groups);
+    RowsArgs d = {};
+    d.m = {(const char *)L.w_expert_down, W, F, s->act_e.p, F8, s->part.p, W8};
+    d.M = M, d.epi = ROWS_SCALE_F32, d.scale = 1.0f, d.w_batch = rows_weight_bytes(dt, W, F), d.active = r.active, d.offset = r.offset, d.list = r.list;
+    if (S) d.shared = {(const char *)L.s_down, W, S, s->act_s.p, S8, s->part_s.p, W8};
+    p.linear(d, groups);
+    if (p.rc) return;
+    CombineArgs c = {};
+    c.part = s->part.p, c.part_s = s->part_s.p, c.ldp = W8, c.place = r.place, c.top = L.top, c.W = W, c.gate = S ? L.shared_gate : nullptr;
+    c.pre = norm_of(L.pre2), c.post = norm_of(L.post2), c.next = next, c.x = s->x.p, c.ldx = W8, c.h = s->h.p, c.ldh = W8;
+    if (dt == PIE_F32) hipLaunchKernelGGL(k_moe_combine<ElemF32>, dim3((unsigned)M), dim3(256), 0, p.st, c);
+    else hipLaunchKernelGGL(k_moe_combine<ElemBF16>, dim3((unsigned)M), dim3(256), 0, p.st, c);
+    if (hipGetLastError() != hipSuccess) p.rc = pie::fail(PIE_E_HIP, "expert combine launch failed");
+    ++p.launches;
+}
+
+int stack_enqueue(pie_stack *s, const pie_stack_batch &b, hipStream_t st) {
+    const int M = b.n_rows, W = s->cfg.width, W8 = up8(W), V = s->cfg.vocab, n = s->cfg.n_layers, dt = s->cfg.dtype;
+    Pass p{s, b, st};
+    if (s->n_route) {
+        hipLaunchKernelGGL(k_route, dim3((unsigned)s->n_route), dim3(1024), (size_t)s->route_lds, st, s->route_dev.p, b.ids, M, V);
+        PIE_LAUNCH_CHECK();
+        ++p.launches;
+    }
+    const PointNorm fin = norm_of(s->cfg.final_norm), first = n ? norm_of(s->layers[0].pre1) : fin;
+    const dim3 ge((unsigned)((W + 255) / 256), (unsigned)M);
+    if (dt == PIE_F32)
+        hipLaunchKernelGGL(k_stack_embed<ElemF32>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, first, s->x.p, W8, (float *)s->h.p, W8);
+    else
+        hipLaunchKernelGGL(k_stack_embed<ElemBF16>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, first, s->x.p, W8, (u16 *)s->h.p, W8);
+    PIE_LAUNCH_CHECK();
+    ++p.launches;
+    for (int i = 0; i < n && !p.rc; ++i) {
+        const pie_stack_layer &L = s->layers[i];
+        const PointNorm after = i + 1 < n ? norm_of(s->layers[i + 1].pre1) : fin;
+        latent_mixer(p, i, L, L.ff == PIE_FF_NONE ? after : norm_of(L.pre2));
+        if (L.ff != PIE_FF_NONE) feed_forward(p, i, L, after);
+        if (b.tap && !p.rc)
+            PIE_HIP_TRY(hipMemcpy2DAsync(b.tap + (size_t)i * M * W, (size_t)W * 4, s->x.p, (size_t)W8 * 4, (size_t)W * 4, (size_t)M, hipMemcpyDeviceToDevice, st));
+    }
+    if (b.n_want > 0) {
+        RowsArgs a = {};
+        a.m = {(const char *)s->cfg.head, V, W, s->h.p, W8, b.logits, V};
+        a.M = b.n_want, a.epi = ROWS_SCALE_F32, a.scale = s->cfg.logit_scale, a.rows = b.want;
+        p.linear(a);
+        if (!p.rc && b.next) {
+            hipLaunchKernelGGL(k_f32_stats, dim3(ST_TILES, (unsigned)b.n_want), dim3(256), 0, st, b.logits, V, s->stats.p);
+            PIE_LAUNCH_CHECK();
+            hipLaunchKernelGGL(k_f32_finish, dim3(b.logprobs ? 32 : 1, (unsigned)b.n_want), dim3(256), 0, st, b.logits, V, s->stats.p, b.logprobs, b.next, b.advance,
+                               b.ids, b.pos, b.history, b.history_len);
+            PIE_LAUNCH_CHECK();
+            p.launches += 2;
+        }
+    }
+    s->launches = p.launches;
+    return p.rc;
+}
+
+}  // namespace
+
+extern "C" {
+
+int pie_stack_create(const pie_stack_config *cfg, pie_stack **out) {
+    PIE_REQUIRE(cfg && out, PIE_E_ARG, "pie_stack_create: null pointer");
+    PIE_REQUIRE(cfg->dtype == PIE_BF16 || cfg->dtype == PIE_F32, PIE_E_ARG, "pie_stack_create: dtype must be PIE_BF16 or PIE_F32");
+    PIE_REQUIRE(cfg->width > 0 && cfg->vocab > 0 && cfg->n_layers >= 0, PIE_E_SHAPE, "pie_stack_create: bad sizes");
+    PIE_REQUIRE(cfg->embed && cfg->head && cfg->final_norm.w && cfg->final_norm.b, PIE_E_ARG, "pie_stack_create: missing weights");
+    pie_stack *s = new (std::nothrow) pie_stack();
+    PIE_REQUIRE(s, PIE_E_HIP, "pie_stack_create: out of host memory");
+    s->cfg = *cfg;
+    s->layers.resize(cfg->n_layers), s->have.assign(cfg->n_layers, 0), s->route.assign(cfg->n_layers, RouteLayer{});
+    *out = s;
+    return PIE_OK;
+}
+
+int pie_stack_destroy(pie_stack *s) {
+    delete s;
+    return PIE_OK;
+}
+
+int pie_stack_set_layer(pie_stack *s, int i, const pie_stack_layer *L) {
+    PIE_REQUIRE(s && L && i >= 0 && i < s->cfg.n_layers, PIE_E_ARG, "pie_stack_set_layer: bad argument");
+    auto norm_ok = [](const pie_point_norm &n) { return n.w && n.b; };
+    PIE_REQUIRE(L->mixer == PIE_MIXER_LATENT, PIE_E_ARG, "pie_stack_set_layer: unknown mixer");
+    PIE_REQUIRE(L->heads > 0 && L->dim > 0 && L->vdim > 0 && L->rank > 0 && L->rank <= 2048, PIE_E_SHAPE, "pie_stack_set_layer: bad mixer sizes (kv_rank at most 2048)");
+    PIE_REQUIRE(L->w_in && L->w_uk && L->w_uv && L->w_o && L->c_norm && norm_ok(L->pre1) && norm_ok(L->post1), PIE_E_ARG, "pie_stack_set_layer: missing mixer weights");
+    PIE_REQUIRE(L->ff == PIE_FF_NONE || (norm_ok(L->pre2) && norm_ok(L->post2) && L->ff_size > 0), PIE_E_ARG, "pie_stack_set_layer: missing feed-forward norms");
+    if (L->ff == PIE_FF_RELU2) PIE_REQUIRE(L->w_up && L->w_down, PIE_E_ARG, "pie_stack_set_layer: missing dense weights");
+    else if (L->ff == PIE_FF_TABLE_MOE) {
+        PIE_REQUIRE(L->experts > 0 && L->experts <= 8192 && L->top > 0 && L->top <= L->experts, PIE_E_SHAPE, "pie_stack_set_layer: bad expert counts");
+        PIE_REQUIRE(L->table && L->w_gate_up && L->w_expert_down, PIE_E_ARG, "pie_stack_set_layer: missing expert weights");
+        PIE_REQUIRE(L->shared_size == 0 || (L->shared_size > 0 && L->s_gate_up && L->s_down && L->shared_gate), PIE_E_ARG, "pie_stack_set_layer: missing shared expert");
+    } else PIE_REQUIRE(L->ff == PIE_FF_NONE, PIE_E_ARG, "pie_stack_set_layer: unknown feed-forward");
+    s->n_route += (L->ff == PIE_FF_TABLE_MOE) - (s->route[i].experts > 0);
+    s->route[i] = RouteLayer{};
+    if (L->ff == PIE_FF_TABLE_MOE) s->route[i].table = L->table, s->route[i].top = L->top, s->route[i].experts = L->experts;
+    s->route_rows = 0;
+    s->layers[i] = *L, s->have[i] = 1;
+    s->drop_graphs();
+    return PIE_OK;
+}
+
+int pie_stack_page_row(const pie_stack *s, int i) { return s && i >= 0 && i < s->cfg.n_layers && s->have[i] ? up8(s->layers[i].rank) : 0; }
+size_t pie_stack_page_bytes(const pie_stack *s, int i) { return (size_t)pie_stack_page_row(s, i) * PAGE_TOKENS * (s ? esize(s) : 0); }
+int pie_stack_launches(const pie_stack *s) { return s ? s->launches : 0; }
+
+int pie_stack_forward(pie_stack *s, const pie_stack_batch *bp, int flags, void *stream) {
+    PIE_REQUIRE(s && bp, PIE_E_ARG, "pie_stack_forward: null pointer");
+    const pie_stack_batch &b = *bp;
+    hipStream_t st = (hipStream_t)stream;
+    for (char h : s->have) PIE_REQUIRE(h, PIE_E_STATE, "pie_stack_forward: a layer has not been set");
+    PIE_REQUIRE(b.n_rows > 0 && b.n_rows <= 65535 && b.n_seqs > 0 && b.table_width > 0 && b.n_runs > 0 && b.n_want >= 0 && b.n_pages > 0, PIE_E_SHAPE,
+                "pie_stack_forward: a pass holds 1 .. 65535 rows of at least one sequence");
+    PIE_REQUIRE(b.ids && b.pos && b.row_seq && b.table && b.runs && b.runs_host && b.slabs, PIE_E_ARG, "pie_stack_forward: null pointer");
+    PIE_REQUIRE(b.n_want == 0 || b.logits, PIE_E_ARG, "pie_stack_forward: logits are asked for but have no buffer");
+    PIE_REQUIRE(b.n_want <= b.n_rows && (b.want || b.n_want == 0 || b.n_want == b.n_rows), PIE_E_ARG, "pie_stack_forward: bad list of wanted rows");
+    PIE_REQUIRE(!b.advance || (b.n_want == b.n_rows && !b.want && b.n_runs == b.n_rows && b.next), PIE_E_ARG, "pie_stack_forward: only a decode step can feed itself");
+    int at = 0;
+    for (int i = 0; i < b.n_runs; ++i) {
+        const int32_t *r = b.runs_host + 4 * i;
+        PIE_REQUIRE(r[0] == at && r[1] > 0 && r[2] >= 0 && r[2] < b.n_seqs, PIE_E_ARG, "pie_stack_forward: the runs must cover the rows in order");
+        at += r[1];
+    }
+    PIE_REQUIRE(at == b.n_rows, PIE_E_ARG, "pie_stack_forward: the runs must cover the rows in order");
+    for (int i = 0; i < s->cfg.n_layers; ++i) PIE_REQUIRE(b.slabs[i], PIE_E_ARG, "pie_stack_forward: a layer has no pages");
+    int rc = stack_reserve(s, b, st);
+    if (rc) return rc;
+    size_t ws = 0;
+    for (const pie_stack_layer &L : s->layers)
+        ws = std::max(ws, latent_attn_ws_floats(b.n_rows, L.heads, L.rank, plan_splits(b, L, stack_tiles(b.runs_host, b.n_runs, L.heads))));
+    bool moved = false;
+    if ((rc = s->attn_ws.need(ws, &moved))) return rc;
+    if (moved) s->drop_graphs();
+    if (!(flags & PIE_STEP_GRAPH) || b.tap) return stack_enqueue(s, b, st);
+
+    GraphKey key;
+    key.b = b;
+    key.b.slabs = nullptr, key.b.runs_host = nullptr;
+    key.slabs.assign(b.slabs, b.slabs + s->cfg.n_layers), key.runs.assign(b.runs_host, b.runs_host + 4 * b.n_runs);
+    GraphSlot *slot = nullptr;
+    for (GraphSlot &g : s->graphs)
+        if (g.key.same(key)) slot = &g;
+    if (!slot) {  // first pass of this shape: runs as launches (and loads every kernel)
+        if (s->graphs.size() >= 4) {
+            size_t old = 0;
+            for (size_t i = 1; i < s->graphs.size(); ++i)
+                if (s->graphs[i].used < s->graphs[old].used) old = i;
+            if (s->graphs[old].exec) (void)hipGraphExecDestroy(s->graphs[old].exec);
+            s->graphs.erase(s->graphs.begin() + old);
+        }
+        s->graphs.push_back({key, nullptr, ++s->tick});
+        return stack_enqueue(s, b, st);
+    }
+    slot->used = ++s->tick;
+    if (!slot->exec) {
+        hipGraph_t graph = nullptr;
+        hipStream_t cs = nullptr;
+        PIE_HIP_TRY(hipStreamCreateWithFlags(&cs, hipStreamNonBlocking));
+        hipError_t e = hipStreamBeginCapture(cs, hipStreamCaptureModeThreadLocal);
+        if (e == hipSuccess) {
+            rc = stack_enqueue(s, b, cs);
+            e = hipStreamEndCapture(cs, &graph);
+        }
+        if (e == hipSuccess && !rc) e = hipGraphInstantiate(&slot->exec, graph, nullptr, nullptr, 0);
+        if (graph) (void)hipGraphDestroy(graph);
+        (void)hipStreamDestroy(cs);
+        if (rc) return rc;
+        PIE_HIP_TRY(e);
+    }
+    PIE_HIP_TRY(hipGraphLaunch(slot->exec, st));
+    return PIE_OK;
+}
+
+}  // extern "C"

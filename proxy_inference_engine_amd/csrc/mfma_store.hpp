@@ -7,6 +7,23 @@
 // 16-byte fragments.  So the rounded tile goes through LDS -- free after the K loop; each wave its own region, rows XOR-swizzled in 8-byte slots:
 // conflict-free both ways -- and leaves as 16 bytes per lane, 8 (or 4) lanes per row.
 #pragma once
+#include "prefill_attn.hpp"  // f32x16_t, the 16-bit traits
+
+// two fp32 -> one packed pair of T in a single v_cvt_pk_* (pack2<T> converts each half separately and ORs them: 3 instructions)
+template <class T>
+__device__ __forceinline__ u32 w4m_pack(float lo, float hi);
+template <>
+__device__ __forceinline__ u32 w4m_pack<BF16>(float lo, float hi) {
+    typedef float f2_t __attribute__((ext_vector_type(2)));
+    typedef __bf16 b2_t __attribute__((ext_vector_type(2)));
+    return __builtin_bit_cast(u32, __builtin_convertvector((f2_t){lo, hi}, b2_t));
+}
+template <>
+__device__ __forceinline__ u32 w4m_pack<F16>(float lo, float hi) {
+    typedef float f2_t __attribute__((ext_vector_type(2)));
+    typedef _Float16 h2_t __attribute__((ext_vector_type(2)));
+    return __builtin_bit_cast(u32, __builtin_convertvector((f2_t){lo, hi}, h2_t));
+}
 
 // acc[s][mi]: strip nt0 + s (32 columns), row block mi of the wave's tile; ot: the wave's LDS region, 32 MB x OB bytes (OB = 64 SW, or 32 SW with
 // SWIGLU); m0: the tile's first row, rows: its live rows; N: the Linear's out_features (stores clipped to it), ldy: output row stride (elements);
@@ -75,4 +92,17 @@ __device__ __forceinline__ void mfma_tile_store(const f32x16_t (&acc)[SW][MB], c
                 if (col + e < ldo) dst[e] = (u16)(w[e >> 1] >> (16 * (e & 1)));
         }
     }
+}
+
+// y = T(sum over z, in z order, of the fp32 partial tiles)
+template <class T>
+__global__ void __launch_bounds__(256) k_w4l_reduce(const float *part, int S, size_t MN, u16 *y) {
+    const size_t i = ((size_t)blockIdx.x * 256 + threadIdx.x) * 4;
+    if (i >= MN) return;
+    float4 a = *reinterpret_cast<const float4 *>(part + i);
+    for (int z = 1; z < S; ++z) {
+        const float4 b = *reinterpret_cast<const float4 *>(part + (size_t)z * MN + i);
+        a.x += b.x, a.y += b.y, a.z += b.z, a.w += b.w;
+    }
+    *reinterpret_cast<uint2 *>(y + i) = make_uint2(w4m_pack<T>(a.x, a.y), w4m_pack<T>(a.z, a.w));
 }

@@ -1,0 +1,251 @@
+// rows_gemm.hip -- the Linear of the layer-stack models: y[M, N] = x[M, K] . W[N, K]^T with the consumer's element-wise work in the epilogue.
+//
+// Few rows (a decode step, a short portion): the weights are read once and everything else is small.  A workgroup of eight waves owns
+// 16 * NW output features; KW waves split K between them (NW * KW = 8).  A wave streams 1-KiB pieces of the W16M tiles (w16_gemm.hpp: 32
+// features x 64 columns in MFMA operand order) -- half a tile row group per instruction, four 256-byte runs -- straight into the A operand of
+// v_mfma_f32_16x16x32_bf16; the B operand is the matching 16 B of up to 16 rows of x, read through L2.  One row of x uses one of the 16 columns,
+// which costs nothing: the matrix cores are idle either way.  The K-split partial sums meet in LDS.
+//
+// The same kernel runs batched over heads (per-head up- / down-projections), grouped over the active experts of a mixture (row lists), and for
+// any M (blockIdx.z walks 16 * NT rows at a time).
+#include "stack_types.hpp"
+
+size_t w16m_size(int N, int K);
+
+typedef __attribute__((ext_vector_type(8))) __bf16 mf_bf16x8;
+typedef __attribute__((ext_vector_type(4))) float mf_f32x4;
+typedef __attribute__((ext_vector_type(4))) u32 mf_u32x4;
+
+namespace {
+
+// What blockIdx.y selects: the matrix, its live rows, and how result rows map to x rows.
+struct RowsWork {
+    const char *w;
+    const void *x;
+    void *y;
+    int N, K, ldx, ldy, count, row0;
+    const int *rows;  // x row of local row i (nullptr: row0 + i)
+    int xoff, yoff;
+};
+__device__ __forceinline__ bool rows_select(const RowsArgs &a, RowsWork &k) {
+    k.w = a.m.w, k.x = a.m.x, k.y = a.m.y, k.N = a.m.N, k.K = a.m.K, k.ldx = a.m.ldx, k.ldy = a.m.ldy;
+    k.count = a.M, k.row0 = 0, k.rows = a.rows, k.xoff = k.yoff = 0;
+    const int b = blockIdx.y;
+    if (a.shared.w && b == (int)gridDim.y - 1) {
+        k.w = a.shared.w, k.x = a.shared.x, k.y = a.shared.y, k.N = a.shared.N, k.K = a.shared.K, k.ldx = a.shared.ldx, k.ldy = a.shared.ldy;
+        return true;
+    }
+    if (a.active) {
+        const int e = a.active[b];
+        if (e < 0) return false;
+        k.row0 = a.offset[e], k.count = a.offset[e + 1] - k.row0;
+        if (a.gather) k.rows = a.list + k.row0;
+        k.w += (size_t)e * a.w_batch;
+        return true;
+    }
+    k.w += (size_t)b * a.w_batch, k.xoff = b * a.x_batch, k.yoff = b * a.y_batch;
+    return true;
+}
+
+// One finished value (m: result row inside the group, n: feature); pair: the value of feature n + 1 (ROWS_SILU_MUL)
+template <class E>
+__device__ __forceinline__ void rows_finish(const RowsArgs &a, const RowsWork &k, int m, int n, float v, float pair) {
+    typedef typename E::type T;
+    const size_t row = (size_t)(k.row0 + m);
+    switch (a.epi) {
+        case ROWS_STORE: ((T *)k.y)[row * k.ldy + k.yoff + n] = E::pack(v); break;
+        case ROWS_SCALE_F32: ((float *)k.y)[row * k.ldy + k.yoff + n] = v * a.scale; break;
+        case ROWS_RELU2: {
+            const float r = fmaxf(v, 0.0f);
+            ((T *)k.y)[row * k.ldy + n] = E::pack(r * r);
+            break;
+        }
+        case ROWS_SILU_MUL:
+            if (!(n & 1)) ((T *)k.y)[row * k.ldy + (n >> 1)] = E::pack(v / (1.0f + expf(-v)) * pair);
+            break;
+        case ROWS_SPLIT:
+            if (n < a.split) ((T *)k.y)[row * k.ldy + n] = E::pack(v);
+            else a.y2[row * a.ldy2 + n - a.split] = v;
+            break;
+        case ROWS_RESIDUAL: {
+            float *xp = a.res + row * a.ld_res + n;
+            const float x = *xp + point_norm(a.post, n, v);
+            *xp = x;
+            ((T *)a.h)[row * a.ldh + n] = E::pack(point_norm(a.next, n, x));
+            break;
+        }
+    }
+}
+
+// NT: blocks of 16 rows of x; KW: waves along K
+template <int NT, int KW>
+__global__ void __launch_bounds__(512) k_rows_w16m(const RowsArgs a) {
+    constexpr int NW = 8 / KW, U = NT >= 4 ? 2 : 4;
+    constexpr int ST = 20;  // floats per (row, 16 features) line of the reduction image
+    __shared__ __attribute__((aligned(16))) float s_red[8 * NT * 16 * ST];
+    RowsWork k;
+    if (!rows_select(a, k)) return;
+    const int i0 = blockIdx.z * 16 * NT;
+    if (i0 >= k.count) return;
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int wn = wave / KW, wk = wave % KW;
+    const int t16 = blockIdx.x * NW + wn;  // this wave's 16 output features
+    if ((int)blockIdx.x * NW * 16 >= k.N) return;
+    const int c = lane & 15, kq = lane >> 4;
+    const int groups = (k.K + 63) >> 6, steps = 2 * groups;
+    const bool live = t16 * 16 < k.N;
+
+    mf_f32x4 acc[NT];
+#pragma unroll
+    for (int t = 0; t < NT; ++t) acc[t] = (mf_f32x4){0.0f, 0.0f, 0.0f, 0.0f};
+    if (live) {
+        const char *wp = k.w + (size_t)(t16 >> 1) * groups * 4096 + ((kq >> 1) * 1024 + ((kq & 1) * 32 + (t16 & 1) * 16 + c) * 16);
+        const u16 *xp[NT];
+#pragma unroll
+        for (int t = 0; t < NT; ++t) {
+            int i = i0 + 16 * t + c;
+            i = i < k.count ? i : k.count - 1;  // rows past the end repeat the last one (never stored)
+            const int xr = k.rows ? k.rows[i] : k.row0 + i;
+            xp[t] = (const u16 *)k.x + (size_t)xr * k.ldx + k.xoff + 8 * kq;
+        }
+        auto fetch = [&](int s, mf_u32x4(&wv)[U], mf_u32x4(&xv)[U][NT]) {
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                const int ss = s + u * KW, cl = ss < steps ? ss : steps - 1;
+                wv[u] = __builtin_nontemporal_load((const mf_u32x4 *)(wp + (size_t)cl * 2048));
+#pragma unroll
+                for (int t = 0; t < NT; ++t) xv[u][t] = *(const mf_u32x4 *)(xp[t] + 32 * cl);
+            }
+        };
+        auto multiply = [&](int s, const mf_u32x4(&wv)[U], const mf_u32x4(&xv)[U][NT]) {
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                mf_u32x4 w = wv[u];
+                if (s + u * KW >= steps) w = (mf_u32x4){0u, 0u, 0u, 0u};
+#pragma unroll
+                for (int t = 0; t < NT; ++t)
+                    acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(mf_bf16x8, w), __builtin_bit_cast(mf_bf16x8, xv[u][t]), acc[t], 0, 0, 0);
+            }
+        };
+        mf_u32x4 w0[U], w1[U], x0[U][NT], x1[U][NT];
+        fetch(wk, w0, x0);
+        for (int s = wk; s < steps; s += 2 * U * KW) {
+            fetch(s + U * KW, w1, x1);
+            multiply(s, w0, x0);
+            fetch(s + 2 * U * KW, w0, x0);
+            multiply(s + U * KW, w1, x1);
+        }
+    }
+    // lane (kq, c) holds features 4 kq .. + 3 of row c
+#pragma unroll
+    for (int t = 0; t < NT; ++t) *(mf_f32x4 *)(s_red + ((wave * NT + t) * 16 + c) * ST + 4 * kq) = acc[t];
+    __syncthreads();
+    for (int id = threadIdx.x; id < NW * NT * 256; id += 512) {
+        const int nl = id & 15, ml = (id >> 4) % (16 * NT), w = id / (256 * NT);
+        const int n = ((int)blockIdx.x * NW + w) * 16 + nl, m = i0 + ml;
+        if (n >= k.N || m >= k.count) continue;
+        if (a.epi == ROWS_SILU_MUL && (nl & 1)) continue;
+        const float *r = s_red + ((w * KW * NT + (ml >> 4)) * 16 + (ml & 15)) * ST + nl;
+        float v = 0.0f, p = 0.0f;
+#pragma unroll
+        for (int q = 0; q < KW; ++q) v += r[q * NT * 16 * ST];
+        if (a.epi == ROWS_SILU_MUL)
+#pragma unroll
+            for (int q = 0; q < KW; ++q) p += r[q * NT * 16 * ST + 1];
+        rows_finish<ElemBF16>(a, k, m, n, v, p);
+    }
+}
+
+// fp32: one output per thread, 16 features x 16 rows per workgroup, both operands through LDS
+__global__ void __launch_bounds__(256) k_rows_f32(const RowsArgs a) {
+    __shared__ float s_w[16][65], s_x[16][65], s_v[16][17];
+    RowsWork k;
+    if (!rows_select(a, k)) return;
+    const int i0 = blockIdx.z * 16, n0 = blockIdx.x * 16;
+    if (i0 >= k.count || n0 >= k.N) return;
+    const int tn = threadIdx.x & 15, tm = threadIdx.x >> 4;
+    const int Kp = (k.K + 63) & ~63;
+    float acc = 0.0f;
+    for (int k0 = 0; k0 < Kp; k0 += 64) {
+        for (int id = threadIdx.x; id < 1024; id += 256) {
+            const int r = id >> 6, c = id & 63;
+            s_w[r][c] = n0 + r < k.N ? ((const float *)k.w)[(size_t)(n0 + r) * Kp + k0 + c] : 0.0f;
+            int i = i0 + r;
+            i = i < k.count ? i : k.count - 1;
+            const int xr = k.rows ? k.rows[i] : k.row0 + i;
+            s_x[r][c] = k0 + c < k.K ? ((const float *)k.x)[(size_t)xr * k.ldx + k.xoff + k0 + c] : 0.0f;
+        }
+        __syncthreads();
+#pragma unroll 16
+        for (int c = 0; c < 64; ++c) acc = fmaf(s_w[tn][c], s_x[tm][c], acc);
+        __syncthreads();
+    }
+    s_v[tm][tn] = acc;
+    __syncthreads();
+    const int n = n0 + tn, m = i0 + tm;
+    if (n < k.N && m < k.count) rows_finish<ElemF32>(a, k, m, n, acc, s_v[tm][tn < 15 ? tn + 1 : 15]);
+}
+
+template <int NT>
+int rows_go(const RowsArgs &a, int n_max, int k_max, int batches, hipStream_t st) {
+    const int steps = 2 * ((k_max + 63) / 64), tiles = (n_max + 15) / 16, z = (a.M + 16 * NT - 1) / (16 * NT);
+    // waves along K: enough steps for each, and enough workgroups for the chip
+    int kw = steps >= 32 ? 8 : steps >= 16 ? 4 : steps >= 8 ? 2 : 1;
+    while (kw < 8 && steps >= 2 * kw && (size_t)((tiles + 8 / kw - 1) / (8 / kw)) * batches * z < 256) kw *= 2;
+    const dim3 grid((unsigned)((tiles + 8 / kw - 1) / (8 / kw)), (unsigned)batches, (unsigned)z);
+    if (kw == 8) hipLaunchKernelGGL((k_rows_w16m<NT, 8>), grid, dim3(512), 0, st, a);
+    else if (kw == 4) hipLaunchKernelGGL((k_rows_w16m<NT, 4>), grid, dim3(512), 0, st, a);
+    else if (kw == 2) hipLaunchKernelGGL((k_rows_w16m<NT, 2>), grid, dim3(512), 0, st, a);
+    else hipLaunchKernelGGL((k_rows_w16m<NT, 1>), grid, dim3(512), 0, st, a);
+    PIE_LAUNCH_CHECK();
+    return PIE_OK;
+}
+
+__global__ void __launch_bounds__(256) k_pack_f32(const u16 *w, int N, int K, int Kp, float *out) {
+    const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= (size_t)N * Kp) return;
+    const int n = (int)(i / Kp), c = (int)(i % Kp);
+    out[i] = c < K ? BF16::to_f32(w[(size_t)n * K + c]) : 0.0f;
+}
+
+}  // namespace
+
+size_t rows_weight_bytes(int dtype, int N, int K) {
+    return dtype == PIE_F32 ? (size_t)N * ((K + 63) & ~63) * 4 : w16m_size(N, K);
+}
+
+int rows_gemm_launch(int dtype, const RowsArgs &a, int batches, hipStream_t st) {
+    if (a.M <= 0 || batches <= 0) return PIE_OK;
+    PIE_REQUIRE(a.m.N > 0 && a.m.K > 0, PIE_E_SHAPE, "row-wise Linear: empty matrix");
+    PIE_REQUIRE(batches <= 65535, PIE_E_SHAPE, "row-wise Linear: too many batches");
+    const int n_max = a.shared.w && a.shared.N > a.m.N ? a.shared.N : a.m.N, k_max = a.shared.w && a.shared.K > a.m.K ? a.shared.K : a.m.K;
+    if (dtype == PIE_F32) {
+        const dim3 grid((unsigned)((n_max + 15) / 16), (unsigned)batches, (unsigned)((a.M + 15) / 16));
+        hipLaunchKernelGGL(k_rows_f32, grid, dim3(256), 0, st, a);
+        PIE_LAUNCH_CHECK();
+        return PIE_OK;
+    }
+    PIE_REQUIRE(a.m.ldx % 8 == 0 && a.x_batch % 8 == 0 && pie_aligned(a.m.x, 16) && pie_aligned(a.m.w, 16), PIE_E_ALIGN, "row-wise Linear: 16-byte alignment required");
+    if (a.M <= 16) return rows_go<1>(a, n_max, k_max, batches, st);
+    if (a.M <= 32) return rows_go<2>(a, n_max, k_max, batches, st);
+    return rows_go<4>(a, n_max, k_max, batches, st);
+}
+
+extern "C" {
+
+size_t pie_stack_weight_bytes(int dtype, int N, int K) {
+    return N > 0 && K > 0 && (dtype == PIE_BF16 || dtype == PIE_F32) ? rows_weight_bytes(dtype, N, K) : 0;
+}
+
+int pie_stack_pack_weight(const void *w, int N, int K, int dtype, void *packed, void *stream) {
+    PIE_REQUIRE(w && packed, PIE_E_ARG, "pie_stack_pack_weight: null pointer");
+    PIE_REQUIRE(N > 0 && K > 0, PIE_E_SHAPE, "pie_stack_pack_weight: empty matrix");
+    if (dtype == PIE_BF16) return pie_repack_w16m(w, N, K, PIE_BF16, packed, stream);
+    PIE_REQUIRE(dtype == PIE_F32, PIE_E_ARG, "pie_stack_pack_weight: dtype must be PIE_BF16 or PIE_F32");
+    const int Kp = (K + 63) & ~63;
+    hipLaunchKernelGGL(k_pack_f32, dim3((unsigned)(((size_t)N * Kp + 255) / 256)), dim3(256), 0, (hipStream_t)stream, (const u16 *)w, N, K, Kp, (float *)packed);
+    PIE_LAUNCH_CHECK();
+    return PIE_OK;
+}
+
+}  // extern "C"

@@ -1,0 +1,103 @@
+// stack_types.hpp -- what the kernels of the layer-stack models share: the element types, the norms that ride in epilogues, and the operand
+// descriptions of the row-wise Linear (rows_gemm.hip) and of the latent attention (latent_attn.hip).
+//
+// Every activation row has a stride that is a multiple of 8 elements; a Linear reads 64 ceil(K / 64) elements of it.  The columns past K meet zero
+// weights, so they only have to be finite: the owner zero-fills its buffers once and keeps 64 elements of slack behind each.
+#pragma once
+#include "common.hpp"
+
+constexpr int PAGE_TOKENS = 64;
+
+// Element types of a stack: 16-bit storage (MFMA products, fp32 accumulation) or fp32 throughout.
+struct ElemBF16 {
+    typedef u16 type;
+    static __device__ __forceinline__ float load(const u16 *p) { return BF16::to_f32(*p); }
+    static __device__ __forceinline__ u16 pack(float v) { return BF16::from_f32(v); }
+};
+struct ElemF32 {
+    typedef float type;
+    static __device__ __forceinline__ float load(const float *p) { return *p; }
+    static __device__ __forceinline__ float pack(float v) { return v; }
+};
+
+// A norm without statistics, applied element by element in fp32: w * tanh(alpha x) + b (Dynamic Tanh).  Because it needs no reduction over the row,
+// the kernel that produces an element can apply both the norm behind its own sublayer and the norm in front of the next one.
+struct PointNorm {
+    const float *w, *b;
+    float alpha;
+};
+__device__ __forceinline__ float point_norm(const PointNorm &n, int i, float x) { return fmaf(tanhf(n.alpha * x), n.w[i], n.b[i]); }
+
+// ---------------------------------------------------------------- the row-wise Linear
+enum RowsEpi {
+    ROWS_STORE = 0,      // y[m][n] = T(v)
+    ROWS_SCALE_F32 = 1,  // y[m][n] = v * scale, fp32 (logits; expert outputs, scale 1)
+    ROWS_RELU2 = 2,      // y[m][n] = T(max(v, 0)^2)
+    ROWS_SILU_MUL = 3,   // rows (2 i, 2 i + 1) = (gate_i, up_i): y[m][i] = T(silu(gate) * up)
+    ROWS_SPLIT = 4,      // n < split: y[m][n] = T(v);  else y2[m][n - split] = v, fp32
+    ROWS_RESIDUAL = 5,   // x[m][n] += post(v);  h[m][n] = T(next(x[m][n]))
+};
+
+struct RowsMat {      // one weight matrix with its operand and result
+    const char *w;    // W16M tiles (bf16) or row-major fp32 [N][64 ceil(K / 64)]
+    int N, K;
+    const void *x;
+    int ldx;          // elements
+    void *y;
+    int ldy;
+};
+struct RowsArgs {
+    RowsMat m;
+    int M;                 // rows of x (grouped: an upper bound for one expert's rows)
+    // batched over blockIdx.y (heads): offsets per batch index
+    size_t w_batch;        // bytes
+    int x_batch, y_batch;  // elements
+    // grouped over blockIdx.y (experts): active[y] = expert or -1; its rows are list[offset[e] .. offset[e + 1])
+    const int *active, *offset, *list;
+    bool gather;           // grouped: x row = list[position] (else x row = position); y row = position always
+    RowsMat shared;        // blockIdx.y == batches - 1 when shared.w: all M rows, this matrix (the expert every token takes)
+    const int *rows;       // ungrouped, nullable: x row of result row i
+    int epi;
+    float scale;
+    int split;
+    float *y2;
+    int ldy2;
+    // ROWS_RESIDUAL
+    float *res;            // [M][ld_res] residual stream
+    int ld_res;
+    PointNorm post, next;
+    void *h;               // [M][ldh]
+    int ldh;
+};
+// batches: blockIdx.y extent (1 for a plain Linear; heads; active experts (+ 1 with a shared expert))
+int rows_gemm_launch(int dtype, const RowsArgs &a, int batches, hipStream_t st);
+// bytes of a packed [N, K] weight of the stack's dtype, and the repack from row-major bf16
+size_t rows_weight_bytes(int dtype, int N, int K);
+
+// ---------------------------------------------------------------- latent attention
+// A pass holds runs of consecutive rows, one run per sequence; a workgroup takes up to 64 (token, head) pairs of ONE run.
+struct RowRun {
+    int row0, n_rows, seq, pad;  // seq: row of the block table
+};
+struct LatentAttnArgs {
+    const void *q;         // [M][H][ldr]: queries in the latent space (W_uk^T q), ldr = row stride in elements
+    const void *slab;      // the layer's latent pages [n_pages][64][ldr]
+    const int *table;      // [n_seqs][table_width] page ids
+    int table_width, n_pages, n_seqs;
+    const int *pos;        // [M]
+    const RowRun *runs;
+    int n_runs, n_tiles;   // n_tiles = sum over the runs of ceil(n_rows * H / 64)
+    bool single;           // every run is one row (a decode step): tile -> run without a search
+    const int *row_seq;    // [M]
+    int H, R, ldr, M;
+    int window;            // keys j with 0 <= i - j < window; <= 0: no limit
+    float scale;
+    int splits;            // > 1: fp32 partials in ws, merged by the combine launch
+    float *ws;             // [splits][M * H] x (R + 2): see latent_attn.hip
+    void *out;             // [M][H][ldr] T: softmax-weighted latents
+};
+int latent_attn_launch(int dtype, const LatentAttnArgs &a, hipStream_t st);
+size_t latent_attn_ws_floats(int M, int H, int R, int splits);
+// c_raw fp32 [M][ldc] -> RMS norm with weight w -> the row of its page
+int latent_append_launch(int dtype, const float *c_raw, int ldc, const float *w, float eps, int M, int R, int ldr, const int *pos, const int *row_seq,
+                         const int *table, int table_width, int n_pages, int n_seqs, void *slab, hipStream_t st);

@@ -55,22 +55,6 @@ __global__ void __launch_bounds__(256) k_w4s_to_w4m(const u32 *w4s, int N, int K
     }
 }
 
-// two fp32 -> one packed pair of T in a single v_cvt_pk_* (pack2<T> converts each half separately and ORs them: 3 instructions)
-template <class T>
-__device__ __forceinline__ u32 w4m_pack(float lo, float hi);
-template <>
-__device__ __forceinline__ u32 w4m_pack<BF16>(float lo, float hi) {
-    typedef float f2_t __attribute__((ext_vector_type(2)));
-    typedef __bf16 b2_t __attribute__((ext_vector_type(2)));
-    return __builtin_bit_cast(u32, __builtin_convertvector((f2_t){lo, hi}, b2_t));
-}
-template <>
-__device__ __forceinline__ u32 w4m_pack<F16>(float lo, float hi) {
-    typedef float f2_t __attribute__((ext_vector_type(2)));
-    typedef _Float16 h2_t __attribute__((ext_vector_type(2)));
-    return __builtin_bit_cast(u32, __builtin_convertvector((f2_t){lo, hi}, h2_t));
-}
-
 #include "mfma_store.hpp"  // the LDS-transposed output epilogue of the one-wave-per-SIMD GEMMs
 
 // 8 codes of one word -> 8 weights in T, the mx.dequantize arithmetic of k_dequant_w4s: T(fp32(s * q) + b), as the MFMA fragment
@@ -603,20 +587,6 @@ __global__ void __launch_bounds__(256) k_w4l2_gemm(const char *w4m, const u16 *x
     mfma_tile_store<T, MB, 2, SWIGLU>(acc, &s_x[0][0] + wave * (MT * (SWIGLU ? 64 : 128)), lane, nt0, m0, rows, N, SWIGLU ? N >> 1 : N, y, nullptr);
 }
 
-// y = T(sum over z, in z order, of the fp32 partial tiles)
-template <class T>
-__global__ void __launch_bounds__(256) k_w4l_reduce(const float *part, int S, size_t MN, u16 *y) {
-    const size_t i = ((size_t)blockIdx.x * 256 + threadIdx.x) * 4;
-    if (i >= MN) return;
-    float4 a = *reinterpret_cast<const float4 *>(part + i);
-    for (int z = 1; z < S; ++z) {
-        const float4 b = *reinterpret_cast<const float4 *>(part + (size_t)z * MN + i);
-        a.x += b.x, a.y += b.y, a.z += b.z, a.w += b.w;
-    }
-    *reinterpret_cast<uint2 *>(y + i) = make_uint2(w4m_pack<T>(a.x, a.y), w4m_pack<T>(a.z, a.w));
-}
-
-
 // K-split factor the launcher will use for [M, N, K]: enough workgroups for the chip, at least 8 groups (512 columns) per split.
 // Decomposition: row tile (64 / 128 / 256 rows) x K split, and which kernel.  The one-wave-per-SIMD form (k_w4l2_gemm) needs a multiple
 // of 4 K groups per split; where it applies, the plan takes the shallowest split that yields ~192 workgroups, and for that split the
@@ -732,162 +702,6 @@ int w4l_gemm_launch(int dtype, const void *w4m, const void *x, int M, int N, int
         if (dtype == PIE_BF16) hipLaunchKernelGGL(k_w4l_reduce<BF16>, rg, dim3(256), 0, st, part, S, MN, (u16 *)y);
         else hipLaunchKernelGGL(k_w4l_reduce<F16>, rg, dim3(256), 0, st, part, S, MN, (u16 *)y);
         PIE_LAUNCH_CHECK();
-    }
-    return PIE_OK;
-}
-
-// ---------------------------------------------------------------- 16-bit weights, many rows (w16_gemm.hpp)
-#include "w16_gemm.hpp"
-int bias_any_launch(int dtype, void *y, const void *bias, int M, int N, hipStream_t st);  // vision.hip
-
-static char *g_w16_zero = nullptr;  // 4 KiB of zeros: the weight tile of the ring's dummy steps
-static std::mutex g_w16_mutex;
-static int w16_zero_block(const char **out) {
-    std::lock_guard<std::mutex> lock(g_w16_mutex);
-    if (!g_w16_zero) {
-        PIE_HIP_TRY(hipMalloc((void **)&g_w16_zero, W16M_TILE_BYTES));
-        PIE_HIP_TRY(hipMemset(g_w16_zero, 0, W16M_TILE_BYTES));
-    }
-    *out = g_w16_zero;
-    return PIE_OK;
-}
-
-size_t w16m_size(int N, int K) { return w16m_bytes(N, K); }
-// row-major [N][K] (any N, K) -> W16M
-int w16m_from_rows_launch(const void *w, int N, int K, void *w16m, hipStream_t st) {
-    const char *zero;
-    if (const int rc = w16_zero_block(&zero)) return rc;  // (first use of the format: never under stream capture)
-    const int groups = (K + 63) / 64;
-    const size_t pieces = w16m_bytes(N, K) / 16;
-    hipLaunchKernelGGL(k_rows_to_w16m, dim3((unsigned)((pieces + 255) / 256)), dim3(256), 0, st, (const u16 *)w, N, K, groups, pieces, (uint4 *)w16m);
-    PIE_LAUNCH_CHECK();
-    return PIE_OK;
-}
-// W16S units (the dense decode stream) -> W16M, packed row order
-int w16m_from_w16s_launch(const void *w16s, int N, int K, void *w16m, hipStream_t st) {
-    const char *zero;
-    if (const int rc = w16_zero_block(&zero)) return rc;
-    const int groups = (K + 63) / 64;
-    const size_t pieces = w16m_bytes(N, K) / 16;
-    hipLaunchKernelGGL(k_w16s_to_w16m, dim3((unsigned)((pieces + 255) / 256)), dim3(256), 0, st, (const uint4 *)w16s, N, K, (K + 511) / 512, groups, pieces,
-                       (uint4 *)w16m);
-    PIE_LAUNCH_CHECK();
-    return PIE_OK;
-}
-
-// Decomposition: row tile (64 / 128 / 256 rows), strips per wave (workgroup = 128 or 256 columns) and K split, by a small cost model
-// calibrated on tools/w16_bench sweep (8B and vision-tower shapes, 64 .. 4096 rows): a K step of a (32 mb) x (128 sw) tile costs
-// t(mb, sw) us -- larger tiles are cheaper per MFMA (0.125 us per 32 x 32 block pair for 64 x 128, 0.09 for 256 x 256) but quantise worse --
-// less when part of the chip idles (the large tiles are power-bound: the clock rises); workgroups run in rounds of 256; few rows
-// are bound by the weight stream (~5.5 TB/s); a launch costs ~4 us of ramp, prologue and epilogue; a K split writes and re-reads its fp32
-// slabs and launches the reduce.
-struct W16Plan {
-    int mb, sw, S;
-};
-static int g_w16_plan_override[3] = {0, 0, 0};  // developer override (tools/w16_bench)
-static int g_w16_block[2] = {4, 8};              // XCD-local traversal block (row tiles x column tiles)
-#ifdef W16L_PROF
-static unsigned long long *g_w16_prof = nullptr;
-#endif
-static int w16_even_splits(int groups, int S) {  // the largest split count <= S whose ceil-sized runs are all non-empty
-    for (;;) {
-        const int per = (groups + S - 1) / S, s2 = (groups + per - 1) / per;
-        if (s2 == S) return S;
-        S = s2;
-    }
-}
-static W16Plan w16_plan(int M, int N, int K, bool no_split = false) {
-    const int groups = (K + 63) / 64;
-    if (g_w16_plan_override[0]) return {g_w16_plan_override[0], g_w16_plan_override[1], w16_even_splits(groups, g_w16_plan_override[2])};
-    const int mb_max = M <= 64 ? 2 : (M <= 128 ? 4 : 8);
-    W16Plan best = {mb_max, 2, 1};
-    double best_us = 1e30;
-    // t(mb, sw) = light + (full - light) * load: one partial round of workgroups runs at a higher clock than sustained full rounds
-    static const double t_light[4][3] = {{0, 0, 0}, {0, 0.25, 0.42}, {0, 0.31, 0.60}, {0, 0.50, 1.45}};  // [log2 mb][sw]
-    static const double t_full[4][3] = {{0, 0, 0}, {0, 0.25, 0.45}, {0, 0.48, 0.80}, {0, 0.83, 1.45}};
-    const double stream_us = 2.0 * N * (64.0 * groups) / 5.5e6;
-    for (int S = 1; S <= (no_split ? 1 : 16) && (S == 1 || 8 * S <= groups); ++S)
-        for (int mb = mb_max; mb >= 2; mb >>= 1)
-            for (int sw = 2; sw >= (no_split ? 2 : 1); --sw) {
-                const int wgs = ((N + 128 * sw - 1) / (128 * sw)) * ((M + 32 * mb - 1) / (32 * mb)) * S;
-                const int steps = ((groups + S - 1) / S + 3) & ~3;
-                const int rounds = (wgs + 255) / 256;
-                const double load = rounds > 1 ? 1.0 : (double)wgs / 256.0;
-                const int mi = mb == 8 ? 3 : (mb == 4 ? 2 : 1);
-                double us = rounds * steps * (t_light[mi][sw] + (t_full[mi][sw] - t_light[mi][sw]) * load);
-                us = (us > stream_us ? us : stream_us) + 4.0;
-                if (S > 1) us += (double)M * N * 4.0 * (2 * S + 0.5) / 4.0e6 + 2.0;
-                if (us < best_us) best_us = us, best = {mb, sw, S};
-            }
-    best.S = w16_even_splits(groups, best.S);
-    return best;
-}
-int w16l_splits(int M, int N, int K) { return w16_plan(M, N, K).S; }
-size_t w16l_workspace_bytes(int M, int N, int K) {
-    if (N & 3) return 0;
-    const int s = w16l_splits(M, N, K);
-    return s > 1 ? (size_t)s * M * N * sizeof(float) : 0;
-}
-
-// y [M, N] = x . W^T (+ bias), W in W16M tiles of an [N, K] Linear; x: M rows of ldx elements (0 = packed) holding 64 ceil(K / 64) used
-// columns, zeros past K.
-// swiglu_act (nullable): the packed gate|up matrix and the caller wants the MLP activation [M, N / 2] there; *fused says whether it got it.
-// workspace: w16l_workspace_bytes() of device scratch (may be null when that is 0).
-// ldy: row stride of the output that is written (y, or the activation; 0 = packed), a multiple of 4.
-int w16l_gemm_launch(int dtype, const void *w16m, const void *x, int ldx, int M, int N, int K, void *y, void *workspace, hipStream_t st, const void *bias,
-                     void *swiglu_act, bool *fused, int ldy) {
-    if (fused) *fused = false;
-    const int Kx = 64 * ((K + 63) / 64);
-    if (ldx == 0) ldx = Kx;
-    PIE_REQUIRE(ldx >= Kx && ldx % 8 == 0 && (size_t)256 * ldx * 2 < (1ull << 32), PIE_E_SHAPE,
-                "16-bit GEMM: x rows must hold 64 * ceil(K / 64) elements (zeros past K) at a stride that is a multiple of 8");
-    PIE_REQUIRE(M >= 1 && N > 0 && K > 0, PIE_E_SHAPE, "16-bit GEMM: empty operand");
-    PIE_REQUIRE(pie_aligned(w16m, 16) && pie_aligned(x, 16) && pie_aligned(y, 8) && (!bias || pie_aligned(bias, (N & 3) ? 2 : 8)), PIE_E_ALIGN, "16-bit GEMM: 16-byte alignment required");
-    PIE_REQUIRE(dtype == PIE_BF16 || dtype == PIE_F16, PIE_E_ARG, "16-bit GEMM: dtype must be PIE_BF16 or PIE_F16");
-    // swiglu_act without `fused`: the caller has no fallback (the C ABI's fused MLP): plan without a K split, two strips per wave
-    W16Plan plan = w16_plan(M, N, K, (swiglu_act && !fused) || (N & 3));  // (the fp32 slabs of a K split are written 16 bytes at a time)
-    const bool sg = swiglu_act && plan.S == 1;
-    if (sg) plan.sw = 2;  // (the fused activation is built for two strips per wave)
-    PIE_REQUIRE(plan.S == 1 || workspace, PIE_E_ARG, "16-bit GEMM: this shape splits K and needs its workspace");
-    W16Args a = {};
-    int rc = w16_zero_block(&a.zero);
-    if (rc) return rc;
-    PIE_REQUIRE(!sg || N % 8 == 0, PIE_E_SHAPE, "16-bit GEMM: a fused SwiGLU needs N % 8 == 0");
-    const int out_cols = sg ? N / 2 : N;
-    if (ldy == 0 || (swiglu_act && !sg)) ldy = out_cols;  // (a declined fusion writes the packed y)
-    PIE_REQUIRE(ldy >= out_cols, PIE_E_SHAPE, "16-bit GEMM: output row stride must cover the row");
-    PIE_REQUIRE(plan.S == 1 || ldy == N, PIE_E_SHAPE, "16-bit GEMM: a K-split shape writes packed rows");
-    a.w16m = (const char *)w16m, a.x = (const u16 *)x, a.M = M, a.N = N, a.K = Kx, a.ldx = ldx, a.ldy = ldy;
-    a.y = (u16 *)(sg ? swiglu_act : y), a.part = plan.S > 1 ? (float *)workspace : nullptr;
-    a.bias = plan.S > 1 ? nullptr : (const u16 *)bias;
-    a.tm = (M + 32 * plan.mb - 1) / (32 * plan.mb), a.tn = (N + 128 * plan.sw - 1) / (128 * plan.sw);
-    a.bm = g_w16_block[0] < a.tm ? g_w16_block[0] : a.tm, a.bc = g_w16_block[1];
-#ifdef W16L_PROF
-    a.prof = g_w16_prof;
-#endif
-    const dim3 grid((unsigned)(8 * ((a.tn + 7) / 8) * a.tm), (unsigned)plan.S);
-#define W16_GO(TT, MB_, SW_, SG_) hipLaunchKernelGGL((k_w16l_gemm<TT, MB_, SW_, SG_>), grid, dim3(256), 0, st, a)
-#define W16_SW(TT, MB_) \
-    if (sg) W16_GO(TT, MB_, 2, true); \
-    else if (plan.sw == 2) W16_GO(TT, MB_, 2, false); \
-    else W16_GO(TT, MB_, 1, false)
-#define W16_MB(TT) \
-    if (plan.mb == 2) { W16_SW(TT, 2); } \
-    else if (plan.mb == 4) { W16_SW(TT, 4); } \
-    else { W16_SW(TT, 8); }
-    if (dtype == PIE_BF16) { W16_MB(BF16) } else { W16_MB(F16) }
-#undef W16_MB
-#undef W16_SW
-#undef W16_GO
-    PIE_LAUNCH_CHECK();
-    if (sg && fused) *fused = true;
-    if (plan.S > 1) {
-        const size_t MN = (size_t)M * N;
-        const dim3 rg((unsigned)((MN / 4 + 255) / 256));
-        if (dtype == PIE_BF16) hipLaunchKernelGGL(k_w4l_reduce<BF16>, rg, dim3(256), 0, st, a.part, plan.S, MN, (u16 *)y);
-        else hipLaunchKernelGGL(k_w4l_reduce<F16>, rg, dim3(256), 0, st, a.part, plan.S, MN, (u16 *)y);
-        PIE_LAUNCH_CHECK();
-        if (bias) return bias_any_launch(dtype, y, bias, M, N, st);
     }
     return PIE_OK;
 }

@@ -159,6 +159,8 @@ class InferenceEngine:
 
         if len(self.prompt_cache.cache) == 0:
             self.prompt_cache.create_kv_cache(self.model)                      # :274-275
+        else:
+            self.prompt_cache.adopt(self.model)
         todo = self.prompt_cache(prompt_ids)                                   # :277
         host_ids = [int(t) for t in (todo.tolist() if isinstance(todo, torch.Tensor) else todo)]
         next_token, logprobs = _inference(torch.tensor(host_ids, dtype=torch.int32))   # :278 (host ids: no read-back)

@@ -1,0 +1,324 @@
+"""Models whose layers are listed one by one, run by the native layer stack (csrc/layer_stack.hip) over a paged latent cache.
+
+A design's module (e.g. models/taduzen) reads its config.json and packs its checkpoint into `pie_stack_layer` descriptions; this class is what every such
+model shares with the engines: the cache protocol (make_cache, enable_paged_kv), the calling convention (`model(inputs, cache=)`), the greedy fast
+path (`step`) and the multi-sequence passes (`step_batch`, `prefill_batch`, `step_mixed`, `step_portions`).  Every one of them is the same pass:
+rows of any sequences, each with its own position, in one batch."""
+from __future__ import annotations
+
+import ctypes as C
+
+import numpy as np
+import torch
+
+from .. import _ffi
+from ..cache.kv_cache import BaseCache, LatentPageAllocator, PagedLatentCache, PagedSequence, SavedLatentCache
+from ..cache.kv_cache.paged import TOKEN_CAPACITY_PER_PAGE
+
+MAX_ROWS = 4096  # rows of one pass; longer prompts run as several
+
+
+def pack_linear(w: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
+    """A Linear weight [N, K] (bf16, device) or a batch of equal ones [B, N, K] in the stack's packed form, as bytes [B * size]."""
+    w = w.to(torch.bfloat16).contiguous()
+    mats = w if w.dim() == 3 else w[None]
+    lib, code = _ffi.base(), _ffi.stack_dtype_code(dtype)
+    n = lib.pie_stack_weight_bytes(code, mats.shape[1], mats.shape[2])
+    out = torch.empty(mats.shape[0] * n, dtype=torch.uint8, device=w.device)
+    for i in range(mats.shape[0]):
+        _ffi.check(lib.pie_stack_pack_weight(mats[i].contiguous().data_ptr(), mats.shape[1], mats.shape[2], code, out.data_ptr() + i * n, _ffi.stream()))
+    return out
+
+
+class LayerStackModel:
+    def __init__(self, args, dtype: torch.dtype, width: int, vocab: int, logit_scale: float, layers: list[dict], embed: torch.Tensor, head: torch.Tensor,
+                 final_norm: tuple):
+        """layers: per layer the fields of pie_stack_layer -- tensors for its pointers, (alpha, w, b) triples for its norms, numbers for the rest
+        (absent fields are zero).  embed: bf16 [vocab, width]; head: packed."""
+        self.args, self.dtype, self.width, self.vocab_size = args, dtype, width, vocab
+        self.device = embed.device
+        self.layers = layers
+        self._held = [embed, head, final_norm]
+        lib = _ffi.base()
+        cfg = _ffi.pie_stack_config(_ffi.stack_dtype_code(dtype), width, vocab, len(layers), logit_scale, embed.data_ptr(), head.data_ptr(), self._norm(final_norm))
+        self._stack = C.c_void_p()
+        _ffi.check(lib.pie_stack_create(C.byref(cfg), C.byref(self._stack)))
+        for i, fields in enumerate(layers):
+            lay = _ffi.pie_stack_layer()
+            for name, v in fields.items():
+                setattr(lay, name, self._norm(v) if isinstance(v, tuple) else v.data_ptr() if isinstance(v, torch.Tensor) else v)
+            _ffi.check(lib.pie_stack_set_layer(self._stack, i, C.byref(lay)))
+        self.row_elems = [lib.pie_stack_page_row(self._stack, i) for i in range(len(layers))]
+        self.history = torch.zeros(1 << 20, dtype=torch.int32, device=self.device)  # history[p] = greedy token chosen for position p
+        self._pool: LatentPageAllocator | None = None
+        self._page_blocks = 16
+        self._bufs: dict = {}      # per decode batch size: the persistent buffers a captured step points at
+        torch.cuda.synchronize(self.device)
+
+    @staticmethod
+    def _norm(n: tuple):
+        alpha, w, b = n
+        return _ffi.pie_point_norm(w.data_ptr(), b.data_ptr(), alpha)
+
+    def __del__(self):
+        s = getattr(self, "_stack", None)
+        if s is not None and s.value:
+            try:
+                _ffi.base().pie_stack_destroy(s)
+            except Exception:  # noqa: BLE001  (interpreter shutdown)
+                pass
+            self._stack = None
+
+    # ------------------------------------------------------------------ caches
+    def enable_paged_kv(self, num_pages: int = 512, max_blocks: int = 16, kv_dtype: torch.dtype | None = None, kv_scales=None) -> LatentPageAllocator:
+        """From now on make_cache() draws on one pool of `num_pages` 64-token pages (all layers).  Returns the pool."""
+        if kv_dtype not in (None, self.dtype) or kv_scales is not None:
+            raise ValueError(f"latent pages are stored in the model's dtype ({self.dtype})")
+        self._pool = LatentPageAllocator(num_pages, self.row_elems, dtype=self.dtype, device=self.device)
+        self._page_blocks = max_blocks
+        return self._pool
+
+    def make_cache(self) -> list[BaseCache]:
+        if self._pool is None:
+            self.enable_paged_kv()
+        return self.make_paged_cache(self._pool, max_blocks=self._page_blocks)
+
+    def make_paged_cache(self, allocator: LatentPageAllocator | None = None, num_pages: int = 512, max_blocks: int = 16) -> list[BaseCache]:
+        if allocator is None:
+            allocator = LatentPageAllocator(num_pages, self.row_elems, dtype=self.dtype, device=self.device)
+        if not isinstance(allocator, LatentPageAllocator) or allocator.row_elems != self.row_elems or allocator.dtype != self.dtype or allocator.device is None:
+            raise ValueError("the allocator's geometry does not match this model")
+        seq = PagedSequence(allocator, max_blocks)
+        return [PagedLatentCache(seq, i) for i in range(len(self.layers))]
+
+    def adopt_cache(self, cache: list[BaseCache]) -> list[BaseCache]:
+        """Latents restored from a file, copied into pages; anything else as it is."""
+        if not isinstance(cache[0], SavedLatentCache):
+            return cache
+        out = self.make_cache()
+        for mine, saved in zip(out, cache):
+            mine.state = (saved.rows[:, :, :saved.offset], None)
+        return out
+
+    def _sequence(self, cache: list[BaseCache]) -> PagedSequence:
+        if len(cache) != len(self.layers) or not isinstance(cache[0], PagedLatentCache):
+            raise TypeError("a layer-stack model runs on its own paged caches (make_cache())")
+        return cache[0].page_manager
+
+    @staticmethod
+    def _sequences(seqs: list[PagedSequence]):
+        a = seqs[0].allocator
+        if any(s.allocator is not a for s in seqs) or len({id(s) for s in seqs}) != len(seqs):
+            raise ValueError("a pass takes distinct sequences of one page pool")
+        return a
+
+    # ------------------------------------------------------------------ the pass
+    def _forward(self, a: LatentPageAllocator, rows: int, ids, pos, row_seq, table, runs, runs_host: np.ndarray, want, n_want: int, logits, logprobs=None,
+                 nxt=None, advance: bool = False, history=None, graph: bool = False, tap=None) -> None:
+        p = lambda t: None if t is None else t.data_ptr()  # noqa: E731
+        slabs = (C.c_void_p * len(a.slabs))(*[s.data_ptr() for s in a.slabs])
+        b = _ffi.pie_stack_batch(rows, table.shape[0], table.shape[1], len(runs_host), n_want, int(advance), 0 if history is None else history.numel(), 0,
+                                 p(ids), p(pos), p(row_seq), p(table), p(runs), runs_host.ctypes.data, p(want), p(logits), p(logprobs), p(nxt), p(history),
+                                 C.cast(slabs, C.c_void_p), a.size(), p(tap))
+        _ffi.check(_ffi.base().pie_stack_forward(self._stack, C.byref(b), _ffi.PIE_STEP_GRAPH if graph else 0, _ffi.stream()))
+
+    def _pass(self, entries: list, want: list[list[int]], tail: bool, tap=None):
+        """entries: (token ids, sequence) in order -- ids a host array, or a device tensor of one token; want: places per entry.
+        Returns (logits [n, V], logprobs, next) of the wanted rows; the sequences advance."""
+        a = self._sequences([s for _, s in entries])
+        for ids, s in entries:
+            s.reserve(len(ids))
+        S, lens = len(entries), np.asarray([len(i) for i, _ in entries], dtype=np.int32)
+        starts = np.concatenate([[0], np.cumsum(lens)]).astype(np.int32)
+        M = int(starts[-1])
+        width = max(len(s.pages) for _, s in entries)
+        host = np.zeros(3 * M + S * width + 4 * S + M, dtype=np.int32)
+        ids, pos, row_seq = host[:M], host[M:2 * M], host[2 * M:3 * M]
+        table, runs = host[3 * M:3 * M + S * width].reshape(S, width), host[3 * M + S * width:3 * M + S * width + 4 * S].reshape(S, 4)
+        on_device = []
+        wanted: list[int] = []
+        for i, (tok, s) in enumerate(entries):
+            lo, hi = starts[i], starts[i + 1]
+            if isinstance(tok, torch.Tensor):
+                on_device.append((lo, tok))
+            else:
+                ids[lo:hi] = tok
+            pos[lo:hi] = np.arange(s.offset, s.offset + lens[i])
+            row_seq[lo:hi] = i
+            table[i, :len(s.pages)] = s.pages
+            runs[i] = (lo, lens[i], i, 0)
+            wanted += [int(lo) + int(k) for k in want[i]]
+        n_want = len(wanted)
+        host[-M:][:n_want] = wanted
+        dev = torch.from_numpy(host).to(self.device)
+        for lo, tok in on_device:
+            dev[lo:lo + 1].copy_(tok.reshape(-1))
+        logits = torch.empty((n_want, self.vocab_size), dtype=torch.float32, device=self.device)
+        logprobs = torch.empty_like(logits) if tail else None
+        nxt = torch.empty(n_want, dtype=torch.int32, device=self.device) if tail else None
+        o = 3 * M
+        self._forward(a, M, dev[:M], dev[M:2 * M], dev[2 * M:o], dev[o:o + S * width].view(S, width), dev[o + S * width:o + S * width + 4 * S], runs,
+                      dev[o + S * width + 4 * S:], n_want, logits, logprobs, nxt, tap=tap)
+        for (_, s), n in zip(entries, lens):
+            s.advance(int(n))
+        return logits, logprobs, nxt
+
+    def _portions(self, entries: list, want: list[list[int]], tail: bool):
+        """_pass in pieces of at most MAX_ROWS rows."""
+        if sum(len(t) for t, _ in entries) <= MAX_ROWS:
+            return self._pass(entries, want, tail)
+        self._sequences([s for _, s in entries])
+        outs, batch, wants, room = [], [], [], MAX_ROWS
+
+        def flush():
+            nonlocal batch, wants, room
+            if batch:
+                outs.append(self._pass(batch, wants, tail))
+            batch, wants, room = [], [], MAX_ROWS
+        for (tok, s), w in zip(entries, want):
+            at = 0
+            while at < len(tok):
+                n = min(room, len(tok) - at)
+                batch.append((tok[at:at + n], s))
+                wants.append([k - at for k in w if at <= k < at + n])
+                at, room = at + n, room - n
+                if room == 0:
+                    flush()
+        flush()
+        return tuple(torch.cat(t) if t[0] is not None else None for t in zip(*outs))
+
+    def step_portions(self, portions: list, want: list[list[int]]) -> torch.Tensor:
+        """portions: (token ids, cache) per sequence -- a whole prompt, the next part of one, or one decoded token; all run as one batch behind what
+        the caches hold.  want: per portion, the places among its tokens whose logits are returned: fp32 [total wanted, vocab]."""
+        for (tok, _), w in zip(portions, want):
+            if len(tok) == 0 or any(not 0 <= int(k) < len(tok) for k in w) or list(w) != sorted(set(w)):
+                raise ValueError("a portion holds at least one token, and its wanted places are increasing places among them")
+        return self._portions([(np.asarray(t, dtype=np.int32), self._sequence(c)) for t, c in portions], want, tail=False)[0]
+
+    # ------------------------------------------------------------------ decode steps
+    def _decode(self, tokens: torch.Tensor | None, seqs: list[PagedSequence], graph: bool, history=None) -> dict:
+        """One token for each of the sequences from persistent buffers (per batch size), replayed as a captured graph.  tokens None: the ids the
+        previous step of this batch left on the device."""
+        a = self._sequences(seqs)
+        B = len(seqs)
+        for s in seqs:
+            s.reserve(1)
+        mb = max(len(s.pages) for s in seqs)
+        buf = self._bufs.pop(B, None)
+        if buf is None or buf["table"].shape[1] < mb:
+            width = max(mb, 2 * buf["table"].shape[1] if buf is not None else 4)
+            i32 = dict(dtype=torch.int32, device=self.device)
+            runs = np.stack([np.arange(B), np.ones(B), np.arange(B), np.zeros(B)], axis=1).astype(np.int32)
+            buf = {"ids": torch.zeros(B, **i32), "pos": torch.zeros(B, **i32), "row_seq": torch.arange(B, **i32), "table": torch.zeros((B, width), **i32),
+                   "runs_host": runs, "runs": torch.from_numpy(runs).to(self.device), "next": torch.empty(B, **i32),
+                   "logits": torch.empty((B, self.vocab_size), dtype=torch.float32, device=self.device),
+                   "logprobs": torch.empty((B, self.vocab_size), dtype=torch.float32, device=self.device), "pages": None, "at": None}
+            if tokens is None:
+                raise RuntimeError("no previous step to continue from")
+        while len(self._bufs) >= 4:
+            self._bufs.pop(next(iter(self._bufs)))
+        self._bufs[B] = buf
+        pages = tuple(tuple(s.pages) for s in seqs)
+        if buf["pages"] != pages:
+            t = np.zeros(tuple(buf["table"].shape), dtype=np.int32)
+            for i, s in enumerate(seqs):
+                t[i, :len(s.pages)] = s.pages
+            buf["table"].copy_(torch.from_numpy(t))
+            buf["pages"] = pages
+        at = [s.offset for s in seqs]
+        if buf["at"] != at:
+            buf["pos"].copy_(torch.tensor(at, dtype=torch.int32))
+        if tokens is not None:
+            buf["ids"].copy_(tokens.reshape(-1))
+        self._forward(a, B, buf["ids"], buf["pos"], buf["row_seq"], buf["table"], buf["runs"], buf["runs_host"], None, B, buf["logits"], buf["logprobs"],
+                      buf["next"], advance=True, history=history, graph=graph)
+        buf["at"] = [n + 1 for n in at]
+        for s in seqs:
+            s.advance(1)
+        return buf
+
+    def step(self, ids: torch.Tensor | None, cache: list[BaseCache], graph: bool = True):
+        """Forwards `ids` [L] and returns (greedy token [1], logprobs [V], logits [V]) of the last position.  None feeds back the previous step's
+        token, which is still on the device.  token stays valid; the other two until the next call."""
+        seq = self._sequence(cache)
+        L = 1 if ids is None else ids.numel()
+        if L == 1:
+            tok = None if ids is None else ids.reshape(-1).to(device=self.device, dtype=torch.int32)
+            if ids is None and self._fed is not seq:
+                raise RuntimeError("step(None) continues the sequence of the previous step")
+            if tok is None and (1 not in self._bufs or self._bufs[1]["at"] != [seq.offset] or self._bufs[1]["table"].shape[1] * TOKEN_CAPACITY_PER_PAGE <= seq.offset):
+                tok = self._last
+            buf = self._decode(tok, [seq], graph, history=self.history)
+            nxt, logprobs, logits = buf["next"], buf["logprobs"], buf["logits"]
+            token = self.history[seq.offset:seq.offset + 1] if seq.offset < self.history.numel() else nxt.clone()
+        else:
+            host = ids.reshape(-1).to(torch.int32).cpu().numpy()
+            logits, logprobs, nxt = self._portions([(host, seq)], [[L - 1]], tail=True)
+            token = nxt
+        self._fed, self._last = seq, token
+        return token, logprobs[0], logits[0]
+
+    _fed = _last = None
+
+    def step_embeds(self, inputs_embeds, cache):
+        raise NotImplementedError("a layer-stack model takes token ids (its experts are chosen by them)")
+
+    def step_batch(self, tokens: torch.Tensor, caches: list[list[BaseCache]], graph: bool = True):
+        """One decode step of several sequences: (next tokens [B], logprobs [B, V], logits [B, V]), buffers valid until the next step of that size."""
+        seqs = [self._sequence(c) for c in caches]
+        tokens = tokens.to(device=self.device, dtype=torch.int32).reshape(-1)
+        if tokens.numel() != len(seqs):
+            raise ValueError("step_batch: one token per sequence")
+        buf = self._decode(tokens, seqs, graph)
+        self._fed = None
+        return buf["next"], buf["logprobs"], buf["logits"]
+
+    def prefill_batch(self, prompts: list, caches: list[list[BaseCache]]):
+        """Several fresh prompts in one pass: (next tokens [S], logprobs, logits) of their last positions."""
+        if any(c[0].offset != 0 for c in caches):
+            raise ValueError("prefill_batch takes fresh caches")
+        return self.step_mixed(None, [], prompts, caches)
+
+    def step_mixed(self, tokens, decode_caches: list[list[BaseCache]], prompts: list, prompt_caches: list[list[BaseCache]]):
+        """Decoding sequences and prompts (fresh, or continuing what their caches hold) in one pass; results as in step_batch, the decoding
+        sequences first, then every prompt's last position."""
+        entries = []
+        if decode_caches:
+            tokens = torch.as_tensor(tokens).to(device=self.device, dtype=torch.int32).reshape(-1)
+            if tokens.numel() != len(decode_caches):
+                raise ValueError("step_mixed: one token per decoding sequence")
+            entries += [(tokens[i:i + 1], self._sequence(c)) for i, c in enumerate(decode_caches)]
+        if any(len(p) == 0 for p in prompts) or len(prompts) != len(prompt_caches):
+            raise ValueError("step_mixed: one non-empty prompt per cache")
+        entries += [(np.asarray(p, dtype=np.int32).reshape(-1), self._sequence(c)) for p, c in zip(prompts, prompt_caches)]
+        if not entries:
+            raise ValueError("step_mixed: an empty batch")
+        self._fed = None
+        logits, logprobs, nxt = self._portions(entries, [[len(t) - 1] for t, _ in entries], tail=True)
+        return nxt, logprobs, logits
+
+    def __call__(self, inputs: torch.Tensor, mask=None, cache: list[BaseCache] | None = None, inputs_embeds=None) -> torch.Tensor:
+        """inputs [1, L] -> logits [1, L, V] (fp32) behind what `cache` holds."""
+        if inputs_embeds is not None:
+            self.step_embeds(inputs_embeds, cache)
+        if inputs.dim() != 2 or inputs.shape[0] != 1:
+            raise ValueError("inputs must be [1, L]")
+        if mask is not None and not (isinstance(mask, str) and mask == "causal"):
+            raise NotImplementedError("a layer-stack model's layers carry their own masks")
+        cache = self.make_cache() if cache is None else cache
+        host = inputs.reshape(-1).to(torch.int32).cpu().numpy()
+        return self._portions([(host, self._sequence(cache))], [list(range(len(host)))], tail=False)[0].unsqueeze(0)
+
+    def layer_outputs(self, ids, cache: list[BaseCache] | None = None) -> torch.Tensor:
+        """The residual stream behind every layer for one portion: fp32 [layers, L, width]."""
+        host = np.asarray(ids, dtype=np.int32).reshape(-1)
+        tap = torch.empty((len(self.layers), len(host), self.width), dtype=torch.float32, device=self.device)
+        self._pass([(host, self._sequence(self.make_cache() if cache is None else cache))], [[]], tail=False, tap=tap)
+        return tap
+
+    def launches(self) -> int:
+        """Kernel launches of the last pass that was not a graph replay."""
+        return int(_ffi.base().pie_stack_launches(self._stack))
+
+
+__all__ = ["LayerStackModel", "pack_linear"]

@@ -16,9 +16,11 @@ from typing import Any
 import torch
 
 from .. import _ffi, hip_ops
+from . import taduzen
 from .llama import Model, ModelArgs
 
 _ARCH_ALIASES = {"llama": "llama", "mistral": "llama"}  # models/utils.py:139-155 (the Llama-shaped subset)
+_ARCHITECTURES = {"Taduzen": taduzen}  # config["architecture"]: designs whose config.json lists the layers one by one
 
 
 @dataclass
@@ -28,8 +30,9 @@ class LargeLanguageModel:
     tokenizer_config: dict
 
 
-def load_model(model_path: str, kv_splits: int = 0) -> tuple[Model, dict]:
-    """Reads config.json + model*.safetensors from a local directory and builds the device model."""
+def load_model(model_path: str, kv_splits: int = 0, dtype: torch.dtype | None = None) -> tuple[Any, dict]:
+    """Reads config.json + model*.safetensors from a local directory and builds the device model.  dtype: compute type of a layer-stack
+    model (bfloat16, or float32 for 32-bit arithmetic throughout); Llama-shaped models run in their checkpoint's."""
     from safetensors import safe_open
 
     path = Path(model_path)
@@ -38,8 +41,10 @@ def load_model(model_path: str, kv_splits: int = 0) -> tuple[Model, dict]:
         raise FileNotFoundError(f"no model*.safetensors under {path}")
     with open(path / "config.json") as f:
         config = json.load(f)
-    if _ARCH_ALIASES.get(config.get("model_type")) != "llama":
-        raise ValueError(f"model_type {config.get('model_type')!r} is not on the MI355X decode path (Llama-shaped only)")
+    design = _ARCHITECTURES.get(config.get("architecture"))
+    if design is None and _ARCH_ALIASES.get(config.get("model_type")) != "llama":
+        raise ValueError(f"neither model_type {config.get('model_type')!r} nor architecture {config.get('architecture')!r} is on the MI355X path "
+                         f"(Llama-shaped models; {', '.join(_ARCHITECTURES)})")
     device = _ffi.require_gpu()
     weights: dict[str, torch.Tensor] = {}
     for wf in files:
@@ -49,7 +54,12 @@ def load_model(model_path: str, kv_splits: int = 0) -> tuple[Model, dict]:
                 if t.dtype in (torch.uint32,):
                     t = t.view(torch.int32)
                 weights[k] = t.to(device)
-    model = Model(ModelArgs(**config), weights, kv_splits=kv_splits)
+    if design is not None:
+        model = design.Model(design.ModelArgs(**config), weights, dtype=dtype or torch.bfloat16)
+    else:
+        if dtype is not None and weights["model.norm.weight"].dtype != dtype:
+            raise ValueError(f"a Llama-shaped model computes in its checkpoint's dtype ({weights['model.norm.weight'].dtype})")
+        model = Model(ModelArgs(**config), weights, kv_splits=kv_splits)
     try:
         with open(path / "tokenizer_config.json") as f:
             tokenizer_config = json.load(f)

@@ -5,7 +5,7 @@ set -e
 cd "$(dirname "$0")/.."
 name=$1; flags=$2; shift 2
 mkdir -p tools/variants/obj tools/variants/$name
-FLAGS="--offload-arch=gfx950 -O3 -std=c++17 -fPIC -ffp-contract=off -fno-fast-math -Wall -Wno-unused-function -D__HIP_PLATFORM_AMD__"
+FLAGS="--offload-arch=gfx950 -O3 -std=c++17 -fPIC -ffp-contract=off -fno-fast-math -Wall -Wno-unused-function -D__HIP_PLATFORM_AMD__ -Xclang -target-feature -Xclang -packed-fp32-ops"
 objs=""
 for o in proxy_inference_engine_amd/lib/obj/*.o; do
   b=$(basename $o .o); hit=0

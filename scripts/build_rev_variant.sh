@@ -6,7 +6,7 @@ cd "$(dirname "$0")/.."
 name=$1; rev=$2
 tmp=$(mktemp -d)
 git archive "$rev" proxy_inference_engine_amd/csrc include | tar -x -C "$tmp"
-FLAGS="--offload-arch=gfx950 -O3 -std=c++17 -fPIC -ffp-contract=off -fno-fast-math -Wall -Wno-unused-function -D__HIP_PLATFORM_AMD__"
+FLAGS="--offload-arch=gfx950 -O3 -std=c++17 -fPIC -ffp-contract=off -fno-fast-math -Wall -Wno-unused-function -D__HIP_PLATFORM_AMD__ -Xclang -target-feature -Xclang -packed-fp32-ops"
 mkdir -p tools/variants/$name "$tmp/obj"
 pids=""
 for src in "$tmp"/proxy_inference_engine_amd/csrc/*.hip "$tmp"/proxy_inference_engine_amd/csrc/*.cpp; do

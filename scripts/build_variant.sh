@@ -7,10 +7,10 @@ set -e
 cd "$(dirname "$0")/.."
 name=$1; src=$2; shift 2
 mkdir -p tools/variants/obj
-FLAGS="--offload-arch=gfx950 -O3 -std=c++17 -fPIC -ffp-contract=off -fno-fast-math -Wall -Wno-unused-function -D__HIP_PLATFORM_AMD__"
+FLAGS="--offload-arch=gfx950 -O3 -std=c++17 -fPIC -ffp-contract=off -fno-fast-math -Wall -Wno-unused-function -D__HIP_PLATFORM_AMD__ -Xclang -target-feature -Xclang -packed-fp32-ops"
 /opt/rocm/bin/hipcc $FLAGS "$@" -c proxy_inference_engine_amd/csrc/$src -o tools/variants/obj/$name.o
 objs=""
-for o in proxy_inference_engine_amd/lib/obj/*.o; do
+for o in proxy_inference_engine_amd/lib/obj/*.o; do  # base and Llama objects in one library
   case "$o" in *"/$src.o") objs="$objs tools/variants/obj/$name.o";; *) objs="$objs $o";; esac
 done
 mkdir -p tools/variants/$name

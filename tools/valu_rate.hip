@@ -26,9 +26,6 @@ __global__ void __launch_bounds__(1024) k_rate(unsigned long long *out, float *s
         } else if (WHICH == 2) {  // v_fma_f32
             REP16(asm volatile("v_fma_f32 %0, %4, %5, %0\n\tv_fma_f32 %1, %5, %4, %1\n\tv_fma_f32 %2, %4, %4, %2\n\tv_fma_f32 %3, %5, %5, %3"
                                : "+v"(a0), "+v"(a1), "+v"(a2), "+v"(a3) : "v"(f0), "v"(f1));)
-        } else if (WHICH == 3) {  // v_pk_fma_f32
-            REP16(asm volatile("v_pk_fma_f32 %0, %2, %3, %0\n\tv_pk_fma_f32 %1, %3, %2, %1\n\tv_pk_fma_f32 %0, %3, %3, %0\n\tv_pk_fma_f32 %1, %2, %2, %1"
-                               : "+v"(p0), "+v"(p1) : "v"(q0), "v"(q1));)
         } else if (WHICH == 4) {  // v_dot2_f32_f16
             REP16(asm volatile("v_dot2_f32_f16 %0, %4, %5, %0\n\tv_dot2_f32_f16 %1, %6, %7, %1\n\tv_dot2_f32_f16 %2, %4, %7, %2\n\tv_dot2_f32_f16 %3, %6, %5, %3"
                                : "+v"(a0), "+v"(a1), "+v"(a2), "+v"(a3) : "v"(w0), "v"(x0), "v"(w1), "v"(x1));)
@@ -100,7 +97,6 @@ int main() {
     run<6>("v_dot2c_f32_f16", d_out, d_sink);
     run<4>("v_dot2_f32_f16", d_out, d_sink);
     run<2>("v_fma_f32", d_out, d_sink);
-    run<3>("v_pk_fma_f32", d_out, d_sink);
     run<5>("v_fma_mix_f32", d_out, d_sink);
     run<7>("v_and/v_lshrrev", d_out, d_sink);
     run<8>("v_dot4_i32_i8", d_out, d_sink);

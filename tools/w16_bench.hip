@@ -13,7 +13,7 @@
 #include <string>
 #include <vector>
 
-#include "../proxy_inference_engine_amd/csrc/w4m_gemm.hip"
+#include "../proxy_inference_engine_amd/csrc/w16_gemm.hip"
 
 __global__ void k_bias_tool(u16 *y, const u16 *bias, int M, int N) {
     const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
