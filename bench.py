@@ -66,6 +66,9 @@ def parse():
                     "IPC-mapped peer memory (default) or RCCL (ncclAllReduce on the launch stream): the comparator for the first run on a real node")
     ap.add_argument("--knob", action="append", default=[], metavar="NAME=VALUE", help="developer: one of the library's test / tuning switches (_ffi.KNOBS) for this run")
     ap.add_argument("--bits", type=int, choices=[2, 4, 6, 8], default=4, help="8 / 6 / 2: MLX int8 / int6 / int2 g=64 weights (W8S / W6S / W2S units; a different workload than the metric's)")
+    ap.add_argument("--design", choices=["taduzen"], help="instead of the metric's workload: prefill and decode throughput of a layer-stack design at sizes that resemble a "
+                    "real model's layers, each beside the dense bf16 Llama of equal size (one JSON line; not the BASELINE.json metric)")
+    ap.add_argument("--design-only", default="", help="--design: run only the cases whose name contains this (e.g. dense4096/new/decode1)")
     ap.add_argument("--dense", action="store_true", help="BASELINE.json configs[2]: unquantised bf16 weights (a different workload than the metric's)")
     return ap.parse_args()
 
@@ -147,6 +150,130 @@ def cpu_baseline(cfg, weights_host, n_tokens, model=None, prompt=None, what="Lla
     return base, parity
 
 
+DESIGN_LAYERS = 4
+# sizes of real models' layers: 8B-class dense layers, and a fine-grained mixture (64 experts, 6 per token, one shared); `like`: the Llama of equal width,
+# heads and active feed-forward width (the mixture's: 6 * 1408 + 2816)
+DESIGN_SIZES = {
+    "dense4096": {"width": 4096, "mixer": {"heads": 32, "dim": 128, "vdim": 128, "kv_rank": 512, "window": 4096}, "mlp": {"ff": 14336},
+                  "like": {"hidden_size": 4096, "intermediate_size": 14336, "num_attention_heads": 32, "num_key_value_heads": 8}},
+    "moe2048": {"width": 2048, "mixer": {"heads": 16, "dim": 128, "vdim": 128, "kv_rank": 512, "window": 4096},
+                "mlp": {"experts": 64, "top": 6, "ff": 1408, "shared": 2816},
+                "like": {"hidden_size": 2048, "intermediate_size": 11264, "num_attention_heads": 16, "num_key_value_heads": 4}},
+}
+DESIGN_VOCAB = 32768
+
+
+def taduzen_checkpoint(size, n_layers, vocab):
+    """(config, device weights) of a random Taduzen model of one of DESIGN_SIZES."""
+    W, mx, ff = size["width"], size["mixer"], size["mlp"]
+    H, D, V, R = mx["heads"], mx["dim"], mx["vdim"], mx["kv_rank"]
+    mixer = {"heads": H, "dim": D, "vdim": V, "kv_rank": R, "scale": D ** -0.5, "mask": {"size": mx["window"]}}
+    mlp = {"kind": "dense", "ff": ff["ff"]} if "experts" not in ff else \
+        {"kind": "moe", "expert": {"ff": ff["ff"]}, "router": {"experts": ff["experts"], "top": ff["top"]}, "shared": {"ff": ff["shared"]}}
+    cfg = {"architecture": "Taduzen", "vocab": vocab, "width": W, "logit_scale": 1.0, "norm": {"eps": 1e-6},
+           "layers": [{"type": "latent_attention", "mixer": mixer, "mlp": mlp}] * n_layers}
+    gen = torch.Generator(device="cuda").manual_seed(0)
+    w = {}
+
+    def put(name, *shape):
+        w[name] = (torch.randn(shape, generator=gen, device="cuda") * shape[-1] ** -0.5).to(torch.bfloat16)
+
+    def norm(name):
+        w[name] = torch.ones(W, dtype=torch.bfloat16, device="cuda")
+        w[name + ".b"] = torch.zeros(W, dtype=torch.bfloat16, device="cuda")
+        w[name + ".alpha"] = torch.tensor(0.5, dtype=torch.bfloat16, device="cuda")
+    put("embed", vocab, W)
+    for i in range(n_layers):
+        p = f"l{i}."
+        for n in ("norm1", "norm1b", "norm2", "norm2b"):
+            norm(p + n)
+        put(p + "mix.q", H * D, W), put(p + "mix.dkv", R, W), put(p + "mix.uk", H * D, R), put(p + "mix.uv", H * V, R), put(p + "mix.o", W, H * V)
+        w[p + "mix.dkv.norm"] = torch.ones(R, dtype=torch.bfloat16, device="cuda")
+        if "experts" not in ff:
+            put(p + "mlp.up", ff["ff"], W), put(p + "mlp.down", W, ff["ff"])
+            continue
+        for e in [f"e{e}" for e in range(ff["experts"])] + ["shared"]:
+            F = ff["shared"] if e == "shared" else ff["ff"]
+            put(f"{p}mlp.{e}.gate", F, W), put(f"{p}mlp.{e}.up", F, W), put(f"{p}mlp.{e}.down", W, F)
+        put(p + "mlp.shared.sg", 1, W)
+        w[p + "mlp.table"] = torch.rand(vocab, ff["experts"], generator=gen, device="cuda").topk(ff["top"], dim=1).indices.to(torch.int32)
+    norm("final.norm")
+    put("head", vocab, W)
+    return cfg, w
+
+
+def design_bench(args):
+    """--design: throughput of a layer-stack design beside the dense bf16 Llama of equal size, DESIGN_LAYERS layers each."""
+    from proxy_inference_engine_amd.models.llama import Model as Llama, ModelArgs as LlamaArgs
+    from proxy_inference_engine_amd.models.taduzen import Model as Taduzen, ModelArgs as TaduzenArgs
+    from proxy_inference_engine_amd.models.utils import synthetic_checkpoint
+    rows = []
+    rng = np.random.default_rng(0)
+
+    def timed(fn, n, warm):
+        for _ in range(warm):
+            fn()
+        torch.cuda.synchronize()
+        t0 = time.perf_counter()
+        for _ in range(n):
+            fn()
+        torch.cuda.synchronize()
+        return 1e3 * (time.perf_counter() - t0) / n
+
+    for name, size in DESIGN_SIZES.items():
+        for which in ("new", "llama"):
+            if not any(args.design_only in f"{name}/{which}/{c}" for c in ("decode1", "decode8", "decode32", "prefill512", "prefill4096")):
+                continue
+            if which == "new":
+                cfg, w = taduzen_checkpoint(size, DESIGN_LAYERS, DESIGN_VOCAB)
+                model = Taduzen(TaduzenArgs(**cfg), w)
+            else:
+                cfg = dict(size["like"], model_type="llama", num_hidden_layers=DESIGN_LAYERS, vocab_size=DESIGN_VOCAB, rms_norm_eps=1e-6, tie_word_embeddings=False,
+                           quantization=None)
+                w = synthetic_checkpoint(cfg, dtype=torch.bfloat16)
+                model = Llama(LlamaArgs(**cfg), w)
+            del w
+            torch.cuda.empty_cache()
+            model.enable_paged_kv(num_pages=32 * 20, max_blocks=80)
+            for L in (512, 4096):
+                if args.design_only not in f"{name}/{which}/prefill{L}":
+                    continue
+                ids = rng.integers(0, DESIGN_VOCAB, L).astype(np.int32)
+                dev = torch.from_numpy(ids).cuda()
+
+                def prompt():
+                    c = model.make_cache()
+                    model.step(dev, c)
+                    c[0].page_manager.release()
+                ms = timed(prompt, 5, 2)
+                rows.append({"size": name, "model": which, "phase": f"prefill {L}", "ms": ms, "tokens_per_s": 1e3 * L / ms})
+            for B in (1, 8, 32):
+                if args.design_only not in f"{name}/{which}/decode{B}":
+                    continue
+                ctx = 1024
+                caches = [model.make_cache() for _ in range(B)]
+                toks = []
+                for c in caches:
+                    toks.append(model.step(torch.from_numpy(rng.integers(0, DESIGN_VOCAB, ctx).astype(np.int32)).cuda(), c)[0].clone())
+                if B == 1:
+                    fn = lambda: model.step(None, caches[0])  # noqa: E731
+                else:
+                    state = [torch.cat(toks)]
+
+                    def fn():
+                        state[0] = model.step_batch(state[0], caches)[0]
+                ms = timed(fn, args.steps, args.warmup)
+                r = {"size": name, "model": which, "phase": f"decode {B} at {ctx}", "ms": ms, "tokens_per_s": 1e3 * B / ms}
+                rows.append(r)
+                for c in caches:
+                    c[0].page_manager.release()
+            del model
+            torch.cuda.empty_cache()
+            print(f"{name} {which} done", file=sys.stderr, flush=True)
+    print(json.dumps({"metric": f"{args.design}: prefill and decode throughput, {DESIGN_LAYERS} layers (NOT the BASELINE.json metric)", "dtype": "bf16", "data": "synthetic",
+                      "layers": DESIGN_LAYERS, "vocab": DESIGN_VOCAB, "rows": rows}), flush=True)
+
+
 def tp_shard(full_cfg, tp, rank, dist, backend):
     """This rank's shard of a synthetic tensor-parallel checkpoint, generated directly in the local shapes (the full 70B checkpoint never
     exists anywhere); the replicated tensors (embedding table, norm weights) are rank 0's, broadcast once.  Returns (local config, weights, HipComm)."""
@@ -226,6 +353,10 @@ def main():
     if world != args.gpus:
         raise SystemExit(f"--gpus {args.gpus} but WORLD_SIZE={world}: launch with torch.distributed.run --nproc-per-node {args.gpus}")
     n_dev = torch.cuda.device_count()
+    if args.design:
+        if world > 1:
+            raise SystemExit("--design measures one GPU")
+        return design_bench(args)
     torch.cuda.set_device(local_rank % max(n_dev, 1))  # one rank per GPU; PIE_BENCH_BACKEND=gloo lets ranks share a card (rehearsal)
     dist = None
     if world > 1:

@@ -544,6 +544,10 @@ int pie_repack_w4s_to_w4m(const void *w4s, int N, int K, void *w4m, void *stream
 int pie_qgemm_w4m(const void *x, const void *w4m, int M, int N, int K, int dtype, void *y, void *stream);
 
 
+/* The tail over fp32 logits [rows][V] (logprobs nullable); workspace: pie_logprobs_argmax_f32_workspace(rows) bytes of device scratch. */
+size_t pie_logprobs_argmax_f32_workspace(int rows);
+int pie_logprobs_argmax_f32(const float *logits, int rows, int V, float *logprobs, int32_t *tokens, void *workspace, void *stream);
+
 /* ---------------------------------------------------------------- layer-stack models (no reference counterpart: models whose layers are listed one by one
  * in config.json, each with its own mixer, feed-forward and sizes).  pie_stack_* runs a whole pass -- prompts, portions of prompts and single decoded
  * tokens side by side, each row with its own position and sequence -- over a paged cache.  dtype PIE_BF16: bf16 products with fp32 accumulation; the
@@ -572,8 +576,8 @@ enum { PIE_MIXER_LATENT = 1 };
 enum { PIE_FF_NONE = 0, PIE_FF_RELU2 = 1, PIE_FF_TABLE_MOE = 2 };
 
 /* One layer: x += post1(mixer(pre1(x))); x += post2(ff(pre2(x))).
- * Latent mixer, with dim8 / vdim8 = dim / vdim rounded up to 8:  w_in packed [heads * dim8 + rank, width] (rows past dim of a head zero, the latent's
- * down-projection last); w_uk heads x packed [rank, dim] (each head's up-projection of keys, transposed); w_uv heads x packed [vdim, rank];
+ * Latent mixer, with dim8 / vdim8 / rank8 = dim / vdim / rank rounded up to 8:  w_in packed [heads * dim8 + rank8, width] (rows past dim of a head and
+ * past rank zero, the latent's down-projection last); w_uk heads x packed [rank, dim] (each head's up-projection of keys, transposed); w_uv heads x packed [vdim, rank];
  * w_o packed [width, heads * vdim8]; w_kv packed [heads * (dim8 + vdim8), rank] (all keys, then all values: long prompts spell K and V out; may be
  * NULL); c_norm fp32 [rank].  window <= 0: no limit.
  * Experts: w_gate_up experts x packed [2 * size, width] with rows (2 i, 2 i + 1) = (gate_i, up_i); w_down experts x packed [width, size];
@@ -603,13 +607,14 @@ size_t pie_stack_page_bytes(const pie_stack *s, int i);
  * `table`), runs in row order, covering all rows.  Every row's latent is appended to its page, then the row attends to its sequence's cached tokens and
  * itself.  want: the rows whose logits are asked for (NULL: all n_rows in order; n_want = n_rows).  logits fp32 [n_want][vocab]; logprobs (nullable)
  * likewise; next (nullable) the greedy tokens.  advance: afterwards ids[i] = next[i] and pos[i] += 1 (all rows wanted, one per run), and with a
- * history, history[pos of row 0] = next[0] at the new position.  tap (nullable): fp32 [n_layers][n_rows][width], the residual stream after each layer.
+ * history, history[pos of row 0] = next[0] at the new position.  ff_size and shared_size are multiples of 8 (zero rows / columns pad a weight).  tap (nullable): fp32 [n_layers][n_rows][width], the residual stream after each layer.
  * flags: PIE_STEP_GRAPH replays a captured graph once a pass of the same shape and addresses has run before. */
 typedef struct {
     int n_rows, n_seqs, table_width, n_runs, n_want, advance, history_len, reserved;
     int32_t *ids, *pos;
     const int32_t *row_seq, *table, *runs;
-    const int32_t *runs_host;  /* the same [n_runs][4] {row0, n_rows, seq, 0} in host memory */
+    const int32_t *runs_host;  /* the same [n_runs][4] {row0, n_rows, seq, first position} in host memory; a run
+                                * of one row may leave its position 0 (its device-side one counts), so that a step keeps its key */
     const int32_t *want;
     float *logits, *logprobs;
     int32_t *next, *history;

@@ -29,7 +29,7 @@ BASE_EXPORTS = [
     "pie_page_ptrs", "pie_page_i8_bytes", "pie_page_scale_ptrs",
     "pie_w16m_bytes", "pie_repack_w16m", "pie_linear_w16m_workspace", "pie_linear_w16m",
     "pie_stack_weight_bytes", "pie_stack_pack_weight", "pie_stack_create", "pie_stack_destroy", "pie_stack_set_layer", "pie_stack_page_row",
-    "pie_stack_page_bytes", "pie_stack_forward", "pie_stack_launches",
+    "pie_stack_page_bytes", "pie_stack_forward", "pie_stack_launches", "pie_logprobs_argmax_f32", "pie_logprobs_argmax_f32_workspace",
 ]
 EXPORTS = BASE_EXPORTS + [
     "pie_quantize_w4g64", "pie_dequantize_w4g64", "pie_w4s_bytes", "pie_repack_w4g64", "pie_w8s_bytes", "pie_repack_w8g64", "pie_qgemv_w8g64", "pie_quantize_g64", "pie_dequantize_g64", "pie_embedding_g64", "pie_w4s32_bytes", "pie_repack_w4g32", "pie_qgemv_w4g32", "pie_w8s32_bytes", "pie_repack_w8g32", "pie_qgemv_w8g32", "pie_embedding_g32",
@@ -131,7 +131,7 @@ def base() -> C.CDLL:
     lib = _open(_PKG / "lib" / "libpie_base.so", BASE_EXPORTS)
     for name in ("pie_hello", "pie_version", "pie_last_error"):
         getattr(lib, name).restype = C.c_char_p
-    for name in ("pie_page_pool_slab_bytes", "pie_page_pool_size", "pie_page_pool_num_free", "pie_stack_weight_bytes", "pie_stack_page_bytes"):
+    for name in ("pie_page_pool_slab_bytes", "pie_page_pool_size", "pie_page_pool_num_free", "pie_stack_weight_bytes", "pie_stack_page_bytes", "pie_logprobs_argmax_f32_workspace"):
         getattr(lib, name).restype = C.c_size_t
     lib.pie_page_pool_slab_bytes.argtypes = [C.c_size_t, C.c_int, C.c_int, C.c_int]
     lib.pie_page_pool_create.argtypes = [C.c_size_t, C.c_int, C.c_int, C.c_int, C.c_void_p, C.POINTER(C.c_void_p)]

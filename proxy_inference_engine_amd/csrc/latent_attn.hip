@@ -218,14 +218,17 @@ __global__ void __launch_bounds__(256) k_latent_attn_rows(const LatentAttnArgs a
         ((T *)a.out)[pr * a.ldr + r] = E::pack((s_o[0][r] * f[0] + s_o[1][r] * f[1] + s_o[2][r] * f[2] + s_o[3][r] * f[3]) / sum);
 }
 
-template <class E>
-__global__ void __launch_bounds__(256) k_latent_append(const float *c_raw, int ldc, const float *w, float eps, int R, int ldr, const int *pos, const int *row_seq,
+template <class E, class X>
+__global__ void __launch_bounds__(256) k_latent_append(const typename X::type *c_raw, int ldc, const float *w, float eps, int R, int ldr, const int *pos, const int *row_seq,
                                                        const int *table, int table_width, int n_pages, int n_seqs, typename E::type *slab) {
     __shared__ float red[4];
     const int m = blockIdx.x;
-    const float *x = c_raw + (size_t)m * ldc;
+    const typename X::type *x = c_raw + (size_t)m * ldc;
     float ss = 0.0f;
-    for (int r = threadIdx.x; r < R; r += 256) ss = fmaf(x[r], x[r], ss);
+    for (int r = threadIdx.x; r < R; r += 256) {
+        const float v = X::load(x + r);
+        ss = fmaf(v, v, ss);
+    }
     ss = wave_sum(ss);
     if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
     __syncthreads();
@@ -233,7 +236,7 @@ __global__ void __launch_bounds__(256) k_latent_append(const float *c_raw, int l
     const int t = pos[m], j = min(t / PAGE_TOKENS, table_width - 1);
     const size_t page = min((unsigned)table[(size_t)min(row_seq[m], n_seqs - 1) * table_width + j], (unsigned)n_pages - 1u);
     typename E::type *dst = slab + (page * PAGE_TOKENS + (t & (PAGE_TOKENS - 1))) * ldr;
-    for (int r = threadIdx.x; r < R; r += 256) dst[r] = E::pack(x[r] * inv * w[r]);
+    for (int r = threadIdx.x; r < R; r += 256) dst[r] = E::pack(X::load(x + r) * inv * w[r]);
 }
 
 }  // namespace
@@ -272,13 +275,16 @@ int latent_attn_launch(int dtype, const LatentAttnArgs &a, hipStream_t st) {
     return PIE_OK;
 }
 
-int latent_append_launch(int dtype, const float *c_raw, int ldc, const float *w, float eps, int M, int R, int ldr, const int *pos, const int *row_seq,
+int latent_append_launch(int dtype, const void *c_raw, bool raw16, int ldc, const float *w, float eps, int M, int R, int ldr, const int *pos, const int *row_seq,
                          const int *table, int table_width, int n_pages, int n_seqs, void *slab, hipStream_t st) {
     if (M <= 0) return PIE_OK;
-    if (dtype == PIE_F32)
-        hipLaunchKernelGGL(k_latent_append<ElemF32>, dim3((unsigned)M), dim3(256), 0, st, c_raw, ldc, w, eps, R, ldr, pos, row_seq, table, table_width, n_pages, n_seqs, (float *)slab);
-    else
-        hipLaunchKernelGGL(k_latent_append<ElemBF16>, dim3((unsigned)M), dim3(256), 0, st, c_raw, ldc, w, eps, R, ldr, pos, row_seq, table, table_width, n_pages, n_seqs, (u16 *)slab);
+#define APPEND_GO(E_, X_) \
+    hipLaunchKernelGGL((k_latent_append<E_, X_>), dim3((unsigned)M), dim3(256), 0, st, (const X_::type *)c_raw, ldc, w, eps, R, ldr, pos, row_seq, table, table_width, n_pages, \
+                       n_seqs, (E_::type *)slab)
+    if (dtype == PIE_F32) APPEND_GO(ElemF32, ElemF32);
+    else if (raw16) APPEND_GO(ElemBF16, ElemBF16);
+    else APPEND_GO(ElemBF16, ElemF32);
+#undef APPEND_GO
     PIE_LAUNCH_CHECK();
     return PIE_OK;
 }

@@ -10,6 +10,9 @@
 //   output projection     Linear; epilogue: x += post1(y), h = pre2(x)
 //   dense: up (relu^2), down; epilogue: x += post2(y), h = next layer's pre1(x)
 //   experts: gate|up (silu * up) and down over the active experts and the shared one, then the weighted sum with the same epilogue
+// A pass of more rows than the weight-streaming Linear is for (BIG_ROWS; bf16) multiplies through the tiled GEMMs instead (w16_gemm.hpp, grouped by expert
+// for mixtures), with the norms in element-wise passes behind them; runs of LONG_RUN rows and more spell their keys and values out (window_attn.hip)
+// while the shorter runs in front of them keep the latent form.
 // The experts of a token are a table lookup, so all layers' row lists are made by one launch in front of the pass.
 #include <cstring>
 #include <algorithm>
@@ -18,13 +21,27 @@
 
 #include "stack_types.hpp"
 
+size_t w16l_workspace_bytes(int M, int N, int K);
+int w16l_gemm_launch(int dtype, const void *w16m, const void *x, int ldx, int M, int N, int K, void *y, void *workspace, hipStream_t st, const void *bias,
+                     void *swiglu_act, bool *fused, int ldy);
+int w16l_relu2_launch(const void *w16m, const void *x, int ldx, int M, int N, int K, void *y, int ldy, hipStream_t st);
+int w16l_grouped_launch(const void *w16m, size_t w_stride, const void *x, int ldx, size_t x_rows, const int *list, const void *tiles, int tm, int tile_rows, int N, int K,
+                        void *y, int ldy, bool swiglu, hipStream_t st);
+
 namespace {
+
+constexpr int BIG_ROWS = 64;  // more rows than this take the tiled GEMMs
+constexpr int LONG_RUN = 64;  // runs of at least this many rows attend with keys and values spelled out
 
 struct RouteLayer {      // one mixture layer's row lists (device pointers)
     const int *table;
     int top, experts, max_active;
     int *active, *offset, *list, *place;  // [max_active], [experts + 1], [M * top] rows by expert, [M * top] position of (row, slot)
+    int4 *tiles;  // {expert, first position, rows, 0}: row tiles of the grouped GEMM
 };
+// rows per tile of the grouped GEMM, and a bound on the number of tiles
+__host__ __device__ inline int route_tile_rows(long M, int top, int experts) { return M * top >= 96l * experts ? 128 : 64; }
+__host__ __device__ inline int route_max_tiles(long M, int top, int experts) { return (int)(M * top / route_tile_rows(M, top, experts)) + experts; }
 
 __global__ void __launch_bounds__(1024) k_route(const RouteLayer *layers, const int *ids, int M, int vocab) {
     extern __shared__ int s_cnt[];  // [experts] counts, then [experts] cursors
@@ -40,7 +57,8 @@ __global__ void __launch_bounds__(1024) k_route(const RouteLayer *layers, const 
     for (int i = threadIdx.x; i < n; i += blockDim.x) atomicAdd(&s_cnt[expert(i)], 1);
     __syncthreads();
     if (threadIdx.x < 64) {
-        int base = 0, n_active = 0;
+        int base = 0, n_active = 0, n_tiles = 0;
+        const int tr = route_tile_rows(M, L.top, L.experts);
         for (int e0 = 0; e0 < L.experts; e0 += 64) {
             const int e = e0 + (int)threadIdx.x, c = e < L.experts ? s_cnt[e] : 0;
             int incl = c;
@@ -53,8 +71,21 @@ __global__ void __launch_bounds__(1024) k_route(const RouteLayer *layers, const 
             const unsigned long long has = __ballot(c > 0);
             const int slot = n_active + __popcll(has & ((1ull << threadIdx.x) - 1ull));
             if (c > 0 && slot < L.max_active) L.active[slot] = e;
+            if (L.tiles) {
+                const int mine = (c + tr - 1) / tr;
+                int ti = mine;
+#pragma unroll
+                for (int o = 1; o < 64; o <<= 1) {
+                    const int v = __shfl_up(ti, o, 64);
+                    if ((int)threadIdx.x >= o) ti += v;
+                }
+                for (int k = 0; k < mine; ++k) L.tiles[n_tiles + ti - mine + k] = make_int4(e, base + incl - c + k * tr, min(tr, c - k * tr), 0);
+                n_tiles += __shfl(ti, 63, 64);
+            }
             base += __shfl(incl, 63, 64), n_active += __popcll(has);
         }
+        if (L.tiles)
+            for (int i = n_tiles + (int)threadIdx.x; i < route_max_tiles(M, L.top, L.experts); i += 64) L.tiles[i] = make_int4(0, 0, 0, 0);
         if (threadIdx.x == 0) L.offset[L.experts] = base;
         for (int i = n_active + (int)threadIdx.x; i < L.max_active; i += 64) L.active[i] = -1;
     }
@@ -79,8 +110,8 @@ __global__ void __launch_bounds__(256) k_stack_embed(const int *ids, const u16 *
 
 // y = sum over the token's slots of its experts' outputs / top (+ sigmoid(gate . input) * shared output); x += post(y); h = next(x)
 struct CombineArgs {
-    const float *part, *part_s;  // [M * top][ldp] by position, [M][ldp]
-    int ldp;
+    const void *part, *part_s;   // [M * top][ldp] by position, [M][ldp_s]
+    int ldp, ldp_s;
     const int *place;
     int top, W;
     const float *gate;           // [W] or nullptr
@@ -90,7 +121,7 @@ struct CombineArgs {
     void *h;
     int ldh;
 };
-template <class E>
+template <class E, class P>  // P: element type of the experts' outputs
 __global__ void __launch_bounds__(256) k_moe_combine(const CombineArgs a) {
     __shared__ float red[4];
     const size_t m = blockIdx.x;
@@ -107,11 +138,33 @@ __global__ void __launch_bounds__(256) k_moe_combine(const CombineArgs a) {
     const float share = 1.0f / (float)a.top;
     for (int n = threadIdx.x; n < a.W; n += 256) {
         float y = 0.0f;
-        for (int s = 0; s < a.top; ++s) y = fmaf(share, a.part[(size_t)a.place[m * a.top + s] * a.ldp + n], y);
-        if (a.gate) y = fmaf(g, a.part_s[m * a.ldp + n], y);
+        for (int s = 0; s < a.top; ++s) y = fmaf(share, P::load((const typename P::type *)a.part + (size_t)a.place[m * a.top + s] * a.ldp + n), y);
+        if (a.gate) y = fmaf(g, P::load((const typename P::type *)a.part_s + m * a.ldp_s + n), y);
         const float v = x[n] + point_norm(a.post, n, y);
         x[n] = v;
         ((typename E::type *)a.h)[m * a.ldh + n] = E::pack(point_norm(a.next, n, v));
+    }
+}
+
+// x += post(y); h = next(x), four columns per thread (y, h: bf16)
+__global__ void __launch_bounds__(256) k_point_residual(const u16 *y, int ldy, PointNorm post, PointNorm next, float *x, int ldx, u16 *h, int ldh, int W) {
+    const size_t m = blockIdx.y;
+    const int n = (blockIdx.x * 256 + threadIdx.x) * 4;
+    if (n >= W) return;
+    if (n + 4 <= W && !(ldy & 3)) {
+        const uint2 yv = *(const uint2 *)(y + m * ldy + n);
+        float4 *xp = (float4 *)(x + m * ldx + n), v = *xp;
+        v.x += point_norm(post, n, lo_f32<BF16>(yv.x)), v.y += point_norm(post, n + 1, hi_f32<BF16>(yv.x));
+        v.z += point_norm(post, n + 2, lo_f32<BF16>(yv.y)), v.w += point_norm(post, n + 3, hi_f32<BF16>(yv.y));
+        *xp = v;
+        *(uint2 *)(h + m * ldh + n) = make_uint2(pack2<BF16>(point_norm(next, n, v.x), point_norm(next, n + 1, v.y)),
+                                                 pack2<BF16>(point_norm(next, n + 2, v.z), point_norm(next, n + 3, v.w)));
+        return;
+    }
+    for (int i = n; i < min(n + 4, W); ++i) {
+        const float v = x[m * ldx + i] + point_norm(post, i, BF16::to_f32(y[m * ldy + i]));
+        x[m * ldx + i] = v;
+        h[m * ldh + i] = BF16::from_f32(point_norm(next, i, v));
     }
 }
 
@@ -170,15 +223,16 @@ __global__ void __launch_bounds__(256) k_f32_finish(const float *logits, int V, 
 }
 
 template <class T>
-struct Buf {  // a device buffer that only grows; new memory is zero (row paddings stay finite), 64 elements of slack behind it
+struct Buf {  // a device buffer that only grows; new memory is zero (row paddings stay finite), with slack for a read past the last row's end
+    static constexpr size_t SLACK = 1024;  // elements (bytes for char)
     T *p = nullptr;
     size_t cap = 0;
     int need(size_t n, bool *moved) {
         if (n <= cap) return PIE_OK;
         if (p) PIE_HIP_TRY(hipFree(p));
         p = nullptr, cap = 0;
-        PIE_HIP_TRY(hipMalloc((void **)&p, (n + 64) * sizeof(T)));
-        PIE_HIP_TRY(hipMemset(p, 0, (n + 64) * sizeof(T)));
+        PIE_HIP_TRY(hipMalloc((void **)&p, (n + SLACK) * sizeof(T)));
+        PIE_HIP_TRY(hipMemset(p, 0, (n + SLACK) * sizeof(T)));
         cap = n, *moved = true;
         return PIE_OK;
     }
@@ -188,6 +242,7 @@ struct Buf {  // a device buffer that only grows; new memory is zero (row paddin
 };
 
 int up8(int n) { return (n + 7) & ~7; }
+int up64(int n) { return (n + 63) & ~63; }
 
 struct GraphKey {
     pie_stack_batch b;
@@ -208,8 +263,8 @@ struct pie_stack {
     std::vector<pie_stack_layer> layers;
     std::vector<char> have;
     // workspace, by rows of a pass
-    Buf<float> x, c_raw, part, part_s, attn_ws;
-    Buf<char> h, q, ql, oc, o, act, act_e, act_s, hsel;
+    Buf<float> x, c_raw, part, part_s, attn_ws, gemm_ws;
+    Buf<char> h, q, ql, oc, o, act, act_e, act_s, y, ctx, kv;
     Buf<RowStat> stats;
     Buf<int> route_ints;
     Buf<RouteLayer> route_dev;
@@ -231,37 +286,77 @@ namespace {
 size_t esize(const pie_stack *s) { return s->cfg.dtype == PIE_F32 ? 4 : 2; }
 PointNorm norm_of(const pie_point_norm &n) { return {n.w, n.b, n.alpha}; }
 
-int stack_reserve(pie_stack *s, const pie_stack_batch &b, hipStream_t st) {
-    const size_t M = (size_t)b.n_rows, E = esize(s), W8 = up8(s->cfg.width);
-    size_t q = 0, c = 0, ql = 0, o = 0, act = 0, act_e = 0, act_s = 0, part = 0, part_s = 0, ints = 0;
+// How a pass is laid out: rows of the leading short runs, and what the long runs behind them see.
+struct Plan {
+    bool big;
+    int short_rows, short_runs, long_tiles;
+};
+Plan plan_pass(const pie_stack *s, const pie_stack_batch &b) {
+    Plan p = {s->cfg.dtype == PIE_BF16 && b.n_rows > BIG_ROWS, 0, 0, 0};
+    while (p.short_runs < b.n_runs && (!p.big || b.runs_host[4 * p.short_runs + 1] < LONG_RUN)) p.short_rows += b.runs_host[4 * p.short_runs++ + 1];
+    for (int i = p.short_runs; i < b.n_runs; ++i) p.long_tiles += (b.runs_host[4 * i + 1] + 127) / 128;
+    return p;
+}
+bool spelled_out(const pie_stack_layer &L) { return L.w_kv && up8(L.dim) <= WINDOW_ATTN_MAX_DIM && up8(L.vdim) <= WINDOW_ATTN_MAX_DIM; }
+// tokens the long runs of a layer see
+size_t plan_context(const pie_stack_batch &b, const Plan &p, int window) {
+    size_t n = 0;
+    for (int i = p.short_runs; i < b.n_runs; ++i) {
+        const int32_t *r = b.runs_host + 4 * i;
+        const int first = window > 0 ? std::max(0, r[3] - window + 1) : 0;
+        n += r[3] + r[1] - first;
+    }
+    return n;
+}
+
+int stack_reserve(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipStream_t st) {
+    const size_t M = (size_t)b.n_rows, E = esize(s), W64 = up64(s->cfg.width);
+    size_t q = 0, c = 0, ql = 0, o = 0, act = 0, act_e = 0, act_s = 0, part = 0, part_s = 0, ints = 0, ctx = 0, kv = 0, ws = 0;
+    auto gemm = [&](int N, int K) { ws = std::max(ws, w16l_workspace_bytes((int)M, N, K) / 4); };
     for (const pie_stack_layer &L : s->layers) {
-        q = std::max(q, (size_t)L.heads * up8(L.dim)), c = std::max(c, (size_t)up8(L.rank)), ql = std::max(ql, (size_t)L.heads * up8(L.rank));
-        o = std::max(o, (size_t)L.heads * up8(L.vdim));
-        if (L.ff == PIE_FF_RELU2) act = std::max(act, (size_t)up8(L.ff_size));
+        const int NI = L.heads * up8(L.dim) + up8(L.rank), KO = L.heads * up8(L.vdim);
+        q = std::max(q, (size_t)NI), c = std::max(c, (size_t)up8(L.rank)), ql = std::max(ql, (size_t)L.heads * up8(L.rank)), o = std::max(o, (size_t)up64(KO));
+        if (plan.big) gemm(NI, s->cfg.width), gemm(s->cfg.width, KO);
+        if (plan.long_tiles && spelled_out(L)) {
+            const size_t n = plan_context(b, plan, L.window), nkv = L.heads * (up8(L.dim) + up8(L.vdim));
+            ctx = std::max(ctx, n * up64(L.rank)), kv = std::max(kv, n * nkv);
+            ws = std::max(ws, w16l_workspace_bytes((int)n, (int)nkv, L.rank) / 4);
+        }
+        if (L.ff == PIE_FF_RELU2) {
+            act = std::max(act, (size_t)up64(L.ff_size));
+            if (plan.big) gemm(s->cfg.width, L.ff_size);
+        }
         if (L.ff == PIE_FF_TABLE_MOE) {
-            act_e = std::max(act_e, (size_t)L.top * up8(L.ff_size)), part = std::max(part, (size_t)L.top * W8);
-            if (L.shared_size) act_s = std::max(act_s, (size_t)up8(L.shared_size)), part_s = W8;
+            act_e = std::max(act_e, (size_t)L.top * up64(L.ff_size)), part = std::max(part, (size_t)L.top * W64);
+            if (L.shared_size) {
+                act_s = std::max(act_s, (size_t)up64(L.shared_size)), part_s = W64;
+                if (plan.big) gemm(s->cfg.width, L.shared_size);
+            }
         }
     }
     bool moved = false;
     int rc = 0;
-    if (M > (size_t)1 << 20) return pie::fail(PIE_E_SHAPE, "pie_stack_forward: too many rows in one pass");
-    if ((rc = s->x.need(M * W8, &moved)) || (rc = s->c_raw.need(M * c, &moved)) || (rc = s->part.need(M * part, &moved)) || (rc = s->part_s.need(M * part_s, &moved)) ||
-        (rc = s->h.need(M * W8 * E, &moved)) || (rc = s->q.need(M * q * E, &moved)) || (rc = s->ql.need(M * ql * E, &moved)) || (rc = s->oc.need(M * ql * E, &moved)) ||
+    if ((rc = s->x.need(M * W64, &moved)) || (rc = s->c_raw.need(M * c, &moved)) || (rc = s->part.need(M * part, &moved)) || (rc = s->part_s.need(M * part_s, &moved)) ||
+        (rc = s->h.need(M * W64 * E, &moved)) || (rc = s->q.need(M * q * E, &moved)) || (rc = s->ql.need(M * ql * E, &moved)) || (rc = s->oc.need(M * ql * E, &moved)) ||
         (rc = s->o.need(M * o * E, &moved)) || (rc = s->act.need(M * act * E, &moved)) || (rc = s->act_e.need(M * act_e * E, &moved)) ||
-        (rc = s->act_s.need(M * act_s * E, &moved)) || (rc = s->stats.need((size_t)b.n_want * ST_TILES, &moved)))
+        (rc = s->act_s.need(M * act_s * E, &moved)) || (rc = s->stats.need((size_t)b.n_want * ST_TILES, &moved)) || (rc = s->y.need(plan.big ? M * W64 * E : 0, &moved)) ||
+        (rc = s->ctx.need(ctx * E, &moved)) || (rc = s->kv.need(kv * E, &moved)) || (rc = s->gemm_ws.need(ws, &moved)))
         return rc;
     if (s->n_route && (int)M > s->route_rows) {
         s->route_rows = (int)M;
+        // (at most this many tiles for any pass of up to M rows: 64-row tiles and one ragged tile per expert)
+        auto tiles = [&](const RouteLayer &r) { return M * r.top / 64 + r.experts + 1; };
         for (const RouteLayer &r : s->route)
-            if (r.experts) ints += r.experts + (size_t)r.experts + 1 + 2 * M * r.top;
+            if (r.experts) ints += (2 * (size_t)r.experts + 1 + 2 * M * r.top + 3) / 4 * 4 + 4 * tiles(r);
         if ((rc = s->route_ints.need(ints, &moved)) || (rc = s->route_dev.need(s->n_route, &moved))) return rc;
         int *p = s->route_ints.p;
         std::vector<RouteLayer> dev;
         s->route_lds = 0;
         for (RouteLayer &r : s->route) {
             if (!r.experts) continue;
-            r.active = p, p += r.experts, r.offset = p, p += r.experts + 1, r.list = p, p += M * r.top, r.place = p, p += M * r.top;
+            r.tiles = (int4 *)p, p += 4 * tiles(r);
+            r.active = p, r.offset = r.active + r.experts, r.list = r.offset + r.experts + 1, r.place = r.list + M * r.top;
+            p += (2 * (size_t)r.experts + 1 + 2 * M * r.top + 3) / 4 * 4;
             r.max_active = r.experts;
             s->route_lds = std::max(s->route_lds, 2 * r.experts * 4);
             dev.push_back(r);
@@ -296,8 +391,23 @@ int stack_tiles(const int32_t *runs, int n_runs, int H) {
 struct Pass {
     pie_stack *s;
     const pie_stack_batch &b;
+    Plan plan;
     hipStream_t st;
     int rc = PIE_OK, launches = 0;
+    // many rows: y = x . W^T rounded to bf16, or the SwiGLU activation of an interleaved matrix
+    void gemm(const void *w, const void *x, int ldx, int M, int N, int K, void *y, int ldy, bool swiglu = false) {
+        if (!rc)
+            rc = w16l_gemm_launch(PIE_BF16, w, x, ldx, M, N, K, swiglu ? nullptr : y, s->gemm_ws.p, st, nullptr, swiglu ? y : nullptr, nullptr, ldy), ++launches;
+    }
+    // x += post(y); h = next(x)
+    void residual(const pie_point_norm &post, const PointNorm &next) {
+        if (rc) return;
+        const int W = s->cfg.width, W64 = up64(W);
+        hipLaunchKernelGGL(k_point_residual, dim3((unsigned)((W + 1023) / 1024), (unsigned)b.n_rows), dim3(256), 0, st, (const u16 *)s->y.p, W, norm_of(post), next, s->x.p, W64,
+                           (u16 *)s->h.p, W64, W);
+        if (hipGetLastError() != hipSuccess) rc = pie::fail(PIE_E_HIP, "residual launch failed");
+        ++launches;
+    }
     void linear(const RowsArgs &a, int batches = 1) {
         if (!rc) rc = rows_gemm_launch(s->cfg.dtype, a, batches, st), ++launches;
     }
@@ -306,73 +416,116 @@ struct Pass {
 void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const PointNorm &next) {
     pie_stack *s = p.s;
     const pie_stack_batch &b = p.b;
-    const int M = b.n_rows, W = s->cfg.width, W8 = up8(W), D8 = up8(L.dim), V8 = up8(L.vdim), R8 = up8(L.rank), H = L.heads, dt = s->cfg.dtype;
-    RowsArgs a = {};
-    a.m = {(const char *)L.w_in, H * D8 + L.rank, W, s->h.p, W8, s->q.p, H * D8};
-    a.M = M, a.epi = ROWS_SPLIT, a.split = H * D8, a.y2 = s->c_raw.p, a.ldy2 = R8;
-    p.linear(a);
-    if (!p.rc)
-        p.rc = latent_append_launch(dt, s->c_raw.p, R8, L.c_norm, L.eps, M, L.rank, R8, b.pos, b.row_seq, b.table, b.table_width, (int)b.n_pages, b.n_seqs,
-                                    b.slabs[li], p.st),
-        ++p.launches;
-    RowsArgs k = {};
-    k.m = {(const char *)L.w_uk, L.rank, L.dim, s->q.p, H * D8, s->ql.p, H * R8};
-    k.M = M, k.epi = ROWS_STORE, k.w_batch = rows_weight_bytes(dt, L.rank, L.dim), k.x_batch = D8, k.y_batch = R8;
-    p.linear(k, H);
-    LatentAttnArgs t = {};
-    t.q = s->ql.p, t.slab = b.slabs[li], t.table = b.table, t.table_width = b.table_width, t.n_pages = (int)b.n_pages, t.n_seqs = b.n_seqs, t.pos = b.pos;
-    t.runs = (const RowRun *)b.runs, t.n_runs = b.n_runs, t.n_tiles = stack_tiles(b.runs_host, b.n_runs, H), t.single = b.n_runs == M, t.row_seq = b.row_seq;
-    t.H = H, t.R = L.rank, t.ldr = R8, t.M = M, t.window = L.window, t.scale = L.scale, t.splits = plan_splits(b, L, t.n_tiles), t.ws = s->attn_ws.p, t.out = s->oc.p;
-    if (!p.rc) p.rc = latent_attn_launch(dt, t, p.st), p.launches += t.splits > 1 ? 2 : 1;
-    RowsArgs v = {};
-    v.m = {(const char *)L.w_uv, L.vdim, L.rank, s->oc.p, H * R8, s->o.p, H * V8};
-    v.M = M, v.epi = ROWS_STORE, v.w_batch = rows_weight_bytes(dt, L.vdim, L.rank), v.x_batch = R8, v.y_batch = V8;
-    p.linear(v, H);
-    RowsArgs o = {};
-    o.m = {(const char *)L.w_o, W, H * V8, s->o.p, H * V8, nullptr, 0};
-    o.M = M, o.epi = ROWS_RESIDUAL, o.res = s->x.p, o.ld_res = W8, o.post = norm_of(L.post1), o.next = next, o.h = s->h.p, o.ldh = W8;
-    p.linear(o);
+    const int W = s->cfg.width, W64 = up64(W), D8 = up8(L.dim), V8 = up8(L.vdim), R8 = up8(L.rank), H = L.heads, NI = H * D8 + R8, KO = H * V8, LO = up64(KO);
+    const int dt = s->cfg.dtype;
+    if (p.plan.big) {
+        p.gemm(L.w_in, s->h.p, W64, b.n_rows, NI, W, s->q.p, NI);
+    } else {
+        RowsArgs a = {};
+        a.m = {(const char *)L.w_in, NI, W, s->h.p, W64, s->q.p, NI};
+        a.M = b.n_rows, a.epi = ROWS_SPLIT, a.split = H * D8, a.y2 = s->c_raw.p, a.ldy2 = R8;
+        p.linear(a);
+    }
+    if (p.rc) return;
+    p.rc = latent_append_launch(dt, p.plan.big ? (const void *)((const u16 *)s->q.p + H * D8) : s->c_raw.p, p.plan.big, p.plan.big ? NI : R8, L.c_norm, L.eps, b.n_rows, L.rank, R8,
+                                b.pos, b.row_seq, b.table, b.table_width, (int)b.n_pages, b.n_seqs, b.slabs[li], p.st);
+    ++p.launches;
+    const bool spell = p.plan.long_tiles && spelled_out(L);
+    const int M = spell ? p.plan.short_rows : b.n_rows, runs = spell ? p.plan.short_runs : b.n_runs;
+    if (M > 0) {  // the latent form
+        RowsArgs k = {};
+        k.m = {(const char *)L.w_uk, L.rank, L.dim, s->q.p, NI, s->ql.p, H * R8};
+        k.M = M, k.epi = ROWS_STORE, k.w_batch = rows_weight_bytes(dt, L.rank, L.dim), k.x_batch = D8, k.y_batch = R8;
+        p.linear(k, H);
+        LatentAttnArgs t = {};
+        t.q = s->ql.p, t.slab = b.slabs[li], t.table = b.table, t.table_width = b.table_width, t.n_pages = (int)b.n_pages, t.n_seqs = b.n_seqs, t.pos = b.pos;
+        t.runs = (const RowRun *)b.runs, t.n_runs = runs, t.n_tiles = stack_tiles(b.runs_host, runs, H), t.single = runs == M, t.row_seq = b.row_seq;
+        t.H = H, t.R = L.rank, t.ldr = R8, t.M = M, t.window = L.window, t.scale = L.scale, t.splits = plan_splits(b, L, t.n_tiles), t.ws = s->attn_ws.p, t.out = s->oc.p;
+        if (!p.rc) p.rc = latent_attn_launch(dt, t, p.st), p.launches += t.splits > 1 ? 2 : 1;
+        RowsArgs v = {};
+        v.m = {(const char *)L.w_uv, L.vdim, L.rank, s->oc.p, H * R8, s->o.p, LO};
+        v.M = M, v.epi = ROWS_STORE, v.w_batch = rows_weight_bytes(dt, L.vdim, L.rank), v.x_batch = R8, v.y_batch = V8;
+        p.linear(v, H);
+    }
+    if (spell && !p.rc) {
+        const RowRun *lr = (const RowRun *)b.runs + p.plan.short_runs;
+        const int n_long = b.n_runs - p.plan.short_runs, n_ctx = (int)plan_context(b, p.plan, L.window), nkv = H * (D8 + V8), LC = up64(L.rank);
+        p.rc = latent_gather_launch(lr, n_long, n_ctx, L.window, b.table, b.table_width, b.n_seqs, (int)b.n_pages, b.slabs[li], R8, s->ctx.p, LC, p.st);
+        p.gemm(L.w_kv, s->ctx.p, LC, n_ctx, nkv, L.rank, s->kv.p, nkv);
+        WindowAttnArgs w = {(const u16 *)s->q.p, (const u16 *)s->kv.p, (u16 *)s->o.p, NI, nkv, LO, H, D8, V8, L.window, L.scale, lr, n_long};
+        if (!p.rc) p.rc = window_attn_launch(w, p.plan.long_tiles, p.st), p.launches += 2;
+    }
+    if (p.plan.big) {
+        p.gemm(L.w_o, s->o.p, LO, b.n_rows, W, KO, s->y.p, W);
+        p.residual(L.post1, next);
+    } else {
+        RowsArgs o = {};
+        o.m = {(const char *)L.w_o, W, KO, s->o.p, LO, nullptr, 0};
+        o.M = b.n_rows, o.epi = ROWS_RESIDUAL, o.res = s->x.p, o.ld_res = W64, o.post = norm_of(L.post1), o.next = next, o.h = s->h.p, o.ldh = W64;
+        p.linear(o);
+    }
 }
 
 void feed_forward(Pass &p, int li, const pie_stack_layer &L, const PointNorm &next) {
     pie_stack *s = p.s;
-    const int M = p.b.n_rows, W = s->cfg.width, W8 = up8(W), F = L.ff_size, F8 = up8(F), dt = s->cfg.dtype;
+    const int M = p.b.n_rows, W = s->cfg.width, W64 = up64(W), F = L.ff_size, F64 = up64(F), dt = s->cfg.dtype;
     if (L.ff == PIE_FF_RELU2) {
+        if (p.plan.big) {
+            if (!p.rc) p.rc = w16l_relu2_launch(L.w_up, s->h.p, W64, M, F, W, s->act.p, F64, p.st), ++p.launches;
+            p.gemm(L.w_down, s->act.p, F64, M, W, F, s->y.p, W);
+            p.residual(L.post2, next);
+            return;
+        }
         RowsArgs u = {};
-        u.m = {(const char *)L.w_up, F, W, s->h.p, W8, s->act.p, F8};
+        u.m = {(const char *)L.w_up, F, W, s->h.p, W64, s->act.p, F64};
         u.M = M, u.epi = ROWS_RELU2;
         p.linear(u);
         RowsArgs d = {};
-        d.m = {(const char *)L.w_down, W, F, s->act.p, F8, nullptr, 0};
-        d.M = M, d.epi = ROWS_RESIDUAL, d.res = s->x.p, d.ld_res = W8, d.post = norm_of(L.post2), d.next = next, d.h = s->h.p, d.ldh = W8;
+        d.m = {(const char *)L.w_down, W, F, s->act.p, F64, nullptr, 0};
+        d.M = M, d.epi = ROWS_RESIDUAL, d.res = s->x.p, d.ld_res = W64, d.post = norm_of(L.post2), d.next = next, d.h = s->h.p, d.ldh = W64;
         p.linear(d);
         return;
     }
     const RouteLayer &r = s->route[li];
-    const int S = L.shared_size, S8 = up8(S), groups = (int)std::min((long)L.experts, (long)M * L.top) + (S ? 1 : 0);
-    RowsArgs u = {};
-    u.m = {(const char *)L.w_gate_up, 2 * F, W, s->h.p, W8, s->act_e.p, F8};
-    u.M = M, u.epi = ROWS_SILU_MUL, u.w_batch = rows_weight_bytes(dt, 2 * F, W), u.active = r.active, u.offset = r.offset, u.list = r.list, u.gather = true;
-    if (S) u.shared = {(const char *)L.s_gate_up, 2 * S, W, s->h.p, W8, s->act_s.p, S8};
-    p.linear(u, groups);
-    RowsArgs d = {};
-    d.m = {(const char *)L.w_expert_down, W, F, s->act_e.p, F8, s->part.p, W8};
-    d.M = M, d.epi = ROWS_SCALE_F32, d.scale = 1.0f, d.w_batch = rows_weight_bytes(dt, W, F), d.active = r.active, d.offset = r.offset, d.list = r.list;
-    if (S) d.shared = {(const char *)L.s_down, W, S, s->act_s.p, S8, s->part_s.p, W8};
-    p.linear(d, groups);
-    if (p.rc) return;
+    const int S = L.shared_size, S64 = up64(S);
+    const size_t gu_stride = rows_weight_bytes(dt, 2 * F, W), dn_stride = rows_weight_bytes(dt, W, F);
     CombineArgs c = {};
-    c.part = s->part.p, c.part_s = s->part_s.p, c.ldp = W8, c.place = r.place, c.top = L.top, c.W = W, c.gate = S ? L.shared_gate : nullptr;
-    c.pre = norm_of(L.pre2), c.post = norm_of(L.post2), c.next = next, c.x = s->x.p, c.ldx = W8, c.h = s->h.p, c.ldh = W8;
-    if (dt == PIE_F32) hipLaunchKernelGGL(k_moe_combine<ElemF32>, dim3((unsigned)M), dim3(256), 0, p.st, c);
-    else hipLaunchKernelGGL(k_moe_combine<ElemBF16>, dim3((unsigned)M), dim3(256), 0, p.st, c);
+    c.part = s->part.p, c.part_s = s->part_s.p, c.ldp = W64, c.ldp_s = p.plan.big ? W : W64, c.place = r.place, c.top = L.top, c.W = W, c.gate = S ? L.shared_gate : nullptr;
+    c.pre = norm_of(L.pre2), c.post = norm_of(L.post2), c.next = next, c.x = s->x.p, c.ldx = W64, c.h = s->h.p, c.ldh = W64;
+    if (p.plan.big) {
+        const int tr = route_tile_rows(M, L.top, L.experts), tm = route_max_tiles(M, L.top, L.experts);
+        if (!p.rc) p.rc = w16l_grouped_launch(L.w_gate_up, gu_stride, s->h.p, W64, (size_t)M, r.list, r.tiles, tm, tr, 2 * F, W, s->act_e.p, F64, true, p.st);
+        if (!p.rc) p.rc = w16l_grouped_launch(L.w_expert_down, dn_stride, s->act_e.p, F64, (size_t)M * L.top, nullptr, r.tiles, tm, tr, W, F, s->part.p, W64, false, p.st);
+        p.launches += 2;
+        if (S) {
+            p.gemm(L.s_gate_up, s->h.p, W64, M, 2 * S, W, s->act_s.p, S64, true);
+            p.gemm(L.s_down, s->act_s.p, S64, M, W, S, s->part_s.p, W);
+        }
+        if (p.rc) return;
+        hipLaunchKernelGGL((k_moe_combine<ElemBF16, ElemBF16>), dim3((unsigned)M), dim3(256), 0, p.st, c);
+    } else {
+        const int groups = (int)std::min((long)L.experts, (long)M * L.top) + (S ? 1 : 0);
+        RowsArgs u = {};
+        u.m = {(const char *)L.w_gate_up, 2 * F, W, s->h.p, W64, s->act_e.p, F64};
+        u.M = M, u.epi = ROWS_SILU_MUL, u.w_batch = gu_stride, u.active = r.active, u.offset = r.offset, u.list = r.list, u.gather = true;
+        if (S) u.shared = {(const char *)L.s_gate_up, 2 * S, W, s->h.p, W64, s->act_s.p, S64};
+        p.linear(u, groups);
+        RowsArgs d = {};
+        d.m = {(const char *)L.w_expert_down, W, F, s->act_e.p, F64, s->part.p, W64};
+        d.M = M, d.epi = ROWS_SCALE_F32, d.scale = 1.0f, d.w_batch = dn_stride, d.active = r.active, d.offset = r.offset, d.list = r.list;
+        if (S) d.shared = {(const char *)L.s_down, W, S, s->act_s.p, S64, s->part_s.p, W64};
+        p.linear(d, groups);
+        if (p.rc) return;
+        if (dt == PIE_F32) hipLaunchKernelGGL((k_moe_combine<ElemF32, ElemF32>), dim3((unsigned)M), dim3(256), 0, p.st, c);
+        else hipLaunchKernelGGL((k_moe_combine<ElemBF16, ElemF32>), dim3((unsigned)M), dim3(256), 0, p.st, c);
+    }
     if (hipGetLastError() != hipSuccess) p.rc = pie::fail(PIE_E_HIP, "expert combine launch failed");
     ++p.launches;
 }
 
-int stack_enqueue(pie_stack *s, const pie_stack_batch &b, hipStream_t st) {
-    const int M = b.n_rows, W = s->cfg.width, W8 = up8(W), V = s->cfg.vocab, n = s->cfg.n_layers, dt = s->cfg.dtype;
-    Pass p{s, b, st};
+int stack_enqueue(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipStream_t st) {
+    const int M = b.n_rows, W = s->cfg.width, W64 = up64(W), V = s->cfg.vocab, n = s->cfg.n_layers, dt = s->cfg.dtype;
+    Pass p{s, b, plan, st};
     if (s->n_route) {
         hipLaunchKernelGGL(k_route, dim3((unsigned)s->n_route), dim3(1024), (size_t)s->route_lds, st, s->route_dev.p, b.ids, M, V);
         PIE_LAUNCH_CHECK();
@@ -381,9 +534,9 @@ int stack_enqueue(pie_stack *s, const pie_stack_batch &b, hipStream_t st) {
     const PointNorm fin = norm_of(s->cfg.final_norm), first = n ? norm_of(s->layers[0].pre1) : fin;
     const dim3 ge((unsigned)((W + 255) / 256), (unsigned)M);
     if (dt == PIE_F32)
-        hipLaunchKernelGGL(k_stack_embed<ElemF32>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, first, s->x.p, W8, (float *)s->h.p, W8);
+        hipLaunchKernelGGL(k_stack_embed<ElemF32>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, first, s->x.p, W64, (float *)s->h.p, W64);
     else
-        hipLaunchKernelGGL(k_stack_embed<ElemBF16>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, first, s->x.p, W8, (u16 *)s->h.p, W8);
+        hipLaunchKernelGGL(k_stack_embed<ElemBF16>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, first, s->x.p, W64, (u16 *)s->h.p, W64);
     PIE_LAUNCH_CHECK();
     ++p.launches;
     for (int i = 0; i < n && !p.rc; ++i) {
@@ -392,11 +545,11 @@ int stack_enqueue(pie_stack *s, const pie_stack_batch &b, hipStream_t st) {
         latent_mixer(p, i, L, L.ff == PIE_FF_NONE ? after : norm_of(L.pre2));
         if (L.ff != PIE_FF_NONE) feed_forward(p, i, L, after);
         if (b.tap && !p.rc)
-            PIE_HIP_TRY(hipMemcpy2DAsync(b.tap + (size_t)i * M * W, (size_t)W * 4, s->x.p, (size_t)W8 * 4, (size_t)W * 4, (size_t)M, hipMemcpyDeviceToDevice, st));
+            PIE_HIP_TRY(hipMemcpy2DAsync(b.tap + (size_t)i * M * W, (size_t)W * 4, s->x.p, (size_t)W64 * 4, (size_t)W * 4, (size_t)M, hipMemcpyDeviceToDevice, st));
     }
     if (b.n_want > 0) {
         RowsArgs a = {};
-        a.m = {(const char *)s->cfg.head, V, W, s->h.p, W8, b.logits, V};
+        a.m = {(const char *)s->cfg.head, V, W, s->h.p, W64, b.logits, V};
         a.M = b.n_want, a.epi = ROWS_SCALE_F32, a.scale = s->cfg.logit_scale, a.rows = b.want;
         p.linear(a);
         if (!p.rc && b.next) {
@@ -440,7 +593,7 @@ int pie_stack_set_layer(pie_stack *s, int i, const pie_stack_layer *L) {
     PIE_REQUIRE(L->mixer == PIE_MIXER_LATENT, PIE_E_ARG, "pie_stack_set_layer: unknown mixer");
     PIE_REQUIRE(L->heads > 0 && L->dim > 0 && L->vdim > 0 && L->rank > 0 && L->rank <= 2048, PIE_E_SHAPE, "pie_stack_set_layer: bad mixer sizes (kv_rank at most 2048)");
     PIE_REQUIRE(L->w_in && L->w_uk && L->w_uv && L->w_o && L->c_norm && norm_ok(L->pre1) && norm_ok(L->post1), PIE_E_ARG, "pie_stack_set_layer: missing mixer weights");
-    PIE_REQUIRE(L->ff == PIE_FF_NONE || (norm_ok(L->pre2) && norm_ok(L->post2) && L->ff_size > 0), PIE_E_ARG, "pie_stack_set_layer: missing feed-forward norms");
+    PIE_REQUIRE(L->ff == PIE_FF_NONE || (norm_ok(L->pre2) && norm_ok(L->post2) && L->ff_size > 0 && L->ff_size % 8 == 0 && L->shared_size % 8 == 0), PIE_E_ARG, "pie_stack_set_layer: missing feed-forward norms");
     if (L->ff == PIE_FF_RELU2) PIE_REQUIRE(L->w_up && L->w_down, PIE_E_ARG, "pie_stack_set_layer: missing dense weights");
     else if (L->ff == PIE_FF_TABLE_MOE) {
         PIE_REQUIRE(L->experts > 0 && L->experts <= 8192 && L->top > 0 && L->top <= L->experts, PIE_E_SHAPE, "pie_stack_set_layer: bad expert counts");
@@ -453,6 +606,17 @@ int pie_stack_set_layer(pie_stack *s, int i, const pie_stack_layer *L) {
     s->route_rows = 0;
     s->layers[i] = *L, s->have[i] = 1;
     s->drop_graphs();
+    return PIE_OK;
+}
+
+size_t pie_logprobs_argmax_f32_workspace(int rows) { return rows > 0 ? (size_t)rows * ST_TILES * sizeof(RowStat) : 0; }
+int pie_logprobs_argmax_f32(const float *logits, int rows, int V, float *logprobs, int32_t *tokens, void *workspace, void *stream) {
+    PIE_REQUIRE(logits && tokens && workspace, PIE_E_ARG, "pie_logprobs_argmax_f32: null pointer");
+    PIE_REQUIRE(rows > 0 && rows <= 65535 && V > 0, PIE_E_SHAPE, "pie_logprobs_argmax_f32: bad shape");
+    hipStream_t st = (hipStream_t)stream;
+    hipLaunchKernelGGL(k_f32_stats, dim3(ST_TILES, (unsigned)rows), dim3(256), 0, st, logits, V, (RowStat *)workspace);
+    hipLaunchKernelGGL(k_f32_finish, dim3(logprobs ? 32 : 1, (unsigned)rows), dim3(256), 0, st, logits, V, (const RowStat *)workspace, logprobs, tokens, 0, nullptr, nullptr, nullptr, 0);
+    PIE_LAUNCH_CHECK();
     return PIE_OK;
 }
 
@@ -479,15 +643,20 @@ int pie_stack_forward(pie_stack *s, const pie_stack_batch *bp, int flags, void *
     }
     PIE_REQUIRE(at == b.n_rows, PIE_E_ARG, "pie_stack_forward: the runs must cover the rows in order");
     for (int i = 0; i < s->cfg.n_layers; ++i) PIE_REQUIRE(b.slabs[i], PIE_E_ARG, "pie_stack_forward: a layer has no pages");
-    int rc = stack_reserve(s, b, st);
+    const Plan plan = plan_pass(s, b);
+    int rc = stack_reserve(s, b, plan, st);
     if (rc) return rc;
     size_t ws = 0;
     for (const pie_stack_layer &L : s->layers)
-        ws = std::max(ws, latent_attn_ws_floats(b.n_rows, L.heads, L.rank, plan_splits(b, L, stack_tiles(b.runs_host, b.n_runs, L.heads))));
+    {
+        const bool spell = plan.long_tiles && spelled_out(L);
+        const int M = spell ? plan.short_rows : b.n_rows, tiles = stack_tiles(b.runs_host, spell ? plan.short_runs : b.n_runs, L.heads);
+        if (tiles) ws = std::max(ws, latent_attn_ws_floats(M, L.heads, L.rank, plan_splits(b, L, tiles)));
+    }
     bool moved = false;
     if ((rc = s->attn_ws.need(ws, &moved))) return rc;
     if (moved) s->drop_graphs();
-    if (!(flags & PIE_STEP_GRAPH) || b.tap) return stack_enqueue(s, b, st);
+    if (!(flags & PIE_STEP_GRAPH) || b.tap) return stack_enqueue(s, b, plan, st);
 
     GraphKey key;
     key.b = b;
@@ -505,7 +674,7 @@ int pie_stack_forward(pie_stack *s, const pie_stack_batch *bp, int flags, void *
             s->graphs.erase(s->graphs.begin() + old);
         }
         s->graphs.push_back({key, nullptr, ++s->tick});
-        return stack_enqueue(s, b, st);
+        return stack_enqueue(s, b, plan, st);
     }
     slot->used = ++s->tick;
     if (!slot->exec) {
@@ -514,7 +683,7 @@ int pie_stack_forward(pie_stack *s, const pie_stack_batch *bp, int flags, void *
         PIE_HIP_TRY(hipStreamCreateWithFlags(&cs, hipStreamNonBlocking));
         hipError_t e = hipStreamBeginCapture(cs, hipStreamCaptureModeThreadLocal);
         if (e == hipSuccess) {
-            rc = stack_enqueue(s, b, cs);
+            rc = stack_enqueue(s, b, plan, cs);
             e = hipStreamEndCapture(cs, &graph);
         }
         if (e == hipSuccess && !rc) e = hipGraphInstantiate(&slot->exec, graph, nullptr, nullptr, 0);

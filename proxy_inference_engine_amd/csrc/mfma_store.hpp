@@ -29,9 +29,18 @@ __device__ __forceinline__ u32 w4m_pack<F16>(float lo, float hi) {
 // SWIGLU); m0: the tile's first row, rows: its live rows; N: the Linear's out_features (stores clipped to it), ldy: output row stride (elements);
 // bias (nullable): T(T(acc) + bias), like the text tower's Linear; SWIGLU: columns (2 i, 2 i + 1) = (gate_i, up_i) -> T(T(silu(g)) * u), N / 2 wide.
 // The caller has made sure nobody still reads the LDS region (a barrier after the K loop).
-template <class T, int MB, int SW, bool SWIGLU>
+// ACT: MFMA_ACT_NONE, MFMA_ACT_SWIGLU (the bool true of the kernels that know only that one), MFMA_ACT_RELU2 (max(T(v), 0)^2, taken where the tile leaves LDS: next to
+// the accumulators it does not fit the registers).
+enum { MFMA_ACT_NONE = 0, MFMA_ACT_SWIGLU = 1, MFMA_ACT_RELU2 = 2 };
+template <class T>
+__device__ __forceinline__ u32 mfma_relu2(u32 w) {
+    const float a = fmaxf(lo_f32<T>(w), 0.0f), b = fmaxf(hi_f32<T>(w), 0.0f);
+    return w4m_pack<T>(a * a, b * b);
+}
+template <class T, int MB, int SW, int ACT>
 __device__ __forceinline__ void mfma_tile_store(const f32x16_t (&acc)[SW][MB], char *ot, int lane, int nt0, int m0, int rows, int N, int ldy, u16 *y,
                                                 const u16 *bias, bool skip_stores = false) {
+    constexpr bool SWIGLU = ACT == MFMA_ACT_SWIGLU;
     constexpr int MT = 32 * MB;
     constexpr int OB = (SWIGLU ? 32 : 64) * SW;  // output bytes per row of the wave's tile
     constexpr int SL = OB / 8, RPB = 256 / OB;    // 8-byte slots per row; rows per 256-byte bank row
@@ -44,7 +53,7 @@ __device__ __forceinline__ void mfma_tile_store(const f32x16_t (&acc)[SW][MB], c
 #pragma unroll
             for (int q = 0; q < 4; ++q) {
                 const int col = 32 * (nt0 + s) + 4 * kh + 8 * q;
-                u32 p01 = w4m_pack<T>(acc[s][mi][4 * q], acc[s][mi][4 * q + 1]), p23 = w4m_pack<T>(acc[s][mi][4 * q + 2], acc[s][mi][4 * q + 3]);  // the Linear's rounding to T
+                u32 p01 = w4m_pack<T>(acc[s][mi][4 * q], acc[s][mi][4 * q + 1]), p23 = w4m_pack<T>(acc[s][mi][4 * q + 2], acc[s][mi][4 * q + 3]);  // the Linear's rounding
                 if (bias && col < N) {
                     uint2 bw;
                     if (col + 4 <= N && !(N & 3)) bw = *reinterpret_cast<const uint2 *>(bias + col);
@@ -76,8 +85,9 @@ __device__ __forceinline__ void mfma_tile_store(const f32x16_t (&acc)[SW][MB], c
     for (int it = 0; it < MT * PR / 64; ++it) {
         const int pc = it * 64 + lane, r = pc / PR, j = pc % PR;
         const int rsv = ((r & 31) / RPB) & (SL - 1);
-        const uint2 lo = *reinterpret_cast<const uint2 *>(ot + r * OB + (((2 * j) ^ rsv) << 3));
-        const uint2 hi = *reinterpret_cast<const uint2 *>(ot + r * OB + (((2 * j + 1) ^ rsv) << 3));
+        uint2 lo = *reinterpret_cast<const uint2 *>(ot + r * OB + (((2 * j) ^ rsv) << 3));
+        uint2 hi = *reinterpret_cast<const uint2 *>(ot + r * OB + (((2 * j + 1) ^ rsv) << 3));
+        if constexpr (ACT == MFMA_ACT_RELU2) lo = make_uint2(mfma_relu2<T>(lo.x), mfma_relu2<T>(lo.y)), hi = make_uint2(mfma_relu2<T>(hi.x), mfma_relu2<T>(hi.y));
         const int col = c0 + 8 * j;
         if (r >= rows || col >= ldo || skip_stores) continue;
         u16 *dst = y + (size_t)(m0 + r) * ldy + col;

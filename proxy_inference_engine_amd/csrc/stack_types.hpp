@@ -77,7 +77,7 @@ size_t rows_weight_bytes(int dtype, int N, int K);
 // ---------------------------------------------------------------- latent attention
 // A pass holds runs of consecutive rows, one run per sequence; a workgroup takes up to 64 (token, head) pairs of ONE run.
 struct RowRun {
-    int row0, n_rows, seq, pad;  // seq: row of the block table
+    int row0, n_rows, seq, pos0;  // seq: row of the block table; pos0: position of row0 (single rows: not used, may be 0)
 };
 struct LatentAttnArgs {
     const void *q;         // [M][H][ldr]: queries in the latent space (W_uk^T q), ldr = row stride in elements
@@ -98,6 +98,20 @@ struct LatentAttnArgs {
 };
 int latent_attn_launch(int dtype, const LatentAttnArgs &a, hipStream_t st);
 size_t latent_attn_ws_floats(int M, int H, int R, int splits);
-// c_raw fp32 [M][ldc] -> RMS norm with weight w -> the row of its page
-int latent_append_launch(int dtype, const float *c_raw, int ldc, const float *w, float eps, int M, int R, int ldr, const int *pos, const int *row_seq,
+// c_raw [M][ldc], fp32 or (raw16) bf16 -> RMS norm with weight w -> the row of its page
+int latent_append_launch(int dtype, const void *c_raw, bool raw16, int ldc, const float *w, float eps, int M, int R, int ldr, const int *pos, const int *row_seq,
                          const int *table, int table_width, int n_pages, int n_seqs, void *slab, hipStream_t st);
+
+// ---------------------------------------------------------------- attention of long runs, keys and values spelled out (window_attn.hip)
+constexpr int WINDOW_ATTN_MAX_DIM = 256;
+struct WindowAttnArgs {
+    const u16 *q, *kv;      // q [M][ld_q], head h at h * D8; kv [context rows][ld_kv]: keys of head h at h * D8, values at H * D8 + h * V8
+    u16 *out;               // [M][ld_out], head h at h * V8
+    int ld_q, ld_kv, ld_out, H, D8, V8, window;
+    float scale;
+    const RowRun *runs;     // the long runs; run r's context = positions [max(0, pos0 - window + 1), pos0 + n_rows), the runs' contexts concatenated in order
+    int n_runs;
+};
+int window_attn_launch(const WindowAttnArgs &a, int n_tiles, hipStream_t st);  // n_tiles = sum of ceil(n_rows / 128)
+int latent_gather_launch(const RowRun *runs, int n_runs, int n_ctx, int window, const int *table, int table_width, int n_seqs, int n_pages, const void *slab, int ldr,
+                         void *out, int ld_out, hipStream_t st);

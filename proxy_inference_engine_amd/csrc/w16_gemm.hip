@@ -34,7 +34,7 @@ int bias_any_launch(int dtype, void *y, const void *bias, int M, int N, hipStrea
 
 static char *g_w16_zero = nullptr;  // 4 KiB of zeros: the weight tile of the ring's dummy steps
 static std::mutex g_w16_mutex;
-static int w16_zero_block(const char **out) {
+int w16_zero_block(const char **out) {
     std::lock_guard<std::mutex> lock(g_w16_mutex);
     if (!g_w16_zero) {
         PIE_HIP_TRY(hipMalloc((void **)&g_w16_zero, W16M_TILE_BYTES));

@@ -25,7 +25,7 @@ constexpr int W16M_TILE_BYTES = 4096;
 static inline size_t w16m_bytes(int N, int K) { return (size_t)((N + 31) / 32) * ((K + 63) / 64) * W16M_TILE_BYTES; }
 
 // row-major [N][K] -> W16M.  One thread per 16-byte piece of the output.
-__global__ void __launch_bounds__(256) k_rows_to_w16m(const u16 *w, int N, int K, int groups, size_t pieces, uint4 *out) {
+static __global__ void __launch_bounds__(256) k_rows_to_w16m(const u16 *w, int N, int K, int groups, size_t pieces, uint4 *out) {
     const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
     if (i >= pieces) return;
     const int l = (int)(i & 63), s = (int)((i >> 6) & 3);
@@ -47,7 +47,7 @@ __global__ void __launch_bounds__(256) k_rows_to_w16m(const u16 *w, int N, int K
 }
 
 // W16S units (w4_gemv.hip: row pair x 512-wide slice, lane (row, 16-element chunk), two 16-byte pieces j) -> W16M, packed row order
-__global__ void __launch_bounds__(256) k_w16s_to_w16m(const uint4 *w16s, int N, int K, int ns, int groups, size_t pieces, uint4 *out) {
+static __global__ void __launch_bounds__(256) k_w16s_to_w16m(const uint4 *w16s, int N, int K, int ns, int groups, size_t pieces, uint4 *out) {
     const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
     if (i >= pieces) return;
     const int l = (int)(i & 63), s = (int)((i >> 6) & 3);
@@ -70,6 +70,10 @@ struct W16Args {
     const u16 *bias;
     const char *zero;  // 4 KiB of zeros (the dummy steps' weight tile)
     int tm, tn;     // row tiles; column tiles (of 128 SW columns)
+    // grouped form (GRP): row tile t multiplies rows [row0, row0 + rows) of expert's matrix; x row = list[row0 + i] (nullptr: row0 + i), y row = row0 + i
+    const int4 *tiles;  // [tm] {expert, row0, rows, 0}; rows = 0: nothing to do
+    const int *list;
+    size_t w_stride;    // bytes between the experts' matrices
     int bm, bc;     // the XCD-local traversal's block: bm row tiles x bc column tiles (bm * bc ~ the 32 workgroups an XCD runs at once)
 #ifdef W16L_PROF
     unsigned long long *prof;  // per workgroup {s_memtime, s_memrealtime} at entry and exit (tools/w16_bench prof)
@@ -82,8 +86,11 @@ struct W16Args {
 // one column tile, then of the column tile 8 further -- they stream the SAME weight tiles at the same time, so each XCD's L2 fetches a
 // weight tile once per pass (16-bit weights are 4x the int4 kernel's bytes: re-read per row tile they would be 3.7 GB of HBM traffic for
 // gate|up at 4096 rows); grid.y = K splits.
-template <class T, int MB, int SW, bool SWIGLU>
+// GRP: many matrices of one shape, each with its own rows (a mixture's experts).  An XCD takes every eighth row tile with all its column tiles, so the
+// x rows and the expert's weight tiles meet in one L2.
+template <class T, int MB, int SW, int ACT, bool GRP = false>
 __global__ void __launch_bounds__(256) k_w16l_gemm(const W16Args a) {
+    constexpr bool SWIGLU = ACT == MFMA_ACT_SWIGLU;
     constexpr int MT = 32 * MB, XJ = MB;  // rows per tile; DMA instructions per wave and tile (MT / 8 row groups over 4 waves)
     constexpr int WL = 4 * SW;            // weight loads per wave and step
     constexpr int XB = 4, CHUNK = MT * 128;  // x buffers (tile v lives in buffer v % 4); bytes each
@@ -97,15 +104,28 @@ __global__ void __launch_bounds__(256) k_w16l_gemm(const W16Args a) {
     // workgroup -> tile: XCD x = blockIdx.x % 8 owns the column tiles c * 8 + x; it walks its [tm][cl] tiles block by block (bc columns,
     // then bm rows inside; row tile fastest), so the ~32 workgroups it runs at once share bm x tiles and bc weight tiles through its L2
     const int xcd = blockIdx.x & 7, sq = blockIdx.x >> 3;
-    const int cl = (a.tn + 7) >> 3;                       // local columns (the grid holds tm * cl workgroups per XCD)
-    const int cb = sq / (a.tm * a.bc), r1 = sq - cb * a.tm * a.bc;
-    const int bce = min(a.bc, cl - cb * a.bc);            // columns of this (maybe last, narrower) column block
-    const int mbi = r1 / (a.bm * bce), r2 = r1 - mbi * a.bm * bce;
-    const int bme = min(a.bm, a.tm - mbi * a.bm);
-    const int mt = mbi * a.bm + r2 % bme, ncol = (cb * a.bc + r2 / bme) * 8 + xcd;
-    if (ncol >= a.tn) return;  // (whole workgroup, before any barrier)
-    const int m0 = mt * MT;
-    const int rows = a.M - m0 < MT ? a.M - m0 : MT;
+    int m0, rows, ncol;
+    const char *weights = a.w16m;
+    if constexpr (GRP) {
+        const int mt = (sq / a.tn) * 8 + xcd;
+        ncol = sq % a.tn;
+        if (mt >= a.tm) return;
+        const int4 tile = a.tiles[mt];
+        m0 = __builtin_amdgcn_readfirstlane(tile.y), rows = __builtin_amdgcn_readfirstlane(tile.z);
+        if (rows <= 0) return;
+        weights += (size_t)__builtin_amdgcn_readfirstlane(tile.x) * a.w_stride;
+    } else {
+        const int cl = (a.tn + 7) >> 3;                       // local columns (the grid holds tm * cl workgroups per XCD)
+        const int cb = sq / (a.tm * a.bc), r1 = sq - cb * a.tm * a.bc;
+        const int bce = min(a.bc, cl - cb * a.bc);            // columns of this (maybe last, narrower) column block
+        const int mbi = r1 / (a.bm * bce), r2 = r1 - mbi * a.bm * bce;
+        const int bme = min(a.bm, a.tm - mbi * a.bm);
+        const int mt = mbi * a.bm + r2 % bme;
+        ncol = (cb * a.bc + r2 / bme) * 8 + xcd;
+        if (ncol >= a.tn) return;  // (whole workgroup, before any barrier)
+        m0 = mt * MT;
+        rows = a.M - m0 < MT ? a.M - m0 : MT;
+    }
     const int n_strips = (a.N + 31) >> 5;
     const int nt0 = (ncol * 4 + wave) * SW;  // this wave's strips: nt0 .. nt0 + SW
 #ifdef W16L_PROF
@@ -116,7 +136,7 @@ __global__ void __launch_bounds__(256) k_w16l_gemm(const W16Args a) {
 #pragma unroll
     for (int s = 0; s < SW; ++s) {
         has[s] = nt0 + s < n_strips;  // wave-uniform; idle waves still stage x and join the barriers
-        strip[s] = a.w16m + ((size_t)(has[s] ? nt0 + s : 0) * all_groups + g_lo) * W16M_TILE_BYTES;
+        strip[s] = weights + ((size_t)(has[s] ? nt0 + s : 0) * all_groups + g_lo) * W16M_TILE_BYTES;
     }
 
     // x staging: wave w moves rows [8 MB w, 8 MB (w + 1)) of the tile with MB DMA instructions of 8 rows each; per-lane byte offsets from
@@ -127,9 +147,10 @@ __global__ void __launch_bounds__(256) k_w16l_gemm(const W16Args a) {
         const int r = 8 * MB * wave + 8 * j + (lane >> 3);
         const int c = (lane & 7) ^ ((r >> 1) & 7);
         const int rr = r < rows ? r : rows - 1;  // ragged tile: rows past the end repeat the last one (never stored)
-        xoffs[j] = (u32)(((size_t)rr * a.ldx + (size_t)c * 8) * 2);
+        const int xr = !GRP ? rr : a.list ? a.list[m0 + rr] : m0 + rr;  // (grouped: offsets from the first row of x; the launcher bounds them)
+        xoffs[j] = (u32)(((size_t)xr * a.ldx + (size_t)c * 8) * 2);
     }
-    const unsigned long long xbase = (unsigned long long)(uintptr_t)(a.x + (size_t)m0 * a.ldx + (size_t)g_lo * 64);
+    const unsigned long long xbase = (unsigned long long)(uintptr_t)(a.x + (GRP ? 0 : (size_t)m0 * a.ldx) + (size_t)g_lo * 64);
     const unsigned lds0 = (unsigned)(size_t)(w4l_lds_void *)s_x;
     // (issued through asm: see k_w4l2_gemm; M0 = the wave's LDS destination)
     auto x_issue1 = [&](int v, int buf, int j) {  // tile v -> buffer buf (= v % 4, spelled statically by the callers)
@@ -275,5 +296,5 @@ __global__ void __launch_bounds__(256) k_w16l_gemm(const W16Args a) {
     }
     static_assert(4 * MT * ((SWIGLU ? 32 : 64) * SW) <= XB * CHUNK, "the output tile fits the x buffers");
     __syncthreads();  // everyone has read its last B fragments
-    mfma_tile_store<T, MB, SW, SWIGLU>(acc, s_x + wave * (MT * (SWIGLU ? 32 : 64) * SW), lane, nt0, m0, rows, a.N, a.ldy, a.y, a.bias, (W16L_ABL & 64) && a.M > 1);
+    mfma_tile_store<T, MB, SW, ACT>(acc, s_x + wave * (MT * (SWIGLU ? 32 : 64) * SW), lane, nt0, m0, rows, a.N, a.ldy, a.y, a.bias, (W16L_ABL & 64) && a.M > 1);
 }

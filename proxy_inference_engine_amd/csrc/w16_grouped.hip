@@ -1,0 +1,52 @@
+// w16_grouped.hip -- forms of k_w16l_gemm (w16_gemm.hpp) that the layer-stack models add: the squared-relu epilogue, and the grouped product of a
+// mixture's experts (every expert its own matrix and its own rows).
+#include "mfma_store.hpp"
+#include "prefill_attn.hpp"
+
+typedef __attribute__((address_space(3))) void w4l_lds_void;
+#include "w16_gemm.hpp"
+
+int w16_zero_block(const char **out);  // w16_gemm.hip
+
+static int w16_fill(W16Args &a, const void *w16m, const void *x, int ldx, int N, int K, void *y, int ldy) {
+    const int Kx = 64 * ((K + 63) / 64);
+    PIE_REQUIRE(N > 0 && K > 0, PIE_E_SHAPE, "16-bit GEMM: empty matrix");
+    PIE_REQUIRE(ldx >= Kx && ldx % 8 == 0 && pie_aligned(w16m, 16) && pie_aligned(x, 16) && pie_aligned(y, 8), PIE_E_ALIGN, "16-bit GEMM: bad operand stride or alignment");
+    if (int rc = w16_zero_block(&a.zero)) return rc;
+    a.w16m = (const char *)w16m, a.x = (const u16 *)x, a.N = N, a.K = Kx, a.ldx = ldx, a.y = (u16 *)y, a.ldy = ldy;
+    a.tn = (N + 255) / 256, a.bm = 4, a.bc = 8;
+    return PIE_OK;
+}
+
+// y = T(max(x . W^T, 0)^2), bf16
+int w16l_relu2_launch(const void *w16m, const void *x, int ldx, int M, int N, int K, void *y, int ldy, hipStream_t st) {
+    W16Args a = {};
+    if (int rc = w16_fill(a, w16m, x, ldx, N, K, y, ldy)) return rc;
+    PIE_REQUIRE((size_t)256 * ldx * 2 < (1ull << 32), PIE_E_SHAPE, "16-bit GEMM: row stride too long");
+    int mb = 8;  // the largest row tile that still gives the chip a round of workgroups
+    while (mb > 2 && (M <= 16 * mb || a.tn * ((M + 32 * mb - 1) / (32 * mb)) < 200)) mb >>= 1;
+    a.M = M, a.tm = (M + 32 * mb - 1) / (32 * mb), a.bm = a.bm < a.tm ? a.bm : a.tm;
+    const dim3 grid((unsigned)(8 * ((a.tn + 7) / 8) * a.tm));
+    if (mb == 2) hipLaunchKernelGGL((k_w16l_gemm<BF16, 2, 2, MFMA_ACT_RELU2>), grid, dim3(256), 0, st, a);
+    else if (mb == 4) hipLaunchKernelGGL((k_w16l_gemm<BF16, 4, 2, MFMA_ACT_RELU2>), grid, dim3(256), 0, st, a);
+    else hipLaunchKernelGGL((k_w16l_gemm<BF16, 8, 2, MFMA_ACT_RELU2>), grid, dim3(256), 0, st, a);
+    PIE_LAUNCH_CHECK();
+    return PIE_OK;
+}
+
+// grouped: tiles [tm] of tile_rows (64 or 128) rows; x_rows: rows of x; swiglu: y = T(silu(gate) up) of the interleaved matrix, N / 2 wide
+int w16l_grouped_launch(const void *w16m, size_t w_stride, const void *x, int ldx, size_t x_rows, const int *list, const void *tiles, int tm, int tile_rows, int N, int K,
+                        void *y, int ldy, bool swiglu, hipStream_t st) {
+    W16Args a = {};
+    if (int rc = w16_fill(a, w16m, x, ldx, N, K, y, ldy)) return rc;
+    PIE_REQUIRE(x_rows * ldx * 2 < (1ull << 32), PIE_E_SHAPE, "grouped GEMM: x too large");
+    PIE_REQUIRE((tile_rows == 64 || tile_rows == 128) && (!swiglu || N % 8 == 0), PIE_E_SHAPE, "grouped GEMM: bad tile or width");
+    a.M = (int)x_rows, a.tm = tm, a.tiles = (const int4 *)tiles, a.list = list, a.w_stride = w_stride;
+    const dim3 grid((unsigned)(8 * ((tm + 7) / 8) * a.tn));
+    if (tile_rows == 64 && swiglu) hipLaunchKernelGGL((k_w16l_gemm<BF16, 2, 2, MFMA_ACT_SWIGLU, true>), grid, dim3(256), 0, st, a);
+    else if (tile_rows == 64) hipLaunchKernelGGL((k_w16l_gemm<BF16, 2, 2, MFMA_ACT_NONE, true>), grid, dim3(256), 0, st, a);
+    else if (swiglu) hipLaunchKernelGGL((k_w16l_gemm<BF16, 4, 2, MFMA_ACT_SWIGLU, true>), grid, dim3(256), 0, st, a);
+    else hipLaunchKernelGGL((k_w16l_gemm<BF16, 4, 2, MFMA_ACT_NONE, true>), grid, dim3(256), 0, st, a);
+    PIE_LAUNCH_CHECK();
+    return PIE_OK;
+}

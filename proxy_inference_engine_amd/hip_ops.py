@@ -509,6 +509,11 @@ def logprobs_argmax(logits: torch.Tensor):
     V = logits.numel()
     lp = torch.empty(V, dtype=torch.float32, device=logits.device)
     tok = torch.empty(1, dtype=torch.int32, device=logits.device)
+    if logits.dtype == torch.float32:
+        lib = _ffi.base()
+        ws = torch.empty(lib.pie_logprobs_argmax_f32_workspace(1), dtype=torch.uint8, device=logits.device)
+        _ffi.check(lib.pie_logprobs_argmax_f32(_ffi.p(logits), 1, V, _ffi.p(lp), _ffi.p(tok), _ffi.p(ws), _ffi.stream()))
+        return tok, lp
     _ffi.check(_ffi.load().pie_logprobs_argmax(_ffi.p(logits), V, _ffi.dtype_code(logits.dtype), _ffi.p(lp), _ffi.p(tok),
                                                _ffi.stream()))
     return tok, lp

@@ -123,14 +123,17 @@ class LayerStackModel:
         _ffi.check(_ffi.base().pie_stack_forward(self._stack, C.byref(b), _ffi.PIE_STEP_GRAPH if graph else 0, _ffi.stream()))
 
     def _pass(self, entries: list, want: list[list[int]], tail: bool, tap=None):
-        """entries: (token ids, sequence) in order -- ids a host array, or a device tensor of one token; want: places per entry.
-        Returns (logits [n, V], logprobs, next) of the wanted rows; the sequences advance."""
+        """entries: (token ids, sequence) -- ids a host array, or a device tensor of one token; want: places per entry.
+        Returns (logits [n, V], logprobs, next) of the wanted rows, in the entries' order; the sequences advance.  The rows are laid out with the short
+        runs first: the native pass serves those in the latent form and the long ones behind them with keys and values spelled out."""
         a = self._sequences([s for _, s in entries])
         for ids, s in entries:
             s.reserve(len(ids))
         S, lens = len(entries), np.asarray([len(i) for i, _ in entries], dtype=np.int32)
-        starts = np.concatenate([[0], np.cumsum(lens)]).astype(np.int32)
-        M = int(starts[-1])
+        order = np.argsort(lens, kind="stable")
+        starts = np.empty(S, dtype=np.int32)
+        starts[order] = np.concatenate([[0], np.cumsum(lens[order])[:-1]])
+        M = int(lens.sum())
         width = max(len(s.pages) for _, s in entries)
         host = np.zeros(3 * M + S * width + 4 * S + M, dtype=np.int32)
         ids, pos, row_seq = host[:M], host[M:2 * M], host[2 * M:3 * M]
@@ -138,7 +141,7 @@ class LayerStackModel:
         on_device = []
         wanted: list[int] = []
         for i, (tok, s) in enumerate(entries):
-            lo, hi = starts[i], starts[i + 1]
+            lo, hi = starts[i], starts[i] + lens[i]
             if isinstance(tok, torch.Tensor):
                 on_device.append((lo, tok))
             else:
@@ -146,8 +149,9 @@ class LayerStackModel:
             pos[lo:hi] = np.arange(s.offset, s.offset + lens[i])
             row_seq[lo:hi] = i
             table[i, :len(s.pages)] = s.pages
-            runs[i] = (lo, lens[i], i, 0)
             wanted += [int(lo) + int(k) for k in want[i]]
+        for j, i in enumerate(order):
+            runs[j] = (starts[i], lens[i], i, entries[i][1].offset)
         n_want = len(wanted)
         host[-M:][:n_want] = wanted
         dev = torch.from_numpy(host).to(self.device)

@@ -63,10 +63,20 @@ class ModelArgs(base.BaseModelArgs):
 
 def _pad_rows(w: torch.Tensor, heads: int, n: int) -> torch.Tensor:
     """[heads * n, K] -> [heads, n rounded up to 8, K], zero rows behind each head."""
-    n8 = (n + 7) // 8 * 8
+    n8 = _up8(n)
     out = torch.zeros(heads, n8, w.shape[1], dtype=w.dtype, device=w.device)
     out[:, :n] = w.view(heads, n, -1)
     return out
+
+
+def _pad(w: torch.Tensor, rows: int, cols: int) -> torch.Tensor:
+    out = torch.zeros(rows, cols, dtype=w.dtype, device=w.device)
+    out[:w.shape[0], :w.shape[1]] = w
+    return out
+
+
+def _up8(n: int) -> int:
+    return (n + 7) // 8 * 8
 
 
 def _interleave(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
@@ -94,6 +104,8 @@ class Model(LayerStackModel):
         def pack(w: torch.Tensor) -> torch.Tensor:
             return pack_linear(w, dtype)
 
+        if not args.layers:
+            raise ValueError("a model has at least one layer")
         layers = []
         for i, lay in enumerate(args.layers):
             p, m, ff = f"l{i}.", lay.mixer, lay.mlp
@@ -106,29 +118,33 @@ class Model(LayerStackModel):
             fields = {
                 "pre1": norm(p + "norm1"), "post1": norm(p + "norm1b"), "mixer": _ffi.PIE_MIXER_LATENT,
                 "heads": H, "dim": D, "vdim": V, "rank": R, "window": m.mask.size if m.mask is not None else 0, "scale": m.scale, "eps": args.norm.eps,
-                "w_in": pack(torch.cat([q.flatten(0, 1), get(p + "mix.dkv", R, W)])),
+                "w_in": pack(torch.cat([q.flatten(0, 1), _pad(get(p + "mix.dkv", R, W), _up8(R), W)])),
                 "w_uk": pack(uk.view(H, D, R).transpose(1, 2)),
                 "w_uv": pack(uv.view(H, V, R)),
                 "w_o": pack(_pad_rows(wo.T, H, V).flatten(0, 1).T),
+                "w_kv": pack(torch.cat([_pad_rows(uk, H, D).flatten(0, 1), _pad_rows(uv, H, V).flatten(0, 1)])),
                 "c_norm": get(p + "mix.dkv.norm", R).float().contiguous(),
             }
             if ff is not None:
                 fields |= {"pre2": norm(p + "norm2"), "post2": norm(p + "norm2b")}
+                # (intermediate widths padded to 8 with zero rows and columns: act(0) = 0 for both activations)
+                def gated(pfx: str, n: int):
+                    n8 = _up8(n)
+                    return (pack(_interleave(_pad(get(pfx + "gate", n, W), n8, W), _pad(get(pfx + "up", n, W), n8, W))), pack(_pad(get(pfx + "down", W, n), W, n8)))
+
                 if ff.kind == "dense":
-                    fields |= {"ff": _ffi.PIE_FF_RELU2, "ff_size": ff.ff, "w_up": pack(get(p + "mlp.up", ff.ff, W)), "w_down": pack(get(p + "mlp.down", W, ff.ff))}
+                    n8 = _up8(ff.ff)
+                    fields |= {"ff": _ffi.PIE_FF_RELU2, "ff_size": n8, "w_up": pack(_pad(get(p + "mlp.up", ff.ff, W), n8, W)),
+                               "w_down": pack(_pad(get(p + "mlp.down", W, ff.ff), W, n8))}
                 elif ff.kind == "moe":
-                    F, E, top = ff.expert.ff, ff.router.experts, ff.router.top
-                    fields |= {
-                        "ff": _ffi.PIE_FF_TABLE_MOE, "ff_size": F, "experts": E, "top": top,
-                        "table": get(p + "mlp.table", args.vocab, top).to(torch.int32).contiguous(),
-                        "w_gate_up": torch.cat([pack(_interleave(get(f"{p}mlp.e{e}.gate", F, W), get(f"{p}mlp.e{e}.up", F, W))) for e in range(E)]),
-                        "w_expert_down": torch.cat([pack(get(f"{p}mlp.e{e}.down", W, F)) for e in range(E)]),
-                    }
+                    E, top = ff.router.experts, ff.router.top
+                    experts = [gated(f"{p}mlp.e{e}.", ff.expert.ff) for e in range(E)]
+                    fields |= {"ff": _ffi.PIE_FF_TABLE_MOE, "ff_size": _up8(ff.expert.ff), "experts": E, "top": top,
+                               "table": get(p + "mlp.table", args.vocab, top).to(torch.int32).contiguous(),
+                               "w_gate_up": torch.cat([e[0] for e in experts]), "w_expert_down": torch.cat([e[1] for e in experts])}
                     if ff.shared is not None:
-                        S = ff.shared.ff
-                        fields |= {"shared_size": S, "s_gate_up": pack(_interleave(get(p + "mlp.shared.gate", S, W), get(p + "mlp.shared.up", S, W))),
-                                   "s_down": pack(get(p + "mlp.shared.down", W, S)),
-                                   "shared_gate": get(p + "mlp.shared.sg", 1, W).float().reshape(-1).contiguous()}
+                        fields["s_gate_up"], fields["s_down"] = gated(p + "mlp.shared.", ff.shared.ff)
+                        fields |= {"shared_size": _up8(ff.shared.ff), "shared_gate": get(p + "mlp.shared.sg", 1, W).float().reshape(-1).contiguous()}
                 else:
                     raise ValueError(f"layer {i}: unknown feed-forward {ff.kind!r}")
             layers.append(fields)

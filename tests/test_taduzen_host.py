@@ -1,0 +1,84 @@
+"""Taduzen without a GPU: configuration, registry, the latent page pool's bookkeeping, and the oracle against itself."""
+import json
+
+import numpy as np
+import pytest
+import torch
+
+import taduzen_util as tu
+from oracle import taduzen_oracle as orc
+from proxy_inference_engine_amd.cache.kv_cache import LatentPageAllocator, PagedLatentCache, PagedSequence
+from proxy_inference_engine_amd.models import utils as mu
+from proxy_inference_engine_amd.models.taduzen import ModelArgs
+
+
+def test_config_is_read_layer_by_layer():
+    cfg = tu.config([(tu.latent(window=7), tu.dense(30)), (tu.latent(heads=3, dim=20, vdim=12, window=None), None), (tu.latent(), tu.moe(shared=None))])
+    a = ModelArgs(**json.loads(json.dumps(cfg)))
+    assert [lay.mixer.heads for lay in a.layers] == [4, 3, 4] and a.layers[0].mixer.mask.size == 7 and a.layers[1].mixer.mask is None
+    assert a.layers[1].mlp is None and a.layers[2].mlp.shared is None and a.layers[2].mlp.router.top == 2 and a.norm.eps == 1e-5
+
+
+def test_registry_refuses_an_unknown_architecture(tmp_path):
+    from safetensors.torch import save_file
+    save_file({"x": torch.zeros(1)}, str(tmp_path / "model.safetensors"))
+    (tmp_path / "config.json").write_text(json.dumps({"architecture": "Nosuch"}))
+    with pytest.raises(ValueError, match="Taduzen"):
+        mu.load_model(str(tmp_path))
+
+
+def test_latent_pages_share_ids_over_layers_of_different_widths():
+    pool = LatentPageAllocator(4, [24, 8], dtype=torch.float32, device="cpu")
+    assert [tuple(s.shape) for s in pool.slabs] == [(4, 64, 24), (4, 64, 8)] and pool.page_bytes == 64 * 32 * 4
+    seq = PagedSequence(pool, 1)
+    cache = [PagedLatentCache(seq, i) for i in range(2)]
+    rows = [torch.randn(1, 1, 70, n) for n in (24, 8)]
+    for c, r in zip(cache, rows):
+        c.state = (r, None)
+    assert seq.offset == 70 and len(seq.pages) == 2 and pool.get_num_free_pages() == 2
+    assert all(torch.equal(c.state[0], r) for c, r in zip(cache, rows))
+    other = seq.fork()                       # the full page shared, the partly filled one copied
+    assert other.pages[0] == seq.pages[0] and other.pages[1] != seq.pages[1]
+    assert torch.equal(PagedLatentCache(other, 1).state[0], rows[1])
+    cache[0].trim(10)
+    assert seq.offset == 60 and len(seq.pages) == 1
+    seq.release(), other.release()
+    assert pool.get_num_free_pages() == 4
+
+
+def test_saved_latents_round_trip(tmp_path):
+    from proxy_inference_engine_amd.cache.kv_cache import BaseCache, SavedLatentCache
+    pool = LatentPageAllocator(2, [16], dtype=torch.bfloat16, device="cpu")
+    c = [PagedLatentCache(PagedSequence(pool, 1), 0)]
+    c[0].state = (torch.randn(1, 1, 9, 16).to(torch.bfloat16), None)
+    BaseCache.save_cache(str(tmp_path / "c.safetensors"), c, {"k": "v"})
+    back, meta = BaseCache.load_cache(str(tmp_path / "c.safetensors"), device="cpu")
+    assert isinstance(back[0], SavedLatentCache) and back[0].offset == 9 and torch.equal(back[0].rows, c[0].state[0]) and meta == {"k": "v"}
+
+
+def test_oracle_window_edges_matter():
+    """The sharpened weights the device tests use: a window one token off changes the logits of the positions it touches, and only those."""
+    cfg = tu.config([(tu.latent(window=9), None)])
+    w, ids = tu.as_numpy(tu.weights(cfg, q_gain=6.0)), tu.tokens(cfg, 30)
+    a = orc.forward(cfg, w, ids)
+    for off in (-1, 1):
+        other = json.loads(json.dumps(cfg))
+        other["layers"][0]["mixer"]["mask"]["size"] += off
+        b = orc.forward(other, w, ids)
+        first = 9 if off > 0 else 8
+        assert np.allclose(a[:first], b[:first]) and tu.err(b[first:], a[first:]) > 0.1
+
+
+def test_oracle_absorbed_form_agrees():
+    """score and value of latent attention written over the latents alone (what the kernels do) equal the spelled-out keys and values."""
+    cfg = tu.config([(tu.latent(heads=2, dim=6, vdim=10, rank=14, window=5), None)])
+    w, m = tu.as_numpy(tu.weights(cfg)), cfg["layers"][0]["mixer"]
+    h = np.random.default_rng(0).normal(size=(11, cfg["width"]))
+    want = orc.latent_attention(h, w, "l0.mix.", 2, 6, 10, m["scale"], 5, 1e-5)
+    c = orc.rms(h @ w["l0.mix.dkv"].T, w["l0.mix.dkv.norm"], 1e-5)
+    q = (h @ w["l0.mix.q"].T).reshape(11, 2, 6)
+    out = []
+    for a in range(2):
+        ql = q[:, a] @ w["l0.mix.uk"].reshape(2, 6, 14)[a]
+        out.append(orc.softmax_rows(ql @ c.T * m["scale"], orc.visible(11, 5)) @ c @ w["l0.mix.uv"].reshape(2, 10, 14)[a].T)
+    assert np.allclose(np.concatenate(out, 1) @ w["l0.mix.o"].T, want)
