@@ -26,38 +26,72 @@ __device__ __forceinline__ int la_page(const LatentAttnArgs &a, int seq, int t) 
 }
 
 template <int RC>
-__device__ __forceinline__ int la_off(int row, int ch) {  // byte offset of 16-byte chunk ch of key row: XOR-swizzled, conflict-free for both kinds of reads
+__device__ __forceinline__ int la_swizzle(int row) {
     const int sw = ((row & 3) << 2) | ((row >> 2) & 3);
-    return row * (RC * 128) + 16 * (ch ^ (RC % 2 ? sw & 7 : sw));
+    return RC % 2 ? sw & 7 : sw;
+}
+template <int RC>
+__device__ __forceinline__ int la_off(int row, int ch) {  // byte offset of 16-byte chunk ch of key row: XOR-swizzled, conflict-free for both kinds of reads
+    return row * (RC * 128) + 16 * (ch ^ la_swizzle<RC>(row));
 }
 
-template <int RC>  // latents of up to 64 RC numbers
+// RC: latents of up to 64 RC numbers.  KH: key groups -- the four waves are 4 / KH tiles of 16 pairs times KH groups that take every KH-th block, so that a
+// decoded token with few heads keeps all waves busy; the groups' sums meet in LDS at the end.
+template <int RC, int KH>
 __global__ void __launch_bounds__(256) k_latent_attn(const LatentAttnArgs a) {
-    __shared__ __attribute__((aligned(16))) char s_c[LA_BK * RC * 128];
+    constexpr int PT = 4 / KH, PAIRS = 16 * PT;
+    constexpr int BLOCK = LA_BK * RC * 128, ROUND = KH * BLOCK;  // bytes: a block of latents; what one round of the groups takes
+    constexpr int NB = 2 * ROUND <= 128 * 1024 ? 2 : 1;          // two buffers (the next round lands while this one is multiplied) where they fit
+    __shared__ __attribute__((aligned(1024))) char s_c[NB * ROUND];
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-    const int c = lane & 15, g = lane >> 4;
+    const int c = lane & 15, g = lane >> 4, pt = wave % PT, kg = wave / PT;
     int run_i = 0, pair0 = blockIdx.x;
     if (a.single) {
-        const int per_run = (a.H + 63) / 64;
+        const int per_run = (a.H + PAIRS - 1) / PAIRS;
         run_i = pair0 / per_run, pair0 %= per_run;
     } else {
         for (;;) {
-            const int n = (a.runs[run_i].n_rows * a.H + 63) / 64;
+            const int n = (a.runs[run_i].n_rows * a.H + PAIRS - 1) / PAIRS;
             if (pair0 < n || run_i + 1 >= a.n_runs) break;
             pair0 -= n, ++run_i;
         }
     }
-    pair0 *= 64;
-    const RowRun tile = a.runs[run_i];
-    const int last = min(64, tile.n_rows * a.H - pair0) - 1;
+    pair0 *= PAIRS;
+    const RowRun tile = a.single ? RowRun{run_i, 1, a.row_seq[run_i], 0} : a.runs[run_i];
+    const int last = min(PAIRS, tile.n_rows * a.H - pair0) - 1;
     if (last < 0) return;  // (a grid larger than the runs need)
     const int row_a = tile.row0 + pair0 / a.H, row_b = tile.row0 + (pair0 + last) / a.H;
     const int t_hi = a.pos[row_b], t_lo = a.window > 0 ? max(0, a.pos[row_a] - a.window + 1) : 0;
-    const int nb = t_hi / LA_BK - t_lo / LA_BK + 1, per = (nb + a.splits - 1) / a.splits;
+    const int nb = t_hi / LA_BK - t_lo / LA_BK + 1, per = ((nb + a.splits - 1) / a.splits + KH - 1) / KH * KH;
     const int b_begin = t_lo / LA_BK + (int)blockIdx.y * per, b_end = min(t_hi / LA_BK + 1, b_begin + per);
 
-    const bool busy = 16 * wave <= last;
-    const int p = pair0 + min(16 * wave + c, last);
+    // Blocks b .. b + KH - 1 into buffer `buf` by LDS-DMA, 1 KiB per wave instruction; the XOR swizzle is on the source side (LDS slot j of a row takes the
+    // chunk that la_off maps there).  Chunks past the latent's end take the row's first one: the queries are zero there, and the sums are not stored.
+    // Blocks behind the end repeat the last one; their group does not look at them.
+    const unsigned lds0 = (unsigned)(size_t)(__attribute__((address_space(3))) void *)s_c;
+    auto fetch = [&](int b, int buf) {
+        unsigned long long src[KH];  // the blocks' first rows: wave-uniform, all looked up before the first DMA (a lookup between two would wait for the first)
+#pragma unroll
+        for (int k = 0; k < KH; ++k) {
+            const int bb = min(b + k, b_end - 1);
+            const unsigned long long v = (unsigned long long)(uintptr_t)((const u16 *)a.slab + ((size_t)la_page(a, tile.seq, bb * LA_BK) * PAGE_TOKENS + (bb & 1) * LA_BK) * a.ldr);
+            src[k] = (unsigned long long)(unsigned)__builtin_amdgcn_readfirstlane((int)(unsigned)v) | ((unsigned long long)(unsigned)__builtin_amdgcn_readfirstlane((int)(unsigned)(v >> 32)) << 32);
+        }
+#pragma unroll
+        for (int j = 0; j < KH * RC; ++j) {  // wave w moves rows of every block: instruction j = (block j / RC, KiB w RC + j % RC of it)
+            const int k = j / RC, q = wave * RC + j % RC, x = q * 64 + lane, r = x / (8 * RC), ch = (x % (8 * RC)) ^ la_swizzle<RC>(r);
+            const unsigned off = (unsigned)((r * a.ldr + (8 * ch < a.ldr ? 8 * ch : 0)) * 2), dst = lds0 + (unsigned)(buf * ROUND + k * BLOCK + q * 1024);
+            unsigned keep;
+            asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %3\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, %2\n\ts_mov_b32 m0, %0"
+                         : "=&s"(keep)
+                         : "v"(off), "s"(src[k]), "s"(dst)
+                         : "memory");
+        }
+    };
+    if (NB == 2 && b_begin < b_end) fetch(b_begin, 0);
+
+    const bool busy = 16 * pt <= last;
+    const int p = pair0 + min(16 * pt + c, last);
     const int row = tile.row0 + p / a.H, head = p % a.H;
     const size_t pr = (size_t)row * a.H + head;
     const int t_q = a.pos[row], t_min = a.window > 0 ? t_q - a.window + 1 : 0;
@@ -66,15 +100,6 @@ __global__ void __launch_bounds__(256) k_latent_attn(const LatentAttnArgs a) {
 #pragma unroll
     for (int s = 0; s < 2 * RC; ++s) qf[s] = 32 * s + 8 * g < a.ldr ? *(const uint4 *)(qp + 32 * s + 8 * g) : make_uint4(0, 0, 0, 0);
 
-    uint4 nx[RC];
-    auto fetch = [&](int b) {
-        const u16 *src = (const u16 *)a.slab + ((size_t)la_page(a, tile.seq, b * LA_BK) * PAGE_TOKENS + (b & 1) * LA_BK) * a.ldr;
-#pragma unroll
-        for (int i = 0; i < RC; ++i) {
-            const int x = threadIdx.x + 256 * i, r = x / (8 * RC), ch = x % (8 * RC);
-            nx[i] = 8 * ch < a.ldr ? *(const uint4 *)(src + (size_t)r * a.ldr + 8 * ch) : make_uint4(0, 0, 0, 0);
-        }
-    };
     la_f32x4 o[4 * RC];
 #pragma unroll
     for (int r = 0; r < 4 * RC; ++r) o[r] = (la_f32x4){0.0f, 0.0f, 0.0f, 0.0f};
@@ -82,27 +107,63 @@ __global__ void __launch_bounds__(256) k_latent_attn(const LatentAttnArgs a) {
     const float sl2 = a.scale * LA_LOG2E;
     const int tq = (lane & 15) >> 2, tp = lane & 3;
 
-    if (b_begin < b_end) fetch(b_begin);
-    for (int b = b_begin; b < b_end; ++b) {
-        __syncthreads();
-#pragma unroll
-        for (int i = 0; i < RC; ++i) {
-            const int x = threadIdx.x + 256 * i;
-            *(uint4 *)(s_c + la_off<RC>(x / (8 * RC), x % (8 * RC))) = nx[i];
+    int buf = 0;
+    bool started = false;
+    for (int b = b_begin; b < b_end; b += KH) {
+        if (NB == 1) {
+            __syncthreads();
+            fetch(b, 0);
         }
-        __syncthreads();
-        if (b + 1 < b_end) fetch(b + 1);
-        if (!busy) continue;
-        la_f32x4 s0 = {0.0f, 0.0f, 0.0f, 0.0f}, s1 = s0;
-#pragma unroll
-        for (int s = 0; s < 2 * RC; ++s) {
-            const la_bf16x8 q = __builtin_bit_cast(la_bf16x8, qf[s]);
-            const uint4 ka = *(const uint4 *)(s_c + la_off<RC>(c, 4 * s + g)), kb = *(const uint4 *)(s_c + la_off<RC>(16 + c, 4 * s + g));
-            s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(la_bf16x8, ka), q, s0, 0, 0, 0);
-            s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(la_bf16x8, kb), q, s1, 0, 0, 0);
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __syncthreads();  // this round's blocks have landed for everyone, and nobody reads the other buffer any more
+        const char *sb = s_c + buf * ROUND + kg * BLOCK;
+        if (NB == 2) {
+            if (b + KH < b_end) fetch(b + KH, buf ^ 1);
+            buf ^= 1;
         }
-        // register i of s0 / s1 <-> key 32 b + 4 g + i (+ 16)
-        const int t0 = b * LA_BK + 4 * g;
+        if (!busy || b + kg >= b_end) continue;
+        // both products read LDS one batch ahead of their MFMAs (pinned: left alone the scheduler waits for every read at its use)
+        constexpr int QB = (2 * RC) % 4 ? 2 : 4;
+        la_f32x4 s0 = {0.0f, 0.0f, 0.0f, 0.0f}, s1 = s0, s2 = s0, s3 = s0;
+        uint4 ka[2][QB], kb[2][QB];
+        auto read_k = [&](int i, int slot) {
+#pragma unroll
+            for (int u = 0; u < QB; ++u) {
+                ka[slot][u] = *(const uint4 *)(sb + la_off<RC>(c, 4 * (i * QB + u) + g));
+                kb[slot][u] = *(const uint4 *)(sb + la_off<RC>(16 + c, 4 * (i * QB + u) + g));
+            }
+        };
+        read_k(0, 0);
+#pragma unroll
+        for (int i = 0; i < 2 * RC / QB; ++i) {
+            if (i + 1 < 2 * RC / QB) read_k(i + 1, (i + 1) & 1);
+            __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+            for (int u = 0; u < QB; u += 2) {
+                const la_bf16x8 qa = __builtin_bit_cast(la_bf16x8, qf[i * QB + u]), qb = __builtin_bit_cast(la_bf16x8, qf[i * QB + u + 1]);
+                s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(la_bf16x8, ka[i & 1][u]), qa, s0, 0, 0, 0);
+                s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(la_bf16x8, kb[i & 1][u]), qa, s1, 0, 0, 0);
+                s2 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(la_bf16x8, ka[i & 1][u + 1]), qb, s2, 0, 0, 0);
+                s3 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(la_bf16x8, kb[i & 1][u + 1]), qb, s3, 0, 0, 0);
+            }
+            __builtin_amdgcn_sched_barrier(0);
+        }
+        s0 += s2, s1 += s3;
+        la_bf16x8 ct[2][4];
+        auto read_c = [&](int i, int slot) {
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                const int ch = 2 * (4 * i + u) + (tp >> 1);
+                const v4s_t a0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) v4s_t *)(sb + la_off<RC>(4 * g + tq, ch) + 8 * (tp & 1)));
+                const v4s_t a1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) v4s_t *)(sb + la_off<RC>(16 + 4 * g + tq, ch) + 8 * (tp & 1)));
+                const uint2 u0 = __builtin_bit_cast(uint2, a0), u1 = __builtin_bit_cast(uint2, a1);
+                ct[slot][u] = __builtin_bit_cast(la_bf16x8, make_uint4(u0.x, u0.y, u1.x, u1.y));
+            }
+        };
+        read_c(0, 0);
+        __builtin_amdgcn_sched_barrier(0);
+        // register i of s0 / s1 <-> key 32 (b + kg) + 4 g + i (+ 16)
+        const int t0 = (b + kg) * LA_BK + 4 * g;
         float sc[8], mloc = LA_NEG;
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
@@ -111,17 +172,19 @@ __global__ void __launch_bounds__(256) k_latent_attn(const LatentAttnArgs a) {
             mloc = fmaxf(mloc, sc[i]);
         }
         mloc = xor32_max(xor16_max(mloc));
-        if (mloc > m_run) {
-            const float alpha = exp2f(m_run - mloc);
+        // The running maximum moves only when a score exceeds it by 2^8 (weights of up to 256 are as exact as weights of up to 1): rescaling is rare.
+        if (!started) m_run = mloc, started = true;
+        else if (__builtin_amdgcn_ballot_w64(mloc > m_run + 8.0f)) {
+            const float mm = fmaxf(m_run, mloc), alpha = __builtin_amdgcn_exp2f(m_run - mm);
             l_run *= alpha;
 #pragma unroll
             for (int r = 0; r < 4 * RC; ++r) o[r] *= alpha;
-            m_run = mloc;
+            m_run = mm;
         }
         u32 hi[4], lo[4];
 #pragma unroll
         for (int i = 0; i < 8; i += 2) {
-            const float pa = sc[i] > LA_NEG ? exp2f(sc[i] - m_run) : 0.0f, pb = sc[i + 1] > LA_NEG ? exp2f(sc[i + 1] - m_run) : 0.0f;
+            const float pa = sc[i] > LA_NEG ? __builtin_amdgcn_exp2f(sc[i] - m_run) : 0.0f, pb = sc[i + 1] > LA_NEG ? __builtin_amdgcn_exp2f(sc[i + 1] - m_run) : 0.0f;
             l_run += pa + pb;
             const float ha = round_T<BF16>(pa), hb = round_T<BF16>(pb);
             hi[i >> 1] = pack2<BF16>(ha, hb);
@@ -130,18 +193,43 @@ __global__ void __launch_bounds__(256) k_latent_attn(const LatentAttnArgs a) {
         const la_bf16x8 ph = __builtin_bit_cast(la_bf16x8, make_uint4(hi[0], hi[1], hi[2], hi[3]));
         const la_bf16x8 pl = __builtin_bit_cast(la_bf16x8, make_uint4(lo[0], lo[1], lo[2], lo[3]));
 #pragma unroll
-        for (int r = 0; r < 4 * RC; ++r) {
-            const int ch = 2 * r + (tp >> 1);
-            const v4s_t a0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) v4s_t *)(s_c + la_off<RC>(4 * g + tq, ch) + 8 * (tp & 1)));
-            const v4s_t a1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) v4s_t *)(s_c + la_off<RC>(16 + 4 * g + tq, ch) + 8 * (tp & 1)));
-            const uint2 u0 = __builtin_bit_cast(uint2, a0), u1 = __builtin_bit_cast(uint2, a1);
-            const la_bf16x8 ct = __builtin_bit_cast(la_bf16x8, make_uint4(u0.x, u0.y, u1.x, u1.y));
-            o[r] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ct, ph, o[r], 0, 0, 0);
-            o[r] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ct, pl, o[r], 0, 0, 0);
+        for (int i = 0; i < RC; ++i) {
+            if (i + 1 < RC) read_c(i + 1, (i + 1) & 1);
+            __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+            for (int u = 0; u < 4; ++u) o[4 * i + u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ct[i & 1][u], ph, o[4 * i + u], 0, 0, 0);
+#pragma unroll
+            for (int u = 0; u < 4; ++u) o[4 * i + u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ct[i & 1][u], pl, o[4 * i + u], 0, 0, 0);
+            __builtin_amdgcn_sched_barrier(0);
         }
     }
-    const float l = xor32_sum(xor16_sum(l_run));
-    if (16 * wave + c > last) return;
+    float l = xor32_sum(xor16_sum(l_run));
+    if constexpr (KH > 1) {  // merge the key groups, halving: group kg + half hands its sums to group kg through LDS (16 pairs x 64 RC floats per pair tile)
+        __shared__ float s_ml[4][16][2];
+#pragma unroll
+        for (int half = KH / 2; half >= 1; half >>= 1) {
+            __syncthreads();
+            float *so = (float *)s_c + ((size_t)(kg % half) * PT + pt) * 16 * 64 * RC;
+            if (kg >= half && kg < 2 * half) {
+#pragma unroll
+                for (int r = 0; r < 4 * RC; ++r) *(la_f32x4 *)(so + (r * 64 + lane) * 4) = o[r];
+                if (g == 0) s_ml[wave - half * PT][c][0] = m_run, s_ml[wave - half * PT][c][1] = l;
+            }
+            __syncthreads();
+            if (kg < half) {
+                const float m2 = s_ml[wave][c][0], l2 = s_ml[wave][c][1], mm = fmaxf(m_run, m2);
+                const float f1 = __builtin_amdgcn_exp2f(m_run - mm), f2 = __builtin_amdgcn_exp2f(m2 - mm);
+#pragma unroll
+                for (int r = 0; r < 4 * RC; ++r) {
+                    const la_f32x4 v = *(const la_f32x4 *)(so + (r * 64 + lane) * 4);
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) o[r][i] = fmaf(f2, v[i], f1 * o[r][i]);
+                }
+                l = l * f1 + l2 * f2, m_run = mm;
+            }
+        }
+    }
+    if (kg > 0 || 16 * pt + c > last) return;
     const size_t MH = (size_t)a.M * a.H;
     if (a.splits == 1) {
         const float inv = 1.0f / l;
@@ -163,26 +251,34 @@ __global__ void __launch_bounds__(256) k_latent_attn(const LatentAttnArgs a) {
     }
 }
 
-// merges the key splits of one (token, head) pair
+// merges the key splits of one (token, head) pair: every wave weighs all splits (at most 64: one per lane), then streams the partial sums, eight in flight
 __global__ void __launch_bounds__(128) k_latent_combine(const LatentAttnArgs a) {
+    __shared__ float s_f[64];
     const size_t pr = blockIdx.x, MH = (size_t)a.M * a.H;
-    const float *ml = a.ws + (size_t)a.splits * MH * a.ldr + pr * 2;
-    float m = LA_NEG;
-    for (int s = 0; s < a.splits; ++s)
-        if (ml[s * MH * 2 + 1] > 0.0f) m = fmaxf(m, ml[s * MH * 2]);
-    float l = 0.0f;
-    for (int s = 0; s < a.splits; ++s) l += ml[s * MH * 2 + 1] > 0.0f ? ml[s * MH * 2 + 1] * exp2f(ml[s * MH * 2] - m) : 0.0f;
-    const float inv = 1.0f / l;
+    const int lane = threadIdx.x & 63;
+    const float2 ml = lane < a.splits ? *(const float2 *)(a.ws + (size_t)a.splits * MH * a.ldr + (lane * MH + pr) * 2) : make_float2(LA_NEG, 0.0f);
+    const float m = wave_max(ml.y > 0.0f ? ml.x : LA_NEG);
+    const float f = ml.y > 0.0f ? __builtin_amdgcn_exp2f(ml.x - m) : 0.0f;  // an empty split wrote no sums and has no weight
+    const float l = wave_sum(ml.y * f);
+    if (threadIdx.x < 64) s_f[lane] = f / l;
+    __syncthreads();
     for (int r = threadIdx.x * 4; r < a.ldr; r += 512) {
         la_f32x4 acc = {0.0f, 0.0f, 0.0f, 0.0f};
-        for (int s = 0; s < a.splits; ++s) {
-            if (!(ml[s * MH * 2 + 1] > 0.0f)) continue;  // an empty split wrote no sums
-            const float f = exp2f(ml[s * MH * 2] - m);
-            const la_f32x4 v = *(const la_f32x4 *)(a.ws + (s * MH + pr) * a.ldr + r);
+        for (int s0 = 0; s0 < a.splits; s0 += 8) {
+            la_f32x4 v[8];
+            float w[8];
 #pragma unroll
-            for (int i = 0; i < 4; ++i) acc[i] = fmaf(f, v[i], acc[i]);
+            for (int u = 0; u < 8; ++u) {
+                const int s = min(s0 + u, a.splits - 1);
+                w[u] = s0 + u < a.splits ? s_f[s] : 0.0f;
+                v[u] = *(const la_f32x4 *)(a.ws + (s * MH + pr) * a.ldr + r);
+            }
+#pragma unroll
+            for (int u = 0; u < 8; ++u)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) acc[i] = w[u] > 0.0f ? fmaf(w[u], v[u][i], acc[i]) : acc[i];
         }
-        *(uint2 *)((u16 *)a.out + pr * a.ldr + r) = make_uint2(pack2<BF16>(acc[0] * inv, acc[1] * inv), pack2<BF16>(acc[2] * inv, acc[3] * inv));
+        *(uint2 *)((u16 *)a.out + pr * a.ldr + r) = make_uint2(pack2<BF16>(acc[0], acc[1]), pack2<BF16>(acc[2], acc[3]));
     }
 }
 
@@ -241,6 +337,11 @@ __global__ void __launch_bounds__(256) k_latent_append(const typename X::type *c
 
 }  // namespace
 
+int latent_attn_pairs(int H, int R, bool single) {
+    if (!single || R > 512) return 64;
+    return H <= 16 ? 16 : H <= 32 ? 32 : 64;
+}
+
 size_t latent_attn_ws_floats(int M, int H, int R, int splits) { return splits > 1 ? (size_t)splits * M * H * (((R + 7) & ~7) + 2) : 0; }
 
 int latent_attn_launch(int dtype, const LatentAttnArgs &a, hipStream_t st) {
@@ -257,15 +358,18 @@ int latent_attn_launch(int dtype, const LatentAttnArgs &a, hipStream_t st) {
     if (a.n_tiles <= 0) return PIE_OK;
     const dim3 grid((unsigned)a.n_tiles, (unsigned)a.splits);
     const int rc = (a.R + 63) / 64;
-#define LA_GO(N) hipLaunchKernelGGL(k_latent_attn<N>, grid, dim3(256), 0, st, a)
-    if (rc <= 1) LA_GO(1);
-    else if (rc <= 2) LA_GO(2);
-    else if (rc <= 3) LA_GO(3);
-    else if (rc <= 4) LA_GO(4);
-    else if (rc <= 6) LA_GO(6);
-    else if (rc <= 8) LA_GO(8);
-    else if (rc <= 10) LA_GO(10);
-    else LA_GO(16);
+#define LA_GO(N) \
+    if (a.pairs == 16) hipLaunchKernelGGL((k_latent_attn<N, 4>), grid, dim3(256), 0, st, a); \
+    else if (a.pairs == 32) hipLaunchKernelGGL((k_latent_attn<N, 2>), grid, dim3(256), 0, st, a); \
+    else hipLaunchKernelGGL((k_latent_attn<N, 1>), grid, dim3(256), 0, st, a)
+    if (rc <= 1) { LA_GO(1); }
+    else if (rc <= 2) { LA_GO(2); }
+    else if (rc <= 3) { LA_GO(3); }
+    else if (rc <= 4) { LA_GO(4); }
+    else if (rc <= 6) { LA_GO(6); }
+    else if (rc <= 8) { LA_GO(8); }
+    else if (rc <= 10) hipLaunchKernelGGL((k_latent_attn<10, 1>), grid, dim3(256), 0, st, a);
+    else hipLaunchKernelGGL((k_latent_attn<16, 1>), grid, dim3(256), 0, st, a);
 #undef LA_GO
     PIE_LAUNCH_CHECK();
     if (a.splits > 1) {

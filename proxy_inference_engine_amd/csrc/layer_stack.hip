@@ -100,12 +100,22 @@ __global__ void __launch_bounds__(1024) k_route(const RouteLayer *layers, const 
 template <class E>
 __global__ void __launch_bounds__(256) k_stack_embed(const int *ids, const u16 *table, int vocab, int W, PointNorm next, float *x, int ldx, typename E::type *h, int ldh) {
     const size_t m = blockIdx.y;
-    const int n = blockIdx.x * 256 + threadIdx.x;
+    const int n = (blockIdx.x * 256 + threadIdx.x) * 4;
     if (n >= W) return;
-    const int t = min(max(ids[m], 0), vocab - 1);
-    const float v = BF16::to_f32(table[(size_t)t * W + n]);
-    x[m * ldx + n] = v;
-    h[m * ldh + n] = E::pack(point_norm(next, n, v));
+    const u16 *src = table + (size_t)min(max(ids[m], 0), vocab - 1) * W + n;
+    if (n + 4 <= W && !(W & 3)) {
+        const uint2 t = *(const uint2 *)src;
+        const float v[4] = {lo_f32<BF16>(t.x), hi_f32<BF16>(t.x), lo_f32<BF16>(t.y), hi_f32<BF16>(t.y)};
+        *(float4 *)(x + m * ldx + n) = make_float4(v[0], v[1], v[2], v[3]);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) h[m * ldh + n + i] = E::pack(point_norm(next, n + i, v[i]));
+        return;
+    }
+    for (int i = 0; i < min(4, W - n); ++i) {
+        const float v = BF16::to_f32(src[i]);
+        x[m * ldx + n + i] = v;
+        h[m * ldh + n + i] = E::pack(point_norm(next, n + i, v));
+    }
 }
 
 // y = sum over the token's slots of its experts' outputs / top (+ sigmoid(gate . input) * shared output); x += post(y); h = next(x)
@@ -116,33 +126,66 @@ struct CombineArgs {
     int top, W;
     const float *gate;           // [W] or nullptr
     PointNorm pre, post, next;   // pre: the sublayer's input norm (the gate's dot product is taken in fp32 on it)
-    float *x;
+    const float *x;
+    float *x_out;                // another buffer: every block of a row reads all of x
     int ldx;
     void *h;
     int ldh;
 };
+// grid (column blocks of 1024, rows): every block of a row takes the gate's dot product itself
+template <class P>
+__device__ __forceinline__ float4 load4(const void *p, size_t i) {
+    if constexpr (sizeof(typename P::type) == 4) return *(const float4 *)((const float *)p + i);
+    else {
+        const uint2 v = *(const uint2 *)((const u16 *)p + i);
+        return make_float4(lo_f32<BF16>(v.x), hi_f32<BF16>(v.x), lo_f32<BF16>(v.y), hi_f32<BF16>(v.y));
+    }
+}
 template <class E, class P>  // P: element type of the experts' outputs
 __global__ void __launch_bounds__(256) k_moe_combine(const CombineArgs a) {
     __shared__ float red[4];
-    const size_t m = blockIdx.x;
-    float *x = a.x + m * a.ldx;
+    const size_t m = blockIdx.y;
+    const float *x = a.x + m * a.ldx;
+    const int n = (blockIdx.x * 256 + threadIdx.x) * 4;
+    const bool in = n < a.W;
+    constexpr int U = 8;  // slots in flight
+    float4 v[U], vs = make_float4(0, 0, 0, 0);
+    auto fetch = [&](int s0) {
+#pragma unroll
+        for (int u = 0; u < U; ++u)
+            if (s0 + u < a.top) v[u] = load4<P>(a.part, (size_t)a.place[m * a.top + s0 + u] * a.ldp + n);
+    };
+    if (in) {  // (rows of part hold 64 ceil(W / 64) columns: a quad that starts inside W is readable)
+        fetch(0);
+        if (a.gate) vs = load4<P>(a.part_s, m * a.ldp_s + n);
+    }
     float g = 0.0f;
     if (a.gate) {
         float d = 0.0f;
-        for (int n = threadIdx.x; n < a.W; n += 256) d = fmaf(point_norm(a.pre, n, x[n]), a.gate[n], d);
+#pragma unroll 4
+        for (int i = threadIdx.x; i < a.W; i += 256) d = fmaf(point_norm(a.pre, i, x[i]), a.gate[i], d);
         d = wave_sum(d);
         if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = d;
         __syncthreads();
         g = 1.0f / (1.0f + expf(-((red[0] + red[1]) + (red[2] + red[3]))));
     }
+    if (!in) return;
     const float share = 1.0f / (float)a.top;
-    for (int n = threadIdx.x; n < a.W; n += 256) {
-        float y = 0.0f;
-        for (int s = 0; s < a.top; ++s) y = fmaf(share, P::load((const typename P::type *)a.part + (size_t)a.place[m * a.top + s] * a.ldp + n), y);
-        if (a.gate) y = fmaf(g, P::load((const typename P::type *)a.part_s + m * a.ldp_s + n), y);
-        const float v = x[n] + point_norm(a.post, n, y);
-        x[n] = v;
-        ((typename E::type *)a.h)[m * a.ldh + n] = E::pack(point_norm(a.next, n, v));
+    float y[4] = {0, 0, 0, 0};
+    for (int s0 = 0; s0 < a.top; s0 += U) {
+        if (s0) fetch(s0);
+#pragma unroll
+        for (int u = 0; u < U; ++u)
+            if (s0 + u < a.top) y[0] = fmaf(share, v[u].x, y[0]), y[1] = fmaf(share, v[u].y, y[1]), y[2] = fmaf(share, v[u].z, y[2]), y[3] = fmaf(share, v[u].w, y[3]);
+    }
+    if (a.gate) y[0] = fmaf(g, vs.x, y[0]), y[1] = fmaf(g, vs.y, y[1]), y[2] = fmaf(g, vs.z, y[2]), y[3] = fmaf(g, vs.w, y[3]);
+    float *xo = a.x_out + m * a.ldx;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        if (n + i >= a.W) break;
+        const float r = x[n + i] + point_norm(a.post, n + i, y[i]);
+        xo[n + i] = r;
+        ((typename E::type *)a.h)[m * a.ldh + n + i] = E::pack(point_norm(a.next, n + i, r));
     }
 }
 
@@ -263,7 +306,7 @@ struct pie_stack {
     std::vector<pie_stack_layer> layers;
     std::vector<char> have;
     // workspace, by rows of a pass
-    Buf<float> x, c_raw, part, part_s, attn_ws, gemm_ws;
+    Buf<float> x, x2, c_raw, part, part_s, attn_ws, gemm_ws;
     Buf<char> h, q, ql, oc, o, act, act_e, act_s, y, ctx, kv;
     Buf<RowStat> stats;
     Buf<int> route_ints;
@@ -310,34 +353,34 @@ size_t plan_context(const pie_stack_batch &b, const Plan &p, int window) {
 }
 
 int stack_reserve(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipStream_t st) {
-    const size_t M = (size_t)b.n_rows, E = esize(s), W64 = up64(s->cfg.width);
+    const size_t M = (size_t)b.n_rows, E = esize(s), W64 = up64(s->cfg.width), WA = act_stride(s->cfg.width);
     size_t q = 0, c = 0, ql = 0, o = 0, act = 0, act_e = 0, act_s = 0, part = 0, part_s = 0, ints = 0, ctx = 0, kv = 0, ws = 0;
     auto gemm = [&](int N, int K) { ws = std::max(ws, w16l_workspace_bytes((int)M, N, K) / 4); };
     for (const pie_stack_layer &L : s->layers) {
         const int NI = L.heads * up8(L.dim) + up8(L.rank), KO = L.heads * up8(L.vdim);
-        q = std::max(q, (size_t)NI), c = std::max(c, (size_t)up8(L.rank)), ql = std::max(ql, (size_t)L.heads * up8(L.rank)), o = std::max(o, (size_t)up64(KO));
-        if (plan.big) gemm(NI, s->cfg.width), gemm(s->cfg.width, KO);
+        q = std::max(q, (size_t)NI), c = std::max(c, (size_t)up8(L.rank)), ql = std::max(ql, (size_t)L.heads * up8(L.rank)), o = std::max(o, (size_t)act_stride(KO));
+        if (plan.big) gemm(NI, s->cfg.width), gemm(L.heads * up8(L.dim), s->cfg.width), gemm(up8(L.rank), s->cfg.width), gemm(s->cfg.width, KO);
         if (plan.long_tiles && spelled_out(L)) {
             const size_t n = plan_context(b, plan, L.window), nkv = L.heads * (up8(L.dim) + up8(L.vdim));
-            ctx = std::max(ctx, n * up64(L.rank)), kv = std::max(kv, n * nkv);
+            ctx = std::max(ctx, n * act_stride(L.rank)), kv = std::max(kv, n * nkv);
             ws = std::max(ws, w16l_workspace_bytes((int)n, (int)nkv, L.rank) / 4);
         }
         if (L.ff == PIE_FF_RELU2) {
-            act = std::max(act, (size_t)up64(L.ff_size));
+            act = std::max(act, (size_t)act_stride(L.ff_size));
             if (plan.big) gemm(s->cfg.width, L.ff_size);
         }
         if (L.ff == PIE_FF_TABLE_MOE) {
-            act_e = std::max(act_e, (size_t)L.top * up64(L.ff_size)), part = std::max(part, (size_t)L.top * W64);
+            act_e = std::max(act_e, (size_t)L.top * act_stride(L.ff_size)), part = std::max(part, (size_t)L.top * W64);
             if (L.shared_size) {
-                act_s = std::max(act_s, (size_t)up64(L.shared_size)), part_s = W64;
+                act_s = std::max(act_s, (size_t)act_stride(L.shared_size)), part_s = W64;
                 if (plan.big) gemm(s->cfg.width, L.shared_size);
             }
         }
     }
     bool moved = false;
     int rc = 0;
-    if ((rc = s->x.need(M * W64, &moved)) || (rc = s->c_raw.need(M * c, &moved)) || (rc = s->part.need(M * part, &moved)) || (rc = s->part_s.need(M * part_s, &moved)) ||
-        (rc = s->h.need(M * W64 * E, &moved)) || (rc = s->q.need(M * q * E, &moved)) || (rc = s->ql.need(M * ql * E, &moved)) || (rc = s->oc.need(M * ql * E, &moved)) ||
+    if ((rc = s->x.need(M * W64, &moved)) || (rc = s->x2.need(s->n_route ? M * W64 : 0, &moved)) || (rc = s->c_raw.need(M * c, &moved)) || (rc = s->part.need(M * part, &moved)) || (rc = s->part_s.need(M * part_s, &moved)) ||
+        (rc = s->h.need(M * WA * E, &moved)) || (rc = s->q.need(M * q * E, &moved)) || (rc = s->ql.need(M * ql * E, &moved)) || (rc = s->oc.need(M * ql * E, &moved)) ||
         (rc = s->o.need(M * o * E, &moved)) || (rc = s->act.need(M * act * E, &moved)) || (rc = s->act_e.need(M * act_e * E, &moved)) ||
         (rc = s->act_s.need(M * act_s * E, &moved)) || (rc = s->stats.need((size_t)b.n_want * ST_TILES, &moved)) || (rc = s->y.need(plan.big ? M * W64 * E : 0, &moved)) ||
         (rc = s->ctx.need(ctx * E, &moved)) || (rc = s->kv.need(kv * E, &moved)) || (rc = s->gemm_ws.need(ws, &moved)))
@@ -376,15 +419,15 @@ int stack_reserve(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
 int plan_splits(const pie_stack_batch &b, const pie_stack_layer &L, int n_tiles) {
     long ctx = (long)b.table_width * PAGE_TOKENS;
     if (L.window > 0 && L.window + 64 < ctx) ctx = L.window + 64;
-    long s = 512 / n_tiles;
+    long s = 256 / n_tiles;
     s = std::min(s, ctx / 64);
     s = std::min(s, 64L);
     return (int)std::max(s, 1L);
 }
 
-int stack_tiles(const int32_t *runs, int n_runs, int H) {
+int stack_tiles(const int32_t *runs, int n_runs, int H, int pairs) {
     int n = 0;
-    for (int i = 0; i < n_runs; ++i) n += (runs[4 * i + 1] * H + 63) / 64;
+    for (int i = 0; i < n_runs; ++i) n += (runs[4 * i + 1] * H + pairs - 1) / pairs;
     return n;
 }
 
@@ -393,6 +436,7 @@ struct Pass {
     const pie_stack_batch &b;
     Plan plan;
     hipStream_t st;
+    float *x, *x_other;  // the residual stream; a mixture's combine moves it to the other buffer
     int rc = PIE_OK, launches = 0;
     // many rows: y = x . W^T rounded to bf16, or the SwiGLU activation of an interleaved matrix
     void gemm(const void *w, const void *x, int ldx, int M, int N, int K, void *y, int ldy, bool swiglu = false) {
@@ -402,9 +446,9 @@ struct Pass {
     // x += post(y); h = next(x)
     void residual(const pie_point_norm &post, const PointNorm &next) {
         if (rc) return;
-        const int W = s->cfg.width, W64 = up64(W);
-        hipLaunchKernelGGL(k_point_residual, dim3((unsigned)((W + 1023) / 1024), (unsigned)b.n_rows), dim3(256), 0, st, (const u16 *)s->y.p, W, norm_of(post), next, s->x.p, W64,
-                           (u16 *)s->h.p, W64, W);
+        const int W = s->cfg.width, W64 = up64(W), WA = act_stride(W);
+        hipLaunchKernelGGL(k_point_residual, dim3((unsigned)((W + 1023) / 1024), (unsigned)b.n_rows), dim3(256), 0, st, (const u16 *)s->y.p, W, norm_of(post), next, x, W64,
+                           (u16 *)s->h.p, WA, W);
         if (hipGetLastError() != hipSuccess) rc = pie::fail(PIE_E_HIP, "residual launch failed");
         ++launches;
     }
@@ -416,30 +460,37 @@ struct Pass {
 void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const PointNorm &next) {
     pie_stack *s = p.s;
     const pie_stack_batch &b = p.b;
-    const int W = s->cfg.width, W64 = up64(W), D8 = up8(L.dim), V8 = up8(L.vdim), R8 = up8(L.rank), H = L.heads, NI = H * D8 + R8, KO = H * V8, LO = up64(KO);
+    const int W = s->cfg.width, W64 = up64(W), WA = act_stride(W), D8 = up8(L.dim), V8 = up8(L.vdim), R8 = up8(L.rank), H = L.heads, NI = H * D8 + R8, KO = H * V8, LO = act_stride(KO);
     const int dt = s->cfg.dtype;
-    if (p.plan.big) {
-        p.gemm(L.w_in, s->h.p, W64, b.n_rows, NI, W, s->q.p, NI);
+    // many rows: q and the latents as two products where the tile rows allow it (together they are a little more than a round of workgroups)
+    const bool two = p.plan.big && (H * D8) % 32 == 0;
+    const int LQ = two ? H * D8 : NI;  // row stride of q
+    if (two) {
+        p.gemm(L.w_in, s->h.p, WA, b.n_rows, H * D8, W, s->q.p, LQ);
+        p.gemm((const char *)L.w_in + (size_t)(H * D8 / 32) * (W64 / 64) * 4096, s->h.p, WA, b.n_rows, R8, W, s->c_raw.p, R8);
+    } else if (p.plan.big) {
+        p.gemm(L.w_in, s->h.p, WA, b.n_rows, NI, W, s->q.p, NI);
     } else {
         RowsArgs a = {};
-        a.m = {(const char *)L.w_in, NI, W, s->h.p, W64, s->q.p, NI};
+        a.m = {(const char *)L.w_in, NI, W, s->h.p, WA, s->q.p, NI};
         a.M = b.n_rows, a.epi = ROWS_SPLIT, a.split = H * D8, a.y2 = s->c_raw.p, a.ldy2 = R8;
         p.linear(a);
     }
     if (p.rc) return;
-    p.rc = latent_append_launch(dt, p.plan.big ? (const void *)((const u16 *)s->q.p + H * D8) : s->c_raw.p, p.plan.big, p.plan.big ? NI : R8, L.c_norm, L.eps, b.n_rows, L.rank, R8,
-                                b.pos, b.row_seq, b.table, b.table_width, (int)b.n_pages, b.n_seqs, b.slabs[li], p.st);
+    p.rc = latent_append_launch(dt, p.plan.big && !two ? (const void *)((const u16 *)s->q.p + H * D8) : s->c_raw.p, p.plan.big, p.plan.big && !two ? NI : R8, L.c_norm, L.eps,
+                                b.n_rows, L.rank, R8, b.pos, b.row_seq, b.table, b.table_width, (int)b.n_pages, b.n_seqs, b.slabs[li], p.st);
     ++p.launches;
     const bool spell = p.plan.long_tiles && spelled_out(L);
     const int M = spell ? p.plan.short_rows : b.n_rows, runs = spell ? p.plan.short_runs : b.n_runs;
     if (M > 0) {  // the latent form
         RowsArgs k = {};
-        k.m = {(const char *)L.w_uk, L.rank, L.dim, s->q.p, NI, s->ql.p, H * R8};
+        k.m = {(const char *)L.w_uk, L.rank, L.dim, s->q.p, LQ, s->ql.p, H * R8};
         k.M = M, k.epi = ROWS_STORE, k.w_batch = rows_weight_bytes(dt, L.rank, L.dim), k.x_batch = D8, k.y_batch = R8;
         p.linear(k, H);
         LatentAttnArgs t = {};
         t.q = s->ql.p, t.slab = b.slabs[li], t.table = b.table, t.table_width = b.table_width, t.n_pages = (int)b.n_pages, t.n_seqs = b.n_seqs, t.pos = b.pos;
-        t.runs = (const RowRun *)b.runs, t.n_runs = runs, t.n_tiles = stack_tiles(b.runs_host, runs, H), t.single = runs == M, t.row_seq = b.row_seq;
+        t.runs = (const RowRun *)b.runs, t.n_runs = runs, t.single = runs == M, t.row_seq = b.row_seq;
+        t.pairs = latent_attn_pairs(H, L.rank, t.single), t.n_tiles = stack_tiles(b.runs_host, runs, H, t.pairs);
         t.H = H, t.R = L.rank, t.ldr = R8, t.M = M, t.window = L.window, t.scale = L.scale, t.splits = plan_splits(b, L, t.n_tiles), t.ws = s->attn_ws.p, t.out = s->oc.p;
         if (!p.rc) p.rc = latent_attn_launch(dt, t, p.st), p.launches += t.splits > 1 ? 2 : 1;
         RowsArgs v = {};
@@ -449,10 +500,10 @@ void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const PointNorm &ne
     }
     if (spell && !p.rc) {
         const RowRun *lr = (const RowRun *)b.runs + p.plan.short_runs;
-        const int n_long = b.n_runs - p.plan.short_runs, n_ctx = (int)plan_context(b, p.plan, L.window), nkv = H * (D8 + V8), LC = up64(L.rank);
+        const int n_long = b.n_runs - p.plan.short_runs, n_ctx = (int)plan_context(b, p.plan, L.window), nkv = H * (D8 + V8), LC = act_stride(L.rank);
         p.rc = latent_gather_launch(lr, n_long, n_ctx, L.window, b.table, b.table_width, b.n_seqs, (int)b.n_pages, b.slabs[li], R8, s->ctx.p, LC, p.st);
         p.gemm(L.w_kv, s->ctx.p, LC, n_ctx, nkv, L.rank, s->kv.p, nkv);
-        WindowAttnArgs w = {(const u16 *)s->q.p, (const u16 *)s->kv.p, (u16 *)s->o.p, NI, nkv, LO, H, D8, V8, L.window, L.scale, lr, n_long};
+        WindowAttnArgs w = {(const u16 *)s->q.p, (const u16 *)s->kv.p, (u16 *)s->o.p, LQ, nkv, LO, H, D8, V8, L.window, L.scale, lr, n_long};
         if (!p.rc) p.rc = window_attn_launch(w, p.plan.long_tiles, p.st), p.launches += 2;
     }
     if (p.plan.big) {
@@ -461,82 +512,84 @@ void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const PointNorm &ne
     } else {
         RowsArgs o = {};
         o.m = {(const char *)L.w_o, W, KO, s->o.p, LO, nullptr, 0};
-        o.M = b.n_rows, o.epi = ROWS_RESIDUAL, o.res = s->x.p, o.ld_res = W64, o.post = norm_of(L.post1), o.next = next, o.h = s->h.p, o.ldh = W64;
+        o.M = b.n_rows, o.epi = ROWS_RESIDUAL, o.res = p.x, o.ld_res = W64, o.post = norm_of(L.post1), o.next = next, o.h = s->h.p, o.ldh = WA;
         p.linear(o);
     }
 }
 
 void feed_forward(Pass &p, int li, const pie_stack_layer &L, const PointNorm &next) {
     pie_stack *s = p.s;
-    const int M = p.b.n_rows, W = s->cfg.width, W64 = up64(W), F = L.ff_size, F64 = up64(F), dt = s->cfg.dtype;
+    const int M = p.b.n_rows, W = s->cfg.width, W64 = up64(W), WA = act_stride(W), F = L.ff_size, FA = act_stride(F), dt = s->cfg.dtype;
     if (L.ff == PIE_FF_RELU2) {
         if (p.plan.big) {
-            if (!p.rc) p.rc = w16l_relu2_launch(L.w_up, s->h.p, W64, M, F, W, s->act.p, F64, p.st), ++p.launches;
-            p.gemm(L.w_down, s->act.p, F64, M, W, F, s->y.p, W);
+            if (!p.rc) p.rc = w16l_relu2_launch(L.w_up, s->h.p, WA, M, F, W, s->act.p, FA, p.st), ++p.launches;
+            p.gemm(L.w_down, s->act.p, FA, M, W, F, s->y.p, W);
             p.residual(L.post2, next);
             return;
         }
         RowsArgs u = {};
-        u.m = {(const char *)L.w_up, F, W, s->h.p, W64, s->act.p, F64};
+        u.m = {(const char *)L.w_up, F, W, s->h.p, WA, s->act.p, FA};
         u.M = M, u.epi = ROWS_RELU2;
         p.linear(u);
         RowsArgs d = {};
-        d.m = {(const char *)L.w_down, W, F, s->act.p, F64, nullptr, 0};
-        d.M = M, d.epi = ROWS_RESIDUAL, d.res = s->x.p, d.ld_res = W64, d.post = norm_of(L.post2), d.next = next, d.h = s->h.p, d.ldh = W64;
+        d.m = {(const char *)L.w_down, W, F, s->act.p, FA, nullptr, 0};
+        d.M = M, d.epi = ROWS_RESIDUAL, d.res = p.x, d.ld_res = W64, d.post = norm_of(L.post2), d.next = next, d.h = s->h.p, d.ldh = WA;
         p.linear(d);
         return;
     }
     const RouteLayer &r = s->route[li];
-    const int S = L.shared_size, S64 = up64(S);
+    const int S = L.shared_size, SA = act_stride(S);
     const size_t gu_stride = rows_weight_bytes(dt, 2 * F, W), dn_stride = rows_weight_bytes(dt, W, F);
     CombineArgs c = {};
-    c.part = s->part.p, c.part_s = s->part_s.p, c.ldp = W64, c.ldp_s = p.plan.big ? W : W64, c.place = r.place, c.top = L.top, c.W = W, c.gate = S ? L.shared_gate : nullptr;
-    c.pre = norm_of(L.pre2), c.post = norm_of(L.post2), c.next = next, c.x = s->x.p, c.ldx = W64, c.h = s->h.p, c.ldh = W64;
+    c.part = s->part.p, c.part_s = s->part_s.p, c.ldp = W64, c.ldp_s = p.plan.big && !(W & 3) ? W : W64, c.place = r.place, c.top = L.top, c.W = W, c.gate = S ? L.shared_gate : nullptr;
+    c.pre = norm_of(L.pre2), c.post = norm_of(L.post2), c.next = next, c.x = p.x, c.x_out = p.x_other, c.ldx = W64, c.h = s->h.p, c.ldh = WA;
+    const dim3 cg((unsigned)((W + 1023) / 1024), (unsigned)M);
     if (p.plan.big) {
         const int tr = route_tile_rows(M, L.top, L.experts), tm = route_max_tiles(M, L.top, L.experts);
-        if (!p.rc) p.rc = w16l_grouped_launch(L.w_gate_up, gu_stride, s->h.p, W64, (size_t)M, r.list, r.tiles, tm, tr, 2 * F, W, s->act_e.p, F64, true, p.st);
-        if (!p.rc) p.rc = w16l_grouped_launch(L.w_expert_down, dn_stride, s->act_e.p, F64, (size_t)M * L.top, nullptr, r.tiles, tm, tr, W, F, s->part.p, W64, false, p.st);
+        if (!p.rc) p.rc = w16l_grouped_launch(L.w_gate_up, gu_stride, s->h.p, WA, (size_t)M, r.list, r.tiles, tm, tr, 2 * F, W, s->act_e.p, FA, true, p.st);
+        if (!p.rc) p.rc = w16l_grouped_launch(L.w_expert_down, dn_stride, s->act_e.p, FA, (size_t)M * L.top, nullptr, r.tiles, tm, tr, W, F, s->part.p, W64, false, p.st);
         p.launches += 2;
         if (S) {
-            p.gemm(L.s_gate_up, s->h.p, W64, M, 2 * S, W, s->act_s.p, S64, true);
-            p.gemm(L.s_down, s->act_s.p, S64, M, W, S, s->part_s.p, W);
+            p.gemm(L.s_gate_up, s->h.p, WA, M, 2 * S, W, s->act_s.p, SA, true);
+            p.gemm(L.s_down, s->act_s.p, SA, M, W, S, s->part_s.p, c.ldp_s);
         }
         if (p.rc) return;
-        hipLaunchKernelGGL((k_moe_combine<ElemBF16, ElemBF16>), dim3((unsigned)M), dim3(256), 0, p.st, c);
+        hipLaunchKernelGGL((k_moe_combine<ElemBF16, ElemBF16>), cg, dim3(256), 0, p.st, c);
     } else {
         const int groups = (int)std::min((long)L.experts, (long)M * L.top) + (S ? 1 : 0);
         RowsArgs u = {};
-        u.m = {(const char *)L.w_gate_up, 2 * F, W, s->h.p, W64, s->act_e.p, F64};
+        u.m = {(const char *)L.w_gate_up, 2 * F, W, s->h.p, WA, s->act_e.p, FA};
         u.M = M, u.epi = ROWS_SILU_MUL, u.w_batch = gu_stride, u.active = r.active, u.offset = r.offset, u.list = r.list, u.gather = true;
-        if (S) u.shared = {(const char *)L.s_gate_up, 2 * S, W, s->h.p, W64, s->act_s.p, S64};
+        if (S) u.shared = {(const char *)L.s_gate_up, 2 * S, W, s->h.p, WA, s->act_s.p, SA};
         p.linear(u, groups);
         RowsArgs d = {};
-        d.m = {(const char *)L.w_expert_down, W, F, s->act_e.p, F64, s->part.p, W64};
+        d.m = {(const char *)L.w_expert_down, W, F, s->act_e.p, FA, s->part.p, W64};
         d.M = M, d.epi = ROWS_SCALE_F32, d.scale = 1.0f, d.w_batch = dn_stride, d.active = r.active, d.offset = r.offset, d.list = r.list;
-        if (S) d.shared = {(const char *)L.s_down, W, S, s->act_s.p, S64, s->part_s.p, W64};
+        if (S) d.shared = {(const char *)L.s_down, W, S, s->act_s.p, SA, s->part_s.p, W64};
         p.linear(d, groups);
         if (p.rc) return;
-        if (dt == PIE_F32) hipLaunchKernelGGL((k_moe_combine<ElemF32, ElemF32>), dim3((unsigned)M), dim3(256), 0, p.st, c);
-        else hipLaunchKernelGGL((k_moe_combine<ElemBF16, ElemF32>), dim3((unsigned)M), dim3(256), 0, p.st, c);
+        if (dt == PIE_F32) hipLaunchKernelGGL((k_moe_combine<ElemF32, ElemF32>), cg, dim3(256), 0, p.st, c);
+        else hipLaunchKernelGGL((k_moe_combine<ElemBF16, ElemF32>), cg, dim3(256), 0, p.st, c);
     }
     if (hipGetLastError() != hipSuccess) p.rc = pie::fail(PIE_E_HIP, "expert combine launch failed");
     ++p.launches;
+    std::swap(p.x, p.x_other);
 }
 
 int stack_enqueue(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipStream_t st) {
-    const int M = b.n_rows, W = s->cfg.width, W64 = up64(W), V = s->cfg.vocab, n = s->cfg.n_layers, dt = s->cfg.dtype;
-    Pass p{s, b, plan, st};
+    const int M = b.n_rows, W = s->cfg.width, W64 = up64(W), WA = act_stride(W), V = s->cfg.vocab, n = s->cfg.n_layers, dt = s->cfg.dtype;
+    Pass p{s, b, plan, st, s->x.p, s->x2.p};
     if (s->n_route) {
         hipLaunchKernelGGL(k_route, dim3((unsigned)s->n_route), dim3(1024), (size_t)s->route_lds, st, s->route_dev.p, b.ids, M, V);
         PIE_LAUNCH_CHECK();
         ++p.launches;
     }
     const PointNorm fin = norm_of(s->cfg.final_norm), first = n ? norm_of(s->layers[0].pre1) : fin;
-    const dim3 ge((unsigned)((W + 255) / 256), (unsigned)M);
+    const dim3 ge((unsigned)((W + 1023) / 1024), (unsigned)M);
     if (dt == PIE_F32)
-        hipLaunchKernelGGL(k_stack_embed<ElemF32>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, first, s->x.p, W64, (float *)s->h.p, W64);
+        hipLaunchKernelGGL(k_stack_embed<ElemF32>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, first, s->x.p, W64, (float *)s->h.p, WA);
     else
-        hipLaunchKernelGGL(k_stack_embed<ElemBF16>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, first, s->x.p, W64, (u16 *)s->h.p, W64);
+        hipLaunchKernelGGL(k_stack_embed<ElemBF16>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, first, s->x.p, W64, (u16 *)s->h.p, WA);
     PIE_LAUNCH_CHECK();
     ++p.launches;
     for (int i = 0; i < n && !p.rc; ++i) {
@@ -545,11 +598,11 @@ int stack_enqueue(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
         latent_mixer(p, i, L, L.ff == PIE_FF_NONE ? after : norm_of(L.pre2));
         if (L.ff != PIE_FF_NONE) feed_forward(p, i, L, after);
         if (b.tap && !p.rc)
-            PIE_HIP_TRY(hipMemcpy2DAsync(b.tap + (size_t)i * M * W, (size_t)W * 4, s->x.p, (size_t)W64 * 4, (size_t)W * 4, (size_t)M, hipMemcpyDeviceToDevice, st));
+            PIE_HIP_TRY(hipMemcpy2DAsync(b.tap + (size_t)i * M * W, (size_t)W * 4, p.x, (size_t)W64 * 4, (size_t)W * 4, (size_t)M, hipMemcpyDeviceToDevice, st));
     }
     if (b.n_want > 0) {
         RowsArgs a = {};
-        a.m = {(const char *)s->cfg.head, V, W, s->h.p, W64, b.logits, V};
+        a.m = {(const char *)s->cfg.head, V, W, s->h.p, WA, b.logits, V};
         a.M = b.n_want, a.epi = ROWS_SCALE_F32, a.scale = s->cfg.logit_scale, a.rows = b.want;
         p.linear(a);
         if (!p.rc && b.next) {
@@ -650,7 +703,8 @@ int pie_stack_forward(pie_stack *s, const pie_stack_batch *bp, int flags, void *
     for (const pie_stack_layer &L : s->layers)
     {
         const bool spell = plan.long_tiles && spelled_out(L);
-        const int M = spell ? plan.short_rows : b.n_rows, tiles = stack_tiles(b.runs_host, spell ? plan.short_runs : b.n_runs, L.heads);
+        const int M = spell ? plan.short_rows : b.n_rows, runs = spell ? plan.short_runs : b.n_runs;
+        const int tiles = stack_tiles(b.runs_host, runs, L.heads, latent_attn_pairs(L.heads, L.rank, runs == M));
         if (tiles) ws = std::max(ws, latent_attn_ws_floats(M, L.heads, L.rank, plan_splits(b, L, tiles)));
     }
     bool moved = false;

@@ -188,7 +188,7 @@ __global__ void __launch_bounds__(256) k_rows_f32(const RowsArgs a) {
 
 template <int NT>
 int rows_go(const RowsArgs &a, int n_max, int k_max, int batches, hipStream_t st) {
-    const int steps = 2 * ((k_max + 63) / 64), tiles = (n_max + 15) / 16, z = (a.M + 16 * NT - 1) / (16 * NT);
+    const int steps = 2 * ((k_max + 63) / 64), tiles = (n_max + 15) / 16, z = (a.M + 16 * NT - 1) / (16 * NT);  // (grouped: most experts have few rows, their later z leave at once)
     // waves along K: enough steps for each, and enough workgroups for the chip
     int kw = steps >= 32 ? 8 : steps >= 16 ? 4 : steps >= 8 ? 2 : 1;
     while (kw < 8 && steps >= 2 * kw && (size_t)((tiles + 8 / kw - 1) / (8 / kw)) * batches * z < 256) kw *= 2;
@@ -226,7 +226,7 @@ int rows_gemm_launch(int dtype, const RowsArgs &a, int batches, hipStream_t st) 
         return PIE_OK;
     }
     PIE_REQUIRE(a.m.ldx % 8 == 0 && a.x_batch % 8 == 0 && pie_aligned(a.m.x, 16) && pie_aligned(a.m.w, 16), PIE_E_ALIGN, "row-wise Linear: 16-byte alignment required");
-    if (a.M <= 16) return rows_go<1>(a, n_max, k_max, batches, st);
+    if (a.M <= 16 || a.active) return rows_go<1>(a, n_max, k_max, batches, st);
     if (a.M <= 32) return rows_go<2>(a, n_max, k_max, batches, st);
     return rows_go<4>(a, n_max, k_max, batches, st);
 }

@@ -1,12 +1,15 @@
 // stack_types.hpp -- what the kernels of the layer-stack models share: the element types, the norms that ride in epilogues, and the operand
 // descriptions of the row-wise Linear (rows_gemm.hip) and of the latent attention (latent_attn.hip).
 //
-// Every activation row has a stride that is a multiple of 8 elements; a Linear reads 64 ceil(K / 64) elements of it.  The columns past K meet zero
+// Every activation row has a stride that is a multiple of 8 elements (act_stride(), or packed); a Linear reads 64 ceil(K / 64) elements of it.  The columns past K meet zero
 // weights, so they only have to be finite: the owner zero-fills its buffers once and keeps 64 elements of slack behind each.
 #pragma once
 #include "common.hpp"
 
 constexpr int PAGE_TOKENS = 64;
+// Row stride (elements) of a 16-bit activation of K columns: an odd number of 256-byte lines, so that the same columns of consecutive rows -- what an
+// MFMA operand load touches -- lie in different cache channels; at a stride of a power of two they would queue up in one.
+static inline int act_stride(int K) { return ((K + 127) / 128 | 1) * 128; }
 
 // Element types of a stack: 16-bit storage (MFMA products, fp32 accumulation) or fp32 throughout.
 struct ElemBF16 {
@@ -26,7 +29,15 @@ struct PointNorm {
     const float *w, *b;
     float alpha;
 };
-__device__ __forceinline__ float point_norm(const PointNorm &n, int i, float x) { return fmaf(tanhf(n.alpha * x), n.w[i], n.b[i]); }
+// tanh to a few units in the last place: below 1/4 the odd Taylor polynomial (next term < 1e-8 of the value), above it 1 - 2 / (e^{2 |z|} + 1)
+__device__ __forceinline__ float fast_tanh(float z) {
+    const float a = fabsf(z), z2 = z * z;
+    const float p = z * fmaf(z2, fmaf(z2, fmaf(z2, fmaf(z2, 62.0f / 2835.0f, -17.0f / 315.0f), 2.0f / 15.0f), -1.0f / 3.0f), 1.0f);
+    const float e = __builtin_amdgcn_exp2f(a * 2.88539008177792681472f);  // e^{2 |z|}; infinite for large |z|: the quotient is then 0
+    const float q = copysignf(1.0f - 2.0f * __builtin_amdgcn_rcpf(e + 1.0f), z);
+    return a < 0.25f ? p : q;
+}
+__device__ __forceinline__ float point_norm(const PointNorm &n, int i, float x) { return fmaf(fast_tanh(n.alpha * x), n.w[i], n.b[i]); }
 
 // ---------------------------------------------------------------- the row-wise Linear
 enum RowsEpi {
@@ -75,7 +86,7 @@ int rows_gemm_launch(int dtype, const RowsArgs &a, int batches, hipStream_t st);
 size_t rows_weight_bytes(int dtype, int N, int K);
 
 // ---------------------------------------------------------------- latent attention
-// A pass holds runs of consecutive rows, one run per sequence; a workgroup takes up to 64 (token, head) pairs of ONE run.
+// A pass holds runs of consecutive rows, one run per sequence; a workgroup takes 16, 32 or 64 (token, head) pairs of ONE run.
 struct RowRun {
     int row0, n_rows, seq, pos0;  // seq: row of the block table; pos0: position of row0 (single rows: not used, may be 0)
 };
@@ -86,7 +97,8 @@ struct LatentAttnArgs {
     int table_width, n_pages, n_seqs;
     const int *pos;        // [M]
     const RowRun *runs;
-    int n_runs, n_tiles;   // n_tiles = sum over the runs of ceil(n_rows * H / 64)
+    int n_runs, n_tiles;   // n_tiles = sum over the runs of ceil(n_rows * H / pairs)
+    int pairs;             // (token, head) pairs per workgroup: latent_attn_pairs()
     bool single;           // every run is one row (a decode step): tile -> run without a search
     const int *row_seq;    // [M]
     int H, R, ldr, M;
@@ -97,6 +109,7 @@ struct LatentAttnArgs {
     void *out;             // [M][H][ldr] T: softmax-weighted latents
 };
 int latent_attn_launch(int dtype, const LatentAttnArgs &a, hipStream_t st);
+int latent_attn_pairs(int H, int R, bool single);  // single decoded tokens of few heads take smaller tiles and split the keys over the waves
 size_t latent_attn_ws_floats(int M, int H, int R, int splits);
 // c_raw [M][ldc], fp32 or (raw16) bf16 -> RMS norm with weight w -> the row of its page
 int latent_append_launch(int dtype, const void *c_raw, bool raw16, int ldc, const float *w, float eps, int M, int R, int ldr, const int *pos, const int *row_seq,
