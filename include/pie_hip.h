@@ -558,7 +558,8 @@ typedef struct pie_stack pie_stack;
 size_t pie_stack_weight_bytes(int dtype, int N, int K);
 int pie_stack_pack_weight(const void *w, int N, int K, int dtype, void *packed, void *stream);
 
-/* Dynamic Tanh: w * tanh(alpha x) + b, element by element.  w, b: fp32 [width] on the device. */
+/* Dynamic Tanh: w * tanh(alpha x) + b, element by element.  w, b: fp32 [width rounded up to 8, zeros past it] on the
+ * device, 16-byte aligned. */
 typedef struct {
     const float *w, *b;
     float alpha;
@@ -581,7 +582,8 @@ enum { PIE_FF_NONE = 0, PIE_FF_RELU2 = 1, PIE_FF_TABLE_MOE = 2 };
  * w_o packed [width, heads * vdim8]; w_kv packed [heads * (dim8 + vdim8), rank] (all keys, then all values: long prompts spell K and V out; may be
  * NULL); c_norm fp32 [rank].  window <= 0: no limit.
  * Experts: w_gate_up experts x packed [2 * size, width] with rows (2 i, 2 i + 1) = (gate_i, up_i); w_down experts x packed [width, size];
- * table int32 [vocab][top].  Shared expert likewise when shared_size > 0, times sigmoid(shared_gate . input), shared_gate fp32 [width]. */
+ * table int32 [vocab][top].  Shared expert likewise when shared_size > 0, times sigmoid(shared_gate . input), shared_gate fp32 [width,
+ * rounded up to 8 with zeros]. */
 typedef struct {
     pie_point_norm pre1, post1, pre2, post2;
     int mixer, heads, dim, vdim, rank, window;

@@ -3,8 +3,7 @@
 // A pass is a batch of rows, each with its own sequence and position: whole prompts, portions and single decoded tokens are the same thing here.
 // Launches per layer (every norm is element-wise and rides in the epilogue of the kernel that produces its input):
 //   [q | latent down]     Linear                                      (rows_gemm.hip)
-//   latent RMS norm + page append                                     (latent_attn.hip)
-//   q -> latent space     Linear per head
+//   q -> latent space     Linear per head; beside it the latents' RMS norm and their append to the pages
 //   attention over the latents [+ merge of the key splits]            (latent_attn.hip)
 //   latents -> values     Linear per head
 //   output projection     Linear; epilogue: x += post1(y), h = pre2(x)
@@ -25,7 +24,7 @@ size_t w16l_workspace_bytes(int M, int N, int K);
 int w16l_gemm_launch(int dtype, const void *w16m, const void *x, int ldx, int M, int N, int K, void *y, void *workspace, hipStream_t st, const void *bias,
                      void *swiglu_act, bool *fused, int ldy);
 int w16l_relu2_launch(const void *w16m, const void *x, int ldx, int M, int N, int K, void *y, int ldy, hipStream_t st);
-int w16l_grouped_launch(const void *w16m, size_t w_stride, const void *x, int ldx, size_t x_rows, const int *list, const void *tiles, int tm, int tile_rows, int N, int K,
+int w16l_grouped_launch(const void *w16m, size_t w_stride, const void *x, int ldx, size_t x_rows, const int *list, const void *tiles, int tm, int block, int tile_rows, int N, int K,
                         void *y, int ldy, bool swiglu, hipStream_t st);
 
 namespace {
@@ -41,7 +40,13 @@ struct RouteLayer {      // one mixture layer's row lists (device pointers)
 };
 // rows per tile of the grouped GEMM, and a bound on the number of tiles
 __host__ __device__ inline int route_tile_rows(long M, int top, int experts) { return M * top >= 96l * experts ? 128 : 64; }
-__host__ __device__ inline int route_max_tiles(long M, int top, int experts) { return (int)(M * top / route_tile_rows(M, top, experts)) + experts; }
+// (an expert's tiles start at a multiple of route_block(): the grouped GEMM runs that many side by side on one XCD, over the same weights)
+// (about as many as an expert has: empty tiles cost a workgroup launch each)
+constexpr int ROUTE_BLOCK_MAX = 4;
+__host__ __device__ inline int route_block(long M, int top, int experts) { return M * top >= 2l * 128 * experts ? 4 : M * top >= 128l * experts ? 2 : 1; }
+__host__ __device__ inline int route_max_tiles(long M, int top, int experts) {
+    return ((int)(M * top / route_tile_rows(M, top, experts)) + route_block(M, top, experts) * experts + 3) / 4 * 4;
+}
 
 __global__ void __launch_bounds__(1024) k_route(const RouteLayer *layers, const int *ids, int M, int vocab) {
     extern __shared__ int s_cnt[];  // [experts] counts, then [experts] cursors
@@ -58,7 +63,7 @@ __global__ void __launch_bounds__(1024) k_route(const RouteLayer *layers, const 
     __syncthreads();
     if (threadIdx.x < 64) {
         int base = 0, n_active = 0, n_tiles = 0;
-        const int tr = route_tile_rows(M, L.top, L.experts);
+        const int tr = route_tile_rows(M, L.top, L.experts), rb = route_block(M, L.top, L.experts);
         for (int e0 = 0; e0 < L.experts; e0 += 64) {
             const int e = e0 + (int)threadIdx.x, c = e < L.experts ? s_cnt[e] : 0;
             int incl = c;
@@ -72,14 +77,14 @@ __global__ void __launch_bounds__(1024) k_route(const RouteLayer *layers, const 
             const int slot = n_active + __popcll(has & ((1ull << threadIdx.x) - 1ull));
             if (c > 0 && slot < L.max_active) L.active[slot] = e;
             if (L.tiles) {
-                const int mine = (c + tr - 1) / tr;
-                int ti = mine;
+                const int mine = (c + tr - 1) / tr, slots = (mine + rb - 1) / rb * rb;
+                int ti = slots;
 #pragma unroll
                 for (int o = 1; o < 64; o <<= 1) {
                     const int v = __shfl_up(ti, o, 64);
                     if ((int)threadIdx.x >= o) ti += v;
                 }
-                for (int k = 0; k < mine; ++k) L.tiles[n_tiles + ti - mine + k] = make_int4(e, base + incl - c + k * tr, min(tr, c - k * tr), 0);
+                for (int k = 0; k < slots; ++k) L.tiles[n_tiles + ti - slots + k] = make_int4(e, base + incl - c + k * tr, max(0, min(tr, c - k * tr)), 0);
                 n_tiles += __shfl(ti, 63, 64);
             }
             base += __shfl(incl, 63, 64), n_active += __popcll(has);
@@ -98,6 +103,11 @@ __global__ void __launch_bounds__(1024) k_route(const RouteLayer *layers, const 
 }
 
 template <class E>
+__device__ __forceinline__ void store4(typename E::type *p, float4 y) {
+    if constexpr (sizeof(typename E::type) == 2) *(uint2 *)p = make_uint2(pack2<BF16>(y.x, y.y), pack2<BF16>(y.z, y.w));
+    else *(float4 *)p = y;
+}
+template <class E>
 __global__ void __launch_bounds__(256) k_stack_embed(const int *ids, const u16 *table, int vocab, int W, PointNorm next, float *x, int ldx, typename E::type *h, int ldh) {
     const size_t m = blockIdx.y;
     const int n = (blockIdx.x * 256 + threadIdx.x) * 4;
@@ -105,10 +115,9 @@ __global__ void __launch_bounds__(256) k_stack_embed(const int *ids, const u16 *
     const u16 *src = table + (size_t)min(max(ids[m], 0), vocab - 1) * W + n;
     if (n + 4 <= W && !(W & 3)) {
         const uint2 t = *(const uint2 *)src;
-        const float v[4] = {lo_f32<BF16>(t.x), hi_f32<BF16>(t.x), lo_f32<BF16>(t.y), hi_f32<BF16>(t.y)};
-        *(float4 *)(x + m * ldx + n) = make_float4(v[0], v[1], v[2], v[3]);
-#pragma unroll
-        for (int i = 0; i < 4; ++i) h[m * ldh + n + i] = E::pack(point_norm(next, n + i, v[i]));
+        const float4 v = make_float4(lo_f32<BF16>(t.x), hi_f32<BF16>(t.x), lo_f32<BF16>(t.y), hi_f32<BF16>(t.y)), y = point_norm4(next, n, v);
+        *(float4 *)(x + m * ldx + n) = v;
+        store4<E>(h + m * ldh + n, y);
         return;
     }
     for (int i = 0; i < min(4, W - n); ++i) {
@@ -126,13 +135,11 @@ struct CombineArgs {
     int top, W;
     const float *gate;           // [W] or nullptr
     PointNorm pre, post, next;   // pre: the sublayer's input norm (the gate's dot product is taken in fp32 on it)
-    const float *x;
-    float *x_out;                // another buffer: every block of a row reads all of x
+    float *x;
     int ldx;
     void *h;
     int ldh;
 };
-// grid (column blocks of 1024, rows): every block of a row takes the gate's dot product itself
 template <class P>
 __device__ __forceinline__ float4 load4(const void *p, size_t i) {
     if constexpr (sizeof(typename P::type) == 4) return *(const float4 *)((const float *)p + i);
@@ -141,51 +148,60 @@ __device__ __forceinline__ float4 load4(const void *p, size_t i) {
         return make_float4(lo_f32<BF16>(v.x), hi_f32<BF16>(v.x), lo_f32<BF16>(v.y), hi_f32<BF16>(v.y));
     }
 }
-template <class E, class P>  // P: element type of the experts' outputs
-__global__ void __launch_bounds__(256) k_moe_combine(const CombineArgs a) {
-    __shared__ float red[4];
-    const size_t m = blockIdx.y;
-    const float *x = a.x + m * a.ldx;
-    const int n = (blockIdx.x * 256 + threadIdx.x) * 4;
-    const bool in = n < a.W;
+template <class E, class P>  // P: element type of the experts' outputs.  One workgroup per row, four columns per thread and pass.
+__global__ void __launch_bounds__(1024) k_moe_combine(const CombineArgs a) {
+    __shared__ float red[16];
+    const size_t m = blockIdx.x;
+    float *x = a.x + m * a.ldx;
     constexpr int U = 8;  // slots in flight
-    float4 v[U], vs = make_float4(0, 0, 0, 0);
+    float4 v[U], vs = make_float4(0, 0, 0, 0), xv = vs;
+    int n = threadIdx.x * 4;
     auto fetch = [&](int s0) {
 #pragma unroll
         for (int u = 0; u < U; ++u)
             if (s0 + u < a.top) v[u] = load4<P>(a.part, (size_t)a.place[m * a.top + s0 + u] * a.ldp + n);
     };
-    if (in) {  // (rows of part hold 64 ceil(W / 64) columns: a quad that starts inside W is readable)
+    auto fetch_row = [&] {  // (rows of x, part and the norms' paddings: a quad that starts inside W is readable up to the next multiple of 4)
         fetch(0);
         if (a.gate) vs = load4<P>(a.part_s, m * a.ldp_s + n);
-    }
+        xv = *(const float4 *)(x + n);
+    };
+    if (n < a.W) fetch_row();
     float g = 0.0f;
     if (a.gate) {
         float d = 0.0f;
-#pragma unroll 4
-        for (int i = threadIdx.x; i < a.W; i += 256) d = fmaf(point_norm(a.pre, i, x[i]), a.gate[i], d);
+        for (int k = n; k < a.W; k += blockDim.x * 4) {
+            const float4 q = point_norm4(a.pre, k, k == n ? xv : *(const float4 *)(x + k)), w = *(const float4 *)(a.gate + k);
+            d += (fmaf(q.x, w.x, q.y * w.y) + fmaf(q.z, w.z, q.w * w.w));  // (columns past W: zero gate weights)
+        }
         d = wave_sum(d);
         if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = d;
         __syncthreads();
-        g = 1.0f / (1.0f + expf(-((red[0] + red[1]) + (red[2] + red[3]))));
+        d = red[0];
+        for (int i = 1; i < (int)blockDim.x / 64; ++i) d += red[i];
+        g = 1.0f / (1.0f + expf(-d));
     }
-    if (!in) return;
     const float share = 1.0f / (float)a.top;
-    float y[4] = {0, 0, 0, 0};
-    for (int s0 = 0; s0 < a.top; s0 += U) {
-        if (s0) fetch(s0);
+    for (; n < a.W; n += blockDim.x * 4) {
+        if (n != (int)threadIdx.x * 4) fetch_row();
+        float y[4] = {0, 0, 0, 0};
+        for (int s0 = 0; s0 < a.top; s0 += U) {
+            if (s0) fetch(s0);
 #pragma unroll
-        for (int u = 0; u < U; ++u)
-            if (s0 + u < a.top) y[0] = fmaf(share, v[u].x, y[0]), y[1] = fmaf(share, v[u].y, y[1]), y[2] = fmaf(share, v[u].z, y[2]), y[3] = fmaf(share, v[u].w, y[3]);
-    }
-    if (a.gate) y[0] = fmaf(g, vs.x, y[0]), y[1] = fmaf(g, vs.y, y[1]), y[2] = fmaf(g, vs.z, y[2]), y[3] = fmaf(g, vs.w, y[3]);
-    float *xo = a.x_out + m * a.ldx;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        if (n + i >= a.W) break;
-        const float r = x[n + i] + point_norm(a.post, n + i, y[i]);
-        xo[n + i] = r;
-        ((typename E::type *)a.h)[m * a.ldh + n + i] = E::pack(point_norm(a.next, n + i, r));
+            for (int u = 0; u < U; ++u)
+                if (s0 + u < a.top) y[0] = fmaf(share, v[u].x, y[0]), y[1] = fmaf(share, v[u].y, y[1]), y[2] = fmaf(share, v[u].z, y[2]), y[3] = fmaf(share, v[u].w, y[3]);
+        }
+        if (a.gate) y[0] = fmaf(g, vs.x, y[0]), y[1] = fmaf(g, vs.y, y[1]), y[2] = fmaf(g, vs.z, y[2]), y[3] = fmaf(g, vs.w, y[3]);
+        const float4 q = point_norm4(a.post, n, make_float4(y[0], y[1], y[2], y[3]));
+        const float4 r = make_float4(xv.x + q.x, xv.y + q.y, xv.z + q.z, xv.w + q.w), hn = point_norm4(a.next, n, r);
+        typename E::type *h = (typename E::type *)a.h + m * a.ldh + n;
+        if (n + 4 <= a.W) {
+            *(float4 *)(x + n) = r;
+            store4<E>(h, hn);
+        } else {
+            const float re[4] = {r.x, r.y, r.z, r.w}, he[4] = {hn.x, hn.y, hn.z, hn.w};
+            for (int i = 0; i < a.W - n; ++i) x[n + i] = re[i], h[i] = E::pack(he[i]);
+        }
     }
 }
 
@@ -197,11 +213,10 @@ __global__ void __launch_bounds__(256) k_point_residual(const u16 *y, int ldy, P
     if (n + 4 <= W && !(ldy & 3)) {
         const uint2 yv = *(const uint2 *)(y + m * ldy + n);
         float4 *xp = (float4 *)(x + m * ldx + n), v = *xp;
-        v.x += point_norm(post, n, lo_f32<BF16>(yv.x)), v.y += point_norm(post, n + 1, hi_f32<BF16>(yv.x));
-        v.z += point_norm(post, n + 2, lo_f32<BF16>(yv.y)), v.w += point_norm(post, n + 3, hi_f32<BF16>(yv.y));
+        const float4 q = point_norm4(post, n, make_float4(lo_f32<BF16>(yv.x), hi_f32<BF16>(yv.x), lo_f32<BF16>(yv.y), hi_f32<BF16>(yv.y)));
+        v.x += q.x, v.y += q.y, v.z += q.z, v.w += q.w;
         *xp = v;
-        *(uint2 *)(h + m * ldh + n) = make_uint2(pack2<BF16>(point_norm(next, n, v.x), point_norm(next, n + 1, v.y)),
-                                                 pack2<BF16>(point_norm(next, n + 2, v.z), point_norm(next, n + 3, v.w)));
+        store4<ElemBF16>(h + m * ldh + n, point_norm4(next, n, v));
         return;
     }
     for (int i = n; i < min(n + 4, W); ++i) {
@@ -306,7 +321,7 @@ struct pie_stack {
     std::vector<pie_stack_layer> layers;
     std::vector<char> have;
     // workspace, by rows of a pass
-    Buf<float> x, x2, c_raw, part, part_s, attn_ws, gemm_ws;
+    Buf<float> x, c_raw, part, part_s, attn_ws, gemm_ws;
     Buf<char> h, q, ql, oc, o, act, act_e, act_s, y, ctx, kv;
     Buf<RowStat> stats;
     Buf<int> route_ints;
@@ -379,7 +394,7 @@ int stack_reserve(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
     }
     bool moved = false;
     int rc = 0;
-    if ((rc = s->x.need(M * W64, &moved)) || (rc = s->x2.need(s->n_route ? M * W64 : 0, &moved)) || (rc = s->c_raw.need(M * c, &moved)) || (rc = s->part.need(M * part, &moved)) || (rc = s->part_s.need(M * part_s, &moved)) ||
+    if ((rc = s->x.need(M * W64, &moved)) || (rc = s->c_raw.need(M * c, &moved)) || (rc = s->part.need(M * part, &moved)) || (rc = s->part_s.need(M * part_s, &moved)) ||
         (rc = s->h.need(M * WA * E, &moved)) || (rc = s->q.need(M * q * E, &moved)) || (rc = s->ql.need(M * ql * E, &moved)) || (rc = s->oc.need(M * ql * E, &moved)) ||
         (rc = s->o.need(M * o * E, &moved)) || (rc = s->act.need(M * act * E, &moved)) || (rc = s->act_e.need(M * act_e * E, &moved)) ||
         (rc = s->act_s.need(M * act_s * E, &moved)) || (rc = s->stats.need((size_t)b.n_want * ST_TILES, &moved)) || (rc = s->y.need(plan.big ? M * W64 * E : 0, &moved)) ||
@@ -387,8 +402,8 @@ int stack_reserve(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
         return rc;
     if (s->n_route && (int)M > s->route_rows) {
         s->route_rows = (int)M;
-        // (at most this many tiles for any pass of up to M rows: 64-row tiles and one ragged tile per expert)
-        auto tiles = [&](const RouteLayer &r) { return M * r.top / 64 + r.experts + 1; };
+        // (at most this many tiles for any pass of up to M rows: 64-row tiles and one ragged block of tiles per expert)
+        auto tiles = [&](const RouteLayer &r) { return (M * r.top / 64 + ROUTE_BLOCK_MAX * r.experts + 3) / 4 * 4; };
         for (const RouteLayer &r : s->route)
             if (r.experts) ints += (2 * (size_t)r.experts + 1 + 2 * M * r.top + 3) / 4 * 4 + 4 * tiles(r);
         if ((rc = s->route_ints.need(ints, &moved)) || (rc = s->route_dev.need(s->n_route, &moved))) return rc;
@@ -425,9 +440,9 @@ int plan_splits(const pie_stack_batch &b, const pie_stack_layer &L, int n_tiles)
     return (int)std::max(s, 1L);
 }
 
-int stack_tiles(const int32_t *runs, int n_runs, int H, int pairs) {
+int stack_tiles(const int32_t *runs, int n_runs, int H) {
     int n = 0;
-    for (int i = 0; i < n_runs; ++i) n += (runs[4 * i + 1] * H + pairs - 1) / pairs;
+    for (int i = 0; i < n_runs; ++i) n += latent_attn_tiles(runs[4 * i + 1], H);
     return n;
 }
 
@@ -436,7 +451,6 @@ struct Pass {
     const pie_stack_batch &b;
     Plan plan;
     hipStream_t st;
-    float *x, *x_other;  // the residual stream; a mixture's combine moves it to the other buffer
     int rc = PIE_OK, launches = 0;
     // many rows: y = x . W^T rounded to bf16, or the SwiGLU activation of an interleaved matrix
     void gemm(const void *w, const void *x, int ldx, int M, int N, int K, void *y, int ldy, bool swiglu = false) {
@@ -447,7 +461,7 @@ struct Pass {
     void residual(const pie_point_norm &post, const PointNorm &next) {
         if (rc) return;
         const int W = s->cfg.width, W64 = up64(W), WA = act_stride(W);
-        hipLaunchKernelGGL(k_point_residual, dim3((unsigned)((W + 1023) / 1024), (unsigned)b.n_rows), dim3(256), 0, st, (const u16 *)s->y.p, W, norm_of(post), next, x, W64,
+        hipLaunchKernelGGL(k_point_residual, dim3((unsigned)((W + 1023) / 1024), (unsigned)b.n_rows), dim3(256), 0, st, (const u16 *)s->y.p, W, norm_of(post), next, s->x.p, W64,
                            (u16 *)s->h.p, WA, W);
         if (hipGetLastError() != hipSuccess) rc = pie::fail(PIE_E_HIP, "residual launch failed");
         ++launches;
@@ -477,20 +491,21 @@ void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const PointNorm &ne
         p.linear(a);
     }
     if (p.rc) return;
-    p.rc = latent_append_launch(dt, p.plan.big && !two ? (const void *)((const u16 *)s->q.p + H * D8) : s->c_raw.p, p.plan.big, p.plan.big && !two ? NI : R8, L.c_norm, L.eps,
-                                b.n_rows, L.rank, R8, b.pos, b.row_seq, b.table, b.table_width, (int)b.n_pages, b.n_seqs, b.slabs[li], p.st);
-    ++p.launches;
+    const LatentAppend append = {p.plan.big && !two ? (const void *)((const u16 *)s->q.p + H * D8) : s->c_raw.p, p.plan.big, p.plan.big && !two ? NI : R8, L.c_norm, L.eps, b.n_rows,
+                                 L.rank, R8, b.pos, b.row_seq, b.table, b.table_width, (int)b.n_pages, b.n_seqs, b.slabs[li]};
+    if (p.plan.big) p.rc = latent_append_launch(dt, append, p.st), ++p.launches;  // (few rows: rides in the next launch)
     const bool spell = p.plan.long_tiles && spelled_out(L);
     const int M = spell ? p.plan.short_rows : b.n_rows, runs = spell ? p.plan.short_runs : b.n_runs;
     if (M > 0) {  // the latent form
         RowsArgs k = {};
         k.m = {(const char *)L.w_uk, L.rank, L.dim, s->q.p, LQ, s->ql.p, H * R8};
         k.M = M, k.epi = ROWS_STORE, k.w_batch = rows_weight_bytes(dt, L.rank, L.dim), k.x_batch = D8, k.y_batch = R8;
+        if (!p.plan.big) k.append = append;
         p.linear(k, H);
         LatentAttnArgs t = {};
         t.q = s->ql.p, t.slab = b.slabs[li], t.table = b.table, t.table_width = b.table_width, t.n_pages = (int)b.n_pages, t.n_seqs = b.n_seqs, t.pos = b.pos;
         t.runs = (const RowRun *)b.runs, t.n_runs = runs, t.single = runs == M, t.row_seq = b.row_seq;
-        t.pairs = latent_attn_pairs(H, L.rank, t.single), t.n_tiles = stack_tiles(b.runs_host, runs, H, t.pairs);
+        t.n_tiles = stack_tiles(b.runs_host, runs, H);
         t.H = H, t.R = L.rank, t.ldr = R8, t.M = M, t.window = L.window, t.scale = L.scale, t.splits = plan_splits(b, L, t.n_tiles), t.ws = s->attn_ws.p, t.out = s->oc.p;
         if (!p.rc) p.rc = latent_attn_launch(dt, t, p.st), p.launches += t.splits > 1 ? 2 : 1;
         RowsArgs v = {};
@@ -512,7 +527,7 @@ void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const PointNorm &ne
     } else {
         RowsArgs o = {};
         o.m = {(const char *)L.w_o, W, KO, s->o.p, LO, nullptr, 0};
-        o.M = b.n_rows, o.epi = ROWS_RESIDUAL, o.res = p.x, o.ld_res = W64, o.post = norm_of(L.post1), o.next = next, o.h = s->h.p, o.ldh = WA;
+        o.M = b.n_rows, o.epi = ROWS_RESIDUAL, o.res = s->x.p, o.ld_res = W64, o.post = norm_of(L.post1), o.next = next, o.h = s->h.p, o.ldh = WA;
         p.linear(o);
     }
 }
@@ -533,7 +548,7 @@ void feed_forward(Pass &p, int li, const pie_stack_layer &L, const PointNorm &ne
         p.linear(u);
         RowsArgs d = {};
         d.m = {(const char *)L.w_down, W, F, s->act.p, FA, nullptr, 0};
-        d.M = M, d.epi = ROWS_RESIDUAL, d.res = p.x, d.ld_res = W64, d.post = norm_of(L.post2), d.next = next, d.h = s->h.p, d.ldh = WA;
+        d.M = M, d.epi = ROWS_RESIDUAL, d.res = s->x.p, d.ld_res = W64, d.post = norm_of(L.post2), d.next = next, d.h = s->h.p, d.ldh = WA;
         p.linear(d);
         return;
     }
@@ -542,19 +557,19 @@ void feed_forward(Pass &p, int li, const pie_stack_layer &L, const PointNorm &ne
     const size_t gu_stride = rows_weight_bytes(dt, 2 * F, W), dn_stride = rows_weight_bytes(dt, W, F);
     CombineArgs c = {};
     c.part = s->part.p, c.part_s = s->part_s.p, c.ldp = W64, c.ldp_s = p.plan.big && !(W & 3) ? W : W64, c.place = r.place, c.top = L.top, c.W = W, c.gate = S ? L.shared_gate : nullptr;
-    c.pre = norm_of(L.pre2), c.post = norm_of(L.post2), c.next = next, c.x = p.x, c.x_out = p.x_other, c.ldx = W64, c.h = s->h.p, c.ldh = WA;
-    const dim3 cg((unsigned)((W + 1023) / 1024), (unsigned)M);
+    c.pre = norm_of(L.pre2), c.post = norm_of(L.post2), c.next = next, c.x = s->x.p, c.ldx = W64, c.h = s->h.p, c.ldh = WA;
+    const dim3 cg((unsigned)M), cb((unsigned)std::min(1024, ((W + 3) / 4 + 63) / 64 * 64));
     if (p.plan.big) {
-        const int tr = route_tile_rows(M, L.top, L.experts), tm = route_max_tiles(M, L.top, L.experts);
-        if (!p.rc) p.rc = w16l_grouped_launch(L.w_gate_up, gu_stride, s->h.p, WA, (size_t)M, r.list, r.tiles, tm, tr, 2 * F, W, s->act_e.p, FA, true, p.st);
-        if (!p.rc) p.rc = w16l_grouped_launch(L.w_expert_down, dn_stride, s->act_e.p, FA, (size_t)M * L.top, nullptr, r.tiles, tm, tr, W, F, s->part.p, W64, false, p.st);
+        const int tr = route_tile_rows(M, L.top, L.experts), tm = route_max_tiles(M, L.top, L.experts), rb = route_block(M, L.top, L.experts);
+        if (!p.rc) p.rc = w16l_grouped_launch(L.w_gate_up, gu_stride, s->h.p, WA, (size_t)M, r.list, r.tiles, tm, rb, tr, 2 * F, W, s->act_e.p, FA, true, p.st);
+        if (!p.rc) p.rc = w16l_grouped_launch(L.w_expert_down, dn_stride, s->act_e.p, FA, (size_t)M * L.top, nullptr, r.tiles, tm, rb, tr, W, F, s->part.p, W64, false, p.st);
         p.launches += 2;
         if (S) {
             p.gemm(L.s_gate_up, s->h.p, WA, M, 2 * S, W, s->act_s.p, SA, true);
             p.gemm(L.s_down, s->act_s.p, SA, M, W, S, s->part_s.p, c.ldp_s);
         }
         if (p.rc) return;
-        hipLaunchKernelGGL((k_moe_combine<ElemBF16, ElemBF16>), cg, dim3(256), 0, p.st, c);
+        hipLaunchKernelGGL((k_moe_combine<ElemBF16, ElemBF16>), cg, cb, 0, p.st, c);
     } else {
         const int groups = (int)std::min((long)L.experts, (long)M * L.top) + (S ? 1 : 0);
         RowsArgs u = {};
@@ -568,17 +583,16 @@ void feed_forward(Pass &p, int li, const pie_stack_layer &L, const PointNorm &ne
         if (S) d.shared = {(const char *)L.s_down, W, S, s->act_s.p, SA, s->part_s.p, W64};
         p.linear(d, groups);
         if (p.rc) return;
-        if (dt == PIE_F32) hipLaunchKernelGGL((k_moe_combine<ElemF32, ElemF32>), cg, dim3(256), 0, p.st, c);
-        else hipLaunchKernelGGL((k_moe_combine<ElemBF16, ElemF32>), cg, dim3(256), 0, p.st, c);
+        if (dt == PIE_F32) hipLaunchKernelGGL((k_moe_combine<ElemF32, ElemF32>), cg, cb, 0, p.st, c);
+        else hipLaunchKernelGGL((k_moe_combine<ElemBF16, ElemF32>), cg, cb, 0, p.st, c);
     }
     if (hipGetLastError() != hipSuccess) p.rc = pie::fail(PIE_E_HIP, "expert combine launch failed");
     ++p.launches;
-    std::swap(p.x, p.x_other);
 }
 
 int stack_enqueue(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipStream_t st) {
     const int M = b.n_rows, W = s->cfg.width, W64 = up64(W), WA = act_stride(W), V = s->cfg.vocab, n = s->cfg.n_layers, dt = s->cfg.dtype;
-    Pass p{s, b, plan, st, s->x.p, s->x2.p};
+    Pass p{s, b, plan, st};
     if (s->n_route) {
         hipLaunchKernelGGL(k_route, dim3((unsigned)s->n_route), dim3(1024), (size_t)s->route_lds, st, s->route_dev.p, b.ids, M, V);
         PIE_LAUNCH_CHECK();
@@ -598,7 +612,7 @@ int stack_enqueue(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
         latent_mixer(p, i, L, L.ff == PIE_FF_NONE ? after : norm_of(L.pre2));
         if (L.ff != PIE_FF_NONE) feed_forward(p, i, L, after);
         if (b.tap && !p.rc)
-            PIE_HIP_TRY(hipMemcpy2DAsync(b.tap + (size_t)i * M * W, (size_t)W * 4, p.x, (size_t)W64 * 4, (size_t)W * 4, (size_t)M, hipMemcpyDeviceToDevice, st));
+            PIE_HIP_TRY(hipMemcpy2DAsync(b.tap + (size_t)i * M * W, (size_t)W * 4, s->x.p, (size_t)W64 * 4, (size_t)W * 4, (size_t)M, hipMemcpyDeviceToDevice, st));
     }
     if (b.n_want > 0) {
         RowsArgs a = {};
@@ -704,7 +718,7 @@ int pie_stack_forward(pie_stack *s, const pie_stack_batch *bp, int flags, void *
     {
         const bool spell = plan.long_tiles && spelled_out(L);
         const int M = spell ? plan.short_rows : b.n_rows, runs = spell ? plan.short_runs : b.n_runs;
-        const int tiles = stack_tiles(b.runs_host, runs, L.heads, latent_attn_pairs(L.heads, L.rank, runs == M));
+        const int tiles = stack_tiles(b.runs_host, runs, L.heads);
         if (tiles) ws = std::max(ws, latent_attn_ws_floats(M, L.heads, L.rank, plan_splits(b, L, tiles)));
     }
     bool moved = false;

@@ -77,27 +77,41 @@ __device__ __forceinline__ void rows_finish(const RowsArgs &a, const RowsWork &k
     }
 }
 
-// NT: blocks of 16 rows of x; KW: waves along K
-template <int NT, int KW>
+template <class E, int THREADS>
+__device__ __forceinline__ bool rows_append(const RowsArgs &a, float *red) {
+    if (a.append.M <= 0 || blockIdx.y + 1 < gridDim.y) return false;
+    if (blockIdx.z == 0)
+        for (int m = blockIdx.x; m < a.append.M; m += gridDim.x) {
+            latent_append_row<E, ElemF32, THREADS>(a.append, m, red);
+            __syncthreads();
+        }
+    return true;
+}
+
+// NT: blocks of 16 rows of x; KW: waves along K; NN: blocks of 16 features per wave (two share the x operands)
+template <int NT, int KW, int NN>
 __global__ void __launch_bounds__(512) k_rows_w16m(const RowsArgs a) {
     constexpr int NW = 8 / KW, U = NT >= 4 ? 2 : 4;
     constexpr int ST = 20;  // floats per (row, 16 features) line of the reduction image
-    __shared__ __attribute__((aligned(16))) float s_red[8 * NT * 16 * ST];
+    __shared__ __attribute__((aligned(16))) float s_red[8 * NN * NT * 16 * ST];
+    if (rows_append<ElemBF16, 512>(a, s_red)) return;
     RowsWork k;
     if (!rows_select(a, k)) return;
     const int i0 = blockIdx.z * 16 * NT;
     if (i0 >= k.count) return;
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int wn = wave / KW, wk = wave % KW;
-    const int t16 = blockIdx.x * NW + wn;  // this wave's 16 output features
-    if ((int)blockIdx.x * NW * 16 >= k.N) return;
+    const int t16 = (blockIdx.x * NW + wn) * NN;  // this wave's first block of 16 output features
+    if ((int)blockIdx.x * NW * NN * 16 >= k.N) return;
     const int c = lane & 15, kq = lane >> 4;
     const int groups = (k.K + 63) >> 6, steps = 2 * groups;
-    const bool live = t16 * 16 < k.N;
+    const bool live = t16 * 16 < k.N;  // (NN = 2: both blocks lie in one 32-row tile, which is stored whole)
 
-    mf_f32x4 acc[NT];
+    mf_f32x4 acc[NN][NT];
 #pragma unroll
-    for (int t = 0; t < NT; ++t) acc[t] = (mf_f32x4){0.0f, 0.0f, 0.0f, 0.0f};
+    for (int n = 0; n < NN; ++n)
+#pragma unroll
+        for (int t = 0; t < NT; ++t) acc[n][t] = (mf_f32x4){0.0f, 0.0f, 0.0f, 0.0f};
     if (live) {
         const char *wp = k.w + (size_t)(t16 >> 1) * groups * 4096 + ((kq >> 1) * 1024 + ((kq & 1) * 32 + (t16 & 1) * 16 + c) * 16);
         const u16 *xp[NT];
@@ -108,26 +122,29 @@ __global__ void __launch_bounds__(512) k_rows_w16m(const RowsArgs a) {
             const int xr = k.rows ? k.rows[i] : k.row0 + i;
             xp[t] = (const u16 *)k.x + (size_t)xr * k.ldx + k.xoff + 8 * kq;
         }
-        auto fetch = [&](int s, mf_u32x4(&wv)[U], mf_u32x4(&xv)[U][NT]) {
+        auto fetch = [&](int s, mf_u32x4(&wv)[U][NN], mf_u32x4(&xv)[U][NT]) {
 #pragma unroll
             for (int u = 0; u < U; ++u) {
                 const int ss = s + u * KW, cl = ss < steps ? ss : steps - 1;
-                wv[u] = __builtin_nontemporal_load((const mf_u32x4 *)(wp + (size_t)cl * 2048));
+#pragma unroll
+                for (int n = 0; n < NN; ++n) wv[u][n] = __builtin_nontemporal_load((const mf_u32x4 *)(wp + (size_t)cl * 2048 + n * 256));
 #pragma unroll
                 for (int t = 0; t < NT; ++t) xv[u][t] = *(const mf_u32x4 *)(xp[t] + 32 * cl);
             }
         };
-        auto multiply = [&](int s, const mf_u32x4(&wv)[U], const mf_u32x4(&xv)[U][NT]) {
+        auto multiply = [&](int s, const mf_u32x4(&wv)[U][NN], const mf_u32x4(&xv)[U][NT]) {
 #pragma unroll
-            for (int u = 0; u < U; ++u) {
-                mf_u32x4 w = wv[u];
-                if (s + u * KW >= steps) w = (mf_u32x4){0u, 0u, 0u, 0u};
+            for (int u = 0; u < U; ++u)
 #pragma unroll
-                for (int t = 0; t < NT; ++t)
-                    acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(mf_bf16x8, w), __builtin_bit_cast(mf_bf16x8, xv[u][t]), acc[t], 0, 0, 0);
-            }
+                for (int n = 0; n < NN; ++n) {
+                    mf_u32x4 w = wv[u][n];
+                    if (s + u * KW >= steps) w = (mf_u32x4){0u, 0u, 0u, 0u};
+#pragma unroll
+                    for (int t = 0; t < NT; ++t)
+                        acc[n][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(mf_bf16x8, w), __builtin_bit_cast(mf_bf16x8, xv[u][t]), acc[n][t], 0, 0, 0);
+                }
         };
-        mf_u32x4 w0[U], w1[U], x0[U][NT], x1[U][NT];
+        mf_u32x4 w0[U][NN], w1[U][NN], x0[U][NT], x1[U][NT];
         fetch(wk, w0, x0);
         for (int s = wk; s < steps; s += 2 * U * KW) {
             fetch(s + U * KW, w1, x1);
@@ -138,20 +155,22 @@ __global__ void __launch_bounds__(512) k_rows_w16m(const RowsArgs a) {
     }
     // lane (kq, c) holds features 4 kq .. + 3 of row c
 #pragma unroll
-    for (int t = 0; t < NT; ++t) *(mf_f32x4 *)(s_red + ((wave * NT + t) * 16 + c) * ST + 4 * kq) = acc[t];
+    for (int n = 0; n < NN; ++n)
+#pragma unroll
+        for (int t = 0; t < NT; ++t) *(mf_f32x4 *)(s_red + (((wave * NN + n) * NT + t) * 16 + c) * ST + 4 * kq) = acc[n][t];
     __syncthreads();
-    for (int id = threadIdx.x; id < NW * NT * 256; id += 512) {
-        const int nl = id & 15, ml = (id >> 4) % (16 * NT), w = id / (256 * NT);
-        const int n = ((int)blockIdx.x * NW + w) * 16 + nl, m = i0 + ml;
+    for (int id = threadIdx.x; id < NW * NN * NT * 256; id += 512) {
+        const int nl = id & 15, ml = (id >> 4) % (16 * NT), wn2 = id / (256 * NT), w = wn2 / NN, nn = wn2 % NN;
+        const int n = ((int)blockIdx.x * NW * NN + wn2) * 16 + nl, m = i0 + ml;
         if (n >= k.N || m >= k.count) continue;
         if (a.epi == ROWS_SILU_MUL && (nl & 1)) continue;
-        const float *r = s_red + ((w * KW * NT + (ml >> 4)) * 16 + (ml & 15)) * ST + nl;
+        const float *r = s_red + (((w * KW * NN + nn) * NT + (ml >> 4)) * 16 + (ml & 15)) * ST + nl;
         float v = 0.0f, p = 0.0f;
 #pragma unroll
-        for (int q = 0; q < KW; ++q) v += r[q * NT * 16 * ST];
+        for (int q = 0; q < KW; ++q) v += r[q * NN * NT * 16 * ST];
         if (a.epi == ROWS_SILU_MUL)
 #pragma unroll
-            for (int q = 0; q < KW; ++q) p += r[q * NT * 16 * ST + 1];
+            for (int q = 0; q < KW; ++q) p += r[q * NN * NT * 16 * ST + 1];
         rows_finish<ElemBF16>(a, k, m, n, v, p);
     }
 }
@@ -159,6 +178,7 @@ __global__ void __launch_bounds__(512) k_rows_w16m(const RowsArgs a) {
 // fp32: one output per thread, 16 features x 16 rows per workgroup, both operands through LDS
 __global__ void __launch_bounds__(256) k_rows_f32(const RowsArgs a) {
     __shared__ float s_w[16][65], s_x[16][65], s_v[16][17];
+    if (rows_append<ElemF32, 256>(a, s_v[0])) return;
     RowsWork k;
     if (!rows_select(a, k)) return;
     const int i0 = blockIdx.z * 16, n0 = blockIdx.x * 16;
@@ -186,17 +206,18 @@ __global__ void __launch_bounds__(256) k_rows_f32(const RowsArgs a) {
     if (n < k.N && m < k.count) rows_finish<ElemF32>(a, k, m, n, acc, s_v[tm][tn < 15 ? tn + 1 : 15]);
 }
 
-template <int NT>
+template <int NT, int NN>
 int rows_go(const RowsArgs &a, int n_max, int k_max, int batches, hipStream_t st) {
-    const int steps = 2 * ((k_max + 63) / 64), tiles = (n_max + 15) / 16, z = (a.M + 16 * NT - 1) / (16 * NT);  // (grouped: most experts have few rows, their later z leave at once)
+    const int steps = 2 * ((k_max + 63) / 64), tiles = (n_max + 16 * NN - 1) / (16 * NN);
+    const int z = (a.M + 16 * NT - 1) / (16 * NT);  // (grouped: most experts have few rows, their later z leave at once)
     // waves along K: enough steps for each, and enough workgroups for the chip
     int kw = steps >= 32 ? 8 : steps >= 16 ? 4 : steps >= 8 ? 2 : 1;
     while (kw < 8 && steps >= 2 * kw && (size_t)((tiles + 8 / kw - 1) / (8 / kw)) * batches * z < 256) kw *= 2;
-    const dim3 grid((unsigned)((tiles + 8 / kw - 1) / (8 / kw)), (unsigned)batches, (unsigned)z);
-    if (kw == 8) hipLaunchKernelGGL((k_rows_w16m<NT, 8>), grid, dim3(512), 0, st, a);
-    else if (kw == 4) hipLaunchKernelGGL((k_rows_w16m<NT, 4>), grid, dim3(512), 0, st, a);
-    else if (kw == 2) hipLaunchKernelGGL((k_rows_w16m<NT, 2>), grid, dim3(512), 0, st, a);
-    else hipLaunchKernelGGL((k_rows_w16m<NT, 1>), grid, dim3(512), 0, st, a);
+    const dim3 grid((unsigned)((tiles + 8 / kw - 1) / (8 / kw)), (unsigned)(batches + (a.append.M > 0 ? 1 : 0)), (unsigned)z);
+    if (kw == 8) hipLaunchKernelGGL((k_rows_w16m<NT, 8, NN>), grid, dim3(512), 0, st, a);
+    else if (kw == 4) hipLaunchKernelGGL((k_rows_w16m<NT, 4, NN>), grid, dim3(512), 0, st, a);
+    else if (kw == 2) hipLaunchKernelGGL((k_rows_w16m<NT, 2, NN>), grid, dim3(512), 0, st, a);
+    else hipLaunchKernelGGL((k_rows_w16m<NT, 1, NN>), grid, dim3(512), 0, st, a);
     PIE_LAUNCH_CHECK();
     return PIE_OK;
 }
@@ -217,18 +238,19 @@ size_t rows_weight_bytes(int dtype, int N, int K) {
 int rows_gemm_launch(int dtype, const RowsArgs &a, int batches, hipStream_t st) {
     if (a.M <= 0 || batches <= 0) return PIE_OK;
     PIE_REQUIRE(a.m.N > 0 && a.m.K > 0, PIE_E_SHAPE, "row-wise Linear: empty matrix");
-    PIE_REQUIRE(batches <= 65535, PIE_E_SHAPE, "row-wise Linear: too many batches");
+    PIE_REQUIRE(batches < 65535 && (a.append.M <= 0 || !(a.shared.w || a.active)), PIE_E_SHAPE, "row-wise Linear: too many batches");
     const int n_max = a.shared.w && a.shared.N > a.m.N ? a.shared.N : a.m.N, k_max = a.shared.w && a.shared.K > a.m.K ? a.shared.K : a.m.K;
     if (dtype == PIE_F32) {
-        const dim3 grid((unsigned)((n_max + 15) / 16), (unsigned)batches, (unsigned)((a.M + 15) / 16));
+        const dim3 grid((unsigned)((n_max + 15) / 16), (unsigned)(batches + (a.append.M > 0 ? 1 : 0)), (unsigned)((a.M + 15) / 16));
         hipLaunchKernelGGL(k_rows_f32, grid, dim3(256), 0, st, a);
         PIE_LAUNCH_CHECK();
         return PIE_OK;
     }
     PIE_REQUIRE(a.m.ldx % 8 == 0 && a.x_batch % 8 == 0 && pie_aligned(a.m.x, 16) && pie_aligned(a.m.w, 16), PIE_E_ALIGN, "row-wise Linear: 16-byte alignment required");
-    if (a.M <= 16 || a.active) return rows_go<1>(a, n_max, k_max, batches, st);
-    if (a.M <= 32) return rows_go<2>(a, n_max, k_max, batches, st);
-    return rows_go<4>(a, n_max, k_max, batches, st);
+    if (a.M <= 16 || a.active) return rows_go<1, 1>(a, n_max, k_max, batches, st);
+    const bool wide = batches == 1 && n_max >= 32 * 140;  // two feature blocks per wave where half as many workgroups still fill most of the chip
+    if (a.M <= 32) return wide ? rows_go<2, 2>(a, n_max, k_max, batches, st) : rows_go<2, 1>(a, n_max, k_max, batches, st);
+    return wide ? rows_go<4, 2>(a, n_max, k_max, batches, st) : rows_go<4, 1>(a, n_max, k_max, batches, st);
 }
 
 extern "C" {

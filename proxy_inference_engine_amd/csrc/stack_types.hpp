@@ -39,6 +39,47 @@ __device__ __forceinline__ float fast_tanh(float z) {
 }
 __device__ __forceinline__ float point_norm(const PointNorm &n, int i, float x) { return fmaf(fast_tanh(n.alpha * x), n.w[i], n.b[i]); }
 
+// four columns i .. i + 3 (i a multiple of 4; w and b hold a multiple of 4 elements)
+__device__ __forceinline__ float4 point_norm4(const PointNorm &n, int i, float4 x) {
+    const float4 w = *(const float4 *)(n.w + i), b = *(const float4 *)(n.b + i);
+    return make_float4(fmaf(fast_tanh(n.alpha * x.x), w.x, b.x), fmaf(fast_tanh(n.alpha * x.y), w.y, b.y), fmaf(fast_tanh(n.alpha * x.z), w.z, b.z),
+                       fmaf(fast_tanh(n.alpha * x.w), w.w, b.w));
+}
+
+// ---------------------------------------------------------------- latent append
+// c_raw [M][ldc], fp32 or (raw16) bf16 -> RMS norm with weight w -> the row of its page
+struct LatentAppend {
+    const void *c_raw;
+    bool raw16;
+    int ldc;
+    const float *w;
+    float eps;
+    int M, R, ldr;
+    const int *pos, *row_seq, *table;
+    int table_width, n_pages, n_seqs;
+    void *slab;
+};
+template <class E, class X, int THREADS>
+__device__ __forceinline__ void latent_append_row(const LatentAppend &a, int m, float *red) {  // red: THREADS / 64 floats of LDS
+    const typename X::type *x = (const typename X::type *)a.c_raw + (size_t)m * a.ldc;
+    const int t = a.pos[m], j = min(t / PAGE_TOKENS, a.table_width - 1);
+    float ss = 0.0f;
+    for (int r = threadIdx.x; r < a.R; r += THREADS) {
+        const float v = X::load(x + r);
+        ss = fmaf(v, v, ss);
+    }
+    ss = wave_sum(ss);
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
+    const size_t page = min((unsigned)a.table[(size_t)min(a.row_seq[m], a.n_seqs - 1) * a.table_width + j], (unsigned)a.n_pages - 1u);
+    __syncthreads();
+    float sum = red[0];
+#pragma unroll
+    for (int i = 1; i < THREADS / 64; ++i) sum += red[i];
+    const float inv = 1.0f / sqrtf(sum / (float)a.R + a.eps);
+    typename E::type *dst = (typename E::type *)a.slab + (page * PAGE_TOKENS + (t & (PAGE_TOKENS - 1))) * a.ldr;
+    for (int r = threadIdx.x; r < a.R; r += THREADS) dst[r] = E::pack(X::load(x + r) * inv * a.w[r]);
+}
+
 // ---------------------------------------------------------------- the row-wise Linear
 enum RowsEpi {
     ROWS_STORE = 0,      // y[m][n] = T(v)
@@ -79,6 +120,7 @@ struct RowsArgs {
     PointNorm post, next;
     void *h;               // [M][ldh]
     int ldh;
+    LatentAppend append;   // append.M > 0: the last blockIdx.y does this instead (it needs the same input and would otherwise be a launch of its own)
 };
 // batches: blockIdx.y extent (1 for a plain Linear; heads; active experts (+ 1 with a shared expert))
 int rows_gemm_launch(int dtype, const RowsArgs &a, int batches, hipStream_t st);
@@ -86,7 +128,7 @@ int rows_gemm_launch(int dtype, const RowsArgs &a, int batches, hipStream_t st);
 size_t rows_weight_bytes(int dtype, int N, int K);
 
 // ---------------------------------------------------------------- latent attention
-// A pass holds runs of consecutive rows, one run per sequence; a workgroup takes 16, 32 or 64 (token, head) pairs of ONE run.
+// A pass holds runs of consecutive rows, one run per sequence; a workgroup takes 32 (token, head) pairs of ONE run.
 struct RowRun {
     int row0, n_rows, seq, pos0;  // seq: row of the block table; pos0: position of row0 (single rows: not used, may be 0)
 };
@@ -97,8 +139,7 @@ struct LatentAttnArgs {
     int table_width, n_pages, n_seqs;
     const int *pos;        // [M]
     const RowRun *runs;
-    int n_runs, n_tiles;   // n_tiles = sum over the runs of ceil(n_rows * H / pairs)
-    int pairs;             // (token, head) pairs per workgroup: latent_attn_pairs()
+    int n_runs, n_tiles;   // n_tiles = sum over the runs of latent_attn_tiles()
     bool single;           // every run is one row (a decode step): tile -> run without a search
     const int *row_seq;    // [M]
     int H, R, ldr, M;
@@ -109,11 +150,9 @@ struct LatentAttnArgs {
     void *out;             // [M][H][ldr] T: softmax-weighted latents
 };
 int latent_attn_launch(int dtype, const LatentAttnArgs &a, hipStream_t st);
-int latent_attn_pairs(int H, int R, bool single);  // single decoded tokens of few heads take smaller tiles and split the keys over the waves
+int latent_attn_tiles(int n_rows, int H);
 size_t latent_attn_ws_floats(int M, int H, int R, int splits);
-// c_raw [M][ldc], fp32 or (raw16) bf16 -> RMS norm with weight w -> the row of its page
-int latent_append_launch(int dtype, const void *c_raw, bool raw16, int ldc, const float *w, float eps, int M, int R, int ldr, const int *pos, const int *row_seq,
-                         const int *table, int table_width, int n_pages, int n_seqs, void *slab, hipStream_t st);
+int latent_append_launch(int dtype, const LatentAppend &a, hipStream_t st);
 
 // ---------------------------------------------------------------- attention of long runs, keys and values spelled out (window_attn.hip)
 constexpr int WINDOW_ATTN_MAX_DIM = 256;

@@ -86,8 +86,8 @@ struct W16Args {
 // one column tile, then of the column tile 8 further -- they stream the SAME weight tiles at the same time, so each XCD's L2 fetches a
 // weight tile once per pass (16-bit weights are 4x the int4 kernel's bytes: re-read per row tile they would be 3.7 GB of HBM traffic for
 // gate|up at 4096 rows); grid.y = K splits.
-// GRP: many matrices of one shape, each with its own rows (a mixture's experts).  An XCD takes every eighth row tile with all its column tiles, so the
-// x rows and the expert's weight tiles meet in one L2.
+// GRP: many matrices of one shape, each with its own rows (a mixture's experts).  An XCD takes every eighth block of bm row tiles -- an
+// expert's tiles start at a block -- with all its column tiles, row tile fastest: a block's tiles stream the same weight tiles through one L2 at the same time.
 template <class T, int MB, int SW, int ACT, bool GRP = false>
 __global__ void __launch_bounds__(256) k_w16l_gemm(const W16Args a) {
     constexpr bool SWIGLU = ACT == MFMA_ACT_SWIGLU;
@@ -107,8 +107,8 @@ __global__ void __launch_bounds__(256) k_w16l_gemm(const W16Args a) {
     int m0, rows, ncol;
     const char *weights = a.w16m;
     if constexpr (GRP) {
-        const int mt = (sq / a.tn) * 8 + xcd;
-        ncol = sq % a.tn;
+        const int in = sq % (a.bm * a.tn), mt = a.bm * ((sq / (a.bm * a.tn)) * 8 + xcd) + in % a.bm;
+        ncol = in / a.bm;
         if (mt >= a.tm) return;
         const int4 tile = a.tiles[mt];
         m0 = __builtin_amdgcn_readfirstlane(tile.y), rows = __builtin_amdgcn_readfirstlane(tile.z);

@@ -99,7 +99,7 @@ class Model(LayerStackModel):
             return t
 
         def norm(name: str) -> tuple:
-            return (float(get(name + ".alpha").float().item()), get(name, W).float().contiguous(), get(name + ".b", W).float().contiguous())
+            return (float(get(name + ".alpha").float().item()), _pad(get(name, W).float()[None], 1, _up8(W))[0], _pad(get(name + ".b", W).float()[None], 1, _up8(W))[0])
 
         def pack(w: torch.Tensor) -> torch.Tensor:
             return pack_linear(w, dtype)
@@ -144,7 +144,7 @@ class Model(LayerStackModel):
                                "w_gate_up": torch.cat([e[0] for e in experts]), "w_expert_down": torch.cat([e[1] for e in experts])}
                     if ff.shared is not None:
                         fields["s_gate_up"], fields["s_down"] = gated(p + "mlp.shared.", ff.shared.ff)
-                        fields |= {"shared_size": _up8(ff.shared.ff), "shared_gate": get(p + "mlp.shared.sg", 1, W).float().reshape(-1).contiguous()}
+                        fields |= {"shared_size": _up8(ff.shared.ff), "shared_gate": _pad(get(p + "mlp.shared.sg", 1, W).float(), 1, _up8(W))[0]}
                 else:
                     raise ValueError(f"layer {i}: unknown feed-forward {ff.kind!r}")
             layers.append(fields)
