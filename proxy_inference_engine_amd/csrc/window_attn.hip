@@ -32,7 +32,7 @@ __global__ void __launch_bounds__(64) k_latent_gather(const RowRun *runs, int n_
 }
 
 template <int DM>  // dim and vdim up to DM (32, 64, 128, 256)
-__global__ void __launch_bounds__(256) k_window_attn(const WindowAttnArgs a) {
+__global__ void __launch_bounds__(256, DM <= 128 ? 2 : 1) k_window_attn(const WindowAttnArgs a) {
     constexpr int CH = DM / 8, KS = DM / 16, DT = DM / 32, CPT = (32 * CH + 255) / 256;
     __shared__ __attribute__((aligned(16))) char k_lds[32 * 2 * DM], v_lds[32 * 2 * DM];
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
