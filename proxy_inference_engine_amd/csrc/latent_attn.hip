@@ -219,34 +219,16 @@ __global__ void __launch_bounds__(256, RC <= 8 ? 2 : 1) k_latent_attn(const Late
     }
 }
 
-// merges the key splits of one (token, head) pair: every wave weighs all splits (at most 64: one per lane), then streams the partial sums, eight in flight
-__global__ void __launch_bounds__(128) k_latent_combine(const LatentAttnArgs a) {
+// merges the key splits of one (token, head) pair
+__global__ void __launch_bounds__(128) k_latent_combine(const LatentMerge a, u16 *out) {
     __shared__ float s_f[64];
-    const size_t pr = blockIdx.x, MH = (size_t)a.M * a.H;
-    const int lane = threadIdx.x & 63;
-    const float2 ml = lane < a.splits ? *(const float2 *)(a.ws + (size_t)a.splits * MH * a.ldr + (lane * MH + pr) * 2) : make_float2(LA_NEG, 0.0f);
-    const float m = wave_max(ml.y > 0.0f ? ml.x : LA_NEG);
-    const float f = ml.y > 0.0f ? __builtin_amdgcn_exp2f(ml.x - m) : 0.0f;  // an empty split wrote no sums and has no weight
-    const float l = wave_sum(ml.y * f);
-    if (threadIdx.x < 64) s_f[lane] = f / l;
+    const size_t pr = blockIdx.x;
+    const float f = latent_split_weight(a, pr, threadIdx.x & 63);
+    if (threadIdx.x < 64) s_f[threadIdx.x] = f;
     __syncthreads();
     for (int r = threadIdx.x * 4; r < a.ldr; r += 512) {
-        la_f32x4 acc = {0.0f, 0.0f, 0.0f, 0.0f};
-        for (int s0 = 0; s0 < a.splits; s0 += 8) {
-            la_f32x4 v[8];
-            float w[8];
-#pragma unroll
-            for (int u = 0; u < 8; ++u) {
-                const int s = min(s0 + u, a.splits - 1);
-                w[u] = s0 + u < a.splits ? s_f[s] : 0.0f;
-                v[u] = *(const la_f32x4 *)(a.ws + (s * MH + pr) * a.ldr + r);
-            }
-#pragma unroll
-            for (int u = 0; u < 8; ++u)
-#pragma unroll
-                for (int i = 0; i < 4; ++i) acc[i] = w[u] > 0.0f ? fmaf(w[u], v[u][i], acc[i]) : acc[i];
-        }
-        *(uint2 *)((u16 *)a.out + pr * a.ldr + r) = make_uint2(pack2<BF16>(acc[0], acc[1]), pack2<BF16>(acc[2], acc[3]));
+        const float4 v = latent_merge4(a, pr, r, [&](int s) { return s_f[s]; });
+        *(uint2 *)(out + pr * a.ldr + r) = make_uint2(pack2<BF16>(v.x, v.y), pack2<BF16>(v.z, v.w));
     }
 }
 
@@ -317,8 +299,9 @@ int latent_attn_launch(int dtype, const LatentAttnArgs &a, hipStream_t st) {
     else LA_GO(16);
 #undef LA_GO
     PIE_LAUNCH_CHECK();
-    if (a.splits > 1) {
-        hipLaunchKernelGGL(k_latent_combine, dim3((unsigned)(a.M * a.H)), dim3(128), 0, st, a);
+    if (a.splits > 1 && a.combine) {
+        const LatentMerge m = {a.ws, a.splits, a.M, a.H, a.ldr};
+        hipLaunchKernelGGL(k_latent_combine, dim3((unsigned)(a.M * a.H)), dim3(128), 0, st, m, (u16 *)a.out);
         PIE_LAUNCH_CHECK();
     }
     return PIE_OK;

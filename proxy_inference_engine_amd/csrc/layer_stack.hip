@@ -4,8 +4,8 @@
 // Launches per layer (every norm is element-wise and rides in the epilogue of the kernel that produces its input):
 //   [q | latent down]     Linear                                      (rows_gemm.hip)
 //   q -> latent space     Linear per head; beside it the latents' RMS norm and their append to the pages
-//   attention over the latents [+ merge of the key splits]            (latent_attn.hip)
-//   latents -> values     Linear per head
+//   attention over the latents                                        (latent_attn.hip)
+//   latents -> values     Linear per head, merging the key splits on the way in (more than a few rows: merged by a launch of its own)
 //   output projection     Linear; epilogue: x += post1(y), h = pre2(x)
 //   dense: up (relu^2), down; epilogue: x += post2(y), h = next layer's pre1(x)
 //   experts: gate|up (silu * up) and down over the active experts and the shared one, then the weighted sum with the same epilogue
@@ -507,10 +507,13 @@ void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const PointNorm &ne
         t.runs = (const RowRun *)b.runs, t.n_runs = runs, t.single = runs == M, t.row_seq = b.row_seq;
         t.n_tiles = stack_tiles(b.runs_host, runs, H);
         t.H = H, t.R = L.rank, t.ldr = R8, t.M = M, t.window = L.window, t.scale = L.scale, t.splits = plan_splits(b, L, t.n_tiles), t.ws = s->attn_ws.p, t.out = s->oc.p;
-        if (!p.rc) p.rc = latent_attn_launch(dt, t, p.st), p.launches += t.splits > 1 ? 2 : 1;
+        const bool merge = t.splits > 1 && M <= MERGE_ROWS && R8 <= MERGE_LDR && dt == PIE_BF16 && L.rank <= 1024;  // few rows: the next launch merges the key splits itself
+        t.combine = !merge;
+        if (!p.rc) p.rc = latent_attn_launch(dt, t, p.st), p.launches += t.splits > 1 && !merge ? 2 : 1;
         RowsArgs v = {};
         v.m = {(const char *)L.w_uv, L.vdim, L.rank, s->oc.p, H * R8, s->o.p, LO};
         v.M = M, v.epi = ROWS_STORE, v.w_batch = rows_weight_bytes(dt, L.vdim, L.rank), v.x_batch = R8, v.y_batch = V8;
+        if (merge) v.merge = {s->attn_ws.p, t.splits, M, H, R8};
         p.linear(v, H);
     }
     if (spell && !p.rc) {

@@ -88,13 +88,30 @@ __device__ __forceinline__ bool rows_append(const RowsArgs &a, float *red) {
     return true;
 }
 
-// NT: blocks of 16 rows of x; KW: waves along K; NN: blocks of 16 features per wave (two share the x operands)
-template <int NT, int KW, int NN>
+// NT: blocks of 16 rows of x; KW: waves along K; NN: blocks of 16 features per wave (two share the x operands); MERGE: x = the merged key splits of head
+// blockIdx.y (RowsArgs::merge), put together in LDS by every workgroup of the head
+template <int NT, int KW, int NN, bool MERGE = false>
 __global__ void __launch_bounds__(512) k_rows_w16m(const RowsArgs a) {
     constexpr int NW = 8 / KW, U = NT >= 4 ? 2 : 4;
     constexpr int ST = 20;  // floats per (row, 16 features) line of the reduction image
     __shared__ __attribute__((aligned(16))) float s_red[8 * NN * NT * 16 * ST];
     if (rows_append<ElemBF16, 512>(a, s_red)) return;
+    __shared__ __attribute__((aligned(16))) u16 s_x[MERGE ? MERGE_ROWS * (MERGE_LDR + 64) : 8];
+    const int ldx_lds = a.merge.ldr + 64;
+    if constexpr (MERGE) {
+        __shared__ float s_f[MERGE_ROWS][64];
+        const int H = a.merge.H, M = a.merge.M, w = threadIdx.x >> 6;
+        if (w < M) s_f[w][threadIdx.x & 63] = latent_split_weight(a.merge, (size_t)w * H + blockIdx.y, threadIdx.x & 63);
+        __syncthreads();
+        const int quads = ldx_lds / 4;
+        for (int i = threadIdx.x; i < M * quads; i += 512) {
+            const int m = i / quads, r = i % quads * 4;
+            float4 v = make_float4(0, 0, 0, 0);  // (columns past the latent meet zero weights: zeros)
+            if (r < a.merge.ldr) v = latent_merge4(a.merge, (size_t)m * H + blockIdx.y, r, [&](int s) { return s_f[m][s]; });
+            *(uint2 *)(s_x + m * ldx_lds + r) = make_uint2(pack2<BF16>(v.x, v.y), pack2<BF16>(v.z, v.w));
+        }
+        __syncthreads();
+    }
     RowsWork k;
     if (!rows_select(a, k)) return;
     const int i0 = blockIdx.z * 16 * NT;
@@ -120,7 +137,7 @@ __global__ void __launch_bounds__(512) k_rows_w16m(const RowsArgs a) {
             int i = i0 + 16 * t + c;
             i = i < k.count ? i : k.count - 1;  // rows past the end repeat the last one (never stored)
             const int xr = k.rows ? k.rows[i] : k.row0 + i;
-            xp[t] = (const u16 *)k.x + (size_t)xr * k.ldx + k.xoff + 8 * kq;
+            xp[t] = MERGE ? s_x + xr * ldx_lds + 8 * kq : (const u16 *)k.x + (size_t)xr * k.ldx + k.xoff + 8 * kq;
         }
         auto fetch = [&](int s, mf_u32x4(&wv)[U][NN], mf_u32x4(&xv)[U][NT]) {
 #pragma unroll
@@ -214,7 +231,12 @@ int rows_go(const RowsArgs &a, int n_max, int k_max, int batches, hipStream_t st
     int kw = steps >= 32 ? 8 : steps >= 16 ? 4 : steps >= 8 ? 2 : 1;
     while (kw < 8 && steps >= 2 * kw && (size_t)((tiles + 8 / kw - 1) / (8 / kw)) * batches * z < 256) kw *= 2;
     const dim3 grid((unsigned)((tiles + 8 / kw - 1) / (8 / kw)), (unsigned)(batches + (a.append.M > 0 ? 1 : 0)), (unsigned)z);
-    if (kw == 8) hipLaunchKernelGGL((k_rows_w16m<NT, 8, NN>), grid, dim3(512), 0, st, a);
+    if (a.merge.splits > 0) {
+        if (kw == 8) hipLaunchKernelGGL((k_rows_w16m<1, 8, 1, true>), grid, dim3(512), 0, st, a);
+        else if (kw == 4) hipLaunchKernelGGL((k_rows_w16m<1, 4, 1, true>), grid, dim3(512), 0, st, a);
+        else if (kw == 2) hipLaunchKernelGGL((k_rows_w16m<1, 2, 1, true>), grid, dim3(512), 0, st, a);
+        else hipLaunchKernelGGL((k_rows_w16m<1, 1, 1, true>), grid, dim3(512), 0, st, a);
+    } else if (kw == 8) hipLaunchKernelGGL((k_rows_w16m<NT, 8, NN>), grid, dim3(512), 0, st, a);
     else if (kw == 4) hipLaunchKernelGGL((k_rows_w16m<NT, 4, NN>), grid, dim3(512), 0, st, a);
     else if (kw == 2) hipLaunchKernelGGL((k_rows_w16m<NT, 2, NN>), grid, dim3(512), 0, st, a);
     else hipLaunchKernelGGL((k_rows_w16m<NT, 1, NN>), grid, dim3(512), 0, st, a);
@@ -246,6 +268,8 @@ int rows_gemm_launch(int dtype, const RowsArgs &a, int batches, hipStream_t st) 
         PIE_LAUNCH_CHECK();
         return PIE_OK;
     }
+    PIE_REQUIRE(a.merge.splits <= 64 && (a.merge.splits <= 0 || (a.merge.M == a.M && a.M <= MERGE_ROWS && a.merge.ldr <= MERGE_LDR && a.merge.ldr % 8 == 0 && !a.active && !a.rows)), PIE_E_SHAPE,
+                "row-wise Linear: too many rows or columns to merge key splits on the way in");
     PIE_REQUIRE(a.m.ldx % 8 == 0 && a.x_batch % 8 == 0 && pie_aligned(a.m.x, 16) && pie_aligned(a.m.w, 16), PIE_E_ALIGN, "row-wise Linear: 16-byte alignment required");
     if (a.M <= 16 || a.active) return rows_go<1, 1>(a, n_max, k_max, batches, st);
     const bool wide = batches == 1 && n_max >= 32 * 140;  // two feature blocks per wave where half as many workgroups still fill most of the chip

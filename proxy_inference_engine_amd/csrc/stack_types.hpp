@@ -80,6 +80,42 @@ __device__ __forceinline__ void latent_append_row(const LatentAppend &a, int m, 
     for (int r = threadIdx.x; r < a.R; r += THREADS) dst[r] = E::pack(X::load(x + r) * inv * a.w[r]);
 }
 
+// ---------------------------------------------------------------- the attention's key splits
+// ws: sums [splits][M * H][ldr] fp32, then (maximum, sum of weights) [splits][M * H][2]; a split that saw no key has weight sum 0 and no sums
+constexpr int MERGE_ROWS = 4, MERGE_LDR = 1024;
+struct LatentMerge {
+    const float *ws;
+    int splits, M, H, ldr;
+};
+// lane s: what split s of pair pr counts in the merged result (base 2 exponents; at most 64 splits)
+__device__ __forceinline__ float latent_split_weight(const LatentMerge &a, size_t pr, int lane) {
+    const size_t MH = (size_t)a.M * a.H;
+    const float2 ml = lane < a.splits ? *(const float2 *)(a.ws + (size_t)a.splits * MH * a.ldr + (lane * MH + pr) * 2) : make_float2(-1e30f, 0.0f);
+    const float m = wave_max(ml.y > 0.0f ? ml.x : -1e30f);
+    const float f = ml.y > 0.0f ? __builtin_amdgcn_exp2f(ml.x - m) : 0.0f;
+    return f / wave_sum(ml.y * f);
+}
+// columns r .. r + 3 of the merged sums of pair pr, eight splits in flight; weight(s): a wave-uniform or per-thread read of split s's weight
+template <class F>
+__device__ __forceinline__ float4 latent_merge4(const LatentMerge &a, size_t pr, int r, F &&weight) {
+    const size_t MH = (size_t)a.M * a.H;
+    float4 acc = make_float4(0, 0, 0, 0);
+    for (int s0 = 0; s0 < a.splits; s0 += 8) {
+        float4 v[8];
+        float w[8];
+#pragma unroll
+        for (int u = 0; u < 8; ++u) {
+            const int s = min(s0 + u, a.splits - 1);
+            w[u] = s0 + u < a.splits ? weight(s) : 0.0f;
+            v[u] = *(const float4 *)(a.ws + (s * MH + pr) * a.ldr + r);
+        }
+#pragma unroll
+        for (int u = 0; u < 8; ++u)
+            if (w[u] > 0.0f) acc.x = fmaf(w[u], v[u].x, acc.x), acc.y = fmaf(w[u], v[u].y, acc.y), acc.z = fmaf(w[u], v[u].z, acc.z), acc.w = fmaf(w[u], v[u].w, acc.w);
+    }
+    return acc;
+}
+
 // ---------------------------------------------------------------- the row-wise Linear
 enum RowsEpi {
     ROWS_STORE = 0,      // y[m][n] = T(v)
@@ -120,6 +156,7 @@ struct RowsArgs {
     PointNorm post, next;
     void *h;               // [M][ldh]
     int ldh;
+    LatentMerge merge;     // merge.splits > 0 (batched over heads, bf16, at most MERGE_ROWS rows): x is merged from the attention's key splits on the way in
     LatentAppend append;   // append.M > 0: the last blockIdx.y does this instead (it needs the same input and would otherwise be a launch of its own)
 };
 // batches: blockIdx.y extent (1 for a plain Linear; heads; active experts (+ 1 with a shared expert))
@@ -145,8 +182,9 @@ struct LatentAttnArgs {
     int H, R, ldr, M;
     int window;            // keys j with 0 <= i - j < window; <= 0: no limit
     float scale;
-    int splits;            // > 1: fp32 partials in ws, merged by the combine launch
-    float *ws;             // [splits][M * H] x (R + 2): see latent_attn.hip
+    int splits;            // > 1: fp32 partials in ws, merged by the combine launch (combine = false: left to the consumer)
+    bool combine;
+    float *ws;             // see LatentMerge
     void *out;             // [M][H][ldr] T: softmax-weighted latents
 };
 int latent_attn_launch(int dtype, const LatentAttnArgs &a, hipStream_t st);

@@ -26,7 +26,8 @@ def pack_linear(w: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
     n = lib.pie_stack_weight_bytes(code, mats.shape[1], mats.shape[2])
     out = torch.empty(mats.shape[0] * n, dtype=torch.uint8, device=w.device)
     for i in range(mats.shape[0]):
-        _ffi.check(lib.pie_stack_pack_weight(mats[i].contiguous().data_ptr(), mats.shape[1], mats.shape[2], code, out.data_ptr() + i * n, _ffi.stream()))
+        mat = mats[i] if mats[i].data_ptr() % 16 == 0 else mats[i].clone()  # (a matrix of odd size starts the next one unaligned)
+        _ffi.check(lib.pie_stack_pack_weight(mat.data_ptr(), mats.shape[1], mats.shape[2], code, out.data_ptr() + i * n, _ffi.stream()))
     return out
 
 

@@ -39,6 +39,8 @@ CONFIGS = {
     "experts_only": tu.config([(tu.latent(heads=1, window=1), tu.moe(shared=None))]),
     "experts_shared": tu.config([(tu.latent(heads=1, window=1), tu.moe(ff=30, experts=7, top=3, shared=50))], width=88, vocab=333),
     "mixed": tu.config(MIXED, width=112, vocab=251, logit_scale=0.7),
+    "odd_sizes": tu.config([(tu.latent(heads=3, dim=9, vdim=5, rank=7, window=11), tu.moe(ff=3, experts=1, top=1, shared=5)),
+                            (tu.latent(heads=2, dim=1, vdim=1, rank=3, window=3), tu.dense(13))], width=21, vocab=53, logit_scale=2.5, eps=1e-3),
     "many_heads": tu.config([(tu.latent(heads=70, dim=8, vdim=8, rank=64, window=50), tu.dense())], width=128),
 }
 

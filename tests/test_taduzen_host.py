@@ -82,3 +82,32 @@ def test_oracle_absorbed_form_agrees():
         ql = q[:, a] @ w["l0.mix.uk"].reshape(2, 6, 14)[a]
         out.append(orc.softmax_rows(ql @ c.T * m["scale"], orc.visible(11, 5)) @ c @ w["l0.mix.uv"].reshape(2, 10, 14)[a].T)
     assert np.allclose(np.concatenate(out, 1) @ w["l0.mix.o"].T, want)
+
+
+@pytest.mark.parametrize("mistake", ["expert", "share", "gate", "post_norm", "norm_bias", "alpha", "latent_norm", "scale", "logit_scale", "act"])
+def test_oracle_mistakes_show(mistake, monkeypatch):
+    """With the weights the device tests use, every mechanism left out or replaced moves the logits by far more than those tests allow."""
+    cfg = tu.config([(tu.latent(), tu.dense()), (tu.latent(heads=2), tu.moe())])
+    w, ids = tu.as_numpy(tu.weights(cfg, seed=3, q_gain=2.0)), tu.tokens(cfg, 60)
+    want = orc.forward(cfg, w, ids)
+    if mistake == "expert":
+        w["l1.mlp.table"] = (w["l1.mlp.table"] + 1) % 5
+    elif mistake == "share":
+        w["l1.mlp.table"] = w["l1.mlp.table"][:, [0, 0]]
+    elif mistake == "gate":
+        monkeypatch.setattr(orc, "sigmoid", lambda z: np.ones_like(z))
+    elif mistake == "post_norm":
+        w["l0.norm1b.alpha"] = w["l0.norm1b.alpha"] * 2
+    elif mistake == "norm_bias":
+        w["l1.norm2.b"] = np.zeros_like(w["l1.norm2.b"])
+    elif mistake == "alpha":
+        w["final.norm.alpha"] = np.ones(())
+    elif mistake == "latent_norm":
+        w["l0.mix.dkv.norm"] = np.ones_like(w["l0.mix.dkv.norm"])
+    elif mistake == "scale":
+        cfg["layers"][1]["mixer"]["scale"] = 1.0
+    elif mistake == "logit_scale":
+        cfg["logit_scale"] = 1.0
+    elif mistake == "act":
+        monkeypatch.setattr(orc, "relu2", lambda z: np.maximum(z, 0.0))
+    assert tu.err(orc.forward(cfg, w, ids), want) > 0.05
