@@ -558,42 +558,64 @@ typedef struct pie_stack pie_stack;
 size_t pie_stack_weight_bytes(int dtype, int N, int K);
 int pie_stack_pack_weight(const void *w, int N, int K, int dtype, void *packed, void *stream);
 
-/* Dynamic Tanh: w * tanh(alpha x) + b, element by element.  w, b: fp32 [width rounded up to 8, zeros past it] on the
- * device, 16-byte aligned. */
+/* A norm.  NONE: the identity.  DYN_TANH: w * tanh(param x) + b, element by element.  RMS: x / sqrt(mean(x^2) + param) * w.
+ * w, b: fp32 [width rounded up to 8, zeros past it] on the device, 16-byte aligned (b: DYN_TANH only). */
+enum { PIE_NORM_NONE = 0, PIE_NORM_DYN_TANH = 1, PIE_NORM_RMS = 2 };
 typedef struct {
     const float *w, *b;
-    float alpha;
-} pie_point_norm;
+    float param;
+    int kind;
+} pie_stack_norm;
 
 typedef struct {
     int dtype, width, vocab, n_layers;
-    float logit_scale;
+    float logit_scale, embed_scale;
     const void *embed;         /* bf16 [vocab][width] */
     const void *head;          /* packed [vocab, width] */
-    pie_point_norm final_norm;
+    pie_stack_norm final_norm;
 } pie_stack_config;
 
-enum { PIE_MIXER_LATENT = 1 };
-enum { PIE_FF_NONE = 0, PIE_FF_RELU2 = 1, PIE_FF_TABLE_MOE = 2 };
+enum { PIE_MIXER_LATENT = 1, PIE_MIXER_ATTENTION = 2, PIE_MIXER_DELTA = 3 };
+enum { PIE_FF_NONE = 0, PIE_FF_RELU2 = 1, PIE_FF_TABLE_MOE = 2, PIE_FF_ROUTED_MOE = 3 };
+enum { PIE_ACT_SILU = 0, PIE_ACT_CLIPPED = 1 };
 
-/* One layer: x += post1(mixer(pre1(x))); x += post2(ff(pre2(x))).
- * Latent mixer, with dim8 / vdim8 / rank8 = dim / vdim / rank rounded up to 8:  w_in packed [heads * dim8 + rank8, width] (rows past dim of a head and
- * past rank zero, the latent's down-projection last); w_uk heads x packed [rank, dim] (each head's up-projection of keys, transposed); w_uv heads x packed [vdim, rank];
- * w_o packed [width, heads * vdim8]; w_kv packed [heads * (dim8 + vdim8), rank] (all keys, then all values: long prompts spell K and V out; may be
- * NULL); c_norm fp32 [rank].  window <= 0: no limit.
- * Experts: w_gate_up experts x packed [2 * size, width] with rows (2 i, 2 i + 1) = (gate_i, up_i); w_down experts x packed [width, size];
- * table int32 [vocab][top].  Shared expert likewise when shared_size > 0, times sigmoid(shared_gate . input), shared_gate fp32 [width,
- * rounded up to 8 with zeros]. */
+/* One layer: x += post1(mixer(pre1(x))); x += post2(ff(pre2(x))).  Below, dim8 / vdim8 / rank8 = dim / vdim / rank rounded up to 8; rows and columns past a
+ * head's size are zero.
+ * Latent mixer:  w_in packed [heads * dim8 + rank8, width] (the latent's down-projection last); w_uk heads x packed [rank, dim] (each head's
+ * up-projection of keys, transposed); w_uv heads x packed [vdim, rank]; w_o packed [width, heads * vdim8]; w_kv packed [heads * (dim8 + vdim8), rank]
+ * (all keys, then all values: long prompts spell K and V out; may be NULL); c_norm fp32 [rank].  window <= 0: no limit.
+ * Attention mixer (softmax attention over cached keys and values):  w_in packed [heads * dim8 (q) + kv_heads * dim8 (k) + kv_heads * vdim8 (v) + heads
+ * rounded up to 8 (gate, when out_gate), width], in_bias bf16 in that order (NULL: none); q and k: RMS norm over dim with q_norm / k_norm (fp32 [dim]; NULL:
+ * none), then the first rot_dims dimensions rotated in neighbouring pairs by position * rot_freq[i] (fp32 [rot_dims / 2]), cos and sin times rot_gain;
+ * value_norm: every head's value over its root mean square; score = scale * q . k; sink: added to the softmax's denominator as sink * exp(0); out_gate:
+ * every head's output times the sigmoid of its gate.  kv_from = j >= 0: no keys and values of its own (no k, v rows in w_in), layer j's cached ones are
+ * read; else -1.  w_o packed [width, heads * vdim8], o_bias bf16 [width] (NULL: none).
+ * Delta mixer (generalised delta rule on a dim x dim state per head):  w_in packed [5 heads * dim8 (r, k, v, gate, removal rate) + rank8 (decay, low rank),
+ * width], in_bias as above; w_decay bf16 [heads * dim][rank8] row-major; decay_bias fp32 [heads * dim]; decay = exp(-decay_scale * sigmoid(w_decay tanh(.) +
+ * decay_bias)); unit key k / sqrt(sum k^2 + unit_eps); o_norm fp32 [heads * dim]; w_o packed [width, heads * dim8].
+ * Experts: w_gate_up experts x packed [2 * size, width] with rows (2 i, 2 i + 1) = (gate_i, up_i); w_down experts x packed [width, size].  act SILU:
+ * silu(g) u; CLIPPED: g = min(gate, act_limit), u = clamp(up, +-act_limit), g sigmoid(act_alpha g) (u + 1).
+ * TABLE_MOE: table int32 [vocab][top], every chosen expert weighs 1 / top.  ROUTED_MOE: w_router packed [experts, width], the `top` experts with the largest
+ * sigmoid(w_router h) + correction (fp32 [experts]), each weighing its sigmoid.
+ * Shared expert likewise when shared_size > 0, times sigmoid(shared_gate . input), shared_gate fp32 [width, rounded up to 8 with zeros]
+ * (element-wise norms only). */
 typedef struct {
-    pie_point_norm pre1, post1, pre2, post2;
+    pie_stack_norm pre1, post1, pre2, post2;
     int mixer, heads, dim, vdim, rank, window;
     float scale, eps;
     const void *w_in, *w_uk, *w_uv, *w_o, *w_kv;
     const float *c_norm;
+    int kv_heads, kv_from, rot_dims, value_norm, out_gate;
+    float rot_gain, sink, decay_scale, unit_eps;
+    const float *rot_freq, *q_norm, *k_norm, *decay_bias, *o_norm;
+    const void *in_bias, *o_bias, *w_decay;
     int ff, ff_size;           /* ff_size: the dense width, or one expert's */
     const void *w_up, *w_down; /* dense */
-    int experts, top, shared_size;
+    int experts, top, shared_size, act;
+    float act_alpha, act_limit;
     const int32_t *table;
+    const void *w_router;
+    const float *correction;
     const void *w_gate_up, *w_expert_down, *s_gate_up, *s_down;
     const float *shared_gate;
 } pie_stack_layer;
@@ -601,11 +623,14 @@ typedef struct {
 int pie_stack_create(const pie_stack_config *cfg, pie_stack **out);
 int pie_stack_destroy(pie_stack *s);
 int pie_stack_set_layer(pie_stack *s, int i, const pie_stack_layer *layer);
-/* elements per cached token of layer i (its page is [64][that many] in the stack's dtype), and bytes of one page */
+/* elements per cached token of layer i (its page is [64][that many] in the stack's dtype; 0: the layer caches no tokens), bytes of one page, and
+ * fp32 numbers of recurrent state per sequence (0: none).  A latent page holds token after token; a page of keys and values is laid out in matrix-core
+ * operand order (csrc/page_attn.hip) and means something as a whole only. */
 int pie_stack_page_row(const pie_stack *s, int i);
+size_t pie_stack_state_floats(const pie_stack *s, int i);
 size_t pie_stack_page_bytes(const pie_stack *s, int i);
 
-/* One pass.  Device arrays unless noted.  Rows are grouped in runs: run r = rows [row0, row0 + n_rows) at consecutive positions of sequence `seq` (a row of
+/* One pass.  Device arrays unless noted.  A sequence's state starts at zero when its row is at position 0 (a slot need not be cleared).  Rows are grouped in runs: run r = rows [row0, row0 + n_rows) at consecutive positions of sequence `seq` (a row of
  * `table`), runs in row order, covering all rows.  Every row's latent is appended to its page, then the row attends to its sequence's cached tokens and
  * itself.  want: the rows whose logits are asked for (NULL: all n_rows in order; n_want = n_rows).  logits fp32 [n_want][vocab]; logprobs (nullable)
  * likewise; next (nullable) the greedy tokens.  advance: afterwards ids[i] = next[i] and pos[i] += 1 (all rows wanted, one per run), and with a
@@ -620,9 +645,12 @@ typedef struct {
     const int32_t *want;
     float *logits, *logprobs;
     int32_t *next, *history;
-    void *const *slabs;        /* host array [n_layers] of device addresses */
+    void *const *slabs;        /* host array [n_layers] of device addresses (NULL where a layer caches no tokens) */
     size_t n_pages;
     float *tap;
+    const int32_t *slots;      /* device [n_seqs]: state slot of each row of `table` (recurrent layers; else NULL) */
+    float *const *states;      /* host array [n_layers] of device addresses [n_slots][state floats] (NULL where a layer has no state) */
+    size_t n_slots;
 } pie_stack_batch;
 int pie_stack_forward(pie_stack *s, const pie_stack_batch *b, int flags, void *stream);
 /* kernel launches of the last pass that was not replayed */

@@ -29,7 +29,7 @@ BASE_EXPORTS = [
     "pie_page_ptrs", "pie_page_i8_bytes", "pie_page_scale_ptrs",
     "pie_w16m_bytes", "pie_repack_w16m", "pie_linear_w16m_workspace", "pie_linear_w16m",
     "pie_stack_weight_bytes", "pie_stack_pack_weight", "pie_stack_create", "pie_stack_destroy", "pie_stack_set_layer", "pie_stack_page_row",
-    "pie_stack_page_bytes", "pie_stack_forward", "pie_stack_launches", "pie_logprobs_argmax_f32", "pie_logprobs_argmax_f32_workspace",
+    "pie_stack_page_bytes", "pie_stack_state_floats", "pie_stack_forward", "pie_stack_launches", "pie_logprobs_argmax_f32", "pie_logprobs_argmax_f32_workspace",
 ]
 EXPORTS = BASE_EXPORTS + [
     "pie_quantize_w4g64", "pie_dequantize_w4g64", "pie_w4s_bytes", "pie_repack_w4g64", "pie_w8s_bytes", "pie_repack_w8g64", "pie_qgemv_w8g64", "pie_quantize_g64", "pie_dequantize_g64", "pie_embedding_g64", "pie_w4s32_bytes", "pie_repack_w4g32", "pie_qgemv_w4g32", "pie_w8s32_bytes", "pie_repack_w8g32", "pie_qgemv_w8g32", "pie_embedding_g32",
@@ -69,33 +69,44 @@ class pie_global_weights(C.Structure):
                 ("fmt_embed", C.c_int), ("fmt_lm_head", C.c_int)]
 
 
-class pie_point_norm(C.Structure):
-    _fields_ = [("w", C.c_void_p), ("b", C.c_void_p), ("alpha", C.c_float)]
+class pie_stack_norm(C.Structure):
+    _fields_ = [("w", C.c_void_p), ("b", C.c_void_p), ("param", C.c_float), ("kind", C.c_int)]
+
+
+def _fields(spec: str, types: dict) -> list:
+    """"f:name name p:name" -> ctypes fields; a prefix holds until the next one."""
+    out, ct = [], None
+    for word in spec.split():
+        if ":" in word:
+            kind, word = word.split(":")
+            ct = types[kind]
+        out.append((word, ct))
+    return out
+
+
+_CT = {"i": C.c_int, "f": C.c_float, "p": C.c_void_p, "z": C.c_size_t, "n": pie_stack_norm}
 
 
 class pie_stack_config(C.Structure):
-    _fields_ = [("dtype", C.c_int), ("width", C.c_int), ("vocab", C.c_int), ("n_layers", C.c_int), ("logit_scale", C.c_float),
-                ("embed", C.c_void_p), ("head", C.c_void_p), ("final_norm", pie_point_norm)]
+    _fields_ = _fields("i:dtype width vocab n_layers f:logit_scale embed_scale p:embed head n:final_norm", _CT)
 
 
 class pie_stack_layer(C.Structure):
-    _fields_ = [("pre1", pie_point_norm), ("post1", pie_point_norm), ("pre2", pie_point_norm), ("post2", pie_point_norm),
-                ("mixer", C.c_int), ("heads", C.c_int), ("dim", C.c_int), ("vdim", C.c_int), ("rank", C.c_int), ("window", C.c_int),
-                ("scale", C.c_float), ("eps", C.c_float),
-                ("w_in", C.c_void_p), ("w_uk", C.c_void_p), ("w_uv", C.c_void_p), ("w_o", C.c_void_p), ("w_kv", C.c_void_p), ("c_norm", C.c_void_p),
-                ("ff", C.c_int), ("ff_size", C.c_int), ("w_up", C.c_void_p), ("w_down", C.c_void_p),
-                ("experts", C.c_int), ("top", C.c_int), ("shared_size", C.c_int), ("table", C.c_void_p),
-                ("w_gate_up", C.c_void_p), ("w_expert_down", C.c_void_p), ("s_gate_up", C.c_void_p), ("s_down", C.c_void_p), ("shared_gate", C.c_void_p)]
+    _fields_ = _fields("n:pre1 post1 pre2 post2 i:mixer heads dim vdim rank window f:scale eps p:w_in w_uk w_uv w_o w_kv c_norm "
+                       "i:kv_heads kv_from rot_dims value_norm out_gate f:rot_gain sink decay_scale unit_eps p:rot_freq q_norm k_norm decay_bias o_norm "
+                       "in_bias o_bias w_decay i:ff ff_size p:w_up w_down i:experts top shared_size act f:act_alpha act_limit p:table w_router correction "
+                       "w_gate_up w_expert_down s_gate_up s_down shared_gate", _CT)
 
 
 class pie_stack_batch(C.Structure):
-    _fields_ = [(n, C.c_int) for n in ("n_rows", "n_seqs", "table_width", "n_runs", "n_want", "advance", "history_len", "reserved")] + \
-               [(n, C.c_void_p) for n in ("ids", "pos", "row_seq", "table", "runs", "runs_host", "want", "logits", "logprobs", "next", "history", "slabs")] + \
-               [("n_pages", C.c_size_t), ("tap", C.c_void_p)]
+    _fields_ = _fields("i:n_rows n_seqs table_width n_runs n_want advance history_len reserved p:ids pos row_seq table runs runs_host want logits logprobs "
+                       "next history slabs z:n_pages p:tap slots states z:n_slots", _CT)
 
 
-PIE_MIXER_LATENT = 1
-PIE_FF_NONE, PIE_FF_RELU2, PIE_FF_TABLE_MOE = 0, 1, 2
+PIE_NORM_NONE, PIE_NORM_DYN_TANH, PIE_NORM_RMS = 0, 1, 2
+PIE_MIXER_LATENT, PIE_MIXER_ATTENTION, PIE_MIXER_DELTA = 1, 2, 3
+PIE_FF_NONE, PIE_FF_RELU2, PIE_FF_TABLE_MOE, PIE_FF_ROUTED_MOE = 0, 1, 2, 3
+PIE_ACT_SILU, PIE_ACT_CLIPPED = 0, 1
 
 
 def set_knob(name: str, value: int | None) -> None:
@@ -131,7 +142,7 @@ def base() -> C.CDLL:
     lib = _open(_PKG / "lib" / "libpie_base.so", BASE_EXPORTS)
     for name in ("pie_hello", "pie_version", "pie_last_error"):
         getattr(lib, name).restype = C.c_char_p
-    for name in ("pie_page_pool_slab_bytes", "pie_page_pool_size", "pie_page_pool_num_free", "pie_stack_weight_bytes", "pie_stack_page_bytes", "pie_logprobs_argmax_f32_workspace"):
+    for name in ("pie_page_pool_slab_bytes", "pie_page_pool_size", "pie_page_pool_num_free", "pie_stack_weight_bytes", "pie_stack_page_bytes", "pie_stack_state_floats", "pie_logprobs_argmax_f32_workspace"):
         getattr(lib, name).restype = C.c_size_t
     lib.pie_page_pool_slab_bytes.argtypes = [C.c_size_t, C.c_int, C.c_int, C.c_int]
     lib.pie_page_pool_create.argtypes = [C.c_size_t, C.c_int, C.c_int, C.c_int, C.c_void_p, C.POINTER(C.c_void_p)]
@@ -146,7 +157,7 @@ def base() -> C.CDLL:
     lib.pie_stack_create.argtypes = [C.POINTER(pie_stack_config), C.POINTER(C.c_void_p)]
     lib.pie_stack_destroy.argtypes = lib.pie_stack_launches.argtypes = [C.c_void_p]
     lib.pie_stack_set_layer.argtypes = [C.c_void_p, C.c_int, C.POINTER(pie_stack_layer)]
-    lib.pie_stack_page_row.argtypes = lib.pie_stack_page_bytes.argtypes = [C.c_void_p, C.c_int]
+    lib.pie_stack_page_row.argtypes = lib.pie_stack_page_bytes.argtypes = lib.pie_stack_state_floats.argtypes = [C.c_void_p, C.c_int]
     lib.pie_stack_forward.argtypes = [C.c_void_p, C.POINTER(pie_stack_batch), C.c_int, C.c_void_p]
     _base = lib
     return lib

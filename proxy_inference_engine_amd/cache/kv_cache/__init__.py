@@ -34,8 +34,8 @@ class BaseCache(ABC):
                 if t is not None:
                     arrays[f"{i}.{j}"] = t.detach().to("cpu").contiguous()
             meta[f"0.{i}"] = str(c.meta_state)
-            # a paged cache is stored as its gathered rows, the layout a ReusableKVCache restores from
-            meta[f"2.{i}"] = {"PagedKVCache": "ReusableKVCache", "PagedLatentCache": "SavedLatentCache"}.get(type(c).__name__, type(c).__name__)
+            # a paged cache is stored as its gathered rows (a layer stack's: as whole pages), the layout its saved class restores from
+            meta[f"2.{i}"] = {"PagedKVCache": "ReusableKVCache", "PagedLatentCache": "SavedLatentCache", "PagedStackCache": "SavedStackCache"}.get(type(c).__name__, type(c).__name__)
         for k, v in (metadata or {}).items():
             meta[f"1.{k}"] = str(v)
         save_file(arrays, file_name, metadata=meta)
@@ -45,7 +45,7 @@ class BaseCache(ABC):
         from safetensors import safe_open
         if device is None:
             device = "cuda" if torch.cuda.is_available() else "cpu"
-        classes = {"ReusableKVCache": ReusableKVCache, "SavedLatentCache": SavedLatentCache}
+        classes = {"ReusableKVCache": ReusableKVCache, "SavedLatentCache": SavedLatentCache, "SavedStackCache": SavedStackCache}
         with safe_open(file_name, framework="pt", device="cpu") as f:
             meta = f.metadata() or {}
             n = sum(1 for k in meta if k.startswith("2."))
@@ -95,5 +95,7 @@ class BaseCache(ABC):
 from .reusable import ReusableKVCache  # noqa: E402
 from .paged import PageAllocator, PagedKVCache, PagedSequence  # noqa: E402
 from .latent import LatentPageAllocator, PagedLatentCache, SavedLatentCache  # noqa: E402
+from .stack import PagedStackCache, SavedStackCache, StackPageAllocator, StackSequence  # noqa: E402
 
-__all__ = ["BaseCache", "ReusableKVCache", "PagedKVCache", "PagedSequence", "PageAllocator", "LatentPageAllocator", "PagedLatentCache", "SavedLatentCache"]
+__all__ = ["BaseCache", "ReusableKVCache", "PagedKVCache", "PagedSequence", "PageAllocator", "LatentPageAllocator", "PagedLatentCache", "SavedLatentCache", "StackPageAllocator",
+           "StackSequence", "PagedStackCache", "SavedStackCache"]

@@ -13,7 +13,7 @@ from .paged import TOKEN_CAPACITY_PER_PAGE, PageAllocator, PagedKVCache, PagedSe
 class LatentPageAllocator(PageAllocator):
     def __init__(self, num_pages: int, row_elems: list[int], dtype: torch.dtype = torch.bfloat16, device: torch.device | str | None = None):
         """row_elems: stored numbers per token, layer by layer (the latent's width, padded as the kernels want it)."""
-        super().__init__(num_pages, 1, max(row_elems, default=1), num_layers=len(row_elems))  # the native pool keeps the ids; it never touches pages
+        super().__init__(num_pages, 1, max([*row_elems, 1]), num_layers=len(row_elems))  # the native pool keeps the ids; it never touches pages
         self.dtype, self.row_elems = dtype, list(row_elems)
         self.slabs = None
         if device is not None:
@@ -91,6 +91,10 @@ class PagedLatentCache(PagedKVCache):
         for j, p in enumerate(seq.pages):
             part = rows[0, 0, j * TOKEN_CAPACITY_PER_PAGE:(j + 1) * TOKEN_CAPACITY_PER_PAGE]
             slab[p, :part.shape[0]] = part.to(device=slab.device, dtype=slab.dtype)
+
+    def adopt(self, saved: SavedLatentCache) -> None:
+        """Takes over what a file held."""
+        self.state = (saved.rows[:, :, :saved.offset], None)
 
 
 __all__ = ["LatentPageAllocator", "PagedLatentCache", "SavedLatentCache", "PagedSequence"]

@@ -20,7 +20,7 @@ import torch
 
 logger = logging.getLogger(__name__)
 
-from .kv_cache import BaseCache, PagedKVCache, ReusableKVCache, SavedLatentCache
+from .kv_cache import BaseCache, PagedKVCache, PagedStackCache, ReusableKVCache, SavedLatentCache
 
 
 def _as_list(ids) -> list[int]:
@@ -82,7 +82,10 @@ class PromptCache:
             if i >= len(ids) - 1 or ids[i] != tok:
                 break
             common += 1
-        if common == 0:
+        stack = isinstance(self.cache[0], PagedStackCache)
+        if stack:  # a recurrent state is the last token's: all of the history is kept, or none
+            common = self.cache[0].reusable(common)
+        if common == 0 and not stack:
             return prompt_ids
         for layer_cache in self.cache:
             assert isinstance(layer_cache, (ReusableKVCache, PagedKVCache, SavedLatentCache))

@@ -1,23 +1,24 @@
 // layer_stack.hip -- native runtime of the layer-stack models: one pass over a list of layers that may all differ (pie_stack_*, include/pie_hip.h).
 //
 // A pass is a batch of rows, each with its own sequence and position: whole prompts, portions and single decoded tokens are the same thing here.
-// Launches per layer (every norm is element-wise and rides in the epilogue of the kernel that produces its input):
-//   [q | latent down]     Linear                                      (rows_gemm.hip)
-//   q -> latent space     Linear per head; beside it the latents' RMS norm and their append to the pages
-//   attention over the latents                                        (latent_attn.hip)
-//   latents -> values     Linear per head, merging the key splits on the way in (more than a few rows: merged by a launch of its own)
-//   output projection     Linear; epilogue: x += post1(y), h = pre2(x)
-//   dense: up (relu^2), down; epilogue: x += post2(y), h = next layer's pre1(x)
-//   experts: gate|up (silu * up) and down over the active experts and the shared one, then the weighted sum with the same epilogue
+// A layer is a mixer and a feed-forward, each between two norms.  Mixers:
+//   latent attention      [q | latent down] Linear; q -> latent space per head (beside it the latents' RMS norm and their append to the pages); attention
+//                         (latent_attn.hip); latents -> values per head, merging the key splits on the way in (more than a few rows: a launch of its own)
+//   attention             [q | k | v | gate] Linear; norms, rotation and page writes; attention over keys and values (page_attn.hip)
+//   delta rule            [r | k | v | gate | rate | decay] Linear; recurrence (delta_rule.hip)
+// and an output projection.  Feed-forwards: dense up (relu^2), down; or experts: gate|up and down over the active experts (and a shared one).
+// Norms: element-wise ones ride in the epilogue of the kernel that produces their input (x += post(y), h = next(x)); a norm over the whole row is applied,
+// with the same additions, by one launch behind the sublayer (row_update.hip), which also takes the experts' weighted sum.
 // A pass of more rows than the weight-streaming Linear is for (BIG_ROWS; bf16) multiplies through the tiled GEMMs instead (w16_gemm.hpp, grouped by expert
-// for mixtures), with the norms in element-wise passes behind them; runs of LONG_RUN rows and more spell their keys and values out (window_attn.hip)
-// while the shorter runs in front of them keep the latent form.
-// The experts of a token are a table lookup, so all layers' row lists are made by one launch in front of the pass.
+// for mixtures); runs of LONG_RUN rows and more use the attentions' long forms (latents: with keys and values spelled out, window_attn.hip) while the
+// shorter runs in front of them keep the short ones.
+// Where a table names a token's experts, all layers' row lists are made by one launch in front of the pass; a router's are made behind its logits.
 #include <cstring>
 #include <algorithm>
 #include <new>
 #include <vector>
 
+#include "mfma_store.hpp"  // MFMA_ACT_*
 #include "stack_types.hpp"
 
 size_t w16l_workspace_bytes(int M, int N, int K);
@@ -25,7 +26,7 @@ int w16l_gemm_launch(int dtype, const void *w16m, const void *x, int ldx, int M,
                      void *swiglu_act, bool *fused, int ldy);
 int w16l_relu2_launch(const void *w16m, const void *x, int ldx, int M, int N, int K, void *y, int ldy, hipStream_t st);
 int w16l_grouped_launch(const void *w16m, size_t w_stride, const void *x, int ldx, size_t x_rows, const int *list, const void *tiles, int tm, int block, int tile_rows, int N, int K,
-                        void *y, int ldy, bool swiglu, hipStream_t st);
+                        void *y, int ldy, int act, float act_alpha, float act_limit, hipStream_t st);
 
 namespace {
 
@@ -33,7 +34,11 @@ constexpr int BIG_ROWS = 64;  // more rows than this take the tiled GEMMs
 constexpr int LONG_RUN = 64;  // runs of at least this many rows attend with keys and values spelled out
 
 struct RouteLayer {      // one mixture layer's row lists (device pointers)
-    const int *table;
+    const int *table;    // experts by token id; nullptr: by the router's logits
+    const float *logits, *correction;  // [M][ld_logits], [experts]
+    int ld_logits;
+    int *chosen;         // [M * top]: the router's choice, best first, and the weights
+    float *weight;
     int top, experts, max_active;
     int *active, *offset, *list, *place;  // [max_active], [experts + 1], [M * top] rows by expert, [M * top] position of (row, slot)
     int4 *tiles;  // {expert, first position, rows, 0}: row tiles of the grouped GEMM
@@ -48,12 +53,56 @@ __host__ __device__ inline int route_max_tiles(long M, int top, int experts) {
     return ((int)(M * top / route_tile_rows(M, top, experts)) + route_block(M, top, experts) * experts + 3) / 4 * 4;
 }
 
-__global__ void __launch_bounds__(1024) k_route(const RouteLayer *layers, const int *ids, int M, int vocab) {
+// One wave: the `top` experts of row m with the largest sigmoid(logit) + correction (equal ones: the first), each with the weight sigmoid(logit).
+// Round k takes the best of what comes behind round k - 1's in that order, so nothing has to be marked as taken.
+__device__ __forceinline__ void route_pick(const RouteLayer &L, int m, int lane) {
+    const float *z = L.logits + (size_t)m * L.ld_logits;
+    constexpr int R = 4;  // scores a lane keeps; more experts than 64 R are scored again in every round
+    float keep[R];
+    auto score = [&](int e) { return 1.0f / (1.0f + expf(-z[e])) + L.correction[e]; };
+#pragma unroll
+    for (int r = 0; r < R; ++r) keep[r] = 64 * r + lane < L.experts ? score(64 * r + lane) : -INFINITY;
+    float last = INFINITY;
+    int last_e = -1;
+    for (int k = 0; k < L.top; ++k) {
+        float best = -INFINITY;
+        int at = 0x7fffffff;
+        auto look = [&](float s, int e) {
+            if ((s < last || (s == last && e > last_e)) && s > best) best = s, at = e;
+        };
+#pragma unroll
+        for (int r = 0; r < R; ++r)
+            if (64 * r + lane < L.experts) look(keep[r], 64 * r + lane);
+        for (int e = 64 * R + lane; e < L.experts; e += 64) look(score(e), e);
+        const float top = wave_max(best);
+        int e = best == top ? at : 0x7fffffff;
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) e = min(e, __shfl_xor(e, o, 64));
+        e = e < L.experts ? e : k;  // (scores that compare with nothing)
+        last = top, last_e = e;
+        if (lane == 0) {
+            L.chosen[(size_t)m * L.top + k] = e;
+            L.weight[(size_t)m * L.top + k] = 1.0f / (1.0f + expf(-z[e]));
+        }
+    }
+}
+__global__ void __launch_bounds__(256) k_route_pick(const RouteLayer *layers, int M) {
+    const int m = blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (m < M) route_pick(layers[0], m, threadIdx.x & 63);
+}
+
+// the row lists of layers[blockIdx.x]; pick: its router's choice is made here too (few rows)
+__global__ void __launch_bounds__(1024) k_route(const RouteLayer *layers, const int *ids, int M, int vocab, bool pick) {
     extern __shared__ int s_cnt[];  // [experts] counts, then [experts] cursors
     const RouteLayer L = layers[blockIdx.x];
     int *s_cur = s_cnt + L.experts;
     const int n = M * L.top;
+    if (pick) {
+        for (int m = threadIdx.x >> 6; m < M; m += 16) route_pick(L, m, threadIdx.x & 63);
+        __syncthreads();
+    }
     auto expert = [&](int i) {
+        if (!L.table) return min(max(L.chosen[i], 0), L.experts - 1);
         const int t = min(max(ids[i / L.top], 0), vocab - 1);
         return min(max(L.table[(size_t)t * L.top + i % L.top], 0), L.experts - 1);
     };
@@ -108,30 +157,33 @@ __device__ __forceinline__ void store4(typename E::type *p, float4 y) {
     else *(float4 *)p = y;
 }
 template <class E>
-__global__ void __launch_bounds__(256) k_stack_embed(const int *ids, const u16 *table, int vocab, int W, PointNorm next, float *x, int ldx, typename E::type *h, int ldh) {
+__global__ void __launch_bounds__(256) k_stack_embed(const int *ids, const u16 *table, int vocab, int W, float scale, bool plain, PointNorm next, float *x, int ldx,
+                                                     typename E::type *h, int ldh) {  // plain: h = x
     const size_t m = blockIdx.y;
     const int n = (blockIdx.x * 256 + threadIdx.x) * 4;
     if (n >= W) return;
     const u16 *src = table + (size_t)min(max(ids[m], 0), vocab - 1) * W + n;
     if (n + 4 <= W && !(W & 3)) {
         const uint2 t = *(const uint2 *)src;
-        const float4 v = make_float4(lo_f32<BF16>(t.x), hi_f32<BF16>(t.x), lo_f32<BF16>(t.y), hi_f32<BF16>(t.y)), y = point_norm4(next, n, v);
+        const float4 v = make_float4(lo_f32<BF16>(t.x) * scale, hi_f32<BF16>(t.x) * scale, lo_f32<BF16>(t.y) * scale, hi_f32<BF16>(t.y) * scale);
+        const float4 y = plain ? v : point_norm4(next, n, v);
         *(float4 *)(x + m * ldx + n) = v;
         store4<E>(h + m * ldh + n, y);
         return;
     }
     for (int i = 0; i < min(4, W - n); ++i) {
-        const float v = BF16::to_f32(src[i]);
+        const float v = BF16::to_f32(src[i]) * scale;
         x[m * ldx + n + i] = v;
-        h[m * ldh + n + i] = E::pack(point_norm(next, n + i, v));
+        h[m * ldh + n + i] = E::pack(plain ? v : point_norm(next, n + i, v));
     }
 }
 
-// y = sum over the token's slots of its experts' outputs / top (+ sigmoid(gate . input) * shared output); x += post(y); h = next(x)
+// y = sum over the token's slots of its experts' weighted outputs (+ sigmoid(gate . input) * shared output); x += post(y); h = next(x)
 struct CombineArgs {
     const void *part, *part_s;   // [M * top][ldp] by position, [M][ldp_s]
     int ldp, ldp_s;
     const int *place;
+    const float *weight;         // [M * top] or nullptr: 1 / top each
     int top, W;
     const float *gate;           // [W] or nullptr
     PointNorm pre, post, next;   // pre: the sublayer's input norm (the gate's dot product is taken in fp32 on it)
@@ -156,10 +208,11 @@ __global__ void __launch_bounds__(1024) k_moe_combine(const CombineArgs a) {
     constexpr int U = 8;  // slots in flight
     float4 v[U], vs = make_float4(0, 0, 0, 0), xv = vs;
     int n = threadIdx.x * 4;
+    float share[U];
     auto fetch = [&](int s0) {
 #pragma unroll
         for (int u = 0; u < U; ++u)
-            if (s0 + u < a.top) v[u] = load4<P>(a.part, (size_t)a.place[m * a.top + s0 + u] * a.ldp + n);
+            if (s0 + u < a.top) share[u] = a.weight ? a.weight[m * a.top + s0 + u] : 1.0f / (float)a.top, v[u] = load4<P>(a.part, (size_t)a.place[m * a.top + s0 + u] * a.ldp + n);
     };
     auto fetch_row = [&] {  // (rows of x, part and the norms' paddings: a quad that starts inside W is readable up to the next multiple of 4)
         fetch(0);
@@ -181,7 +234,6 @@ __global__ void __launch_bounds__(1024) k_moe_combine(const CombineArgs a) {
         for (int i = 1; i < (int)blockDim.x / 64; ++i) d += red[i];
         g = 1.0f / (1.0f + expf(-d));
     }
-    const float share = 1.0f / (float)a.top;
     for (; n < a.W; n += blockDim.x * 4) {
         if (n != (int)threadIdx.x * 4) fetch_row();
         float y[4] = {0, 0, 0, 0};
@@ -189,7 +241,7 @@ __global__ void __launch_bounds__(1024) k_moe_combine(const CombineArgs a) {
             if (s0) fetch(s0);
 #pragma unroll
             for (int u = 0; u < U; ++u)
-                if (s0 + u < a.top) y[0] = fmaf(share, v[u].x, y[0]), y[1] = fmaf(share, v[u].y, y[1]), y[2] = fmaf(share, v[u].z, y[2]), y[3] = fmaf(share, v[u].w, y[3]);
+                if (s0 + u < a.top) y[0] = fmaf(share[u], v[u].x, y[0]), y[1] = fmaf(share[u], v[u].y, y[1]), y[2] = fmaf(share[u], v[u].z, y[2]), y[3] = fmaf(share[u], v[u].w, y[3]);
         }
         if (a.gate) y[0] = fmaf(g, vs.x, y[0]), y[1] = fmaf(g, vs.y, y[1]), y[2] = fmaf(g, vs.z, y[2]), y[3] = fmaf(g, vs.w, y[3]);
         const float4 q = point_norm4(a.post, n, make_float4(y[0], y[1], y[2], y[3]));
@@ -305,8 +357,9 @@ int up64(int n) { return (n + 63) & ~63; }
 struct GraphKey {
     pie_stack_batch b;
     std::vector<void *> slabs;
+    std::vector<float *> states;
     std::vector<int32_t> runs;
-    bool same(const GraphKey &o) const { return memcmp(&b, &o.b, sizeof b) == 0 && slabs == o.slabs && runs == o.runs; }
+    bool same(const GraphKey &o) const { return memcmp(&b, &o.b, sizeof b) == 0 && slabs == o.slabs && states == o.states && runs == o.runs; }
 };
 struct GraphSlot {
     GraphKey key;
@@ -321,13 +374,14 @@ struct pie_stack {
     std::vector<pie_stack_layer> layers;
     std::vector<char> have;
     // workspace, by rows of a pass
-    Buf<float> x, c_raw, part, part_s, attn_ws, gemm_ws;
+    Buf<float> x, c_raw, part, part_s, attn_ws, gemm_ws, y32, logits_e;
     Buf<char> h, q, ql, oc, o, act, act_e, act_s, y, ctx, kv;
     Buf<RowStat> stats;
     Buf<int> route_ints;
     Buf<RouteLayer> route_dev;
     std::vector<RouteLayer> route;  // per layer; experts == 0: not a mixture
-    int route_rows = 0, n_route = 0, route_lds = 0;
+    int route_rows = 0, n_table = 0, route_lds = 0;  // n_table: mixtures whose experts a table names (in front in route_dev)
+    std::vector<int> route_at;      // layer -> entry of route_dev
     std::vector<GraphSlot> graphs;
     unsigned long long tick = 0;
     int launches = 0;
@@ -342,17 +396,28 @@ struct pie_stack {
 namespace {
 
 size_t esize(const pie_stack *s) { return s->cfg.dtype == PIE_F32 ? 4 : 2; }
-PointNorm norm_of(const pie_point_norm &n) { return {n.w, n.b, n.alpha}; }
+bool pointwise(const pie_stack_norm &n) { return n.kind == PIE_NORM_DYN_TANH; }
+PointNorm norm_of(const pie_stack_norm &n) { return {n.w, n.b, n.param}; }
+StackNorm row_norm_of(const pie_stack_norm &n) { return {n.w, n.b, n.param, n.kind}; }
+bool is_moe(const pie_stack_layer &L) { return L.ff == PIE_FF_TABLE_MOE || L.ff == PIE_FF_ROUTED_MOE; }
+KvGeometry geometry(const pie_stack_layer &L) { return kv_geometry(L.heads, L.kv_heads, L.dim, L.vdim); }
+// columns of the mixer's input projection, and what its output projection reads
+int in_columns(const pie_stack_layer &L) {
+    if (L.mixer == PIE_MIXER_LATENT) return L.heads * up8(L.dim) + up8(L.rank);
+    if (L.mixer == PIE_MIXER_DELTA) return 5 * L.heads * up8(L.dim) + up8(L.rank);
+    return L.heads * up8(L.dim) + (L.kv_from < 0 ? L.kv_heads * (up8(L.dim) + up8(L.vdim)) : 0) + (L.out_gate ? up8(L.heads) : 0);
+}
+int out_columns(const pie_stack_layer &L) { return L.heads * up8(L.mixer == PIE_MIXER_DELTA ? L.dim : L.vdim); }
 
 // How a pass is laid out: rows of the leading short runs, and what the long runs behind them see.
 struct Plan {
     bool big;
-    int short_rows, short_runs, long_tiles;
+    int short_rows, short_runs, long_rows;
 };
 Plan plan_pass(const pie_stack *s, const pie_stack_batch &b) {
     Plan p = {s->cfg.dtype == PIE_BF16 && b.n_rows > BIG_ROWS, 0, 0, 0};
     while (p.short_runs < b.n_runs && (!p.big || b.runs_host[4 * p.short_runs + 1] < LONG_RUN)) p.short_rows += b.runs_host[4 * p.short_runs++ + 1];
-    for (int i = p.short_runs; i < b.n_runs; ++i) p.long_tiles += (b.runs_host[4 * i + 1] + 127) / 128;
+    p.long_rows = b.n_rows - p.short_rows;
     return p;
 }
 bool spelled_out(const pie_stack_layer &L) { return L.w_kv && up8(L.dim) <= WINDOW_ATTN_MAX_DIM && up8(L.vdim) <= WINDOW_ATTN_MAX_DIM; }
@@ -369,23 +434,28 @@ size_t plan_context(const pie_stack_batch &b, const Plan &p, int window) {
 
 int stack_reserve(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipStream_t st) {
     const size_t M = (size_t)b.n_rows, E = esize(s), W64 = up64(s->cfg.width), WA = act_stride(s->cfg.width);
-    size_t q = 0, c = 0, ql = 0, o = 0, act = 0, act_e = 0, act_s = 0, part = 0, part_s = 0, ints = 0, ctx = 0, kv = 0, ws = 0;
+    size_t q = 0, c = 0, ql = 0, o = 0, act = 0, act_e = 0, act_s = 0, part = 0, part_s = 0, ints = 0, ctx = 0, kv = 0, ws = 0, le = 0;
     auto gemm = [&](int N, int K) { ws = std::max(ws, w16l_workspace_bytes((int)M, N, K) / 4); };
     for (const pie_stack_layer &L : s->layers) {
-        const int NI = L.heads * up8(L.dim) + up8(L.rank), KO = L.heads * up8(L.vdim);
-        q = std::max(q, (size_t)NI), c = std::max(c, (size_t)up8(L.rank)), ql = std::max(ql, (size_t)L.heads * up8(L.rank)), o = std::max(o, (size_t)act_stride(KO));
-        if (plan.big) gemm(NI, s->cfg.width), gemm(L.heads * up8(L.dim), s->cfg.width), gemm(up8(L.rank), s->cfg.width), gemm(s->cfg.width, KO);
-        if (plan.long_tiles && spelled_out(L)) {
-            const size_t n = plan_context(b, plan, L.window), nkv = L.heads * (up8(L.dim) + up8(L.vdim));
-            ctx = std::max(ctx, n * act_stride(L.rank)), kv = std::max(kv, n * nkv);
-            ws = std::max(ws, w16l_workspace_bytes((int)n, (int)nkv, L.rank) / 4);
+        const int NI = in_columns(L), KO = out_columns(L);
+        q = std::max(q, (size_t)NI), o = std::max(o, (size_t)act_stride(KO));
+        if (plan.big) gemm(NI, s->cfg.width), gemm(s->cfg.width, KO);
+        if (L.mixer == PIE_MIXER_LATENT) {
+            c = std::max(c, (size_t)up8(L.rank)), ql = std::max(ql, (size_t)L.heads * up8(L.rank));
+            if (plan.big) gemm(L.heads * up8(L.dim), s->cfg.width), gemm(up8(L.rank), s->cfg.width);
+            if (plan.long_rows && spelled_out(L)) {
+                const size_t n = plan_context(b, plan, L.window), nkv = L.heads * (up8(L.dim) + up8(L.vdim));
+                ctx = std::max(ctx, n * act_stride(L.rank)), kv = std::max(kv, n * nkv);
+                ws = std::max(ws, w16l_workspace_bytes((int)n, (int)nkv, L.rank) / 4);
+            }
         }
         if (L.ff == PIE_FF_RELU2) {
             act = std::max(act, (size_t)act_stride(L.ff_size));
             if (plan.big) gemm(s->cfg.width, L.ff_size);
         }
-        if (L.ff == PIE_FF_TABLE_MOE) {
+        if (is_moe(L)) {
             act_e = std::max(act_e, (size_t)L.top * act_stride(L.ff_size)), part = std::max(part, (size_t)L.top * W64);
+            if (L.ff == PIE_FF_ROUTED_MOE) le = std::max(le, (size_t)up8(L.experts));
             if (L.shared_size) {
                 act_s = std::max(act_s, (size_t)act_stride(L.shared_size)), part_s = W64;
                 if (plan.big) gemm(s->cfg.width, L.shared_size);
@@ -398,26 +468,34 @@ int stack_reserve(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
         (rc = s->h.need(M * WA * E, &moved)) || (rc = s->q.need(M * q * E, &moved)) || (rc = s->ql.need(M * ql * E, &moved)) || (rc = s->oc.need(M * ql * E, &moved)) ||
         (rc = s->o.need(M * o * E, &moved)) || (rc = s->act.need(M * act * E, &moved)) || (rc = s->act_e.need(M * act_e * E, &moved)) ||
         (rc = s->act_s.need(M * act_s * E, &moved)) || (rc = s->stats.need((size_t)b.n_want * ST_TILES, &moved)) || (rc = s->y.need(plan.big ? M * W64 * E : 0, &moved)) ||
-        (rc = s->ctx.need(ctx * E, &moved)) || (rc = s->kv.need(kv * E, &moved)) || (rc = s->gemm_ws.need(ws, &moved)))
+        (rc = s->y32.need(plan.big ? 0 : M * W64, &moved)) || (rc = s->logits_e.need(M * le, &moved)) || (rc = s->ctx.need(ctx * E, &moved)) ||
+        (rc = s->kv.need(kv * E, &moved)) || (rc = s->gemm_ws.need(ws, &moved)))
         return rc;
-    if (s->n_route && (int)M > s->route_rows) {
-        s->route_rows = (int)M;
-        // (at most this many tiles for any pass of up to M rows: 64-row tiles and one ragged block of tiles per expert)
-        auto tiles = [&](const RouteLayer &r) { return (M * r.top / 64 + ROUTE_BLOCK_MAX * r.experts + 3) / 4 * 4; };
+    int n_moe = 0;
+    s->n_table = 0;
+    for (const pie_stack_layer &L : s->layers) n_moe += is_moe(L), s->n_table += L.ff == PIE_FF_TABLE_MOE;
+    if (n_moe && ((int)M > s->route_rows || moved)) {
+        s->route_rows = std::max(s->route_rows, (int)M);
+        const size_t R = (size_t)s->route_rows;
+        // (at most this many tiles for any pass of up to R rows: 64-row tiles and one ragged block of tiles per expert)
+        auto tiles = [&](const RouteLayer &r) { return (R * r.top / 64 + ROUTE_BLOCK_MAX * r.experts + 3) / 4 * 4; };
+        auto lists = [&](const RouteLayer &r) { return (2 * (size_t)r.experts + 1 + 2 * R * r.top + (r.table ? 0 : 2 * R * r.top) + 3) / 4 * 4; };
         for (const RouteLayer &r : s->route)
-            if (r.experts) ints += (2 * (size_t)r.experts + 1 + 2 * M * r.top + 3) / 4 * 4 + 4 * tiles(r);
-        if ((rc = s->route_ints.need(ints, &moved)) || (rc = s->route_dev.need(s->n_route, &moved))) return rc;
-        int *p = s->route_ints.p;
-        std::vector<RouteLayer> dev;
-        s->route_lds = 0;
-        for (RouteLayer &r : s->route) {
+            if (r.experts) ints += lists(r) + 4 * tiles(r);
+        if ((rc = s->route_ints.need(ints, &moved)) || (rc = s->route_dev.need(n_moe, &moved))) return rc;
+        int *p = s->route_ints.p, at[2] = {0, s->n_table};
+        std::vector<RouteLayer> dev(n_moe);
+        s->route_lds = 0, s->route_at.assign(s->layers.size(), 0);
+        for (size_t i = 0; i < s->layers.size(); ++i) {
+            RouteLayer &r = s->route[i];
             if (!r.experts) continue;
             r.tiles = (int4 *)p, p += 4 * tiles(r);
-            r.active = p, r.offset = r.active + r.experts, r.list = r.offset + r.experts + 1, r.place = r.list + M * r.top;
-            p += (2 * (size_t)r.experts + 1 + 2 * M * r.top + 3) / 4 * 4;
+            r.active = p, r.offset = r.active + r.experts, r.list = r.offset + r.experts + 1, r.place = r.list + R * r.top;
+            if (!r.table) r.chosen = r.place + R * r.top, r.weight = (float *)(r.chosen + R * r.top), r.logits = s->logits_e.p, r.ld_logits = up8(r.experts);
+            p += lists(r);
             r.max_active = r.experts;
             s->route_lds = std::max(s->route_lds, 2 * r.experts * 4);
-            dev.push_back(r);
+            dev[s->route_at[i] = at[r.table ? 0 : 1]++] = r;
         }
         PIE_HIP_TRY(hipStreamSynchronize(st));
         PIE_HIP_TRY(hipMemcpy(s->route_dev.p, dev.data(), dev.size() * sizeof(RouteLayer), hipMemcpyHostToDevice));
@@ -432,6 +510,7 @@ int stack_reserve(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
 
 // key splits of a layer's attention: enough workgroups for the chip, at least 64 keys each; from capacities only, so that a captured step keeps its plan
 int plan_splits(const pie_stack_batch &b, const pie_stack_layer &L, int n_tiles) {
+    if (n_tiles <= 0) return 1;
     long ctx = (long)b.table_width * PAGE_TOKENS;
     if (L.window > 0 && L.window + 64 < ctx) ctx = L.window + 64;
     long s = 256 / n_tiles;
@@ -440,10 +519,23 @@ int plan_splits(const pie_stack_batch &b, const pie_stack_layer &L, int n_tiles)
     return (int)std::max(s, 1L);
 }
 
-int stack_tiles(const int32_t *runs, int n_runs, int H) {
-    int n = 0;
-    for (int i = 0; i < n_runs; ++i) n += latent_attn_tiles(runs[4 * i + 1], H);
-    return n;
+// the rows and runs of a pass that take a layer's short attention form, and their tiles
+struct ShortPart {
+    int M, runs, tiles;
+};
+ShortPart short_part(const pie_stack *s, const pie_stack_batch &b, const Plan &plan, const pie_stack_layer &L) {
+    const bool attn = L.mixer == PIE_MIXER_ATTENTION, split = plan.long_rows && (attn ? page_attn_mfma(s->cfg.dtype, geometry(L)) : spelled_out(L));
+    ShortPart p = {split ? plan.short_rows : b.n_rows, split ? plan.short_runs : b.n_runs, 0};
+    for (int i = 0; i < p.runs; ++i) p.tiles += attn ? page_attn_tiles(b.runs_host[4 * i + 1], geometry(L)) : latent_attn_tiles(b.runs_host[4 * i + 1], L.heads);
+    return p;
+}
+// floats of key-split workspace a layer's attention needs
+size_t attn_ws(const pie_stack *s, const pie_stack_batch &b, const Plan &plan, const pie_stack_layer &L) {
+    if (L.mixer == PIE_MIXER_DELTA) return 0;
+    const ShortPart p = short_part(s, b, plan, L);
+    if (!p.tiles) return 0;
+    const int splits = plan_splits(b, L, p.tiles);
+    return L.mixer == PIE_MIXER_ATTENTION ? page_attn_ws_floats(p.M, geometry(L), splits) : latent_attn_ws_floats(p.M, L.heads, L.rank, splits);
 }
 
 struct Pass {
@@ -457,21 +549,46 @@ struct Pass {
         if (!rc)
             rc = w16l_gemm_launch(PIE_BF16, w, x, ldx, M, N, K, swiglu ? nullptr : y, s->gemm_ws.p, st, nullptr, swiglu ? y : nullptr, nullptr, ldy), ++launches;
     }
-    // x += post(y); h = next(x)
-    void residual(const pie_point_norm &post, const PointNorm &next) {
+    // x += post(y); h = next(x) over y = s->y (bf16; many rows) or s->y32
+    void update(const pie_stack_norm &post, const pie_stack_norm &next, const u16 *bias = nullptr) {
         if (rc) return;
         const int W = s->cfg.width, W64 = up64(W), WA = act_stride(W);
-        hipLaunchKernelGGL(k_point_residual, dim3((unsigned)((W + 1023) / 1024), (unsigned)b.n_rows), dim3(256), 0, st, (const u16 *)s->y.p, W, norm_of(post), next, s->x.p, W64,
-                           (u16 *)s->h.p, WA, W);
-        if (hipGetLastError() != hipSuccess) rc = pie::fail(PIE_E_HIP, "residual launch failed");
+        if (plan.big && pointwise(post) && pointwise(next) && !bias) {
+            hipLaunchKernelGGL(k_point_residual, dim3((unsigned)((W + 1023) / 1024), (unsigned)b.n_rows), dim3(256), 0, st, (const u16 *)s->y.p, W, norm_of(post), norm_of(next), s->x.p, W64,
+                               (u16 *)s->h.p, WA, W);
+            if (hipGetLastError() != hipSuccess) rc = pie::fail(PIE_E_HIP, "residual launch failed");
+        } else {
+            RowUpdateArgs a = {};
+            a.y = plan.big ? (const void *)s->y.p : s->y32.p, a.y32 = !plan.big, a.ldy = plan.big ? W : W64, a.bias = bias;
+            a.post = row_norm_of(post), a.next = row_norm_of(next), a.x = s->x.p, a.ldx = W64, a.h = s->h.p, a.ldh = WA, a.M = b.n_rows, a.W = W;
+            rc = row_update_launch(s->cfg.dtype, a, st);
+        }
         ++launches;
+    }
+    // a sublayer's last product [W, K], its norm, the residual sum and the next sublayer's norm
+    void output(const void *w, const void *x, int ldx, int K, const pie_stack_norm &post, const pie_stack_norm &next, const u16 *bias = nullptr) {
+        const int W = s->cfg.width, W64 = up64(W), WA = act_stride(W), M = b.n_rows;
+        if (plan.big) {
+            gemm(w, x, ldx, M, W, K, s->y.p, W);
+            return update(post, next, bias);
+        }
+        RowsArgs o = {};
+        o.m = {(const char *)w, W, K, x, ldx, s->y32.p, W64};
+        o.M = M;
+        if (pointwise(post) && pointwise(next) && !bias) {
+            o.epi = ROWS_RESIDUAL, o.res = s->x.p, o.ld_res = W64, o.post = norm_of(post), o.next = norm_of(next), o.h = s->h.p, o.ldh = WA;
+            return linear(o);
+        }
+        o.epi = ROWS_SCALE_F32, o.scale = 1.0f;
+        linear(o);
+        update(post, next, bias);
     }
     void linear(const RowsArgs &a, int batches = 1) {
         if (!rc) rc = rows_gemm_launch(s->cfg.dtype, a, batches, st), ++launches;
     }
 };
 
-void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const PointNorm &next) {
+void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm &next) {
     pie_stack *s = p.s;
     const pie_stack_batch &b = p.b;
     const int W = s->cfg.width, W64 = up64(W), WA = act_stride(W), D8 = up8(L.dim), V8 = up8(L.vdim), R8 = up8(L.rank), H = L.heads, NI = H * D8 + R8, KO = H * V8, LO = act_stride(KO);
@@ -494,8 +611,9 @@ void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const PointNorm &ne
     const LatentAppend append = {p.plan.big && !two ? (const void *)((const u16 *)s->q.p + H * D8) : s->c_raw.p, p.plan.big, p.plan.big && !two ? NI : R8, L.c_norm, L.eps, b.n_rows,
                                  L.rank, R8, b.pos, b.row_seq, b.table, b.table_width, (int)b.n_pages, b.n_seqs, b.slabs[li]};
     if (p.plan.big) p.rc = latent_append_launch(dt, append, p.st), ++p.launches;  // (few rows: rides in the next launch)
-    const bool spell = p.plan.long_tiles && spelled_out(L);
-    const int M = spell ? p.plan.short_rows : b.n_rows, runs = spell ? p.plan.short_runs : b.n_runs;
+    const bool spell = p.plan.long_rows && spelled_out(L);
+    const ShortPart sp = short_part(s, b, p.plan, L);
+    const int M = sp.M, runs = sp.runs;
     if (M > 0) {  // the latent form
         RowsArgs k = {};
         k.m = {(const char *)L.w_uk, L.rank, L.dim, s->q.p, LQ, s->ql.p, H * R8};
@@ -505,7 +623,7 @@ void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const PointNorm &ne
         LatentAttnArgs t = {};
         t.q = s->ql.p, t.slab = b.slabs[li], t.table = b.table, t.table_width = b.table_width, t.n_pages = (int)b.n_pages, t.n_seqs = b.n_seqs, t.pos = b.pos;
         t.runs = (const RowRun *)b.runs, t.n_runs = runs, t.single = runs == M, t.row_seq = b.row_seq;
-        t.n_tiles = stack_tiles(b.runs_host, runs, H);
+        t.n_tiles = sp.tiles;
         t.H = H, t.R = L.rank, t.ldr = R8, t.M = M, t.window = L.window, t.scale = L.scale, t.splits = plan_splits(b, L, t.n_tiles), t.ws = s->attn_ws.p, t.out = s->oc.p;
         const bool merge = t.splits > 1 && M <= MERGE_ROWS && R8 <= MERGE_LDR && dt == PIE_BF16 && L.rank <= 1024;  // few rows: the next launch merges the key splits itself
         t.combine = !merge;
@@ -522,62 +640,128 @@ void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const PointNorm &ne
         p.rc = latent_gather_launch(lr, n_long, n_ctx, L.window, b.table, b.table_width, b.n_seqs, (int)b.n_pages, b.slabs[li], R8, s->ctx.p, LC, p.st);
         p.gemm(L.w_kv, s->ctx.p, LC, n_ctx, nkv, L.rank, s->kv.p, nkv);
         WindowAttnArgs w = {(const u16 *)s->q.p, (const u16 *)s->kv.p, (u16 *)s->o.p, LQ, nkv, LO, H, D8, V8, L.window, L.scale, lr, n_long};
-        if (!p.rc) p.rc = window_attn_launch(w, p.plan.long_tiles, p.st), p.launches += 2;
+        int tiles = 0;
+        for (int i = p.plan.short_runs; i < b.n_runs; ++i) tiles += (b.runs_host[4 * i + 1] + 127) / 128;
+        if (!p.rc) p.rc = window_attn_launch(w, tiles, p.st), p.launches += 2;
     }
-    if (p.plan.big) {
-        p.gemm(L.w_o, s->o.p, LO, b.n_rows, W, KO, s->y.p, W);
-        p.residual(L.post1, next);
-    } else {
-        RowsArgs o = {};
-        o.m = {(const char *)L.w_o, W, KO, s->o.p, LO, nullptr, 0};
-        o.M = b.n_rows, o.epi = ROWS_RESIDUAL, o.res = s->x.p, o.ld_res = W64, o.post = norm_of(L.post1), o.next = next, o.h = s->h.p, o.ldh = WA;
-        p.linear(o);
-    }
+    p.output(L.w_o, s->o.p, LO, KO, L.post1, next);
 }
 
-void feed_forward(Pass &p, int li, const pie_stack_layer &L, const PointNorm &next) {
+// y = h . W^T in the stack's dtype
+void project(Pass &p, const void *w, int N, void *y) {
+    pie_stack *s = p.s;
+    const int W = s->cfg.width, WA = act_stride(W);
+    if (p.plan.big) return p.gemm(w, s->h.p, WA, p.b.n_rows, N, W, y, N);
+    RowsArgs a = {};
+    a.m = {(const char *)w, N, W, s->h.p, WA, y, N};
+    a.M = p.b.n_rows, a.epi = ROWS_STORE;
+    p.linear(a);
+}
+
+void attention_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm &next) {
+    pie_stack *s = p.s;
+    const pie_stack_batch &b = p.b;
+    const int NI = in_columns(L), KO = out_columns(L), LO = act_stride(KO), dt = s->cfg.dtype;
+    const bool own = L.kv_from < 0;
+    const KvGeometry geo = geometry(L);
+    void *slab = b.slabs[own ? li : L.kv_from];
+    const PageTable pages = {b.table, b.table_width, (int)b.n_pages, b.n_seqs};
+    project(p, L.w_in, NI, s->q.p);
+    if (p.rc) return;
+    KvPrepArgs k = {};
+    k.raw = s->q.p, k.ld = NI, k.M = b.n_rows, k.bias = (const u16 *)L.in_bias, k.geo = geo, k.own = own, k.value_norm = L.value_norm != 0;
+    k.q_norm = L.q_norm, k.k_norm = L.k_norm, k.eps = L.eps, k.freq = L.rot_freq, k.rot_dims = L.rot_dims, k.rot_gain = L.rot_gain;
+    k.pos = b.pos, k.row_seq = b.row_seq, k.pages = pages, k.slab = slab;
+    p.rc = kv_prep_launch(dt, k, p.st), ++p.launches;
+    PageAttnArgs a = {};
+    a.q = s->q.p, a.ldq = NI, a.slab = slab, a.pages = pages, a.geo = geo, a.pos = b.pos, a.row_seq = b.row_seq, a.runs = (const RowRun *)b.runs;
+    a.window = L.window, a.scale = L.scale, a.sink = L.sink, a.out = s->o.p, a.ld_out = LO, a.ws = s->attn_ws.p;
+    if (L.out_gate) {
+        const int at = NI - up8(L.heads);
+        a.gate = (const char *)s->q.p + at * esize(s), a.ldg = NI, a.gate_bias = L.in_bias ? (const u16 *)L.in_bias + at : nullptr;
+    }
+    const ShortPart sp = short_part(s, b, p.plan, L);
+    a.n_runs = sp.runs, a.n_tiles = sp.tiles, a.M = sp.M, a.single = sp.runs == sp.M, a.splits = plan_splits(b, L, sp.tiles);
+    if (!p.rc && sp.M > 0) p.rc = page_attn_launch(dt, a, p.st), p.launches += page_attn_mfma(dt, geo) && a.splits > 1 ? 2 : 1;
+    if (!p.rc && sp.M < b.n_rows) {
+        a.runs += sp.runs, a.n_runs = b.n_runs - sp.runs, a.n_tiles = 0, a.M = b.n_rows, a.single = false, a.splits = 1;
+        for (int i = sp.runs; i < b.n_runs; ++i) a.n_tiles += page_attn_long_tiles(b.runs_host[4 * i + 1], geo);
+        p.rc = page_attn_long_launch(a, p.st), ++p.launches;
+    }
+    p.output(L.w_o, s->o.p, LO, KO, L.post1, next, (const u16 *)L.o_bias);
+}
+
+void delta_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm &next) {
+    pie_stack *s = p.s;
+    const pie_stack_batch &b = p.b;
+    const int NI = in_columns(L), KO = out_columns(L), LO = act_stride(KO);
+    project(p, L.w_in, NI, s->q.p);
+    if (p.rc) return;
+    DeltaArgs d = {};
+    d.raw = s->q.p, d.ld = NI, d.M = b.n_rows, d.H = L.heads, d.D = L.dim, d.D8 = up8(L.dim), d.rank = L.rank, d.R8 = up8(L.rank), d.bias = (const u16 *)L.in_bias;
+    d.w_decay = (const u16 *)L.w_decay, d.decay_bias = L.decay_bias, d.o_norm = L.o_norm, d.decay_scale = L.decay_scale, d.unit_eps = L.unit_eps, d.eps = L.eps;
+    d.pos = b.pos, d.row_seq = b.row_seq, d.slots = b.slots, d.n_seqs = b.n_seqs, d.n_slots = (int)b.n_slots, d.runs = (const RowRun *)b.runs, d.n_runs = b.n_runs;
+    d.state = b.states[li], d.out = s->o.p, d.ld_out = LO;
+    p.rc = delta_step_launch(s->cfg.dtype, d, p.st), ++p.launches;
+    p.output(L.w_o, s->o.p, LO, KO, L.post1, next);
+}
+
+void feed_forward(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm &next) {
     pie_stack *s = p.s;
     const int M = p.b.n_rows, W = s->cfg.width, W64 = up64(W), WA = act_stride(W), F = L.ff_size, FA = act_stride(F), dt = s->cfg.dtype;
     if (L.ff == PIE_FF_RELU2) {
         if (p.plan.big) {
             if (!p.rc) p.rc = w16l_relu2_launch(L.w_up, s->h.p, WA, M, F, W, s->act.p, FA, p.st), ++p.launches;
-            p.gemm(L.w_down, s->act.p, FA, M, W, F, s->y.p, W);
-            p.residual(L.post2, next);
-            return;
+        } else {
+            RowsArgs u = {};
+            u.m = {(const char *)L.w_up, F, W, s->h.p, WA, s->act.p, FA};
+            u.M = M, u.epi = ROWS_RELU2;
+            p.linear(u);
         }
-        RowsArgs u = {};
-        u.m = {(const char *)L.w_up, F, W, s->h.p, WA, s->act.p, FA};
-        u.M = M, u.epi = ROWS_RELU2;
-        p.linear(u);
-        RowsArgs d = {};
-        d.m = {(const char *)L.w_down, W, F, s->act.p, FA, nullptr, 0};
-        d.M = M, d.epi = ROWS_RESIDUAL, d.res = s->x.p, d.ld_res = W64, d.post = norm_of(L.post2), d.next = next, d.h = s->h.p, d.ldh = WA;
-        p.linear(d);
-        return;
+        return p.output(L.w_down, s->act.p, FA, F, L.post2, next);
     }
     const RouteLayer &r = s->route[li];
     const int S = L.shared_size, SA = act_stride(S);
     const size_t gu_stride = rows_weight_bytes(dt, 2 * F, W), dn_stride = rows_weight_bytes(dt, W, F);
+    const bool clipped = L.act == PIE_ACT_CLIPPED;
+    if (L.ff == PIE_FF_ROUTED_MOE) {  // logits, then the choice and its row lists
+        RowsArgs z = {};
+        z.m = {(const char *)L.w_router, L.experts, W, s->h.p, WA, s->logits_e.p, up8(L.experts)};
+        z.M = M, z.epi = ROWS_SCALE_F32, z.scale = 1.0f;
+        p.linear(z);
+        if (p.rc) return;
+        const RouteLayer *dev = s->route_dev.p + s->route_at[li];
+        const bool few = M <= 64;
+        if (!few) {
+            hipLaunchKernelGGL(k_route_pick, dim3((unsigned)((M + 3) / 4)), dim3(256), 0, p.st, dev, M);
+            ++p.launches;
+        }
+        hipLaunchKernelGGL(k_route, dim3(1), dim3(1024), (size_t)2 * L.experts * 4, p.st, dev, p.b.ids, M, s->cfg.vocab, few);
+        if (hipGetLastError() != hipSuccess) p.rc = pie::fail(PIE_E_HIP, "routing launch failed");
+        ++p.launches;
+    }
     CombineArgs c = {};
-    c.part = s->part.p, c.part_s = s->part_s.p, c.ldp = W64, c.ldp_s = p.plan.big && !(W & 3) ? W : W64, c.place = r.place, c.top = L.top, c.W = W, c.gate = S ? L.shared_gate : nullptr;
-    c.pre = norm_of(L.pre2), c.post = norm_of(L.post2), c.next = next, c.x = s->x.p, c.ldx = W64, c.h = s->h.p, c.ldh = WA;
+    c.part = s->part.p, c.part_s = s->part_s.p, c.ldp = W64, c.ldp_s = p.plan.big && !(W & 3) ? W : W64, c.place = r.place, c.weight = r.weight, c.top = L.top, c.W = W, c.gate = S ? L.shared_gate : nullptr;
+    c.pre = norm_of(L.pre2), c.post = norm_of(L.post2), c.next = norm_of(next), c.x = s->x.p, c.ldx = W64, c.h = s->h.p, c.ldh = WA;
+    const bool elementwise = pointwise(L.post2) && pointwise(next);
     const dim3 cg((unsigned)M), cb((unsigned)std::min(1024, ((W + 3) / 4 + 63) / 64 * 64));
     if (p.plan.big) {
         const int tr = route_tile_rows(M, L.top, L.experts), tm = route_max_tiles(M, L.top, L.experts), rb = route_block(M, L.top, L.experts);
-        if (!p.rc) p.rc = w16l_grouped_launch(L.w_gate_up, gu_stride, s->h.p, WA, (size_t)M, r.list, r.tiles, tm, rb, tr, 2 * F, W, s->act_e.p, FA, true, p.st);
-        if (!p.rc) p.rc = w16l_grouped_launch(L.w_expert_down, dn_stride, s->act_e.p, FA, (size_t)M * L.top, nullptr, r.tiles, tm, rb, tr, W, F, s->part.p, W64, false, p.st);
+        if (!p.rc) p.rc = w16l_grouped_launch(L.w_gate_up, gu_stride, s->h.p, WA, (size_t)M, r.list, r.tiles, tm, rb, tr, 2 * F, W, s->act_e.p, FA, clipped ? MFMA_ACT_CLIPPED : MFMA_ACT_SWIGLU, L.act_alpha, L.act_limit,
+                                               p.st);
+        if (!p.rc) p.rc = w16l_grouped_launch(L.w_expert_down, dn_stride, s->act_e.p, FA, (size_t)M * L.top, nullptr, r.tiles, tm, rb, tr, W, F, s->part.p, W64, MFMA_ACT_NONE, 0.0f, 0.0f, p.st);
         p.launches += 2;
         if (S) {
             p.gemm(L.s_gate_up, s->h.p, WA, M, 2 * S, W, s->act_s.p, SA, true);
             p.gemm(L.s_down, s->act_s.p, SA, M, W, S, s->part_s.p, c.ldp_s);
         }
         if (p.rc) return;
-        hipLaunchKernelGGL((k_moe_combine<ElemBF16, ElemBF16>), cg, cb, 0, p.st, c);
+        if (elementwise) hipLaunchKernelGGL((k_moe_combine<ElemBF16, ElemBF16>), cg, cb, 0, p.st, c);
     } else {
         const int groups = (int)std::min((long)L.experts, (long)M * L.top) + (S ? 1 : 0);
         RowsArgs u = {};
         u.m = {(const char *)L.w_gate_up, 2 * F, W, s->h.p, WA, s->act_e.p, FA};
-        u.M = M, u.epi = ROWS_SILU_MUL, u.w_batch = gu_stride, u.active = r.active, u.offset = r.offset, u.list = r.list, u.gather = true;
+        u.M = M, u.epi = clipped ? ROWS_CLIP_MUL : ROWS_SILU_MUL, u.act_alpha = L.act_alpha, u.act_limit = L.act_limit, u.w_batch = gu_stride, u.active = r.active, u.offset = r.offset, u.list = r.list, u.gather = true;
         if (S) u.shared = {(const char *)L.s_gate_up, 2 * S, W, s->h.p, WA, s->act_s.p, SA};
         p.linear(u, groups);
         RowsArgs d = {};
@@ -586,34 +770,49 @@ void feed_forward(Pass &p, int li, const pie_stack_layer &L, const PointNorm &ne
         if (S) d.shared = {(const char *)L.s_down, W, S, s->act_s.p, SA, s->part_s.p, W64};
         p.linear(d, groups);
         if (p.rc) return;
-        if (dt == PIE_F32) hipLaunchKernelGGL((k_moe_combine<ElemF32, ElemF32>), cg, cb, 0, p.st, c);
+        if (!elementwise) {
+        } else if (dt == PIE_F32) hipLaunchKernelGGL((k_moe_combine<ElemF32, ElemF32>), cg, cb, 0, p.st, c);
         else hipLaunchKernelGGL((k_moe_combine<ElemBF16, ElemF32>), cg, cb, 0, p.st, c);
     }
-    if (hipGetLastError() != hipSuccess) p.rc = pie::fail(PIE_E_HIP, "expert combine launch failed");
+    if (!elementwise) {
+        RowUpdateArgs a = {};
+        a.y = s->part.p, a.y32 = !p.plan.big, a.ldy = W64, a.place = r.place, a.weight = r.weight, a.top = L.top;
+        a.post = row_norm_of(L.post2), a.next = row_norm_of(next), a.x = s->x.p, a.ldx = W64, a.h = s->h.p, a.ldh = WA, a.M = M, a.W = W;
+        p.rc = row_update_launch(dt, a, p.st);
+    } else if (hipGetLastError() != hipSuccess) p.rc = pie::fail(PIE_E_HIP, "expert combine launch failed");
     ++p.launches;
 }
 
 int stack_enqueue(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipStream_t st) {
     const int M = b.n_rows, W = s->cfg.width, W64 = up64(W), WA = act_stride(W), V = s->cfg.vocab, n = s->cfg.n_layers, dt = s->cfg.dtype;
     Pass p{s, b, plan, st};
-    if (s->n_route) {
-        hipLaunchKernelGGL(k_route, dim3((unsigned)s->n_route), dim3(1024), (size_t)s->route_lds, st, s->route_dev.p, b.ids, M, V);
+    if (s->n_table) {
+        hipLaunchKernelGGL(k_route, dim3((unsigned)s->n_table), dim3(1024), (size_t)s->route_lds, st, s->route_dev.p, b.ids, M, V, false);
         PIE_LAUNCH_CHECK();
         ++p.launches;
     }
-    const PointNorm fin = norm_of(s->cfg.final_norm), first = n ? norm_of(s->layers[0].pre1) : fin;
+    const pie_stack_norm &fin = s->cfg.final_norm, &first = n ? s->layers[0].pre1 : fin;
     const dim3 ge((unsigned)((W + 1023) / 1024), (unsigned)M);
     if (dt == PIE_F32)
-        hipLaunchKernelGGL(k_stack_embed<ElemF32>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, first, s->x.p, W64, (float *)s->h.p, WA);
+        hipLaunchKernelGGL(k_stack_embed<ElemF32>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, s->cfg.embed_scale, !pointwise(first), norm_of(first), s->x.p, W64,
+                           (float *)s->h.p, WA);
     else
-        hipLaunchKernelGGL(k_stack_embed<ElemBF16>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, first, s->x.p, W64, (u16 *)s->h.p, WA);
+        hipLaunchKernelGGL(k_stack_embed<ElemBF16>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, s->cfg.embed_scale, !pointwise(first), norm_of(first), s->x.p, W64,
+                           (u16 *)s->h.p, WA);
     PIE_LAUNCH_CHECK();
     ++p.launches;
+    if (first.kind == PIE_NORM_RMS) {
+        RowUpdateArgs a = {};
+        a.next = row_norm_of(first), a.x = s->x.p, a.ldx = W64, a.h = s->h.p, a.ldh = WA, a.M = M, a.W = W;
+        p.rc = row_update_launch(dt, a, st), ++p.launches;
+    }
     for (int i = 0; i < n && !p.rc; ++i) {
         const pie_stack_layer &L = s->layers[i];
-        const PointNorm after = i + 1 < n ? norm_of(s->layers[i + 1].pre1) : fin;
-        latent_mixer(p, i, L, L.ff == PIE_FF_NONE ? after : norm_of(L.pre2));
-        if (L.ff != PIE_FF_NONE) feed_forward(p, i, L, after);
+        const pie_stack_norm &after = i + 1 < n ? s->layers[i + 1].pre1 : fin, &next = L.ff == PIE_FF_NONE ? after : L.pre2;
+        if (L.mixer == PIE_MIXER_LATENT) latent_mixer(p, i, L, next);
+        else if (L.mixer == PIE_MIXER_ATTENTION) attention_mixer(p, i, L, next);
+        else delta_mixer(p, i, L, next);
+        if (L.ff != PIE_FF_NONE && !p.rc) feed_forward(p, i, L, after);
         if (b.tap && !p.rc)
             PIE_HIP_TRY(hipMemcpy2DAsync(b.tap + (size_t)i * M * W, (size_t)W * 4, s->x.p, (size_t)W64 * 4, (size_t)W * 4, (size_t)M, hipMemcpyDeviceToDevice, st));
     }
@@ -635,6 +834,31 @@ int stack_enqueue(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
     return p.rc;
 }
 
+bool norm_ok(const pie_stack_norm &n) {
+    return n.kind == PIE_NORM_NONE || (n.kind == PIE_NORM_DYN_TANH && n.w && n.b) || (n.kind == PIE_NORM_RMS && n.w);
+}
+int mixer_ok(const pie_stack *s, int i, const pie_stack_layer &L) {
+    PIE_REQUIRE(L.heads > 0 && L.dim > 0 && L.w_in && L.w_o && norm_ok(L.pre1) && norm_ok(L.post1), PIE_E_ARG, "pie_stack_set_layer: missing mixer weights or sizes");
+    if (L.mixer == PIE_MIXER_LATENT) {
+        PIE_REQUIRE(L.vdim > 0 && L.rank > 0 && L.rank <= 2048, PIE_E_SHAPE, "pie_stack_set_layer: bad mixer sizes (kv_rank at most 2048)");
+        PIE_REQUIRE(L.w_uk && L.w_uv && L.c_norm, PIE_E_ARG, "pie_stack_set_layer: missing mixer weights");
+    } else if (L.mixer == PIE_MIXER_ATTENTION) {
+        PIE_REQUIRE(L.vdim > 0 && L.kv_heads > 0 && L.heads % L.kv_heads == 0 && L.dim <= PAGE_ATTN_ROWS_DIM && L.vdim <= PAGE_ATTN_ROWS_DIM, PIE_E_SHAPE,
+                    "pie_stack_set_layer: bad mixer sizes (heads of at most 1024 numbers, a multiple of kv_heads)");
+        PIE_REQUIRE(L.rot_dims >= 0 && L.rot_dims <= L.dim && L.rot_dims % 2 == 0 && (L.rot_dims == 0 || L.rot_freq), PIE_E_SHAPE, "pie_stack_set_layer: bad rotation");
+        if (L.kv_from >= 0) {
+            PIE_REQUIRE(L.kv_from < i && s->have[L.kv_from], PIE_E_ARG, "pie_stack_set_layer: kv_from names an earlier layer");
+            const pie_stack_layer &F = s->layers[L.kv_from];
+            PIE_REQUIRE(F.mixer == PIE_MIXER_ATTENTION && F.kv_from < 0 && F.kv_heads == L.kv_heads && F.dim == L.dim && F.vdim == L.vdim, PIE_E_SHAPE,
+                        "pie_stack_set_layer: kv_from names an attention layer with keys and values of its own, of the same sizes");
+        }
+    } else if (L.mixer == PIE_MIXER_DELTA) {
+        PIE_REQUIRE(L.dim <= DELTA_MAX_DIM && L.rank > 0 && L.rank <= DELTA_MAX_RANK, PIE_E_SHAPE, "pie_stack_set_layer: bad mixer sizes (delta rule: dim at most 256, rank at most 1024)");
+        PIE_REQUIRE(L.w_decay && L.decay_bias && L.o_norm, PIE_E_ARG, "pie_stack_set_layer: missing mixer weights");
+    } else PIE_REQUIRE(false, PIE_E_ARG, "pie_stack_set_layer: unknown mixer");
+    return PIE_OK;
+}
+
 }  // namespace
 
 extern "C" {
@@ -643,7 +867,7 @@ int pie_stack_create(const pie_stack_config *cfg, pie_stack **out) {
     PIE_REQUIRE(cfg && out, PIE_E_ARG, "pie_stack_create: null pointer");
     PIE_REQUIRE(cfg->dtype == PIE_BF16 || cfg->dtype == PIE_F32, PIE_E_ARG, "pie_stack_create: dtype must be PIE_BF16 or PIE_F32");
     PIE_REQUIRE(cfg->width > 0 && cfg->vocab > 0 && cfg->n_layers >= 0, PIE_E_SHAPE, "pie_stack_create: bad sizes");
-    PIE_REQUIRE(cfg->embed && cfg->head && cfg->final_norm.w && cfg->final_norm.b, PIE_E_ARG, "pie_stack_create: missing weights");
+    PIE_REQUIRE(cfg->embed && cfg->head && norm_ok(cfg->final_norm), PIE_E_ARG, "pie_stack_create: missing weights");
     pie_stack *s = new (std::nothrow) pie_stack();
     PIE_REQUIRE(s, PIE_E_HIP, "pie_stack_create: out of host memory");
     s->cfg = *cfg;
@@ -659,20 +883,18 @@ int pie_stack_destroy(pie_stack *s) {
 
 int pie_stack_set_layer(pie_stack *s, int i, const pie_stack_layer *L) {
     PIE_REQUIRE(s && L && i >= 0 && i < s->cfg.n_layers, PIE_E_ARG, "pie_stack_set_layer: bad argument");
-    auto norm_ok = [](const pie_point_norm &n) { return n.w && n.b; };
-    PIE_REQUIRE(L->mixer == PIE_MIXER_LATENT, PIE_E_ARG, "pie_stack_set_layer: unknown mixer");
-    PIE_REQUIRE(L->heads > 0 && L->dim > 0 && L->vdim > 0 && L->rank > 0 && L->rank <= 2048, PIE_E_SHAPE, "pie_stack_set_layer: bad mixer sizes (kv_rank at most 2048)");
-    PIE_REQUIRE(L->w_in && L->w_uk && L->w_uv && L->w_o && L->c_norm && norm_ok(L->pre1) && norm_ok(L->post1), PIE_E_ARG, "pie_stack_set_layer: missing mixer weights");
+    if (const int rc = mixer_ok(s, i, *L)) return rc;
     PIE_REQUIRE(L->ff == PIE_FF_NONE || (norm_ok(L->pre2) && norm_ok(L->post2) && L->ff_size > 0 && L->ff_size % 8 == 0 && L->shared_size % 8 == 0), PIE_E_ARG, "pie_stack_set_layer: missing feed-forward norms");
     if (L->ff == PIE_FF_RELU2) PIE_REQUIRE(L->w_up && L->w_down, PIE_E_ARG, "pie_stack_set_layer: missing dense weights");
-    else if (L->ff == PIE_FF_TABLE_MOE) {
+    else if (is_moe(*L)) {
         PIE_REQUIRE(L->experts > 0 && L->experts <= 8192 && L->top > 0 && L->top <= L->experts, PIE_E_SHAPE, "pie_stack_set_layer: bad expert counts");
-        PIE_REQUIRE(L->table && L->w_gate_up && L->w_expert_down, PIE_E_ARG, "pie_stack_set_layer: missing expert weights");
-        PIE_REQUIRE(L->shared_size == 0 || (L->shared_size > 0 && L->s_gate_up && L->s_down && L->shared_gate), PIE_E_ARG, "pie_stack_set_layer: missing shared expert");
+        PIE_REQUIRE((L->ff == PIE_FF_TABLE_MOE ? L->table != nullptr : L->w_router && L->correction) && L->w_gate_up && L->w_expert_down, PIE_E_ARG, "pie_stack_set_layer: missing expert weights");
+        PIE_REQUIRE(L->act == PIE_ACT_SILU || L->act == PIE_ACT_CLIPPED, PIE_E_ARG, "pie_stack_set_layer: unknown activation");
+        PIE_REQUIRE(L->shared_size == 0 || (L->shared_size > 0 && L->s_gate_up && L->s_down && L->shared_gate && L->act == PIE_ACT_SILU && pointwise(L->pre2) && pointwise(L->post2)),
+                    PIE_E_ARG, "pie_stack_set_layer: a shared expert needs its weights, SiLU and element-wise norms");
     } else PIE_REQUIRE(L->ff == PIE_FF_NONE, PIE_E_ARG, "pie_stack_set_layer: unknown feed-forward");
-    s->n_route += (L->ff == PIE_FF_TABLE_MOE) - (s->route[i].experts > 0);
     s->route[i] = RouteLayer{};
-    if (L->ff == PIE_FF_TABLE_MOE) s->route[i].table = L->table, s->route[i].top = L->top, s->route[i].experts = L->experts;
+    if (is_moe(*L)) s->route[i].table = L->ff == PIE_FF_TABLE_MOE ? L->table : nullptr, s->route[i].correction = L->correction, s->route[i].top = L->top, s->route[i].experts = L->experts;
     s->route_rows = 0;
     s->layers[i] = *L, s->have[i] = 1;
     s->drop_graphs();
@@ -690,7 +912,15 @@ int pie_logprobs_argmax_f32(const float *logits, int rows, int V, float *logprob
     return PIE_OK;
 }
 
-int pie_stack_page_row(const pie_stack *s, int i) { return s && i >= 0 && i < s->cfg.n_layers && s->have[i] ? up8(s->layers[i].rank) : 0; }
+int pie_stack_page_row(const pie_stack *s, int i) {
+    if (!s || i < 0 || i >= s->cfg.n_layers || !s->have[i]) return 0;
+    const pie_stack_layer &L = s->layers[i];
+    if (L.mixer == PIE_MIXER_LATENT) return up8(L.rank);
+    return L.mixer == PIE_MIXER_ATTENTION && L.kv_from < 0 ? (int)(geometry(L).page_elems() / PAGE_TOKENS) : 0;
+}
+size_t pie_stack_state_floats(const pie_stack *s, int i) {
+    return s && i >= 0 && i < s->cfg.n_layers && s->have[i] && s->layers[i].mixer == PIE_MIXER_DELTA ? (size_t)s->layers[i].heads * s->layers[i].dim * s->layers[i].dim : 0;
+}
 size_t pie_stack_page_bytes(const pie_stack *s, int i) { return (size_t)pie_stack_page_row(s, i) * PAGE_TOKENS * (s ? esize(s) : 0); }
 int pie_stack_launches(const pie_stack *s) { return s ? s->launches : 0; }
 
@@ -712,18 +942,15 @@ int pie_stack_forward(pie_stack *s, const pie_stack_batch *bp, int flags, void *
         at += r[1];
     }
     PIE_REQUIRE(at == b.n_rows, PIE_E_ARG, "pie_stack_forward: the runs must cover the rows in order");
-    for (int i = 0; i < s->cfg.n_layers; ++i) PIE_REQUIRE(b.slabs[i], PIE_E_ARG, "pie_stack_forward: a layer has no pages");
+    for (int i = 0; i < s->cfg.n_layers; ++i) {
+        PIE_REQUIRE(b.slabs[i] || !pie_stack_page_row(s, i), PIE_E_ARG, "pie_stack_forward: a layer has no pages");
+        PIE_REQUIRE(!pie_stack_state_floats(s, i) || (b.slots && b.states && b.states[i] && b.n_slots > 0), PIE_E_ARG, "pie_stack_forward: a recurrent layer has no state slots");
+    }
     const Plan plan = plan_pass(s, b);
     int rc = stack_reserve(s, b, plan, st);
     if (rc) return rc;
     size_t ws = 0;
-    for (const pie_stack_layer &L : s->layers)
-    {
-        const bool spell = plan.long_tiles && spelled_out(L);
-        const int M = spell ? plan.short_rows : b.n_rows, runs = spell ? plan.short_runs : b.n_runs;
-        const int tiles = stack_tiles(b.runs_host, runs, L.heads);
-        if (tiles) ws = std::max(ws, latent_attn_ws_floats(M, L.heads, L.rank, plan_splits(b, L, tiles)));
-    }
+    for (const pie_stack_layer &L : s->layers) ws = std::max(ws, attn_ws(s, b, plan, L));
     bool moved = false;
     if ((rc = s->attn_ws.need(ws, &moved))) return rc;
     if (moved) s->drop_graphs();
@@ -731,7 +958,8 @@ int pie_stack_forward(pie_stack *s, const pie_stack_batch *bp, int flags, void *
 
     GraphKey key;
     key.b = b;
-    key.b.slabs = nullptr, key.b.runs_host = nullptr;
+    key.b.slabs = nullptr, key.b.runs_host = nullptr, key.b.states = nullptr;
+    if (b.states) key.states.assign(b.states, b.states + s->cfg.n_layers);
     key.slabs.assign(b.slabs, b.slabs + s->cfg.n_layers), key.runs.assign(b.runs_host, b.runs_host + 4 * b.n_runs);
     GraphSlot *slot = nullptr;
     for (GraphSlot &g : s->graphs)

@@ -30,8 +30,9 @@ __device__ __forceinline__ u32 w4m_pack<F16>(float lo, float hi) {
 // bias (nullable): T(T(acc) + bias), like the text tower's Linear; SWIGLU: columns (2 i, 2 i + 1) = (gate_i, up_i) -> T(T(silu(g)) * u), N / 2 wide.
 // The caller has made sure nobody still reads the LDS region (a barrier after the K loop).
 // ACT: MFMA_ACT_NONE, MFMA_ACT_SWIGLU (the bool true of the kernels that know only that one), MFMA_ACT_RELU2 (max(T(v), 0)^2, taken where the tile leaves LDS: next to
-// the accumulators it does not fit the registers).
-enum { MFMA_ACT_NONE = 0, MFMA_ACT_SWIGLU = 1, MFMA_ACT_RELU2 = 2 };
+// the accumulators it does not fit the registers), MFMA_ACT_CLIPPED (columns paired as for SWIGLU: g sigmoid(alpha g) (u + 1) with g = min(gate, limit),
+// u = clamp(up, +-limit) of the rounded pair).
+enum { MFMA_ACT_NONE = 0, MFMA_ACT_SWIGLU = 1, MFMA_ACT_RELU2 = 2, MFMA_ACT_CLIPPED = 3 };
 template <class T>
 __device__ __forceinline__ u32 mfma_relu2(u32 w) {
     const float a = fmaxf(lo_f32<T>(w), 0.0f), b = fmaxf(hi_f32<T>(w), 0.0f);
@@ -39,8 +40,8 @@ __device__ __forceinline__ u32 mfma_relu2(u32 w) {
 }
 template <class T, int MB, int SW, int ACT>
 __device__ __forceinline__ void mfma_tile_store(const f32x16_t (&acc)[SW][MB], char *ot, int lane, int nt0, int m0, int rows, int N, int ldy, u16 *y,
-                                                const u16 *bias, bool skip_stores = false) {
-    constexpr bool SWIGLU = ACT == MFMA_ACT_SWIGLU;
+                                                const u16 *bias, bool skip_stores = false, float act_alpha = 0.0f, float act_limit = 0.0f) {
+    constexpr bool SWIGLU = ACT == MFMA_ACT_SWIGLU || ACT == MFMA_ACT_CLIPPED;  // two columns make one
     constexpr int MT = 32 * MB;
     constexpr int OB = (SWIGLU ? 32 : 64) * SW;  // output bytes per row of the wave's tile
     constexpr int SL = OB / 8, RPB = 256 / OB;    // 8-byte slots per row; rows per 256-byte bank row
@@ -69,6 +70,14 @@ __device__ __forceinline__ void mfma_tile_store(const f32x16_t (&acc)[SW][MB], c
                 char *row = ot + (32 * mi + n) * OB;
                 if (SWIGLU) {  // two activations, 4 bytes at byte 32 s + 8 q + 4 kh of the row
                     const float g0 = lo_f32<T>(p01), u0 = hi_f32<T>(p01), g1 = lo_f32<T>(p23), u1 = hi_f32<T>(p23);
+                    if constexpr (ACT == MFMA_ACT_CLIPPED) {
+                        auto glu = [&](float g, float u) {
+                            g = fminf(g, act_limit), u = fminf(fmaxf(u, -act_limit), act_limit);
+                            return g / (1.0f + expf(-act_alpha * g)) * (u + 1.0f);
+                        };
+                        *reinterpret_cast<u32 *>(row + (((4 * s + q) ^ sv) << 3) + 4 * kh) = w4m_pack<T>(glu(g0, u0), glu(g1, u1));
+                        continue;
+                    }
                     const u16 o0 = T::from_f32(round_T<T>(g0 / (1.0f + expf(-g0))) * u0), o1 = T::from_f32(round_T<T>(g1 / (1.0f + expf(-g1))) * u1);
                     *reinterpret_cast<u32 *>(row + (((4 * s + q) ^ sv) << 3) + 4 * kh) = (u32)o0 | ((u32)o1 << 16);
                 } else {       // 8 bytes at byte 64 s + 16 q + 8 kh

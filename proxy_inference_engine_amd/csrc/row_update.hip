@@ -1,0 +1,181 @@
+// row_update.hip -- what stands between two sublayers when a norm needs the whole row: x += post(y); h = next(x).
+//
+// One workgroup per row.  y is a sublayer's output (plus a bias), or the weighted sum of a row's experts; the row stays in registers from the first read to
+// the last store, so the norms' sums cost one exchange through LDS each and x, y and h pass through memory once.
+#include "stack_types.hpp"
+
+namespace {
+
+template <int THREADS>
+__device__ __forceinline__ float block_sum(float v, float *red) {  // red: THREADS / 64 floats, free again behind the next barrier
+    v = wave_sum(v);
+    if constexpr (THREADS == 64) return v;
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+    __syncthreads();
+    float s = red[0];
+#pragma unroll
+    for (int i = 1; i < THREADS / 64; ++i) s += red[i];
+    return s;
+}
+
+__device__ __forceinline__ float4 load_quad(const void *p, bool is32, size_t row, int n, int W, int stride) {
+    if (is32) {  // (fp32 rows are padded to a multiple of 64)
+        return *(const float4 *)((const float *)p + row * stride + n);
+    }
+    const u16 *q = (const u16 *)p + row * stride + n;
+    if (!(stride & 3)) {
+        const uint2 v = *(const uint2 *)q;
+        return make_float4(lo_f32<BF16>(v.x), hi_f32<BF16>(v.x), lo_f32<BF16>(v.y), hi_f32<BF16>(v.y));
+    }
+    float e[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) e[i] = n + i < W ? BF16::to_f32(q[i]) : 0.0f;
+    return make_float4(e[0], e[1], e[2], e[3]);
+}
+
+// y[q] <- norm(y[q]) for the row's quads; n0 + 4 THREADS q: first column of quad q
+template <int THREADS, int NQ>
+__device__ __forceinline__ void norm_row(const StackNorm &m, int W, float (&y)[NQ][4], float *red) {
+    const int n0 = threadIdx.x * 4;
+    if (m.kind == PIE_NORM_RMS) {
+        float ss = 0.0f;
+#pragma unroll
+        for (int q = 0; q < NQ; ++q)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) ss = fmaf(y[q][i], y[q][i], ss);
+        const float inv = 1.0f / sqrtf(block_sum<THREADS>(ss, red) / (float)W + m.param);
+#pragma unroll
+        for (int q = 0; q < NQ; ++q) {
+            const int n = n0 + 4 * THREADS * q;
+            if (n >= W) break;
+            const float4 w = *(const float4 *)(m.w + n);
+            y[q][0] *= inv * w.x, y[q][1] *= inv * w.y, y[q][2] *= inv * w.z, y[q][3] *= inv * w.w;
+        }
+    } else if (m.kind == PIE_NORM_DYN_TANH) {
+        const PointNorm pn = {m.w, m.b, m.param};
+#pragma unroll
+        for (int q = 0; q < NQ; ++q) {
+            const int n = n0 + 4 * THREADS * q;
+            if (n >= W) break;
+            const float4 v = point_norm4(pn, n, make_float4(y[q][0], y[q][1], y[q][2], y[q][3]));
+            y[q][0] = v.x, y[q][1] = v.y, y[q][2] = v.z, y[q][3] = v.w;
+        }
+    }
+}
+
+template <class E, int THREADS, int NQ>
+__global__ void __launch_bounds__(THREADS) k_row_update(const RowUpdateArgs a) {
+    typedef typename E::type T;
+    __shared__ float red[2][THREADS / 64];
+    const size_t m = blockIdx.x;
+    const int n0 = threadIdx.x * 4;
+    float *x = a.x + m * a.ldx;
+    float xv[NQ][4], y[NQ][4];
+#pragma unroll
+    for (int q = 0; q < NQ; ++q) {
+        const int n = n0 + 4 * THREADS * q;
+        float4 v = make_float4(0, 0, 0, 0);
+        if (n < a.W) v = *(const float4 *)(x + n);
+        xv[q][0] = v.x, xv[q][1] = v.y, xv[q][2] = v.z, xv[q][3] = v.w;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) y[q][i] = 0.0f;
+    }
+    if (a.y) {
+        if (a.place) {
+            constexpr int U = NQ >= 4 ? 4 : 8;  // slots in flight
+            const float share = 1.0f / (float)a.top;
+            for (int s0 = 0; s0 < a.top; s0 += U) {
+                float w[U];
+                int at[U];
+#pragma unroll
+                for (int u = 0; u < U; ++u) {
+                    const size_t i = m * a.top + min(s0 + u, a.top - 1);
+                    at[u] = a.place[i], w[u] = s0 + u < a.top ? (a.weight ? a.weight[i] : share) : 0.0f;
+                }
+#pragma unroll
+                for (int q = 0; q < NQ; ++q) {
+                    const int n = n0 + 4 * THREADS * q;
+                    if (n >= a.W) break;
+                    float4 v[U];
+#pragma unroll
+                    for (int u = 0; u < U; ++u) v[u] = load_quad(a.y, a.y32, at[u], n, a.W, a.ldy);
+#pragma unroll
+                    for (int u = 0; u < U; ++u)
+                        y[q][0] = fmaf(w[u], v[u].x, y[q][0]), y[q][1] = fmaf(w[u], v[u].y, y[q][1]), y[q][2] = fmaf(w[u], v[u].z, y[q][2]), y[q][3] = fmaf(w[u], v[u].w, y[q][3]);
+                }
+            }
+        } else {
+#pragma unroll
+            for (int q = 0; q < NQ; ++q) {
+                const int n = n0 + 4 * THREADS * q;
+                if (n >= a.W) break;
+                const float4 v = load_quad(a.y, a.y32, m, n, a.W, a.ldy);
+                y[q][0] = v.x, y[q][1] = v.y, y[q][2] = v.z, y[q][3] = v.w;
+                if (a.bias)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) y[q][i] += BF16::to_f32(a.bias[min(n + i, a.W - 1)]);
+            }
+        }
+#pragma unroll
+        for (int q = 0; q < NQ; ++q)  // columns past the row's end: nothing
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+                if (n0 + 4 * THREADS * q + i >= a.W) y[q][i] = xv[q][i] = 0.0f;
+        norm_row<THREADS, NQ>(a.post, a.W, y, red[0]);
+#pragma unroll
+        for (int q = 0; q < NQ; ++q) {
+            const int n = n0 + 4 * THREADS * q;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) xv[q][i] += y[q][i];
+            if (n + 4 <= a.W) *(float4 *)(x + n) = make_float4(xv[q][0], xv[q][1], xv[q][2], xv[q][3]);
+            else
+                for (int i = 0; i < a.W - n; ++i) x[n + i] = xv[q][i];
+        }
+    } else {
+#pragma unroll
+        for (int q = 0; q < NQ; ++q)
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+                if (n0 + 4 * THREADS * q + i >= a.W) xv[q][i] = 0.0f;
+    }
+    norm_row<THREADS, NQ>(a.next, a.W, xv, red[1]);
+    T *h = (T *)a.h + m * a.ldh;
+#pragma unroll
+    for (int q = 0; q < NQ; ++q) {
+        const int n = n0 + 4 * THREADS * q;
+        if (n + 4 <= a.W) {
+            if constexpr (sizeof(T) == 2) *(uint2 *)(h + n) = make_uint2(pack2<BF16>(xv[q][0], xv[q][1]), pack2<BF16>(xv[q][2], xv[q][3]));
+            else *(float4 *)(h + n) = make_float4(xv[q][0], xv[q][1], xv[q][2], xv[q][3]);
+        } else
+            for (int i = 0; i < a.W - n; ++i) h[n + i] = E::pack(xv[q][i]);
+    }
+}
+
+template <class E>
+void row_go(const RowUpdateArgs &a, hipStream_t st) {
+    const dim3 grid((unsigned)a.M);
+#define ROW_GO(T_, Q_) hipLaunchKernelGGL((k_row_update<E, T_, Q_>), grid, dim3(T_), 0, st, a)
+    if (a.W <= 256) ROW_GO(64, 1);
+    else if (a.W <= 1024) ROW_GO(256, 1);
+    else if (a.M >= 512 && a.W <= 4096) {  // many rows: fewer, longer-lived workgroups per row
+        if (a.W <= 2048) ROW_GO(256, 2);
+        else ROW_GO(256, 4);
+    } else if (a.W <= 2048) ROW_GO(512, 1);
+    else if (a.W <= 4096) ROW_GO(1024, 1);
+    else if (a.W <= 8192) ROW_GO(1024, 2);
+    else if (a.W <= 16384) ROW_GO(1024, 4);
+    else ROW_GO(1024, 8);
+#undef ROW_GO
+}
+
+}  // namespace
+
+int row_update_launch(int dtype, const RowUpdateArgs &a, hipStream_t st) {
+    if (a.M <= 0) return PIE_OK;
+    PIE_REQUIRE(a.W > 0 && a.W <= ROW_UPDATE_MAX_WIDTH, PIE_E_SHAPE, "row update: widths up to 32768");
+    PIE_REQUIRE(a.ldx % 4 == 0 && a.ldh % 4 == 0 && (!a.y32 || a.ldy % 4 == 0), PIE_E_ALIGN, "row update: row strides must be multiples of 4");
+    if (dtype == PIE_F32) row_go<ElemF32>(a, st);
+    else row_go<ElemBF16>(a, st);
+    PIE_LAUNCH_CHECK();
+    return PIE_OK;
+}

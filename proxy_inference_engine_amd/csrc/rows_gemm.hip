@@ -47,7 +47,7 @@ __device__ __forceinline__ bool rows_select(const RowsArgs &a, RowsWork &k) {
     return true;
 }
 
-// One finished value (m: result row inside the group, n: feature); pair: the value of feature n + 1 (ROWS_SILU_MUL)
+// One finished value (m: result row inside the group, n: feature); pair: the value of feature n + 1 (ROWS_SILU_MUL, ROWS_CLIP_MUL)
 template <class E>
 __device__ __forceinline__ void rows_finish(const RowsArgs &a, const RowsWork &k, int m, int n, float v, float pair) {
     typedef typename E::type T;
@@ -62,6 +62,9 @@ __device__ __forceinline__ void rows_finish(const RowsArgs &a, const RowsWork &k
         }
         case ROWS_SILU_MUL:
             if (!(n & 1)) ((T *)k.y)[row * k.ldy + (n >> 1)] = E::pack(v / (1.0f + expf(-v)) * pair);
+            break;
+        case ROWS_CLIP_MUL:
+            if (!(n & 1)) ((T *)k.y)[row * k.ldy + (n >> 1)] = E::pack(clipped_glu(v, pair, a.act_alpha, a.act_limit));
             break;
         case ROWS_SPLIT:
             if (n < a.split) ((T *)k.y)[row * k.ldy + n] = E::pack(v);
@@ -176,16 +179,17 @@ __global__ void __launch_bounds__(512) k_rows_w16m(const RowsArgs a) {
 #pragma unroll
         for (int t = 0; t < NT; ++t) *(mf_f32x4 *)(s_red + (((wave * NN + n) * NT + t) * 16 + c) * ST + 4 * kq) = acc[n][t];
     __syncthreads();
+    const bool paired = a.epi == ROWS_SILU_MUL || a.epi == ROWS_CLIP_MUL;
     for (int id = threadIdx.x; id < NW * NN * NT * 256; id += 512) {
         const int nl = id & 15, ml = (id >> 4) % (16 * NT), wn2 = id / (256 * NT), w = wn2 / NN, nn = wn2 % NN;
         const int n = ((int)blockIdx.x * NW * NN + wn2) * 16 + nl, m = i0 + ml;
         if (n >= k.N || m >= k.count) continue;
-        if (a.epi == ROWS_SILU_MUL && (nl & 1)) continue;
+        if (paired && (nl & 1)) continue;
         const float *r = s_red + (((w * KW * NN + nn) * NT + (ml >> 4)) * 16 + (ml & 15)) * ST + nl;
         float v = 0.0f, p = 0.0f;
 #pragma unroll
         for (int q = 0; q < KW; ++q) v += r[q * NN * NT * 16 * ST];
-        if (a.epi == ROWS_SILU_MUL)
+        if (paired)
 #pragma unroll
             for (int q = 0; q < KW; ++q) p += r[q * NN * NT * 16 * ST + 1];
         rows_finish<ElemBF16>(a, k, m, n, v, p);

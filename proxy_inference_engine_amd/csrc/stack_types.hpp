@@ -1,5 +1,6 @@
 // stack_types.hpp -- what the kernels of the layer-stack models share: the element types, the norms that ride in epilogues, and the operand
-// descriptions of the row-wise Linear (rows_gemm.hip) and of the latent attention (latent_attn.hip).
+// descriptions of the row-wise Linear (rows_gemm.hip), the attentions (latent_attn.hip, window_attn.hip, page_attn.hip), the recurrence (delta_rule.hip) and
+// the row norms (row_update.hip).
 //
 // Every activation row has a stride that is a multiple of 8 elements (act_stride(), or packed); a Linear reads 64 ceil(K / 64) elements of it.  The columns past K meet zero
 // weights, so they only have to be finite: the owner zero-fills its buffers once and keeps 64 elements of slack behind each.
@@ -124,7 +125,13 @@ enum RowsEpi {
     ROWS_SILU_MUL = 3,   // rows (2 i, 2 i + 1) = (gate_i, up_i): y[m][i] = T(silu(gate) * up)
     ROWS_SPLIT = 4,      // n < split: y[m][n] = T(v);  else y2[m][n - split] = v, fp32
     ROWS_RESIDUAL = 5,   // x[m][n] += post(v);  h[m][n] = T(next(x[m][n]))
+    ROWS_CLIP_MUL = 6,   // rows (2 i, 2 i + 1) = (gate_i, up_i): y[m][i] = T(clipped_glu(gate, up))
 };
+// g sigmoid(alpha g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit)
+__device__ __forceinline__ float clipped_glu(float gate, float up, float alpha, float limit) {
+    const float g = fminf(gate, limit), u = fminf(fmaxf(up, -limit), limit);
+    return g / (1.0f + expf(-alpha * g)) * (u + 1.0f);
+}
 
 struct RowsMat {      // one weight matrix with its operand and result
     const char *w;    // W16M tiles (bf16) or row-major fp32 [N][64 ceil(K / 64)]
@@ -147,6 +154,7 @@ struct RowsArgs {
     const int *rows;       // ungrouped, nullable: x row of result row i
     int epi;
     float scale;
+    float act_alpha, act_limit;  // ROWS_CLIP_MUL
     int split;
     float *y2;
     int ldy2;
@@ -205,3 +213,120 @@ struct WindowAttnArgs {
 int window_attn_launch(const WindowAttnArgs &a, int n_tiles, hipStream_t st);  // n_tiles = sum of ceil(n_rows / 128)
 int latent_gather_launch(const RowRun *runs, int n_runs, int n_ctx, int window, const int *table, int table_width, int n_seqs, int n_pages, const void *slab, int ldr,
                          void *out, int ld_out, hipStream_t st);
+
+// ---------------------------------------------------------------- softmax attention over paged keys and values (page_attn.hip)
+// A page of one layer holds, per key/value head, 64 keys and 64 values in matrix-core operand order: every operand load of a wave is one contiguous KiB.
+//   key t (0 .. 63), dimension d:    two blocks of 32 keys, each [D16 / 8 chunks of 8 dimensions][32 keys][8]
+//   value t, dimension d:            two blocks of 32 tokens, each [V32 / 32 blocks of 32 dimensions][2 halves of 16 tokens][2][32 dimensions][8 tokens], where the
+//                                    8 tokens of (half s, h) are 16 s + 4 h + {0 .. 3, 8 .. 11}: the order in which the score product leaves its weights
+// D16 = dim rounded up to 16, V32 = vdim rounded up to 32; what is never written stays zero.  fp32 stacks use the same order.
+struct KvGeometry {
+    int H, G, dim, vdim, D8, V8, D16, V32;  // D8, V8: head strides of activations
+    __host__ __device__ size_t head_elems() const { return (size_t)PAGE_TOKENS * (D16 + V32); }
+    __host__ __device__ size_t page_elems() const { return G * head_elems(); }
+    __host__ __device__ int key(int t, int d) const { return (t >> 5) * 32 * D16 + ((d >> 3) * 32 + (t & 31)) * 8 + (d & 7); }
+    __host__ __device__ int value(int t, int d) const {
+        return PAGE_TOKENS * D16 + (t >> 5) * 32 * V32 + (d >> 5) * 1024 + ((t >> 4) & 1) * 512 + ((t >> 2) & 1) * 256 + (d & 31) * 8 + ((t & 3) | ((t >> 3) & 1) << 2);
+    }
+};
+static inline KvGeometry kv_geometry(int H, int G, int dim, int vdim) {
+    return {H, G, dim, vdim, (dim + 7) & ~7, (vdim + 7) & ~7, (dim + 15) & ~15, (vdim + 31) & ~31};
+}
+constexpr int PAGE_ATTN_MAX_DIM = 256;  // wider heads take the vector ALU (up to PAGE_ATTN_ROWS_DIM)
+constexpr int PAGE_ATTN_ROWS_DIM = 1024;
+
+struct PageTable {  // where a sequence's pages are
+    const int *table;
+    int table_width, n_pages, n_seqs;
+};
+__device__ __forceinline__ int page_of(const PageTable &p, int seq, int t) {
+    const int j = min(t / PAGE_TOKENS, p.table_width - 1);
+    return (int)min((unsigned)p.table[(size_t)min(seq, p.n_seqs - 1) * p.table_width + j], (unsigned)p.n_pages - 1u);
+}
+
+// raw projections -> normed and rotated queries (in place), keys and values of the pass's rows into their pages
+struct KvPrepArgs {
+    void *raw;              // [M][ld] T: q [H][D8], k [G][D8], v [G][V8] (own), gate
+    int ld, M;
+    const u16 *bias;        // bf16, same order; nullable
+    KvGeometry geo;
+    bool own, value_norm;   // own: the layer has keys and values of its own
+    const float *q_norm, *k_norm;
+    float eps;
+    const float *freq;
+    int rot_dims;
+    float rot_gain;
+    const int *pos, *row_seq;
+    PageTable pages;
+    void *slab;
+};
+int kv_prep_launch(int dtype, const KvPrepArgs &a, hipStream_t st);
+
+struct PageAttnArgs {
+    const void *q;          // [M][ldq] T, head h at h * D8
+    int ldq;
+    const void *slab;
+    PageTable pages;
+    KvGeometry geo;
+    const int *pos, *row_seq;
+    const RowRun *runs;
+    int n_runs, n_tiles, M;
+    bool single;            // every run is one row
+    int window;             // keys j with 0 <= i - j < window; <= 0: no limit
+    float scale, sink;      // sink: what the softmax's denominator has besides the keys, as the weight of one more score of 0
+    const void *gate;       // [M][ldg] T logits per head, nullable: every head's output times their sigmoid
+    const u16 *gate_bias;   // bf16 [H], nullable
+    int ldg;
+    int splits;
+    float *ws;              // see LatentMerge (ldr = V32)
+    void *out;              // [M][ld_out] T, head h at h * V8
+    int ld_out;
+};
+int page_attn_tiles(int n_rows, const KvGeometry &g);       // of the short form
+int page_attn_long_tiles(int n_rows, const KvGeometry &g);  // of the long form
+size_t page_attn_ws_floats(int M, const KvGeometry &g, int splits);
+bool page_attn_mfma(int dtype, const KvGeometry &g);        // matrix-core forms exist for this shape (else: one launch for any rows)
+int page_attn_launch(int dtype, const PageAttnArgs &a, hipStream_t st);
+int page_attn_long_launch(const PageAttnArgs &a, hipStream_t st);
+
+// ---------------------------------------------------------------- generalised delta rule (delta_rule.hip)
+constexpr int DELTA_MAX_DIM = 256, DELTA_MAX_RANK = 1024;
+struct DeltaArgs {
+    const void *raw;        // [M][ld] T: r, k, v, gate, rate [H][D8] each, then the decay's low-rank input [rank]
+    int ld, M, H, D, D8, rank, R8;
+    const u16 *bias;        // bf16, same order; nullable
+    const u16 *w_decay;     // bf16 [H * D][R8]
+    const float *decay_bias, *o_norm;
+    float decay_scale, unit_eps, eps;
+    const int *pos, *row_seq, *slots;
+    int n_seqs, n_slots;
+    const RowRun *runs;
+    int n_runs;
+    float *state;           // [n_slots][H][D][D] (key channel, value column)
+    void *out;              // [M][ld_out] T, head h at h * D8
+    int ld_out;
+};
+int delta_step_launch(int dtype, const DeltaArgs &a, hipStream_t st);
+
+// ---------------------------------------------------------------- x += post(y); h = next(x) with norms that need the whole row (row_update.hip)
+struct StackNorm {
+    const float *w, *b;
+    float param;
+    int kind;
+};
+constexpr int ROW_UPDATE_MAX_WIDTH = 32768;
+struct RowUpdateArgs {
+    const void *y;          // [M][ldy] (nullptr: x stays as it is, h = next(x)); experts: [M * top][ldy] by position
+    bool y32;               // y is fp32 (else bf16)
+    int ldy;
+    const u16 *bias;        // bf16 [W] added to y; nullable
+    const int *place;       // experts (nullable): y of row m = sum over its slots s of weight[m * top + s] * y[place[m * top + s]]
+    const float *weight;    // nullable: 1 / top each
+    int top;
+    StackNorm post, next;
+    float *x;               // [M][ldx]
+    int ldx;
+    void *h;                // [M][ldh] T
+    int ldh, M, W;
+};
+int row_update_launch(int dtype, const RowUpdateArgs &a, hipStream_t st);

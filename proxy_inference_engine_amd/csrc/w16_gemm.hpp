@@ -68,6 +68,7 @@ struct W16Args {
     u16 *y;         // [M][N], or the MLP activation [M][N / 2] (SWIGLU)
     float *part;    // gridDim.y > 1: fp32 slabs [z][M][N]
     const u16 *bias;
+    float act_alpha, act_limit;  // MFMA_ACT_CLIPPED
     const char *zero;  // 4 KiB of zeros (the dummy steps' weight tile)
     int tm, tn;     // row tiles; column tiles (of 128 SW columns)
     // grouped form (GRP): row tile t multiplies rows [row0, row0 + rows) of expert's matrix; x row = list[row0 + i] (nullptr: row0 + i), y row = row0 + i
@@ -90,7 +91,7 @@ struct W16Args {
 // expert's tiles start at a block -- with all its column tiles, row tile fastest: a block's tiles stream the same weight tiles through one L2 at the same time.
 template <class T, int MB, int SW, int ACT, bool GRP = false>
 __global__ void __launch_bounds__(256) k_w16l_gemm(const W16Args a) {
-    constexpr bool SWIGLU = ACT == MFMA_ACT_SWIGLU;
+    constexpr bool SWIGLU = ACT == MFMA_ACT_SWIGLU || ACT == MFMA_ACT_CLIPPED;
     constexpr int MT = 32 * MB, XJ = MB;  // rows per tile; DMA instructions per wave and tile (MT / 8 row groups over 4 waves)
     constexpr int WL = 4 * SW;            // weight loads per wave and step
     constexpr int XB = 4, CHUNK = MT * 128;  // x buffers (tile v lives in buffer v % 4); bytes each
@@ -296,5 +297,5 @@ __global__ void __launch_bounds__(256) k_w16l_gemm(const W16Args a) {
     }
     static_assert(4 * MT * ((SWIGLU ? 32 : 64) * SW) <= XB * CHUNK, "the output tile fits the x buffers");
     __syncthreads();  // everyone has read its last B fragments
-    mfma_tile_store<T, MB, SW, ACT>(acc, s_x + wave * (MT * (SWIGLU ? 32 : 64) * SW), lane, nt0, m0, rows, a.N, a.ldy, a.y, a.bias, (W16L_ABL & 64) && a.M > 1);
+    mfma_tile_store<T, MB, SW, ACT>(acc, s_x + wave * (MT * (SWIGLU ? 32 : 64) * SW), lane, nt0, m0, rows, a.N, a.ldy, a.y, a.bias, (W16L_ABL & 64) && a.M > 1, a.act_alpha, a.act_limit);
 }

@@ -34,20 +34,22 @@ int w16l_relu2_launch(const void *w16m, const void *x, int ldx, int M, int N, in
     return PIE_OK;
 }
 
-// grouped: tiles [tm] of tile_rows (64 or 128) rows, `block` of them side by side on an XCD; x_rows: rows of x; swiglu: y = T(silu(gate) up) of the interleaved matrix, N / 2 wide
+// grouped: tiles [tm] of tile_rows (64 or 128) rows, `block` of them side by side on an XCD; x_rows: rows of x; act: MFMA_ACT_NONE, or MFMA_ACT_SWIGLU / _CLIPPED of the interleaved matrix, N / 2 wide
 int w16l_grouped_launch(const void *w16m, size_t w_stride, const void *x, int ldx, size_t x_rows, const int *list, const void *tiles, int tm, int block, int tile_rows, int N, int K,
-                        void *y, int ldy, bool swiglu, hipStream_t st) {
+                        void *y, int ldy, int act, float act_alpha, float act_limit, hipStream_t st) {
     W16Args a = {};
     if (int rc = w16_fill(a, w16m, x, ldx, N, K, y, ldy)) return rc;
     PIE_REQUIRE(x_rows * ldx * 2 < (1ull << 32), PIE_E_SHAPE, "grouped GEMM: x too large");
-    PIE_REQUIRE((tile_rows == 64 || tile_rows == 128) && (!swiglu || N % 8 == 0), PIE_E_SHAPE, "grouped GEMM: bad tile or width");
-    a.M = (int)x_rows, a.tm = tm, a.tiles = (const int4 *)tiles, a.list = list, a.w_stride = w_stride;
+    PIE_REQUIRE((tile_rows == 64 || tile_rows == 128) && (act == MFMA_ACT_NONE || N % 8 == 0), PIE_E_SHAPE, "grouped GEMM: bad tile or width");
+    a.M = (int)x_rows, a.tm = tm, a.tiles = (const int4 *)tiles, a.list = list, a.w_stride = w_stride, a.act_alpha = act_alpha, a.act_limit = act_limit;
     a.bm = block;
     const dim3 grid((unsigned)(8 * ((tm + 8 * block - 1) / (8 * block)) * block * a.tn));
-    if (tile_rows == 64 && swiglu) hipLaunchKernelGGL((k_w16l_gemm<BF16, 2, 2, MFMA_ACT_SWIGLU, true>), grid, dim3(256), 0, st, a);
-    else if (tile_rows == 64) hipLaunchKernelGGL((k_w16l_gemm<BF16, 2, 2, MFMA_ACT_NONE, true>), grid, dim3(256), 0, st, a);
-    else if (swiglu) hipLaunchKernelGGL((k_w16l_gemm<BF16, 4, 2, MFMA_ACT_SWIGLU, true>), grid, dim3(256), 0, st, a);
-    else hipLaunchKernelGGL((k_w16l_gemm<BF16, 4, 2, MFMA_ACT_NONE, true>), grid, dim3(256), 0, st, a);
+#define GRP_GO(MB_) \
+    if (act == MFMA_ACT_SWIGLU) hipLaunchKernelGGL((k_w16l_gemm<BF16, MB_, 2, MFMA_ACT_SWIGLU, true>), grid, dim3(256), 0, st, a); \
+    else if (act == MFMA_ACT_CLIPPED) hipLaunchKernelGGL((k_w16l_gemm<BF16, MB_, 2, MFMA_ACT_CLIPPED, true>), grid, dim3(256), 0, st, a); \
+    else hipLaunchKernelGGL((k_w16l_gemm<BF16, MB_, 2, MFMA_ACT_NONE, true>), grid, dim3(256), 0, st, a)
+    if (tile_rows == 64) { GRP_GO(2); } else { GRP_GO(4); }
+#undef GRP_GO
     PIE_LAUNCH_CHECK();
     return PIE_OK;
 }

@@ -33,7 +33,8 @@ class BatchedEngine:
         """kv_dtype=torch.int8 (+ kv_scales = (k, v) float16 [n_layers, n_kv_heads]): the pool holds the reference KVPage's int8 pages with
         per-head scales (page.hpp:25-32) -- half the cache bytes per token, so twice the sequences / context per pool."""
         self.model = model
-        self.pool = model.enable_paged_kv(num_pages=num_pages, kv_dtype=kv_dtype, kv_scales=kv_scales)
+        slots = {"max_sequences": max_batch + 1} if getattr(model, "recurrent", False) else {}  # (+ 1: the sequence that holds a shared prefix)
+        self.pool = model.enable_paged_kv(num_pages=num_pages, kv_dtype=kv_dtype, kv_scales=kv_scales, **slots)
         self._i8 = self.pool.dtype == torch.int8   # int8 pages are written by the batch paths only: lone prompts go through prefill_batch too
         self.max_batch = max_batch
         self.stop_tokens = set(int(t) for t in stop_tokens)

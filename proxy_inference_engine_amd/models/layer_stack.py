@@ -1,21 +1,73 @@
-"""Models whose layers are listed one by one, run by the native layer stack (csrc/layer_stack.hip) over a paged latent cache.
+"""Models whose layers are listed one by one, run by the native layer stack (csrc/layer_stack.hip) over paged caches and recurrent state.
 
-A design's module (e.g. models/taduzen) reads its config.json and packs its checkpoint into `pie_stack_layer` descriptions; this class is what every such
+A design's module (models/taduzen, models/kodupel) reads its config.json and packs its checkpoint into `pie_stack_layer` descriptions; this class is what every such
 model shares with the engines: the cache protocol (make_cache, enable_paged_kv), the calling convention (`model(inputs, cache=)`), the greedy fast
 path (`step`) and the multi-sequence passes (`step_batch`, `prefill_batch`, `step_mixed`, `step_portions`).  Every one of them is the same pass:
 rows of any sequences, each with its own position, in one batch."""
 from __future__ import annotations
 
 import ctypes as C
+import math
+from typing import NamedTuple
 
 import numpy as np
 import torch
 
 from .. import _ffi
-from ..cache.kv_cache import BaseCache, LatentPageAllocator, PagedLatentCache, PagedSequence, SavedLatentCache
+from ..cache.kv_cache import BaseCache, LatentPageAllocator, PagedLatentCache, PagedSequence, PagedStackCache, SavedLatentCache, StackPageAllocator, StackSequence
 from ..cache.kv_cache.paged import TOKEN_CAPACITY_PER_PAGE
 
 MAX_ROWS = 4096  # rows of one pass; longer prompts run as several
+
+
+class Norm(NamedTuple):
+    """A norm of the stack: kind PIE_NORM_*, param (DYN_TANH: alpha; RMS: eps), fp32 w and b [width rounded up to 8]."""
+    kind: int
+    param: float
+    w: torch.Tensor
+    b: torch.Tensor | None = None
+
+
+def up8(n: int) -> int:
+    return (n + 7) // 8 * 8
+
+
+def pad(w: torch.Tensor, rows: int, cols: int) -> torch.Tensor:
+    """w in the corner of a [rows, cols] matrix of zeros."""
+    out = torch.zeros(rows, cols, dtype=w.dtype, device=w.device)
+    out[:w.shape[0], :w.shape[1]] = w
+    return out
+
+
+def pad_head_rows(w: torch.Tensor, heads: int, n: int) -> torch.Tensor:
+    """[heads * n, K] -> [heads * (n rounded up to 8), K], zero rows behind each head."""
+    out = torch.zeros(heads, up8(n), w.shape[1], dtype=w.dtype, device=w.device)
+    out[:, :n] = w.reshape(heads, n, -1)
+    return out.flatten(0, 1)
+
+
+def pad_head_columns(w: torch.Tensor, heads: int, n: int) -> torch.Tensor:
+    """[N, heads * n] -> [N, heads * (n rounded up to 8)], zero columns behind each head."""
+    return pad_head_rows(w.T, heads, n).T
+
+
+def interleave(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
+    """Rows (2 i, 2 i + 1) = (gate_i, up_i)."""
+    return torch.stack([gate, up], dim=-2).flatten(-3, -2)
+
+
+def yarn_frequencies(dims: int, base: float, scaling: tuple[float, float, float, float] | None = None) -> tuple[torch.Tensor, float]:
+    """(fp32 [dims / 2] angle per position of every rotated pair, the factor on cos and sin).  scaling = (factor, original, fast, slow): pairs that turn
+    more than `fast` times over the original context keep their frequency, pairs that turn less than `slow` times have it divided by factor, those between
+    are mixed linearly (YaRN)."""
+    freq = [base ** (-2.0 * i / dims) for i in range(dims // 2)]
+    if scaling is None:
+        return torch.tensor(freq, dtype=torch.float32), 1.0
+    factor, original, fast, slow = scaling
+    at = lambda turns: dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))  # noqa: E731
+    lo, hi = max(math.floor(at(fast)), 0), min(math.ceil(at(slow)), dims - 1)
+    mix = [min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0) for i in range(dims // 2)]
+    return torch.tensor([f * (m / factor + 1.0 - m) for f, m in zip(freq, mix)], dtype=torch.float32), 0.1 * math.log(factor) + 1.0
 
 
 def pack_linear(w: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
@@ -33,23 +85,27 @@ def pack_linear(w: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
 
 class LayerStackModel:
     def __init__(self, args, dtype: torch.dtype, width: int, vocab: int, logit_scale: float, layers: list[dict], embed: torch.Tensor, head: torch.Tensor,
-                 final_norm: tuple):
-        """layers: per layer the fields of pie_stack_layer -- tensors for its pointers, (alpha, w, b) triples for its norms, numbers for the rest
+                 final_norm: Norm, embed_scale: float = 1.0):
+        """layers: per layer the fields of pie_stack_layer -- tensors for its pointers, Norms for its norms, numbers for the rest
         (absent fields are zero).  embed: bf16 [vocab, width]; head: packed."""
         self.args, self.dtype, self.width, self.vocab_size = args, dtype, width, vocab
         self.device = embed.device
         self.layers = layers
         self._held = [embed, head, final_norm]
         lib = _ffi.base()
-        cfg = _ffi.pie_stack_config(_ffi.stack_dtype_code(dtype), width, vocab, len(layers), logit_scale, embed.data_ptr(), head.data_ptr(), self._norm(final_norm))
+        cfg = _ffi.pie_stack_config(_ffi.stack_dtype_code(dtype), width, vocab, len(layers), logit_scale, embed_scale, embed.data_ptr(), head.data_ptr(), self._norm(final_norm))
         self._stack = C.c_void_p()
         _ffi.check(lib.pie_stack_create(C.byref(cfg), C.byref(self._stack)))
         for i, fields in enumerate(layers):
             lay = _ffi.pie_stack_layer()
             for name, v in fields.items():
-                setattr(lay, name, self._norm(v) if isinstance(v, tuple) else v.data_ptr() if isinstance(v, torch.Tensor) else v)
+                setattr(lay, name, self._norm(v) if isinstance(v, Norm) else v.data_ptr() if isinstance(v, torch.Tensor) else v)
             _ffi.check(lib.pie_stack_set_layer(self._stack, i, C.byref(lay)))
         self.row_elems = [lib.pie_stack_page_row(self._stack, i) for i in range(len(layers))]
+        self.state_floats = [int(lib.pie_stack_state_floats(self._stack, i)) for i in range(len(layers))]
+        self.recurrent = any(self.state_floats)
+        # a latent layer's pages hold token after token; anything else is kept, shared and saved by whole pages, beside the recurrent state
+        self._plain_pages = not self.recurrent and all(lay["mixer"] == _ffi.PIE_MIXER_LATENT for lay in layers)
         self.history = torch.zeros(1 << 20, dtype=torch.int32, device=self.device)  # history[p] = greedy token chosen for position p
         self._pool: LatentPageAllocator | None = None
         self._page_blocks = 16
@@ -57,9 +113,8 @@ class LayerStackModel:
         torch.cuda.synchronize(self.device)
 
     @staticmethod
-    def _norm(n: tuple):
-        alpha, w, b = n
-        return _ffi.pie_point_norm(w.data_ptr(), b.data_ptr(), alpha)
+    def _norm(n: Norm):
+        return _ffi.pie_stack_norm(n.w.data_ptr(), None if n.b is None else n.b.data_ptr(), n.param, n.kind)
 
     def __del__(self):
         s = getattr(self, "_stack", None)
@@ -71,11 +126,18 @@ class LayerStackModel:
             self._stack = None
 
     # ------------------------------------------------------------------ caches
-    def enable_paged_kv(self, num_pages: int = 512, max_blocks: int = 16, kv_dtype: torch.dtype | None = None, kv_scales=None) -> LatentPageAllocator:
-        """From now on make_cache() draws on one pool of `num_pages` 64-token pages (all layers).  Returns the pool."""
+    def _allocator(self, num_pages: int, max_sequences: int) -> LatentPageAllocator:
+        if self._plain_pages:
+            return LatentPageAllocator(num_pages, self.row_elems, dtype=self.dtype, device=self.device)
+        return StackPageAllocator(num_pages, self.row_elems, self.state_floats, max_sequences, dtype=self.dtype, device=self.device)
+
+    def enable_paged_kv(self, num_pages: int = 512, max_blocks: int = 16, kv_dtype: torch.dtype | None = None, kv_scales=None,
+                        max_sequences: int = 32) -> LatentPageAllocator:
+        """From now on make_cache() draws on one pool of `num_pages` 64-token pages (all layers) and, for recurrent layers, state slots for
+        `max_sequences` live sequences.  Returns the pool."""
         if kv_dtype not in (None, self.dtype) or kv_scales is not None:
-            raise ValueError(f"latent pages are stored in the model's dtype ({self.dtype})")
-        self._pool = LatentPageAllocator(num_pages, self.row_elems, dtype=self.dtype, device=self.device)
+            raise ValueError(f"a layer-stack model's pages are stored in its dtype ({self.dtype})")
+        self._pool = self._allocator(num_pages, max_sequences)
         self._page_blocks = max_blocks
         return self._pool
 
@@ -86,19 +148,23 @@ class LayerStackModel:
 
     def make_paged_cache(self, allocator: LatentPageAllocator | None = None, num_pages: int = 512, max_blocks: int = 16) -> list[BaseCache]:
         if allocator is None:
-            allocator = LatentPageAllocator(num_pages, self.row_elems, dtype=self.dtype, device=self.device)
-        if not isinstance(allocator, LatentPageAllocator) or allocator.row_elems != self.row_elems or allocator.dtype != self.dtype or allocator.device is None:
+            allocator = self._allocator(num_pages, 32)
+        if not isinstance(allocator, LatentPageAllocator if self._plain_pages else StackPageAllocator) or allocator.row_elems != self.row_elems or \
+                allocator.dtype != self.dtype or allocator.device is None or (not self._plain_pages and allocator.state_floats != self.state_floats):
             raise ValueError("the allocator's geometry does not match this model")
-        seq = PagedSequence(allocator, max_blocks)
-        return [PagedLatentCache(seq, i) for i in range(len(self.layers))]
+        if self._plain_pages:
+            seq: PagedSequence = PagedSequence(allocator, max_blocks)
+            return [PagedLatentCache(seq, i) for i in range(len(self.layers))]
+        seq = StackSequence(allocator, max_blocks)
+        return [PagedStackCache(seq, i) for i in range(len(self.layers))]
 
     def adopt_cache(self, cache: list[BaseCache]) -> list[BaseCache]:
-        """Latents restored from a file, copied into pages; anything else as it is."""
+        """A cache restored from a file, copied into pages (and a state slot); anything else as it is."""
         if not isinstance(cache[0], SavedLatentCache):
             return cache
         out = self.make_cache()
         for mine, saved in zip(out, cache):
-            mine.state = (saved.rows[:, :, :saved.offset], None)
+            mine.adopt(saved)
         return out
 
     def _sequence(self, cache: list[BaseCache]) -> PagedSequence:
@@ -114,13 +180,15 @@ class LayerStackModel:
         return a
 
     # ------------------------------------------------------------------ the pass
-    def _forward(self, a: LatentPageAllocator, rows: int, ids, pos, row_seq, table, runs, runs_host: np.ndarray, want, n_want: int, logits, logprobs=None,
+    def _forward(self, a: LatentPageAllocator, rows: int, ids, pos, row_seq, table, slots, runs, runs_host: np.ndarray, want, n_want: int, logits, logprobs=None,
                  nxt=None, advance: bool = False, history=None, graph: bool = False, tap=None) -> None:
         p = lambda t: None if t is None else t.data_ptr()  # noqa: E731
-        slabs = (C.c_void_p * len(a.slabs))(*[s.data_ptr() for s in a.slabs])
+        slabs = (C.c_void_p * len(a.slabs))(*[s.data_ptr() if s.numel() else None for s in a.slabs])
+        states = (C.c_void_p * len(a.slabs))(*[None if s is None else s.data_ptr() for s in a.states]) if self.recurrent else None
         b = _ffi.pie_stack_batch(rows, table.shape[0], table.shape[1], len(runs_host), n_want, int(advance), 0 if history is None else history.numel(), 0,
                                  p(ids), p(pos), p(row_seq), p(table), p(runs), runs_host.ctypes.data, p(want), p(logits), p(logprobs), p(nxt), p(history),
-                                 C.cast(slabs, C.c_void_p), a.size(), p(tap))
+                                 C.cast(slabs, C.c_void_p), a.size(), p(tap), p(slots), None if states is None else C.cast(states, C.c_void_p),
+                                 a.num_slots if self.recurrent else 0)
         _ffi.check(_ffi.base().pie_stack_forward(self._stack, C.byref(b), _ffi.PIE_STEP_GRAPH if graph else 0, _ffi.stream()))
 
     def _pass(self, entries: list, want: list[list[int]], tail: bool, tap=None):
@@ -136,7 +204,7 @@ class LayerStackModel:
         starts[order] = np.concatenate([[0], np.cumsum(lens[order])[:-1]])
         M = int(lens.sum())
         width = max(len(s.pages) for _, s in entries)
-        host = np.zeros(3 * M + S * width + 4 * S + M, dtype=np.int32)
+        host = np.zeros(3 * M + S * width + 4 * S + S + M, dtype=np.int32)
         ids, pos, row_seq = host[:M], host[M:2 * M], host[2 * M:3 * M]
         table, runs = host[3 * M:3 * M + S * width].reshape(S, width), host[3 * M + S * width:3 * M + S * width + 4 * S].reshape(S, 4)
         on_device = []
@@ -150,6 +218,8 @@ class LayerStackModel:
             pos[lo:hi] = np.arange(s.offset, s.offset + lens[i])
             row_seq[lo:hi] = i
             table[i, :len(s.pages)] = s.pages
+            if self.recurrent:
+                host[len(host) - M - S + i] = s.slot
             wanted += [int(lo) + int(k) for k in want[i]]
         for j, i in enumerate(order):
             runs[j] = (starts[i], lens[i], i, entries[i][1].offset)
@@ -162,8 +232,8 @@ class LayerStackModel:
         logprobs = torch.empty_like(logits) if tail else None
         nxt = torch.empty(n_want, dtype=torch.int32, device=self.device) if tail else None
         o = 3 * M
-        self._forward(a, M, dev[:M], dev[M:2 * M], dev[2 * M:o], dev[o:o + S * width].view(S, width), dev[o + S * width:o + S * width + 4 * S], runs,
-                      dev[o + S * width + 4 * S:], n_want, logits, logprobs, nxt, tap=tap)
+        self._forward(a, M, dev[:M], dev[M:2 * M], dev[2 * M:o], dev[o:o + S * width].view(S, width), dev[-M - S:-M], dev[o + S * width:o + S * width + 4 * S], runs,
+                      dev[-M:], n_want, logits, logprobs, nxt, tap=tap)
         for (_, s), n in zip(entries, lens):
             s.advance(int(n))
         return logits, logprobs, nxt
@@ -217,7 +287,8 @@ class LayerStackModel:
             buf = {"ids": torch.zeros(B, **i32), "pos": torch.zeros(B, **i32), "row_seq": torch.arange(B, **i32), "table": torch.zeros((B, width), **i32),
                    "runs_host": runs, "runs": torch.from_numpy(runs).to(self.device), "next": torch.empty(B, **i32),
                    "logits": torch.empty((B, self.vocab_size), dtype=torch.float32, device=self.device),
-                   "logprobs": torch.empty((B, self.vocab_size), dtype=torch.float32, device=self.device), "pages": None, "at": None}
+                   "logprobs": torch.empty((B, self.vocab_size), dtype=torch.float32, device=self.device), "slots": torch.zeros(B, **i32),
+                   "pages": None, "held": None, "at": None}
             if tokens is None:
                 raise RuntimeError("no previous step to continue from")
         while len(self._bufs) >= 4:
@@ -230,12 +301,17 @@ class LayerStackModel:
                 t[i, :len(s.pages)] = s.pages
             buf["table"].copy_(torch.from_numpy(t))
             buf["pages"] = pages
+        if self.recurrent:
+            held = [s.slot for s in seqs]
+            if buf["held"] != held:
+                buf["slots"].copy_(torch.tensor(held, dtype=torch.int32))
+                buf["held"] = held
         at = [s.offset for s in seqs]
         if buf["at"] != at:
             buf["pos"].copy_(torch.tensor(at, dtype=torch.int32))
         if tokens is not None:
             buf["ids"].copy_(tokens.reshape(-1))
-        self._forward(a, B, buf["ids"], buf["pos"], buf["row_seq"], buf["table"], buf["runs"], buf["runs_host"], None, B, buf["logits"], buf["logprobs"],
+        self._forward(a, B, buf["ids"], buf["pos"], buf["row_seq"], buf["table"], buf["slots"], buf["runs"], buf["runs_host"], None, B, buf["logits"], buf["logprobs"],
                       buf["next"], advance=True, history=history, graph=graph)
         buf["at"] = [n + 1 for n in at]
         for s in seqs:
@@ -326,4 +402,4 @@ class LayerStackModel:
         return int(_ffi.base().pie_stack_launches(self._stack))
 
 
-__all__ = ["LayerStackModel", "pack_linear"]
+__all__ = ["LayerStackModel", "Norm", "interleave", "pack_linear", "pad", "pad_head_columns", "pad_head_rows", "up8", "yarn_frequencies"]

@@ -9,7 +9,7 @@ import torch
 
 from .. import base
 from ... import _ffi
-from ..layer_stack import LayerStackModel, pack_linear
+from ..layer_stack import LayerStackModel, Norm, interleave, pack_linear, pad, pad_head_columns, pad_head_rows, up8
 
 
 class MaskArgs(base.BaseModelArgs):
@@ -61,28 +61,6 @@ class ModelArgs(base.BaseModelArgs):
     norm: NormArgs
 
 
-def _pad_rows(w: torch.Tensor, heads: int, n: int) -> torch.Tensor:
-    """[heads * n, K] -> [heads, n rounded up to 8, K], zero rows behind each head."""
-    n8 = _up8(n)
-    out = torch.zeros(heads, n8, w.shape[1], dtype=w.dtype, device=w.device)
-    out[:, :n] = w.view(heads, n, -1)
-    return out
-
-
-def _pad(w: torch.Tensor, rows: int, cols: int) -> torch.Tensor:
-    out = torch.zeros(rows, cols, dtype=w.dtype, device=w.device)
-    out[:w.shape[0], :w.shape[1]] = w
-    return out
-
-
-def _up8(n: int) -> int:
-    return (n + 7) // 8 * 8
-
-
-def _interleave(gate: torch.Tensor, up: torch.Tensor) -> torch.Tensor:
-    return torch.stack([gate, up], dim=-2).flatten(-3, -2)
-
-
 class Model(LayerStackModel):
     model_type = "taduzen"
 
@@ -98,8 +76,8 @@ class Model(LayerStackModel):
                 raise ValueError(f"{name}: expected {list(shape)}, got {list(t.shape)}")
             return t
 
-        def norm(name: str) -> tuple:
-            return (float(get(name + ".alpha").float().item()), _pad(get(name, W).float()[None], 1, _up8(W))[0], _pad(get(name + ".b", W).float()[None], 1, _up8(W))[0])
+        def norm(name: str) -> Norm:
+            return Norm(_ffi.PIE_NORM_DYN_TANH, float(get(name + ".alpha").float().item()), pad(get(name, W).float()[None], 1, up8(W))[0], pad(get(name + ".b", W).float()[None], 1, up8(W))[0])
 
         def pack(w: torch.Tensor) -> torch.Tensor:
             return pack_linear(w, dtype)
@@ -112,39 +90,39 @@ class Model(LayerStackModel):
             if lay.type != "latent_attention":
                 raise ValueError(f"layer {i}: unknown mixer {lay.type!r}")
             H, D, V, R = m.heads, m.dim, m.vdim, m.kv_rank
-            q = _pad_rows(get(p + "mix.q", H * D, W), H, D)
+            q = pad_head_rows(get(p + "mix.q", H * D, W), H, D)
             uk, uv = get(p + "mix.uk", H * D, R), get(p + "mix.uv", H * V, R)
             wo = get(p + "mix.o", W, H * V)
             fields = {
                 "pre1": norm(p + "norm1"), "post1": norm(p + "norm1b"), "mixer": _ffi.PIE_MIXER_LATENT,
                 "heads": H, "dim": D, "vdim": V, "rank": R, "window": m.mask.size if m.mask is not None else 0, "scale": m.scale, "eps": args.norm.eps,
-                "w_in": pack(torch.cat([q.flatten(0, 1), _pad(get(p + "mix.dkv", R, W), _up8(R), W)])),
+                "w_in": pack(torch.cat([q, pad(get(p + "mix.dkv", R, W), up8(R), W)])),
                 "w_uk": pack(uk.view(H, D, R).transpose(1, 2)),
                 "w_uv": pack(uv.view(H, V, R)),
-                "w_o": pack(_pad_rows(wo.T, H, V).flatten(0, 1).T),
-                "w_kv": pack(torch.cat([_pad_rows(uk, H, D).flatten(0, 1), _pad_rows(uv, H, V).flatten(0, 1)])),
+                "w_o": pack(pad_head_columns(wo, H, V)),
+                "w_kv": pack(torch.cat([pad_head_rows(uk, H, D), pad_head_rows(uv, H, V)])),
                 "c_norm": get(p + "mix.dkv.norm", R).float().contiguous(),
             }
             if ff is not None:
                 fields |= {"pre2": norm(p + "norm2"), "post2": norm(p + "norm2b")}
                 # (intermediate widths padded to 8 with zero rows and columns: act(0) = 0 for both activations)
                 def gated(pfx: str, n: int):
-                    n8 = _up8(n)
-                    return (pack(_interleave(_pad(get(pfx + "gate", n, W), n8, W), _pad(get(pfx + "up", n, W), n8, W))), pack(_pad(get(pfx + "down", W, n), W, n8)))
+                    n8 = up8(n)
+                    return (pack(interleave(pad(get(pfx + "gate", n, W), n8, W), pad(get(pfx + "up", n, W), n8, W))), pack(pad(get(pfx + "down", W, n), W, n8)))
 
                 if ff.kind == "dense":
-                    n8 = _up8(ff.ff)
-                    fields |= {"ff": _ffi.PIE_FF_RELU2, "ff_size": n8, "w_up": pack(_pad(get(p + "mlp.up", ff.ff, W), n8, W)),
-                               "w_down": pack(_pad(get(p + "mlp.down", W, ff.ff), W, n8))}
+                    n8 = up8(ff.ff)
+                    fields |= {"ff": _ffi.PIE_FF_RELU2, "ff_size": n8, "w_up": pack(pad(get(p + "mlp.up", ff.ff, W), n8, W)),
+                               "w_down": pack(pad(get(p + "mlp.down", W, ff.ff), W, n8))}
                 elif ff.kind == "moe":
                     E, top = ff.router.experts, ff.router.top
                     experts = [gated(f"{p}mlp.e{e}.", ff.expert.ff) for e in range(E)]
-                    fields |= {"ff": _ffi.PIE_FF_TABLE_MOE, "ff_size": _up8(ff.expert.ff), "experts": E, "top": top,
+                    fields |= {"ff": _ffi.PIE_FF_TABLE_MOE, "ff_size": up8(ff.expert.ff), "experts": E, "top": top,
                                "table": get(p + "mlp.table", args.vocab, top).to(torch.int32).contiguous(),
                                "w_gate_up": torch.cat([e[0] for e in experts]), "w_expert_down": torch.cat([e[1] for e in experts])}
                     if ff.shared is not None:
                         fields["s_gate_up"], fields["s_down"] = gated(p + "mlp.shared.", ff.shared.ff)
-                        fields |= {"shared_size": _up8(ff.shared.ff), "shared_gate": _pad(get(p + "mlp.shared.sg", 1, W).float(), 1, _up8(W))[0]}
+                        fields |= {"shared_size": up8(ff.shared.ff), "shared_gate": pad(get(p + "mlp.shared.sg", 1, W).float(), 1, up8(W))[0]}
                 else:
                     raise ValueError(f"layer {i}: unknown feed-forward {ff.kind!r}")
             layers.append(fields)
