@@ -119,14 +119,20 @@ def clipped_expert(h, w, p, limit):
 
 
 def choose_experts(h, w, p, top):
-    """([n, top] expert numbers, [n, top] their weights): the choice counts the correction, the weights do not."""
+    """([n, top] expert numbers, [n, top] their weights, [n] how far the last chosen is ahead of the first that is not): the choice counts the correction,
+    the weights do not."""
     s = sigmoid(h @ w[p + "router"].T)
-    best = np.argsort(-(s + w[p + "correction"]), axis=-1, kind="stable")[:, :top]
-    return best, np.take_along_axis(s, best, axis=-1)
+    counted = s + w[p + "correction"]
+    order = np.argsort(-counted, axis=-1, kind="stable")
+    best, ranked = order[:, :top], np.take_along_axis(counted, order, axis=-1)
+    lead = ranked[:, top - 1] - ranked[:, top] if top < s.shape[-1] else np.full(len(s), np.inf)
+    return best, np.take_along_axis(s, best, axis=-1), lead
 
 
-def mixture(h, w, p, ff):
-    best, weight = choose_experts(h, w, p, ff["router"]["top"])
+def mixture(h, w, p, ff, leads=None):
+    best, weight, lead = choose_experts(h, w, p, ff["router"]["top"])
+    if leads is not None:
+        leads.append(lead)
     y = np.zeros_like(h)
     for e in range(ff["router"]["experts"]):
         row, slot = np.nonzero(best == e)
@@ -136,8 +142,8 @@ def mixture(h, w, p, ff):
 
 
 # ------------------------------------------------------------------ the model
-def forward(cfg, w, ids, layers_out=None):
-    """Logits [n, vocab] of one sequence; layers_out (a list) receives the residual stream after every layer."""
+def forward(cfg, w, ids, layers_out=None, leads=None):
+    """Logits [n, vocab] of one sequence; layers_out (a list) receives the residual stream after every layer, leads every mixture's closest calls."""
     eps = cfg["norm"]["eps"]
     x = w["embed"][np.asarray(ids)] * cfg["embedding"]["scale"]
     cached = {}
@@ -151,7 +157,7 @@ def forward(cfg, w, ids, layers_out=None):
             y = attention(x, w, p + "mix.", mx, cached[i], eps)
         x = x + zero_centred_norm(y, w[p + "norm1"], eps)
         if ff is not None:
-            x = x + zero_centred_norm(mixture(x, w, p + "mlp.", ff), w[p + "norm2"], eps)
+            x = x + zero_centred_norm(mixture(x, w, p + "mlp.", ff, leads), w[p + "norm2"], eps)
         if layers_out is not None:
             layers_out.append(x.copy())
     return zero_centred_norm(x, w["final.norm"], eps) @ w["head"].T
