@@ -66,7 +66,7 @@ def parse():
                     "IPC-mapped peer memory (default) or RCCL (ncclAllReduce on the launch stream): the comparator for the first run on a real node")
     ap.add_argument("--knob", action="append", default=[], metavar="NAME=VALUE", help="developer: one of the library's test / tuning switches (_ffi.KNOBS) for this run")
     ap.add_argument("--bits", type=int, choices=[2, 4, 6, 8], default=4, help="8 / 6 / 2: MLX int8 / int6 / int2 g=64 weights (W8S / W6S / W2S units; a different workload than the metric's)")
-    ap.add_argument("--design", choices=["taduzen"], help="instead of the metric's workload: prefill and decode throughput of a layer-stack design at sizes that resemble a "
+    ap.add_argument("--design", choices=["taduzen", "kodupel"], help="instead of the metric's workload: prefill and decode throughput of a layer-stack design at sizes that resemble a "
                     "real model's layers, each beside the dense bf16 Llama of equal size (one JSON line; not the BASELINE.json metric)")
     ap.add_argument("--design-only", default="", help="--design: run only the cases whose name contains this (e.g. dense4096/new/decode1)")
     ap.add_argument("--dense", action="store_true", help="BASELINE.json configs[2]: unquantised bf16 weights (a different workload than the metric's)")
@@ -151,20 +151,28 @@ def cpu_baseline(cfg, weights_host, n_tokens, model=None, prompt=None, what="Lla
 
 
 DESIGN_LAYERS = 4
-# sizes of real models' layers: 8B-class dense layers, and a fine-grained mixture (64 experts, 6 per token, one shared); `like`: the Llama of equal width,
-# heads and active feed-forward width (the mixture's: 6 * 1408 + 2816)
+# sizes of real models' layers: 8B-class dense layers, and fine-grained mixtures; `like`: the Llama of equal width, heads and active feed-forward width
 DESIGN_SIZES = {
-    "dense4096": {"width": 4096, "mixer": {"heads": 32, "dim": 128, "vdim": 128, "kv_rank": 512, "window": 4096}, "mlp": {"ff": 14336},
-                  "like": {"hidden_size": 4096, "intermediate_size": 14336, "num_attention_heads": 32, "num_key_value_heads": 8}},
-    "moe2048": {"width": 2048, "mixer": {"heads": 16, "dim": 128, "vdim": 128, "kv_rank": 512, "window": 4096},
-                "mlp": {"experts": 64, "top": 6, "ff": 1408, "shared": 2816},
-                "like": {"hidden_size": 2048, "intermediate_size": 11264, "num_attention_heads": 16, "num_key_value_heads": 4}},
+    "taduzen": {
+        "dense4096": {"width": 4096, "mixer": {"heads": 32, "dim": 128, "vdim": 128, "kv_rank": 512, "window": 4096}, "mlp": {"ff": 14336},
+                      "like": {"hidden_size": 4096, "intermediate_size": 14336, "num_attention_heads": 32, "num_key_value_heads": 8}},
+        "moe2048": {"width": 2048, "mixer": {"heads": 16, "dim": 128, "vdim": 128, "kv_rank": 512, "window": 4096},
+                    "mlp": {"experts": 64, "top": 6, "ff": 1408, "shared": 2816},
+                    "like": {"hidden_size": 2048, "intermediate_size": 11264, "num_attention_heads": 16, "num_key_value_heads": 4}},
+    },
+    # layers: attention, delta rule, attention on the first layer's keys and values, delta rule
+    "kodupel": {
+        "wide4096": {"width": 4096, "heads": 32, "kv_heads": 8, "dim": 128, "delta_heads": 32, "rank": 128, "mlp": {"experts": 16, "top": 4, "ff": 3584},
+                     "like": {"hidden_size": 4096, "intermediate_size": 14336, "num_attention_heads": 32, "num_key_value_heads": 8}},
+        "fine2048": {"width": 2048, "heads": 16, "kv_heads": 4, "dim": 128, "delta_heads": 16, "rank": 64, "mlp": {"experts": 64, "top": 6, "ff": 1408},
+                     "like": {"hidden_size": 2048, "intermediate_size": 8448, "num_attention_heads": 16, "num_key_value_heads": 4}},
+    },
 }
 DESIGN_VOCAB = 32768
 
 
 def taduzen_checkpoint(size, n_layers, vocab):
-    """(config, device weights) of a random Taduzen model of one of DESIGN_SIZES."""
+    """(config, device weights) of a random Taduzen model of one of its DESIGN_SIZES."""
     W, mx, ff = size["width"], size["mixer"], size["mlp"]
     H, D, V, R = mx["heads"], mx["dim"], mx["vdim"], mx["kv_rank"]
     mixer = {"heads": H, "dim": D, "vdim": V, "kv_rank": R, "scale": D ** -0.5, "mask": {"size": mx["window"]}}
@@ -202,11 +210,49 @@ def taduzen_checkpoint(size, n_layers, vocab):
     return cfg, w
 
 
+def kodupel_checkpoint(size, n_layers, vocab):
+    """(config, device weights) of a random Kodupel model of one of its DESIGN_SIZES."""
+    W, H, G, D, HD, R, ff = size["width"], size["heads"], size["kv_heads"], size["dim"], size["delta_heads"], size["rank"], size["mlp"]
+    mlp = {"kind": "moe", "expert": {"ff": ff["ff"], "limit": 7.0}, "router": {"experts": ff["experts"], "top": ff["top"]}}
+    attn = {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5,
+            "rot": {"base": 500000.0, "dims": D // 2, "scaling": {"factor": 4.0, "original": 2048, "fast": 32.0, "slow": 1.0}}}
+    layers = [{"type": "general_delta", "mixer": {"heads": HD, "dim": D}, "mlp": mlp} if i % 2 else
+              {"type": "attention", "mixer": dict(attn, kv_from=0) if i % 4 else attn, "mlp": mlp} for i in range(n_layers)]
+    cfg = {"architecture": "Kodupel", "vocab": vocab, "width": W, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-6}, "layers": layers}
+    gen = torch.Generator(device="cuda").manual_seed(0)
+    w = {}
+
+    def put(name, *shape, std=None, mean=0.0):
+        w[name] = (torch.randn(shape, generator=gen, device="cuda") * (shape[-1] ** -0.5 if std is None else std) + mean).to(torch.bfloat16)
+    put("embed", vocab, W, std=1.0)
+    for i, lay in enumerate(layers):
+        p = f"l{i}."
+        put(p + "norm1", W, std=0.02), put(p + "norm2", W, std=0.02)
+        if lay["type"] == "attention":
+            for n, heads in (("q", H), *((("k", G), ("v", G)) if "kv_from" not in lay["mixer"] else ())):
+                put(p + f"mix.{n}", heads * D, W), put(p + f"mix.{n}.b", heads * D, std=0.02)
+                if n != "v":
+                    put(p + f"mix.{n}.norm", D, std=0.02, mean=1.0)
+            put(p + "mix.g", H, W), put(p + "mix.o", W, H * D), put(p + "mix.o.b", W, std=0.02)
+        else:
+            for n in "rkvga":
+                put(p + f"mix.{n}", HD * D, W)
+            put(p + "mix.a.b", HD * D, std=1.0), put(p + "mix.w0", HD * D, std=1.0, mean=-3.0), put(p + "mix.w1", R, W), put(p + "mix.w2", HD * D, R)
+            put(p + "mix.norm", HD * D, std=0.02, mean=1.0), put(p + "mix.o", W, HD * D)
+        for e in range(ff["experts"]):
+            put(f"{p}mlp.e{e}.gate", ff["ff"], W), put(f"{p}mlp.e{e}.up", ff["ff"], W), put(f"{p}mlp.e{e}.down", W, ff["ff"])
+        put(p + "mlp.router", ff["experts"], W), put(p + "mlp.correction", ff["experts"], std=0.01)
+    put("final.norm", W, std=0.02)
+    put("head", vocab, W)
+    return cfg, w
+
+
 def design_bench(args):
     """--design: throughput of a layer-stack design beside the dense bf16 Llama of equal size, DESIGN_LAYERS layers each."""
     from proxy_inference_engine_amd.models.llama import Model as Llama, ModelArgs as LlamaArgs
-    from proxy_inference_engine_amd.models.taduzen import Model as Taduzen, ModelArgs as TaduzenArgs
+    from proxy_inference_engine_amd.models import kodupel, taduzen
     from proxy_inference_engine_amd.models.utils import synthetic_checkpoint
+    design, checkpoint = (taduzen, taduzen_checkpoint) if args.design == "taduzen" else (kodupel, kodupel_checkpoint)
     rows = []
     rng = np.random.default_rng(0)
 
@@ -220,13 +266,13 @@ def design_bench(args):
         torch.cuda.synchronize()
         return 1e3 * (time.perf_counter() - t0) / n
 
-    for name, size in DESIGN_SIZES.items():
+    for name, size in DESIGN_SIZES[args.design].items():
         for which in ("new", "llama"):
             if not any(args.design_only in f"{name}/{which}/{c}" for c in ("decode1", "decode8", "decode32", "prefill512", "prefill4096")):
                 continue
             if which == "new":
-                cfg, w = taduzen_checkpoint(size, DESIGN_LAYERS, DESIGN_VOCAB)
-                model = Taduzen(TaduzenArgs(**cfg), w)
+                cfg, w = checkpoint(size, DESIGN_LAYERS, DESIGN_VOCAB)
+                model = design.Model(design.ModelArgs(**cfg), w)
             else:
                 cfg = dict(size["like"], model_type="llama", num_hidden_layers=DESIGN_LAYERS, vocab_size=DESIGN_VOCAB, rms_norm_eps=1e-6, tie_word_embeddings=False,
                            quantization=None)

@@ -31,7 +31,8 @@ int w16l_grouped_launch(const void *w16m, size_t w_stride, const void *x, int ld
 namespace {
 
 constexpr int BIG_ROWS = 64;  // more rows than this take the tiled GEMMs
-constexpr int LONG_RUN = 64;  // runs of at least this many rows attend with keys and values spelled out
+constexpr int LONG_RUN = 64;  // runs of at least this many rows take the attentions' long forms
+constexpr int DELTA_RUN = 8;  // runs of at least this many rows take the recurrence's chunk form
 
 struct RouteLayer {      // one mixture layer's row lists (device pointers)
     const int *table;    // experts by token id; nullptr: by the router's logits
@@ -374,7 +375,7 @@ struct pie_stack {
     std::vector<pie_stack_layer> layers;
     std::vector<char> have;
     // workspace, by rows of a pass
-    Buf<float> x, c_raw, part, part_s, attn_ws, gemm_ws, y32, logits_e;
+    Buf<float> x, c_raw, part, part_s, attn_ws, gemm_ws, y32, logits_e, delta_ws, delta_o;
     Buf<char> h, q, ql, oc, o, act, act_e, act_s, y, ctx, kv;
     Buf<RowStat> stats;
     Buf<int> route_ints;
@@ -432,9 +433,21 @@ size_t plan_context(const pie_stack_batch &b, const Plan &p, int window) {
     return n;
 }
 
+// the leading runs that take the recurrence's step form, their rows, and the chunks of those behind them
+struct DeltaPart {
+    int runs, rows, chunks;
+};
+DeltaPart delta_part(const pie_stack_batch &b) {
+    DeltaPart p = {0, 0, 0};
+    while (p.runs < b.n_runs && b.runs_host[4 * p.runs + 1] < DELTA_RUN) p.rows += b.runs_host[4 * p.runs++ + 1];
+    for (int i = p.runs; i < b.n_runs; ++i) p.chunks += delta_chunks(b.runs_host[4 * i + 1]);
+    return p;
+}
+
 int stack_reserve(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipStream_t st) {
     const size_t M = (size_t)b.n_rows, E = esize(s), W64 = up64(s->cfg.width), WA = act_stride(s->cfg.width);
-    size_t q = 0, c = 0, ql = 0, o = 0, act = 0, act_e = 0, act_s = 0, part = 0, part_s = 0, ints = 0, ctx = 0, kv = 0, ws = 0, le = 0;
+    size_t q = 0, c = 0, ql = 0, o = 0, act = 0, act_e = 0, act_s = 0, part = 0, part_s = 0, ints = 0, ctx = 0, kv = 0, ws = 0, le = 0, dw = 0, dout = 0;
+    const DeltaPart dp = delta_part(b);
     auto gemm = [&](int N, int K) { ws = std::max(ws, w16l_workspace_bytes((int)M, N, K) / 4); };
     for (const pie_stack_layer &L : s->layers) {
         const int NI = in_columns(L), KO = out_columns(L);
@@ -449,6 +462,7 @@ int stack_reserve(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
                 ws = std::max(ws, w16l_workspace_bytes((int)n, (int)nkv, L.rank) / 4);
             }
         }
+        if (L.mixer == PIE_MIXER_DELTA && dp.chunks) dw = std::max(dw, delta_ws_floats(dp.chunks, L.heads, L.dim)), dout = std::max(dout, (size_t)L.heads * up8(L.dim));
         if (L.ff == PIE_FF_RELU2) {
             act = std::max(act, (size_t)act_stride(L.ff_size));
             if (plan.big) gemm(s->cfg.width, L.ff_size);
@@ -468,7 +482,7 @@ int stack_reserve(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
         (rc = s->h.need(M * WA * E, &moved)) || (rc = s->q.need(M * q * E, &moved)) || (rc = s->ql.need(M * ql * E, &moved)) || (rc = s->oc.need(M * ql * E, &moved)) ||
         (rc = s->o.need(M * o * E, &moved)) || (rc = s->act.need(M * act * E, &moved)) || (rc = s->act_e.need(M * act_e * E, &moved)) ||
         (rc = s->act_s.need(M * act_s * E, &moved)) || (rc = s->stats.need((size_t)b.n_want * ST_TILES, &moved)) || (rc = s->y.need(plan.big ? M * W64 * E : 0, &moved)) ||
-        (rc = s->y32.need(plan.big ? 0 : M * W64, &moved)) || (rc = s->logits_e.need(M * le, &moved)) || (rc = s->ctx.need(ctx * E, &moved)) ||
+        (rc = s->y32.need(plan.big ? 0 : M * W64, &moved)) || (rc = s->logits_e.need(M * le, &moved)) || (rc = s->delta_ws.need(dw, &moved)) || (rc = s->delta_o.need(M * dout, &moved)) || (rc = s->ctx.need(ctx * E, &moved)) ||
         (rc = s->kv.need(kv * E, &moved)) || (rc = s->gemm_ws.need(ws, &moved)))
         return rc;
     int n_moe = 0;
@@ -702,7 +716,13 @@ void delta_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm
     d.w_decay = (const u16 *)L.w_decay, d.decay_bias = L.decay_bias, d.o_norm = L.o_norm, d.decay_scale = L.decay_scale, d.unit_eps = L.unit_eps, d.eps = L.eps;
     d.pos = b.pos, d.row_seq = b.row_seq, d.slots = b.slots, d.n_seqs = b.n_seqs, d.n_slots = (int)b.n_slots, d.runs = (const RowRun *)b.runs, d.n_runs = b.n_runs;
     d.state = b.states[li], d.out = s->o.p, d.ld_out = LO;
-    p.rc = delta_step_launch(s->cfg.dtype, d, p.st), ++p.launches;
+    const DeltaPart dp = delta_part(b);
+    d.ws = s->delta_ws.p, d.o = s->delta_o.p, d.n_runs = dp.runs;
+    if (dp.runs) p.rc = delta_step_launch(s->cfg.dtype, d, p.st), ++p.launches;
+    if (!p.rc && dp.chunks) {
+        d.runs += dp.runs, d.n_runs = b.n_runs - dp.runs;
+        p.rc = delta_chunks_launch(s->cfg.dtype, d, dp.chunks, dp.rows, b.n_rows - dp.rows, p.st), p.launches += 3;
+    }
     p.output(L.w_o, s->o.p, LO, KO, L.post1, next);
 }
 

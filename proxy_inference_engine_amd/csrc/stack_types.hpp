@@ -303,10 +303,15 @@ struct DeltaArgs {
     const RowRun *runs;
     int n_runs;
     float *state;           // [n_slots][H][D][D] (key channel, value column)
+    float *ws, *o;          // chunk form: delta_ws_floats(); outputs [M][H][D8] in front of norm and gate
     void *out;              // [M][ld_out] T, head h at h * D8
     int ld_out;
 };
-int delta_step_launch(int dtype, const DeltaArgs &a, hipStream_t st);
+int delta_step_launch(int dtype, const DeltaArgs &a, hipStream_t st);  // token by token
+// runs of many tokens, covering rows [row0, row0 + rows); chunks: sum of delta_chunks() over the runs
+int delta_chunks_launch(int dtype, const DeltaArgs &a, int chunks, int row0, int rows, hipStream_t st);
+int delta_chunks(int n_rows);
+size_t delta_ws_floats(int chunks, int H, int D);
 
 // ---------------------------------------------------------------- x += post(y); h = next(x) with norms that need the whole row (row_update.hip)
 struct StackNorm {

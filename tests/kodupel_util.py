@@ -112,7 +112,7 @@ CONFIGS = {
     "delta_only": config([(delta(), None)]),
     "experts": config([(attention(heads=1, kv_heads=1), moe(ff=30, experts=7, top=3))], width=88, vocab=333),
     "mixed": config(MIXED, width=112, vocab=251, scale=0.7),
-    "odd_sizes": config([(attention(heads=3, kv_heads=3, dim=9, vdim=5, dims=6), moe(ff=3, experts=1, top=1)), (delta(heads=1, dim=1, rank=1), moe(ff=5, experts=2, top=1)),
-                         (delta(heads=5, dim=7, rank=13), None)], width=21, vocab=53, scale=2.5, eps=1e-3),
+    "odd_sizes": config([(attention(heads=3, kv_heads=3, dim=9, vdim=5, dims=6), moe(ff=3, experts=1, top=1)), (delta(heads=1, dim=15, rank=1), moe(ff=5, experts=2, top=1)),
+                         (delta(heads=5, dim=13, rank=13), None)], width=21, vocab=53, scale=2.5, eps=1e-3),
     "many_heads": config([(attention(heads=72, kv_heads=2, dim=8, vdim=8, dims=4), None), (delta(heads=40, dim=8, rank=64), None)], width=128),
 }
