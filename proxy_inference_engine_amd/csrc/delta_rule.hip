@@ -25,6 +25,7 @@ typedef __attribute__((ext_vector_type(8))) __bf16 dr_bf16x8;
 namespace {
 
 constexpr int DC = 16;  // tokens of a chunk
+constexpr size_t DELTA_SEGMENT_BYTES = 96u << 20;
 
 
 template <class E, int CP, int NT>  // CP: power of two >= D; NT threads
@@ -128,6 +129,17 @@ __host__ __device__ __forceinline__ size_t dr_chunk_floats(int D) { return (size
 
 __device__ __forceinline__ dr_f32x4 dr_mfma(float a, float b, const dr_f32x4 &c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
 
+// exp(x) and 1 / (1 + exp(-x)): fp32 stacks take the library's, 16-bit ones the exponential unit (a few units in the last place)
+constexpr float DR_LOG2E = 1.44269504088896340736f;
+template <bool F32>
+__device__ __forceinline__ float dr_exp(float x) {
+    return F32 ? expf(x) : __builtin_amdgcn_exp2f(x * DR_LOG2E);
+}
+template <bool F32>
+__device__ __forceinline__ float dr_sigmoid(float x) {
+    return F32 ? 1.0f / (1.0f + expf(-x)) : __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(x * -DR_LOG2E));
+}
+
 struct DeltaChunk {
     int row0, n;  // rows [row0, row0 + n)
 };
@@ -148,49 +160,76 @@ __global__ void __launch_bounds__(256) k_delta_prep(const DeltaArgs a) {
     constexpr bool F32 = sizeof(T) == 4;
     constexpr int LD = 64 * NB + 4, CH = 64 * NB, PARTS = 256 / CH, TP = DC / PARTS, LM = 20;
     extern __shared__ __attribute__((aligned(16))) char lds[];
-    float *s_l = (float *)lds, *s_m = s_l + DC * LD, *s_unit = s_m + 5 * DC * LM, *s_wc = s_unit + DC;  // log decays; A, B, A', B', T; 1 / |k|; W_16
+    float *s_l = (float *)lds, *s_m = s_l + DC * LD, *s_unit = s_m + 5 * DC * LM, *s_wc = s_unit + DC;  // log decays; A, B (transposed), A', B', T; 1 / |k|; W_16
     float *s_u = s_wc + CH, *s_r = s_u + DC * LD, *s_k = s_r + DC * LD, *s_a = s_k + DC * LD;
     // (the low-rank input of the decay lies where the channel vectors come later)
     const int D = a.D, nblk = dr_blocks(D), lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), n16 = lane & 15, q = lane >> 4;
     const int head = blockIdx.y, HD8 = a.H * a.D8;
-    const DeltaChunk c = dr_chunk(a, blockIdx.x);
+    const DeltaChunk c = dr_chunk(a, a.chunk_lo + (int)blockIdx.x);
     if (c.n <= 0) return;
     const T *raw = (const T *)a.raw + (size_t)c.row0 * a.ld;
     const int R32 = (a.R8 + 31) & ~31, LR = R32 + 8;
     u16 *s_hi = (u16 *)s_u, *s_lo = s_hi + DC * LR;
     float *s_low = s_u;
+    const T *x = raw + head * a.D8;  // this head's r; k, v, gate, rate behind it at HD8 each
+    const u16 *bias = a.bias ? a.bias + head * a.D8 : nullptr;
+    auto channel = [&](int what, int t, int d) { return E::load(x + (size_t)t * a.ld + what * HD8 + d) + (bias ? BF16::to_f32(bias[what * HD8 + d]) : 0.0f); };
+    // (all loads without branches around them: they leave together, and what lies outside is dropped afterwards)
+    float kv[4 * NB];  // a sixteenth of token threadIdx.x / 16's key
+    {
+        const int t = min((int)threadIdx.x >> 4, c.n - 1);
+#pragma unroll
+        for (int j = 0; j < 4 * NB; ++j) kv[j] = channel(1, t, min((int)(threadIdx.x & 15) + 16 * j, D - 1));
+    }
     for (int i = threadIdx.x; i < DC * R32; i += 256) {
         const int t = i / R32, j = i % R32;
-        const float v = t < c.n && j < a.rank ? tanhf(E::load(raw + (size_t)t * a.ld + 5 * HD8 + j) + (a.bias ? BF16::to_f32(a.bias[5 * HD8 + j]) : 0.0f)) : 0.0f;
+        const float z = E::load(raw + (size_t)min(t, c.n - 1) * a.ld + 5 * HD8 + min(j, a.rank - 1)) + (a.bias ? BF16::to_f32(a.bias[5 * HD8 + min(j, a.rank - 1)]) : 0.0f);
+        const float v = t < c.n && j < a.rank ? F32 ? tanhf(z) : fast_tanh(z) : 0.0f;
         if constexpr (F32) s_low[t * LR + j] = v;
         else {
             const u16 hi = BF16::from_f32(v);
             s_hi[t * LR + j] = hi, s_lo[t * LR + j] = BF16::from_f32(v - BF16::to_f32(hi));
         }
     }
-    const T *x = raw + head * a.D8;  // this head's r; k, v, gate, rate behind it at HD8 each
-    const u16 *bias = a.bias ? a.bias + head * a.D8 : nullptr;
-    auto channel = [&](int what, int t, int d) { return E::load(x + (size_t)t * a.ld + what * HD8 + d) + (bias ? BF16::to_f32(bias[what * HD8 + d]) : 0.0f); };
     {
-        const int t = threadIdx.x >> 4;
         float ss = 0.0f;
-        if (t < c.n)
-            for (int d = threadIdx.x & 15; d < D; d += 16) {
-                const float k = channel(1, t, d);
-                ss = fmaf(k, k, ss);
-            }
+#pragma unroll
+        for (int j = 0; j < 4 * NB; ++j) ss = (int)(threadIdx.x & 15) + 16 * j < D ? fmaf(kv[j], kv[j], ss) : ss;
         ss = lanes16_sum(ss);
-        if ((threadIdx.x & 15) == 0) s_unit[t] = 1.0f / sqrtf(ss + a.unit_eps);
+        if ((threadIdx.x & 15) == 0) s_unit[threadIdx.x >> 4] = 1.0f / sqrtf(ss + a.unit_eps);
+    }
+    // the decay's weights (the first WS steps) and the channel vectors, on their way during the barrier and the decay's product
+    constexpr int WS = 4;
+    uint4 wd[F32 ? 1 : NB][WS];
+    float db[NB];
+    auto decay_weights = [&](int j, int s) {
+        const int d = 16 * (wave * NB + j) + n16, at = 32 * s + 8 * q;
+        const uint4 w = *(const uint4 *)(a.w_decay + (size_t)(head * D + min(d, D - 1)) * a.R8 + min(at, a.R8 - 8));
+        return d < D && at < a.R8 ? w : make_uint4(0, 0, 0, 0);
+    };
+    if constexpr (!F32)
+#pragma unroll
+        for (int j = 0; j < NB; ++j) {
+#pragma unroll
+            for (int s = 0; s < WS; ++s) wd[j][s] = decay_weights(j, s);
+            db[j] = a.decay_bias[head * D + min(16 * (wave * NB + j) + n16, D - 1)];
+        }
+    const int pd = threadIdx.x % CH, part = threadIdx.x / CH;
+    float xr[TP], xk[TP], xa[TP];
+#pragma unroll
+    for (int j = 0; j < TP; ++j) {
+        const int t = min(part * TP + j, c.n - 1), d = min(pd, D - 1);
+        xr[j] = channel(0, t, d), xk[j] = channel(1, t, d), xa[j] = channel(4, t, d);
     }
     __syncthreads();
-    auto log_decay = [&](int t, int d, float z) { s_l[t * LD + d] = t < c.n && d < D ? -a.decay_scale / (1.0f + expf(-(z + a.decay_bias[head * D + min(d, D - 1)]))) : 0.0f; };
+    auto log_decay = [&](int t, int d, float z) { s_l[t * LD + d] = t < c.n && d < D ? -a.decay_scale * dr_sigmoid<F32>(z) : 0.0f; };
     if constexpr (F32) {
         for (int i = threadIdx.x; i < DC * 16 * nblk; i += 256) {
             const int t = i / (16 * nblk), d = i % (16 * nblk);
             float z = 0.0f;
             if (d < D)
                 for (int j = 0; j < a.rank; ++j) z = fmaf(s_low[t * LR + j], BF16::to_f32(a.w_decay[(size_t)(head * D + d) * a.R8 + j]), z);
-            log_decay(t, d, z);
+            log_decay(t, d, z + a.decay_bias[head * D + min(d, D - 1)]);
         }
     } else {
 #pragma unroll
@@ -198,36 +237,37 @@ __global__ void __launch_bounds__(256) k_delta_prep(const DeltaArgs a) {
             const int b = wave * NB + j, d = 16 * b + n16;
             if (b >= nblk) break;
             dr_f32x4 z = {0.0f, 0.0f, 0.0f, 0.0f};
-            for (int s = 0; s < R32; s += 32) {
-                const int at = s + 8 * q;
-                const uint4 w = d < D && at < a.R8 ? *(const uint4 *)(a.w_decay + (size_t)(head * D + d) * a.R8 + at) : make_uint4(0, 0, 0, 0);
-                const uint4 hi = *(const uint4 *)(s_hi + n16 * LR + at), lo = *(const uint4 *)(s_lo + n16 * LR + at);
+            auto product = [&](int s, const uint4 &w) {
+                const uint4 hi = *(const uint4 *)(s_hi + n16 * LR + 32 * s + 8 * q), lo = *(const uint4 *)(s_lo + n16 * LR + 32 * s + 8 * q);
                 z = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(dr_bf16x8, hi), __builtin_bit_cast(dr_bf16x8, w), z, 0, 0, 0);
                 z = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(dr_bf16x8, lo), __builtin_bit_cast(dr_bf16x8, w), z, 0, 0, 0);
-            }
+            };
 #pragma unroll
-            for (int i = 0; i < 4; ++i) log_decay(4 * q + i, d, z[i]);
+            for (int s = 0; s < WS; ++s)
+                if (32 * s < R32) product(s, wd[j][s]);
+            for (int s = WS; 32 * s < R32; ++s) product(s, decay_weights(j, s));
+#pragma unroll
+            for (int i = 0; i < 4; ++i) log_decay(4 * q + i, d, z[i] + db[j]);
         }
     }
     __syncthreads();  // the low-rank input has been read
     {
-        const int d = threadIdx.x % CH, part = threadIdx.x / CH;
+        const int d = pd;
         if (part < PARTS && d < 16 * nblk) {
             float L = 0.0f;
             for (int t = 0; t < part * TP; ++t) L += s_l[t * LD + d];
+            float before = dr_exp<F32>(L);
 #pragma unroll
             for (int j = 0; j < TP; ++j) {
                 const int t = part * TP + j;
                 const bool live = t < c.n && d < D;
-                const float before = expf(L);
                 L += s_l[t * LD + d];
-                const float e = expf(L), back = expf(-L);
-                float r = 0.0f, k = 0.0f, ra = 0.0f;
-                if (live) r = channel(0, t, d), k = channel(1, t, d), ra = 1.0f / (1.0f + expf(-channel(4, t, d)));
-                const float u = k * s_unit[t];
-                s_u[t * LD + d] = u * before, s_r[t * LD + d] = r * e, s_k[t * LD + d] = k * back, s_a[t * LD + d] = ra * u * back;
+                const float e = dr_exp<F32>(L), back = dr_exp<F32>(-L);
+                const float r = live ? xr[j] : 0.0f, k = live ? xk[j] : 0.0f, u = k * s_unit[t];
+                s_u[t * LD + d] = u * before, s_r[t * LD + d] = r * e, s_k[t * LD + d] = k * back, s_a[t * LD + d] = dr_sigmoid<F32>(xa[j]) * u * back;
+                before = e;
             }
-            if (part == PARTS - 1) s_wc[d] = expf(L);
+            if (part == PARTS - 1) s_wc[d] = before;
         }
     }
     __syncthreads();
@@ -240,21 +280,29 @@ __global__ void __launch_bounds__(256) k_delta_prep(const DeltaArgs a) {
             for (int i = 0; i < 4; ++i) acc = dr_mfma(lv[i], rv[i], acc);
         }
 #pragma unroll
-        for (int i = 0; i < 4; ++i) s_m[(wave * DC + 4 * q + i) * LM + n16] = n16 < 4 * q + i + (wave >= 2) ? acc[i] : 0.0f;
+        for (int i = 0; i < 4; ++i) acc[i] = n16 < 4 * q + i + (wave >= 2) ? acc[i] : 0.0f;
+        if (wave == 1) *(dr_f32x4 *)(s_m + (DC + n16) * LM + 4 * q) = acc;  // (B transposed)
+        else
+#pragma unroll
+            for (int i = 0; i < 4; ++i) s_m[(wave * DC + 4 * q + i) * LM + n16] = acc[i];
     }
     __syncthreads();
     float *out = a.ws + ((size_t)blockIdx.x * a.H + head) * dr_chunk_floats(D);
     float *o_r = out + nblk * 256, *o_k = o_r + nblk * 256, *o_a = o_k + nblk * 256, *o_m = o_a + nblk * 256;
     float *s_t = s_m + 4 * DC * LM;
     if (wave == 0) {
-        float tc[DC];  // column n16 of (I + B)^-1
+        float tc[DC];  // column n16 of (I + B)^-1: forward substitution, column by column of B (stored transposed: rows are read whole)
 #pragma unroll
-        for (int t = 0; t < DC; ++t) {
-            float v = t == n16 ? 1.0f : 0.0f;
+        for (int t = 0; t < DC; ++t) tc[t] = t == n16 ? 1.0f : 0.0f;
 #pragma unroll
-            for (int i = 0; i < t; ++i) v = fmaf(-s_m[(DC + t) * LM + i], tc[i], v);
-            tc[t] = v;
-        }
+        for (int i = 0; i < DC - 1; ++i)
+#pragma unroll
+            for (int t4 = i / 4; t4 < DC / 4; ++t4) {
+                const dr_f32x4 col = *(const dr_f32x4 *)(s_m + (DC + i) * LM + 4 * t4);
+#pragma unroll
+                for (int k = 0; k < 4; ++k)
+                    if (4 * t4 + k > i) tc[4 * t4 + k] = fmaf(-col[k], tc[i], tc[4 * t4 + k]);
+            }
         if (q == 0)
 #pragma unroll
             for (int t = 0; t < DC; ++t) s_t[t * LM + n16] = tc[t];
@@ -290,19 +338,32 @@ __global__ void __launch_bounds__(256) k_delta_prep(const DeltaArgs a) {
     }
 }
 
+// A chunk's operands are further away than a chunk takes, so they travel through LDS by DMA, RING - 1 chunks ahead; every wave fetches, waits for and reads
+// only its own.
 template <class E, int NB>
-__global__ void __launch_bounds__(256) k_delta_scan(const DeltaArgs a) {
+struct ScanLds {
+    static constexpr int DW = 16 * sizeof(typename E::type) / 4, VI = 16 * DW / 64;  // dwords of a token's 16 values; DMA instructions for the chunk's
+    static constexpr int OPS = 4 * NB + 2 + VI;                                      // DMA instructions per wave and chunk
+    static constexpr int WAVE = (4 * NB + 2) * 1024 + VI * 256, SLOT = 4 * WAVE;
+    static constexpr int PB = NB <= 3 ? 2 : 1;  // buffers of the exchanges between the waves
+    static constexpr int RING = 5 * SLOT <= 128 * 1024 ? 5 : 3 * SLOT <= 136 * 1024 ? 3 : 2;
+};
+template <class E, int NB>
+__global__ void __launch_bounds__(256, 1) k_delta_scan(const DeltaArgs a) {
     typedef typename E::type T;
-    __shared__ dr_f32x4 s_p[2][4][64], s_o[2][4][64];
+    typedef ScanLds<E, NB> L;
+    __shared__ __attribute__((aligned(1024))) char s_ring[L::RING * L::SLOT];
+    __shared__ dr_f32x4 s_p[L::PB][4][64], s_o[L::PB][4][64];
     const int D = a.D, nblk = dr_blocks(D), lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), n16 = lane & 15, q = lane >> 4;
     const int head = (int)blockIdx.x % a.H, cb = (int)blockIdx.x / a.H, col = 16 * cb + n16;  // (head fastest: the column blocks of a head share an L2 where H is a multiple of 8)
     const RowRun run = a.runs[blockIdx.y];
     int chunk0 = 0;
     for (int r = 0; r < (int)blockIdx.y; ++r) chunk0 += (a.runs[r].n_rows + DC - 1) / DC;
-    const int chunks = (run.n_rows + DC - 1) / DC;
+    const int c_lo = max(a.chunk_lo - chunk0, 0), c_hi = min(a.chunk_hi - chunk0, (run.n_rows + DC - 1) / DC);  // this launch's chunks of the run
+    if (c_lo >= c_hi) return;
     const size_t slot = min((unsigned)a.slots[min(a.row_seq[run.row0], a.n_seqs - 1)], (unsigned)a.n_slots - 1u);
     float *state = a.state + (slot * a.H + head) * D * D;
-    const bool fresh = a.pos[run.row0] == 0;
+    const bool fresh = c_lo == 0 && a.pos[run.row0] == 0;
     dr_f32x4 S[NB];  // S[16 b + 4 q + i][col]
 #pragma unroll
     for (int j = 0; j < NB; ++j)
@@ -312,84 +373,117 @@ __global__ void __launch_bounds__(256) k_delta_scan(const DeltaArgs a) {
             S[j][i] = !fresh && d < D && col < D ? state[(size_t)d * D + col] : 0.0f;
         }
     const size_t per = dr_chunk_floats(D);
-    const float *ws = a.ws + ((size_t)chunk0 * a.H + head) * per;
-    const T *vp = (const T *)a.raw + (size_t)run.row0 * a.ld + 2 * a.H * a.D8 + head * a.D8 + min(col, D - 1);
+    const float *ws = a.ws + ((ptrdiff_t)(chunk0 - a.chunk_lo) * a.H + head) * (ptrdiff_t)per;  // chunk c of the run at c * H * per
+    const char *vp = (const char *)((const T *)a.raw + (size_t)run.row0 * a.ld + 2 * a.H * a.D8 + head * a.D8 + 16 * cb);
     const float vbias = a.bias ? BF16::to_f32(a.bias[2 * a.H * a.D8 + head * a.D8 + min(col, D - 1)]) : 0.0f;
-    struct Operands {
-        dr_f32x4 u[NB], r[NB], k[NB], m[NB], w[NB], v, x;  // x: T A (wave 0), A' (wave 1), -B' (wave 2)
+    const unsigned lds0 = (unsigned)(size_t)(__attribute__((address_space(3))) void *)s_ring + (unsigned)(wave * L::WAVE);
+    auto scalar = [&](const void *p) {
+        const unsigned long long v = (unsigned long long)(uintptr_t)p;
+        return (unsigned long long)(unsigned)__builtin_amdgcn_readfirstlane((int)(unsigned)v) | ((unsigned long long)(unsigned)__builtin_amdgcn_readfirstlane((int)(unsigned)(v >> 32)) << 32);
     };
-    const dr_f32x4 zero = {0.0f, 0.0f, 0.0f, 0.0f};
-    auto load = [&](int c, Operands &o) {
-        const float *p = ws + (size_t)c * a.H * per;
+    auto fetch = [&](int cc, int at) {  // chunk cc (behind the end: the last one again, the waits count instructions) into ring slot `at`
+        const int c = min(cc, c_hi - 1);
+        const unsigned dst0 = lds0 + (unsigned)(at * L::SLOT);
+        const unsigned long long base = scalar(ws + (size_t)c * a.H * per);
+        auto piece = [&](unsigned byte, unsigned dst) {
+            unsigned keep;
+            asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %3\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, %2\n\ts_mov_b32 m0, %0"
+                         : "=&s"(keep)
+                         : "v"(byte + (unsigned)lane * 16u), "s"(base), "s"(dst)
+                         : "memory");
+        };
 #pragma unroll
         for (int j = 0; j < NB; ++j) {
-            const int b = wave * NB + j;
-            if (b < nblk) {
-                const float *pb = p + b * 256 + lane * 4;
-                o.u[j] = *(const dr_f32x4 *)pb, o.r[j] = *(const dr_f32x4 *)(pb + nblk * 256), o.k[j] = *(const dr_f32x4 *)(pb + 2 * nblk * 256), o.m[j] = *(const dr_f32x4 *)(pb + 3 * nblk * 256);
-                o.w[j] = *(const dr_f32x4 *)(p + nblk * 1024 + 768 + 16 * b + 4 * q);
-            } else o.u[j] = o.r[j] = o.k[j] = o.m[j] = o.w[j] = zero;
-        }
-        o.x = *(const dr_f32x4 *)(p + nblk * 1024 + min(wave, 2) * 256 + lane * 4);
+            const int b = min(wave * NB + j, nblk - 1);  // (blocks past the end meet channels that stay zero)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int t = DC * c + 4 * q + i;
-            const float v = E::load(vp + (size_t)min(t, run.n_rows - 1) * a.ld) + vbias;
-            o.v[i] = t < run.n_rows && col < D ? v : 0.0f;
+            for (int k = 0; k < 4; ++k) piece((unsigned)(k * nblk + b) * 1024u, dst0 + (unsigned)(4 * j + k) * 1024u);
+        }
+        piece((unsigned)nblk * 4096u + (unsigned)min(wave, 2) * 1024u, dst0 + 4096u * NB);
+        piece((unsigned)nblk * 4096u + 3072u, dst0 + 4096u * NB + 1024u);  // W_16 of all channels (and what lies behind it)
+        const unsigned long long vbase = scalar(vp + (size_t)(DC * c) * a.ld * sizeof(T));
+#pragma unroll
+        for (int k = 0; k < L::VI; ++k) {
+            const int t = min((64 / L::DW) * k + lane / L::DW, run.n_rows - 1 - DC * c);
+            const unsigned off = (unsigned)(t * a.ld) * (unsigned)sizeof(T) + (unsigned)(lane % L::DW) * 4u;
+            unsigned keep;
+            asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %3\n\ts_nop 0\n\tglobal_load_lds_dword %1, %2\n\ts_mov_b32 m0, %0"
+                         : "=&s"(keep)
+                         : "v"(off), "s"(vbase), "s"(dst0 + 4096u * NB + 2048u + 256u * k)
+                         : "memory");
         }
     };
+    const dr_f32x4 zero = {0.0f, 0.0f, 0.0f, 0.0f};
     auto store_o = [&](int c) {  // chunk c's outputs: one per thread
-        const float *p = (const float *)s_o[c & 1] + threadIdx.x;
+        const float *p = (const float *)s_o[c % L::PB] + threadIdx.x;
         const float o = (p[0] + p[256]) + (p[512] + p[768]);
         const int l = threadIdx.x >> 2, t = DC * c + 4 * (l >> 4) + (threadIdx.x & 3), d = 16 * cb + (l & 15);
         if (t < run.n_rows && d < D) a.o[((size_t)(run.row0 + t) * a.H + head) * a.D8 + d] = o;
     };
-    auto step = [&](int c, const Operands &o) {
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // (the state's loads: the waits below count DMAs)
+#pragma unroll
+    for (int i = 0; i < L::RING - 1; ++i) fetch(c_lo + i, i);
+    int at = 0;
+    for (int c = c_lo; c < c_hi; ++c) {
+        asm volatile("s_waitcnt vmcnt(%0)" ::"n"((L::RING - 2) * L::OPS) : "memory");
+        fetch(c + L::RING - 1, at ? at - 1 : L::RING - 1);  // into the previous chunk's slot
+        const char *mine = s_ring + at * L::SLOT + wave * L::WAVE;
+        at = at + 1 < L::RING ? at + 1 : 0;
+        auto operand = [&](int piece) { return *(const dr_f32x4 *)(mine + piece * 1024 + lane * 16); };
+        dr_f32x4 u[NB], r[NB], k[NB], m[NB], w[NB], v, x = operand(4 * NB);
+#pragma unroll
+        for (int j = 0; j < NB; ++j) u[j] = operand(4 * j);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int t = 4 * q + i;
+            const float e = E::load((const T *)(mine + (4 * NB + 2) * 1024) + t * 16 + n16) + vbias;
+            v[i] = DC * c + t < run.n_rows && col < D ? e : 0.0f;
+        }
+#pragma unroll
+        for (int j = 0; j < NB; ++j) r[j] = operand(4 * j + 1), k[j] = operand(4 * j + 2), w[j] = *(const dr_f32x4 *)(mine + (4 * NB + 1) * 1024 + (16 * min(wave * NB + j, nblk - 1) + 4 * q) * 4);
         dr_f32x4 P = zero, O = zero;
 #pragma unroll
         for (int j = 0; j < NB; ++j)
 #pragma unroll
-            for (int i = 0; i < 4; ++i) P = dr_mfma(o.u[j][i], S[j][i], P);
+            for (int i = 0; i < 4; ++i) P = dr_mfma(u[j][i], S[j][i], P);
         if (wave == 0)
 #pragma unroll
-            for (int i = 0; i < 4; ++i) P = dr_mfma(o.x[i], o.v[i], P);
-        s_p[c & 1][wave][lane] = P;
+            for (int i = 0; i < 4; ++i) P = dr_mfma(x[i], v[i], P);
+        s_p[c % L::PB][wave][lane] = P;
+#pragma unroll
+        for (int j = 0; j < NB; ++j) m[j] = operand(4 * j + 3);
 #pragma unroll
         for (int j = 0; j < NB; ++j)
 #pragma unroll
-            for (int i = 0; i < 4; ++i) O = dr_mfma(o.r[j][i], S[j][i], O);
+            for (int i = 0; i < 4; ++i) O = dr_mfma(r[j][i], S[j][i], O);
         if (wave == 1)
 #pragma unroll
-            for (int i = 0; i < 4; ++i) O = dr_mfma(o.x[i], o.v[i], O);
+            for (int i = 0; i < 4; ++i) O = dr_mfma(x[i], v[i], O);
 #pragma unroll
-        for (int j = 0; j < NB; ++j) S[j] *= o.w[j];
-#pragma unroll
-        for (int i = 0; i < 4; ++i)
-#pragma unroll
-            for (int j = 0; j < NB; ++j) S[j] = dr_mfma(o.k[j][i], o.v[i], S[j]);
-        __syncthreads();
-        P = (s_p[c & 1][0][lane] + s_p[c & 1][1][lane]) + (s_p[c & 1][2][lane] + s_p[c & 1][3][lane]);
-        if (c > 0) store_o(c - 1);
+        for (int j = 0; j < NB; ++j) S[j] *= w[j];
 #pragma unroll
         for (int i = 0; i < 4; ++i)
 #pragma unroll
-            for (int j = 0; j < NB; ++j) S[j] = dr_mfma(o.m[j][i], P[i], S[j]);
+            for (int j = 0; j < NB; ++j) S[j] = dr_mfma(k[j][i], v[i], S[j]);
+        // the four waves' shares of P meet (LDS only: the DMAs stay in flight)
+        asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+        P = (s_p[c % L::PB][0][lane] + s_p[c % L::PB][1][lane]) + (s_p[c % L::PB][2][lane] + s_p[c % L::PB][3][lane]);
+        if (c > c_lo) store_o(c - 1);
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+#pragma unroll
+            for (int j = 0; j < NB; ++j) S[j] = dr_mfma(m[j][i], P[i], S[j]);
         if (wave == 2)
 #pragma unroll
-            for (int i = 0; i < 4; ++i) O = dr_mfma(o.x[i], P[i], O);
-        s_o[c & 1][wave][lane] = O;
-    };
-    Operands even, odd;
-    load(0, even);
-    for (int c = 0; c < chunks; c += 2) {
-        load(min(c + 1, chunks - 1), odd);
-        step(c, even);
-        if (c + 1 >= chunks) break;
-        load(min(c + 2, chunks - 1), even);
-        step(c + 1, odd);
+            for (int i = 0; i < 4; ++i) O = dr_mfma(x[i], P[i], O);
+#pragma unroll
+        for (int j = 0; j < NB; ++j)
+            if (wave * NB + j >= nblk) S[j] = zero;  // (a block that does not exist saw another's operands)
+        if constexpr (L::PB == 1) asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");  // everyone has read P and the previous outputs
+        s_o[c % L::PB][wave][lane] = O;
     }
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // the look-ahead DMAs: LDS is handed on when the workgroup ends
     __syncthreads();
-    store_o(chunks - 1);
+    store_o(c_hi - 1);
 #pragma unroll
     for (int j = 0; j < NB; ++j)
 #pragma unroll
@@ -422,6 +516,12 @@ __global__ void __launch_bounds__(256) k_delta_out(const DeltaArgs a, int row0) 
     }
 }
 
+// chunks whose operands are made and used at a time
+int delta_segment(int H, int D) {
+    const size_t bytes = H * dr_chunk_floats(D) * 4;
+    return (int)std::max((size_t)16, DELTA_SEGMENT_BYTES / bytes);
+}
+
 size_t delta_prep_lds(int NB, int R8) {
     const int R32 = (R8 + 31) & ~31;
     const size_t vec = (size_t)DC * (64 * NB + 4) * 4, low = (size_t)DC * (R32 + 8) * 4;  // (fp32, or bf16 halves)
@@ -437,10 +537,15 @@ int delta_chunks_nb(const DeltaArgs &a, int chunks, int row0, int rows, hipStrea
         PIE_HIP_TRY(hipFuncSetAttribute((const void *)k_delta_prep<E, NB>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024));
         raised = true;
     }
-    hipLaunchKernelGGL((k_delta_prep<E, NB>), dim3((unsigned)chunks, (unsigned)a.H), dim3(256), lds, st, a);
-    PIE_LAUNCH_CHECK();
-    hipLaunchKernelGGL((k_delta_scan<E, NB>), dim3((unsigned)(a.H * dr_blocks(a.D)), (unsigned)a.n_runs), dim3(256), 0, st, a);
-    PIE_LAUNCH_CHECK();
+    DeltaArgs seg = a;
+    const int step = delta_segment(a.H, a.D);
+    for (int c = 0; c < chunks; c += step) {  // a segment's operands are read back before they leave the last-level cache
+        seg.chunk_lo = c, seg.chunk_hi = std::min(chunks, c + step);
+        hipLaunchKernelGGL((k_delta_prep<E, NB>), dim3((unsigned)(seg.chunk_hi - c), (unsigned)a.H), dim3(256), lds, st, seg);
+        PIE_LAUNCH_CHECK();
+        hipLaunchKernelGGL((k_delta_scan<E, NB>), dim3((unsigned)(a.H * dr_blocks(a.D)), (unsigned)a.n_runs), dim3(256), 0, st, seg);
+        PIE_LAUNCH_CHECK();
+    }
     hipLaunchKernelGGL(k_delta_out<E>, dim3((unsigned)rows, (unsigned)((a.H + 3) / 4)), dim3(256), 0, st, a, row0);
     PIE_LAUNCH_CHECK();
     return PIE_OK;
@@ -470,7 +575,8 @@ int delta_step_go(const DeltaArgs &a, hipStream_t st) {
 }  // namespace
 
 int delta_chunks(int n_rows) { return (n_rows + DC - 1) / DC; }
-size_t delta_ws_floats(int chunks, int H, int D) { return (size_t)chunks * H * dr_chunk_floats(D); }
+size_t delta_ws_floats(int chunks, int H, int D) { return (size_t)std::min(chunks, delta_segment(H, D)) * H * dr_chunk_floats(D); }
+int delta_launches(int chunks, int H, int D) { return 2 * ((chunks + delta_segment(H, D) - 1) / delta_segment(H, D)) + 1; }
 
 static int delta_check(const DeltaArgs &a) {
     PIE_REQUIRE(a.D > 0 && a.D <= DELTA_MAX_DIM && a.rank > 0 && a.rank <= DELTA_MAX_RANK && a.H > 0 && a.H <= 65535, PIE_E_SHAPE,

@@ -721,7 +721,7 @@ void delta_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm
     if (dp.runs) p.rc = delta_step_launch(s->cfg.dtype, d, p.st), ++p.launches;
     if (!p.rc && dp.chunks) {
         d.runs += dp.runs, d.n_runs = b.n_runs - dp.runs;
-        p.rc = delta_chunks_launch(s->cfg.dtype, d, dp.chunks, dp.rows, b.n_rows - dp.rows, p.st), p.launches += 3;
+        p.rc = delta_chunks_launch(s->cfg.dtype, d, dp.chunks, dp.rows, b.n_rows - dp.rows, p.st), p.launches += delta_launches(dp.chunks, L.heads, L.dim);
     }
     p.output(L.w_o, s->o.p, LO, KO, L.post1, next);
 }

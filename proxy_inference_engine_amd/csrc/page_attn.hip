@@ -20,50 +20,92 @@ namespace {
 constexpr float PG_NEG = -1e30f, PG_LOG2E = 1.44269504088896340736f;
 
 // ---------------------------------------------------------------- projections -> queries, pages
-// one wave per (row, head): heads [0, H) queries, [H, H + G) keys, [H + G, H + 2 G) values
-template <class E>
+// One wave per row and run of PREP_HEADS heads: heads [0, H) queries, [H, H + G) keys, [H + G, H + 2 G) values.  Lane l holds the dimension pairs l, l + 64, ...
+// of a head; their angles are taken once for all heads of the wave.  NP: pairs per lane.
+constexpr int PREP_HEADS = 8;
+template <class E, int NP>
 __global__ void __launch_bounds__(256) k_kv_prep(const KvPrepArgs a) {
     typedef typename E::type T;
     const KvGeometry &geo = a.geo;
-    const int m = blockIdx.x, head = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-    if (head >= geo.H + (a.own ? 2 * geo.G : 0)) return;
-    const bool is_q = head < geo.H, is_v = head >= geo.H + geo.G;
-    const int g = is_q ? head : head - geo.H - (is_v ? geo.G : 0), n = is_v ? geo.vdim : geo.dim;
-    const int off = is_q ? head * geo.D8 : geo.H * geo.D8 + (is_v ? geo.G * geo.D8 + g * geo.V8 : g * geo.D8);
-    T *x = (T *)a.raw + (size_t)m * a.ld + off;
-    const u16 *bias = a.bias ? a.bias + off : nullptr;
-    const int t = a.pos[m];
-    auto elem = [&](int d) { return d < n ? E::load(x + d) + (bias ? BF16::to_f32(bias[d]) : 0.0f) : 0.0f; };
-    const float *w = is_v ? nullptr : is_q ? a.q_norm : a.k_norm;
-    float inv = 1.0f;
-    if (is_v ? a.value_norm : w != nullptr) {
-        float ss = 0.0f;
-        for (int d = 2 * lane; d < n; d += 128) {
-            const float u = elem(d), v = elem(d + 1);
-            ss = fmaf(u, u, fmaf(v, v, ss));
+    const int m = blockIdx.x, lane = threadIdx.x & 63, heads = geo.H + (a.own ? 2 * geo.G : 0), head0 = (blockIdx.y * 4 + (threadIdx.x >> 6)) * PREP_HEADS;
+    if (head0 >= heads) return;
+    const int t = a.pos[m], tl = t & (PAGE_TOKENS - 1);
+    T *page = a.own && head0 + PREP_HEADS > geo.H ? (T *)a.slab + (size_t)page_of(a.pages, a.row_seq[m], t) * geo.page_elems() : nullptr;
+    float sn[NP], cs[NP];
+    if (head0 < geo.H + geo.G)
+#pragma unroll
+        for (int j = 0; j < NP; ++j) {
+            const int d = 2 * (lane + 64 * j);
+            sn[j] = 0.0f, cs[j] = 1.0f;
+            if (d + 1 < a.rot_dims) {
+                sincosf((float)t * a.freq[d >> 1], &sn[j], &cs[j]);
+                sn[j] *= a.rot_gain, cs[j] *= a.rot_gain;
+            }
         }
-        inv = 1.0f / sqrtf(wave_sum(ss) / (float)n + a.eps);
-    }
-    T *page = nullptr;
-    if (!is_q) page = (T *)a.slab + (size_t)page_of(a.pages, a.row_seq[m], t) * geo.page_elems() + g * geo.head_elems();
-    const int tl = t & (PAGE_TOKENS - 1);
-    for (int d = 2 * lane; d < n; d += 128) {
-        float u = elem(d) * inv, v = elem(d + 1) * inv;
-        if (w) u *= w[d], v = d + 1 < n ? v * w[d + 1] : 0.0f;
-        if (!is_v && d + 1 < a.rot_dims) {
-            float s, c;
-            sincosf((float)t * a.freq[d >> 1], &s, &c);
-            s *= a.rot_gain, c *= a.rot_gain;
-            const float u2 = u * c - v * s;
-            v = v * c + u * s, u = u2;
+    constexpr int HB = NP == 1 ? 8 : NP == 2 ? 4 : 1;  // heads in flight
+    static_assert(PREP_HEADS % HB == 0, "whole batches of heads");
+    for (int h0 = head0; h0 < min(head0 + PREP_HEADS, heads); h0 += HB) {
+        float u[HB][NP], v[HB][NP];
+        auto offset = [&](int head) {
+            return head < geo.H + geo.G ? head * geo.D8 : (geo.H + geo.G) * geo.D8 + (head - geo.H - geo.G) * geo.V8;
+        };
+#pragma unroll
+        for (int k = 0; k < HB; ++k) {
+            const int head = min(h0 + k, heads - 1), n = head >= geo.H + geo.G ? geo.vdim : geo.dim, off = offset(head);
+            const T *x = (const T *)a.raw + (size_t)m * a.ld + off;
+#pragma unroll
+            for (int j = 0; j < NP; ++j) {
+                const int d = 2 * (lane + 64 * j), dd = min(d, (n - 1) & ~1);
+                float p, r;  // (an odd head's last partner is its padding: zero)
+                if constexpr (sizeof(T) == 2) {
+                    const u32 w = *(const u32 *)(x + dd);
+                    p = lo_f32<BF16>(w), r = hi_f32<BF16>(w);
+                } else {
+                    const float2 w = *(const float2 *)(x + dd);
+                    p = w.x, r = w.y;
+                }
+                if (a.bias) {
+                    const u32 w = *(const u32 *)(a.bias + off + dd);  // (padded like the head)
+                    p += lo_f32<BF16>(w), r += hi_f32<BF16>(w);
+                }
+                u[k][j] = d < n ? p : 0.0f, v[k][j] = d + 1 < n ? r : 0.0f;
+            }
         }
-        if (is_v) {
-            page[geo.value(tl, d)] = E::pack(u);
-            if (d + 1 < n) page[geo.value(tl, d + 1)] = E::pack(v);
-        } else {
-            T *dst = is_q ? x + d : page + geo.key(tl, d);  // (d even: both in one 8-dimension chunk, and the pair aligned)
-            if constexpr (sizeof(T) == 2) *(u32 *)dst = pack2<BF16>(u, v);  // (an odd head's last partner is its padding: zero)
-            else *(float2 *)dst = make_float2(u, v);
+#pragma unroll
+        for (int k = 0; k < HB; ++k) {
+            const int head = h0 + k;
+            if (head >= min(head0 + PREP_HEADS, heads)) break;
+            const bool is_q = head < geo.H, is_v = head >= geo.H + geo.G;
+            const int g = is_q ? head : head - geo.H - (is_v ? geo.G : 0), n = is_v ? geo.vdim : geo.dim;
+            const float *w = is_v ? nullptr : is_q ? a.q_norm : a.k_norm;
+            float inv = 1.0f;
+            if (is_v ? a.value_norm : w != nullptr) {
+                float ss = 0.0f;
+#pragma unroll
+                for (int j = 0; j < NP; ++j) ss = fmaf(u[k][j], u[k][j], fmaf(v[k][j], v[k][j], ss));
+                inv = 1.0f / sqrtf(wave_sum(ss) / (float)n + a.eps);
+            }
+            T *x = (T *)a.raw + (size_t)m * a.ld + offset(head);
+#pragma unroll
+            for (int j = 0; j < NP; ++j) {
+                const int d = 2 * (lane + 64 * j);
+                if (d >= n) break;
+                float p = u[k][j] * inv, r = v[k][j] * inv;
+                if (is_v) {
+                    T *dst = page + g * geo.head_elems();
+                    dst[geo.value(tl, d)] = E::pack(p);
+                    if (d + 1 < n) dst[geo.value(tl, d + 1)] = E::pack(r);
+                    continue;
+                }
+                if (w) p *= w[d], r = d + 1 < n ? r * w[d + 1] : 0.0f;
+                if (d + 1 < a.rot_dims) {
+                    const float p2 = p * cs[j] - r * sn[j];
+                    r = r * cs[j] + p * sn[j], p = p2;
+                }
+                T *dst = is_q ? x + d : page + g * geo.head_elems() + geo.key(tl, d);  // (d even: both in one 8-dimension chunk, and the pair aligned)
+                if constexpr (sizeof(T) == 2) *(u32 *)dst = pack2<BF16>(p, r);
+                else *(float2 *)dst = make_float2(p, r);
+            }
         }
     }
 }
@@ -411,9 +453,13 @@ bool page_attn_mfma(int dtype, const KvGeometry &g) { return dtype == PIE_BF16 &
 
 int kv_prep_launch(int dtype, const KvPrepArgs &a, hipStream_t st) {
     if (a.M <= 0) return PIE_OK;
-    const dim3 grid((unsigned)a.M, (unsigned)((a.geo.H + (a.own ? 2 * a.geo.G : 0) + 3) / 4));
-    if (dtype == PIE_F32) hipLaunchKernelGGL(k_kv_prep<ElemF32>, grid, dim3(256), 0, st, a);
-    else hipLaunchKernelGGL(k_kv_prep<ElemBF16>, grid, dim3(256), 0, st, a);
+    const dim3 grid((unsigned)a.M, (unsigned)((a.geo.H + (a.own ? 2 * a.geo.G : 0) + 4 * PREP_HEADS - 1) / (4 * PREP_HEADS)));
+    const int wide = a.geo.dim > a.geo.vdim ? a.geo.dim : a.geo.vdim;
+#define PREP_GO(NP_) \
+    if (dtype == PIE_F32) hipLaunchKernelGGL((k_kv_prep<ElemF32, NP_>), grid, dim3(256), 0, st, a); \
+    else hipLaunchKernelGGL((k_kv_prep<ElemBF16, NP_>), grid, dim3(256), 0, st, a)
+    if (wide <= 128) { PREP_GO(1); } else if (wide <= 256) { PREP_GO(2); } else { PREP_GO(8); }
+#undef PREP_GO
     PIE_LAUNCH_CHECK();
     return PIE_OK;
 }

@@ -304,6 +304,7 @@ struct DeltaArgs {
     int n_runs;
     float *state;           // [n_slots][H][D][D] (key channel, value column)
     float *ws, *o;          // chunk form: delta_ws_floats(); outputs [M][H][D8] in front of norm and gate
+    int chunk_lo, chunk_hi; // (set by the launcher: the chunks of one segment)
     void *out;              // [M][ld_out] T, head h at h * D8
     int ld_out;
 };
@@ -312,6 +313,7 @@ int delta_step_launch(int dtype, const DeltaArgs &a, hipStream_t st);  // token 
 int delta_chunks_launch(int dtype, const DeltaArgs &a, int chunks, int row0, int rows, hipStream_t st);
 int delta_chunks(int n_rows);
 size_t delta_ws_floats(int chunks, int H, int D);
+int delta_launches(int chunks, int H, int D);
 
 // ---------------------------------------------------------------- x += post(y); h = next(x) with norms that need the whole row (row_update.hip)
 struct StackNorm {
