@@ -153,52 +153,63 @@ __device__ __forceinline__ DeltaChunk dr_chunk(const DeltaArgs &a, int i) {
     return {a.runs[r].row0 + DC * i, min(DC, a.runs[r].n_rows - DC * i)};
 }
 
-// NB: 16-channel blocks per wave (D <= 64 NB).  Dynamic LDS: see delta_prep_lds().
+__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }  // (loads and stores stay in flight)
+
+// One workgroup per (chunk, head).  A wave owns four tokens; its lanes own channel pairs.
+// NB: 16-channel blocks per wave in the products (D <= 64 NB).  Dynamic LDS: see delta_prep_lds().
 template <class E, int NB>
 __global__ void __launch_bounds__(256) k_delta_prep(const DeltaArgs a) {
     typedef typename E::type T;
     constexpr bool F32 = sizeof(T) == 4;
-    constexpr int LD = 64 * NB + 4, CH = 64 * NB, PARTS = 256 / CH, TP = DC / PARTS, LM = 20;
+    constexpr int LD = 64 * NB + 4, NP = (NB + 1) / 2, TP = DC / 4, LM = 20;  // NP: channel pairs per lane; TP: tokens per wave
     extern __shared__ __attribute__((aligned(16))) char lds[];
-    float *s_l = (float *)lds, *s_m = s_l + DC * LD, *s_unit = s_m + 5 * DC * LM, *s_wc = s_unit + DC;  // log decays; A, B (transposed), A', B', T; 1 / |k|; W_16
-    float *s_u = s_wc + CH, *s_r = s_u + DC * LD, *s_k = s_r + DC * LD, *s_a = s_k + DC * LD;
+    float *s_l = (float *)lds, *s_m = s_l + DC * LD, *s_wc = s_m + 5 * DC * LM;  // log decays; A, B (transposed), A', B', T; W_16
+    float *s_u = s_wc + 64 * NB, *s_r = s_u + DC * LD, *s_k = s_r + DC * LD, *s_a = s_k + DC * LD;
     // (the low-rank input of the decay lies where the channel vectors come later)
     const int D = a.D, nblk = dr_blocks(D), lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), n16 = lane & 15, q = lane >> 4;
-    const int head = blockIdx.y, HD8 = a.H * a.D8;
-    const DeltaChunk c = dr_chunk(a, a.chunk_lo + (int)blockIdx.x);
+    const int head = blockIdx.x, HD8 = a.H * a.D8;  // (head fastest: workgroups that run together read whole rows)
+    const DeltaChunk c = dr_chunk(a, a.chunk_lo + (int)blockIdx.y);
     if (c.n <= 0) return;
-    const T *raw = (const T *)a.raw + (size_t)c.row0 * a.ld;
     const int R32 = (a.R8 + 31) & ~31, LR = R32 + 8;
     u16 *s_hi = (u16 *)s_u, *s_lo = s_hi + DC * LR;
     float *s_low = s_u;
-    const T *x = raw + head * a.D8;  // this head's r; k, v, gate, rate behind it at HD8 each
-    const u16 *bias = a.bias ? a.bias + head * a.D8 : nullptr;
-    auto channel = [&](int what, int t, int d) { return E::load(x + (size_t)t * a.ld + what * HD8 + d) + (bias ? BF16::to_f32(bias[what * HD8 + d]) : 0.0f); };
-    // (all loads without branches around them: they leave together, and what lies outside is dropped afterwards)
-    float kv[4 * NB];  // a sixteenth of token threadIdx.x / 16's key
-    {
-        const int t = min((int)threadIdx.x >> 4, c.n - 1);
-#pragma unroll
-        for (int j = 0; j < 4 * NB; ++j) kv[j] = channel(1, t, min((int)(threadIdx.x & 15) + 16 * j, D - 1));
-    }
-    for (int i = threadIdx.x; i < DC * R32; i += 256) {
-        const int t = i / R32, j = i % R32;
-        const float z = E::load(raw + (size_t)min(t, c.n - 1) * a.ld + 5 * HD8 + min(j, a.rank - 1)) + (a.bias ? BF16::to_f32(a.bias[5 * HD8 + min(j, a.rank - 1)]) : 0.0f);
-        const float v = t < c.n && j < a.rank ? F32 ? tanhf(z) : fast_tanh(z) : 0.0f;
-        if constexpr (F32) s_low[t * LR + j] = v;
+    struct Pair {
+        float x, y;
+    };
+    auto pair_at = [&](const T *p) -> Pair {
+        if constexpr (F32) return {((const float2 *)p)->x, ((const float2 *)p)->y};
         else {
-            const u16 hi = BF16::from_f32(v);
-            s_hi[t * LR + j] = hi, s_lo[t * LR + j] = BF16::from_f32(v - BF16::to_f32(hi));
+            const u32 w = *(const u32 *)p;
+            return {lo_f32<BF16>(w), hi_f32<BF16>(w)};
         }
-    }
-    {
-        float ss = 0.0f;
+    };
+    auto bias_at = [&](int at) -> Pair {
+        if (!a.bias) return {0.0f, 0.0f};
+        const u32 w = *(const u32 *)(a.bias + at);
+        return {lo_f32<BF16>(w), hi_f32<BF16>(w)};
+    };
+    // All loads without branches around them: they leave together, and what lies outside is dropped afterwards.
+    const T *raw = (const T *)a.raw + (size_t)c.row0 * a.ld;
+    constexpr int LN = 4;  // pairs of the low-rank input per thread that travel ahead (ranks up to 128): sixteen lanes per token
+    const int tr = threadIdx.x >> 4, lr = 2 * (threadIdx.x & 15);
+    Pair low[LN], lowb[LN];
 #pragma unroll
-        for (int j = 0; j < 4 * NB; ++j) ss = (int)(threadIdx.x & 15) + 16 * j < D ? fmaf(kv[j], kv[j], ss) : ss;
-        ss = lanes16_sum(ss);
-        if ((threadIdx.x & 15) == 0) s_unit[threadIdx.x >> 4] = 1.0f / sqrtf(ss + a.unit_eps);
+    for (int j = 0; j < LN; ++j) {
+        const int at = 5 * HD8 + min(lr + 32 * j, a.R8 - 2);
+        low[j] = pair_at(raw + (size_t)min(tr, c.n - 1) * a.ld + at), lowb[j] = bias_at(at);
     }
-    // the decay's weights (the first WS steps) and the channel vectors, on their way during the barrier and the decay's product
+    Pair xr[NP][TP], xk[NP][TP], xa[NP][TP], bx[NP][3];
+#pragma unroll
+    for (int p = 0; p < NP; ++p) {
+        const int d = min(2 * (lane + 64 * p), a.D8 - 2) + head * a.D8;  // (heads are padded to a multiple of 8)
+#pragma unroll
+        for (int j = 0; j < TP; ++j) {
+            const T *x = raw + (size_t)min(TP * wave + j, c.n - 1) * a.ld;
+            xr[p][j] = pair_at(x + d), xk[p][j] = pair_at(x + HD8 + d), xa[p][j] = pair_at(x + 4 * HD8 + d);
+        }
+        bx[p][0] = bias_at(d), bx[p][1] = bias_at(HD8 + d), bx[p][2] = bias_at(4 * HD8 + d);
+    }
+    // the decay's weights (the first WS steps)
     constexpr int WS = 4;
     uint4 wd[F32 ? 1 : NB][WS];
     float db[NB];
@@ -214,14 +225,23 @@ __global__ void __launch_bounds__(256) k_delta_prep(const DeltaArgs a) {
             for (int s = 0; s < WS; ++s) wd[j][s] = decay_weights(j, s);
             db[j] = a.decay_bias[head * D + min(16 * (wave * NB + j) + n16, D - 1)];
         }
-    const int pd = threadIdx.x % CH, part = threadIdx.x / CH;
-    float xr[TP], xk[TP], xa[TP];
+    auto put_low = [&](int j, const Pair &v, const Pair &b) {
+        auto f = [&](int i, float z) { return tr < c.n && i < a.rank ? F32 ? tanhf(z) : fast_tanh(z) : 0.0f; };
+        const float x = f(j, v.x + b.x), y = f(j + 1, v.y + b.y);
+        if constexpr (F32) s_low[tr * LR + j] = x, s_low[tr * LR + j + 1] = y;
+        else {
+            const u32 hi = pack2<BF16>(x, y);
+            *(u32 *)(s_hi + tr * LR + j) = hi, *(u32 *)(s_lo + tr * LR + j) = pack2<BF16>(x - lo_f32<BF16>(hi), y - hi_f32<BF16>(hi));
+        }
+    };
 #pragma unroll
-    for (int j = 0; j < TP; ++j) {
-        const int t = min(part * TP + j, c.n - 1), d = min(pd, D - 1);
-        xr[j] = channel(0, t, d), xk[j] = channel(1, t, d), xa[j] = channel(4, t, d);
+    for (int j = 0; j < LN; ++j)
+        if (32 * j < R32) put_low(lr + 32 * j, low[j], lowb[j]);
+    for (int j = lr + 32 * LN; j < R32; j += 32) {
+        const int at = 5 * HD8 + min(j, a.R8 - 2);
+        put_low(j, pair_at(raw + (size_t)min(tr, c.n - 1) * a.ld + at), bias_at(at));
     }
-    __syncthreads();
+    lds_barrier();
     auto log_decay = [&](int t, int d, float z) { s_l[t * LD + d] = t < c.n && d < D ? -a.decay_scale * dr_sigmoid<F32>(z) : 0.0f; };
     if constexpr (F32) {
         for (int i = threadIdx.x; i < DC * 16 * nblk; i += 256) {
@@ -250,27 +270,48 @@ __global__ void __launch_bounds__(256) k_delta_prep(const DeltaArgs a) {
             for (int i = 0; i < 4; ++i) log_decay(4 * q + i, d, z[i] + db[j]);
         }
     }
-    __syncthreads();  // the low-rank input has been read
+    lds_barrier();  // the low-rank input has been read
     {
-        const int d = pd;
-        if (part < PARTS && d < 16 * nblk) {
-            float L = 0.0f;
-            for (int t = 0; t < part * TP; ++t) L += s_l[t * LD + d];
-            float before = dr_exp<F32>(L);
+        float unit[TP];
+#pragma unroll
+        for (int j = 0; j < TP; ++j) {
+            float ss = 0.0f;
+#pragma unroll
+            for (int p = 0; p < NP; ++p) {
+                const int d = 2 * (lane + 64 * p);
+                xk[p][j].x = d < D && TP * wave + j < c.n ? xk[p][j].x + bx[p][1].x : 0.0f, xk[p][j].y = d + 1 < D && TP * wave + j < c.n ? xk[p][j].y + bx[p][1].y : 0.0f;
+                ss = fmaf(xk[p][j].x, xk[p][j].x, fmaf(xk[p][j].y, xk[p][j].y, ss));
+            }
+            unit[j] = 1.0f / sqrtf(wave_sum(ss) + a.unit_eps);
+        }
+#pragma unroll
+        for (int p = 0; p < NP; ++p) {
+            const int d = 2 * (lane + 64 * p);
+            if (d >= 16 * nblk) break;
+            float2 L = make_float2(0.0f, 0.0f);
+            for (int t = 0; t < TP * wave; ++t) {
+                const float2 l = *(const float2 *)(s_l + t * LD + d);
+                L.x += l.x, L.y += l.y;
+            }
+            float2 before = make_float2(dr_exp<F32>(L.x), dr_exp<F32>(L.y));
 #pragma unroll
             for (int j = 0; j < TP; ++j) {
-                const int t = part * TP + j;
-                const bool live = t < c.n && d < D;
-                L += s_l[t * LD + d];
-                const float e = dr_exp<F32>(L), back = dr_exp<F32>(-L);
-                const float r = live ? xr[j] : 0.0f, k = live ? xk[j] : 0.0f, u = k * s_unit[t];
-                s_u[t * LD + d] = u * before, s_r[t * LD + d] = r * e, s_k[t * LD + d] = k * back, s_a[t * LD + d] = dr_sigmoid<F32>(xa[j]) * u * back;
+                const int t = TP * wave + j, at = t * LD + d;
+                const bool lx = t < c.n && d < D, ly = t < c.n && d + 1 < D;
+                const float2 l = *(const float2 *)(s_l + at);
+                L.x += l.x, L.y += l.y;
+                const float2 e = make_float2(dr_exp<F32>(L.x), dr_exp<F32>(L.y)), back = make_float2(dr_exp<F32>(-L.x), dr_exp<F32>(-L.y));
+                const float2 k = make_float2(xk[p][j].x, xk[p][j].y), u = make_float2(k.x * unit[j], k.y * unit[j]);
+                *(float2 *)(s_u + at) = make_float2(u.x * before.x, u.y * before.y);
+                *(float2 *)(s_r + at) = make_float2(lx ? (xr[p][j].x + bx[p][0].x) * e.x : 0.0f, ly ? (xr[p][j].y + bx[p][0].y) * e.y : 0.0f);
+                *(float2 *)(s_k + at) = make_float2(k.x * back.x, k.y * back.y);
+                *(float2 *)(s_a + at) = make_float2(dr_sigmoid<F32>(xa[p][j].x + bx[p][2].x) * u.x * back.x, dr_sigmoid<F32>(xa[p][j].y + bx[p][2].y) * u.y * back.y);
                 before = e;
             }
-            if (part == PARTS - 1) s_wc[d] = before;
+            if (wave == 3) *(float2 *)(s_wc + d) = before;
         }
     }
-    __syncthreads();
+    lds_barrier();
     {  // wave 0: A = U K^T, 1: B = U A^T, 2: A' = R K^T, 3: B' = R A^T
         const float *l = wave < 2 ? s_u : s_r, *r = wave & 1 ? s_a : s_k;
         dr_f32x4 acc = {0.0f, 0.0f, 0.0f, 0.0f};
@@ -286,8 +327,8 @@ __global__ void __launch_bounds__(256) k_delta_prep(const DeltaArgs a) {
 #pragma unroll
             for (int i = 0; i < 4; ++i) s_m[(wave * DC + 4 * q + i) * LM + n16] = acc[i];
     }
-    __syncthreads();
-    float *out = a.ws + ((size_t)blockIdx.x * a.H + head) * dr_chunk_floats(D);
+    lds_barrier();
+    float *out = a.ws + ((size_t)blockIdx.y * a.H + head) * dr_chunk_floats(D);
     float *o_r = out + nblk * 256, *o_k = o_r + nblk * 256, *o_a = o_k + nblk * 256, *o_m = o_a + nblk * 256;
     float *s_t = s_m + 4 * DC * LM;
     if (wave == 0) {
@@ -325,7 +366,7 @@ __global__ void __launch_bounds__(256) k_delta_prep(const DeltaArgs a) {
         if (wave == 1)
             for (int d = lane; d < 16 * nblk; d += 64) o_m[768 + d] = s_wc[d];
     }
-    __syncthreads();
+    lds_barrier();
     const dr_f32x4 tv = *(const dr_f32x4 *)(s_t + n16 * LM + 4 * q);
 #pragma unroll
     for (int j = 0; j < NB; ++j) {
@@ -541,7 +582,7 @@ int delta_chunks_nb(const DeltaArgs &a, int chunks, int row0, int rows, hipStrea
     const int step = delta_segment(a.H, a.D);
     for (int c = 0; c < chunks; c += step) {  // a segment's operands are read back before they leave the last-level cache
         seg.chunk_lo = c, seg.chunk_hi = std::min(chunks, c + step);
-        hipLaunchKernelGGL((k_delta_prep<E, NB>), dim3((unsigned)(seg.chunk_hi - c), (unsigned)a.H), dim3(256), lds, st, seg);
+        hipLaunchKernelGGL((k_delta_prep<E, NB>), dim3((unsigned)a.H, (unsigned)(seg.chunk_hi - c)), dim3(256), lds, st, seg);
         PIE_LAUNCH_CHECK();
         hipLaunchKernelGGL((k_delta_scan<E, NB>), dim3((unsigned)(a.H * dr_blocks(a.D)), (unsigned)a.n_runs), dim3(256), 0, st, seg);
         PIE_LAUNCH_CHECK();
