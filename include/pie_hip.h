@@ -596,7 +596,8 @@ enum { PIE_ACT_SILU = 0, PIE_ACT_CLIPPED = 1 };
  * Experts: w_gate_up experts x packed [2 * size, width] with rows (2 i, 2 i + 1) = (gate_i, up_i); w_down experts x packed [width, size].  act SILU:
  * silu(g) u; CLIPPED: g = min(gate, act_limit), u = clamp(up, +-act_limit), g sigmoid(act_alpha g) (u + 1).
  * TABLE_MOE: table int32 [vocab][top], every chosen expert weighs 1 / top.  ROUTED_MOE: w_router packed [experts, width], the `top` experts with the largest
- * sigmoid(w_router h) + correction (fp32 [experts]), each weighing its sigmoid.
+ * sigmoid(w_router h) + correction (fp32 [experts]), each weighing its sigmoid; w_router_rows (may be NULL): the same weights as bf16 [experts][width rounded
+ * up to 8], zeros past width -- passes of few rows choose beside the norm then.
  * Shared expert likewise when shared_size > 0, times sigmoid(shared_gate . input), shared_gate fp32 [width, rounded up to 8 with zeros]
  * (element-wise norms only). */
 typedef struct {
@@ -614,7 +615,7 @@ typedef struct {
     int experts, top, shared_size, act;
     float act_alpha, act_limit;
     const int32_t *table;
-    const void *w_router;
+    const void *w_router, *w_router_rows;
     const float *correction;
     const void *w_gate_up, *w_expert_down, *s_gate_up, *s_down;
     const float *shared_gate;

@@ -94,7 +94,7 @@ class pie_stack_config(C.Structure):
 class pie_stack_layer(C.Structure):
     _fields_ = _fields("n:pre1 post1 pre2 post2 i:mixer heads dim vdim rank window f:scale eps p:w_in w_uk w_uv w_o w_kv c_norm "
                        "i:kv_heads kv_from rot_dims value_norm out_gate f:rot_gain sink decay_scale unit_eps p:rot_freq q_norm k_norm decay_bias o_norm "
-                       "in_bias o_bias w_decay i:ff ff_size p:w_up w_down i:experts top shared_size act f:act_alpha act_limit p:table w_router correction "
+                       "in_bias o_bias w_decay i:ff ff_size p:w_up w_down i:experts top shared_size act f:act_alpha act_limit p:table w_router w_router_rows correction "
                        "w_gate_up w_expert_down s_gate_up s_down shared_gate", _CT)
 
 

@@ -19,6 +19,7 @@
 #include <vector>
 
 #include "mfma_store.hpp"  // MFMA_ACT_*
+#include "route.hpp"
 #include "stack_types.hpp"
 
 size_t w16l_workspace_bytes(int M, int N, int K);
@@ -32,18 +33,10 @@ namespace {
 
 constexpr int BIG_ROWS = 64;  // more rows than this take the tiled GEMMs
 constexpr int LONG_RUN = 64;  // runs of at least this many rows take the attentions' long forms
+constexpr int ROUTE_FEW_ROWS = 64;              // up to this many rows, and router weights that one workgroup reads in a few us: chosen beside the norm
+constexpr long ROUTE_FEW_WEIGHTS = 256l << 10;
 constexpr int DELTA_RUN = 8;  // runs of at least this many rows take the recurrence's chunk form
 
-struct RouteLayer {      // one mixture layer's row lists (device pointers)
-    const int *table;    // experts by token id; nullptr: by the router's logits
-    const float *logits, *correction;  // [M][ld_logits], [experts]
-    int ld_logits;
-    int *chosen;         // [M * top]: the router's choice, best first, and the weights
-    float *weight;
-    int top, experts, max_active;
-    int *active, *offset, *list, *place;  // [max_active], [experts + 1], [M * top] rows by expert, [M * top] position of (row, slot)
-    int4 *tiles;  // {expert, first position, rows, 0}: row tiles of the grouped GEMM
-};
 // rows per tile of the grouped GEMM, and a bound on the number of tiles
 __host__ __device__ inline int route_tile_rows(long M, int top, int experts) { return M * top >= 96l * experts ? 128 : 64; }
 // (an expert's tiles start at a multiple of route_block(): the grouped GEMM runs that many side by side on one XCD, over the same weights)
@@ -54,102 +47,25 @@ __host__ __device__ inline int route_max_tiles(long M, int top, int experts) {
     return ((int)(M * top / route_tile_rows(M, top, experts)) + route_block(M, top, experts) * experts + 3) / 4 * 4;
 }
 
-// One wave: the `top` experts of row m with the largest sigmoid(logit) + correction (equal ones: the first), each with the weight sigmoid(logit).
-// Round k takes the best of what comes behind round k - 1's in that order, so nothing has to be marked as taken.
-__device__ __forceinline__ void route_pick(const RouteLayer &L, int m, int lane) {
-    const float *z = L.logits + (size_t)m * L.ld_logits;
-    constexpr int R = 4;  // scores a lane keeps; more experts than 64 R are scored again in every round
-    float keep[R];
-    auto score = [&](int e) { return 1.0f / (1.0f + expf(-z[e])) + L.correction[e]; };
-#pragma unroll
-    for (int r = 0; r < R; ++r) keep[r] = 64 * r + lane < L.experts ? score(64 * r + lane) : -INFINITY;
-    float last = INFINITY;
-    int last_e = -1;
-    for (int k = 0; k < L.top; ++k) {
-        float best = -INFINITY;
-        int at = 0x7fffffff;
-        auto look = [&](float s, int e) {
-            if ((s < last || (s == last && e > last_e)) && s > best) best = s, at = e;
-        };
-#pragma unroll
-        for (int r = 0; r < R; ++r)
-            if (64 * r + lane < L.experts) look(keep[r], 64 * r + lane);
-        for (int e = 64 * R + lane; e < L.experts; e += 64) look(score(e), e);
-        const float top = wave_max(best);
-        int e = best == top ? at : 0x7fffffff;
-#pragma unroll
-        for (int o = 32; o > 0; o >>= 1) e = min(e, __shfl_xor(e, o, 64));
-        e = e < L.experts ? e : k;  // (scores that compare with nothing)
-        last = top, last_e = e;
-        if (lane == 0) {
-            L.chosen[(size_t)m * L.top + k] = e;
-            L.weight[(size_t)m * L.top + k] = 1.0f / (1.0f + expf(-z[e]));
-        }
-    }
-}
 __global__ void __launch_bounds__(256) k_route_pick(const RouteLayer *layers, int M) {
     const int m = blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (m < M) route_pick(layers[0], m, threadIdx.x & 63);
+    const RouteLayer L = layers[0];
+    if (m < M)
+        route_pick(L, L.logits + (size_t)m * L.ld_logits, threadIdx.x & 63, [&](int k, int e, float w) { L.chosen[(size_t)m * L.top + k] = e, L.weight[(size_t)m * L.top + k] = w; });
 }
 
-// the row lists of layers[blockIdx.x]; pick: its router's choice is made here too (few rows)
-__global__ void __launch_bounds__(1024) k_route(const RouteLayer *layers, const int *ids, int M, int vocab, bool pick) {
+// the row lists of layers[blockIdx.x]
+__global__ void __launch_bounds__(1024) k_route(const RouteLayer *layers, const int *ids, int M, int vocab) {
     extern __shared__ int s_cnt[];  // [experts] counts, then [experts] cursors
     const RouteLayer L = layers[blockIdx.x];
-    int *s_cur = s_cnt + L.experts;
-    const int n = M * L.top;
-    if (pick) {
-        for (int m = threadIdx.x >> 6; m < M; m += 16) route_pick(L, m, threadIdx.x & 63);
-        __syncthreads();
-    }
-    auto expert = [&](int i) {
-        if (!L.table) return min(max(L.chosen[i], 0), L.experts - 1);
-        const int t = min(max(ids[i / L.top], 0), vocab - 1);
-        return min(max(L.table[(size_t)t * L.top + i % L.top], 0), L.experts - 1);
-    };
-    for (int e = threadIdx.x; e < L.experts; e += blockDim.x) s_cnt[e] = 0;
-    __syncthreads();
-    for (int i = threadIdx.x; i < n; i += blockDim.x) atomicAdd(&s_cnt[expert(i)], 1);
-    __syncthreads();
-    if (threadIdx.x < 64) {
-        int base = 0, n_active = 0, n_tiles = 0;
-        const int tr = route_tile_rows(M, L.top, L.experts), rb = route_block(M, L.top, L.experts);
-        for (int e0 = 0; e0 < L.experts; e0 += 64) {
-            const int e = e0 + (int)threadIdx.x, c = e < L.experts ? s_cnt[e] : 0;
-            int incl = c;
-#pragma unroll
-            for (int o = 1; o < 64; o <<= 1) {
-                const int v = __shfl_up(incl, o, 64);
-                if ((int)threadIdx.x >= o) incl += v;
-            }
-            if (e < L.experts) s_cur[e] = L.offset[e] = base + incl - c;
-            const unsigned long long has = __ballot(c > 0);
-            const int slot = n_active + __popcll(has & ((1ull << threadIdx.x) - 1ull));
-            if (c > 0 && slot < L.max_active) L.active[slot] = e;
-            if (L.tiles) {
-                const int mine = (c + tr - 1) / tr, slots = (mine + rb - 1) / rb * rb;
-                int ti = slots;
-#pragma unroll
-                for (int o = 1; o < 64; o <<= 1) {
-                    const int v = __shfl_up(ti, o, 64);
-                    if ((int)threadIdx.x >= o) ti += v;
-                }
-                for (int k = 0; k < slots; ++k) L.tiles[n_tiles + ti - slots + k] = make_int4(e, base + incl - c + k * tr, max(0, min(tr, c - k * tr)), 0);
-                n_tiles += __shfl(ti, 63, 64);
-            }
-            base += __shfl(incl, 63, 64), n_active += __popcll(has);
-        }
-        if (L.tiles)
-            for (int i = n_tiles + (int)threadIdx.x; i < route_max_tiles(M, L.top, L.experts); i += 64) L.tiles[i] = make_int4(0, 0, 0, 0);
-        if (threadIdx.x == 0) L.offset[L.experts] = base;
-        for (int i = n_active + (int)threadIdx.x; i < L.max_active; i += 64) L.active[i] = -1;
-    }
-    __syncthreads();
-    for (int i = threadIdx.x; i < n; i += blockDim.x) {
-        const int p = atomicAdd(&s_cur[expert(i)], 1);
-        L.list[p] = i / L.top;
-        L.place[i] = p;
-    }
+    const int tr = route_tile_rows(M, L.top, L.experts), rb = route_block(M, L.top, L.experts);
+    route_lists(
+        L, M, s_cnt,
+        [&](int i) {
+            if (!L.table) return L.chosen[i];
+            return L.table[(size_t)min(max(ids[i / L.top], 0), vocab - 1) * L.top + i % L.top];
+        },
+        tr, rb, route_max_tiles(M, L.top, L.experts));
 }
 
 template <class E>
@@ -380,6 +296,7 @@ struct pie_stack {
     Buf<RowStat> stats;
     Buf<int> route_ints;
     Buf<RouteLayer> route_dev;
+    Buf<int> arrived;               // rows that have chosen their experts (zero between launches)
     std::vector<RouteLayer> route;  // per layer; experts == 0: not a mixture
     int route_rows = 0, n_table = 0, route_lds = 0;  // n_table: mixtures whose experts a table names (in front in route_dev)
     std::vector<int> route_at;      // layer -> entry of route_dev
@@ -496,7 +413,7 @@ int stack_reserve(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
         auto lists = [&](const RouteLayer &r) { return (2 * (size_t)r.experts + 1 + 2 * R * r.top + (r.table ? 0 : 2 * R * r.top) + 3) / 4 * 4; };
         for (const RouteLayer &r : s->route)
             if (r.experts) ints += lists(r) + 4 * tiles(r);
-        if ((rc = s->route_ints.need(ints, &moved)) || (rc = s->route_dev.need(n_moe, &moved))) return rc;
+        if ((rc = s->route_ints.need(ints, &moved)) || (rc = s->route_dev.need(n_moe, &moved)) || (rc = s->arrived.need(1, &moved))) return rc;
         int *p = s->route_ints.p, at[2] = {0, s->n_table};
         std::vector<RouteLayer> dev(n_moe);
         s->route_lds = 0, s->route_at.assign(s->layers.size(), 0);
@@ -564,7 +481,8 @@ struct Pass {
             rc = w16l_gemm_launch(PIE_BF16, w, x, ldx, M, N, K, swiglu ? nullptr : y, s->gemm_ws.p, st, nullptr, swiglu ? y : nullptr, nullptr, ldy), ++launches;
     }
     // x += post(y); h = next(x) over y = s->y (bf16; many rows) or s->y32
-    void update(const pie_stack_norm &post, const pie_stack_norm &next, const u16 *bias = nullptr) {
+    // route (few rows): the layer whose experts the rows choose on their way
+    void update(const pie_stack_norm &post, const pie_stack_norm &next, const u16 *bias = nullptr, int route = -1) {
         if (rc) return;
         const int W = s->cfg.width, W64 = up64(W), WA = act_stride(W);
         if (plan.big && pointwise(post) && pointwise(next) && !bias) {
@@ -575,12 +493,14 @@ struct Pass {
             RowUpdateArgs a = {};
             a.y = plan.big ? (const void *)s->y.p : s->y32.p, a.y32 = !plan.big, a.ldy = plan.big ? W : W64, a.bias = bias;
             a.post = row_norm_of(post), a.next = row_norm_of(next), a.x = s->x.p, a.ldx = W64, a.h = s->h.p, a.ldh = WA, a.M = b.n_rows, a.W = W;
+            if (route >= 0) a.route = s->route_dev.p + s->route_at[route], a.experts = s->layers[route].experts, a.router = (const u16 *)s->layers[route].w_router_rows, a.arrived = s->arrived.p;
             rc = row_update_launch(s->cfg.dtype, a, st);
         }
         ++launches;
     }
     // a sublayer's last product [W, K], its norm, the residual sum and the next sublayer's norm
-    void output(const void *w, const void *x, int ldx, int K, const pie_stack_norm &post, const pie_stack_norm &next, const u16 *bias = nullptr) {
+    void output(const void *w, const void *x, int ldx, int K, const pie_stack_norm &post, const pie_stack_norm &next, const u16 *bias = nullptr,
+                int route = -1) {
         const int W = s->cfg.width, W64 = up64(W), WA = act_stride(W), M = b.n_rows;
         if (plan.big) {
             gemm(w, x, ldx, M, W, K, s->y.p, W);
@@ -589,20 +509,20 @@ struct Pass {
         RowsArgs o = {};
         o.m = {(const char *)w, W, K, x, ldx, s->y32.p, W64};
         o.M = M;
-        if (pointwise(post) && pointwise(next) && !bias) {
+        if (pointwise(post) && pointwise(next) && !bias && route < 0) {
             o.epi = ROWS_RESIDUAL, o.res = s->x.p, o.ld_res = W64, o.post = norm_of(post), o.next = norm_of(next), o.h = s->h.p, o.ldh = WA;
             return linear(o);
         }
         o.epi = ROWS_SCALE_F32, o.scale = 1.0f;
         linear(o);
-        update(post, next, bias);
+        update(post, next, bias, route);
     }
     void linear(const RowsArgs &a, int batches = 1) {
         if (!rc) rc = rows_gemm_launch(s->cfg.dtype, a, batches, st), ++launches;
     }
 };
 
-void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm &next) {
+void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm &next, int route) {
     pie_stack *s = p.s;
     const pie_stack_batch &b = p.b;
     const int W = s->cfg.width, W64 = up64(W), WA = act_stride(W), D8 = up8(L.dim), V8 = up8(L.vdim), R8 = up8(L.rank), H = L.heads, NI = H * D8 + R8, KO = H * V8, LO = act_stride(KO);
@@ -658,7 +578,7 @@ void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_nor
         for (int i = p.plan.short_runs; i < b.n_runs; ++i) tiles += (b.runs_host[4 * i + 1] + 127) / 128;
         if (!p.rc) p.rc = window_attn_launch(w, tiles, p.st), p.launches += 2;
     }
-    p.output(L.w_o, s->o.p, LO, KO, L.post1, next);
+    p.output(L.w_o, s->o.p, LO, KO, L.post1, next, nullptr, route);
 }
 
 // y = h . W^T in the stack's dtype
@@ -672,7 +592,7 @@ void project(Pass &p, const void *w, int N, void *y) {
     p.linear(a);
 }
 
-void attention_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm &next) {
+void attention_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm &next, int route) {
     pie_stack *s = p.s;
     const pie_stack_batch &b = p.b;
     const int NI = in_columns(L), KO = out_columns(L), LO = act_stride(KO), dt = s->cfg.dtype;
@@ -702,10 +622,10 @@ void attention_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_
         for (int i = sp.runs; i < b.n_runs; ++i) a.n_tiles += page_attn_long_tiles(b.runs_host[4 * i + 1], geo);
         p.rc = page_attn_long_launch(a, p.st), ++p.launches;
     }
-    p.output(L.w_o, s->o.p, LO, KO, L.post1, next, (const u16 *)L.o_bias);
+    p.output(L.w_o, s->o.p, LO, KO, L.post1, next, (const u16 *)L.o_bias, route);
 }
 
-void delta_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm &next) {
+void delta_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm &next, int route) {
     pie_stack *s = p.s;
     const pie_stack_batch &b = p.b;
     const int NI = in_columns(L), KO = out_columns(L), LO = act_stride(KO);
@@ -723,10 +643,10 @@ void delta_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm
         d.runs += dp.runs, d.n_runs = b.n_runs - dp.runs;
         p.rc = delta_chunks_launch(s->cfg.dtype, d, dp.chunks, dp.rows, b.n_rows - dp.rows, p.st), p.launches += delta_launches(dp.chunks, L.heads, L.dim);
     }
-    p.output(L.w_o, s->o.p, LO, KO, L.post1, next);
+    p.output(L.w_o, s->o.p, LO, KO, L.post1, next, nullptr, route);
 }
 
-void feed_forward(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm &next) {
+void feed_forward(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm &next, bool routed) {  // routed: the experts have been chosen already
     pie_stack *s = p.s;
     const int M = p.b.n_rows, W = s->cfg.width, W64 = up64(W), WA = act_stride(W), F = L.ff_size, FA = act_stride(F), dt = s->cfg.dtype;
     if (L.ff == PIE_FF_RELU2) {
@@ -744,21 +664,17 @@ void feed_forward(Pass &p, int li, const pie_stack_layer &L, const pie_stack_nor
     const int S = L.shared_size, SA = act_stride(S);
     const size_t gu_stride = rows_weight_bytes(dt, 2 * F, W), dn_stride = rows_weight_bytes(dt, W, F);
     const bool clipped = L.act == PIE_ACT_CLIPPED;
-    if (L.ff == PIE_FF_ROUTED_MOE) {  // logits, then the choice and its row lists
+    if (L.ff == PIE_FF_ROUTED_MOE && !routed) {  // logits, then the choice and its row lists
         RowsArgs z = {};
         z.m = {(const char *)L.w_router, L.experts, W, s->h.p, WA, s->logits_e.p, up8(L.experts)};
         z.M = M, z.epi = ROWS_SCALE_F32, z.scale = 1.0f;
         p.linear(z);
         if (p.rc) return;
         const RouteLayer *dev = s->route_dev.p + s->route_at[li];
-        const bool few = M <= 64;
-        if (!few) {
-            hipLaunchKernelGGL(k_route_pick, dim3((unsigned)((M + 3) / 4)), dim3(256), 0, p.st, dev, M);
-            ++p.launches;
-        }
-        hipLaunchKernelGGL(k_route, dim3(1), dim3(1024), (size_t)2 * L.experts * 4, p.st, dev, p.b.ids, M, s->cfg.vocab, few);
+        hipLaunchKernelGGL(k_route_pick, dim3((unsigned)((M + 3) / 4)), dim3(256), 0, p.st, dev, M);
+        hipLaunchKernelGGL(k_route, dim3(1), dim3(1024), (size_t)2 * L.experts * 4, p.st, dev, p.b.ids, M, s->cfg.vocab);
         if (hipGetLastError() != hipSuccess) p.rc = pie::fail(PIE_E_HIP, "routing launch failed");
-        ++p.launches;
+        p.launches += 2;
     }
     CombineArgs c = {};
     c.part = s->part.p, c.part_s = s->part_s.p, c.ldp = W64, c.ldp_s = p.plan.big && !(W & 3) ? W : W64, c.place = r.place, c.weight = r.weight, c.top = L.top, c.W = W, c.gate = S ? L.shared_gate : nullptr;
@@ -807,7 +723,7 @@ int stack_enqueue(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
     const int M = b.n_rows, W = s->cfg.width, W64 = up64(W), WA = act_stride(W), V = s->cfg.vocab, n = s->cfg.n_layers, dt = s->cfg.dtype;
     Pass p{s, b, plan, st};
     if (s->n_table) {
-        hipLaunchKernelGGL(k_route, dim3((unsigned)s->n_table), dim3(1024), (size_t)s->route_lds, st, s->route_dev.p, b.ids, M, V, false);
+        hipLaunchKernelGGL(k_route, dim3((unsigned)s->n_table), dim3(1024), (size_t)s->route_lds, st, s->route_dev.p, b.ids, M, V);
         PIE_LAUNCH_CHECK();
         ++p.launches;
     }
@@ -829,10 +745,12 @@ int stack_enqueue(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
     for (int i = 0; i < n && !p.rc; ++i) {
         const pie_stack_layer &L = s->layers[i];
         const pie_stack_norm &after = i + 1 < n ? s->layers[i + 1].pre1 : fin, &next = L.ff == PIE_FF_NONE ? after : L.pre2;
-        if (L.mixer == PIE_MIXER_LATENT) latent_mixer(p, i, L, next);
-        else if (L.mixer == PIE_MIXER_ATTENTION) attention_mixer(p, i, L, next);
-        else delta_mixer(p, i, L, next);
-        if (L.ff != PIE_FF_NONE && !p.rc) feed_forward(p, i, L, after);
+        // few rows: the launch that makes the router's input also chooses the experts
+        const bool routed = L.ff == PIE_FF_ROUTED_MOE && !plan.big && L.w_router_rows && M <= ROUTE_FEW_ROWS && (long)L.experts * W <= ROUTE_FEW_WEIGHTS && W <= 8192;
+        if (L.mixer == PIE_MIXER_LATENT) latent_mixer(p, i, L, next, routed ? i : -1);
+        else if (L.mixer == PIE_MIXER_ATTENTION) attention_mixer(p, i, L, next, routed ? i : -1);
+        else delta_mixer(p, i, L, next, routed ? i : -1);
+        if (L.ff != PIE_FF_NONE && !p.rc) feed_forward(p, i, L, after, routed);
         if (b.tap && !p.rc)
             PIE_HIP_TRY(hipMemcpy2DAsync(b.tap + (size_t)i * M * W, (size_t)W * 4, s->x.p, (size_t)W64 * 4, (size_t)W * 4, (size_t)M, hipMemcpyDeviceToDevice, st));
     }

@@ -2,6 +2,10 @@
 //
 // One workgroup per row.  y is a sublayer's output (plus a bias), or the weighted sum of a row's experts; the row stays in registers from the first read to
 // the last store, so the norms' sums cost one exchange through LDS each and x, y and h pass through memory once.
+//
+// Few rows in front of a mixture: the workgroup goes on with its row's router logits (the row is in LDS, a wave per expert), chooses the experts, and the
+// last workgroup to arrive makes the row lists -- the router, the choice and the lists are no launches of their own.
+#include "route.hpp"
 #include "stack_types.hpp"
 
 namespace {
@@ -63,7 +67,51 @@ __device__ __forceinline__ void norm_row(const StackNorm &m, int W, float (&y)[N
     }
 }
 
-template <class E, int THREADS, int NQ>
+// xv: next(x) of row blockIdx.x, quads as in k_row_update
+template <int THREADS, int NQ>
+__device__ __forceinline__ void row_route(const RowUpdateArgs &a, const float (&xv)[NQ][4]) {
+    extern __shared__ __attribute__((aligned(16))) float s_dyn[];  // [W rounded up to 8] the row, [experts] logits, [2 * experts] list counters
+    const int W8 = (a.W + 7) & ~7, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, m = blockIdx.x;
+    float *s_z = s_dyn + W8;
+    int *s_cnt = (int *)(s_z + a.experts);
+    __shared__ int s_last;
+    const RouteLayer L = *a.route;
+#pragma unroll
+    for (int q = 0; q < NQ; ++q) {
+        const int n = threadIdx.x * 4 + 4 * THREADS * q;
+        if (n < W8) *(float4 *)(s_dyn + n) = make_float4(xv[q][0], xv[q][1], xv[q][2], xv[q][3]);  // (zeros past W)
+    }
+    __syncthreads();
+    for (int e = wave; e < a.experts; e += THREADS / 64) {
+        const u16 *w = a.router + (size_t)e * W8;
+        float z = 0.0f;
+#pragma unroll 4
+        for (int k = lane * 8; k < W8; k += 512) {
+            const uint4 v = *(const uint4 *)(w + k);
+            const float4 h0 = *(const float4 *)(s_dyn + k), h1 = *(const float4 *)(s_dyn + k + 4);
+            z = fmaf(lo_f32<BF16>(v.x), h0.x, fmaf(hi_f32<BF16>(v.x), h0.y, fmaf(lo_f32<BF16>(v.y), h0.z, fmaf(hi_f32<BF16>(v.y), h0.w, z))));
+            z = fmaf(lo_f32<BF16>(v.z), h1.x, fmaf(hi_f32<BF16>(v.z), h1.y, fmaf(lo_f32<BF16>(v.w), h1.z, fmaf(hi_f32<BF16>(v.w), h1.w, z))));
+        }
+        z = wave_sum(z);
+        if (lane == 0) s_z[e] = z;
+    }
+    __syncthreads();
+    if (wave == 0) {
+        route_pick(L, s_z, lane, [&](int k, int e, float w) {
+            const size_t i = (size_t)m * L.top + k;
+            __hip_atomic_store(L.chosen + i, e, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);  // (seen by whichever workgroup arrives last, on any XCD)
+            L.weight[i] = w;
+        });
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        if (lane == 0) s_last = __hip_atomic_fetch_add(a.arrived, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) == (int)gridDim.x - 1;
+    }
+    __syncthreads();
+    if (!s_last) return;
+    if (threadIdx.x == 0) __hip_atomic_store(a.arrived, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    route_lists(L, a.M, s_cnt, [&](int i) { return __hip_atomic_load(L.chosen + i, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); }, 0, 0, 0);
+}
+
+template <class E, int THREADS, int NQ, bool ROUTE = false>
 __global__ void __launch_bounds__(THREADS) k_row_update(const RowUpdateArgs a) {
     typedef typename E::type T;
     __shared__ float red[2][THREADS / 64];
@@ -149,11 +197,21 @@ __global__ void __launch_bounds__(THREADS) k_row_update(const RowUpdateArgs a) {
         } else
             for (int i = 0; i < a.W - n; ++i) h[n + i] = E::pack(xv[q][i]);
     }
+    if constexpr (ROUTE) row_route<THREADS, NQ>(a, xv);
 }
 
 template <class E>
 void row_go(const RowUpdateArgs &a, hipStream_t st) {
     const dim3 grid((unsigned)a.M);
+    if (a.route) {  // (at least eight waves: they share the experts)
+        const size_t lds = ((size_t)((a.W + 7) & ~7) + 3 * a.experts) * 4;
+#define ROW_GO(T_, Q_) hipLaunchKernelGGL((k_row_update<E, T_, Q_, true>), grid, dim3(T_), lds, st, a)
+        if (a.W <= 2048) ROW_GO(512, 1);
+        else if (a.W <= 4096) ROW_GO(1024, 1);
+        else ROW_GO(1024, 4);
+#undef ROW_GO
+        return;
+    }
 #define ROW_GO(T_, Q_) hipLaunchKernelGGL((k_row_update<E, T_, Q_>), grid, dim3(T_), 0, st, a)
     if (a.W <= 256) ROW_GO(64, 1);
     else if (a.W <= 1024) ROW_GO(256, 1);
@@ -174,6 +232,7 @@ int row_update_launch(int dtype, const RowUpdateArgs &a, hipStream_t st) {
     if (a.M <= 0) return PIE_OK;
     PIE_REQUIRE(a.W > 0 && a.W <= ROW_UPDATE_MAX_WIDTH, PIE_E_SHAPE, "row update: widths up to 32768");
     PIE_REQUIRE(a.ldx % 4 == 0 && a.ldh % 4 == 0 && (!a.y32 || a.ldy % 4 == 0), PIE_E_ALIGN, "row update: row strides must be multiples of 4");
+    PIE_REQUIRE(!a.route || (a.router && a.arrived && a.experts > 0 && ((size_t)a.W + 8 + 3 * a.experts) * 4 <= 64 * 1024 - 1024 && a.W <= 16384), PIE_E_SHAPE, "row update: too wide to route beside");
     if (dtype == PIE_F32) row_go<ElemF32>(a, st);
     else row_go<ElemBF16>(a, st);
     PIE_LAUNCH_CHECK();

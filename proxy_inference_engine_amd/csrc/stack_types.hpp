@@ -335,5 +335,10 @@ struct RowUpdateArgs {
     int ldx;
     void *h;                // [M][ldh] T
     int ldh, M, W;
+    // nullable: the rows choose their experts on the way, by the router's logits of next(x) (fp32); lists as k_route makes them, without tiles
+    const struct RouteLayer *route;
+    int experts;
+    const u16 *router;      // bf16 [experts][W rounded up to 8], zeros past W
+    int *arrived;           // one int, zero before and after
 };
 int row_update_launch(int dtype, const RowUpdateArgs &a, hipStream_t st);

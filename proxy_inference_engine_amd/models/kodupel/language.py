@@ -150,7 +150,8 @@ class Model(LayerStackModel):
                 return (pack(interleave(pad(get(q + "gate", F, W), F8, W), pad(get(q + "up", F, W), F8, W))), pack(pad(get(q + "down", W, F), W, F8)))
             experts = [gated(f"{p}e{e}.") for e in range(E)]
             return {"ff": _ffi.PIE_FF_ROUTED_MOE, "ff_size": F8, "experts": E, "top": ff.router.top, "act": _ffi.PIE_ACT_CLIPPED, "act_alpha": EXPERT_SLOPE,
-                    "act_limit": ff.expert.limit, "w_router": pack(get(p + "router", E, W)), "correction": flat(p + "correction", E),
+                    "act_limit": ff.expert.limit, "w_router": pack(get(p + "router", E, W)), "w_router_rows": pad(get(p + "router", E, W).to(torch.bfloat16), E, up8(W)),
+                    "correction": flat(p + "correction", E),
                     "w_gate_up": torch.cat([e[0] for e in experts]), "w_expert_down": torch.cat([e[1] for e in experts])}
 
         if not args.layers:
