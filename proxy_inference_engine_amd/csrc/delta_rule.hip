@@ -28,8 +28,11 @@ constexpr int DC = 16;  // tokens of a chunk
 constexpr size_t DELTA_SEGMENT_BYTES = 96u << 20;
 
 
-template <class E, int CP, int NT>  // CP: power of two >= D; NT threads
-__global__ void __launch_bounds__(NT) k_delta_step(const DeltaArgs a) {
+__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }  // (loads and stores stay in flight)
+
+// CP: power of two >= D; NT threads; AHEAD: few workgroups, where latency counts and registers do not
+template <class E, int CP, int NT, bool AHEAD>
+__global__ void __launch_bounds__(NT, AHEAD ? 1 : 4) k_delta_step(const DeltaArgs a) {
     typedef typename E::type T;
     constexpr int SL = NT / CP, RPT = CP / SL;  // channel slices; channels per thread
     static_assert(NT % CP == 0 && CP % SL == 0 && NT % 64 == 0, "slices");
@@ -45,6 +48,19 @@ __global__ void __launch_bounds__(NT) k_delta_step(const DeltaArgs a) {
 #pragma unroll
     for (int i = 0; i < RPT; ++i) S[i] = !fresh && col < D && d0 + i < D ? state[(size_t)(d0 + i) * D + col] : 0.0f;
     const int HD8 = a.H * a.D8;
+    // AHEAD: what all tokens share leaves together with the state -- the decay's weights (eight lanes per channel, the first WS pieces) and the head's norm
+    constexpr int CPT = (CP + NT / 8 - 1) / (NT / 8), WS = 2;
+    uint4 wd[AHEAD ? CPT : 1][WS];
+    float db[AHEAD ? CPT : 1], o_norm = 0.0f;
+    auto decay_weights = [&](int d, int i) { return *(const uint4 *)(a.w_decay + (size_t)(head * D + min(d, D - 1)) * a.R8 + min(i, a.R8 - 8)); };
+    if constexpr (AHEAD) o_norm = a.o_norm[head * D + min((int)threadIdx.x, D - 1)];
+#pragma unroll
+    for (int c = 0; c < (AHEAD ? CPT : 0); ++c) {
+        const int d = (threadIdx.x >> 3) + c * (NT / 8);
+#pragma unroll
+        for (int s = 0; s < WS; ++s) wd[c][s] = decay_weights(d, (threadIdx.x & 7) * 8 + 64 * s);
+        db[c] = a.decay_bias[head * D + min(d, D - 1)];
+    }
 
     for (int j = 0; j < run.n_rows; ++j) {
         const size_t m = run.row0 + j;
@@ -61,22 +77,34 @@ __global__ void __launch_bounds__(NT) k_delta_step(const DeltaArgs a) {
             const float z = i < a.rank ? E::load((const T *)a.raw + m * a.ld + 5 * HD8 + i) + (a.bias ? BF16::to_f32(a.bias[5 * HD8 + i]) : 0.0f) : 0.0f;
             s_low[i] = tanhf(z);
         }
-        __syncthreads();
-        // the decay: eight lanes per channel
-        for (int d = threadIdx.x >> 3; d < CP; d += NT / 8) {
-            float z = 0.0f;
-            if (d < D) {
-                const u16 *wr = a.w_decay + (size_t)(head * D + d) * a.R8;
-                for (int i = (threadIdx.x & 7) * 8; i < a.R8; i += 64) {
-                    const uint4 q = *(const uint4 *)(wr + i);
-                    const float4 l0 = *(const float4 *)(s_low + i), l1 = *(const float4 *)(s_low + i + 4);
-                    z = fmaf(lo_f32<BF16>(q.x), l0.x, fmaf(hi_f32<BF16>(q.x), l0.y, fmaf(lo_f32<BF16>(q.y), l0.z, fmaf(hi_f32<BF16>(q.y), l0.w, z))));
-                    z = fmaf(lo_f32<BF16>(q.z), l1.x, fmaf(hi_f32<BF16>(q.z), l1.y, fmaf(lo_f32<BF16>(q.w), l1.z, fmaf(hi_f32<BF16>(q.w), l1.w, z))));
-                }
-            }
+        lds_barrier();
+        auto part = [&](float z, int i, const uint4 &w) {
+            const float4 l0 = *(const float4 *)(s_low + i), l1 = *(const float4 *)(s_low + i + 4);
+            z = fmaf(lo_f32<BF16>(w.x), l0.x, fmaf(hi_f32<BF16>(w.x), l0.y, fmaf(lo_f32<BF16>(w.y), l0.z, fmaf(hi_f32<BF16>(w.y), l0.w, z))));
+            return fmaf(lo_f32<BF16>(w.z), l1.x, fmaf(hi_f32<BF16>(w.z), l1.y, fmaf(lo_f32<BF16>(w.w), l1.z, fmaf(hi_f32<BF16>(w.w), l1.w, z))));
+        };
+        auto put_decay = [&](int d, float z, float bias) {
             z = lanes8_sum(z);
-            if ((threadIdx.x & 7) == 0) s_w[d] = d < D ? expf(-a.decay_scale / (1.0f + expf(-(z + a.decay_bias[head * D + d])))) : 1.0f;
-        }
+            if ((threadIdx.x & 7) == 0 && d < CP) s_w[d] = d < D ? expf(-a.decay_scale / (1.0f + expf(-(z + bias)))) : 1.0f;
+        };
+        if constexpr (AHEAD)
+#pragma unroll
+            for (int c = 0; c < CPT; ++c) {
+                const int d = (threadIdx.x >> 3) + c * (NT / 8);
+                float z = 0.0f;
+#pragma unroll
+                for (int s = 0; s < WS; ++s)
+                    if ((int)(threadIdx.x & 7) * 8 + 64 * s < a.R8) z = part(z, (threadIdx.x & 7) * 8 + 64 * s, wd[c][s]);
+                for (int i = (threadIdx.x & 7) * 8 + 64 * WS; i < a.R8; i += 64) z = part(z, i, decay_weights(d, i));
+                put_decay(d, z, db[c]);
+            }
+        else
+#pragma unroll 1
+            for (int d = threadIdx.x >> 3; d < CP; d += NT / 8) {
+                float z = 0.0f;
+                for (int i = (threadIdx.x & 7) * 8; i < a.R8; i += 64) z = part(z, i, decay_weights(d, i));
+                put_decay(d, z, a.decay_bias[head * D + min(d, D - 1)]);
+            }
         float ss = 0.0f;  // every wave: the key's length
         for (int d = lane; d < CP; d += 64) ss = fmaf(s_k[d], s_k[d], ss);
         const float unit = 1.0f / sqrtf(wave_sum(ss) + a.unit_eps);
@@ -84,7 +112,7 @@ __global__ void __launch_bounds__(NT) k_delta_step(const DeltaArgs a) {
 #pragma unroll
         for (int i = 0; i < RPT; ++i) p = fmaf(s_k[d0 + i], S[i], p);
         s_p[slice][col] = p * unit;
-        __syncthreads();
+        lds_barrier();
         p = 0.0f;
 #pragma unroll
         for (int i = 0; i < SL; ++i) p += s_p[i][col];
@@ -97,7 +125,7 @@ __global__ void __launch_bounds__(NT) k_delta_step(const DeltaArgs a) {
             o = fmaf(s_r[d0 + i], S[i], o);
         }
         s_o[slice][col] = o;
-        __syncthreads();
+        lds_barrier();
         if (threadIdx.x < (CP < 64 ? 64 : CP)) {  // whole waves
             o = 0.0f;
             if (threadIdx.x < CP)
@@ -106,15 +134,15 @@ __global__ void __launch_bounds__(NT) k_delta_step(const DeltaArgs a) {
             const float sum = wave_sum(o * o);
             if (lane == 0) s_ss[threadIdx.x >> 6] = sum;
         }
-        __syncthreads();
+        lds_barrier();
         if (threadIdx.x < D) {
             float sum = s_ss[0];
 #pragma unroll
             for (int i = 1; i < (CP + 63) / 64; ++i) sum += s_ss[i];
-            const float y = o * (1.0f / sqrtf(sum / (float)D + a.eps)) * a.o_norm[head * D + threadIdx.x] * s_g[threadIdx.x];
+            const float y = o * (1.0f / sqrtf(sum / (float)D + a.eps)) * (AHEAD ? o_norm : a.o_norm[head * D + threadIdx.x]) * s_g[threadIdx.x];
             ((T *)a.out)[m * a.ld_out + head * a.D8 + threadIdx.x] = E::pack(y);
         }
-        __syncthreads();  // the channel vectors are written again
+        lds_barrier();  // the channel vectors are written again
     }
     if (col < D)
 #pragma unroll
@@ -152,8 +180,6 @@ __device__ __forceinline__ DeltaChunk dr_chunk(const DeltaArgs &a, int i) {
     }
     return {a.runs[r].row0 + DC * i, min(DC, a.runs[r].n_rows - DC * i)};
 }
-
-__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }  // (loads and stores stay in flight)
 
 // One workgroup per (chunk, head).  A wave owns four tokens; its lanes own channel pairs.
 // NB: 16-channel blocks per wave in the products (D <= 64 NB).  Dynamic LDS: see delta_prep_lds().
@@ -602,12 +628,15 @@ int delta_chunks_go(const DeltaArgs &a, int chunks, int row0, int rows, hipStrea
 template <class E>
 int delta_step_go(const DeltaArgs &a, hipStream_t st) {
     const dim3 grid((unsigned)a.n_runs, (unsigned)a.H);
-#define DS_GO(CP_, NT_) hipLaunchKernelGGL((k_delta_step<E, CP_, NT_>), grid, dim3(NT_), 0, st, a)
-    if (a.D <= 16) DS_GO(16, 128);
-    else if (a.D <= 32) DS_GO(32, 256);
-    else if (a.D <= 64) DS_GO(64, 256);
-    else if (a.D <= 128) DS_GO(128, 512);
-    else DS_GO(256, 1024);
+    const bool ahead = (long)a.n_runs * a.H <= 256 && a.D <= 128;
+#define DS_GO(CP_, NT_) \
+    if (ahead) hipLaunchKernelGGL((k_delta_step<E, CP_, NT_, CP_ <= 128>), grid, dim3(NT_), 0, st, a); \
+    else hipLaunchKernelGGL((k_delta_step<E, CP_, NT_, false>), grid, dim3(NT_), 0, st, a)
+    if (a.D <= 16) { DS_GO(16, 128); }
+    else if (a.D <= 32) { DS_GO(32, 256); }
+    else if (a.D <= 64) { DS_GO(64, 256); }
+    else if (a.D <= 128) { DS_GO(128, 512); }
+    else { DS_GO(256, 1024); }
 #undef DS_GO
     PIE_LAUNCH_CHECK();
     return PIE_OK;

@@ -67,6 +67,34 @@ __device__ __forceinline__ void norm_row(const StackNorm &m, int W, float (&y)[N
     }
 }
 
+// the router's logits of the row in s_row; EB: experts of a wave in flight (the weights come from memory, and a wave has few of them)
+template <int EB, int NW>
+__device__ __forceinline__ void row_logits(const RowUpdateArgs &a, const float *s_row, float *s_z, int W8) {
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    for (int e0 = wave; e0 < a.experts; e0 += EB * NW) {
+        float z[EB];
+#pragma unroll
+        for (int i = 0; i < EB; ++i) z[i] = 0.0f;
+#pragma unroll 4
+        for (int k = lane * 8; k < W8; k += 512) {
+            uint4 v[EB];
+#pragma unroll
+            for (int i = 0; i < EB; ++i) v[i] = *(const uint4 *)(a.router + (size_t)min(e0 + i * NW, a.experts - 1) * W8 + k);
+            const float4 h0 = *(const float4 *)(s_row + k), h1 = *(const float4 *)(s_row + k + 4);
+#pragma unroll
+            for (int i = 0; i < EB; ++i) {
+                z[i] = fmaf(lo_f32<BF16>(v[i].x), h0.x, fmaf(hi_f32<BF16>(v[i].x), h0.y, fmaf(lo_f32<BF16>(v[i].y), h0.z, fmaf(hi_f32<BF16>(v[i].y), h0.w, z[i]))));
+                z[i] = fmaf(lo_f32<BF16>(v[i].z), h1.x, fmaf(hi_f32<BF16>(v[i].z), h1.y, fmaf(lo_f32<BF16>(v[i].w), h1.z, fmaf(hi_f32<BF16>(v[i].w), h1.w, z[i]))));
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < EB; ++i) {
+            const float sum = wave_sum(z[i]);
+            if (lane == 0 && e0 + i * NW < a.experts) s_z[e0 + i * NW] = sum;
+        }
+    }
+}
+
 // xv: next(x) of row blockIdx.x, quads as in k_row_update
 template <int THREADS, int NQ>
 __device__ __forceinline__ void row_route(const RowUpdateArgs &a, const float (&xv)[NQ][4]) {
@@ -82,19 +110,10 @@ __device__ __forceinline__ void row_route(const RowUpdateArgs &a, const float (&
         if (n < W8) *(float4 *)(s_dyn + n) = make_float4(xv[q][0], xv[q][1], xv[q][2], xv[q][3]);  // (zeros past W)
     }
     __syncthreads();
-    for (int e = wave; e < a.experts; e += THREADS / 64) {
-        const u16 *w = a.router + (size_t)e * W8;
-        float z = 0.0f;
-#pragma unroll 4
-        for (int k = lane * 8; k < W8; k += 512) {
-            const uint4 v = *(const uint4 *)(w + k);
-            const float4 h0 = *(const float4 *)(s_dyn + k), h1 = *(const float4 *)(s_dyn + k + 4);
-            z = fmaf(lo_f32<BF16>(v.x), h0.x, fmaf(hi_f32<BF16>(v.x), h0.y, fmaf(lo_f32<BF16>(v.y), h0.z, fmaf(hi_f32<BF16>(v.y), h0.w, z))));
-            z = fmaf(lo_f32<BF16>(v.z), h1.x, fmaf(hi_f32<BF16>(v.z), h1.y, fmaf(lo_f32<BF16>(v.w), h1.z, fmaf(hi_f32<BF16>(v.w), h1.w, z))));
-        }
-        z = wave_sum(z);
-        if (lane == 0) s_z[e] = z;
-    }
+    constexpr int NW = THREADS / 64;
+    if (a.experts <= NW) row_logits<1, NW>(a, s_dyn, s_z, W8);
+    else if (a.experts <= 2 * NW) row_logits<2, NW>(a, s_dyn, s_z, W8);
+    else row_logits<4, NW>(a, s_dyn, s_z, W8);
     __syncthreads();
     if (wave == 0) {
         route_pick(L, s_z, lane, [&](int k, int e, float w) {
@@ -203,11 +222,10 @@ __global__ void __launch_bounds__(THREADS) k_row_update(const RowUpdateArgs a) {
 template <class E>
 void row_go(const RowUpdateArgs &a, hipStream_t st) {
     const dim3 grid((unsigned)a.M);
-    if (a.route) {  // (at least eight waves: they share the experts)
+    if (a.route) {  // (always sixteen waves: they share the experts)
         const size_t lds = ((size_t)((a.W + 7) & ~7) + 3 * a.experts) * 4;
 #define ROW_GO(T_, Q_) hipLaunchKernelGGL((k_row_update<E, T_, Q_, true>), grid, dim3(T_), lds, st, a)
-        if (a.W <= 2048) ROW_GO(512, 1);
-        else if (a.W <= 4096) ROW_GO(1024, 1);
+        if (a.W <= 4096) ROW_GO(1024, 1);
         else ROW_GO(1024, 4);
 #undef ROW_GO
         return;
