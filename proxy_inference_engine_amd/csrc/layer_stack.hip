@@ -33,7 +33,7 @@ namespace {
 
 constexpr int BIG_ROWS = 64;  // more rows than this take the tiled GEMMs
 constexpr int LONG_RUN = 64;  // runs of at least this many rows take the attentions' long forms
-constexpr int ROUTE_FEW_ROWS = 64;              // up to this many rows, and router weights that one workgroup reads in a few us: chosen beside the norm
+constexpr int ROUTE_MIN_ROWS = 6, ROUTE_FEW_ROWS = 64;              // up to this many rows, and router weights that one workgroup reads in a few us: chosen beside the norm
 constexpr long ROUTE_FEW_WEIGHTS = 256l << 10;
 constexpr int DELTA_RUN = 8;  // runs of at least this many rows take the recurrence's chunk form
 
@@ -47,17 +47,35 @@ __host__ __device__ inline int route_max_tiles(long M, int top, int experts) {
     return ((int)(M * top / route_tile_rows(M, top, experts)) + route_block(M, top, experts) * experts + 3) / 4 * 4;
 }
 
+__device__ __forceinline__ void route_row(const RouteLayer &L, int m, int lane, const float (&corr)[ROUTE_KEPT]) {
+    route_pick(L, L.logits + (size_t)m * L.ld_logits, lane, corr, [&](int k, int e, float w) {
+        if (lane == 0) L.chosen[(size_t)m * L.top + k] = e, L.weight[(size_t)m * L.top + k] = w;
+    });
+}
 __global__ void __launch_bounds__(256) k_route_pick(const RouteLayer *layers, int M) {
-    const int m = blockIdx.x * 4 + (threadIdx.x >> 6);
+    const int m = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
     const RouteLayer L = layers[0];
-    if (m < M)
-        route_pick(L, L.logits + (size_t)m * L.ld_logits, threadIdx.x & 63, [&](int k, int e, float w) { L.chosen[(size_t)m * L.top + k] = e, L.weight[(size_t)m * L.top + k] = w; });
+    if (m >= M) return;
+    float corr[ROUTE_KEPT];
+    route_corrections(L, lane, corr);
+    route_row(L, m, lane, corr);
 }
 
-// the row lists of layers[blockIdx.x]
-__global__ void __launch_bounds__(1024) k_route(const RouteLayer *layers, const int *ids, int M, int vocab) {
+// the row lists of layers[blockIdx.x]; pick: its router's choice is made here too (few rows: no tiles)
+__global__ void __launch_bounds__(1024) k_route(const RouteLayer *layers, const int *ids, int M, int vocab, bool pick) {
     extern __shared__ int s_cnt[];  // [experts] counts, then [experts] cursors
     const RouteLayer L = layers[blockIdx.x];
+    if (pick) {
+        const int lane = threadIdx.x & 63;
+        float corr[ROUTE_KEPT];
+        route_corrections(L, lane, corr);
+        if (M == 1 && L.top <= 64) {
+            if (threadIdx.x < 64) route_single(L, L.logits, lane, corr);
+            return;
+        }
+        for (int m = threadIdx.x >> 6; m < M; m += 16) route_row(L, m, lane, corr);
+        __syncthreads();
+    }
     const int tr = route_tile_rows(M, L.top, L.experts), rb = route_block(M, L.top, L.experts);
     route_lists(
         L, M, s_cnt,
@@ -65,7 +83,7 @@ __global__ void __launch_bounds__(1024) k_route(const RouteLayer *layers, const 
             if (!L.table) return L.chosen[i];
             return L.table[(size_t)min(max(ids[i / L.top], 0), vocab - 1) * L.top + i % L.top];
         },
-        tr, rb, route_max_tiles(M, L.top, L.experts));
+        tr, rb, pick ? 0 : route_max_tiles(M, L.top, L.experts));
 }
 
 template <class E>
@@ -671,10 +689,14 @@ void feed_forward(Pass &p, int li, const pie_stack_layer &L, const pie_stack_nor
         p.linear(z);
         if (p.rc) return;
         const RouteLayer *dev = s->route_dev.p + s->route_at[li];
-        hipLaunchKernelGGL(k_route_pick, dim3((unsigned)((M + 3) / 4)), dim3(256), 0, p.st, dev, M);
-        hipLaunchKernelGGL(k_route, dim3(1), dim3(1024), (size_t)2 * L.experts * 4, p.st, dev, p.b.ids, M, s->cfg.vocab);
+        const bool few = !p.plan.big && M <= ROUTE_FEW_ROWS;
+        if (!few) {
+            hipLaunchKernelGGL(k_route_pick, dim3((unsigned)((M + 3) / 4)), dim3(256), 0, p.st, dev, M);
+            ++p.launches;
+        }
+        hipLaunchKernelGGL(k_route, dim3(1), dim3(few && M == 1 ? 64 : 1024), (size_t)2 * L.experts * 4, p.st, dev, p.b.ids, M, s->cfg.vocab, few);
         if (hipGetLastError() != hipSuccess) p.rc = pie::fail(PIE_E_HIP, "routing launch failed");
-        p.launches += 2;
+        ++p.launches;
     }
     CombineArgs c = {};
     c.part = s->part.p, c.part_s = s->part_s.p, c.ldp = W64, c.ldp_s = p.plan.big && !(W & 3) ? W : W64, c.place = r.place, c.weight = r.weight, c.top = L.top, c.W = W, c.gate = S ? L.shared_gate : nullptr;
@@ -723,7 +745,7 @@ int stack_enqueue(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
     const int M = b.n_rows, W = s->cfg.width, W64 = up64(W), WA = act_stride(W), V = s->cfg.vocab, n = s->cfg.n_layers, dt = s->cfg.dtype;
     Pass p{s, b, plan, st};
     if (s->n_table) {
-        hipLaunchKernelGGL(k_route, dim3((unsigned)s->n_table), dim3(1024), (size_t)s->route_lds, st, s->route_dev.p, b.ids, M, V);
+        hipLaunchKernelGGL(k_route, dim3((unsigned)s->n_table), dim3(1024), (size_t)s->route_lds, st, s->route_dev.p, b.ids, M, V, false);
         PIE_LAUNCH_CHECK();
         ++p.launches;
     }
@@ -745,8 +767,8 @@ int stack_enqueue(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
     for (int i = 0; i < n && !p.rc; ++i) {
         const pie_stack_layer &L = s->layers[i];
         const pie_stack_norm &after = i + 1 < n ? s->layers[i + 1].pre1 : fin, &next = L.ff == PIE_FF_NONE ? after : L.pre2;
-        // few rows: the launch that makes the router's input also chooses the experts
-        const bool routed = L.ff == PIE_FF_ROUTED_MOE && !plan.big && L.w_router_rows && M <= ROUTE_FEW_ROWS && (long)L.experts * W <= ROUTE_FEW_WEIGHTS && W <= 8192;
+        // some rows: the launch that makes the router's input also chooses the experts (for very few rows, spreading the router over the chip takes less time)
+        const bool routed = L.ff == PIE_FF_ROUTED_MOE && !plan.big && L.w_router_rows && M >= ROUTE_MIN_ROWS && M <= ROUTE_FEW_ROWS && (long)L.experts * W <= ROUTE_FEW_WEIGHTS && W <= 8192;
         if (L.mixer == PIE_MIXER_LATENT) latent_mixer(p, i, L, next, routed ? i : -1);
         else if (L.mixer == PIE_MIXER_ATTENTION) attention_mixer(p, i, L, next, routed ? i : -1);
         else delta_mixer(p, i, L, next, routed ? i : -1);

@@ -13,35 +13,78 @@ struct RouteLayer {      // one mixture layer's row lists (device pointers)
     int4 *tiles;  // {expert, first position, rows, 0}: row tiles of the grouped GEMM
 };
 
-// One wave: the `top` experts of a row with the largest sigmoid(logit) + correction (equal ones: the first), each with the weight sigmoid(logit).
-// Round k takes the best of what comes behind round k - 1's in that order, so nothing has to be marked as taken.
-// put(k, expert, weight) is called by one lane, in the order of the choice.
-template <class Put>
-__device__ __forceinline__ void route_pick(const RouteLayer &L, const float *z, int lane, Put &&put) {
-    constexpr int R = 4;  // scores a lane keeps; more experts than 64 R are scored again in every round
-    float keep[R];
-    auto score = [&](int e) { return 1.0f / (1.0f + expf(-z[e])) + L.correction[e]; };
+// sum / maximum over the wave without LDS, in every lane
+__device__ __forceinline__ float lanes_sum(float v) { return xor32_sum(xor16_sum(lanes16_sum(v))); }
+__device__ __forceinline__ float lanes_max(float v) {
+    v = fmaxf(v, __builtin_amdgcn_update_dpp(v, v, 0xB1, 0xF, 0xF, true));   // quad_perm [1,0,3,2]
+    v = fmaxf(v, __builtin_amdgcn_update_dpp(v, v, 0x4E, 0xF, 0xF, true));   // quad_perm [2,3,0,1]
+    v = fmaxf(v, __builtin_amdgcn_update_dpp(v, v, 0x141, 0xF, 0xF, true));  // row_half_mirror
+    v = fmaxf(v, __builtin_amdgcn_update_dpp(v, v, 0x140, 0xF, 0xF, true));  // row_mirror
+    return xor32_max(xor16_max(v));
+}
+
+constexpr int ROUTE_KEPT = 4;  // scores a lane keeps: up to 64 ROUTE_KEPT experts
+__device__ __forceinline__ void route_corrections(const RouteLayer &L, int lane, float (&corr)[ROUTE_KEPT]) {
 #pragma unroll
-    for (int r = 0; r < R; ++r) keep[r] = 64 * r + lane < L.experts ? score(64 * r + lane) : -INFINITY;
+    for (int r = 0; r < ROUTE_KEPT; ++r) corr[r] = L.correction[min(64 * r + lane, L.experts - 1)];
+}
+// One wave: the `top` experts of a row with the largest sigmoid(logit) + correction (equal ones: the first), each with the weight sigmoid(logit).
+// corr: what route_corrections() read.  put(k, expert, weight) is called by all lanes with the same arguments, in the order of the choice.
+template <class Put>
+__device__ __forceinline__ void route_pick(const RouteLayer &L, const float *z, int lane, const float (&corr)[ROUTE_KEPT], Put &&put) {
+    constexpr int R = ROUTE_KEPT;
+    auto sigmoid = [&](int e) { return 1.0f / (1.0f + expf(-z[e])); };
+    if (L.experts <= 64 * R) {  // a chosen score is taken out
+        float keep[R];
+#pragma unroll
+        for (int r = 0; r < R; ++r) keep[r] = 64 * r + lane < L.experts ? sigmoid(64 * r + lane) + corr[r] : -INFINITY;
+        for (int k = 0; k < L.top; ++k) {
+            const float top = lanes_max(fmaxf(fmaxf(keep[0], keep[1]), fmaxf(keep[2], keep[3])));
+            int e = L.experts;
+#pragma unroll
+            for (int r = R - 1; r >= 0; --r) {
+                const unsigned long long has = __ballot(keep[r] == top);
+                if (has) e = 64 * r + __builtin_ctzll(has);
+            }
+            e = e < L.experts ? e : k;  // (scores that compare with nothing)
+#pragma unroll
+            for (int r = 0; r < R; ++r)
+                if (64 * r + lane == e) keep[r] = -INFINITY;
+            put(k, e, sigmoid(e));
+        }
+        return;
+    }
+    // many experts: scored again in every round, which takes the best of what comes behind the round before in the order of the choice
     float last = INFINITY;
     int last_e = -1;
     for (int k = 0; k < L.top; ++k) {
         float best = -INFINITY;
         int at = 0x7fffffff;
-        auto look = [&](float s, int e) {
+        for (int e = lane; e < L.experts; e += 64) {
+            const float s = sigmoid(e) + L.correction[e];
             if ((s < last || (s == last && e > last_e)) && s > best) best = s, at = e;
-        };
-#pragma unroll
-        for (int r = 0; r < R; ++r)
-            if (64 * r + lane < L.experts) look(keep[r], 64 * r + lane);
-        for (int e = 64 * R + lane; e < L.experts; e += 64) look(score(e), e);
-        const float top = wave_max(best);
+        }
+        const float top = lanes_max(best);
         int e = best == top ? at : 0x7fffffff;
 #pragma unroll
         for (int o = 32; o > 0; o >>= 1) e = min(e, __shfl_xor(e, o, 64));
-        e = e < L.experts ? e : k;  // (scores that compare with nothing)
+        e = e < L.experts ? e : k;
         last = top, last_e = e;
-        if (lane == 0) put(k, e, 1.0f / (1.0f + expf(-z[e])));
+        put(k, e, sigmoid(e));
+    }
+}
+
+// One wave: the lists of a single row, without counting: every chosen expert has it, in the order of their numbers.  top <= 64.
+__device__ __forceinline__ void route_single(const RouteLayer &L, const float *z, int lane, const float (&corr)[ROUTE_KEPT]) {
+    int mine = 0x7fffffff, rank = 0;
+    float weight = 0.0f;
+    route_pick(L, z, lane, corr, [&](int k, int e, float w) {
+        if (lane == k) mine = e, weight = w;
+    });
+    for (int k = 0; k < L.top; ++k) rank += __builtin_amdgcn_readlane(mine, k) < mine;
+    if (lane < L.top) {
+        L.weight[lane] = weight, L.place[lane] = rank, L.list[rank] = 0, L.active[rank] = mine;
+        L.offset[mine] = rank, L.offset[mine + 1] = rank + 1;  // (neighbours that are both chosen agree)
     }
 }
 

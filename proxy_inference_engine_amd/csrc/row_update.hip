@@ -12,7 +12,7 @@ namespace {
 
 template <int THREADS>
 __device__ __forceinline__ float block_sum(float v, float *red) {  // red: THREADS / 64 floats, free again behind the next barrier
-    v = wave_sum(v);
+    v = lanes_sum(v);
     if constexpr (THREADS == 64) return v;
     if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
     __syncthreads();
@@ -89,7 +89,7 @@ __device__ __forceinline__ void row_logits(const RowUpdateArgs &a, const float *
         }
 #pragma unroll
         for (int i = 0; i < EB; ++i) {
-            const float sum = wave_sum(z[i]);
+            const float sum = lanes_sum(z[i]);
             if (lane == 0 && e0 + i * NW < a.experts) s_z[e0 + i * NW] = sum;
         }
     }
@@ -104,6 +104,8 @@ __device__ __forceinline__ void row_route(const RowUpdateArgs &a, const float (&
     int *s_cnt = (int *)(s_z + a.experts);
     __shared__ int s_last;
     const RouteLayer L = *a.route;
+    float corr[ROUTE_KEPT];
+    route_corrections(L, lane, corr);
 #pragma unroll
     for (int q = 0; q < NQ; ++q) {
         const int n = threadIdx.x * 4 + 4 * THREADS * q;
@@ -116,7 +118,8 @@ __device__ __forceinline__ void row_route(const RowUpdateArgs &a, const float (&
     else row_logits<4, NW>(a, s_dyn, s_z, W8);
     __syncthreads();
     if (wave == 0) {
-        route_pick(L, s_z, lane, [&](int k, int e, float w) {
+        route_pick(L, s_z, lane, corr, [&](int k, int e, float w) {
+            if (lane) return;
             const size_t i = (size_t)m * L.top + k;
             __hip_atomic_store(L.chosen + i, e, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);  // (seen by whichever workgroup arrives last, on any XCD)
             L.weight[i] = w;
