@@ -20,92 +20,95 @@ namespace {
 constexpr float PG_NEG = -1e30f, PG_LOG2E = 1.44269504088896340736f;
 
 // ---------------------------------------------------------------- projections -> queries, pages
-// One wave per row and run of PREP_HEADS heads: heads [0, H) queries, [H, H + G) keys, [H + G, H + 2 G) values.  Lane l holds the dimension pairs l, l + 64, ...
-// of a head; their angles are taken once for all heads of the wave.  NP: pairs per lane.
-constexpr int PREP_HEADS = 8;
-template <class E, int NP>
+// sin and cos of an angle: the library's in fp32 stacks; else reduced to one turn in two steps, then the trigonometric unit (absolute error about 1e-6)
+template <bool F32>
+__device__ __forceinline__ void pg_sincos(float a, float &s, float &c) {
+    if constexpr (F32) sincosf(a, &s, &c);
+    else {
+        const float n = rintf(a * 0.15915494309189533577f), r = fmaf(n, 1.7484556e-7f, fmaf(n, -6.2831855f, a)) * 0.15915494309189533577f;  // (6.2831855f is 2 pi + 1.7484556e-7)
+        s = __builtin_amdgcn_sinf(r), c = __builtin_amdgcn_cosf(r);
+    }
+}
+
+// One wave per row and run of HB heads of one kind (queries, keys or values).  Lane l holds the dimension pairs l, l + 64, ... of a head; angles and places in a
+// page are taken once for all heads of the wave.  NP: pairs per lane.
+template <class E, int NP, int HB>
 __global__ void __launch_bounds__(256) k_kv_prep(const KvPrepArgs a) {
     typedef typename E::type T;
+    constexpr bool F32 = sizeof(T) == 4;
     const KvGeometry &geo = a.geo;
-    const int m = blockIdx.x, lane = threadIdx.x & 63, heads = geo.H + (a.own ? 2 * geo.G : 0), head0 = (blockIdx.y * 4 + (threadIdx.x >> 6)) * PREP_HEADS;
-    if (head0 >= heads) return;
+    const int nq = (geo.H + HB - 1) / HB, nk = a.own ? (geo.G + HB - 1) / HB : 0, lane = threadIdx.x & 63, m = blockIdx.x;
+    int unit = __builtin_amdgcn_readfirstlane(blockIdx.y * 4 + (threadIdx.x >> 6));
+    if (unit >= nq + 2 * nk) return;
+    const bool is_q = unit < nq, is_v = unit >= nq + nk;
+    unit -= is_q ? 0 : is_v ? nq + nk : nq;
+    const int h0 = unit * HB, count = min(HB, (is_q ? geo.H : geo.G) - h0), n = is_v ? geo.vdim : geo.dim, stride = is_v ? geo.V8 : geo.D8;
+    const int off = (is_q ? 0 : is_v ? (geo.H + geo.G) * geo.D8 : geo.H * geo.D8) + h0 * stride;
+    T *x = (T *)a.raw + (size_t)m * a.ld + off;
+    float u[HB][NP], v[HB][NP];
+#pragma unroll
+    for (int k = 0; k < HB; ++k)
+#pragma unroll
+        for (int j = 0; j < NP; ++j) {
+            const int d = 2 * (lane + 64 * j), at = min(k, count - 1) * stride + min(d, (n - 1) & ~1);
+            float p, r;  // (an odd head's last partner is its padding: zero)
+            if constexpr (!F32) {
+                const u32 w = *(const u32 *)(x + at);
+                p = lo_f32<BF16>(w), r = hi_f32<BF16>(w);
+            } else {
+                const float2 w = *(const float2 *)(x + at);
+                p = w.x, r = w.y;
+            }
+            if (a.bias) {
+                const u32 w = *(const u32 *)(a.bias + off + at);  // (padded like the head)
+                p += lo_f32<BF16>(w), r += hi_f32<BF16>(w);
+            }
+            u[k][j] = d < n ? p : 0.0f, v[k][j] = d + 1 < n ? r : 0.0f;
+        }
     const int t = a.pos[m], tl = t & (PAGE_TOKENS - 1);
-    T *page = a.own && head0 + PREP_HEADS > geo.H ? (T *)a.slab + (size_t)page_of(a.pages, a.row_seq[m], t) * geo.page_elems() : nullptr;
-    float sn[NP], cs[NP];
-    if (head0 < geo.H + geo.G)
+    T *page = is_q ? nullptr : (T *)a.slab + (size_t)page_of(a.pages, a.row_seq[m], t) * geo.page_elems() + h0 * geo.head_elems();
+    const float *w = is_v ? nullptr : is_q ? a.q_norm : a.k_norm;
+    const bool normed = is_v ? a.value_norm : w != nullptr;
+    float sn[NP], cs[NP], wu[NP], wv[NP];
+    int place[NP], place1[NP];
+#pragma unroll
+    for (int j = 0; j < NP; ++j) {
+        const int d = 2 * (lane + 64 * j);
+        sn[j] = 0.0f, cs[j] = 1.0f, wu[j] = wv[j] = 1.0f;
+        if (w) wu[j] = w[min(d, n - 1)], wv[j] = w[min(d + 1, n - 1)];
+        if (!is_v && d + 1 < a.rot_dims) {
+            pg_sincos<F32>((float)t * a.freq[d >> 1], sn[j], cs[j]);
+            sn[j] *= a.rot_gain, cs[j] *= a.rot_gain;
+        }
+        place[j] = is_q ? d : is_v ? geo.value(tl, d) : geo.key(tl, d), place1[j] = is_v ? geo.value(tl, d + 1) : 0;
+    }
+    const float inv_n = 1.0f / (float)n;
+#pragma unroll
+    for (int k = 0; k < HB; ++k) {
+        if (k >= count) break;
+        float inv = 1.0f;
+        if (normed) {
+            float ss = 0.0f;
+#pragma unroll
+            for (int j = 0; j < NP; ++j) ss = fmaf(u[k][j], u[k][j], fmaf(v[k][j], v[k][j], ss));
+            ss = lanes_sum(ss) * inv_n + a.eps;
+            inv = F32 ? 1.0f / sqrtf(ss) : __builtin_amdgcn_rsqf(ss);
+        }
 #pragma unroll
         for (int j = 0; j < NP; ++j) {
             const int d = 2 * (lane + 64 * j);
-            sn[j] = 0.0f, cs[j] = 1.0f;
-            if (d + 1 < a.rot_dims) {
-                sincosf((float)t * a.freq[d >> 1], &sn[j], &cs[j]);
-                sn[j] *= a.rot_gain, cs[j] *= a.rot_gain;
+            if (d >= n) break;
+            const float p = u[k][j] * inv * wu[j], r = v[k][j] * inv * wv[j];
+            const float p2 = p * cs[j] - r * sn[j], r2 = r * cs[j] + p * sn[j];
+            if (is_v) {
+                T *dst = page + k * geo.head_elems();
+                dst[place[j]] = E::pack(p);
+                if (d + 1 < n) dst[place1[j]] = E::pack(r);
+                continue;
             }
-        }
-    constexpr int HB = NP == 1 ? 8 : NP == 2 ? 4 : 1;  // heads in flight
-    static_assert(PREP_HEADS % HB == 0, "whole batches of heads");
-    for (int h0 = head0; h0 < min(head0 + PREP_HEADS, heads); h0 += HB) {
-        float u[HB][NP], v[HB][NP];
-        auto offset = [&](int head) {
-            return head < geo.H + geo.G ? head * geo.D8 : (geo.H + geo.G) * geo.D8 + (head - geo.H - geo.G) * geo.V8;
-        };
-#pragma unroll
-        for (int k = 0; k < HB; ++k) {
-            const int head = min(h0 + k, heads - 1), n = head >= geo.H + geo.G ? geo.vdim : geo.dim, off = offset(head);
-            const T *x = (const T *)a.raw + (size_t)m * a.ld + off;
-#pragma unroll
-            for (int j = 0; j < NP; ++j) {
-                const int d = 2 * (lane + 64 * j), dd = min(d, (n - 1) & ~1);
-                float p, r;  // (an odd head's last partner is its padding: zero)
-                if constexpr (sizeof(T) == 2) {
-                    const u32 w = *(const u32 *)(x + dd);
-                    p = lo_f32<BF16>(w), r = hi_f32<BF16>(w);
-                } else {
-                    const float2 w = *(const float2 *)(x + dd);
-                    p = w.x, r = w.y;
-                }
-                if (a.bias) {
-                    const u32 w = *(const u32 *)(a.bias + off + dd);  // (padded like the head)
-                    p += lo_f32<BF16>(w), r += hi_f32<BF16>(w);
-                }
-                u[k][j] = d < n ? p : 0.0f, v[k][j] = d + 1 < n ? r : 0.0f;
-            }
-        }
-#pragma unroll
-        for (int k = 0; k < HB; ++k) {
-            const int head = h0 + k;
-            if (head >= min(head0 + PREP_HEADS, heads)) break;
-            const bool is_q = head < geo.H, is_v = head >= geo.H + geo.G;
-            const int g = is_q ? head : head - geo.H - (is_v ? geo.G : 0), n = is_v ? geo.vdim : geo.dim;
-            const float *w = is_v ? nullptr : is_q ? a.q_norm : a.k_norm;
-            float inv = 1.0f;
-            if (is_v ? a.value_norm : w != nullptr) {
-                float ss = 0.0f;
-#pragma unroll
-                for (int j = 0; j < NP; ++j) ss = fmaf(u[k][j], u[k][j], fmaf(v[k][j], v[k][j], ss));
-                inv = 1.0f / sqrtf(wave_sum(ss) / (float)n + a.eps);
-            }
-            T *x = (T *)a.raw + (size_t)m * a.ld + offset(head);
-#pragma unroll
-            for (int j = 0; j < NP; ++j) {
-                const int d = 2 * (lane + 64 * j);
-                if (d >= n) break;
-                float p = u[k][j] * inv, r = v[k][j] * inv;
-                if (is_v) {
-                    T *dst = page + g * geo.head_elems();
-                    dst[geo.value(tl, d)] = E::pack(p);
-                    if (d + 1 < n) dst[geo.value(tl, d + 1)] = E::pack(r);
-                    continue;
-                }
-                if (w) p *= w[d], r = d + 1 < n ? r * w[d + 1] : 0.0f;
-                if (d + 1 < a.rot_dims) {
-                    const float p2 = p * cs[j] - r * sn[j];
-                    r = r * cs[j] + p * sn[j], p = p2;
-                }
-                T *dst = is_q ? x + d : page + g * geo.head_elems() + geo.key(tl, d);  // (d even: both in one 8-dimension chunk, and the pair aligned)
-                if constexpr (sizeof(T) == 2) *(u32 *)dst = pack2<BF16>(p, r);
-                else *(float2 *)dst = make_float2(p, r);
-            }
+            T *dst = (is_q ? x + k * stride : page + k * geo.head_elems()) + place[j];  // (d even: both in one 8-dimension chunk, and the pair aligned)
+            if constexpr (!F32) *(u32 *)dst = pack2<BF16>(p2, r2);
+            else *(float2 *)dst = make_float2(p2, r2);
         }
     }
 }
@@ -453,12 +456,18 @@ bool page_attn_mfma(int dtype, const KvGeometry &g) { return dtype == PIE_BF16 &
 
 int kv_prep_launch(int dtype, const KvPrepArgs &a, hipStream_t st) {
     if (a.M <= 0) return PIE_OK;
-    const dim3 grid((unsigned)a.M, (unsigned)((a.geo.H + (a.own ? 2 * a.geo.G : 0) + 4 * PREP_HEADS - 1) / (4 * PREP_HEADS)));
     const int wide = a.geo.dim > a.geo.vdim ? a.geo.dim : a.geo.vdim;
-#define PREP_GO(NP_) \
-    if (dtype == PIE_F32) hipLaunchKernelGGL((k_kv_prep<ElemF32, NP_>), grid, dim3(256), 0, st, a); \
-    else hipLaunchKernelGGL((k_kv_prep<ElemBF16, NP_>), grid, dim3(256), 0, st, a)
-    if (wide <= 128) { PREP_GO(1); } else if (wide <= 256) { PREP_GO(2); } else { PREP_GO(8); }
+    const int hb = a.M < 64 || wide > 256 ? 1 : wide > 128 ? 4 : 8;  // few rows: a wave per head
+    auto units = [&](int n) { return (n + hb - 1) / hb; };
+    const dim3 grid((unsigned)a.M, (unsigned)((units(a.geo.H) + (a.own ? 2 * units(a.geo.G) : 0) + 3) / 4));
+#define PREP_GO(NP_, HB_) \
+    if (dtype == PIE_F32) hipLaunchKernelGGL((k_kv_prep<ElemF32, NP_, HB_>), grid, dim3(256), 0, st, a); \
+    else hipLaunchKernelGGL((k_kv_prep<ElemBF16, NP_, HB_>), grid, dim3(256), 0, st, a)
+    if (wide <= 128) {
+        if (hb == 1) { PREP_GO(1, 1); } else { PREP_GO(1, 8); }
+    } else if (wide <= 256) {
+        if (hb == 1) { PREP_GO(2, 1); } else { PREP_GO(2, 4); }
+    } else { PREP_GO(8, 1); }
 #undef PREP_GO
     PIE_LAUNCH_CHECK();
     return PIE_OK;

@@ -13,16 +13,6 @@ struct RouteLayer {      // one mixture layer's row lists (device pointers)
     int4 *tiles;  // {expert, first position, rows, 0}: row tiles of the grouped GEMM
 };
 
-// sum / maximum over the wave without LDS, in every lane
-__device__ __forceinline__ float lanes_sum(float v) { return xor32_sum(xor16_sum(lanes16_sum(v))); }
-__device__ __forceinline__ float lanes_max(float v) {
-    v = fmaxf(v, __builtin_amdgcn_update_dpp(v, v, 0xB1, 0xF, 0xF, true));   // quad_perm [1,0,3,2]
-    v = fmaxf(v, __builtin_amdgcn_update_dpp(v, v, 0x4E, 0xF, 0xF, true));   // quad_perm [2,3,0,1]
-    v = fmaxf(v, __builtin_amdgcn_update_dpp(v, v, 0x141, 0xF, 0xF, true));  // row_half_mirror
-    v = fmaxf(v, __builtin_amdgcn_update_dpp(v, v, 0x140, 0xF, 0xF, true));  // row_mirror
-    return xor32_max(xor16_max(v));
-}
-
 constexpr int ROUTE_KEPT = 4;  // scores a lane keeps: up to 64 ROUTE_KEPT experts
 __device__ __forceinline__ void route_corrections(const RouteLayer &L, int lane, float (&corr)[ROUTE_KEPT]) {
 #pragma unroll

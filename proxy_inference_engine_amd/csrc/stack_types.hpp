@@ -47,6 +47,16 @@ __device__ __forceinline__ float4 point_norm4(const PointNorm &n, int i, float4 
                        fmaf(fast_tanh(n.alpha * x.w), w.w, b.w));
 }
 
+// sum / maximum over the wave without LDS, in every lane
+__device__ __forceinline__ float lanes_sum(float v) { return xor32_sum(xor16_sum(lanes16_sum(v))); }
+__device__ __forceinline__ float lanes_max(float v) {
+    v = fmaxf(v, __builtin_amdgcn_update_dpp(v, v, 0xB1, 0xF, 0xF, true));   // quad_perm [1,0,3,2]
+    v = fmaxf(v, __builtin_amdgcn_update_dpp(v, v, 0x4E, 0xF, 0xF, true));   // quad_perm [2,3,0,1]
+    v = fmaxf(v, __builtin_amdgcn_update_dpp(v, v, 0x141, 0xF, 0xF, true));  // row_half_mirror
+    v = fmaxf(v, __builtin_amdgcn_update_dpp(v, v, 0x140, 0xF, 0xF, true));  // row_mirror
+    return xor32_max(xor16_max(v));
+}
+
 // ---------------------------------------------------------------- latent append
 // c_raw [M][ldc], fp32 or (raw16) bf16 -> RMS norm with weight w -> the row of its page
 struct LatentAppend {
