@@ -560,26 +560,53 @@ __global__ void __launch_bounds__(256, 1) k_delta_scan(const DeltaArgs a) {
         }
 }
 
-// the head's norm and the output gate over the chunk form's outputs: one wave per (row, head)
-template <class E>
+// the head's norm and the output gate over the chunk form's outputs: one wave per row and HB heads; lanes own channel pairs, NP each
+template <class E, int NP, int HB>
 __global__ void __launch_bounds__(256) k_delta_out(const DeltaArgs a, int row0) {
     typedef typename E::type T;
+    constexpr bool F32 = sizeof(T) == 4;
     const size_t m = row0 + blockIdx.x;
-    const int head = blockIdx.y * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-    if (head >= a.H) return;
-    constexpr int R = DELTA_MAX_DIM / 64;
-    const float *o = a.o + (m * a.H + head) * a.D8;
-    float v[R], ss = 0.0f;
+    const int h0 = (blockIdx.y * 4 + (threadIdx.x >> 6)) * HB, lane = threadIdx.x & 63, D = a.D;
+    if (h0 >= a.H) return;
+    const int count = min(HB, a.H - h0), g0 = 3 * a.H * a.D8;
+    float2 o[HB][NP], g[HB][NP], w[HB][NP];
 #pragma unroll
-    for (int r = 0; r < R; ++r) v[r] = 64 * r + lane < a.D ? o[64 * r + lane] : 0.0f, ss = fmaf(v[r], v[r], ss);
-    const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)a.D + a.eps);
-    const int at = 3 * a.H * a.D8 + head * a.D8;
+    for (int k = 0; k < HB; ++k)
 #pragma unroll
-    for (int r = 0; r < R; ++r) {
-        const int d = 64 * r + lane;
-        if (d >= a.D) break;
-        const float g = E::load((const T *)a.raw + m * a.ld + at + d) + (a.bias ? BF16::to_f32(a.bias[at + d]) : 0.0f);
-        ((T *)a.out)[m * a.ld_out + head * a.D8 + d] = E::pack(v[r] * inv * a.o_norm[head * a.D + d] / (1.0f + expf(-g)));
+        for (int p = 0; p < NP; ++p) {
+            const int head = h0 + min(k, count - 1), d = 2 * (lane + 64 * p), dd = min(d, a.D8 - 2), at = head * a.D8 + dd;
+            o[k][p] = *(const float2 *)(a.o + m * a.H * a.D8 + at);
+            if (d >= D) o[k][p].x = 0.0f;
+            if (d + 1 >= D) o[k][p].y = 0.0f;
+            if constexpr (F32) g[k][p] = *(const float2 *)((const T *)a.raw + m * a.ld + g0 + at);
+            else {
+                const u32 v = *(const u32 *)((const T *)a.raw + m * a.ld + g0 + at);
+                g[k][p] = make_float2(lo_f32<BF16>(v), hi_f32<BF16>(v));
+            }
+            if (a.bias) {
+                const u32 v = *(const u32 *)(a.bias + g0 + at);
+                g[k][p].x += lo_f32<BF16>(v), g[k][p].y += hi_f32<BF16>(v);
+            }
+            w[k][p] = make_float2(a.o_norm[head * D + min(d, D - 1)], a.o_norm[head * D + min(d + 1, D - 1)]);
+        }
+    const float inv_d = 1.0f / (float)D;
+#pragma unroll
+    for (int k = 0; k < HB; ++k) {
+        if (k >= count) break;
+        float ss = 0.0f;
+#pragma unroll
+        for (int p = 0; p < NP; ++p) ss = fmaf(o[k][p].x, o[k][p].x, fmaf(o[k][p].y, o[k][p].y, ss));
+        ss = lanes_sum(ss) * inv_d + a.eps;
+        const float inv = F32 ? 1.0f / sqrtf(ss) : __builtin_amdgcn_rsqf(ss);
+        T *out = (T *)a.out + m * a.ld_out + (h0 + k) * a.D8;
+#pragma unroll
+        for (int p = 0; p < NP; ++p) {
+            const int d = 2 * (lane + 64 * p);
+            if (d >= D) break;
+            const float x = o[k][p].x * inv * w[k][p].x * dr_sigmoid<F32>(g[k][p].x), y = o[k][p].y * inv * w[k][p].y * dr_sigmoid<F32>(g[k][p].y);  // (past an odd head's end: zero)
+            if constexpr (F32) *(float2 *)(out + d) = make_float2(x, y);
+            else *(u32 *)(out + d) = pack2<BF16>(x, y);
+        }
     }
 }
 
@@ -613,7 +640,8 @@ int delta_chunks_nb(const DeltaArgs &a, int chunks, int row0, int rows, hipStrea
         hipLaunchKernelGGL((k_delta_scan<E, NB>), dim3((unsigned)(a.H * dr_blocks(a.D)), (unsigned)a.n_runs), dim3(256), 0, st, seg);
         PIE_LAUNCH_CHECK();
     }
-    hipLaunchKernelGGL(k_delta_out<E>, dim3((unsigned)rows, (unsigned)((a.H + 3) / 4)), dim3(256), 0, st, a, row0);
+    constexpr int NP = NB <= 2 ? 1 : 2, HB = NB <= 2 ? 8 : 4;
+    hipLaunchKernelGGL((k_delta_out<E, NP, HB>), dim3((unsigned)rows, (unsigned)((a.H + 4 * HB - 1) / (4 * HB))), dim3(256), 0, st, a, row0);
     PIE_LAUNCH_CHECK();
     return PIE_OK;
 }
