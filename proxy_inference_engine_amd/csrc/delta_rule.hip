@@ -13,8 +13,8 @@
 //   S  <- W_16 S + sum_i (W_16 / W_i) (k_i v_i^T - a_i u_i p_i^T)
 // Everything but S and p is known beforehand: one launch (all chunks of all heads in parallel) takes the channel vectors, A, B, A', B' and T = (I + B)^-1 and
 // leaves T U, R, K, -A and T A, A', -B' in matrix operand order; a second walks the chunks, one workgroup per head and 16 value columns, whose four waves
-// split the key channels of S (which stays in accumulators and is its own B operand); a third takes the heads' norm and gate.  Decays are above exp(-0.61), so
-// W_16 > 6e-5: the quotients are formed as W_t times 1 / W_i in fp32 without loss.
+// split the key channels of S (which stays in accumulators and is its own B operand); a third takes the heads' norm and gate.  W_16 is
+// above exp(-16 decay_scale): the quotients are formed as W_t times 1 / W_i, which fp32 holds up to DELTA_MAX_DECAY.
 #include <algorithm>
 
 #include "stack_types.hpp"
@@ -26,7 +26,6 @@ namespace {
 
 constexpr int DC = 16;  // tokens of a chunk
 constexpr size_t DELTA_SEGMENT_BYTES = 96u << 20;
-
 
 __device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }  // (loads and stores stay in flight)
 

@@ -815,6 +815,7 @@ int mixer_ok(const pie_stack *s, int i, const pie_stack_layer &L) {
     } else if (L.mixer == PIE_MIXER_DELTA) {
         PIE_REQUIRE(L.dim <= DELTA_MAX_DIM && L.rank > 0 && L.rank <= DELTA_MAX_RANK, PIE_E_SHAPE, "pie_stack_set_layer: bad mixer sizes (delta rule: dim at most 256, rank at most 1024)");
         PIE_REQUIRE(L.w_decay && L.decay_bias && L.o_norm, PIE_E_ARG, "pie_stack_set_layer: missing mixer weights");
+        PIE_REQUIRE(L.decay_scale >= 0 && L.decay_scale <= DELTA_MAX_DECAY, PIE_E_ARG, "pie_stack_set_layer: decay_scale must be in [0, 2] (the chunk form divides by sixteen decays)");
     } else PIE_REQUIRE(false, PIE_E_ARG, "pie_stack_set_layer: unknown mixer");
     return PIE_OK;
 }

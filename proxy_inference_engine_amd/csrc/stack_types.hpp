@@ -301,6 +301,7 @@ int page_attn_long_launch(const PageAttnArgs &a, hipStream_t st);
 
 // ---------------------------------------------------------------- generalised delta rule (delta_rule.hip)
 constexpr int DELTA_MAX_DIM = 256, DELTA_MAX_RANK = 1024;
+constexpr float DELTA_MAX_DECAY = 2.0f;
 struct DeltaArgs {
     const void *raw;        // [M][ld] T: r, k, v, gate, rate [H][D8] each, then the decay's low-rank input [rank]
     int ld, M, H, D, D8, rank, R8;
