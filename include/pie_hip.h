@@ -573,17 +573,34 @@ typedef struct {
     const void *embed;         /* bf16 [vocab][width] */
     const void *head;          /* packed [vocab, width] */
     pie_stack_norm final_norm;
+    /* streams > 0: hyper-connections over that many residual streams (at most 16; every layer then has hyper1, and hyper2 with a feed-forward); 0: one plain
+     * residual.  The streams start as equal copies, and the final norm reads their sum. */
+    int streams;
+    int max_positions;         /* rows of `positions`; 0: no position vectors.  A pass may not go beyond them. */
+    const void *positions;     /* bf16 [max_positions][width], added to the embedding by position */
+    const void *bigram;        /* bf16 [buckets + 1][width], or NULL: row (previous token * mul_prev + token * mul_cur) mod buckets is added to the embedding,
+                                * at a sequence's first token row `buckets`; the previous token stands at the end of layer 0's state */
+    long long mul_prev, mul_cur;
+    int buckets, reserved;
 } pie_stack_config;
 
-enum { PIE_MIXER_LATENT = 1, PIE_MIXER_ATTENTION = 2, PIE_MIXER_DELTA = 3 };
-enum { PIE_FF_NONE = 0, PIE_FF_RELU2 = 1, PIE_FF_TABLE_MOE = 2, PIE_FF_ROUTED_MOE = 3 };
+enum { PIE_MIXER_LATENT = 1, PIE_MIXER_ATTENTION = 2, PIE_MIXER_DELTA = 3, PIE_MIXER_MLSTM = 4, PIE_MIXER_MINGRU = 5 };
+enum { PIE_FF_NONE = 0, PIE_FF_RELU2 = 1, PIE_FF_TABLE_MOE = 2, PIE_FF_ROUTED_MOE = 3, PIE_FF_XIELU = 4 };
 enum { PIE_ACT_SILU = 0, PIE_ACT_CLIPPED = 1 };
 
-/* One layer: x += post1(mixer(pre1(x))); x += post2(ff(pre2(x))).  Below, dim8 / vdim8 / rank8 = dim / vdim / rank rounded up to 8; rows and columns past a
+/* One layer: x += post1(mixer(pre1(x))); x += post2(ff(pre2(x))).  With hyper-connections (hyper1, hyper2: fp32 [streams (in) + streams (out) + streams *
+ * streams (mix, [from][to])]; RMS norms in front, none behind) instead: u = sum in[s] x_s, y = sublayer(pre(u)), x_t <- sum mix[s][t] x_s + out[t] y.
+ * conv_taps > 0: the mixer reads h + conv(h), h = pre1(.), conv(h)_t = sum_j conv[j] h_(t - taps + 1 + j) per channel with zeros in front of the sequence; conv
+ * fp32 [conv_taps][width rounded up to 64]; the last conv_taps - 1 inputs are part of the layer's state.  Below, dim8 / vdim8 / rank8 = dim / vdim / rank rounded up to 8; rows and columns past a
  * head's size are zero.
  * Latent mixer:  w_in packed [heads * dim8 + rank8, width] (the latent's down-projection last); w_uk heads x packed [rank, dim] (each head's
  * up-projection of keys, transposed); w_uv heads x packed [vdim, rank]; w_o packed [width, heads * vdim8]; w_kv packed [heads * (dim8 + vdim8), rank]
  * (all keys, then all values: long prompts spell K and V out; may be NULL); c_norm fp32 [rank].  window <= 0: no limit.
+ * With q_rank > 0: w_in packed [q_rank8 (query latent) + rank8 (latent) + rot_dim8 (key part that all heads share, rotated, not normed) + heads rounded up to 8
+ * (gate, when out_gate), width] (kv_from >= 0: no latent and key part; layer j's cached ones are read); q = w_uq RMSnorm(query latent, q_norm fp32 [q_rank]) with w_uq
+ * packed [heads * dim8 (unrotated) + heads * rot_dim8 (rotated), q_rank]; score = scale * (unrotated parts' + rotated parts' products); rotation: the first
+ * rot_dims numbers of a rotated part, number i with i + rot_dims / 2, by position * rot_freq[i], cos and sin times rot_gain.  head_sink fp32 [heads] (NULL: none): the
+ * softmax's denominator also has exp(head_sink).  out_gate as below.
  * Attention mixer (softmax attention over cached keys and values):  w_in packed [heads * dim8 (q) + kv_heads * dim8 (k) + kv_heads * vdim8 (v) + heads
  * rounded up to 8 (gate, when out_gate), width], in_bias bf16 in that order (NULL: none); q and k: RMS norm over dim with q_norm / k_norm (fp32 [dim]; NULL:
  * none), then the first rot_dims dimensions rotated in neighbouring pairs by position * rot_freq[i] (fp32 [rot_dims / 2]), cos and sin times rot_gain;
@@ -593,6 +610,14 @@ enum { PIE_ACT_SILU = 0, PIE_ACT_CLIPPED = 1 };
  * Delta mixer (generalised delta rule on a dim x dim state per head):  w_in packed [5 heads * dim8 (r, k, v, gate, removal rate) + rank8 (decay, low rank),
  * width], in_bias as above; w_decay bf16 [heads * dim][rank8] row-major; decay_bias fp32 [heads * dim]; decay = exp(-decay_scale * sigmoid(w_decay tanh(.) +
  * decay_bias)); unit key k / sqrt(sum k^2 + unit_eps); o_norm fp32 [heads * dim]; w_o packed [width, heads * dim8].
+ * mLSTM mixer (matrix memory with exponential gates):  w_in packed [heads * dim8 (q) + heads * dim8 (k) + heads * vdim8 (v) + heads * vdim8 (output gate) + heads
+ * rounded up to 8 (input gate) + the same (forget gate), width]; the two gates plus gate_bias; q times scale; log gates i = c(.), f = log sigmoid(c(.)), c(z) = gate_cap
+ * tanh(z / gate_cap); m_t = max(f + m_(t-1), i) from m = 0; S_t = exp(f + m_(t-1) - m_t) S_(t-1) + exp(i - m_t) k v^T, n_t likewise with k alone; o = S_t^T q /
+ * (max(|n_t . q|, exp(-m_t)) + unit_eps); then every head over its root mean square (eps), times o_norm (fp32 [heads * vdim]) and the sigmoid of the output gate;
+ * w_o packed [width, heads * vdim8].
+ * minGRU mixer:  heads = 1, dim = its size; w_in packed [dim8 (update gate) + dim8 (candidate) + dim8 (output gate), width], in_bias as above; z = sigmoid(.), candidate
+ * u + 1/2 where u >= 0, else sigmoid(u); S_t = (1 - z) S_(t-1) + z candidate; output S_t silu(output gate); w_o packed [width, dim8].
+ * Dense feed-forwards: w_down act(w_up h), act RELU2: max(z, 0)^2; XIELU: act_alpha z^2 + z / 2 for z > 0, act_beta (exp(z) - 1 - z) + z / 2 else.
  * Experts: w_gate_up experts x packed [2 * size, width] with rows (2 i, 2 i + 1) = (gate_i, up_i); w_down experts x packed [width, size].  act SILU:
  * silu(g) u; CLIPPED: g = min(gate, act_limit), u = clamp(up, +-act_limit), g sigmoid(act_alpha g) (u + 1).
  * TABLE_MOE: table int32 [vocab][top], every chosen expert weighs 1 / top.  ROUTED_MOE: w_router packed [experts, width], the `top` experts with the largest
@@ -619,13 +644,19 @@ typedef struct {
     const float *correction;
     const void *w_gate_up, *w_expert_down, *s_gate_up, *s_down;
     const float *shared_gate;
+    const float *hyper1, *hyper2, *conv;
+    int conv_taps, q_rank, rot_dim;
+    float gate_cap, act_beta;
+    const float *gate_bias;    /* mLSTM: fp32 [2][heads], input then forget gate */
+    const void *w_uq;
+    const float *head_sink;
 } pie_stack_layer;
 
 int pie_stack_create(const pie_stack_config *cfg, pie_stack **out);
 int pie_stack_destroy(pie_stack *s);
 int pie_stack_set_layer(pie_stack *s, int i, const pie_stack_layer *layer);
 /* elements per cached token of layer i (its page is [64][that many] in the stack's dtype; 0: the layer caches no tokens), bytes of one page, and
- * fp32 numbers of recurrent state per sequence (0: none).  A latent page holds token after token; a page of keys and values is laid out in matrix-core
+ * fp32 numbers of recurrent state per sequence (0: none; the mixer's, then the convolution's last inputs, then -- layer 0 -- the embedding's previous token).  A latent page holds token after token; a page of keys and values is laid out in matrix-core
  * operand order (csrc/page_attn.hip) and means something as a whole only. */
 int pie_stack_page_row(const pie_stack *s, int i);
 size_t pie_stack_state_floats(const pie_stack *s, int i);

@@ -41,7 +41,7 @@ __global__ void __launch_bounds__(NT, AHEAD ? 1 : 4) k_delta_step(const DeltaArg
     const int col = threadIdx.x % CP, slice = threadIdx.x / CP, d0 = slice * RPT;
     const int seq = min(a.row_seq[run.row0], a.n_seqs - 1);
     const size_t slot = min((unsigned)a.slots[seq], (unsigned)a.n_slots - 1u);
-    float *state = a.state + (slot * a.H + head) * D * D;
+    float *state = a.state + slot * a.slot_floats + (size_t)head * D * D;
     float S[RPT];
     const bool fresh = a.pos[run.row0] == 0;
 #pragma unroll
@@ -156,17 +156,6 @@ __host__ __device__ __forceinline__ size_t dr_chunk_floats(int D) { return (size
 
 __device__ __forceinline__ dr_f32x4 dr_mfma(float a, float b, const dr_f32x4 &c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
 
-// exp(x) and 1 / (1 + exp(-x)): fp32 stacks take the library's, 16-bit ones the exponential unit (a few units in the last place)
-constexpr float DR_LOG2E = 1.44269504088896340736f;
-template <bool F32>
-__device__ __forceinline__ float dr_exp(float x) {
-    return F32 ? expf(x) : __builtin_amdgcn_exp2f(x * DR_LOG2E);
-}
-template <bool F32>
-__device__ __forceinline__ float dr_sigmoid(float x) {
-    return F32 ? 1.0f / (1.0f + expf(-x)) : __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(x * -DR_LOG2E));
-}
-
 struct DeltaChunk {
     int row0, n;  // rows [row0, row0 + n)
 };
@@ -267,7 +256,7 @@ __global__ void __launch_bounds__(256) k_delta_prep(const DeltaArgs a) {
         put_low(j, pair_at(raw + (size_t)min(tr, c.n - 1) * a.ld + at), bias_at(at));
     }
     lds_barrier();
-    auto log_decay = [&](int t, int d, float z) { s_l[t * LD + d] = t < c.n && d < D ? -a.decay_scale * dr_sigmoid<F32>(z) : 0.0f; };
+    auto log_decay = [&](int t, int d, float z) { s_l[t * LD + d] = t < c.n && d < D ? -a.decay_scale * stack_sigmoid<F32>(z) : 0.0f; };
     if constexpr (F32) {
         for (int i = threadIdx.x; i < DC * 16 * nblk; i += 256) {
             const int t = i / (16 * nblk), d = i % (16 * nblk);
@@ -318,19 +307,19 @@ __global__ void __launch_bounds__(256) k_delta_prep(const DeltaArgs a) {
                 const float2 l = *(const float2 *)(s_l + t * LD + d);
                 L.x += l.x, L.y += l.y;
             }
-            float2 before = make_float2(dr_exp<F32>(L.x), dr_exp<F32>(L.y));
+            float2 before = make_float2(stack_exp<F32>(L.x), stack_exp<F32>(L.y));
 #pragma unroll
             for (int j = 0; j < TP; ++j) {
                 const int t = TP * wave + j, at = t * LD + d;
                 const bool lx = t < c.n && d < D, ly = t < c.n && d + 1 < D;
                 const float2 l = *(const float2 *)(s_l + at);
                 L.x += l.x, L.y += l.y;
-                const float2 e = make_float2(dr_exp<F32>(L.x), dr_exp<F32>(L.y)), back = make_float2(dr_exp<F32>(-L.x), dr_exp<F32>(-L.y));
+                const float2 e = make_float2(stack_exp<F32>(L.x), stack_exp<F32>(L.y)), back = make_float2(stack_exp<F32>(-L.x), stack_exp<F32>(-L.y));
                 const float2 k = make_float2(xk[p][j].x, xk[p][j].y), u = make_float2(k.x * unit[j], k.y * unit[j]);
                 *(float2 *)(s_u + at) = make_float2(u.x * before.x, u.y * before.y);
                 *(float2 *)(s_r + at) = make_float2(lx ? (xr[p][j].x + bx[p][0].x) * e.x : 0.0f, ly ? (xr[p][j].y + bx[p][0].y) * e.y : 0.0f);
                 *(float2 *)(s_k + at) = make_float2(k.x * back.x, k.y * back.y);
-                *(float2 *)(s_a + at) = make_float2(dr_sigmoid<F32>(xa[p][j].x + bx[p][2].x) * u.x * back.x, dr_sigmoid<F32>(xa[p][j].y + bx[p][2].y) * u.y * back.y);
+                *(float2 *)(s_a + at) = make_float2(stack_sigmoid<F32>(xa[p][j].x + bx[p][2].x) * u.x * back.x, stack_sigmoid<F32>(xa[p][j].y + bx[p][2].y) * u.y * back.y);
                 before = e;
             }
             if (wave == 3) *(float2 *)(s_wc + d) = before;
@@ -428,7 +417,7 @@ __global__ void __launch_bounds__(256, 1) k_delta_scan(const DeltaArgs a) {
     const int c_lo = max(a.chunk_lo - chunk0, 0), c_hi = min(a.chunk_hi - chunk0, (run.n_rows + DC - 1) / DC);  // this launch's chunks of the run
     if (c_lo >= c_hi) return;
     const size_t slot = min((unsigned)a.slots[min(a.row_seq[run.row0], a.n_seqs - 1)], (unsigned)a.n_slots - 1u);
-    float *state = a.state + (slot * a.H + head) * D * D;
+    float *state = a.state + slot * a.slot_floats + (size_t)head * D * D;
     const bool fresh = c_lo == 0 && a.pos[run.row0] == 0;
     dr_f32x4 S[NB];  // S[16 b + 4 q + i][col]
 #pragma unroll
@@ -559,56 +548,6 @@ __global__ void __launch_bounds__(256, 1) k_delta_scan(const DeltaArgs a) {
         }
 }
 
-// the head's norm and the output gate over the chunk form's outputs: one wave per row and HB heads; lanes own channel pairs, NP each
-template <class E, int NP, int HB>
-__global__ void __launch_bounds__(256) k_delta_out(const DeltaArgs a, int row0) {
-    typedef typename E::type T;
-    constexpr bool F32 = sizeof(T) == 4;
-    const size_t m = row0 + blockIdx.x;
-    const int h0 = (blockIdx.y * 4 + (threadIdx.x >> 6)) * HB, lane = threadIdx.x & 63, D = a.D;
-    if (h0 >= a.H) return;
-    const int count = min(HB, a.H - h0), g0 = 3 * a.H * a.D8;
-    float2 o[HB][NP], g[HB][NP], w[HB][NP];
-#pragma unroll
-    for (int k = 0; k < HB; ++k)
-#pragma unroll
-        for (int p = 0; p < NP; ++p) {
-            const int head = h0 + min(k, count - 1), d = 2 * (lane + 64 * p), dd = min(d, a.D8 - 2), at = head * a.D8 + dd;
-            o[k][p] = *(const float2 *)(a.o + m * a.H * a.D8 + at);
-            if (d >= D) o[k][p].x = 0.0f;
-            if (d + 1 >= D) o[k][p].y = 0.0f;
-            if constexpr (F32) g[k][p] = *(const float2 *)((const T *)a.raw + m * a.ld + g0 + at);
-            else {
-                const u32 v = *(const u32 *)((const T *)a.raw + m * a.ld + g0 + at);
-                g[k][p] = make_float2(lo_f32<BF16>(v), hi_f32<BF16>(v));
-            }
-            if (a.bias) {
-                const u32 v = *(const u32 *)(a.bias + g0 + at);
-                g[k][p].x += lo_f32<BF16>(v), g[k][p].y += hi_f32<BF16>(v);
-            }
-            w[k][p] = make_float2(a.o_norm[head * D + min(d, D - 1)], a.o_norm[head * D + min(d + 1, D - 1)]);
-        }
-    const float inv_d = 1.0f / (float)D;
-#pragma unroll
-    for (int k = 0; k < HB; ++k) {
-        if (k >= count) break;
-        float ss = 0.0f;
-#pragma unroll
-        for (int p = 0; p < NP; ++p) ss = fmaf(o[k][p].x, o[k][p].x, fmaf(o[k][p].y, o[k][p].y, ss));
-        ss = lanes_sum(ss) * inv_d + a.eps;
-        const float inv = F32 ? 1.0f / sqrtf(ss) : __builtin_amdgcn_rsqf(ss);
-        T *out = (T *)a.out + m * a.ld_out + (h0 + k) * a.D8;
-#pragma unroll
-        for (int p = 0; p < NP; ++p) {
-            const int d = 2 * (lane + 64 * p);
-            if (d >= D) break;
-            const float x = o[k][p].x * inv * w[k][p].x * dr_sigmoid<F32>(g[k][p].x), y = o[k][p].y * inv * w[k][p].y * dr_sigmoid<F32>(g[k][p].y);  // (past an odd head's end: zero)
-            if constexpr (F32) *(float2 *)(out + d) = make_float2(x, y);
-            else *(u32 *)(out + d) = pack2<BF16>(x, y);
-        }
-    }
-}
-
 // chunks whose operands are made and used at a time
 int delta_segment(int H, int D) {
     const size_t bytes = H * dr_chunk_floats(D) * 4;
@@ -639,10 +578,9 @@ int delta_chunks_nb(const DeltaArgs &a, int chunks, int row0, int rows, hipStrea
         hipLaunchKernelGGL((k_delta_scan<E, NB>), dim3((unsigned)(a.H * dr_blocks(a.D)), (unsigned)a.n_runs), dim3(256), 0, st, seg);
         PIE_LAUNCH_CHECK();
     }
-    constexpr int NP = NB <= 2 ? 1 : 2, HB = NB <= 2 ? 8 : 4;
-    hipLaunchKernelGGL((k_delta_out<E, NP, HB>), dim3((unsigned)rows, (unsigned)((a.H + 4 * HB - 1) / (4 * HB))), dim3(256), 0, st, a, row0);
-    PIE_LAUNCH_CHECK();
-    return PIE_OK;
+    const int g0 = 3 * a.H * a.D8;
+    const HeadOutArgs h = {a.o, nullptr, (const typename E::type *)a.raw + g0, a.bias ? a.bias + g0 : nullptr, a.ld, a.H, a.D, a.D8, a.o_norm, a.eps, a.out, a.ld_out};
+    return head_out_launch(sizeof(typename E::type) == 4 ? PIE_F32 : PIE_BF16, h, row0, rows, st);
 }
 template <class E>
 int delta_chunks_go(const DeltaArgs &a, int chunks, int row0, int rows, hipStream_t st) {

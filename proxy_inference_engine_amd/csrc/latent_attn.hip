@@ -6,8 +6,10 @@
 // latents is staged once in LDS and serves both products:
 //   S^T[key, pair] = C . Q'^T         A = rows of C (ds_read_b128), B = the pairs' queries, kept in registers;
 //   online softmax in fp32, base 2;   the reduction over keys runs over registers and one lane exchange;
-//   O^T[r, pair] += C^T . P^T         A = C^T by ds_read_b64_tr_b16, B = P^T as the score layout leaves it, split into hi + lo bf16 halves: weights
+//   O^T[r, pair] += C^T . P^T         (r: the latent's own numbers) A = C^T by ds_read_b64_tr_b16, B = P^T as the score layout leaves it, split into hi + lo bf16 halves: weights
 //                                     keep ~16 bits.
+// A cached row may hold more than the latent: numbers behind it that scores read too (a rotated key part all heads share), against a second part of the queries.
+// Where the sums are finished the denominator takes the head's sink, and the result the head's gate.
 // Scores, weights, their sums and the accumulators are fp32.  A sliding window is a bound on i - j: blocks outside it are never read.
 #include "mfma_store.hpp"    // w4m_pack
 #include "prefill_attn.hpp"  // MfmaT, f32x16_t
@@ -95,10 +97,14 @@ __global__ void __launch_bounds__(256, RC <= 8 ? 2 : 1) k_latent_attn(const Late
     const size_t pr = (size_t)row * a.H + head;
     const int t_q = a.pos[row], t_min = a.window > 0 ? t_q - a.window + 1 : 0;
     const int col0 = 16 * RC * wave;  // the wave's columns of the latent
-    const u16 *qp = (const u16 *)a.q + pr * a.ldr + col0;
     uint4 qf[RC];
 #pragma unroll
-    for (int s = 0; s < RC; ++s) qf[s] = col0 + 16 * s + 8 * h < a.ldr ? *(const uint4 *)(qp + 16 * s + 8 * h) : make_uint4(0, 0, 0, 0);
+    for (int s = 0; s < RC; ++s) {
+        const int at = col0 + 16 * s + 8 * h;
+        const u16 *qp = (const u16 *)a.q + pr * a.ldq + at;
+        if (at >= a.ldq) qp = (const u16 *)a.q_rot + (size_t)row * a.ld_rot + head * (a.ldr - a.ldq) + at - a.ldq;
+        qf[s] = at < a.ldr ? *(const uint4 *)qp : make_uint4(0, 0, 0, 0);
+    }
 
     f32x16_t o[RC / 2];
 #pragma unroll
@@ -179,6 +185,7 @@ __global__ void __launch_bounds__(256, RC <= 8 ? 2 : 1) k_latent_attn(const Late
         }
 #pragma unroll
         for (int d = 0; d < RC / 2; ++d) {
+            if (col0 + 32 * d >= a.ldq) break;  // (wave-uniform: nothing but score numbers, or nothing at all)
             if (d + 1 < RC / 2) ct[(d + 1) & 1][0] = read_c(0, d + 1), ct[(d + 1) & 1][1] = read_c(1, d + 1);
             __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
@@ -194,26 +201,26 @@ __global__ void __launch_bounds__(256, RC <= 8 ? 2 : 1) k_latent_attn(const Late
     if (c > last) return;
     const size_t MH = (size_t)a.M * a.H;
     if (a.splits == 1) {
-        const float inv = 1.0f / l;
-        u16 *dst = (u16 *)a.out + pr * a.ldr + col0;
+        const float inv = head_gate<false>(a.finish, row, head) / (l + head_sink2(a.finish, head, m_run));
+        u16 *dst = (u16 *)a.out + pr * a.ldq + col0;
 #pragma unroll
         for (int d = 0; d < RC / 2; ++d)
 #pragma unroll
             for (int k = 0; k < 4; ++k)  // registers 4k .. 4k + 3 <-> columns 32 d + 8 k + 4 h + {0..3}
-                if (col0 + 32 * d + 8 * k + 4 * h < a.ldr)
+                if (col0 + 32 * d + 8 * k + 4 * h < a.ldq)
                     *(uint2 *)(dst + 32 * d + 8 * k + 4 * h) =
                         make_uint2(w4m_pack<BF16>(o[d][4 * k] * inv, o[d][4 * k + 1] * inv), w4m_pack<BF16>(o[d][4 * k + 2] * inv, o[d][4 * k + 3] * inv));
     } else {
-        float *dst = a.ws + ((size_t)blockIdx.y * MH + pr) * a.ldr + col0;
+        float *dst = a.ws + ((size_t)blockIdx.y * MH + pr) * a.ldq + col0;
         if (l > 0.0f)
 #pragma unroll
             for (int d = 0; d < RC / 2; ++d)
 #pragma unroll
                 for (int k = 0; k < 4; ++k)
-                    if (col0 + 32 * d + 8 * k + 4 * h < a.ldr)
+                    if (col0 + 32 * d + 8 * k + 4 * h < a.ldq)
                         *(la_f32x4 *)(dst + 32 * d + 8 * k + 4 * h) = (la_f32x4){o[d][4 * k], o[d][4 * k + 1], o[d][4 * k + 2], o[d][4 * k + 3]};
         if (wave == 0 && h == 0) {
-            float *ml = a.ws + (size_t)a.splits * MH * a.ldr + ((size_t)blockIdx.y * MH + pr) * 2;
+            float *ml = a.ws + (size_t)a.splits * MH * a.ldq + ((size_t)blockIdx.y * MH + pr) * 2;
             ml[0] = m_run, ml[1] = l;
         }
     }
@@ -240,8 +247,10 @@ __global__ void __launch_bounds__(256) k_latent_attn_rows(const LatentAttnArgs a
     __shared__ float s_o[4][LA_RMAX], s_q[LA_RMAX], s_m[4], s_l[4];
     const int row = blockIdx.x, head = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const size_t pr = (size_t)row * a.H + head;
-    for (int r = threadIdx.x; r < a.R; r += 256) s_q[r] = E::load((const T *)a.q + pr * a.ldr + r);
-    for (int r = lane; r < a.R; r += 64) s_o[wave][r] = 0.0f;
+    for (int r = threadIdx.x; r < a.R; r += 256)
+        s_q[r] = E::load(r < a.ldq ? (const T *)a.q + pr * a.ldq + r : (const T *)a.q_rot + (size_t)row * a.ld_rot + head * (a.ldr - a.ldq) + r - a.ldq);
+    const int RO = min(a.R, a.ldq);
+    for (int r = lane; r < RO; r += 64) s_o[wave][r] = 0.0f;
     __syncthreads();
     const int t_q = a.pos[row], t_lo = a.window > 0 ? max(0, t_q - a.window + 1) : 0, seq = a.row_seq[row];
     float m = LA_NEG, l = 0.0f;
@@ -252,22 +261,84 @@ __global__ void __launch_bounds__(256) k_latent_attn_rows(const LatentAttnArgs a
         d = wave_sum(d) * a.scale;
         const float m2 = fmaxf(m, d), f = expf(m - m2), w = expf(d - m2);
         l = l * f + w, m = m2;
-        for (int r = lane; r < a.R; r += 64) s_o[wave][r] = fmaf(w, E::load(cp + r), s_o[wave][r] * f);
+        for (int r = lane; r < RO; r += 64) s_o[wave][r] = fmaf(w, E::load(cp + r), s_o[wave][r] * f);
     }
     if (lane == 0) s_m[wave] = m, s_l[wave] = l;
     __syncthreads();
     const float mx = fmaxf(fmaxf(s_m[0], s_m[1]), fmaxf(s_m[2], s_m[3]));
-    float f[4], sum = 0.0f;
+    const float sink = a.finish.sink ? a.finish.sink[head] : LA_NEG;
+    float f[4], sum = expf(sink - mx);
 #pragma unroll
     for (int w = 0; w < 4; ++w) f[w] = s_l[w] > 0.0f ? expf(s_m[w] - mx) : 0.0f, sum += s_l[w] * f[w];
-    for (int r = threadIdx.x; r < a.R; r += 256)
-        ((T *)a.out)[pr * a.ldr + r] = E::pack((s_o[0][r] * f[0] + s_o[1][r] * f[1] + s_o[2][r] * f[2] + s_o[3][r] * f[3]) / sum);
+    const float gate = head_gate<sizeof(T) == 4>(a.finish, row, head);
+    for (int r = threadIdx.x; r < RO; r += 256)
+        ((T *)a.out)[pr * a.ldq + r] = E::pack((s_o[0][r] * f[0] + s_o[1][r] * f[1] + s_o[2][r] * f[2] + s_o[3][r] * f[3]) * gate / sum);
 }
 
 template <class E, class X>
 __global__ void __launch_bounds__(256) k_latent_append(const LatentAppend a) {
     __shared__ float red[4];
     latent_append_row<E, X, 256>(a, blockIdx.x, red);
+}
+
+// One workgroup per row: the query latent's norm, the latent's norm into the page, and the shared key part's rotation.
+template <class E>
+__global__ void __launch_bounds__(256) k_latent_prep(const LatentPrepArgs a) {
+    typedef typename E::type T;
+    constexpr bool F32 = sizeof(T) == 4;
+    __shared__ float red[2][4];
+    const int m = blockIdx.x, wave = threadIdx.x >> 6;
+    const T *q = (const T *)a.raw + (size_t)m * a.ld, *c = q + a.Q8, *k = c + a.R8;
+    float sq = 0.0f, sc = 0.0f;
+    for (int i = threadIdx.x; i < a.Q; i += 256) sq = fmaf(E::load(q + i), E::load(q + i), sq);
+    if (a.own)
+        for (int i = threadIdx.x; i < a.R; i += 256) sc = fmaf(E::load(c + i), E::load(c + i), sc);
+    sq = lanes_sum(sq), sc = lanes_sum(sc);
+    if ((threadIdx.x & 63) == 0) red[0][wave] = sq, red[1][wave] = sc;
+    const int t = a.pos[m];
+    T *row = nullptr;
+    if (a.own) {
+        const size_t page = min((unsigned)a.table[(size_t)min(a.row_seq[m], a.n_seqs - 1) * a.table_width + min(t / PAGE_TOKENS, a.table_width - 1)], (unsigned)a.n_pages - 1u);
+        row = (T *)a.slab + (page * PAGE_TOKENS + (t & (PAGE_TOKENS - 1))) * (a.R8 + a.T8);
+    }
+    __syncthreads();
+    const float iq = 1.0f / sqrtf(((red[0][0] + red[0][1]) + (red[0][2] + red[0][3])) / (float)a.Q + a.eps);
+    T *cq = (T *)a.cq + (size_t)m * a.ldc;
+    for (int i = threadIdx.x; i < a.Q; i += 256) cq[i] = E::pack(E::load(q + i) * iq * a.q_norm[i]);
+    if (!a.own) return;
+    const float ic = 1.0f / sqrtf(((red[1][0] + red[1][1]) + (red[1][2] + red[1][3])) / (float)a.R + a.eps);
+    for (int i = threadIdx.x; i < a.R; i += 256) row[i] = E::pack(E::load(c + i) * ic * a.c_norm[i]);
+    row += a.R8;
+    const int half = a.rot.dims / 2;
+    for (int i = threadIdx.x; i < half; i += 256) {
+        float s, co;
+        stack_sincos<F32>((float)t * a.rot.freq[i], s, co);
+        s *= a.rot.gain, co *= a.rot.gain;
+        const float u = E::load(k + i), v = E::load(k + half + i);
+        row[i] = E::pack(u * co - v * s), row[half + i] = E::pack(v * co + u * s);
+    }
+    for (int i = 2 * half + threadIdx.x; i < a.T; i += 256) row[i] = k[i];
+}
+
+// One workgroup per row; a thread keeps one pair's angle for all heads it takes.
+template <class E>
+__global__ void __launch_bounds__(256) k_rotate_heads(const RotateArgs a) {
+    typedef typename E::type T;
+    constexpr bool F32 = sizeof(T) == 4;
+    const int m = blockIdx.x, half = a.rot.dims / 2;
+    int lanes = 1;
+    while (lanes < half && lanes < 256) lanes <<= 1;
+    const float t = (float)a.pos[m];
+    for (int i = threadIdx.x & (lanes - 1); i < half; i += lanes) {
+        float s, c;
+        stack_sincos<F32>(t * a.rot.freq[i], s, c);
+        s *= a.rot.gain, c *= a.rot.gain;
+        for (int h = threadIdx.x / lanes; h < a.H; h += 256 / lanes) {
+            T *p = (T *)a.q + (size_t)m * a.ld + h * a.stride + i;
+            const float u = E::load(p), v = E::load(p + half);
+            p[0] = E::pack(u * c - v * s), p[half] = E::pack(v * c + u * s);
+        }
+    }
 }
 
 }  // namespace
@@ -280,6 +351,7 @@ int latent_attn_launch(int dtype, const LatentAttnArgs &a, hipStream_t st) {
     if (a.M <= 0) return PIE_OK;
     PIE_REQUIRE(a.R > 0 && a.R <= LA_RMAX && a.H > 0 && a.H <= 65535, PIE_E_SHAPE, "latent attention: kv_rank must be 1 .. 2048");
     PIE_REQUIRE(a.splits >= 1 && (a.splits == 1 || a.ws), PIE_E_ARG, "latent attention: a key split needs its workspace");
+    PIE_REQUIRE(a.ldq % 8 == 0 && a.ldr % 8 == 0 && a.R <= a.ldr && (a.ldq == a.ldr || (a.ldq < a.ldr && a.q_rot && a.ld_rot % 8 == 0)), PIE_E_ALIGN, "latent attention: row strides");
     if (dtype == PIE_F32 || a.R > 1024) {
         const dim3 grid((unsigned)a.M, (unsigned)a.H);
         if (dtype == PIE_F32) hipLaunchKernelGGL(k_latent_attn_rows<ElemF32>, grid, dim3(256), 0, st, a);
@@ -295,12 +367,13 @@ int latent_attn_launch(int dtype, const LatentAttnArgs &a, hipStream_t st) {
     else if (rc <= 4) LA_GO(4);
     else if (rc <= 6) LA_GO(6);
     else if (rc <= 8) LA_GO(8);
+    else if (rc <= 10) LA_GO(10);
     else if (rc <= 12) LA_GO(12);
     else LA_GO(16);
 #undef LA_GO
     PIE_LAUNCH_CHECK();
     if (a.splits > 1 && a.combine) {
-        const LatentMerge m = {a.ws, a.splits, a.M, a.H, a.ldr};
+        const LatentMerge m = {a.ws, a.splits, a.M, a.H, a.ldq, a.finish};
         hipLaunchKernelGGL(k_latent_combine, dim3((unsigned)(a.M * a.H)), dim3(128), 0, st, m, (u16 *)a.out);
         PIE_LAUNCH_CHECK();
     }
@@ -313,6 +386,24 @@ int latent_append_launch(int dtype, const LatentAppend &a, hipStream_t st) {
     if (dtype == PIE_F32) hipLaunchKernelGGL((k_latent_append<ElemF32, ElemF32>), grid, dim3(256), 0, st, a);
     else if (a.raw16) hipLaunchKernelGGL((k_latent_append<ElemBF16, ElemBF16>), grid, dim3(256), 0, st, a);
     else hipLaunchKernelGGL((k_latent_append<ElemBF16, ElemF32>), grid, dim3(256), 0, st, a);
+    PIE_LAUNCH_CHECK();
+    return PIE_OK;
+}
+
+int latent_prep_launch(int dtype, const LatentPrepArgs &a, hipStream_t st) {
+    if (a.M <= 0) return PIE_OK;
+    PIE_REQUIRE(a.rot.dims >= 0 && a.rot.dims <= a.T && a.rot.dims % 2 == 0 && (a.rot.dims == 0 || a.rot.freq), PIE_E_SHAPE, "latent attention: bad rotation");
+    if (dtype == PIE_F32) hipLaunchKernelGGL(k_latent_prep<ElemF32>, dim3((unsigned)a.M), dim3(256), 0, st, a);
+    else hipLaunchKernelGGL(k_latent_prep<ElemBF16>, dim3((unsigned)a.M), dim3(256), 0, st, a);
+    PIE_LAUNCH_CHECK();
+    return PIE_OK;
+}
+
+int rotate_heads_launch(int dtype, const RotateArgs &a, hipStream_t st) {
+    if (a.M <= 0 || a.rot.dims <= 0) return PIE_OK;
+    PIE_REQUIRE(a.rot.dims % 2 == 0 && a.rot.dims <= a.stride && a.rot.freq, PIE_E_SHAPE, "rotation: an even number of a head's numbers");
+    if (dtype == PIE_F32) hipLaunchKernelGGL(k_rotate_heads<ElemF32>, dim3((unsigned)a.M), dim3(256), 0, st, a);
+    else hipLaunchKernelGGL(k_rotate_heads<ElemBF16>, dim3((unsigned)a.M), dim3(256), 0, st, a);
     PIE_LAUNCH_CHECK();
     return PIE_OK;
 }

@@ -3,12 +3,17 @@
 // A pass is a batch of rows, each with its own sequence and position: whole prompts, portions and single decoded tokens are the same thing here.
 // A layer is a mixer and a feed-forward, each between two norms.  Mixers:
 //   latent attention      [q | latent down] Linear; q -> latent space per head (beside it the latents' RMS norm and their append to the pages); attention
-//                         (latent_attn.hip); latents -> values per head, merging the key splits on the way in (more than a few rows: a launch of its own)
+//                         (latent_attn.hip); latents -> values per head, merging the key splits on the way in (more than a few rows: a launch of its own).
+//                         With a query latent: [query latent | latent | rotated key | gate] Linear; norms, key rotation, append; queries out of their latent, rotated
 //   attention             [q | k | v | gate] Linear; norms, rotation and page writes; attention over keys and values (page_attn.hip)
 //   delta rule            [r | k | v | gate | rate | decay] Linear; recurrence (delta_rule.hip)
-// and an output projection.  Feed-forwards: dense up (relu^2), down; or experts: gate|up and down over the active experts (and a shared one).
+//   mLSTM                 [q | k | v | gate | i | f] Linear; recurrence (mlstm.hip); head norm and gate (head_out.hip)
+//   minGRU                [z | candidate | gate] Linear; recurrence (mingru.hip)
+// and an output projection.  Feed-forwards: dense up (relu^2 or xIELU), down; or experts: gate|up and down over the active experts (and a shared one).
 // Norms: element-wise ones ride in the epilogue of the kernel that produces their input (x += post(y), h = next(x)); a norm over the whole row is applied,
 // with the same additions, by one launch behind the sublayer (row_update.hip), which also takes the experts' weighted sum.
+// Hyper-connections keep several residual streams: one launch behind every sublayer mixes them, takes the next sublayer's input out of them, and norms (and, for a mixer,
+// convolves) it (stream_update.hip); the first one starts the streams from the embedding.
 // A pass of more rows than the weight-streaming Linear is for (BIG_ROWS; bf16) multiplies through the tiled GEMMs instead (w16_gemm.hpp, grouped by expert
 // for mixtures); runs of LONG_RUN rows and more use the attentions' long forms (latents: with keys and values spelled out, window_attn.hip) while the
 // shorter runs in front of them keep the short ones.
@@ -25,7 +30,7 @@
 size_t w16l_workspace_bytes(int M, int N, int K);
 int w16l_gemm_launch(int dtype, const void *w16m, const void *x, int ldx, int M, int N, int K, void *y, void *workspace, hipStream_t st, const void *bias,
                      void *swiglu_act, bool *fused, int ldy);
-int w16l_relu2_launch(const void *w16m, const void *x, int ldx, int M, int N, int K, void *y, int ldy, hipStream_t st);
+int w16l_act_launch(const void *w16m, const void *x, int ldx, int M, int N, int K, void *y, int ldy, int act, float alpha, float beta, hipStream_t st);
 int w16l_grouped_launch(const void *w16m, size_t w_stride, const void *x, int ldx, size_t x_rows, const int *list, const void *tiles, int tm, int block, int tile_rows, int N, int K,
                         void *y, int ldy, int act, float act_alpha, float act_limit, hipStream_t st);
 
@@ -35,7 +40,7 @@ constexpr int BIG_ROWS = 64;  // more rows than this take the tiled GEMMs
 constexpr int LONG_RUN = 64;  // runs of at least this many rows take the attentions' long forms
 constexpr int ROUTE_MIN_ROWS = 6, ROUTE_FEW_ROWS = 64;              // up to this many rows, and router weights that one workgroup reads in a few us: chosen beside the norm
 constexpr long ROUTE_FEW_WEIGHTS = 256l << 10;
-constexpr int DELTA_RUN = 8;  // runs of at least this many rows take the recurrence's chunk form
+constexpr int CHUNK_RUN = 8;  // runs of at least this many rows take the recurrences' chunk forms
 
 // rows per tile of the grouped GEMM, and a bound on the number of tiles
 __host__ __device__ inline int route_tile_rows(long M, int top, int experts) { return M * top >= 96l * experts ? 128 : 64; }
@@ -309,8 +314,8 @@ struct pie_stack {
     std::vector<pie_stack_layer> layers;
     std::vector<char> have;
     // workspace, by rows of a pass
-    Buf<float> x, c_raw, part, part_s, attn_ws, gemm_ws, y32, logits_e, delta_ws, delta_o;
-    Buf<char> h, q, ql, oc, o, act, act_e, act_s, y, ctx, kv;
+    Buf<float> x, c_raw, part, part_s, attn_ws, gemm_ws, y32, logits_e, rec_ws, rec_o, rec_den;
+    Buf<char> h, hc, q, qu, cq, ql, oc, o, act, act_e, act_s, y, ctx, kv;
     Buf<RowStat> stats;
     Buf<int> route_ints;
     Buf<RouteLayer> route_dev;
@@ -337,13 +342,40 @@ PointNorm norm_of(const pie_stack_norm &n) { return {n.w, n.b, n.param}; }
 StackNorm row_norm_of(const pie_stack_norm &n) { return {n.w, n.b, n.param, n.kind}; }
 bool is_moe(const pie_stack_layer &L) { return L.ff == PIE_FF_TABLE_MOE || L.ff == PIE_FF_ROUTED_MOE; }
 KvGeometry geometry(const pie_stack_layer &L) { return kv_geometry(L.heads, L.kv_heads, L.dim, L.vdim); }
+bool is_dense(const pie_stack_layer &L) { return L.ff == PIE_FF_RELU2 || L.ff == PIE_FF_XIELU; }
+bool own_cache(const pie_stack_layer &L) { return (L.mixer == PIE_MIXER_LATENT && (!L.q_rank || L.kv_from < 0)) || (L.mixer == PIE_MIXER_ATTENTION && L.kv_from < 0); }
 // columns of the mixer's input projection, and what its output projection reads
 int in_columns(const pie_stack_layer &L) {
-    if (L.mixer == PIE_MIXER_LATENT) return L.heads * up8(L.dim) + up8(L.rank);
-    if (L.mixer == PIE_MIXER_DELTA) return 5 * L.heads * up8(L.dim) + up8(L.rank);
-    return L.heads * up8(L.dim) + (L.kv_from < 0 ? L.kv_heads * (up8(L.dim) + up8(L.vdim)) : 0) + (L.out_gate ? up8(L.heads) : 0);
+    const int gate = L.out_gate ? up8(L.heads) : 0;
+    switch (L.mixer) {
+        case PIE_MIXER_LATENT:
+            if (L.q_rank) return up8(L.q_rank) + (own_cache(L) ? up8(L.rank) + up8(L.rot_dim) : 0) + gate;
+            return L.heads * up8(L.dim) + up8(L.rank);
+        case PIE_MIXER_DELTA: return 5 * L.heads * up8(L.dim) + up8(L.rank);
+        case PIE_MIXER_MLSTM: return 2 * L.heads * (up8(L.dim) + up8(L.vdim)) + 2 * up8(L.heads);
+        case PIE_MIXER_MINGRU: return 3 * up8(L.dim);
+        default: return L.heads * up8(L.dim) + (own_cache(L) ? L.kv_heads * (up8(L.dim) + up8(L.vdim)) : 0) + gate;
+    }
 }
-int out_columns(const pie_stack_layer &L) { return L.heads * up8(L.mixer == PIE_MIXER_DELTA ? L.dim : L.vdim); }
+int out_columns(const pie_stack_layer &L) { return L.heads * up8(L.mixer == PIE_MIXER_DELTA || L.mixer == PIE_MIXER_MINGRU ? L.dim : L.vdim); }
+int up4(int n) { return (n + 3) & ~3; }
+int latent_row(const pie_stack_layer &L) { return up8(L.rank) + up8(L.rot_dim); }  // numbers of a cached latent row
+
+// A layer's recurrent state: the mixer's, the last inputs of the convolution in front of it, and (layer 0) the embedding's previous token
+struct StateLayout {
+    size_t conv, prev, total;  // where the second and the third begin
+};
+StateLayout state_layout(const pie_stack *s, int i) {
+    const pie_stack_layer &L = s->layers[i];
+    size_t mixer = 0;
+    if (L.mixer == PIE_MIXER_DELTA) mixer = (size_t)L.heads * L.dim * L.dim;
+    else if (L.mixer == PIE_MIXER_MLSTM) mixer = mlstm_state_floats(L.heads, L.dim, L.vdim);
+    else if (L.mixer == PIE_MIXER_MINGRU) mixer = L.dim;
+    const size_t conv = L.conv_taps > 1 ? (size_t)(L.conv_taps - 1) * up4(s->cfg.width) : 0, prev = i == 0 && s->cfg.bigram ? 4 : 0;
+    if (!conv && !prev && (L.mixer == PIE_MIXER_DELTA || !mixer)) return {mixer, mixer, mixer};
+    mixer = (mixer + 3) / 4 * 4;
+    return {mixer, mixer + conv, mixer + conv + prev};
+}
 
 // How a pass is laid out: rows of the leading short runs, and what the long runs behind them see.
 struct Plan {
@@ -356,7 +388,7 @@ Plan plan_pass(const pie_stack *s, const pie_stack_batch &b) {
     p.long_rows = b.n_rows - p.short_rows;
     return p;
 }
-bool spelled_out(const pie_stack_layer &L) { return L.w_kv && up8(L.dim) <= WINDOW_ATTN_MAX_DIM && up8(L.vdim) <= WINDOW_ATTN_MAX_DIM; }
+bool spelled_out(const pie_stack_layer &L) { return L.w_kv && up8(L.dim) + up8(L.rot_dim) <= WINDOW_ATTN_MAX_DIM && up8(L.vdim) <= WINDOW_ATTN_MAX_DIM; }
 // tokens the long runs of a layer see
 size_t plan_context(const pie_stack_batch &b, const Plan &p, int window) {
     size_t n = 0;
@@ -368,21 +400,26 @@ size_t plan_context(const pie_stack_batch &b, const Plan &p, int window) {
     return n;
 }
 
-// the leading runs that take the recurrence's step form, their rows, and the chunks of those behind them
-struct DeltaPart {
+// the leading runs that take a recurrence's step form, their rows, and the chunks of those behind them
+struct ChunkPart {
     int runs, rows, chunks;
 };
-DeltaPart delta_part(const pie_stack_batch &b) {
-    DeltaPart p = {0, 0, 0};
-    while (p.runs < b.n_runs && b.runs_host[4 * p.runs + 1] < DELTA_RUN) p.rows += b.runs_host[4 * p.runs++ + 1];
-    for (int i = p.runs; i < b.n_runs; ++i) p.chunks += delta_chunks(b.runs_host[4 * i + 1]);
+bool chunk_form(const pie_stack *s, const pie_stack_layer &L) { return L.mixer != PIE_MIXER_MLSTM || (s->cfg.dtype == PIE_BF16 && L.dim <= MLSTM_CHUNK_MAX_DIM); }
+ChunkPart chunk_part(const pie_stack *s, const pie_stack_batch &b, const pie_stack_layer &L) {
+    ChunkPart p = {0, 0, 0};
+    const bool chunks = chunk_form(s, L);
+    while (p.runs < b.n_runs && (!chunks || b.runs_host[4 * p.runs + 1] < CHUNK_RUN)) p.rows += b.runs_host[4 * p.runs++ + 1];
+    for (int i = p.runs; i < b.n_runs; ++i) {
+        const int n = b.runs_host[4 * i + 1];
+        p.chunks += L.mixer == PIE_MIXER_DELTA ? delta_chunks(n) : L.mixer == PIE_MIXER_MLSTM ? mlstm_chunks(n) : mingru_chunks(n);
+    }
     return p;
 }
 
 int stack_reserve(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipStream_t st) {
     const size_t M = (size_t)b.n_rows, E = esize(s), W64 = up64(s->cfg.width), WA = act_stride(s->cfg.width);
-    size_t q = 0, c = 0, ql = 0, o = 0, act = 0, act_e = 0, act_s = 0, part = 0, part_s = 0, ints = 0, ctx = 0, kv = 0, ws = 0, le = 0, dw = 0, dout = 0;
-    const DeltaPart dp = delta_part(b);
+    size_t q = 0, c = 0, ql = 0, o = 0, act = 0, act_e = 0, act_s = 0, part = 0, part_s = 0, ints = 0, ctx = 0, kv = 0, ws = 0, le = 0, rw = 0, ro = 0, rd = 0, hc = 0, qu = 0, cq = 0;
+    const size_t streams = std::max(s->cfg.streams, 1);
     auto gemm = [&](int N, int K) { ws = std::max(ws, w16l_workspace_bytes((int)M, N, K) / 4); };
     for (const pie_stack_layer &L : s->layers) {
         const int NI = in_columns(L), KO = out_columns(L);
@@ -390,15 +427,26 @@ int stack_reserve(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
         if (plan.big) gemm(NI, s->cfg.width), gemm(s->cfg.width, KO);
         if (L.mixer == PIE_MIXER_LATENT) {
             c = std::max(c, (size_t)up8(L.rank)), ql = std::max(ql, (size_t)L.heads * up8(L.rank));
-            if (plan.big) gemm(L.heads * up8(L.dim), s->cfg.width), gemm(up8(L.rank), s->cfg.width);
+            if (L.q_rank) {
+                const int NQ = L.heads * (up8(L.dim) + up8(L.rot_dim));
+                qu = std::max(qu, (size_t)NQ), cq = std::max(cq, (size_t)act_stride(L.q_rank));
+                if (plan.big) gemm(NQ, L.q_rank);
+            } else if (plan.big) gemm(L.heads * up8(L.dim), s->cfg.width), gemm(up8(L.rank), s->cfg.width);
             if (plan.long_rows && spelled_out(L)) {
                 const size_t n = plan_context(b, plan, L.window), nkv = L.heads * (up8(L.dim) + up8(L.vdim));
-                ctx = std::max(ctx, n * act_stride(L.rank)), kv = std::max(kv, n * nkv);
+                ctx = std::max(ctx, n * act_stride(latent_row(L))), kv = std::max(kv, n * nkv);
                 ws = std::max(ws, w16l_workspace_bytes((int)n, (int)nkv, L.rank) / 4);
             }
         }
-        if (L.mixer == PIE_MIXER_DELTA && dp.chunks) dw = std::max(dw, delta_ws_floats(dp.chunks, L.heads, L.dim)), dout = std::max(dout, (size_t)L.heads * up8(L.dim));
-        if (L.ff == PIE_FF_RELU2) {
+        if (L.conv_taps > 0 && b.n_runs < b.n_rows) hc = WA;
+        if (L.mixer == PIE_MIXER_MLSTM) ro = std::max(ro, (size_t)L.heads * up8(L.vdim)), rd = std::max(rd, (size_t)L.heads);
+        if (L.mixer == PIE_MIXER_DELTA || L.mixer == PIE_MIXER_MLSTM || L.mixer == PIE_MIXER_MINGRU) {
+            const int chunks = chunk_part(s, b, L).chunks;
+            if (chunks && L.mixer == PIE_MIXER_DELTA) rw = std::max(rw, delta_ws_floats(chunks, L.heads, L.dim)), ro = std::max(ro, (size_t)L.heads * up8(L.dim));
+            else if (chunks && L.mixer == PIE_MIXER_MLSTM) rw = std::max(rw, mlstm_ws_floats(chunks, L.heads, L.dim));
+            else if (chunks) rw = std::max(rw, mingru_ws_floats(chunks, L.dim));
+        }
+        if (is_dense(L)) {
             act = std::max(act, (size_t)act_stride(L.ff_size));
             if (plan.big) gemm(s->cfg.width, L.ff_size);
         }
@@ -413,11 +461,12 @@ int stack_reserve(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
     }
     bool moved = false;
     int rc = 0;
-    if ((rc = s->x.need(M * W64, &moved)) || (rc = s->c_raw.need(M * c, &moved)) || (rc = s->part.need(M * part, &moved)) || (rc = s->part_s.need(M * part_s, &moved)) ||
+    if ((rc = s->x.need(M * streams * W64, &moved)) || (rc = s->c_raw.need(M * c, &moved)) || (rc = s->part.need(M * part, &moved)) || (rc = s->part_s.need(M * part_s, &moved)) ||
         (rc = s->h.need(M * WA * E, &moved)) || (rc = s->q.need(M * q * E, &moved)) || (rc = s->ql.need(M * ql * E, &moved)) || (rc = s->oc.need(M * ql * E, &moved)) ||
         (rc = s->o.need(M * o * E, &moved)) || (rc = s->act.need(M * act * E, &moved)) || (rc = s->act_e.need(M * act_e * E, &moved)) ||
         (rc = s->act_s.need(M * act_s * E, &moved)) || (rc = s->stats.need((size_t)b.n_want * ST_TILES, &moved)) || (rc = s->y.need(plan.big ? M * W64 * E : 0, &moved)) ||
-        (rc = s->y32.need(plan.big ? 0 : M * W64, &moved)) || (rc = s->logits_e.need(M * le, &moved)) || (rc = s->delta_ws.need(dw, &moved)) || (rc = s->delta_o.need(M * dout, &moved)) || (rc = s->ctx.need(ctx * E, &moved)) ||
+        (rc = s->y32.need(plan.big ? 0 : M * W64, &moved)) || (rc = s->logits_e.need(M * le, &moved)) || (rc = s->rec_ws.need(rw, &moved)) || (rc = s->rec_o.need(M * ro, &moved)) ||
+        (rc = s->rec_den.need(M * rd, &moved)) || (rc = s->hc.need(M * hc * E, &moved)) || (rc = s->qu.need(M * qu * E, &moved)) || (rc = s->cq.need(M * cq * E, &moved)) || (rc = s->ctx.need(ctx * E, &moved)) ||
         (rc = s->kv.need(kv * E, &moved)) || (rc = s->gemm_ws.need(ws, &moved)))
         return rc;
     int n_moe = 0;
@@ -480,12 +529,19 @@ ShortPart short_part(const pie_stack *s, const pie_stack_batch &b, const Plan &p
 }
 // floats of key-split workspace a layer's attention needs
 size_t attn_ws(const pie_stack *s, const pie_stack_batch &b, const Plan &plan, const pie_stack_layer &L) {
-    if (L.mixer == PIE_MIXER_DELTA) return 0;
+    if (L.mixer != PIE_MIXER_LATENT && L.mixer != PIE_MIXER_ATTENTION) return 0;
     const ShortPart p = short_part(s, b, plan, L);
     if (!p.tiles) return 0;
     const int splits = plan_splits(b, L, p.tiles);
     return L.mixer == PIE_MIXER_ATTENTION ? page_attn_ws_floats(p.M, geometry(L), splits) : latent_attn_ws_floats(p.M, L.heads, L.rank, splits);
 }
+
+// what a sublayer's input is made of: the norm in front of it, with hyper-connections the streams' shares (nullptr: their sum), and the layer whose convolution follows (or -1)
+struct Into {
+    const pie_stack_norm *norm;
+    const float *in;
+    int conv;
+};
 
 struct Pass {
     pie_stack *s;
@@ -498,10 +554,48 @@ struct Pass {
         if (!rc)
             rc = w16l_gemm_launch(PIE_BF16, w, x, ldx, M, N, K, swiglu ? nullptr : y, s->gemm_ws.p, st, nullptr, swiglu ? y : nullptr, nullptr, ldy), ++launches;
     }
+    // the slots and runs a layer's state belongs to (at: its place in the state)
+    ConvArgs conv_args(int li, size_t at) const {
+        ConvArgs c = {};
+        c.pos = b.pos, c.row_seq = b.row_seq, c.slots = b.slots, c.n_seqs = b.n_seqs, c.n_slots = (int)b.n_slots, c.runs = (const RowRun *)b.runs, c.n_runs = b.n_runs;
+        if (b.states && b.states[li]) c.state = b.states[li] + at, c.slot_floats = state_layout(s, li).total;
+        return c;
+    }
+    // the streams take y = s->y (bf16; many rows) or s->y32 (hyper: the sublayer's connections), or start from the embedding (hyper null); h = the next sublayer's input
+    void streams(const float *hyper, const Into &next) {
+        if (rc) return;
+        const int W = s->cfg.width, WA = act_stride(W), S = s->cfg.streams;
+        StreamUpdateArgs a = {};
+        a.x = s->x.p, a.ldx = up64(W), a.S = S, a.in = next.in, a.next = row_norm_of(*next.norm), a.ldh = WA, a.M = b.n_rows, a.W = W, a.single = b.n_runs == b.n_rows;
+        ConvArgs conv = {};
+        if (next.conv >= 0) {
+            conv = conv_args(next.conv, state_layout(s, next.conv).conv);
+            conv.w = s->layers[next.conv].conv, conv.taps = s->layers[next.conv].conv_taps, conv.ldw = up64(W);
+        }
+        const bool behind = next.conv >= 0 && !a.single;  // the convolution has its own launch
+        if (hyper) {
+            a.y = plan.big ? (const void *)s->y.p : s->y32.p, a.y32 = !plan.big, a.ldy = plan.big ? W : up64(W), a.out = hyper + S, a.mix = hyper + 2 * S;
+            if (next.conv >= 0) a.conv = conv;
+        } else {
+            a.conv = next.conv >= 0 ? conv : conv_args(0, 0);
+            StackEmbed &e = a.embed;
+            e.ids = b.ids, e.table = (const u16 *)s->cfg.embed, e.scale = s->cfg.embed_scale, e.vocab = s->cfg.vocab;
+            e.positions = (const u16 *)s->cfg.positions, e.max_positions = s->cfg.max_positions;
+            e.bigram = (const u16 *)s->cfg.bigram, e.buckets = s->cfg.buckets, e.mul_prev = s->cfg.mul_prev, e.mul_cur = s->cfg.mul_cur;
+            if (e.bigram) e.prev = b.states[0] + state_layout(s, 0).prev;
+        }
+        a.h = behind ? s->hc.p : s->h.p;
+        rc = stream_update_launch(s->cfg.dtype, a, st), ++launches;
+        if (rc || !behind) return;
+        int tiles = 0;
+        for (int i = 0; i < b.n_runs; ++i) tiles += conv_tiles(b.runs_host[4 * i + 1]);
+        rc = conv_launch(s->cfg.dtype, conv, s->hc.p, s->h.p, WA, W, tiles, st), ++launches;
+    }
     // x += post(y); h = next(x) over y = s->y (bf16; many rows) or s->y32
     // route (few rows): the layer whose experts the rows choose on their way
-    void update(const pie_stack_norm &post, const pie_stack_norm &next, const u16 *bias = nullptr, int route = -1) {
+    void update(const pie_stack_norm &post, const Into &into, const u16 *bias = nullptr, int route = -1) {
         if (rc) return;
+        const pie_stack_norm &next = *into.norm;
         const int W = s->cfg.width, W64 = up64(W), WA = act_stride(W);
         if (plan.big && pointwise(post) && pointwise(next) && !bias) {
             hipLaunchKernelGGL(k_point_residual, dim3((unsigned)((W + 1023) / 1024), (unsigned)b.n_rows), dim3(256), 0, st, (const u16 *)s->y.p, W, norm_of(post), norm_of(next), s->x.p, W64,
@@ -516,35 +610,98 @@ struct Pass {
         }
         ++launches;
     }
-    // a sublayer's last product [W, K], its norm, the residual sum and the next sublayer's norm
-    void output(const void *w, const void *x, int ldx, int K, const pie_stack_norm &post, const pie_stack_norm &next, const u16 *bias = nullptr,
+    // a sublayer's last product [W, K], its norm, the residual sum and the next sublayer's norm; hyper (or null): its connections
+    void output(const void *w, const void *x, int ldx, int K, const pie_stack_norm &post, const Into &next, const float *hyper, const u16 *bias = nullptr,
                 int route = -1) {
         const int W = s->cfg.width, W64 = up64(W), WA = act_stride(W), M = b.n_rows;
         if (plan.big) {
             gemm(w, x, ldx, M, W, K, s->y.p, W);
-            return update(post, next, bias);
+            return hyper ? streams(hyper, next) : update(post, next, bias);
         }
         RowsArgs o = {};
         o.m = {(const char *)w, W, K, x, ldx, s->y32.p, W64};
         o.M = M;
-        if (pointwise(post) && pointwise(next) && !bias && route < 0) {
-            o.epi = ROWS_RESIDUAL, o.res = s->x.p, o.ld_res = W64, o.post = norm_of(post), o.next = norm_of(next), o.h = s->h.p, o.ldh = WA;
+        if (!hyper && pointwise(post) && pointwise(*next.norm) && !bias && route < 0) {
+            o.epi = ROWS_RESIDUAL, o.res = s->x.p, o.ld_res = W64, o.post = norm_of(post), o.next = norm_of(*next.norm), o.h = s->h.p, o.ldh = WA;
             return linear(o);
         }
         o.epi = ROWS_SCALE_F32, o.scale = 1.0f;
         linear(o);
-        update(post, next, bias, route);
+        if (hyper) streams(hyper, next);
+        else update(post, next, bias, route);
     }
     void linear(const RowsArgs &a, int batches = 1) {
         if (!rc) rc = rows_gemm_launch(s->cfg.dtype, a, batches, st), ++launches;
     }
 };
 
-void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm &next, int route) {
+// y = h . W^T in the stack's dtype
+void project(Pass &p, const void *w, int N, void *y) {
+    pie_stack *s = p.s;
+    const int W = s->cfg.width, WA = act_stride(W);
+    if (p.plan.big) return p.gemm(w, s->h.p, WA, p.b.n_rows, N, W, y, N);
+    RowsArgs a = {};
+    a.m = {(const char *)w, N, W, s->h.p, WA, y, N};
+    a.M = p.b.n_rows, a.epi = ROWS_STORE;
+    p.linear(a);
+}
+
+// where a pass's queries of a latent layer are: [M][ld], head h at h * D8; their rotated parts (rot_dim > 0) at q_rot, same row stride
+struct LatentQueries {
+    const void *q, *q_rot;
+    int ld;
+    HeadFinish finish;
+};
+// Attention and output of a latent layer whose latents are in their pages (append: not yet, few rows: they ride in the first launch)
+void latent_attend(Pass &p, int li, const pie_stack_layer &L, const LatentQueries &q, const LatentAppend *append, const Into &next, int route) {
     pie_stack *s = p.s;
     const pie_stack_batch &b = p.b;
-    const int W = s->cfg.width, W64 = up64(W), WA = act_stride(W), D8 = up8(L.dim), V8 = up8(L.vdim), R8 = up8(L.rank), H = L.heads, NI = H * D8 + R8, KO = H * V8, LO = act_stride(KO);
-    const int dt = s->cfg.dtype;
+    const int D8 = up8(L.dim), V8 = up8(L.vdim), R8 = up8(L.rank), T8 = up8(L.rot_dim), H = L.heads, KO = H * V8, LO = act_stride(KO), dt = s->cfg.dtype;
+    const void *slab = b.slabs[own_cache(L) ? li : L.kv_from];
+    const bool spell = p.plan.long_rows && spelled_out(L);
+    const ShortPart sp = short_part(s, b, p.plan, L);
+    const int M = sp.M, runs = sp.runs;
+    if (M > 0) {  // the latent form
+        RowsArgs k = {};
+        k.m = {(const char *)L.w_uk, L.rank, L.dim, q.q, q.ld, s->ql.p, H * R8};
+        k.M = M, k.epi = ROWS_STORE, k.w_batch = rows_weight_bytes(dt, L.rank, L.dim), k.x_batch = D8, k.y_batch = R8;
+        if (append) k.append = *append;
+        p.linear(k, H);
+        LatentAttnArgs t = {};
+        t.q = s->ql.p, t.ldq = R8, t.q_rot = q.q_rot, t.ld_rot = q.ld, t.finish = q.finish;
+        t.slab = slab, t.table = b.table, t.table_width = b.table_width, t.n_pages = (int)b.n_pages, t.n_seqs = b.n_seqs, t.pos = b.pos;
+        t.runs = (const RowRun *)b.runs, t.n_runs = runs, t.single = runs == M, t.row_seq = b.row_seq;
+        t.n_tiles = sp.tiles;
+        t.H = H, t.R = T8 ? R8 + T8 : L.rank, t.ldr = R8 + T8, t.M = M, t.window = L.window, t.scale = L.scale, t.splits = plan_splits(b, L, t.n_tiles), t.ws = s->attn_ws.p, t.out = s->oc.p;
+        const bool merge = t.splits > 1 && M <= MERGE_ROWS && R8 <= MERGE_LDR && dt == PIE_BF16 && R8 + T8 <= 1024;  // few rows: the next launch merges the key splits itself
+        t.combine = !merge;
+        if (!p.rc) p.rc = latent_attn_launch(dt, t, p.st), p.launches += t.splits > 1 && !merge ? 2 : 1;
+        RowsArgs v = {};
+        v.m = {(const char *)L.w_uv, L.vdim, L.rank, s->oc.p, H * R8, s->o.p, LO};
+        v.M = M, v.epi = ROWS_STORE, v.w_batch = rows_weight_bytes(dt, L.vdim, L.rank), v.x_batch = R8, v.y_batch = V8;
+        if (merge) v.merge = {s->attn_ws.p, t.splits, M, H, R8, q.finish};
+        p.linear(v, H);
+    }
+    if (spell && !p.rc) {
+        const RowRun *lr = (const RowRun *)b.runs + p.plan.short_runs;
+        const int n_long = b.n_runs - p.plan.short_runs, n_ctx = (int)plan_context(b, p.plan, L.window), nkv = H * (D8 + V8), LC = act_stride(R8 + T8);
+        p.rc = latent_gather_launch(lr, n_long, n_ctx, L.window, b.table, b.table_width, b.n_seqs, (int)b.n_pages, slab, R8 + T8, s->ctx.p, LC, p.st);
+        p.gemm(L.w_kv, s->ctx.p, LC, n_ctx, nkv, L.rank, s->kv.p, nkv);
+        WindowAttnArgs w = {};
+        w.q = (const u16 *)q.q, w.kv = (const u16 *)s->kv.p, w.out = (u16 *)s->o.p, w.ld_q = q.ld, w.ld_kv = nkv, w.ld_out = LO, w.H = H, w.D8 = D8, w.V8 = V8, w.window = L.window;
+        w.q_rot = (const u16 *)q.q_rot, w.k_rot = (const u16 *)s->ctx.p + R8, w.T8 = T8, w.ld_krot = LC, w.finish = q.finish, w.scale = L.scale, w.runs = lr, w.n_runs = n_long;
+        int tiles = 0;
+        for (int i = p.plan.short_runs; i < b.n_runs; ++i) tiles += (b.runs_host[4 * i + 1] + 127) / 128;
+        if (!p.rc) p.rc = window_attn_launch(w, tiles, p.st), p.launches += 2;
+    }
+    p.output(L.w_o, s->o.p, LO, KO, L.post1, next, L.hyper1, nullptr, route);
+}
+
+// queries straight from the layer's input
+void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next, int route) {
+    pie_stack *s = p.s;
+    const pie_stack_batch &b = p.b;
+    const int W = s->cfg.width, W64 = up64(W), WA = act_stride(W), D8 = up8(L.dim), R8 = up8(L.rank), H = L.heads, NI = H * D8 + R8;
     // many rows: q and the latents as two products where the tile rows allow it (together they are a little more than a round of workgroups)
     const bool two = p.plan.big && (H * D8) % 32 == 0;
     const int LQ = two ? H * D8 : NI;  // row stride of q
@@ -562,55 +719,38 @@ void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_nor
     if (p.rc) return;
     const LatentAppend append = {p.plan.big && !two ? (const void *)((const u16 *)s->q.p + H * D8) : s->c_raw.p, p.plan.big, p.plan.big && !two ? NI : R8, L.c_norm, L.eps, b.n_rows,
                                  L.rank, R8, b.pos, b.row_seq, b.table, b.table_width, (int)b.n_pages, b.n_seqs, b.slabs[li]};
-    if (p.plan.big) p.rc = latent_append_launch(dt, append, p.st), ++p.launches;  // (few rows: rides in the next launch)
-    const bool spell = p.plan.long_rows && spelled_out(L);
-    const ShortPart sp = short_part(s, b, p.plan, L);
-    const int M = sp.M, runs = sp.runs;
-    if (M > 0) {  // the latent form
-        RowsArgs k = {};
-        k.m = {(const char *)L.w_uk, L.rank, L.dim, s->q.p, LQ, s->ql.p, H * R8};
-        k.M = M, k.epi = ROWS_STORE, k.w_batch = rows_weight_bytes(dt, L.rank, L.dim), k.x_batch = D8, k.y_batch = R8;
-        if (!p.plan.big) k.append = append;
-        p.linear(k, H);
-        LatentAttnArgs t = {};
-        t.q = s->ql.p, t.slab = b.slabs[li], t.table = b.table, t.table_width = b.table_width, t.n_pages = (int)b.n_pages, t.n_seqs = b.n_seqs, t.pos = b.pos;
-        t.runs = (const RowRun *)b.runs, t.n_runs = runs, t.single = runs == M, t.row_seq = b.row_seq;
-        t.n_tiles = sp.tiles;
-        t.H = H, t.R = L.rank, t.ldr = R8, t.M = M, t.window = L.window, t.scale = L.scale, t.splits = plan_splits(b, L, t.n_tiles), t.ws = s->attn_ws.p, t.out = s->oc.p;
-        const bool merge = t.splits > 1 && M <= MERGE_ROWS && R8 <= MERGE_LDR && dt == PIE_BF16 && L.rank <= 1024;  // few rows: the next launch merges the key splits itself
-        t.combine = !merge;
-        if (!p.rc) p.rc = latent_attn_launch(dt, t, p.st), p.launches += t.splits > 1 && !merge ? 2 : 1;
-        RowsArgs v = {};
-        v.m = {(const char *)L.w_uv, L.vdim, L.rank, s->oc.p, H * R8, s->o.p, LO};
-        v.M = M, v.epi = ROWS_STORE, v.w_batch = rows_weight_bytes(dt, L.vdim, L.rank), v.x_batch = R8, v.y_batch = V8;
-        if (merge) v.merge = {s->attn_ws.p, t.splits, M, H, R8};
-        p.linear(v, H);
-    }
-    if (spell && !p.rc) {
-        const RowRun *lr = (const RowRun *)b.runs + p.plan.short_runs;
-        const int n_long = b.n_runs - p.plan.short_runs, n_ctx = (int)plan_context(b, p.plan, L.window), nkv = H * (D8 + V8), LC = act_stride(L.rank);
-        p.rc = latent_gather_launch(lr, n_long, n_ctx, L.window, b.table, b.table_width, b.n_seqs, (int)b.n_pages, b.slabs[li], R8, s->ctx.p, LC, p.st);
-        p.gemm(L.w_kv, s->ctx.p, LC, n_ctx, nkv, L.rank, s->kv.p, nkv);
-        WindowAttnArgs w = {(const u16 *)s->q.p, (const u16 *)s->kv.p, (u16 *)s->o.p, LQ, nkv, LO, H, D8, V8, L.window, L.scale, lr, n_long};
-        int tiles = 0;
-        for (int i = p.plan.short_runs; i < b.n_runs; ++i) tiles += (b.runs_host[4 * i + 1] + 127) / 128;
-        if (!p.rc) p.rc = window_attn_launch(w, tiles, p.st), p.launches += 2;
-    }
-    p.output(L.w_o, s->o.p, LO, KO, L.post1, next, nullptr, route);
+    if (p.plan.big) p.rc = latent_append_launch(s->cfg.dtype, append, p.st), ++p.launches;  // (few rows: rides in the next launch)
+    latent_attend(p, li, L, {s->q.p, nullptr, LQ, {}}, p.plan.big ? nullptr : &append, next, route);
 }
 
-// y = h . W^T in the stack's dtype
-void project(Pass &p, const void *w, int N, void *y) {
+// queries out of a latent of their own, with rotated parts
+void latent_query_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next, int route) {
     pie_stack *s = p.s;
-    const int W = s->cfg.width, WA = act_stride(W);
-    if (p.plan.big) return p.gemm(w, s->h.p, WA, p.b.n_rows, N, W, y, N);
-    RowsArgs a = {};
-    a.m = {(const char *)w, N, W, s->h.p, WA, y, N};
-    a.M = p.b.n_rows, a.epi = ROWS_STORE;
-    p.linear(a);
+    const pie_stack_batch &b = p.b;
+    const int D8 = up8(L.dim), T8 = up8(L.rot_dim), H = L.heads, NI = in_columns(L), NQ = H * (D8 + T8), CQ = act_stride(L.q_rank), dt = s->cfg.dtype;
+    project(p, L.w_in, NI, s->q.p);
+    if (p.rc) return;
+    LatentPrepArgs a = {};
+    a.raw = s->q.p, a.ld = NI, a.M = b.n_rows, a.Q = L.q_rank, a.Q8 = up8(L.q_rank), a.R = L.rank, a.R8 = up8(L.rank), a.T = L.rot_dim, a.T8 = T8;
+    a.q_norm = L.q_norm, a.c_norm = L.c_norm, a.eps = L.eps, a.rot = {L.rot_freq, L.rot_dims, L.rot_gain}, a.own = own_cache(L);
+    a.pos = b.pos, a.row_seq = b.row_seq, a.table = b.table, a.table_width = b.table_width, a.n_pages = (int)b.n_pages, a.n_seqs = b.n_seqs;
+    a.cq = s->cq.p, a.ldc = CQ, a.slab = b.slabs[li];
+    p.rc = latent_prep_launch(dt, a, p.st), ++p.launches;
+    if (p.plan.big) p.gemm(L.w_uq, s->cq.p, CQ, b.n_rows, NQ, L.q_rank, s->qu.p, NQ);
+    else {
+        RowsArgs u = {};
+        u.m = {(const char *)L.w_uq, NQ, L.q_rank, s->cq.p, CQ, s->qu.p, NQ};
+        u.M = b.n_rows, u.epi = ROWS_STORE;
+        p.linear(u);
+    }
+    if (p.rc) return;
+    char *q_rot = (char *)s->qu.p + (size_t)H * D8 * esize(s);
+    if (L.rot_dims > 0) p.rc = rotate_heads_launch(dt, {q_rot, NQ, T8, H, b.n_rows, {L.rot_freq, L.rot_dims, L.rot_gain}, b.pos}, p.st), ++p.launches;
+    const HeadFinish finish = {L.head_sink, L.out_gate ? (const char *)s->q.p + (size_t)(NI - up8(H)) * esize(s) : nullptr, NI};
+    latent_attend(p, li, L, {s->qu.p, q_rot, NQ, finish}, nullptr, next, route);
 }
 
-void attention_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm &next, int route) {
+void attention_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next, int route) {
     pie_stack *s = p.s;
     const pie_stack_batch &b = p.b;
     const int NI = in_columns(L), KO = out_columns(L), LO = act_stride(KO), dt = s->cfg.dtype;
@@ -640,10 +780,10 @@ void attention_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_
         for (int i = sp.runs; i < b.n_runs; ++i) a.n_tiles += page_attn_long_tiles(b.runs_host[4 * i + 1], geo);
         p.rc = page_attn_long_launch(a, p.st), ++p.launches;
     }
-    p.output(L.w_o, s->o.p, LO, KO, L.post1, next, (const u16 *)L.o_bias, route);
+    p.output(L.w_o, s->o.p, LO, KO, L.post1, next, L.hyper1, (const u16 *)L.o_bias, route);
 }
 
-void delta_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm &next, int route) {
+void delta_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next, int route) {
     pie_stack *s = p.s;
     const pie_stack_batch &b = p.b;
     const int NI = in_columns(L), KO = out_columns(L), LO = act_stride(KO);
@@ -653,30 +793,73 @@ void delta_mixer(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm
     d.raw = s->q.p, d.ld = NI, d.M = b.n_rows, d.H = L.heads, d.D = L.dim, d.D8 = up8(L.dim), d.rank = L.rank, d.R8 = up8(L.rank), d.bias = (const u16 *)L.in_bias;
     d.w_decay = (const u16 *)L.w_decay, d.decay_bias = L.decay_bias, d.o_norm = L.o_norm, d.decay_scale = L.decay_scale, d.unit_eps = L.unit_eps, d.eps = L.eps;
     d.pos = b.pos, d.row_seq = b.row_seq, d.slots = b.slots, d.n_seqs = b.n_seqs, d.n_slots = (int)b.n_slots, d.runs = (const RowRun *)b.runs, d.n_runs = b.n_runs;
-    d.state = b.states[li], d.out = s->o.p, d.ld_out = LO;
-    const DeltaPart dp = delta_part(b);
-    d.ws = s->delta_ws.p, d.o = s->delta_o.p, d.n_runs = dp.runs;
+    d.state = b.states[li], d.slot_floats = state_layout(s, li).total, d.out = s->o.p, d.ld_out = LO;
+    const ChunkPart dp = chunk_part(s, b, L);
+    d.ws = s->rec_ws.p, d.o = s->rec_o.p, d.n_runs = dp.runs;
     if (dp.runs) p.rc = delta_step_launch(s->cfg.dtype, d, p.st), ++p.launches;
     if (!p.rc && dp.chunks) {
         d.runs += dp.runs, d.n_runs = b.n_runs - dp.runs;
         p.rc = delta_chunks_launch(s->cfg.dtype, d, dp.chunks, dp.rows, b.n_rows - dp.rows, p.st), p.launches += delta_launches(dp.chunks, L.heads, L.dim);
     }
-    p.output(L.w_o, s->o.p, LO, KO, L.post1, next, nullptr, route);
+    p.output(L.w_o, s->o.p, LO, KO, L.post1, next, L.hyper1, nullptr, route);
 }
 
-void feed_forward(Pass &p, int li, const pie_stack_layer &L, const pie_stack_norm &next, bool routed) {  // routed: the experts have been chosen already
+RecurrentArgs recurrent_args(const Pass &p, int li, int ld) {
+    const pie_stack_batch &b = p.b;
+    return {p.s->q.p, ld, b.n_rows, b.pos, b.row_seq, b.slots, b.n_seqs, (int)b.n_slots, (const RowRun *)b.runs, b.n_runs, b.states[li], state_layout(p.s, li).total, p.s->rec_ws.p};
+}
+
+void mlstm_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next, int route) {
+    pie_stack *s = p.s;
+    const pie_stack_batch &b = p.b;
+    const int NI = in_columns(L), KO = out_columns(L), LO = act_stride(KO), D8 = up8(L.dim), V8 = up8(L.vdim), H = L.heads, dt = s->cfg.dtype;
+    project(p, L.w_in, NI, s->q.p);
+    if (p.rc) return;
+    MlstmArgs m = {recurrent_args(p, li, NI), L.gate_bias, H, L.dim, D8, L.vdim, V8, up8(H), L.scale, L.gate_cap, L.unit_eps, s->rec_o.p, s->rec_den.p};
+    const ChunkPart cp = chunk_part(s, b, L);
+    m.r.n_runs = cp.runs;
+    if (cp.runs) p.rc = mlstm_step_launch(dt, m, p.st), ++p.launches;
+    if (!p.rc && cp.chunks) {
+        m.r.runs += cp.runs, m.r.n_runs = b.n_runs - cp.runs;
+        p.rc = mlstm_chunks_launch(m, cp.chunks, p.st), p.launches += 2;
+    }
+    const HeadOutArgs h = {s->rec_o.p, s->rec_den.p, (const char *)s->q.p + (size_t)H * (2 * D8 + V8) * esize(s), nullptr, NI, H, L.vdim, V8, L.o_norm, L.eps, s->o.p, LO};
+    if (!p.rc) p.rc = head_out_launch(dt, h, 0, b.n_rows, p.st), ++p.launches;
+    p.output(L.w_o, s->o.p, LO, KO, L.post1, next, L.hyper1, nullptr, route);
+}
+
+void mingru_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next, int route) {
+    pie_stack *s = p.s;
+    const pie_stack_batch &b = p.b;
+    const int NI = in_columns(L), KO = out_columns(L), LO = act_stride(KO), dt = s->cfg.dtype;
+    project(p, L.w_in, NI, s->q.p);
+    if (p.rc) return;
+    MingruArgs m = {recurrent_args(p, li, NI), (const u16 *)L.in_bias, L.dim, up8(L.dim), s->o.p, LO};
+    const ChunkPart cp = chunk_part(s, b, L);
+    m.r.n_runs = cp.runs;
+    if (cp.runs) p.rc = mingru_step_launch(dt, m, p.st), ++p.launches;
+    if (!p.rc && cp.chunks) {
+        m.r.runs += cp.runs, m.r.n_runs = b.n_runs - cp.runs;
+        p.rc = mingru_chunks_launch(dt, m, cp.chunks, p.st), p.launches += 3;
+    }
+    p.output(L.w_o, s->o.p, LO, KO, L.post1, next, L.hyper1, nullptr, route);
+}
+
+void feed_forward(Pass &p, int li, const pie_stack_layer &L, const Into &into, bool routed) {  // routed: the experts have been chosen already
     pie_stack *s = p.s;
     const int M = p.b.n_rows, W = s->cfg.width, W64 = up64(W), WA = act_stride(W), F = L.ff_size, FA = act_stride(F), dt = s->cfg.dtype;
-    if (L.ff == PIE_FF_RELU2) {
+    const pie_stack_norm &next = *into.norm;
+    if (is_dense(L)) {
+        const bool relu = L.ff == PIE_FF_RELU2;
         if (p.plan.big) {
-            if (!p.rc) p.rc = w16l_relu2_launch(L.w_up, s->h.p, WA, M, F, W, s->act.p, FA, p.st), ++p.launches;
+            if (!p.rc) p.rc = w16l_act_launch(L.w_up, s->h.p, WA, M, F, W, s->act.p, FA, relu ? MFMA_ACT_RELU2 : MFMA_ACT_XIELU, L.act_alpha, L.act_beta, p.st), ++p.launches;
         } else {
             RowsArgs u = {};
             u.m = {(const char *)L.w_up, F, W, s->h.p, WA, s->act.p, FA};
-            u.M = M, u.epi = ROWS_RELU2;
+            u.M = M, u.epi = relu ? ROWS_RELU2 : ROWS_XIELU, u.act_alpha = L.act_alpha, u.act_limit = L.act_beta;
             p.linear(u);
         }
-        return p.output(L.w_down, s->act.p, FA, F, L.post2, next);
+        return p.output(L.w_down, s->act.p, FA, F, L.post2, into, L.hyper2);
     }
     const RouteLayer &r = s->route[li];
     const int S = L.shared_size, SA = act_stride(S);
@@ -749,31 +932,44 @@ int stack_enqueue(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
         PIE_LAUNCH_CHECK();
         ++p.launches;
     }
-    const pie_stack_norm &fin = s->cfg.final_norm, &first = n ? s->layers[0].pre1 : fin;
+    // what sublayer 1 of layer i (n: the final norm) takes in, and sublayer 2
+    const int S = s->cfg.streams;
+    auto mixer_in = [&](int i) -> Into {
+        if (i >= n) return {&s->cfg.final_norm, nullptr, -1};
+        return {&s->layers[i].pre1, s->layers[i].hyper1, s->layers[i].conv_taps > 0 ? i : -1};
+    };
+    const pie_stack_norm &first = *mixer_in(0).norm;
     const dim3 ge((unsigned)((W + 1023) / 1024), (unsigned)M);
-    if (dt == PIE_F32)
+    if (S) p.streams(nullptr, mixer_in(0));
+    else if (dt == PIE_F32)
         hipLaunchKernelGGL(k_stack_embed<ElemF32>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, s->cfg.embed_scale, !pointwise(first), norm_of(first), s->x.p, W64,
                            (float *)s->h.p, WA);
     else
         hipLaunchKernelGGL(k_stack_embed<ElemBF16>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, s->cfg.embed_scale, !pointwise(first), norm_of(first), s->x.p, W64,
                            (u16 *)s->h.p, WA);
     PIE_LAUNCH_CHECK();
-    ++p.launches;
-    if (first.kind == PIE_NORM_RMS) {
+    p.launches += !S;
+    if (!S && first.kind == PIE_NORM_RMS) {
         RowUpdateArgs a = {};
         a.next = row_norm_of(first), a.x = s->x.p, a.ldx = W64, a.h = s->h.p, a.ldh = WA, a.M = M, a.W = W;
         p.rc = row_update_launch(dt, a, st), ++p.launches;
     }
     for (int i = 0; i < n && !p.rc; ++i) {
         const pie_stack_layer &L = s->layers[i];
-        const pie_stack_norm &after = i + 1 < n ? s->layers[i + 1].pre1 : fin, &next = L.ff == PIE_FF_NONE ? after : L.pre2;
+        const Into after = mixer_in(i + 1), next = L.ff == PIE_FF_NONE ? after : Into{&L.pre2, L.hyper2, -1};
         // some rows: the launch that makes the router's input also chooses the experts (for very few rows, spreading the router over the chip takes less time)
         const bool routed = L.ff == PIE_FF_ROUTED_MOE && !plan.big && L.w_router_rows && M >= ROUTE_MIN_ROWS && M <= ROUTE_FEW_ROWS && (long)L.experts * W <= ROUTE_FEW_WEIGHTS && W <= 8192;
-        if (L.mixer == PIE_MIXER_LATENT) latent_mixer(p, i, L, next, routed ? i : -1);
-        else if (L.mixer == PIE_MIXER_ATTENTION) attention_mixer(p, i, L, next, routed ? i : -1);
-        else delta_mixer(p, i, L, next, routed ? i : -1);
+        const int route = routed ? i : -1;
+        switch (L.mixer) {
+            case PIE_MIXER_LATENT: L.q_rank ? latent_query_mixer(p, i, L, next, route) : latent_mixer(p, i, L, next, route); break;
+            case PIE_MIXER_ATTENTION: attention_mixer(p, i, L, next, route); break;
+            case PIE_MIXER_DELTA: delta_mixer(p, i, L, next, route); break;
+            case PIE_MIXER_MLSTM: mlstm_mixer(p, i, L, next, route); break;
+            default: mingru_mixer(p, i, L, next, route); break;
+        }
         if (L.ff != PIE_FF_NONE && !p.rc) feed_forward(p, i, L, after, routed);
-        if (b.tap && !p.rc)
+        if (b.tap && !p.rc && S) p.rc = stream_sum_launch(s->x.p, W64, S, b.tap + (size_t)i * M * W, M, W, st);
+        else if (b.tap && !p.rc)
             PIE_HIP_TRY(hipMemcpy2DAsync(b.tap + (size_t)i * M * W, (size_t)W * 4, s->x.p, (size_t)W64 * 4, (size_t)W * 4, (size_t)M, hipMemcpyDeviceToDevice, st));
     }
     if (b.n_want > 0) {
@@ -800,8 +996,17 @@ bool norm_ok(const pie_stack_norm &n) {
 int mixer_ok(const pie_stack *s, int i, const pie_stack_layer &L) {
     PIE_REQUIRE(L.heads > 0 && L.dim > 0 && L.w_in && L.w_o && norm_ok(L.pre1) && norm_ok(L.post1), PIE_E_ARG, "pie_stack_set_layer: missing mixer weights or sizes");
     if (L.mixer == PIE_MIXER_LATENT) {
-        PIE_REQUIRE(L.vdim > 0 && L.rank > 0 && L.rank <= 2048, PIE_E_SHAPE, "pie_stack_set_layer: bad mixer sizes (kv_rank at most 2048)");
-        PIE_REQUIRE(L.w_uk && L.w_uv && L.c_norm, PIE_E_ARG, "pie_stack_set_layer: missing mixer weights");
+        PIE_REQUIRE(L.vdim > 0 && L.rank > 0 && L.q_rank >= 0 && L.rot_dim >= 0 && latent_row(L) <= 2048, PIE_E_SHAPE, "pie_stack_set_layer: bad mixer sizes (kv_rank + rot_dim at most 2048)");
+        PIE_REQUIRE(L.w_uk && L.w_uv && (L.c_norm || !own_cache(L)), PIE_E_ARG, "pie_stack_set_layer: missing mixer weights");
+        PIE_REQUIRE(L.q_rank ? L.w_uq && L.q_norm : !L.rot_dim && !L.out_gate && !L.head_sink, PIE_E_ARG,
+                    "pie_stack_set_layer: rotation, gate and sink of latent attention go with a query latent, which needs its weights");
+        PIE_REQUIRE(L.rot_dims >= 0 && L.rot_dims <= L.rot_dim && L.rot_dims % 2 == 0 && (L.rot_dims == 0 || L.rot_freq), PIE_E_SHAPE, "pie_stack_set_layer: bad rotation");
+        if (!own_cache(L)) {
+            PIE_REQUIRE(L.kv_from < i && s->have[L.kv_from], PIE_E_ARG, "pie_stack_set_layer: kv_from names an earlier layer");
+            const pie_stack_layer &F = s->layers[L.kv_from];
+            PIE_REQUIRE(F.mixer == PIE_MIXER_LATENT && own_cache(F) && F.rank == L.rank && F.rot_dim == L.rot_dim, PIE_E_SHAPE,
+                        "pie_stack_set_layer: kv_from names a latent layer with a cache of its own, of the same sizes");
+        }
     } else if (L.mixer == PIE_MIXER_ATTENTION) {
         PIE_REQUIRE(L.vdim > 0 && L.kv_heads > 0 && L.heads % L.kv_heads == 0 && L.dim <= PAGE_ATTN_ROWS_DIM && L.vdim <= PAGE_ATTN_ROWS_DIM, PIE_E_SHAPE,
                     "pie_stack_set_layer: bad mixer sizes (heads of at most 1024 numbers, a multiple of kv_heads)");
@@ -816,7 +1021,17 @@ int mixer_ok(const pie_stack *s, int i, const pie_stack_layer &L) {
         PIE_REQUIRE(L.dim <= DELTA_MAX_DIM && L.rank > 0 && L.rank <= DELTA_MAX_RANK, PIE_E_SHAPE, "pie_stack_set_layer: bad mixer sizes (delta rule: dim at most 256, rank at most 1024)");
         PIE_REQUIRE(L.w_decay && L.decay_bias && L.o_norm, PIE_E_ARG, "pie_stack_set_layer: missing mixer weights");
         PIE_REQUIRE(L.decay_scale >= 0 && L.decay_scale <= DELTA_MAX_DECAY, PIE_E_ARG, "pie_stack_set_layer: decay_scale must be in [0, 2] (the chunk form divides by sixteen decays)");
+    } else if (L.mixer == PIE_MIXER_MLSTM) {
+        PIE_REQUIRE(L.vdim > 0 && L.dim <= MLSTM_MAX_DIM && L.vdim <= HEAD_OUT_MAX_DIM && L.gate_cap > 0, PIE_E_SHAPE, "pie_stack_set_layer: bad mixer sizes (mLSTM: dim at most 1024, vdim at most 2048)");
+        PIE_REQUIRE(L.gate_bias && L.o_norm, PIE_E_ARG, "pie_stack_set_layer: missing mixer weights");
+    } else if (L.mixer == PIE_MIXER_MINGRU) {
+        PIE_REQUIRE(L.heads == 1, PIE_E_SHAPE, "pie_stack_set_layer: a minGRU has one head");
     } else PIE_REQUIRE(false, PIE_E_ARG, "pie_stack_set_layer: unknown mixer");
+    if (s->cfg.streams) {
+        PIE_REQUIRE(L.hyper1 && (L.ff == PIE_FF_NONE || L.hyper2) && L.post1.kind == PIE_NORM_NONE && (L.ff == PIE_FF_NONE || L.post2.kind == PIE_NORM_NONE) && !is_moe(L) && !L.o_bias, PIE_E_ARG,
+                    "pie_stack_set_layer: hyper-connections need their weights, dense feed-forwards, and neither norms nor biases behind the sublayers");
+        PIE_REQUIRE(L.conv_taps >= 0 && L.conv_taps <= CONV_MAX_TAPS && (!L.conv_taps || L.conv), PIE_E_SHAPE, "pie_stack_set_layer: a convolution of 1 .. 16 taps, with its weights");
+    } else PIE_REQUIRE(!L.hyper1 && !L.hyper2 && !L.conv_taps, PIE_E_ARG, "pie_stack_set_layer: hyper-connections and convolutions go with several streams");
     return PIE_OK;
 }
 
@@ -829,6 +1044,9 @@ int pie_stack_create(const pie_stack_config *cfg, pie_stack **out) {
     PIE_REQUIRE(cfg->dtype == PIE_BF16 || cfg->dtype == PIE_F32, PIE_E_ARG, "pie_stack_create: dtype must be PIE_BF16 or PIE_F32");
     PIE_REQUIRE(cfg->width > 0 && cfg->vocab > 0 && cfg->n_layers >= 0, PIE_E_SHAPE, "pie_stack_create: bad sizes");
     PIE_REQUIRE(cfg->embed && cfg->head && norm_ok(cfg->final_norm), PIE_E_ARG, "pie_stack_create: missing weights");
+    PIE_REQUIRE(cfg->streams >= 0 && cfg->streams <= STREAMS_MAX && (cfg->streams == 0 || cfg->width <= ROW_UPDATE_MAX_WIDTH), PIE_E_SHAPE, "pie_stack_create: at most 16 streams, of at most 32768 numbers");
+    PIE_REQUIRE((!cfg->positions && !cfg->bigram) || (cfg->streams > 0 && (!cfg->positions || cfg->max_positions > 0) && (!cfg->bigram || (cfg->buckets > 0 && cfg->n_layers > 0))), PIE_E_ARG,
+                "pie_stack_create: position and bigram vectors go with streams, and need their sizes");
     pie_stack *s = new (std::nothrow) pie_stack();
     PIE_REQUIRE(s, PIE_E_HIP, "pie_stack_create: out of host memory");
     s->cfg = *cfg;
@@ -846,7 +1064,7 @@ int pie_stack_set_layer(pie_stack *s, int i, const pie_stack_layer *L) {
     PIE_REQUIRE(s && L && i >= 0 && i < s->cfg.n_layers, PIE_E_ARG, "pie_stack_set_layer: bad argument");
     if (const int rc = mixer_ok(s, i, *L)) return rc;
     PIE_REQUIRE(L->ff == PIE_FF_NONE || (norm_ok(L->pre2) && norm_ok(L->post2) && L->ff_size > 0 && L->ff_size % 8 == 0 && L->shared_size % 8 == 0), PIE_E_ARG, "pie_stack_set_layer: missing feed-forward norms");
-    if (L->ff == PIE_FF_RELU2) PIE_REQUIRE(L->w_up && L->w_down, PIE_E_ARG, "pie_stack_set_layer: missing dense weights");
+    if (is_dense(*L)) PIE_REQUIRE(L->w_up && L->w_down, PIE_E_ARG, "pie_stack_set_layer: missing dense weights");
     else if (is_moe(*L)) {
         PIE_REQUIRE(L->experts > 0 && L->experts <= 8192 && L->top > 0 && L->top <= L->experts, PIE_E_SHAPE, "pie_stack_set_layer: bad expert counts");
         PIE_REQUIRE((L->ff == PIE_FF_TABLE_MOE ? L->table != nullptr : L->w_router && L->correction) && L->w_gate_up && L->w_expert_down, PIE_E_ARG, "pie_stack_set_layer: missing expert weights");
@@ -876,11 +1094,11 @@ int pie_logprobs_argmax_f32(const float *logits, int rows, int V, float *logprob
 int pie_stack_page_row(const pie_stack *s, int i) {
     if (!s || i < 0 || i >= s->cfg.n_layers || !s->have[i]) return 0;
     const pie_stack_layer &L = s->layers[i];
-    if (L.mixer == PIE_MIXER_LATENT) return up8(L.rank);
-    return L.mixer == PIE_MIXER_ATTENTION && L.kv_from < 0 ? (int)(geometry(L).page_elems() / PAGE_TOKENS) : 0;
+    if (!own_cache(L)) return 0;
+    return L.mixer == PIE_MIXER_LATENT ? latent_row(L) : (int)(geometry(L).page_elems() / PAGE_TOKENS);
 }
 size_t pie_stack_state_floats(const pie_stack *s, int i) {
-    return s && i >= 0 && i < s->cfg.n_layers && s->have[i] && s->layers[i].mixer == PIE_MIXER_DELTA ? (size_t)s->layers[i].heads * s->layers[i].dim * s->layers[i].dim : 0;
+    return s && i >= 0 && i < s->cfg.n_layers && s->have[i] ? state_layout(s, i).total : 0;
 }
 size_t pie_stack_page_bytes(const pie_stack *s, int i) { return (size_t)pie_stack_page_row(s, i) * PAGE_TOKENS * (s ? esize(s) : 0); }
 int pie_stack_launches(const pie_stack *s) { return s ? s->launches : 0; }

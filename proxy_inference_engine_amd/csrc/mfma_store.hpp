@@ -8,6 +8,7 @@
 // conflict-free both ways -- and leaves as 16 bytes per lane, 8 (or 4) lanes per row.
 #pragma once
 #include "prefill_attn.hpp"  // f32x16_t, the 16-bit traits
+#include "stack_types.hpp"   // xielu
 
 // two fp32 -> one packed pair of T in a single v_cvt_pk_* (pack2<T> converts each half separately and ORs them: 3 instructions)
 template <class T>
@@ -32,11 +33,16 @@ __device__ __forceinline__ u32 w4m_pack<F16>(float lo, float hi) {
 // ACT: MFMA_ACT_NONE, MFMA_ACT_SWIGLU (the bool true of the kernels that know only that one), MFMA_ACT_RELU2 (max(T(v), 0)^2, taken where the tile leaves LDS: next to
 // the accumulators it does not fit the registers), MFMA_ACT_CLIPPED (columns paired as for SWIGLU: g sigmoid(alpha g) (u + 1) with g = min(gate, limit),
 // u = clamp(up, +-limit) of the rounded pair).
-enum { MFMA_ACT_NONE = 0, MFMA_ACT_SWIGLU = 1, MFMA_ACT_RELU2 = 2, MFMA_ACT_CLIPPED = 3 };
+// MFMA_ACT_XIELU: of the rounded value, like RELU2 on the way out of LDS (act_alpha, act_limit: its two factors).
+enum { MFMA_ACT_NONE = 0, MFMA_ACT_SWIGLU = 1, MFMA_ACT_RELU2 = 2, MFMA_ACT_CLIPPED = 3, MFMA_ACT_XIELU = 4 };
 template <class T>
 __device__ __forceinline__ u32 mfma_relu2(u32 w) {
     const float a = fmaxf(lo_f32<T>(w), 0.0f), b = fmaxf(hi_f32<T>(w), 0.0f);
     return w4m_pack<T>(a * a, b * b);
+}
+template <class T>
+__device__ __forceinline__ u32 mfma_xielu(u32 w, float up, float down) {
+    return w4m_pack<T>(xielu<false>(lo_f32<T>(w), up, down), xielu<false>(hi_f32<T>(w), up, down));
 }
 template <class T, int MB, int SW, int ACT>
 __device__ __forceinline__ void mfma_tile_store(const f32x16_t (&acc)[SW][MB], char *ot, int lane, int nt0, int m0, int rows, int N, int ldy, u16 *y,
@@ -97,6 +103,9 @@ __device__ __forceinline__ void mfma_tile_store(const f32x16_t (&acc)[SW][MB], c
         uint2 lo = *reinterpret_cast<const uint2 *>(ot + r * OB + (((2 * j) ^ rsv) << 3));
         uint2 hi = *reinterpret_cast<const uint2 *>(ot + r * OB + (((2 * j + 1) ^ rsv) << 3));
         if constexpr (ACT == MFMA_ACT_RELU2) lo = make_uint2(mfma_relu2<T>(lo.x), mfma_relu2<T>(lo.y)), hi = make_uint2(mfma_relu2<T>(hi.x), mfma_relu2<T>(hi.y));
+        if constexpr (ACT == MFMA_ACT_XIELU)
+            lo = make_uint2(mfma_xielu<T>(lo.x, act_alpha, act_limit), mfma_xielu<T>(lo.y, act_alpha, act_limit)),
+            hi = make_uint2(mfma_xielu<T>(hi.x, act_alpha, act_limit), mfma_xielu<T>(hi.y, act_alpha, act_limit));
         const int col = c0 + 8 * j;
         if (r >= rows || col >= ldo || skip_stores) continue;
         u16 *dst = y + (size_t)(m0 + r) * ldy + col;

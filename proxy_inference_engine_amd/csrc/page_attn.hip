@@ -20,16 +20,6 @@ namespace {
 constexpr float PG_NEG = -1e30f, PG_LOG2E = 1.44269504088896340736f;
 
 // ---------------------------------------------------------------- projections -> queries, pages
-// sin and cos of an angle: the library's in fp32 stacks; else reduced to one turn in two steps, then the trigonometric unit (absolute error about 1e-6)
-template <bool F32>
-__device__ __forceinline__ void pg_sincos(float a, float &s, float &c) {
-    if constexpr (F32) sincosf(a, &s, &c);
-    else {
-        const float n = rintf(a * 0.15915494309189533577f), r = fmaf(n, 1.7484556e-7f, fmaf(n, -6.2831855f, a)) * 0.15915494309189533577f;  // (6.2831855f is 2 pi + 1.7484556e-7)
-        s = __builtin_amdgcn_sinf(r), c = __builtin_amdgcn_cosf(r);
-    }
-}
-
 // One wave per row and run of HB heads of one kind (queries, keys or values).  Lane l holds the dimension pairs l, l + 64, ... of a head; angles and places in a
 // page are taken once for all heads of the wave.  NP: pairs per lane.
 template <class E, int NP, int HB>
@@ -77,7 +67,7 @@ __global__ void __launch_bounds__(256) k_kv_prep(const KvPrepArgs a) {
         sn[j] = 0.0f, cs[j] = 1.0f, wu[j] = wv[j] = 1.0f;
         if (w) wu[j] = w[min(d, n - 1)], wv[j] = w[min(d + 1, n - 1)];
         if (!is_v && d + 1 < a.rot_dims) {
-            pg_sincos<F32>((float)t * a.freq[d >> 1], sn[j], cs[j]);
+            stack_sincos<F32>((float)t * a.freq[d >> 1], sn[j], cs[j]);
             sn[j] *= a.rot_gain, cs[j] *= a.rot_gain;
         }
         place[j] = is_q ? d : is_v ? geo.value(tl, d) : geo.key(tl, d), place1[j] = is_v ? geo.value(tl, d + 1) : 0;

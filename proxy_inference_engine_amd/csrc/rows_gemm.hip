@@ -60,6 +60,7 @@ __device__ __forceinline__ void rows_finish(const RowsArgs &a, const RowsWork &k
             ((T *)k.y)[row * k.ldy + n] = E::pack(r * r);
             break;
         }
+        case ROWS_XIELU: ((T *)k.y)[row * k.ldy + n] = E::pack(xielu<sizeof(T) == 4>(v, a.act_alpha, a.act_limit)); break;
         case ROWS_SILU_MUL:
             if (!(n & 1)) ((T *)k.y)[row * k.ldy + (n >> 1)] = E::pack(v / (1.0f + expf(-v)) * pair);
             break;

@@ -1,6 +1,6 @@
 // stack_types.hpp -- what the kernels of the layer-stack models share: the element types, the norms that ride in epilogues, and the operand
-// descriptions of the row-wise Linear (rows_gemm.hip), the attentions (latent_attn.hip, window_attn.hip, page_attn.hip), the recurrence (delta_rule.hip) and
-// the row norms (row_update.hip).
+// descriptions of the row-wise Linear (rows_gemm.hip), the attentions (latent_attn.hip, window_attn.hip, page_attn.hip), the recurrences (delta_rule.hip, mlstm.hip,
+// mingru.hip) and what stands between sublayers (row_update.hip, stream_update.hip).
 //
 // Every activation row has a stride that is a multiple of 8 elements (act_stride(), or packed); a Linear reads 64 ceil(K / 64) elements of it.  The columns past K meet zero
 // weights, so they only have to be finite: the owner zero-fills its buffers once and keeps 64 elements of slack behind each.
@@ -45,6 +45,36 @@ __device__ __forceinline__ float4 point_norm4(const PointNorm &n, int i, float4 
     const float4 w = *(const float4 *)(n.w + i), b = *(const float4 *)(n.b + i);
     return make_float4(fmaf(fast_tanh(n.alpha * x.x), w.x, b.x), fmaf(fast_tanh(n.alpha * x.y), w.y, b.y), fmaf(fast_tanh(n.alpha * x.z), w.z, b.z),
                        fmaf(fast_tanh(n.alpha * x.w), w.w, b.w));
+}
+
+// exp(x) and 1 / (1 + exp(-x)): fp32 stacks take the library's, 16-bit ones the exponential unit (a few units in the last place)
+constexpr float STACK_LOG2E = 1.44269504088896340736f;
+template <bool F32>
+__device__ __forceinline__ float stack_exp(float x) {
+    return F32 ? expf(x) : __builtin_amdgcn_exp2f(x * STACK_LOG2E);
+}
+template <bool F32>
+__device__ __forceinline__ float stack_sigmoid(float x) {
+    return F32 ? 1.0f / (1.0f + expf(-x)) : __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(x * -STACK_LOG2E));
+}
+
+// sin and cos of an angle: the library's in fp32 stacks; else reduced to one turn in two steps, then the trigonometric unit (absolute error about 1e-6)
+template <bool F32>
+__device__ __forceinline__ void stack_sincos(float a, float &s, float &c) {
+    if constexpr (F32) sincosf(a, &s, &c);
+    else {
+        const float n = rintf(a * 0.15915494309189533577f), r = fmaf(n, 1.7484556e-7f, fmaf(n, -6.2831855f, a)) * 0.15915494309189533577f;  // (6.2831855f is 2 pi + 1.7484556e-7)
+        s = __builtin_amdgcn_sinf(r), c = __builtin_amdgcn_cosf(r);
+    }
+}
+
+// up z^2 + z / 2 for z > 0, down (e^z - 1 - z) + z / 2 for z <= 0 (xIELU); e^z - 1 - z by its series near zero, where the difference would cancel
+template <bool F32>
+__device__ __forceinline__ float xielu(float z, float up, float down) {
+    const float n = fminf(z, 0.0f);
+    const float series = 0.5f * n * n * fmaf(n * (1.0f / 3.0f), fmaf(n * 0.25f, fmaf(n * 0.2f, fmaf(n * (1.0f / 6.0f), fmaf(n * (1.0f / 7.0f), 1.0f, 1.0f), 1.0f), 1.0f), 1.0f), 1.0f);
+    const float g = n > -0.25f ? series : stack_exp<F32>(n) - 1.0f - n;
+    return fmaf(0.5f, z, z > 0.0f ? up * z * z : down * g);
 }
 
 // sum / maximum over the wave without LDS, in every lane
@@ -94,9 +124,23 @@ __device__ __forceinline__ void latent_append_row(const LatentAppend &a, int m, 
 // ---------------------------------------------------------------- the attention's key splits
 // ws: sums [splits][M * H][ldr] fp32, then (maximum, sum of weights) [splits][M * H][2]; a split that saw no key has weight sum 0 and no sums
 constexpr int MERGE_ROWS = 4, MERGE_LDR = 1024;
+// what a head's sums are finished with: fp32 [H] a sink score in the denominator (nullable), [M][ldg] gate logits in the stack's dtype (nullable)
+struct HeadFinish {
+    const float *sink;
+    const void *gate;
+    int ldg;
+};
+template <bool F32>
+__device__ __forceinline__ float head_gate(const HeadFinish &f, size_t row, int head) {
+    if (!f.gate) return 1.0f;
+    return 1.0f / (1.0f + expf(-(F32 ? ((const float *)f.gate)[row * f.ldg + head] : BF16::to_f32(((const u16 *)f.gate)[row * f.ldg + head]))));
+}
+// the sink's share of a denominator whose weights are relative to the exponent m (base 2)
+__device__ __forceinline__ float head_sink2(const HeadFinish &f, int head, float m) { return f.sink ? __builtin_amdgcn_exp2f(f.sink[head] * STACK_LOG2E - m) : 0.0f; }
 struct LatentMerge {
     const float *ws;
     int splits, M, H, ldr;
+    HeadFinish finish;
 };
 // lane s: what split s of pair pr counts in the merged result (base 2 exponents; at most 64 splits)
 __device__ __forceinline__ float latent_split_weight(const LatentMerge &a, size_t pr, int lane) {
@@ -104,7 +148,7 @@ __device__ __forceinline__ float latent_split_weight(const LatentMerge &a, size_
     const float2 ml = lane < a.splits ? *(const float2 *)(a.ws + (size_t)a.splits * MH * a.ldr + (lane * MH + pr) * 2) : make_float2(-1e30f, 0.0f);
     const float m = wave_max(ml.y > 0.0f ? ml.x : -1e30f);
     const float f = ml.y > 0.0f ? __builtin_amdgcn_exp2f(ml.x - m) : 0.0f;
-    return f / wave_sum(ml.y * f);
+    return f * head_gate<false>(a.finish, pr / a.H, (int)(pr % a.H)) / (wave_sum(ml.y * f) + head_sink2(a.finish, (int)(pr % a.H), m));
 }
 // columns r .. r + 3 of the merged sums of pair pr, eight splits in flight; weight(s): a wave-uniform or per-thread read of split s's weight
 template <class F>
@@ -136,6 +180,7 @@ enum RowsEpi {
     ROWS_SPLIT = 4,      // n < split: y[m][n] = T(v);  else y2[m][n - split] = v, fp32
     ROWS_RESIDUAL = 5,   // x[m][n] += post(v);  h[m][n] = T(next(x[m][n]))
     ROWS_CLIP_MUL = 6,   // rows (2 i, 2 i + 1) = (gate_i, up_i): y[m][i] = T(clipped_glu(gate, up))
+    ROWS_XIELU = 7,      // y[m][n] = T(xielu(v))
 };
 // g sigmoid(alpha g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit)
 __device__ __forceinline__ float clipped_glu(float gate, float up, float alpha, float limit) {
@@ -164,7 +209,7 @@ struct RowsArgs {
     const int *rows;       // ungrouped, nullable: x row of result row i
     int epi;
     float scale;
-    float act_alpha, act_limit;  // ROWS_CLIP_MUL
+    float act_alpha, act_limit;  // ROWS_CLIP_MUL; ROWS_XIELU: its two factors
     int split;
     float *y2;
     int ldy2;
@@ -188,8 +233,10 @@ struct RowRun {
     int row0, n_rows, seq, pos0;  // seq: row of the block table; pos0: position of row0 (single rows: not used, may be 0)
 };
 struct LatentAttnArgs {
-    const void *q;         // [M][H][ldr]: queries in the latent space (W_uk^T q), ldr = row stride in elements
-    const void *slab;      // the layer's latent pages [n_pages][64][ldr]
+    const void *q;         // [M][H][ldq]: queries in the latent space (W_uk^T q), ldq = row stride in elements
+    const void *q_rot;     // nullable: [M][ld_rot], head h at h * (ldr - ldq): what meets the numbers of a cached row behind the latent
+    int ldq, ld_rot;
+    const void *slab;      // the layer's latent pages [n_pages][64][ldr]: the latent [ldq], and what scores read beside it
     const int *table;      // [n_seqs][table_width] page ids
     int table_width, n_pages, n_seqs;
     const int *pos;        // [M]
@@ -197,18 +244,49 @@ struct LatentAttnArgs {
     int n_runs, n_tiles;   // n_tiles = sum over the runs of latent_attn_tiles()
     bool single;           // every run is one row (a decode step): tile -> run without a search
     const int *row_seq;    // [M]
-    int H, R, ldr, M;
+    int H, R, ldr, M;      // R: numbers of a row that scores read
+    HeadFinish finish;
     int window;            // keys j with 0 <= i - j < window; <= 0: no limit
     float scale;
     int splits;            // > 1: fp32 partials in ws, merged by the combine launch (combine = false: left to the consumer)
     bool combine;
     float *ws;             // see LatentMerge
-    void *out;             // [M][H][ldr] T: softmax-weighted latents
+    void *out;             // [M][H][ldq] T: softmax-weighted latents
 };
 int latent_attn_launch(int dtype, const LatentAttnArgs &a, hipStream_t st);
 int latent_attn_tiles(int n_rows, int H);
 size_t latent_attn_ws_floats(int M, int H, int R, int splits);
 int latent_append_launch(int dtype, const LatentAppend &a, hipStream_t st);
+
+// rotation in halves: number i of a vector with number i + dims / 2, by position * freq[i], cos and sin times gain; what lies behind dims stays
+struct Rotation {
+    const float *freq;
+    int dims;
+    float gain;
+};
+// one row's projections -> its normed query latent, and (own) its normed latent and rotated key part into the page
+struct LatentPrepArgs {
+    const void *raw;       // [M][ld] T: query latent [Q8], latent [R8], key part [T8]
+    int ld, M, Q, Q8, R, R8, T, T8;
+    const float *q_norm, *c_norm;
+    float eps;
+    Rotation rot;
+    bool own;
+    const int *pos, *row_seq, *table;
+    int table_width, n_pages, n_seqs;
+    void *cq;              // [M][ldc] T
+    int ldc;
+    void *slab;            // [n_pages][64][R8 + T8]
+};
+int latent_prep_launch(int dtype, const LatentPrepArgs &a, hipStream_t st);
+// the heads' vectors of every row, in place: row m, head h at q + m * ld + h * stride
+struct RotateArgs {
+    void *q;
+    int ld, stride, H, M;
+    Rotation rot;
+    const int *pos;
+};
+int rotate_heads_launch(int dtype, const RotateArgs &a, hipStream_t st);
 
 // ---------------------------------------------------------------- attention of long runs, keys and values spelled out (window_attn.hip)
 constexpr int WINDOW_ATTN_MAX_DIM = 256;
@@ -216,6 +294,9 @@ struct WindowAttnArgs {
     const u16 *q, *kv;      // q [M][ld_q], head h at h * D8; kv [context rows][ld_kv]: keys of head h at h * D8, values at H * D8 + h * V8
     u16 *out;               // [M][ld_out], head h at h * V8
     int ld_q, ld_kv, ld_out, H, D8, V8, window;
+    const u16 *q_rot, *k_rot;  // T8 > 0: a second part of queries (row stride ld_q, head h at h * T8) and of keys (row stride ld_krot, the same for all heads)
+    int T8, ld_krot;
+    HeadFinish finish;
     float scale;
     const RowRun *runs;     // the long runs; run r's context = positions [max(0, pos0 - window + 1), pos0 + n_rows), the runs' contexts concatenated in order
     int n_runs;
@@ -313,7 +394,8 @@ struct DeltaArgs {
     int n_seqs, n_slots;
     const RowRun *runs;
     int n_runs;
-    float *state;           // [n_slots][H][D][D] (key channel, value column)
+    float *state;           // [n_slots][slot_floats], of which [H][D][D] (key channel, value column)
+    size_t slot_floats;
     float *ws, *o;          // chunk form: delta_ws_floats(); outputs [M][H][D8] in front of norm and gate
     int chunk_lo, chunk_hi; // (set by the launcher: the chunks of one segment)
     void *out;              // [M][ld_out] T, head h at h * D8
@@ -325,6 +407,78 @@ int delta_chunks_launch(int dtype, const DeltaArgs &a, int chunks, int row0, int
 int delta_chunks(int n_rows);
 size_t delta_ws_floats(int chunks, int H, int D);
 int delta_launches(int chunks, int H, int D);
+
+// every head's output over its root mean square, times w and the sigmoid of its gate (head_out.hip)
+struct HeadOutArgs {
+    const float *o;         // [M][H][D8]
+    const float *den;       // [M][H], what o is divided by first; nullable
+    const void *gate;       // [M][ldg] T logits, head h at h * D8
+    const u16 *gate_bias;   // bf16 [H * D8]; nullable
+    int ldg, H, D, D8;
+    const float *w;         // [H][D]
+    float eps;
+    void *out;              // [M][ld_out] T, head h at h * D8
+    int ld_out;
+};
+constexpr int HEAD_OUT_MAX_DIM = 2048;
+int head_out_launch(int dtype, const HeadOutArgs &a, int row0, int rows, hipStream_t st);
+
+// ---------------------------------------------------------------- recurrences whose gates read the current token only
+struct RecurrentArgs {
+    const void *raw;        // [M][ld] T, the mixer's projections
+    int ld, M;
+    const int *pos, *row_seq, *slots;
+    int n_seqs, n_slots;
+    const RowRun *runs;
+    int n_runs;
+    float *state;           // [n_slots][slot_floats]
+    size_t slot_floats;
+    float *ws;              // chunk forms
+};
+__device__ __forceinline__ float *recurrent_state(const RecurrentArgs &a, const RowRun &run) {
+    return a.state + min((unsigned)a.slots[min(a.row_seq[run.row0], a.n_seqs - 1)], (unsigned)a.n_slots - 1u) * a.slot_floats;
+}
+// chunk i of the runs in pieces of `size` rows
+struct RowChunk {
+    int run, row0, n, pos;  // pos: places of the run in front of it
+};
+__device__ __forceinline__ RowChunk row_chunk(const RowRun *runs, int n_runs, int i, int size) {
+    int r = 0;
+    for (;;) {
+        const int n = (runs[r].n_rows + size - 1) / size;
+        if (i < n || r + 1 >= n_runs) break;
+        i -= n, ++r;
+    }
+    return {r, runs[r].row0 + size * i, min(size, runs[r].n_rows - size * i), size * i};
+}
+
+// minGRU (mingru.hip): S_t = (1 - z) S_(t-1) + z candidate per channel; out = S_t silu(gate)
+struct MingruArgs {
+    RecurrentArgs r;        // raw: z, candidate, gate [D8] each
+    const u16 *bias;        // bf16, same order; nullable
+    int D, D8;
+    void *out;              // [M][ld_out] T
+    int ld_out;
+};
+int mingru_step_launch(int dtype, const MingruArgs &a, hipStream_t st);                 // token by token
+int mingru_chunks_launch(int dtype, const MingruArgs &a, int chunks, hipStream_t st);  // runs of many tokens
+int mingru_chunks(int n_rows);
+size_t mingru_ws_floats(int chunks, int D);
+
+// mLSTM (mlstm.hip): a matrix memory per head with exponential gates
+struct MlstmArgs {
+    RecurrentArgs r;        // raw: q, k [H][D8] each, v, output gate [H][V8] each, input gate, forget gate [H8] each
+    const float *gate_bias; // [2][H]: input, forget
+    int H, D, D8, V, V8, H8;
+    float scale, cap, den_eps;
+    float *o, *den;         // [M][H][V8] sums, [M][H] what they are divided by
+};
+constexpr int MLSTM_MAX_DIM = 1024, MLSTM_CHUNK_MAX_DIM = 512;
+size_t mlstm_state_floats(int H, int D, int V);
+int mlstm_step_launch(int dtype, const MlstmArgs &a, hipStream_t st);       // token by token
+int mlstm_chunks_launch(const MlstmArgs &a, int chunks, hipStream_t st);   // runs of many tokens (bf16)
+int mlstm_chunks(int n_rows);
+size_t mlstm_ws_floats(int chunks, int H, int D);
 
 // ---------------------------------------------------------------- x += post(y); h = next(x) with norms that need the whole row (row_update.hip)
 struct StackNorm {
@@ -353,3 +507,46 @@ struct RowUpdateArgs {
     int *arrived;           // one int, zero before and after
 };
 int row_update_launch(int dtype, const RowUpdateArgs &a, hipStream_t st);
+
+// ---------------------------------------------------------------- residual streams (stream_update.hip)
+// x_t <- sum_s mix[s][t] x_s + out[t] y;  h = next(sum_s in[s] x_s), and the causal convolution over time in front of a mixer: h + conv(h)
+constexpr int STREAMS_MAX = 16, CONV_MAX_TAPS = 16;
+struct StackEmbed {
+    const int *ids;         // nullptr: the streams are in memory already
+    const u16 *table, *bigram, *positions;  // bf16 [vocab][W]; [buckets + 1][W], [max_positions][W], nullable
+    float scale;
+    int vocab, buckets, max_positions;
+    long long mul_prev, mul_cur;
+    float *prev;            // [n_slots][slot_floats]: the sequences' previous tokens (as integers)
+};
+struct ConvArgs {
+    const float *w;         // [taps][ldw], tap taps - 1 reads the row itself; nullptr: none
+    int taps, ldw;
+    float *state;           // [n_slots][slot_floats], of which [taps - 1][W rounded up to 4]: the last inputs, oldest first
+    const int *pos, *row_seq, *slots;
+    int n_seqs, n_slots;
+    size_t slot_floats;
+    const RowRun *runs;
+    int n_runs;
+};
+struct StreamUpdateArgs {
+    StackEmbed embed;
+    const void *y;          // [M][ldy]; nullptr: the streams stay as they are
+    bool y32;               // y is fp32 (else bf16)
+    int ldy;
+    const float *out, *mix; // [S], [S][S] (from, to)
+    float *x;               // [M][S][ldx]
+    int ldx, S;
+    const float *in;        // [S]; nullptr: the streams' sum
+    StackNorm next;
+    ConvArgs conv;          // single: taken here (conv.w may be nullptr); else only its slots are used, and conv_launch follows
+    bool single;            // every run is one row
+    void *h;                // [M][ldh] T
+    int ldh, M, W;
+};
+int stream_update_launch(int dtype, const StreamUpdateArgs &a, hipStream_t st);
+// h = hc + conv(hc) over runs of several rows; carries the state
+int conv_launch(int dtype, const ConvArgs &a, const void *hc, void *h, int ldh, int W, int tiles, hipStream_t st);
+int conv_tiles(int n_rows);
+// out[m][W] = sum of the streams
+int stream_sum_launch(const float *x, int ldx, int S, float *out, int M, int W, hipStream_t st);

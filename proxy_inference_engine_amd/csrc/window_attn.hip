@@ -7,7 +7,8 @@
 //
 // A workgroup owns 128 query rows (4 waves x 32) of one head and walks the 32-key blocks of their union of windows; K and V blocks are staged once in
 // LDS.  Per wave and block: S^T = K . Q^T (32x32x16 MFMAs, keys in registers, rows in lanes), online softmax in fp32, O^T += V^T . P^T with V read
-// transposed from LDS and P split into hi + lo bf16 halves.  Blocks outside a wave's own window are skipped, blocks inside it for every row are not masked.
+// transposed from LDS and P split into hi + lo bf16 halves.  Keys and queries may have a second part (a rotated one; the keys' is the same for all heads and comes
+// from the latents' rows): scores simply run over both.  Blocks outside a wave's own window are skipped, blocks inside it for every row are not masked.
 #include "mfma_store.hpp"  // w4m_pack
 #include "prefill_attn.hpp"
 #include "stack_types.hpp"
@@ -31,10 +32,10 @@ __global__ void __launch_bounds__(64) k_latent_gather(const RowRun *runs, int n_
     for (int c = threadIdx.x * 8; c < ldr; c += 512) *(uint4 *)(out + (size_t)blockIdx.x * ld_out + c) = *(const uint4 *)(src + c);
 }
 
-template <int DM>  // dim and vdim up to DM (32, 64, 128, 256)
-__global__ void __launch_bounds__(256, DM <= 128 ? 2 : 1) k_window_attn(const WindowAttnArgs a) {
-    constexpr int CH = DM / 8, KS = DM / 16, DT = DM / 32, CPT = (32 * CH + 255) / 256;
-    __shared__ __attribute__((aligned(16))) char k_lds[32 * 2 * DM], v_lds[32 * 2 * DM];
+template <int DK, int DV>  // scores over up to DK numbers, values of up to DV
+__global__ void __launch_bounds__(256, DV <= 128 ? 2 : 1) k_window_attn(const WindowAttnArgs a) {
+    constexpr int KC = DK / 8, VC = DV / 8, KS = DK / 16, DT = DV / 32, KPT = (32 * KC + 255) / 256, VPT = (32 * VC + 255) / 256;
+    __shared__ __attribute__((aligned(16))) char k_lds[32 * 2 * DK], v_lds[32 * 2 * DV];
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int c = lane & 31, h = lane >> 5;
     const int head = (int)blockIdx.x % a.H;  // fastest: an XCD keeps meeting the same heads' keys
@@ -54,15 +55,23 @@ __global__ void __launch_bounds__(256, DM <= 128 ? 2 : 1) k_window_attn(const Wi
     const int t_first = a.window > 0 ? max(0, run.pos0 + w0 - a.window + 1) : 0;
     const u16 *kbase = a.kv + (size_t)ctx * a.ld_kv + head * a.D8, *vbase = a.kv + (size_t)ctx * a.ld_kv + a.H * a.D8 + head * a.V8;
 
-    uint4 kr[CPT], vr[CPT];
+    const u16 *krot = a.k_rot + (size_t)ctx * a.ld_krot;
+    uint4 kr[KPT], vr[VPT];
     auto fetch = [&](int t0) {
 #pragma unroll
-        for (int i = 0; i < CPT; ++i) {
-            const int x = threadIdx.x + 256 * i, row = x / CH, ch = x % CH;
+        for (int i = 0; i < KPT; ++i) {
+            const int x = threadIdx.x + 256 * i, row = x / KC, d = 8 * (x % KC);
             const int t = min(max(t0 + row, first), t_last);  // (clamped rows are masked)
-            const bool in = 32 * CH >= 256 || x < 32 * CH;
-            kr[i] = in && 8 * ch < a.D8 ? *(const uint4 *)(kbase + (size_t)(t - first) * a.ld_kv + 8 * ch) : make_uint4(0, 0, 0, 0);
-            vr[i] = in && 8 * ch < a.V8 ? *(const uint4 *)(vbase + (size_t)(t - first) * a.ld_kv + 8 * ch) : make_uint4(0, 0, 0, 0);
+            const bool in = 32 * KC >= 256 || x < 32 * KC;
+            const u16 *p = d < a.D8 ? kbase + (size_t)(t - first) * a.ld_kv + d : krot + (size_t)(t - first) * a.ld_krot + d - a.D8;
+            kr[i] = in && d < a.D8 + a.T8 ? *(const uint4 *)p : make_uint4(0, 0, 0, 0);
+        }
+#pragma unroll
+        for (int i = 0; i < VPT; ++i) {
+            const int x = threadIdx.x + 256 * i, row = x / VC, d = 8 * (x % VC);
+            const int t = min(max(t0 + row, first), t_last);
+            const bool in = 32 * VC >= 256 || x < 32 * VC;
+            vr[i] = in && d < a.V8 ? *(const uint4 *)(vbase + (size_t)(t - first) * a.ld_kv + d) : make_uint4(0, 0, 0, 0);
         }
     };
     const int b0 = t_first / 32, b1 = t_last / 32;
@@ -76,8 +85,11 @@ __global__ void __launch_bounds__(256, DM <= 128 ? 2 : 1) k_window_attn(const Wi
     const int k_lo = a.window > 0 ? q_lo - a.window + 1 : 0, k_full = a.window > 0 ? q_hi - a.window + 1 : 0;
     uint4 qf[KS];
 #pragma unroll
-    for (int s = 0; s < KS; ++s)
-        qf[s] = 16 * s + 8 * h < a.D8 ? *(const uint4 *)(a.q + (size_t)row * a.ld_q + head * a.D8 + 16 * s + 8 * h) : make_uint4(0, 0, 0, 0);
+    for (int s = 0; s < KS; ++s) {
+        const int d = 16 * s + 8 * h;
+        const u16 *p = d < a.D8 ? a.q + (size_t)row * a.ld_q + head * a.D8 + d : a.q_rot + (size_t)row * a.ld_q + head * a.T8 + d - a.D8;
+        qf[s] = d < a.D8 + a.T8 ? *(const uint4 *)p : make_uint4(0, 0, 0, 0);
+    }
     const float sl2 = a.scale * ATTN_LOG2E;
     f32x16_t oacc[DT];
 #pragma unroll
@@ -91,12 +103,14 @@ __global__ void __launch_bounds__(256, DM <= 128 ? 2 : 1) k_window_attn(const Wi
         const int t0 = b * 32;
         __syncthreads();
 #pragma unroll
-        for (int i = 0; i < CPT; ++i) {
+        for (int i = 0; i < KPT; ++i) {
             const int x = threadIdx.x + 256 * i;
-            if (32 * CH >= 256 || x < 32 * CH) {
-                *(uint4 *)(k_lds + pa_off<DM>(x / CH, x % CH)) = kr[i];
-                *(uint4 *)(v_lds + pa_off<DM>(x / CH, x % CH)) = vr[i];
-            }
+            if (32 * KC >= 256 || x < 32 * KC) *(uint4 *)(k_lds + pa_off<DK>(x / KC, x % KC)) = kr[i];
+        }
+#pragma unroll
+        for (int i = 0; i < VPT; ++i) {
+            const int x = threadIdx.x + 256 * i;
+            if (32 * VC >= 256 || x < 32 * VC) *(uint4 *)(v_lds + pa_off<DV>(x / VC, x % VC)) = vr[i];
         }
         __syncthreads();
         if (b < b1) fetch(t0 + 32);
@@ -105,7 +119,7 @@ __global__ void __launch_bounds__(256, DM <= 128 ? 2 : 1) k_window_attn(const Wi
 #pragma unroll
         for (int i = 0; i < 16; ++i) sacc[i] = 0.0f;
 #pragma unroll
-        for (int s = 0; s < KS; ++s) sacc = MfmaT<BF16>::run(*(const uint4 *)(k_lds + pa_off<DM>(c, 2 * s + h)), qf[s], sacc);
+        for (int s = 0; s < KS; ++s) sacc = MfmaT<BF16>::run(*(const uint4 *)(k_lds + pa_off<DK>(c, 2 * s + h)), qf[s], sacc);
         // register i <-> key t0 + (i & 3) + 8 (i >> 2) + 4 h
         float sc[16], mloc = ATTN_NEG;
         if (t0 + 31 <= q_lo && t0 >= k_full) {  // wave-uniform: every row of the wave sees the whole block
@@ -146,9 +160,9 @@ __global__ void __launch_bounds__(256, DM <= 128 ? 2 : 1) k_window_attn(const Wi
             for (int d = 0; d < DT; ++d) {
                 const int ch = 4 * d + 2 * (grp & 1) + (tp >> 1);
                 const v4i16_t lo4 = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-                    (__attribute__((address_space(3))) v4i16_t *)(v_lds + pa_off<DM>(16 * s + 4 * h + tq, ch) + 8 * (tp & 1)));
+                    (__attribute__((address_space(3))) v4i16_t *)(v_lds + pa_off<DV>(16 * s + 4 * h + tq, ch) + 8 * (tp & 1)));
                 const v4i16_t hi4 = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-                    (__attribute__((address_space(3))) v4i16_t *)(v_lds + pa_off<DM>(16 * s + 8 + 4 * h + tq, ch) + 8 * (tp & 1)));
+                    (__attribute__((address_space(3))) v4i16_t *)(v_lds + pa_off<DV>(16 * s + 8 + 4 * h + tq, ch) + 8 * (tp & 1)));
                 const uint2 a0 = __builtin_bit_cast(uint2, lo4), a1 = __builtin_bit_cast(uint2, hi4);
                 const uint4 vf = make_uint4(a0.x, a0.y, a1.x, a1.y);
                 oacc[d] = MfmaT<BF16>::run(vf, bh, oacc[d]);
@@ -156,8 +170,9 @@ __global__ void __launch_bounds__(256, DM <= 128 ? 2 : 1) k_window_attn(const Wi
             }
         }
     }
-    const float inv = 1.0f / xor32_sum(l_run);
+    const float l = xor32_sum(l_run);
     if (r0 + c >= run.n_rows) return;
+    const float inv = head_gate<false>(a.finish, row, head) / (l + head_sink2(a.finish, head, m_run));
     u16 *dst = a.out + (size_t)row * a.ld_out + head * a.V8;
 #pragma unroll
     for (int d = 0; d < DT; ++d)
@@ -178,13 +193,17 @@ int latent_gather_launch(const RowRun *runs, int n_runs, int n_ctx, int window, 
 }
 
 int window_attn_launch(const WindowAttnArgs &a, int n_tiles, hipStream_t st) {
-    const int d = a.D8 > a.V8 ? a.D8 : a.V8;
-    PIE_REQUIRE(d <= WINDOW_ATTN_MAX_DIM, PIE_E_SHAPE, "window attention: heads of at most 256 numbers");
+    const int k = a.D8 + a.T8, v = a.V8;
+    PIE_REQUIRE(k <= WINDOW_ATTN_MAX_DIM && v <= WINDOW_ATTN_MAX_DIM && (a.T8 == 0 || (a.q_rot && a.k_rot && a.ld_krot % 8 == 0)), PIE_E_SHAPE, "window attention: heads of at most 256 numbers");
     const dim3 grid((unsigned)(n_tiles * a.H));
-    if (d <= 32) hipLaunchKernelGGL(k_window_attn<32>, grid, dim3(256), 0, st, a);
-    else if (d <= 64) hipLaunchKernelGGL(k_window_attn<64>, grid, dim3(256), 0, st, a);
-    else if (d <= 128) hipLaunchKernelGGL(k_window_attn<128>, grid, dim3(256), 0, st, a);
-    else hipLaunchKernelGGL(k_window_attn<256>, grid, dim3(256), 0, st, a);
+#define WA_GO(K_, V_) hipLaunchKernelGGL((k_window_attn<K_, V_>), grid, dim3(256), 0, st, a)
+    if (k <= 32 && v <= 32) WA_GO(32, 32);
+    else if (k <= 64 && v <= 64) WA_GO(64, 64);
+    else if (k <= 128 && v <= 64) WA_GO(128, 64);
+    else if (k <= 128 && v <= 128) WA_GO(128, 128);
+    else if (k <= 192 && v <= 128) WA_GO(192, 128);
+    else WA_GO(256, 256);
+#undef WA_GO
     PIE_LAUNCH_CHECK();
     return PIE_OK;
 }

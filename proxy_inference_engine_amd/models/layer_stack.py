@@ -1,6 +1,6 @@
 """Models whose layers are listed one by one, run by the native layer stack (csrc/layer_stack.hip) over paged caches and recurrent state.
 
-A design's module (models/taduzen, models/kodupel) reads its config.json and packs its checkpoint into `pie_stack_layer` descriptions; this class is what every such
+A design's module (models/taduzen, models/kodupel, models/bezutar) reads its config.json and packs its checkpoint into `pie_stack_layer` descriptions; this class is what every such
 model shares with the engines: the cache protocol (make_cache, enable_paged_kv), the calling convention (`model(inputs, cache=)`), the greedy fast
 path (`step`) and the multi-sequence passes (`step_batch`, `prefill_batch`, `step_mixed`, `step_portions`).  Every one of them is the same pass:
 rows of any sequences, each with its own position, in one batch."""
@@ -26,6 +26,16 @@ class Norm(NamedTuple):
     param: float
     w: torch.Tensor
     b: torch.Tensor | None = None
+
+
+class Embedding(NamedTuple):
+    """What the residual starts from besides the token's vector.  streams > 0: equal copies of it (hyper-connections); positions: bf16 [rows, width] by position -- no sequence
+    grows beyond them; bigram: bf16 [buckets + 1, width] by (previous token * mul_prev + token * mul_cur) mod buckets, the last row at a sequence's first token."""
+    streams: int = 0
+    positions: torch.Tensor | None = None
+    bigram: torch.Tensor | None = None
+    mul_prev: int = 0
+    mul_cur: int = 0
 
 
 def up8(n: int) -> int:
@@ -85,15 +95,18 @@ def pack_linear(w: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
 
 class LayerStackModel:
     def __init__(self, args, dtype: torch.dtype, width: int, vocab: int, logit_scale: float, layers: list[dict], embed: torch.Tensor, head: torch.Tensor,
-                 final_norm: Norm, embed_scale: float = 1.0):
+                 final_norm: Norm, embed_scale: float = 1.0, embedding: Embedding = Embedding()):
         """layers: per layer the fields of pie_stack_layer -- tensors for its pointers, Norms for its norms, numbers for the rest
         (absent fields are zero).  embed: bf16 [vocab, width]; head: packed."""
         self.args, self.dtype, self.width, self.vocab_size = args, dtype, width, vocab
         self.device = embed.device
         self.layers = layers
-        self._held = [embed, head, final_norm]
+        self._held = [embed, head, final_norm, embedding]
+        self.max_positions = None if embedding.positions is None else embedding.positions.shape[0]  # tokens a sequence can have
         lib = _ffi.base()
-        cfg = _ffi.pie_stack_config(_ffi.stack_dtype_code(dtype), width, vocab, len(layers), logit_scale, embed_scale, embed.data_ptr(), head.data_ptr(), self._norm(final_norm))
+        cfg = _ffi.pie_stack_config(_ffi.stack_dtype_code(dtype), width, vocab, len(layers), logit_scale, embed_scale, embed.data_ptr(), head.data_ptr(), self._norm(final_norm), embedding.streams, self.max_positions or 0,
+                                    *(None if t is None else t.data_ptr() for t in (embedding.positions, embedding.bigram)), embedding.mul_prev, embedding.mul_cur,
+                                    0 if embedding.bigram is None else embedding.bigram.shape[0] - 1)
         self._stack = C.c_void_p()
         _ffi.check(lib.pie_stack_create(C.byref(cfg), C.byref(self._stack)))
         for i, fields in enumerate(layers):
@@ -179,6 +192,12 @@ class LayerStackModel:
             raise ValueError("a pass takes distinct sequences of one page pool")
         return a
 
+    def _reserve(self, seq: PagedSequence, n: int) -> None:
+        """Room for n more tokens."""
+        if self.max_positions is not None and seq.offset + n > self.max_positions:
+            raise ValueError(f"a sequence of {seq.offset + n} tokens: this model has {self.max_positions} positions")
+        seq.reserve(n)
+
     # ------------------------------------------------------------------ the pass
     def _forward(self, a: LatentPageAllocator, rows: int, ids, pos, row_seq, table, slots, runs, runs_host: np.ndarray, want, n_want: int, logits, logprobs=None,
                  nxt=None, advance: bool = False, history=None, graph: bool = False, tap=None) -> None:
@@ -197,7 +216,7 @@ class LayerStackModel:
         runs first: the native pass serves those in the latent form and the long ones behind them with keys and values spelled out."""
         a = self._sequences([s for _, s in entries])
         for ids, s in entries:
-            s.reserve(len(ids))
+            self._reserve(s, len(ids))
         S, lens = len(entries), np.asarray([len(i) for i, _ in entries], dtype=np.int32)
         order = np.argsort(lens, kind="stable")
         starts = np.empty(S, dtype=np.int32)
@@ -277,7 +296,7 @@ class LayerStackModel:
         a = self._sequences(seqs)
         B = len(seqs)
         for s in seqs:
-            s.reserve(1)
+            self._reserve(s, 1)
         mb = max(len(s.pages) for s in seqs)
         buf = self._bufs.pop(B, None)
         if buf is None or buf["table"].shape[1] < mb:
@@ -402,4 +421,4 @@ class LayerStackModel:
         return int(_ffi.base().pie_stack_launches(self._stack))
 
 
-__all__ = ["LayerStackModel", "Norm", "interleave", "pack_linear", "pad", "pad_head_columns", "pad_head_rows", "up8", "yarn_frequencies"]
+__all__ = ["Embedding", "LayerStackModel", "Norm", "interleave", "pack_linear", "pad", "pad_head_columns", "pad_head_rows", "up8", "yarn_frequencies"]
