@@ -66,7 +66,7 @@ def parse():
                     "IPC-mapped peer memory (default) or RCCL (ncclAllReduce on the launch stream): the comparator for the first run on a real node")
     ap.add_argument("--knob", action="append", default=[], metavar="NAME=VALUE", help="developer: one of the library's test / tuning switches (_ffi.KNOBS) for this run")
     ap.add_argument("--bits", type=int, choices=[2, 4, 6, 8], default=4, help="8 / 6 / 2: MLX int8 / int6 / int2 g=64 weights (W8S / W6S / W2S units; a different workload than the metric's)")
-    ap.add_argument("--design", choices=["taduzen", "kodupel"], help="instead of the metric's workload: prefill and decode throughput of a layer-stack design at sizes that resemble a "
+    ap.add_argument("--design", choices=["taduzen", "kodupel", "bezutar"], help="instead of the metric's workload: prefill and decode throughput of a layer-stack design at sizes that resemble a "
                     "real model's layers, each beside the dense bf16 Llama of equal size (one JSON line; not the BASELINE.json metric)")
     ap.add_argument("--design-only", default="", help="--design: run only the cases whose name contains this (e.g. dense4096/new/decode1)")
     ap.add_argument("--dense", action="store_true", help="BASELINE.json configs[2]: unquantised bf16 weights (a different workload than the metric's)")
@@ -167,6 +167,16 @@ DESIGN_SIZES = {
         "fine2048": {"width": 2048, "heads": 16, "kv_heads": 4, "dim": 128, "delta_heads": 16, "rank": 64, "mlp": {"experts": 64, "top": 6, "ff": 1408},
                      "like": {"hidden_size": 2048, "intermediate_size": 8448, "num_attention_heads": 16, "num_key_value_heads": 4}},
     },
+    # layers: latent attention, minGRU, mLSTM, latent attention on the first layer's latents; `near`: the Taduzen (latent attention without positions, dense squared relu) of equal
+    # width, heads, ranks and feed-forward width
+    "bezutar": {
+        "wide4096": {"width": 4096, "streams": 4, "heads": 32, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "q_rank": 1536, "mlstm": {"heads": 8, "dim": 256, "vdim": 512},
+                     "gru": 4096, "ff": 14336, "near": {"width": 4096, "mixer": {"heads": 32, "dim": 128, "vdim": 128, "kv_rank": 512, "window": None}, "mlp": {"ff": 14336}},
+                     "like": {"hidden_size": 4096, "intermediate_size": 14336, "num_attention_heads": 32, "num_key_value_heads": 8}},
+        "slim2048": {"width": 2048, "streams": 2, "heads": 16, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "q_rank": 768, "mlstm": {"heads": 8, "dim": 128, "vdim": 256},
+                     "gru": 2048, "ff": 8192, "near": {"width": 2048, "mixer": {"heads": 16, "dim": 128, "vdim": 128, "kv_rank": 512, "window": None}, "mlp": {"ff": 8192}},
+                     "like": {"hidden_size": 2048, "intermediate_size": 8192, "num_attention_heads": 16, "num_key_value_heads": 4}},
+    },
 }
 DESIGN_VOCAB = 32768
 
@@ -175,7 +185,7 @@ def taduzen_checkpoint(size, n_layers, vocab):
     """(config, device weights) of a random Taduzen model of one of its DESIGN_SIZES."""
     W, mx, ff = size["width"], size["mixer"], size["mlp"]
     H, D, V, R = mx["heads"], mx["dim"], mx["vdim"], mx["kv_rank"]
-    mixer = {"heads": H, "dim": D, "vdim": V, "kv_rank": R, "scale": D ** -0.5, "mask": {"size": mx["window"]}}
+    mixer = {"heads": H, "dim": D, "vdim": V, "kv_rank": R, "scale": D ** -0.5, "mask": mx["window"] and {"size": mx["window"]}}
     mlp = {"kind": "dense", "ff": ff["ff"]} if "experts" not in ff else \
         {"kind": "moe", "expert": {"ff": ff["ff"]}, "router": {"experts": ff["experts"], "top": ff["top"]}, "shared": {"ff": ff["shared"]}}
     cfg = {"architecture": "Taduzen", "vocab": vocab, "width": W, "logit_scale": 1.0, "norm": {"eps": 1e-6},
@@ -247,12 +257,50 @@ def kodupel_checkpoint(size, n_layers, vocab):
     return cfg, w
 
 
+def bezutar_checkpoint(size, n_layers, vocab):
+    """(config, device weights) of a random Bezutar model of one of its DESIGN_SIZES."""
+    W, S, H, D, T, U, R, Q, N, F, mem = (size[k] for k in ("width", "streams", "heads", "dim", "rot_dim", "vdim", "kv_rank", "q_rank", "gru", "ff", "mlstm"))
+    attn = {"heads": H, "dim": D, "rot_dim": T, "vdim": U, "kv_rank": R, "q_rank": Q, "scale": (D + T) ** -0.5,
+            "rot": {"base": 500000.0, "dims": T, "scaling": {"factor": 4.0, "original": 2048, "fast": 32.0, "slow": 1.0}}}
+    kinds = [("latent_attention", attn), ("mingru", {"width": N}), ("mlstm", dict(mem, gate_cap=15.0)), ("latent_attention", dict(attn, kv_from=0))]
+    layers = [{"type": kinds[i % 4][0], "mixer": kinds[i % 4][1], "mlp": {"kind": "dense", "ff": F}} for i in range(n_layers)]
+    cfg = {"architecture": "Bezutar", "vocab": vocab, "width": W, "streams": S, "max_positions": 8192, "canon": {"taps": 4}, "norm": {"eps": 1e-6},
+           "embedding": {"bigram": {"buckets": 65521, "mul_prev": 31, "mul_cur": 7}}, "layers": layers}
+    gen = torch.Generator(device="cuda").manual_seed(0)
+    w = {}
+
+    def put(name, *shape, std=None, mean=0.0):
+        w[name] = (torch.randn(shape, generator=gen, device="cuda") * (shape[-1] ** -0.5 if std is None else std) + mean).to(torch.bfloat16)
+    put("embed", vocab, W, std=1.0), put("bigram", 65522, W, std=0.5), put("pos", 8192, W, std=0.2)
+    for i, lay in enumerate(layers):
+        p = f"l{i}."
+        put(p + "norm1", W, std=0.02), put(p + "norm2", W, std=0.02), put(p + "canon1", W, 4, std=0.2)
+        for q in ("hc1.", "hc2."):
+            put(p + q + "in", S, std=0.1, mean=1.0 / S), put(p + q + "out", S, std=0.1, mean=1.0), put(p + q + "mix", S, S, std=0.05)
+            w[p + q + "mix"] += 0.9 * torch.eye(S, dtype=torch.bfloat16, device="cuda")
+        if lay["type"] == "latent_attention":
+            put(p + "mix.dq", Q, W), put(p + "mix.dq.norm", Q, std=0.02, mean=1.0), put(p + "mix.uq", H * (D + T), Q), put(p + "mix.uk", H * D, R), put(p + "mix.uv", H * U, R)
+            if "kv_from" not in lay["mixer"]:
+                put(p + "mix.dkv", R + T, W), put(p + "mix.dkv.norm", R, std=0.02, mean=1.0)
+            put(p + "mix.sink", H, std=1.0), put(p + "mix.g", H, W), put(p + "mix.o", W, H * U)
+        elif lay["type"] == "mingru":
+            put(p + "mix.z", N, W), put(p + "mix.z.b", N, std=1.0, mean=-2.0), put(p + "mix.x", N, W), put(p + "mix.x.b", N, std=0.1), put(p + "mix.g", N, W), put(p + "mix.o", W, N)
+        else:
+            h, d, v = mem["heads"], mem["dim"], mem["vdim"]
+            put(p + "mix.q", h * d, W), put(p + "mix.k", h * d, W), put(p + "mix.v", h * v, W), put(p + "mix.g", h * v, W), put(p + "mix.norm", h * v, std=0.02, mean=1.0)
+            put(p + "mix.i", h, W), put(p + "mix.i.b", h, std=0.1), put(p + "mix.f", h, W), put(p + "mix.f.b", h, std=0.1, mean=4.0), put(p + "mix.o", W, h * v)
+        put(p + "mlp.up", F, W), put(p + "mlp.down", W, F), put(p + "mlp.act", 2, std=0.1)
+    put("final.norm", W, std=0.02)
+    put("head", vocab, W)
+    return cfg, w
+
+
 def design_bench(args):
-    """--design: throughput of a layer-stack design beside the dense bf16 Llama of equal size, DESIGN_LAYERS layers each."""
+    """--design: throughput of a layer-stack design beside the dense bf16 Llama of equal size (and, where one is close, another design), DESIGN_LAYERS layers each."""
     from proxy_inference_engine_amd.models.llama import Model as Llama, ModelArgs as LlamaArgs
-    from proxy_inference_engine_amd.models import kodupel, taduzen
+    from proxy_inference_engine_amd.models import bezutar, kodupel, taduzen
     from proxy_inference_engine_amd.models.utils import synthetic_checkpoint
-    design, checkpoint = (taduzen, taduzen_checkpoint) if args.design == "taduzen" else (kodupel, kodupel_checkpoint)
+    design, checkpoint = {"taduzen": (taduzen, taduzen_checkpoint), "kodupel": (kodupel, kodupel_checkpoint), "bezutar": (bezutar, bezutar_checkpoint)}[args.design]
     rows = []
     rng = np.random.default_rng(0)
 
@@ -267,12 +315,15 @@ def design_bench(args):
         return 1e3 * (time.perf_counter() - t0) / n
 
     for name, size in DESIGN_SIZES[args.design].items():
-        for which in ("new", "llama"):
+        for which in ("new", *(("taduzen",) if "near" in size else ()), "llama"):
             if not any(args.design_only in f"{name}/{which}/{c}" for c in ("decode1", "decode8", "decode32", "prefill512", "prefill4096")):
                 continue
             if which == "new":
                 cfg, w = checkpoint(size, DESIGN_LAYERS, DESIGN_VOCAB)
                 model = design.Model(design.ModelArgs(**cfg), w)
+            elif which == "taduzen":
+                cfg, w = taduzen_checkpoint(size["near"], DESIGN_LAYERS, DESIGN_VOCAB)
+                model = taduzen.Model(taduzen.ModelArgs(**cfg), w)
             else:
                 cfg = dict(size["like"], model_type="llama", num_hidden_layers=DESIGN_LAYERS, vocab_size=DESIGN_VOCAB, rms_norm_eps=1e-6, tie_word_embeddings=False,
                            quantization=None)

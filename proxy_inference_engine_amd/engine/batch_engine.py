@@ -57,9 +57,14 @@ class BatchedEngine:
         return (n_tokens + TOKEN_CAPACITY_PER_PAGE - 1) // TOKEN_CAPACITY_PER_PAGE
 
     def generate(self, prompts: list, max_new_tokens: int) -> list[list[int]]:
-        """Token ids generated for every prompt (in order), at most max_new_tokens each, ending early at a stop token."""
+        """Token ids generated for every prompt (in order), at most max_new_tokens each, ending early at a stop token or where the model has no more positions."""
         if max_new_tokens < 1:
             return [[] for _ in prompts]
+        positions = getattr(self.model, "max_positions", None)
+        if positions is not None and any(len(p) > positions for p in prompts):
+            raise ValueError(f"a prompt is longer than the model's {positions} positions")
+        # (a request's last token is not fed back: it needs no position)
+        most = [max_new_tokens if positions is None else min(max_new_tokens, positions - len(p) + 1) for p in prompts]
         for p in prompts:
             if self._pages_for(len(p) + max_new_tokens) > self.pool.size():
                 raise ValueError("a prompt does not fit the page pool")
@@ -99,7 +104,7 @@ class BatchedEngine:
                 keep = []
                 for a, t in zip(active, host):
                     a.generated.append(int(t))
-                    if int(t) in self.stop_tokens or len(a.generated) >= max_new_tokens:
+                    if int(t) in self.stop_tokens or len(a.generated) >= most[a.request]:
                         out[a.request] = a.generated
                         a.cache[0].page_manager.release()
                         reserved -= need.pop(a.request)

@@ -202,6 +202,10 @@ class InferenceEngine:
             if max_completion_tokens > 0 and token_count >= max_completion_tokens:
                 stop_reason = "length"
                 break
+            positions = getattr(self.model, "max_positions", None)
+            if positions is not None and self.prompt_cache.cache[0].offset >= positions:  # the model has no place for the token just generated
+                stop_reason = "length"
+                break
         return stop_reason
 
 

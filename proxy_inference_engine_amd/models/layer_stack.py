@@ -194,9 +194,12 @@ class LayerStackModel:
 
     def _reserve(self, seq: PagedSequence, n: int) -> None:
         """Room for n more tokens."""
+        self._check_length(seq, n)
+        seq.reserve(n)
+
+    def _check_length(self, seq: PagedSequence, n: int) -> None:
         if self.max_positions is not None and seq.offset + n > self.max_positions:
             raise ValueError(f"a sequence of {seq.offset + n} tokens: this model has {self.max_positions} positions")
-        seq.reserve(n)
 
     # ------------------------------------------------------------------ the pass
     def _forward(self, a: LatentPageAllocator, rows: int, ids, pos, row_seq, table, slots, runs, runs_host: np.ndarray, want, n_want: int, logits, logprobs=None,
@@ -262,6 +265,8 @@ class LayerStackModel:
         if sum(len(t) for t, _ in entries) <= MAX_ROWS:
             return self._pass(entries, want, tail)
         self._sequences([s for _, s in entries])
+        for t, s in entries:
+            self._check_length(s, len(t))
         outs, batch, wants, room = [], [], [], MAX_ROWS
 
         def flush():
@@ -361,7 +366,7 @@ class LayerStackModel:
     _fed = _last = None
 
     def step_embeds(self, inputs_embeds, cache):
-        raise NotImplementedError("a layer-stack model takes token ids (its experts are chosen by them)")
+        raise NotImplementedError("a layer-stack model takes token ids (its experts or bigrams are chosen by them)")
 
     def step_batch(self, tokens: torch.Tensor, caches: list[list[BaseCache]], graph: bool = True):
         """One decode step of several sequences: (next tokens [B], logprobs [B, V], logits [B, V]), buffers valid until the next step of that size."""
