@@ -597,7 +597,7 @@ enum { PIE_ACT_SILU = 0, PIE_ACT_CLIPPED = 1 };
  * up-projection of keys, transposed); w_uv heads x packed [vdim, rank]; w_o packed [width, heads * vdim8]; w_kv packed [heads * (dim8 + vdim8), rank]
  * (all keys, then all values: long prompts spell K and V out; may be NULL); c_norm fp32 [rank].  window <= 0: no limit.
  * With q_rank > 0: w_in packed [q_rank8 (query latent) + rank8 (latent) + rot_dim8 (key part that all heads share, rotated, not normed) + heads rounded up to 8
- * (gate, when out_gate), width] (kv_from >= 0: no latent and key part; layer j's cached ones are read); q = w_uq RMSnorm(query latent, q_norm fp32 [q_rank]) with w_uq
+ * (gate, when out_gate), width] (kv_from >= 0: no latent and key part; layer j's cached ones are read); q = w_uq RMSnorm(query latent) times q_norm (fp32 [q_rank]; NULL: folded into w_uq) with w_uq
  * packed [heads * dim8 (unrotated) + heads * rot_dim8 (rotated), q_rank]; score = scale * (unrotated parts' + rotated parts' products); rotation: the first
  * rot_dims numbers of a rotated part, number i with i + rot_dims / 2, by position * rot_freq[i], cos and sin times rot_gain.  head_sink fp32 [heads] (NULL: none): the
  * softmax's denominator also has exp(head_sink).  out_gate as below.

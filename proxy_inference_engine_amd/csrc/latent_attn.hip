@@ -285,60 +285,25 @@ __global__ void __launch_bounds__(256) k_latent_append(const LatentAppend a) {
 template <class E>
 __global__ void __launch_bounds__(256) k_latent_prep(const LatentPrepArgs a) {
     typedef typename E::type T;
-    constexpr bool F32 = sizeof(T) == 4;
     __shared__ float red[2][4];
-    const int m = blockIdx.x, wave = threadIdx.x >> 6;
-    const T *q = (const T *)a.raw + (size_t)m * a.ld, *c = q + a.Q8, *k = c + a.R8;
-    float sq = 0.0f, sc = 0.0f;
-    for (int i = threadIdx.x; i < a.Q; i += 256) sq = fmaf(E::load(q + i), E::load(q + i), sq);
-    if (a.own)
-        for (int i = threadIdx.x; i < a.R; i += 256) sc = fmaf(E::load(c + i), E::load(c + i), sc);
-    sq = lanes_sum(sq), sc = lanes_sum(sc);
-    if ((threadIdx.x & 63) == 0) red[0][wave] = sq, red[1][wave] = sc;
-    const int t = a.pos[m];
-    T *row = nullptr;
-    if (a.own) {
-        const size_t page = min((unsigned)a.table[(size_t)min(a.row_seq[m], a.n_seqs - 1) * a.table_width + min(t / PAGE_TOKENS, a.table_width - 1)], (unsigned)a.n_pages - 1u);
-        row = (T *)a.slab + (page * PAGE_TOKENS + (t & (PAGE_TOKENS - 1))) * (a.R8 + a.T8);
+    const int m = blockIdx.x;
+    if (a.cq) {
+        const T *q = (const T *)a.raw + (size_t)m * a.ld;
+        float ss = 0.0f;
+        for (int i = threadIdx.x; i < a.Q; i += 256) ss = fmaf(E::load(q + i), E::load(q + i), ss);
+        ss = lanes_sum(ss);
+        if ((threadIdx.x & 63) == 0) red[0][threadIdx.x >> 6] = ss;
+        __syncthreads();
+        const float inv = 1.0f / sqrtf(((red[0][0] + red[0][1]) + (red[0][2] + red[0][3])) / (float)a.Q + a.eps);
+        T *cq = (T *)a.cq + (size_t)m * a.ldc;
+        for (int i = threadIdx.x; i < a.Q; i += 256) cq[i] = E::pack(E::load(q + i) * inv * (a.q_norm ? a.q_norm[i] : 1.0f));
     }
-    __syncthreads();
-    const float iq = 1.0f / sqrtf(((red[0][0] + red[0][1]) + (red[0][2] + red[0][3])) / (float)a.Q + a.eps);
-    T *cq = (T *)a.cq + (size_t)m * a.ldc;
-    for (int i = threadIdx.x; i < a.Q; i += 256) cq[i] = E::pack(E::load(q + i) * iq * a.q_norm[i]);
-    if (!a.own) return;
-    const float ic = 1.0f / sqrtf(((red[1][0] + red[1][1]) + (red[1][2] + red[1][3])) / (float)a.R + a.eps);
-    for (int i = threadIdx.x; i < a.R; i += 256) row[i] = E::pack(E::load(c + i) * ic * a.c_norm[i]);
-    row += a.R8;
-    const int half = a.rot.dims / 2;
-    for (int i = threadIdx.x; i < half; i += 256) {
-        float s, co;
-        stack_sincos<F32>((float)t * a.rot.freq[i], s, co);
-        s *= a.rot.gain, co *= a.rot.gain;
-        const float u = E::load(k + i), v = E::load(k + half + i);
-        row[i] = E::pack(u * co - v * s), row[half + i] = E::pack(v * co + u * s);
-    }
-    for (int i = 2 * half + threadIdx.x; i < a.T; i += 256) row[i] = k[i];
+    if (a.own) latent_cache_row<E, 256>(a, m, red[1]);
 }
 
-// One workgroup per row; a thread keeps one pair's angle for all heads it takes.
 template <class E>
 __global__ void __launch_bounds__(256) k_rotate_heads(const RotateArgs a) {
-    typedef typename E::type T;
-    constexpr bool F32 = sizeof(T) == 4;
-    const int m = blockIdx.x, half = a.rot.dims / 2;
-    int lanes = 1;
-    while (lanes < half && lanes < 256) lanes <<= 1;
-    const float t = (float)a.pos[m];
-    for (int i = threadIdx.x & (lanes - 1); i < half; i += lanes) {
-        float s, c;
-        stack_sincos<F32>(t * a.rot.freq[i], s, c);
-        s *= a.rot.gain, c *= a.rot.gain;
-        for (int h = threadIdx.x / lanes; h < a.H; h += 256 / lanes) {
-            T *p = (T *)a.q + (size_t)m * a.ld + h * a.stride + i;
-            const float u = E::load(p), v = E::load(p + half);
-            p[0] = E::pack(u * c - v * s), p[half] = E::pack(v * c + u * s);
-        }
-    }
+    rotate_row<E, 256>(a, blockIdx.x);
 }
 
 }  // namespace

@@ -652,8 +652,8 @@ struct LatentQueries {
     int ld;
     HeadFinish finish;
 };
-// Attention and output of a latent layer whose latents are in their pages (append: not yet, few rows: they ride in the first launch)
-void latent_attend(Pass &p, int li, const pie_stack_layer &L, const LatentQueries &q, const LatentAppend *append, const Into &next, int route) {
+// Attention and output of a latent layer whose latents are in their pages, or (riders, few rows) get there, and whose queries are rotated, along with the first launch
+void latent_attend(Pass &p, int li, const pie_stack_layer &L, const LatentQueries &q, const RowsArgs &riders, const Into &next, int route) {
     pie_stack *s = p.s;
     const pie_stack_batch &b = p.b;
     const int D8 = up8(L.dim), V8 = up8(L.vdim), R8 = up8(L.rank), T8 = up8(L.rot_dim), H = L.heads, KO = H * V8, LO = act_stride(KO), dt = s->cfg.dtype;
@@ -662,10 +662,9 @@ void latent_attend(Pass &p, int li, const pie_stack_layer &L, const LatentQuerie
     const ShortPart sp = short_part(s, b, p.plan, L);
     const int M = sp.M, runs = sp.runs;
     if (M > 0) {  // the latent form
-        RowsArgs k = {};
+        RowsArgs k = riders;
         k.m = {(const char *)L.w_uk, L.rank, L.dim, q.q, q.ld, s->ql.p, H * R8};
         k.M = M, k.epi = ROWS_STORE, k.w_batch = rows_weight_bytes(dt, L.rank, L.dim), k.x_batch = D8, k.y_batch = R8;
-        if (append) k.append = *append;
         p.linear(k, H);
         LatentAttnArgs t = {};
         t.q = s->ql.p, t.ldq = R8, t.q_rot = q.q_rot, t.ld_rot = q.ld, t.finish = q.finish;
@@ -720,7 +719,9 @@ void latent_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next, i
     const LatentAppend append = {p.plan.big && !two ? (const void *)((const u16 *)s->q.p + H * D8) : s->c_raw.p, p.plan.big, p.plan.big && !two ? NI : R8, L.c_norm, L.eps, b.n_rows,
                                  L.rank, R8, b.pos, b.row_seq, b.table, b.table_width, (int)b.n_pages, b.n_seqs, b.slabs[li]};
     if (p.plan.big) p.rc = latent_append_launch(s->cfg.dtype, append, p.st), ++p.launches;  // (few rows: rides in the next launch)
-    latent_attend(p, li, L, {s->q.p, nullptr, LQ, {}}, p.plan.big ? nullptr : &append, next, route);
+    RowsArgs riders = {};
+    if (!p.plan.big) riders.append = append;
+    latent_attend(p, li, L, {s->q.p, nullptr, LQ, {}}, riders, next, route);
 }
 
 // queries out of a latent of their own, with rotated parts
@@ -735,19 +736,25 @@ void latent_query_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &n
     a.q_norm = L.q_norm, a.c_norm = L.c_norm, a.eps = L.eps, a.rot = {L.rot_freq, L.rot_dims, L.rot_gain}, a.own = own_cache(L);
     a.pos = b.pos, a.row_seq = b.row_seq, a.table = b.table, a.table_width = b.table_width, a.n_pages = (int)b.n_pages, a.n_seqs = b.n_seqs;
     a.cq = s->cq.p, a.ldc = CQ, a.slab = b.slabs[li];
-    p.rc = latent_prep_launch(dt, a, p.st), ++p.launches;
+    char *q_rot = (char *)s->qu.p + (size_t)H * D8 * esize(s);
+    const RotateArgs rotate = {q_rot, NQ, T8, H, b.n_rows, a.rot, b.pos};
+    RowsArgs riders = {};
+    const bool few = !p.plan.big && dt == PIE_BF16 && b.n_rows <= 16 && !L.q_norm;  // the norm rides in the queries' product, cache and rotation in the one behind it
+    if (few) {
+        if (a.own) riders.cache = a;
+        if (L.rot_dims > 0) riders.rotate = rotate;
+    } else p.rc = latent_prep_launch(dt, a, p.st), ++p.launches;
     if (p.plan.big) p.gemm(L.w_uq, s->cq.p, CQ, b.n_rows, NQ, L.q_rank, s->qu.p, NQ);
     else {
         RowsArgs u = {};
-        u.m = {(const char *)L.w_uq, NQ, L.q_rank, s->cq.p, CQ, s->qu.p, NQ};
-        u.M = b.n_rows, u.epi = ROWS_STORE;
+        u.m = {(const char *)L.w_uq, NQ, L.q_rank, few ? s->q.p : s->cq.p, few ? NI : CQ, s->qu.p, NQ};
+        u.M = b.n_rows, u.epi = ROWS_STORE, u.x_norm = few, u.x_eps = L.eps;
         p.linear(u);
     }
     if (p.rc) return;
-    char *q_rot = (char *)s->qu.p + (size_t)H * D8 * esize(s);
-    if (L.rot_dims > 0) p.rc = rotate_heads_launch(dt, {q_rot, NQ, T8, H, b.n_rows, {L.rot_freq, L.rot_dims, L.rot_gain}, b.pos}, p.st), ++p.launches;
+    if (!few && L.rot_dims > 0) p.rc = rotate_heads_launch(dt, rotate, p.st), ++p.launches;
     const HeadFinish finish = {L.head_sink, L.out_gate ? (const char *)s->q.p + (size_t)(NI - up8(H)) * esize(s) : nullptr, NI};
-    latent_attend(p, li, L, {s->qu.p, q_rot, NQ, finish}, nullptr, next, route);
+    latent_attend(p, li, L, {s->qu.p, q_rot, NQ, finish}, riders, next, route);
 }
 
 void attention_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next, int route) {
@@ -998,7 +1005,7 @@ int mixer_ok(const pie_stack *s, int i, const pie_stack_layer &L) {
     if (L.mixer == PIE_MIXER_LATENT) {
         PIE_REQUIRE(L.vdim > 0 && L.rank > 0 && L.q_rank >= 0 && L.rot_dim >= 0 && latent_row(L) <= 2048, PIE_E_SHAPE, "pie_stack_set_layer: bad mixer sizes (kv_rank + rot_dim at most 2048)");
         PIE_REQUIRE(L.w_uk && L.w_uv && (L.c_norm || !own_cache(L)), PIE_E_ARG, "pie_stack_set_layer: missing mixer weights");
-        PIE_REQUIRE(L.q_rank ? L.w_uq && L.q_norm : !L.rot_dim && !L.out_gate && !L.head_sink, PIE_E_ARG,
+        PIE_REQUIRE(L.q_rank ? L.w_uq != nullptr : !L.rot_dim && !L.out_gate && !L.head_sink, PIE_E_ARG,
                     "pie_stack_set_layer: rotation, gate and sink of latent attention go with a query latent, which needs its weights");
         PIE_REQUIRE(L.rot_dims >= 0 && L.rot_dims <= L.rot_dim && L.rot_dims % 2 == 0 && (L.rot_dims == 0 || L.rot_freq), PIE_E_SHAPE, "pie_stack_set_layer: bad rotation");
         if (!own_cache(L)) {

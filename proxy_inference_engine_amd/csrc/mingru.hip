@@ -43,7 +43,7 @@ __device__ __forceinline__ void mg_store(const MingruArgs &a, size_t m, int d, f
     else *(u32 *)out = pack2<BF16>(x, y);
 }
 
-constexpr int MG_AHEAD = 8;  // tokens in flight
+constexpr int MG_AHEAD = 16;  // tokens in flight
 
 // walks rows [row0, row0 + n) from (sx, sy); OUT: writes the outputs; else accumulates the factors' products
 template <class E, bool OUT>
@@ -61,7 +61,7 @@ __device__ __forceinline__ void mg_walk(const MingruArgs &a, int row0, int n, in
         }
 #pragma unroll
         for (int t = 0; t < MG_AHEAD; ++t) {
-            if (t0 + t >= n) break;
+            if (t0 + t >= n) continue;
             const MgPair p = mg_gate<F32>(z[t].x + bz.x, u[t].x + bu.x), q = mg_gate<F32>(z[t].y + bz.y, u[t].y + bu.y);
             sx = fmaf(p.x, sx, p.y), sy = fmaf(q.x, sy, q.y);
             if constexpr (OUT) mg_store<E>(a, row0 + t0 + t, d, sx, sy, g[t], bg);

@@ -175,7 +175,7 @@ __global__ void __launch_bounds__(256) k_mlstm_prep(const MlstmArgs a) {
         }
         s_b[lane] = b, s_c[lane] = m, s_g[lane] = g.i;
         const float bl = __shfl(b, 63, 64), cl = __shfl(m, 63, 64);
-        o_s[lane] = b, o_s[ML + lane] = m, o_s[2 * ML + lane] = lane < c.n ? expf(bl - b + g.i - cl) : 0.0f;
+        o_s[lane] = b, o_s[ML + lane] = m, o_s[2 * ML + lane] = lane < c.n ? stack_exp<false>(bl - b + g.i - cl) : 0.0f;
     }
     ml_f32x4 acc[4];
 #pragma unroll
@@ -204,7 +204,7 @@ __global__ void __launch_bounds__(256) k_mlstm_prep(const MlstmArgs a) {
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int row = 16 * wave + 4 * q4 + i, s = 16 * t + n16;
-            float x = s <= row && row < c.n ? a.scale * acc[t][i] * expf(s_b[row] - s_b[s] + s_g[s] - s_c[row]) : 0.0f, y = 0.0f;
+            float x = s <= row && row < c.n ? a.scale * acc[t][i] * stack_exp<false>(s_b[row] - s_b[s] + s_g[s] - s_c[row]) : 0.0f, y = 0.0f;
             const u16 hi = BF16::from_f32(x);
             y = x - BF16::to_f32(hi);
             s_p[0][row][s] = hi, s_p[1][row][s] = BF16::from_f32(y);
@@ -218,15 +218,9 @@ __global__ void __launch_bounds__(256) k_mlstm_prep(const MlstmArgs a) {
         for (int k = 0; k < 2; ++k) *(uint4 *)(o_p + (s * 2 + k) * 1024 + lane * 16) = *(const uint4 *)&s_p[k][16 * wave + n16][32 * s + 8 * q4];
 }
 
-// NPW: 32-channel pairs per wave (D <= 128 NPW)
+// NPW: 32-channel pairs per wave (D <= 128 NPW).  A chunk's operands are loaded where the previous chunk's have just been used.
 template <int NPW>
-struct MlOps {
-    uint4 q[4][NPW], k[NPW][2][2], p[2][2];
-    u16 v[16];
-    float b, c, w;
-};
-template <int NPW>
-__global__ void __launch_bounds__(256, 1) k_mlstm_scan(const MlstmArgs a) {
+__global__ void __launch_bounds__(256, NPW <= 2 ? 2 : 1) k_mlstm_scan(const MlstmArgs a) {
     __shared__ __attribute__((aligned(16))) ml_f32x4 s_o[2][4][4][64];
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), n16 = lane & 15, q4 = lane >> 4;
     const int head = (int)blockIdx.x % a.H, cb = (int)blockIdx.x / a.H, blocks = ml_blocks(a.V), V4 = ml_up4(a.V), D = a.D, np = ml_pairs(D);  // (head fastest: a head's columns share an L2 where H is a multiple of 8)
@@ -255,38 +249,52 @@ __global__ void __launch_bounds__(256, 1) k_mlstm_scan(const MlstmArgs a) {
                 S[j][e][i] = !fresh && p ? *p : 0.0f;
             }
     float m = fresh ? 0.0f : st.m[cb];
-    const size_t per = ml_chunk_bytes(D);
+    const size_t per = ml_chunk_bytes(D), step = per * a.H;
+    const char *ws0 = (const char *)a.r.ws + ((size_t)chunk0 * a.H + head) * per;
     const u16 *rv = (const u16 *)a.r.raw + (size_t)run.row0 * a.r.ld + 2 * a.H * a.D8 + head * a.V8 + min(col, a.V - 1);
-    auto fetch = [&](int cc, MlOps<NPW> &o) {
-        const int ch = min(cc, chunks - 1);
-        const char *ws = (const char *)a.r.ws + ((size_t)(chunk0 + ch) * a.H + head) * per + lane * 16;
+    uint4 q[4][NPW], k[NPW][2][2], p[2][2];
+    u16 v[16];
+    float nb, nc, nw;
+    auto load_q = [&](int ch) {
+        const char *ws = ws0 + (size_t)min(ch, chunks - 1) * step + lane * 16;
 #pragma unroll
-        for (int j = 0; j < NPW; ++j) {
-            const int p = min(wave * NPW + j, np - 1);
+        for (int t = 0; t < 4; ++t)
 #pragma unroll
-            for (int t = 0; t < 4; ++t) o.q[t][j] = *(const uint4 *)(ws + ((size_t)t * np + p) * 1024);
+            for (int j = 0; j < NPW; ++j) q[t][j] = *(const uint4 *)(ws + ((size_t)t * np + min(wave * NPW + j, np - 1)) * 1024);
+    };
+    auto load_k = [&](int ch) {
+        const char *ws = ws0 + (size_t)min(ch, chunks - 1) * step + (size_t)np * 4096 + lane * 16;
+#pragma unroll
+        for (int j = 0; j < NPW; ++j)
 #pragma unroll
             for (int e = 0; e < 2; ++e)
 #pragma unroll
-                for (int s = 0; s < 2; ++s) o.k[j][e][s] = *(const uint4 *)(ws + (size_t)np * 4096 + (size_t)(4 * p + 2 * e + s) * 1024);
-        }
+                for (int s = 0; s < 2; ++s) k[j][e][s] = *(const uint4 *)(ws + (size_t)(4 * min(wave * NPW + j, np - 1) + 2 * e + s) * 1024);
+    };
+    auto load_pv = [&](int ch) {
+        const int c = min(ch, chunks - 1);
+        const char *ws = ws0 + (size_t)c * step + (size_t)np * 8192 + wave * 4096 + lane * 16;
 #pragma unroll
         for (int s = 0; s < 2; ++s)
 #pragma unroll
-            for (int k = 0; k < 2; ++k) o.p[s][k] = *(const uint4 *)(ws + (size_t)np * 8192 + wave * 4096 + (s * 2 + k) * 1024);
-        const float *sc = (const float *)(ws - lane * 16 + (size_t)np * 8192 + 16384);
-        o.b = sc[lane], o.c = sc[ML + lane], o.w = sc[2 * ML + lane];
+            for (int h = 0; h < 2; ++h) p[s][h] = *(const uint4 *)(ws + (s * 2 + h) * 1024);
 #pragma unroll
-        for (int i = 0; i < 16; ++i) o.v[i] = has_n ? (u16)0x3F80 : rv[(size_t)min(ML * ch + 32 * (i >> 3) + 8 * q4 + (i & 7), run.n_rows - 1) * a.r.ld];
+        for (int i = 0; i < 16; ++i) v[i] = rv[(size_t)min(ML * c + 32 * (i >> 3) + 8 * q4 + (i & 7), run.n_rows - 1) * a.r.ld];
     };
+    auto load_scalars = [&](int ch) {
+        const float *sc = (const float *)(ws0 + (size_t)min(ch, chunks - 1) * step + (size_t)np * 8192 + 16384);
+        nb = sc[lane], nc = sc[ML + lane], nw = sc[2 * ML + lane];
+    };
+    load_scalars(0), load_q(0), load_pv(0), load_k(0);
     const ml_f32x4 zero = {0.0f, 0.0f, 0.0f, 0.0f};
-    auto chunk = [&](int ch, const MlOps<NPW> &x) {
-        const float bl = __shfl(x.b, 63, 64), cl = __shfl(x.c, 63, 64), next = fmaxf(m + bl, cl), keep = expf(m + bl - next), add = expf(cl - next);
+    for (int ch = 0; ch < chunks; ++ch) {
+        const float cb_ = nb, cc = nc, cw = nw;
+        load_scalars(ch + 1);
+        const float bl = __shfl(cb_, 63, 64), cl = __shfl(cc, 63, 64), next = fmaxf(m + bl, cl), keep = stack_exp<false>(m + bl - next), add = stack_exp<false>(cl - next);
         // S^T q of the chunk's 64 rows: the wave's channels
         ml_f32x4 acc[4] = {zero, zero, zero, zero};
 #pragma unroll
         for (int j = 0; j < NPW; ++j) {
-            if (wave * NPW + j >= np) continue;
             float f[8];
             u32 hi[4], lo[4];
 #pragma unroll
@@ -295,67 +303,74 @@ __global__ void __launch_bounds__(256, 1) k_mlstm_scan(const MlstmArgs a) {
             for (int i = 0; i < 4; ++i) hi[i] = ml_part(f[2 * i], f[2 * i + 1]), lo[i] = pack2<BF16>(f[2 * i], f[2 * i + 1]);
             const uint4 h = make_uint4(hi[0], hi[1], hi[2], hi[3]), l = make_uint4(lo[0], lo[1], lo[2], lo[3]);
 #pragma unroll
-            for (int t = 0; t < 4; ++t) acc[t] = ml_mfma(x.q[t][j], h, acc[t]);
+            for (int t = 0; t < 4; ++t) acc[t] = ml_mfma(q[t][j], h, acc[t]);
 #pragma unroll
-            for (int t = 0; t < 4; ++t) acc[t] = ml_mfma(x.q[t][j], l, acc[t]);
+            for (int t = 0; t < 4; ++t) acc[t] = ml_mfma(q[t][j], l, acc[t]);
         }
+        load_q(ch + 1);
 #pragma unroll
         for (int t = 0; t < 4; ++t) s_o[ch & 1][wave][t][lane] = acc[t];
         // the wave's own rows among themselves
         ml_f32x4 own = zero;
-        uint4 v[2];
+        float f[2][8];
 #pragma unroll
-        for (int s = 0; s < 2; ++s)
-            v[s] = make_uint4(x.v[8 * s] | (u32)x.v[8 * s + 1] << 16, x.v[8 * s + 2] | (u32)x.v[8 * s + 3] << 16, x.v[8 * s + 4] | (u32)x.v[8 * s + 5] << 16, x.v[8 * s + 6] | (u32)x.v[8 * s + 7] << 16);
+        for (int s = 0; s < 2; ++s) {
+            u32 w[4];
 #pragma unroll
-        for (int s = 0; s < 2; ++s) own = ml_mfma(x.p[s][0], v[s], own), own = ml_mfma(x.p[s][1], v[s], own);
+            for (int i = 0; i < 4; ++i) w[i] = has_n ? 0x3F803F80u : (u32)v[8 * s + 2 * i] | (u32)v[8 * s + 2 * i + 1] << 16;  // (n: v = 1)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                f[s][2 * i] = lo_f32<BF16>(w[i]) * (add * __shfl(cw, 32 * s + 8 * q4 + 2 * i, 64));
+                f[s][2 * i + 1] = hi_f32<BF16>(w[i]) * (add * __shfl(cw, 32 * s + 8 * q4 + 2 * i + 1, 64));
+            }
+            const uint4 vv = make_uint4(w[0], w[1], w[2], w[3]);
+            own = ml_mfma(p[s][0], vv, own), own = ml_mfma(p[s][1], vv, own);
+        }
+        load_pv(ch + 1);
         // the state behind the chunk: values times their key weights, in three parts
 #pragma unroll
         for (int j = 0; j < NPW; ++j)
 #pragma unroll
             for (int e = 0; e < 2; ++e) S[j][e] *= keep;
 #pragma unroll
-        for (int s = 0; s < 2; ++s) {
-            float f[8];
+        for (int s = 0; s < 2; ++s)
 #pragma unroll
-            for (int i = 0; i < 8; ++i) f[i] = BF16::to_f32(x.v[8 * s + i]) * (add * __shfl(x.w, 32 * s + 8 * q4 + i, 64));
-#pragma unroll
-            for (int k = 0; k < 3; ++k) {
+            for (int h = 0; h < 3; ++h) {
                 u32 w[4];
 #pragma unroll
-                for (int i = 0; i < 4; ++i) w[i] = ml_part(f[2 * i], f[2 * i + 1]);
+                for (int i = 0; i < 4; ++i) w[i] = ml_part(f[s][2 * i], f[s][2 * i + 1]);
                 const uint4 part = make_uint4(w[0], w[1], w[2], w[3]);
 #pragma unroll
-                for (int j = 0; j < NPW; ++j) {
-                    if (wave * NPW + j >= np) continue;
+                for (int j = 0; j < NPW; ++j)
 #pragma unroll
-                    for (int e = 0; e < 2; ++e) S[j][e] = ml_mfma(x.k[j][e][s], part, S[j][e]);
-                }
+                    for (int e = 0; e < 2; ++e) S[j][e] = ml_mfma(k[j][e][s], part, S[j][e]);
             }
-        }
+        load_k(ch + 1);
+#pragma unroll
+        for (int j = 0; j < NPW; ++j)
+            if (wave * NPW + j >= np) S[j][0] = S[j][1] = zero;  // (channels that do not exist saw another pair's keys)
         asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");  // (LDS only: the next chunk's loads stay in flight)
         const ml_f32x4 all = (s_o[ch & 1][0][wave][lane] + s_o[ch & 1][1][wave][lane]) + (s_o[ch & 1][2][wave][lane] + s_o[ch & 1][3][wave][lane]);
+        float o[4], mt[4];
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int t = 16 * wave + 4 * q4 + i;
-            const float b = __shfl(x.b, t, 64), c = __shfl(x.c, t, 64), mt = fmaxf(m + b, c);
-            const float o = fmaf(a.scale * expf(m + b - mt), all[i], expf(c - mt) * own[i]);
-            const size_t at = ((size_t)run.row0 + ML * ch + t) * a.H + head;
-            if (ML * ch + t >= run.n_rows) continue;
-            if (has_n) {
-                if (n16 == 0) a.den[at] = fmaxf(fabsf(o), expf(-mt)) + a.den_eps;
-            } else if (col < a.V) a.o[at * a.V8 + col] = o;
+            const float b = __shfl(cb_, t, 64), c = __shfl(cc, t, 64);
+            mt[i] = fmaxf(m + b, c);
+            o[i] = fmaf(a.scale * stack_exp<false>(m + b - mt[i]), all[i], stack_exp<false>(c - mt[i]) * own[i]);
         }
+        const int t0 = ML * ch + 16 * wave + 4 * q4;
+        const size_t at = ((size_t)run.row0 + t0) * a.H + head;
+        if (has_n) {
+            if (n16 == 0)
+#pragma unroll
+                for (int i = 0; i < 4; ++i)
+                    if (t0 + i < run.n_rows) a.den[at + (size_t)i * a.H] = fmaxf(fabsf(o[i]), stack_exp<false>(-mt[i])) + a.den_eps;
+        } else if (col < a.V)
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+                if (t0 + i < run.n_rows) a.o[(at + (size_t)i * a.H) * a.V8 + col] = o[i];
         m = next;
-    };
-    MlOps<NPW> x0, x1;
-    fetch(0, x0);
-    for (int ch = 0; ch < chunks; ch += 2) {
-        fetch(ch + 1, x1);
-        chunk(ch, x0);
-        if (ch + 1 >= chunks) break;
-        fetch(ch + 2, x0);
-        chunk(ch + 1, x1);
     }
 #pragma unroll
     for (int j = 0; j < NPW; ++j)
@@ -363,7 +378,7 @@ __global__ void __launch_bounds__(256, 1) k_mlstm_scan(const MlstmArgs a) {
         for (int e = 0; e < 2; ++e)
 #pragma unroll
             for (int i = 0; i < 4; ++i)
-                if (float *p = place(j, e, i)) *p = S[j][e][i];
+                if (float *x = place(j, e, i)) *x = S[j][e][i];
     if (threadIdx.x == 0) st.m[cb] = m;
 }
 

@@ -81,25 +81,36 @@ __device__ __forceinline__ void rows_finish(const RowsArgs &a, const RowsWork &k
     }
 }
 
+__host__ __device__ __forceinline__ int rows_riders(const RowsArgs &a) { return (a.append.M > 0) + (a.cache.M > 0) + (a.rotate.M > 0); }
+// the last blockIdx.y: what rides along
 template <class E, int THREADS>
-__device__ __forceinline__ bool rows_append(const RowsArgs &a, float *red) {
-    if (a.append.M <= 0 || blockIdx.y + 1 < gridDim.y) return false;
-    if (blockIdx.z == 0)
-        for (int m = blockIdx.x; m < a.append.M; m += gridDim.x) {
-            latent_append_row<E, ElemF32, THREADS>(a.append, m, red);
-            __syncthreads();
-        }
+__device__ __forceinline__ bool rows_ride(const RowsArgs &a, float *red) {
+    int i = (int)(gridDim.y - 1 - blockIdx.y);
+    if (i >= rows_riders(a)) return false;
+    if (blockIdx.z) return true;
+    const bool append = a.append.M > 0 && i == 0;
+    i -= a.append.M > 0;
+    const bool cache = a.cache.M > 0 && i == 0;
+    const int M = append ? a.append.M : cache ? a.cache.M : a.rotate.M;
+    for (int m = blockIdx.x; m < M; m += gridDim.x) {
+        if (append) latent_append_row<E, ElemF32, THREADS>(a.append, m, red);
+        else if (cache) latent_cache_row<E, THREADS>(a.cache, m, red);
+        else rotate_row<E, THREADS>(a.rotate, m);
+        __syncthreads();
+    }
     return true;
 }
 
 // NT: blocks of 16 rows of x; KW: waves along K; NN: blocks of 16 features per wave (two share the x operands); MERGE: x = the merged key splits of head
-// blockIdx.y (RowsArgs::merge), put together in LDS by every workgroup of the head
-template <int NT, int KW, int NN, bool MERGE = false>
+// blockIdx.y (RowsArgs::merge), put together in LDS by every workgroup of the head; NORM: RowsArgs::x_norm (every workgroup sees its rows whole)
+template <int NT, int KW, int NN, bool MERGE = false, bool NORM = false>
 __global__ void __launch_bounds__(512) k_rows_w16m(const RowsArgs a) {
     constexpr int NW = 8 / KW, U = NT >= 4 ? 2 : 4;
     constexpr int ST = 20;  // floats per (row, 16 features) line of the reduction image
     __shared__ __attribute__((aligned(16))) float s_red[8 * NN * NT * 16 * ST];
-    if (rows_append<ElemBF16, 512>(a, s_red)) return;
+    __shared__ float s_ss[NORM ? 8 : 1][16];
+    static_assert(!NORM || NT == 1, "norms: sixteen rows");
+    if (rows_ride<ElemBF16, 512>(a, s_red)) return;
     __shared__ __attribute__((aligned(16))) u16 s_x[MERGE ? MERGE_ROWS * (MERGE_LDR + 64) : 8];
     const int ldx_lds = a.merge.ldr + 64;
     if constexpr (MERGE) {
@@ -128,6 +139,7 @@ __global__ void __launch_bounds__(512) k_rows_w16m(const RowsArgs a) {
     const int groups = (k.K + 63) >> 6, steps = 2 * groups;
     const bool live = t16 * 16 < k.N;  // (NN = 2: both blocks lie in one 32-row tile, which is stored whole)
 
+    float ss = 0.0f;
     mf_f32x4 acc[NN][NT];
 #pragma unroll
     for (int n = 0; n < NN; ++n)
@@ -160,6 +172,10 @@ __global__ void __launch_bounds__(512) k_rows_w16m(const RowsArgs a) {
                 for (int n = 0; n < NN; ++n) {
                     mf_u32x4 w = wv[u][n];
                     if (s + u * KW >= steps) w = (mf_u32x4){0u, 0u, 0u, 0u};
+                    if constexpr (NORM)
+                        if (n == 0 && s + u * KW < steps && 32 * (s + u * KW) + 8 * kq < k.K)  // (what lies behind the row belongs to others; a row's padding to 8 is zero)
+#pragma unroll
+                            for (int i = 0; i < 4; ++i) ss = fmaf(lo_f32<BF16>(xv[u][0][i]), lo_f32<BF16>(xv[u][0][i]), fmaf(hi_f32<BF16>(xv[u][0][i]), hi_f32<BF16>(xv[u][0][i]), ss));
 #pragma unroll
                     for (int t = 0; t < NT; ++t)
                         acc[n][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(mf_bf16x8, w), __builtin_bit_cast(mf_bf16x8, xv[u][t]), acc[n][t], 0, 0, 0);
@@ -173,6 +189,10 @@ __global__ void __launch_bounds__(512) k_rows_w16m(const RowsArgs a) {
             fetch(s + 2 * U * KW, w0, x0);
             multiply(s + U * KW, w1, x1);
         }
+    }
+    if constexpr (NORM) {
+        ss = xor32_sum(xor16_sum(ss));
+        if (kq == 0) s_ss[wave][c] = ss;
     }
     // lane (kq, c) holds features 4 kq .. + 3 of row c
 #pragma unroll
@@ -193,6 +213,12 @@ __global__ void __launch_bounds__(512) k_rows_w16m(const RowsArgs a) {
         if (paired)
 #pragma unroll
             for (int q = 0; q < KW; ++q) p += r[q * NN * NT * 16 * ST + 1];
+        if constexpr (NORM) {
+            float sum = 0.0f;
+#pragma unroll
+            for (int q = 0; q < KW; ++q) sum += s_ss[w * KW + q][ml];
+            v *= 1.0f / sqrtf(sum / (float)k.K + a.x_eps);
+        }
         rows_finish<ElemBF16>(a, k, m, n, v, p);
     }
 }
@@ -200,7 +226,7 @@ __global__ void __launch_bounds__(512) k_rows_w16m(const RowsArgs a) {
 // fp32: one output per thread, 16 features x 16 rows per workgroup, both operands through LDS
 __global__ void __launch_bounds__(256) k_rows_f32(const RowsArgs a) {
     __shared__ float s_w[16][65], s_x[16][65], s_v[16][17];
-    if (rows_append<ElemF32, 256>(a, s_v[0])) return;
+    if (rows_ride<ElemF32, 256>(a, s_v[0])) return;
     RowsWork k;
     if (!rows_select(a, k)) return;
     const int i0 = blockIdx.z * 16, n0 = blockIdx.x * 16;
@@ -235,8 +261,13 @@ int rows_go(const RowsArgs &a, int n_max, int k_max, int batches, hipStream_t st
     // waves along K: enough steps for each, and enough workgroups for the chip
     int kw = steps >= 32 ? 8 : steps >= 16 ? 4 : steps >= 8 ? 2 : 1;
     while (kw < 8 && steps >= 2 * kw && (size_t)((tiles + 8 / kw - 1) / (8 / kw)) * batches * z < 256) kw *= 2;
-    const dim3 grid((unsigned)((tiles + 8 / kw - 1) / (8 / kw)), (unsigned)(batches + (a.append.M > 0 ? 1 : 0)), (unsigned)z);
-    if (a.merge.splits > 0) {
+    const dim3 grid((unsigned)((tiles + 8 / kw - 1) / (8 / kw)), (unsigned)(batches + rows_riders(a)), (unsigned)z);
+    if (a.x_norm) {
+        if (kw == 8) hipLaunchKernelGGL((k_rows_w16m<1, 8, 1, false, true>), grid, dim3(512), 0, st, a);
+        else if (kw == 4) hipLaunchKernelGGL((k_rows_w16m<1, 4, 1, false, true>), grid, dim3(512), 0, st, a);
+        else if (kw == 2) hipLaunchKernelGGL((k_rows_w16m<1, 2, 1, false, true>), grid, dim3(512), 0, st, a);
+        else hipLaunchKernelGGL((k_rows_w16m<1, 1, 1, false, true>), grid, dim3(512), 0, st, a);
+    } else if (a.merge.splits > 0) {
         if (kw == 8) hipLaunchKernelGGL((k_rows_w16m<1, 8, 1, true>), grid, dim3(512), 0, st, a);
         else if (kw == 4) hipLaunchKernelGGL((k_rows_w16m<1, 4, 1, true>), grid, dim3(512), 0, st, a);
         else if (kw == 2) hipLaunchKernelGGL((k_rows_w16m<1, 2, 1, true>), grid, dim3(512), 0, st, a);
@@ -265,10 +296,11 @@ size_t rows_weight_bytes(int dtype, int N, int K) {
 int rows_gemm_launch(int dtype, const RowsArgs &a, int batches, hipStream_t st) {
     if (a.M <= 0 || batches <= 0) return PIE_OK;
     PIE_REQUIRE(a.m.N > 0 && a.m.K > 0, PIE_E_SHAPE, "row-wise Linear: empty matrix");
-    PIE_REQUIRE(batches < 65535 && (a.append.M <= 0 || !(a.shared.w || a.active)), PIE_E_SHAPE, "row-wise Linear: too many batches");
+    PIE_REQUIRE(batches < 65535 && (!rows_riders(a) || !(a.shared.w || a.active)), PIE_E_SHAPE, "row-wise Linear: too many batches");
     const int n_max = a.shared.w && a.shared.N > a.m.N ? a.shared.N : a.m.N, k_max = a.shared.w && a.shared.K > a.m.K ? a.shared.K : a.m.K;
+    PIE_REQUIRE(!a.x_norm || (dtype == PIE_BF16 && a.M <= 16 && batches == 1 && !a.active && !a.shared.w && !a.rows && a.merge.splits <= 0), PIE_E_SHAPE, "row-wise Linear: too many rows to norm on the way in");
     if (dtype == PIE_F32) {
-        const dim3 grid((unsigned)((n_max + 15) / 16), (unsigned)(batches + (a.append.M > 0 ? 1 : 0)), (unsigned)((a.M + 15) / 16));
+        const dim3 grid((unsigned)((n_max + 15) / 16), (unsigned)(batches + rows_riders(a)), (unsigned)((a.M + 15) / 16));
         hipLaunchKernelGGL(k_rows_f32, grid, dim3(256), 0, st, a);
         PIE_LAUNCH_CHECK();
         return PIE_OK;

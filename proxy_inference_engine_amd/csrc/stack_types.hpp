@@ -72,6 +72,10 @@ __device__ __forceinline__ void stack_sincos(float a, float &s, float &c) {
 template <bool F32>
 __device__ __forceinline__ float xielu(float z, float up, float down) {
     const float n = fminf(z, 0.0f);
+    if constexpr (!F32) {  // (the difference's absolute error of 1e-7 is below what the result is rounded to)
+        const float p = fmaxf(z, 0.0f), e = __builtin_amdgcn_exp2f(n * STACK_LOG2E);
+        return fmaf(p, fmaf(up, p, 0.5f), fmaf(0.5f - down, n, fmaf(down, e, -down)));
+    }
     const float series = 0.5f * n * n * fmaf(n * (1.0f / 3.0f), fmaf(n * 0.25f, fmaf(n * 0.2f, fmaf(n * (1.0f / 6.0f), fmaf(n * (1.0f / 7.0f), 1.0f, 1.0f), 1.0f), 1.0f), 1.0f), 1.0f);
     const float g = n > -0.25f ? series : stack_exp<F32>(n) - 1.0f - n;
     return fmaf(0.5f, z, z > 0.0f ? up * z * z : down * g);
@@ -119,6 +123,83 @@ __device__ __forceinline__ void latent_append_row(const LatentAppend &a, int m, 
     const float inv = 1.0f / sqrtf(sum / (float)a.R + a.eps);
     typename E::type *dst = (typename E::type *)a.slab + (page * PAGE_TOKENS + (t & (PAGE_TOKENS - 1))) * a.ldr;
     for (int r = threadIdx.x; r < a.R; r += THREADS) dst[r] = E::pack(X::load(x + r) * inv * a.w[r]);
+}
+
+// rotation in halves: number i of a vector with number i + dims / 2, by position * freq[i], cos and sin times gain; what lies behind dims stays
+struct Rotation {
+    const float *freq;
+    int dims;
+    float gain;
+};
+// one row's projections -> its normed query latent (cq; nullptr: not made), and (own) its normed latent and rotated key part into the page
+struct LatentPrepArgs {
+    const void *raw;       // [M][ld] T: query latent [Q8], latent [R8], key part [T8]
+    int ld, M, Q, Q8, R, R8, T, T8;
+    const float *q_norm, *c_norm;  // q_norm nullable: no weight
+    float eps;
+    Rotation rot;
+    bool own;
+    const int *pos, *row_seq, *table;
+    int table_width, n_pages, n_seqs;
+    void *cq;              // [M][ldc] T
+    int ldc;
+    void *slab;            // [n_pages][64][R8 + T8]
+};
+// the heads' vectors of every row, in place: row m, head h at q + m * ld + h * stride
+struct RotateArgs {
+    void *q;
+    int ld, stride, H, M;
+    Rotation rot;
+    const int *pos;
+};
+template <class E>
+__device__ __forceinline__ void rotate_pair(const typename E::type *u, const typename E::type *v, typename E::type *du, typename E::type *dv, float s, float c) {
+    const float a = E::load(u), b = E::load(v);
+    *du = E::pack(a * c - b * s), *dv = E::pack(b * c + a * s);
+}
+// row m's latent and key part into its page
+template <class E, int THREADS>
+__device__ __forceinline__ void latent_cache_row(const LatentPrepArgs &a, int m, float *red) {  // red: THREADS / 64 floats of LDS
+    typedef typename E::type T;
+    const T *c = (const T *)a.raw + (size_t)m * a.ld + a.Q8, *k = c + a.R8;
+    const int t = a.pos[m];
+    float ss = 0.0f;
+    for (int i = threadIdx.x; i < a.R; i += THREADS) ss = fmaf(E::load(c + i), E::load(c + i), ss);
+    ss = lanes_sum(ss);
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
+    const size_t page = min((unsigned)a.table[(size_t)min(a.row_seq[m], a.n_seqs - 1) * a.table_width + min(t / PAGE_TOKENS, a.table_width - 1)], (unsigned)a.n_pages - 1u);
+    T *row = (T *)a.slab + (page * PAGE_TOKENS + (t & (PAGE_TOKENS - 1))) * (a.R8 + a.T8), *rot = row + a.R8;
+    const int half = a.rot.dims / 2;
+    for (int i = threadIdx.x; i < half; i += THREADS) {
+        float s, co;
+        stack_sincos<sizeof(T) == 4>((float)t * a.rot.freq[i], s, co);
+        rotate_pair<E>(k + i, k + half + i, rot + i, rot + half + i, s * a.rot.gain, co * a.rot.gain);
+    }
+    for (int i = 2 * half + threadIdx.x; i < a.T; i += THREADS) rot[i] = k[i];
+    __syncthreads();
+    float sum = red[0];
+#pragma unroll
+    for (int i = 1; i < THREADS / 64; ++i) sum += red[i];
+    const float inv = 1.0f / sqrtf(sum / (float)a.R + a.eps);
+    for (int i = threadIdx.x; i < a.R; i += THREADS) row[i] = E::pack(E::load(c + i) * inv * a.c_norm[i]);
+}
+// all heads of row m; a thread keeps one pair's angle for the heads it takes
+template <class E, int THREADS>
+__device__ __forceinline__ void rotate_row(const RotateArgs &a, int m) {
+    typedef typename E::type T;
+    const int half = a.rot.dims / 2;
+    int lanes = 1;
+    while (lanes < half && lanes < THREADS) lanes <<= 1;
+    const float t = (float)a.pos[m];
+    for (int i = threadIdx.x & (lanes - 1); i < half; i += lanes) {
+        float s, c;
+        stack_sincos<sizeof(T) == 4>(t * a.rot.freq[i], s, c);
+        s *= a.rot.gain, c *= a.rot.gain;
+        for (int h = threadIdx.x / lanes; h < a.H; h += THREADS / lanes) {
+            T *p = (T *)a.q + (size_t)m * a.ld + h * a.stride + i;
+            rotate_pair<E>(p, p + half, p, p + half, s, c);
+        }
+    }
 }
 
 // ---------------------------------------------------------------- the attention's key splits
@@ -220,7 +301,12 @@ struct RowsArgs {
     void *h;               // [M][ldh]
     int ldh;
     LatentMerge merge;     // merge.splits > 0 (batched over heads, bf16, at most MERGE_ROWS rows): x is merged from the attention's key splits on the way in
-    LatentAppend append;   // append.M > 0: the last blockIdx.y does this instead (it needs the same input and would otherwise be a launch of its own)
+    bool x_norm;           // every row of x over its root mean square on the way in (fp32; with x_eps; ungrouped, bf16, at most 16 rows)
+    float x_eps;
+    // What rides along (M > 0) on blockIdx.y past the batches: it needs what this launch needs and would otherwise be launches of its own
+    LatentAppend append;
+    LatentPrepArgs cache;  // (the latent and key part only)
+    RotateArgs rotate;     // (numbers of the same rows that this product does not read)
 };
 // batches: blockIdx.y extent (1 for a plain Linear; heads; active experts (+ 1 with a shared expert))
 int rows_gemm_launch(int dtype, const RowsArgs &a, int batches, hipStream_t st);
@@ -258,34 +344,7 @@ int latent_attn_tiles(int n_rows, int H);
 size_t latent_attn_ws_floats(int M, int H, int R, int splits);
 int latent_append_launch(int dtype, const LatentAppend &a, hipStream_t st);
 
-// rotation in halves: number i of a vector with number i + dims / 2, by position * freq[i], cos and sin times gain; what lies behind dims stays
-struct Rotation {
-    const float *freq;
-    int dims;
-    float gain;
-};
-// one row's projections -> its normed query latent, and (own) its normed latent and rotated key part into the page
-struct LatentPrepArgs {
-    const void *raw;       // [M][ld] T: query latent [Q8], latent [R8], key part [T8]
-    int ld, M, Q, Q8, R, R8, T, T8;
-    const float *q_norm, *c_norm;
-    float eps;
-    Rotation rot;
-    bool own;
-    const int *pos, *row_seq, *table;
-    int table_width, n_pages, n_seqs;
-    void *cq;              // [M][ldc] T
-    int ldc;
-    void *slab;            // [n_pages][64][R8 + T8]
-};
 int latent_prep_launch(int dtype, const LatentPrepArgs &a, hipStream_t st);
-// the heads' vectors of every row, in place: row m, head h at q + m * ld + h * stride
-struct RotateArgs {
-    void *q;
-    int ld, stride, H, M;
-    Rotation rot;
-    const int *pos;
-};
 int rotate_heads_launch(int dtype, const RotateArgs &a, hipStream_t st);
 
 // ---------------------------------------------------------------- attention of long runs, keys and values spelled out (window_attn.hip)

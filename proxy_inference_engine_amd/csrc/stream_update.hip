@@ -172,7 +172,7 @@ __global__ void __launch_bounds__(THREADS) k_stream_update(const StreamUpdateArg
 }
 
 // ---------------------------------------------------------------- the convolution over longer runs
-constexpr int CONV_ROWS = 32;
+constexpr int CONV_ROWS = 16;
 
 // TAPS: taps at most.  A thread owns four columns and walks CONV_ROWS rows of one run with the last inputs in registers; the run's first tile carries the state.
 template <class E, int TAPS>
@@ -199,11 +199,17 @@ __global__ void __launch_bounds__(256) k_conv(const ConvArgs a, const typename E
         const int n_rows = a.runs[c.run].n_rows;
         for (int j = 0; j < taps - 1; ++j) *(float4 *)(held + (size_t)j * W4) = at(n_rows - (taps - 1) + j);  // (an older place is read before it is written)
     }
-#pragma unroll 4
-    for (int i = 0; i < c.n; ++i) {
+    constexpr int AHEAD = 8;  // rows in flight
+    float4 x[AHEAD];
+#pragma unroll
+    for (int i = 0; i < CONV_ROWS; ++i) {
+        if (i % AHEAD == 0)
+#pragma unroll
+            for (int k = 0; k < AHEAD; ++k) x[k] = load_h4<E>(hc + (size_t)(c.row0 + min(i + k, c.n - 1)) * ldh + n);
+        if (i >= c.n) break;
 #pragma unroll
         for (int j = 0; j + 1 < TAPS; ++j) v[j] = v[j + 1];
-        v[TAPS - 1] = load_h4<E>(hc + (size_t)(c.row0 + i) * ldh + n);
+        v[TAPS - 1] = x[i % AHEAD];
         float4 y = fma4(w[TAPS - 1], v[TAPS - 1], v[TAPS - 1]);
 #pragma unroll
         for (int j = 0; j + 1 < TAPS; ++j) y = fma4(w[j], v[j], y);

@@ -124,10 +124,13 @@ class Model(LayerStackModel):
                 down = get(p + "dkv", R + T, W)
                 rows += [pad(down[:R], up8(R), W), pad(down[R:], up8(T), W)]
             rows.append(pad(get(p + "g", H, W), up8(H), W))
-            up = get(p + "uq", H * (D + T), Q).view(H, D + T, Q)
+            q_norm, up = flat(p + "dq.norm", Q), get(p + "uq", H * (D + T), Q)
+            if dtype == torch.bfloat16:  # the norm's weight goes into the matrix behind it: few rows are normed on their way into that product
+                q_norm, up = None, (up.float() * q_norm).to(torch.bfloat16)
+            up = up.view(H, D + T, Q)
             uk, uv = get(p + "uk", H * D, R), get(p + "uv", H * V, R)
             out = {"mixer": _ffi.PIE_MIXER_LATENT, "heads": H, "dim": D, "vdim": V, "rank": R, "q_rank": Q, "rot_dim": T, "kv_from": -1 if own else m.kv_from, "scale": m.scale,
-                   "out_gate": 1, "head_sink": flat(p + "sink", H), "w_in": pack(torch.cat(rows)), "q_norm": flat(p + "dq.norm", Q),
+                   "out_gate": 1, "head_sink": flat(p + "sink", H), "w_in": pack(torch.cat(rows)), "q_norm": q_norm,
                    "w_uq": pack(torch.cat([pad_head_rows(up[:, :D].flatten(0, 1), H, D), pad_head_rows(up[:, D:].flatten(0, 1), H, T)])),
                    "w_uk": pack(uk.view(H, D, R).transpose(1, 2)), "w_uv": pack(uv.view(H, V, R)), "w_kv": pack(torch.cat([pad_head_rows(uk, H, D), pad_head_rows(uv, H, V)])),
                    "w_o": pack(pad_head_columns(get(p + "o", W, H * V), H, V))}
