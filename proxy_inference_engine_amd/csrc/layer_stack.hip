@@ -443,7 +443,7 @@ int stack_reserve(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
         if (L.mixer == PIE_MIXER_DELTA || L.mixer == PIE_MIXER_MLSTM || L.mixer == PIE_MIXER_MINGRU) {
             const int chunks = chunk_part(s, b, L).chunks;
             if (chunks && L.mixer == PIE_MIXER_DELTA) rw = std::max(rw, delta_ws_floats(chunks, L.heads, L.dim)), ro = std::max(ro, (size_t)L.heads * up8(L.dim));
-            else if (chunks && L.mixer == PIE_MIXER_MLSTM) rw = std::max(rw, mlstm_ws_floats(chunks, L.heads, L.dim));
+            else if (chunks && L.mixer == PIE_MIXER_MLSTM) rw = std::max(rw, mlstm_ws_floats(chunks, L.heads, L.dim, L.vdim));
             else if (chunks) rw = std::max(rw, mingru_ws_floats(chunks, L.dim));
         }
         if (is_dense(L)) {

@@ -11,7 +11,7 @@
 // Chunk form, 64 tokens at a time.  With b_t the sum of f inside the chunk, c_t = max over s <= t of (b_t - b_s + i_s), M and S in front of the chunk,
 //   m_t = max(M + b_t, c_t),   sums_t = e^(M + b_t - m_t) S^T q_t + e^(c_t - m_t) sum_{s <= t} P_ts v_s,   P_ts = e^(b_t - b_s + i_s - c_t) q_t . k_s
 //   S <- e^(M + b_L - m_L) S + e^(c_L - m_L) sum_s e^(b_L - b_s + i_s - c_L) k_s v_s^T
-// where no exponent is above zero.  One launch (all chunks of all heads in parallel) makes b, c, P and the key weights, and leaves q, k^T and P in matrix operand order; a
+// where no exponent is above zero.  One launch (all chunks of all heads in parallel) makes b, c, P and the key weights, and leaves q, k^T, v and P in matrix operand order; a
 // second walks the chunks, one workgroup per head and 16 value columns (and one per head for n: v = 1), whose four waves split the key channels of S.
 // q, k and v are bf16 numbers, so their products are exact in fp32; what meets them as an operand is fp32 split into bf16 parts: the weighted values that enter the
 // state in three (24 bits), P and the state where it is read in two.
@@ -138,8 +138,15 @@ __global__ void __launch_bounds__(256) k_mlstm_step(const MlstmArgs a) {
 
 // ---------------------------------------------------------------- chunk form
 __host__ __device__ __forceinline__ int ml_pairs(int D) { return (D + 31) / 32; }  // 32-channel steps of the keys
-// per (chunk, head), bytes: q [4 row tiles][pairs] KiB; k^T [pairs][2][2 token steps] KiB; P [4 row tiles][2 token steps][hi, lo] KiB; b, c, key weights [64] fp32
-__host__ __device__ __forceinline__ size_t ml_chunk_bytes(int D) { return (size_t)ml_pairs(D) * 8192 + 16384 + 3 * ML * 4; }
+// per (chunk, head), bytes: q [4 row tiles][pairs] KiB; k^T [pairs][2][2 token steps] KiB; P [4 row tiles][2 token steps][hi, lo] KiB; b, c, key weights [64] fp32 in a KiB;
+// v [16-column blocks][2 token steps] KiB
+struct MlChunk {
+    size_t k, p, s, v, bytes;  // where they begin
+};
+__host__ __device__ __forceinline__ MlChunk ml_chunk(int D, int V) {
+    const size_t np = ml_pairs(D);
+    return {np * 4096, np * 8192, np * 8192 + 16384, np * 8192 + 17408, np * 8192 + 17408 + (size_t)ml_blocks(V) * 2048};
+}
 
 __device__ __forceinline__ ml_f32x4 ml_mfma(const uint4 &a, const uint4 &b, const ml_f32x4 &c) {
     return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(ml_bf16x8, a), __builtin_bit_cast(ml_bf16x8, b), c, 0, 0, 0);
@@ -151,19 +158,53 @@ __device__ __forceinline__ u32 ml_part(float &x, float &y) {
     return w;
 }
 
-// One workgroup per (chunk, head); wave w owns the chunk's rows 16 w .. + 15.
+constexpr int ML_VB = 4;  // 16-column blocks of v per wave
+// One workgroup per (chunk, head), wave w owning the chunk's rows 16 w .. + 15; behind them (blockIdx.z > 0) the ones that turn v round.
 __global__ void __launch_bounds__(256) k_mlstm_prep(const MlstmArgs a) {
     __shared__ __attribute__((aligned(16))) u16 s_p[2][ML][ML + 8];
     __shared__ __attribute__((aligned(16))) float s_b[ML], s_c[ML], s_g[ML];
+    constexpr int LV = 18;  // u16 per row of a transposed block: odd dwords
+    __shared__ __attribute__((aligned(16))) u16 s_v[4][ML * LV];  // (of the workgroups that turn v round)
     const int head = blockIdx.x, lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), n16 = lane & 15, q4 = lane >> 4;
     const RowChunk c = row_chunk(a.r.runs, a.r.n_runs, blockIdx.y, ML);
     if (c.n <= 0) return;
     const int np = ml_pairs(a.D), ld = a.r.ld;
-    char *ws = (char *)a.r.ws + ((size_t)blockIdx.y * a.H + head) * ml_chunk_bytes(a.D);
-    float *o_s = (float *)(ws + (size_t)np * 8192 + 16384);
+    const MlChunk at = ml_chunk(a.D, a.V);
+    char *ws = (char *)a.r.ws + ((size_t)blockIdx.y * a.H + head) * at.bytes;
+    float *o_s = (float *)(ws + at.s);
     const u16 *raw = (const u16 *)a.r.raw + (size_t)c.row0 * ld + head * a.D8, *rk = raw + a.H * a.D8;
     auto piece = [&](const u16 *p, int row, int d) { return d < a.D8 ? *(const uint4 *)(p + (size_t)min(row, c.n - 1) * ld + d) : make_uint4(0, 0, 0, 0); };
 
+    if (blockIdx.z) {
+        // v: operand (block b, token step s) has column 16 b + n16 in lane n16, tokens 32 s + 8 q4 ..; a wave takes a block's 64 rows (a row per lane) through LDS
+        const u16 *rv = (const u16 *)a.r.raw + (size_t)(c.row0 + min(lane, c.n - 1)) * ld + 2 * a.H * a.D8 + head * a.V8;
+        const int b0 = ((int)blockIdx.z - 1) * 4 * ML_VB + wave * ML_VB;
+        uint4 x[ML_VB][2];
+#pragma unroll
+        for (int j = 0; j < ML_VB; ++j)
+#pragma unroll
+            for (int h = 0; h < 2; ++h) x[j][h] = 16 * (b0 + j) + 8 * h < a.V8 ? *(const uint4 *)(rv + 16 * (b0 + j) + 8 * h) : make_uint4(0, 0, 0, 0);
+        u16 *t = s_v[wave];
+#pragma unroll
+        for (int j = 0; j < ML_VB; ++j) {
+            if (b0 + j >= ml_blocks(a.V)) break;
+#pragma unroll
+            for (int h = 0; h < 2; ++h) {
+                u32 *d = (u32 *)(t + lane * LV + 8 * h);
+                d[0] = x[j][h].x, d[1] = x[j][h].y, d[2] = x[j][h].z, d[3] = x[j][h].w;
+            }
+            asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // (a wave reads what it wrote)
+#pragma unroll
+            for (int s = 0; s < 2; ++s) {
+                u32 w[4];
+#pragma unroll
+                for (int i = 0; i < 4; ++i) w[i] = t[(32 * s + 8 * q4 + 2 * i) * LV + n16] | (u32)t[(32 * s + 8 * q4 + 2 * i + 1) * LV + n16] << 16;
+                *(uint4 *)(ws + at.v + (size_t)(2 * (b0 + j) + s) * 1024 + lane * 16) = make_uint4(w[0], w[1], w[2], w[3]);
+            }
+            asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+        }
+        return;
+    }
     if (wave == 0) {  // lane: token
         MlGates g = {ML_NEG, 0.0f};
         if (lane < c.n) g = ml_gates<u16>(a, c.row0 + lane, head);
@@ -195,7 +236,7 @@ __global__ void __launch_bounds__(256) k_mlstm_prep(const MlstmArgs a) {
         for (int k = 0; k < 8; ++k) v[k] = rk[(size_t)min(32 * s + 8 * q4 + k, c.n - 1) * ld + min(d, a.D8 - 1)];
         uint4 w = make_uint4(v[0] | (u32)v[1] << 16, v[2] | (u32)v[3] << 16, v[4] | (u32)v[5] << 16, v[6] | (u32)v[7] << 16);
         if (d >= a.D) w = make_uint4(0, 0, 0, 0);
-        *(uint4 *)(ws + (size_t)np * 4096 + (size_t)i * 1024 + lane * 16) = w;
+        *(uint4 *)(ws + at.k + (size_t)i * 1024 + lane * 16) = w;
     }
     __syncthreads();
     // rows 16 wave + 4 q4 + i, columns 16 t + n16
@@ -211,17 +252,19 @@ __global__ void __launch_bounds__(256) k_mlstm_prep(const MlstmArgs a) {
         }
     // (a wave reads the rows it wrote)
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-    char *o_p = ws + (size_t)np * 8192 + (size_t)wave * 4096;
+    char *o_p = ws + at.p + (size_t)wave * 4096;
 #pragma unroll
     for (int s = 0; s < 2; ++s)
 #pragma unroll
         for (int k = 0; k < 2; ++k) *(uint4 *)(o_p + (s * 2 + k) * 1024 + lane * 16) = *(const uint4 *)&s_p[k][16 * wave + n16][32 * s + 8 * q4];
 }
 
-// NPW: 32-channel pairs per wave (D <= 128 NPW).  A chunk's operands are loaded where the previous chunk's have just been used.
+// NPW: 32-channel pairs per wave (D <= 128 NPW).  A chunk's operands are loaded where the previous chunk's have just been used, out of the L2: a head's workgroups share
+// the reading of the chunk behind that from further away, a line per thread (into LDS that nobody reads).
 template <int NPW>
 __global__ void __launch_bounds__(256, NPW <= 2 ? 2 : 1) k_mlstm_scan(const MlstmArgs a) {
     __shared__ __attribute__((aligned(16))) ml_f32x4 s_o[2][4][4][64];
+    __shared__ __attribute__((aligned(1024))) char s_warm[1024];
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), n16 = lane & 15, q4 = lane >> 4;
     const int head = (int)blockIdx.x % a.H, cb = (int)blockIdx.x / a.H, blocks = ml_blocks(a.V), V4 = ml_up4(a.V), D = a.D, np = ml_pairs(D);  // (head fastest: a head's columns share an L2 where H is a multiple of 8)
     const bool has_n = cb == blocks;  // this workgroup carries n
@@ -249,12 +292,13 @@ __global__ void __launch_bounds__(256, NPW <= 2 ? 2 : 1) k_mlstm_scan(const Mlst
                 S[j][e][i] = !fresh && p ? *p : 0.0f;
             }
     float m = fresh ? 0.0f : st.m[cb];
-    const size_t per = ml_chunk_bytes(D), step = per * a.H;
-    const char *ws0 = (const char *)a.r.ws + ((size_t)chunk0 * a.H + head) * per;
-    const u16 *rv = (const u16 *)a.r.raw + (size_t)run.row0 * a.r.ld + 2 * a.H * a.D8 + head * a.V8 + min(col, a.V - 1);
+    const MlChunk place_of = ml_chunk(D, a.V);
+    const size_t step = place_of.bytes * a.H;
+    const char *ws0 = (const char *)a.r.ws + ((size_t)chunk0 * a.H + head) * place_of.bytes;
     uint4 q[4][NPW], k[NPW][2][2], p[2][2];
-    u16 v[16];
-    float nb, nc, nw;
+    uint4 v[2];
+    ml_f32x4 w[2][2], nb, nc;  // key weights of the lane's tokens; b and c of its output rows
+    float nbl, ncl;
     auto load_q = [&](int ch) {
         const char *ws = ws0 + (size_t)min(ch, chunks - 1) * step + lane * 16;
 #pragma unroll
@@ -263,7 +307,7 @@ __global__ void __launch_bounds__(256, NPW <= 2 ? 2 : 1) k_mlstm_scan(const Mlst
             for (int j = 0; j < NPW; ++j) q[t][j] = *(const uint4 *)(ws + ((size_t)t * np + min(wave * NPW + j, np - 1)) * 1024);
     };
     auto load_k = [&](int ch) {
-        const char *ws = ws0 + (size_t)min(ch, chunks - 1) * step + (size_t)np * 4096 + lane * 16;
+        const char *ws = ws0 + (size_t)min(ch, chunks - 1) * step + place_of.k + lane * 16;
 #pragma unroll
         for (int j = 0; j < NPW; ++j)
 #pragma unroll
@@ -272,25 +316,35 @@ __global__ void __launch_bounds__(256, NPW <= 2 ? 2 : 1) k_mlstm_scan(const Mlst
                 for (int s = 0; s < 2; ++s) k[j][e][s] = *(const uint4 *)(ws + (size_t)(4 * min(wave * NPW + j, np - 1) + 2 * e + s) * 1024);
     };
     auto load_pv = [&](int ch) {
-        const int c = min(ch, chunks - 1);
-        const char *ws = ws0 + (size_t)c * step + (size_t)np * 8192 + wave * 4096 + lane * 16;
+        const char *ws = ws0 + (size_t)min(ch, chunks - 1) * step + lane * 16;
 #pragma unroll
-        for (int s = 0; s < 2; ++s)
+        for (int s = 0; s < 2; ++s) {
 #pragma unroll
-            for (int h = 0; h < 2; ++h) p[s][h] = *(const uint4 *)(ws + (s * 2 + h) * 1024);
+            for (int h = 0; h < 2; ++h) p[s][h] = *(const uint4 *)(ws + place_of.p + wave * 4096 + (s * 2 + h) * 1024);
+            v[s] = *(const uint4 *)(ws + place_of.v + (size_t)(2 * min(cb, blocks - 1) + s) * 1024);
 #pragma unroll
-        for (int i = 0; i < 16; ++i) v[i] = rv[(size_t)min(ML * c + 32 * (i >> 3) + 8 * q4 + (i & 7), run.n_rows - 1) * a.r.ld];
+            for (int h = 0; h < 2; ++h) w[s][h] = *(const ml_f32x4 *)((const float *)(ws - lane * 16 + place_of.s) + 2 * ML + 32 * s + 8 * q4 + 4 * h);
+        }
     };
     auto load_scalars = [&](int ch) {
-        const float *sc = (const float *)(ws0 + (size_t)min(ch, chunks - 1) * step + (size_t)np * 8192 + 16384);
-        nb = sc[lane], nc = sc[ML + lane], nw = sc[2 * ML + lane];
+        const float *sc = (const float *)(ws0 + (size_t)min(ch, chunks - 1) * step + place_of.s);
+        nb = *(const ml_f32x4 *)(sc + 16 * wave + 4 * q4), nc = *(const ml_f32x4 *)(sc + ML + 16 * wave + 4 * q4), nbl = sc[ML - 1], ncl = sc[2 * ML - 1];
     };
-    load_scalars(0), load_q(0), load_pv(0), load_k(0);
+    const unsigned line = (unsigned)min((cb * 256 + (int)threadIdx.x) * 128, (int)place_of.bytes - 4) & ~3u, warm_lds = (unsigned)(size_t)(__attribute__((address_space(3))) void *)s_warm + 256u * wave;
+    auto warm = [&](int ch) {
+        const unsigned long long v = (unsigned long long)(uintptr_t)(ws0 + (size_t)min(ch, chunks - 1) * step);
+        const unsigned long long src =
+            (unsigned long long)(unsigned)__builtin_amdgcn_readfirstlane((int)(unsigned)v) | ((unsigned long long)(unsigned)__builtin_amdgcn_readfirstlane((int)(unsigned)(v >> 32)) << 32);
+        unsigned keep;
+        asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %3\n\ts_nop 0\n\tglobal_load_lds_dword %1, %2\n\ts_mov_b32 m0, %0" : "=&s"(keep) : "v"(line), "s"(src), "s"(warm_lds) : "memory");
+    };
+    load_scalars(0), load_q(0), load_pv(0), load_k(0), warm(1);
     const ml_f32x4 zero = {0.0f, 0.0f, 0.0f, 0.0f};
     for (int ch = 0; ch < chunks; ++ch) {
-        const float cb_ = nb, cc = nc, cw = nw;
+        const ml_f32x4 cbv = nb, ccv = nc;
+        const float bl = nbl, cl = ncl;
         load_scalars(ch + 1);
-        const float bl = __shfl(cb_, 63, 64), cl = __shfl(cc, 63, 64), next = fmaxf(m + bl, cl), keep = stack_exp<false>(m + bl - next), add = stack_exp<false>(cl - next);
+        const float next = fmaxf(m + bl, cl), keep = stack_exp<false>(m + bl - next), add = stack_exp<false>(cl - next);
         // S^T q of the chunk's 64 rows: the wave's channels
         ml_f32x4 acc[4] = {zero, zero, zero, zero};
 #pragma unroll
@@ -315,15 +369,15 @@ __global__ void __launch_bounds__(256, NPW <= 2 ? 2 : 1) k_mlstm_scan(const Mlst
         float f[2][8];
 #pragma unroll
         for (int s = 0; s < 2; ++s) {
-            u32 w[4];
+            u32 x[4] = {v[s].x, v[s].y, v[s].z, v[s].w};
 #pragma unroll
-            for (int i = 0; i < 4; ++i) w[i] = has_n ? 0x3F803F80u : (u32)v[8 * s + 2 * i] | (u32)v[8 * s + 2 * i + 1] << 16;  // (n: v = 1)
+            for (int i = 0; i < 4; ++i) x[i] = has_n ? 0x3F803F80u : x[i];  // (n: v = 1)
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
-                f[s][2 * i] = lo_f32<BF16>(w[i]) * (add * __shfl(cw, 32 * s + 8 * q4 + 2 * i, 64));
-                f[s][2 * i + 1] = hi_f32<BF16>(w[i]) * (add * __shfl(cw, 32 * s + 8 * q4 + 2 * i + 1, 64));
+                f[s][2 * i] = lo_f32<BF16>(x[i]) * (add * w[s][i >> 1][2 * (i & 1)]);
+                f[s][2 * i + 1] = hi_f32<BF16>(x[i]) * (add * w[s][i >> 1][2 * (i & 1) + 1]);
             }
-            const uint4 vv = make_uint4(w[0], w[1], w[2], w[3]);
+            const uint4 vv = make_uint4(x[0], x[1], x[2], x[3]);
             own = ml_mfma(p[s][0], vv, own), own = ml_mfma(p[s][1], vv, own);
         }
         load_pv(ch + 1);
@@ -336,16 +390,17 @@ __global__ void __launch_bounds__(256, NPW <= 2 ? 2 : 1) k_mlstm_scan(const Mlst
         for (int s = 0; s < 2; ++s)
 #pragma unroll
             for (int h = 0; h < 3; ++h) {
-                u32 w[4];
+                u32 x[4];
 #pragma unroll
-                for (int i = 0; i < 4; ++i) w[i] = ml_part(f[s][2 * i], f[s][2 * i + 1]);
-                const uint4 part = make_uint4(w[0], w[1], w[2], w[3]);
+                for (int i = 0; i < 4; ++i) x[i] = ml_part(f[s][2 * i], f[s][2 * i + 1]);
+                const uint4 part = make_uint4(x[0], x[1], x[2], x[3]);
 #pragma unroll
                 for (int j = 0; j < NPW; ++j)
 #pragma unroll
                     for (int e = 0; e < 2; ++e) S[j][e] = ml_mfma(k[j][e][s], part, S[j][e]);
             }
         load_k(ch + 1);
+        warm(ch + 2);
 #pragma unroll
         for (int j = 0; j < NPW; ++j)
             if (wave * NPW + j >= np) S[j][0] = S[j][1] = zero;  // (channels that do not exist saw another pair's keys)
@@ -354,10 +409,8 @@ __global__ void __launch_bounds__(256, NPW <= 2 ? 2 : 1) k_mlstm_scan(const Mlst
         float o[4], mt[4];
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-            const int t = 16 * wave + 4 * q4 + i;
-            const float b = __shfl(cb_, t, 64), c = __shfl(cc, t, 64);
-            mt[i] = fmaxf(m + b, c);
-            o[i] = fmaf(a.scale * stack_exp<false>(m + b - mt[i]), all[i], stack_exp<false>(c - mt[i]) * own[i]);
+            mt[i] = fmaxf(m + cbv[i], ccv[i]);
+            o[i] = fmaf(a.scale * stack_exp<false>(m + cbv[i] - mt[i]), all[i], stack_exp<false>(ccv[i] - mt[i]) * own[i]);
         }
         const int t0 = ML * ch + 16 * wave + 4 * q4;
         const size_t at = ((size_t)run.row0 + t0) * a.H + head;
@@ -366,10 +419,17 @@ __global__ void __launch_bounds__(256, NPW <= 2 ? 2 : 1) k_mlstm_scan(const Mlst
 #pragma unroll
                 for (int i = 0; i < 4; ++i)
                     if (t0 + i < run.n_rows) a.den[at + (size_t)i * a.H] = fmaxf(fabsf(o[i]), stack_exp<false>(-mt[i])) + a.den_eps;
-        } else if (col < a.V)
+        } else if (col < a.V) {
+            float *dst = a.o + at * a.V8 + col;
+            const int row = a.H * a.V8;
+            if (ML * (ch + 1) <= run.n_rows)
 #pragma unroll
-            for (int i = 0; i < 4; ++i)
-                if (t0 + i < run.n_rows) a.o[(at + (size_t)i * a.H) * a.V8 + col] = o[i];
+                for (int i = 0; i < 4; ++i) dst[i * row] = o[i];
+            else
+#pragma unroll
+                for (int i = 0; i < 4; ++i)
+                    if (t0 + i < run.n_rows) dst[i * row] = o[i];
+        }
         m = next;
     }
 #pragma unroll
@@ -380,6 +440,7 @@ __global__ void __launch_bounds__(256, NPW <= 2 ? 2 : 1) k_mlstm_scan(const Mlst
             for (int i = 0; i < 4; ++i)
                 if (float *x = place(j, e, i)) *x = S[j][e][i];
     if (threadIdx.x == 0) st.m[cb] = m;
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // (what was read ahead: LDS is handed on when the workgroup ends)
 }
 
 int mlstm_check(const MlstmArgs &a) {
@@ -405,7 +466,7 @@ void mlstm_step_go(const MlstmArgs &a, hipStream_t st) {
 
 size_t mlstm_state_floats(int H, int D, int V) { return (size_t)H * D * ml_up4(V) + (size_t)H * ml_up4(D) + (size_t)H * (ml_blocks(V) + 1); }
 int mlstm_chunks(int n_rows) { return (n_rows + ML - 1) / ML; }
-size_t mlstm_ws_floats(int chunks, int H, int D) { return (size_t)chunks * H * ml_chunk_bytes(D) / 4; }
+size_t mlstm_ws_floats(int chunks, int H, int D, int V) { return (size_t)chunks * H * ml_chunk(D, V).bytes / 4; }
 
 int mlstm_step_launch(int dtype, const MlstmArgs &a, hipStream_t st) {
     if (a.r.n_runs <= 0) return PIE_OK;
@@ -420,7 +481,7 @@ int mlstm_chunks_launch(const MlstmArgs &a, int chunks, hipStream_t st) {
     if (a.r.n_runs <= 0) return PIE_OK;
     if (const int rc = mlstm_check(a)) return rc;
     PIE_REQUIRE(a.r.ws && chunks > 0 && chunks <= 65535 && a.D <= MLSTM_CHUNK_MAX_DIM, PIE_E_ARG, "mLSTM: the chunk form needs its workspace, and keys of at most 512 channels");
-    hipLaunchKernelGGL(k_mlstm_prep, dim3((unsigned)a.H, (unsigned)chunks), dim3(256), 0, st, a);
+    hipLaunchKernelGGL(k_mlstm_prep, dim3((unsigned)a.H, (unsigned)chunks, (unsigned)(1 + (ml_blocks(a.V) + 4 * ML_VB - 1) / (4 * ML_VB))), dim3(256), 0, st, a);
     PIE_LAUNCH_CHECK();
     const dim3 grid((unsigned)(a.H * (ml_blocks(a.V) + 1)), (unsigned)a.r.n_runs);
     if (a.D <= 128) hipLaunchKernelGGL(k_mlstm_scan<1>, grid, dim3(256), 0, st, a);

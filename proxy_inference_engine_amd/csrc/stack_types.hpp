@@ -537,7 +537,7 @@ size_t mlstm_state_floats(int H, int D, int V);
 int mlstm_step_launch(int dtype, const MlstmArgs &a, hipStream_t st);       // token by token
 int mlstm_chunks_launch(const MlstmArgs &a, int chunks, hipStream_t st);   // runs of many tokens (bf16)
 int mlstm_chunks(int n_rows);
-size_t mlstm_ws_floats(int chunks, int H, int D);
+size_t mlstm_ws_floats(int chunks, int H, int D, int V);
 
 // ---------------------------------------------------------------- x += post(y); h = next(x) with norms that need the whole row (row_update.hip)
 struct StackNorm {

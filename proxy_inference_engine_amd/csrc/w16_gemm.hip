@@ -96,7 +96,9 @@ static W16Plan w16_plan(int M, int N, int K, bool no_split = false) {
     double best_us = 1e30;
     // t(mb, sw) = light + (full - light) * load: one partial round of workgroups runs at a higher clock than sustained full rounds
     static const double t_light[4][3] = {{0, 0, 0}, {0, 0.25, 0.42}, {0, 0.31, 0.60}, {0, 0.50, 1.45}};  // [log2 mb][sw]
-    static const double t_full[4][3] = {{0, 0, 0}, {0, 0.25, 0.45}, {0, 0.48, 0.80}, {0, 0.83, 1.45}};
+    static const double t_rows[4][3] = {{0, 0, 0}, {0, 0.25, 0.45}, {0, 0.48, 0.80}, {0, 0.83, 1.45}};
+    static const double t_tall[4][3] = {{0, 0, 0}, {0, 0.31, 0.53}, {0, 0.46, 0.84}, {0, 0.90, 1.45}};  // many row tiles: small tiles re-read the weights from beyond their XCD's L2
+    const double (&t_full)[4][3] = M > 512 ? t_tall : t_rows;
     const double stream_us = 2.0 * N * (64.0 * groups) / 5.5e6;
     for (int S = 1; S <= (no_split ? 1 : 16) && (S == 1 || 8 * S <= groups); ++S)
         for (int mb = mb_max; mb >= 2; mb >>= 1)
