@@ -828,7 +828,7 @@ void mlstm_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next, in
     if (cp.runs) p.rc = mlstm_step_launch(dt, m, p.st), ++p.launches;
     if (!p.rc && cp.chunks) {
         m.r.runs += cp.runs, m.r.n_runs = b.n_runs - cp.runs;
-        p.rc = mlstm_chunks_launch(m, cp.chunks, p.st), p.launches += 2;
+        p.rc = mlstm_chunks_launch(m, cp.chunks, p.st), p.launches += 4;
     }
     const HeadOutArgs h = {s->rec_o.p, s->rec_den.p, (const char *)s->q.p + (size_t)H * (2 * D8 + V8) * esize(s), nullptr, NI, H, L.vdim, V8, L.o_norm, L.eps, s->o.p, LO};
     if (!p.rc) p.rc = head_out_launch(dt, h, 0, b.n_rows, p.st), ++p.launches;

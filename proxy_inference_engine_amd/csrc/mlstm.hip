@@ -11,10 +11,12 @@
 // Chunk form, 64 tokens at a time.  With b_t the sum of f inside the chunk, c_t = max over s <= t of (b_t - b_s + i_s), M and S in front of the chunk,
 //   m_t = max(M + b_t, c_t),   sums_t = e^(M + b_t - m_t) S^T q_t + e^(c_t - m_t) sum_{s <= t} P_ts v_s,   P_ts = e^(b_t - b_s + i_s - c_t) q_t . k_s
 //   S <- e^(M + b_L - m_L) S + e^(c_L - m_L) sum_s e^(b_L - b_s + i_s - c_L) k_s v_s^T
-// where no exponent is above zero.  One launch (all chunks of all heads in parallel) makes b, c, P and the key weights, and leaves q, k^T, v and P in matrix operand order; a
-// second walks the chunks, one workgroup per head and 16 value columns (and one per head for n: v = 1), whose four waves split the key channels of S.
+// where no exponent is above zero.  One launch (all chunks of all heads in parallel) makes b, c, P and the key weights, and leaves q, k^T, v and P in matrix operand order; one
+// walks the chunks, a workgroup per head and 16 value columns, whose four waves split the key channels of S.  n is chained by a launch of its own (its additions are known
+// beforehand: k summed with its weights), and the denominators follow from it, all chunks in parallel.
 // q, k and v are bf16 numbers, so their products are exact in fp32; what meets them as an operand is fp32 split into bf16 parts: the weighted values that enter the
 // state in three (24 bits), P and the state where it is read in two.
+#include "mfma_store.hpp"  // w4m_pack
 #include "stack_types.hpp"
 
 typedef __attribute__((ext_vector_type(4))) float ml_f32x4;
@@ -138,14 +140,15 @@ __global__ void __launch_bounds__(256) k_mlstm_step(const MlstmArgs a) {
 
 // ---------------------------------------------------------------- chunk form
 __host__ __device__ __forceinline__ int ml_pairs(int D) { return (D + 31) / 32; }  // 32-channel steps of the keys
-// per (chunk, head), bytes: q [4 row tiles][pairs] KiB; k^T [pairs][2][2 token steps] KiB; P [4 row tiles][2 token steps][hi, lo] KiB; b, c, key weights [64] fp32 in a KiB;
-// v [16-column blocks][2 token steps] KiB
+// per (chunk, head), bytes: q [4 row tiles][pairs] KiB; k^T [pairs][2][2 token steps] KiB; P [4 row tiles][2 token steps][hi, lo] KiB; b, c, key weights, sums of P's rows [64]
+// fp32 each; v [16-column blocks][2 token steps] KiB; [32 pairs] fp32 k summed with its weights (once chained: n in front of the chunk) and the maximum in front of it
 struct MlChunk {
-    size_t k, p, s, v, bytes;  // where they begin
+    size_t k, p, s, v, n, bytes;  // where they begin
 };
 __host__ __device__ __forceinline__ MlChunk ml_chunk(int D, int V) {
     const size_t np = ml_pairs(D);
-    return {np * 4096, np * 8192, np * 8192 + 16384, np * 8192 + 17408, np * 8192 + 17408 + (size_t)ml_blocks(V) * 2048};
+    const size_t n = np * 8192 + 17408 + (size_t)ml_blocks(V) * 2048;
+    return {np * 4096, np * 8192, np * 8192 + 16384, np * 8192 + 17408, n, n + np * 128 + 128};
 }
 
 __device__ __forceinline__ ml_f32x4 ml_mfma(const uint4 &a, const uint4 &b, const ml_f32x4 &c) {
@@ -153,7 +156,7 @@ __device__ __forceinline__ ml_f32x4 ml_mfma(const uint4 &a, const uint4 &b, cons
 }
 // two fp32 numbers -> their leading bf16 parts; what is left stays in (x, y)
 __device__ __forceinline__ u32 ml_part(float &x, float &y) {
-    const u32 w = pack2<BF16>(x, y);
+    const u32 w = w4m_pack<BF16>(x, y);
     x -= lo_f32<BF16>(w), y -= hi_f32<BF16>(w);
     return w;
 }
@@ -161,10 +164,9 @@ __device__ __forceinline__ u32 ml_part(float &x, float &y) {
 constexpr int ML_VB = 4;  // 16-column blocks of v per wave
 // One workgroup per (chunk, head), wave w owning the chunk's rows 16 w .. + 15; behind them (blockIdx.z > 0) the ones that turn v round.
 __global__ void __launch_bounds__(256) k_mlstm_prep(const MlstmArgs a) {
-    __shared__ __attribute__((aligned(16))) u16 s_p[2][ML][ML + 8];
-    __shared__ __attribute__((aligned(16))) float s_b[ML], s_c[ML], s_g[ML];
-    constexpr int LV = 18;  // u16 per row of a transposed block: odd dwords
-    __shared__ __attribute__((aligned(16))) u16 s_v[4][ML * LV];  // (of the workgroups that turn v round)
+    constexpr int LP = ML + 8, LV = 16 * ML_VB + 2;  // u16 per row of P's parts, and of what is turned round (odd dwords)
+    __shared__ __attribute__((aligned(16))) u16 s_t[2 * ML * LP > 4 * ML * LV ? 2 * ML * LP : 4 * ML * LV];
+    __shared__ __attribute__((aligned(16))) float s_b[ML], s_c[ML], s_g[ML], s_w[ML];
     const int head = blockIdx.x, lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), n16 = lane & 15, q4 = lane >> 4;
     const RowChunk c = row_chunk(a.r.runs, a.r.n_runs, blockIdx.y, ML);
     if (c.n <= 0) return;
@@ -176,32 +178,30 @@ __global__ void __launch_bounds__(256) k_mlstm_prep(const MlstmArgs a) {
     auto piece = [&](const u16 *p, int row, int d) { return d < a.D8 ? *(const uint4 *)(p + (size_t)min(row, c.n - 1) * ld + d) : make_uint4(0, 0, 0, 0); };
 
     if (blockIdx.z) {
-        // v: operand (block b, token step s) has column 16 b + n16 in lane n16, tokens 32 s + 8 q4 ..; a wave takes a block's 64 rows (a row per lane) through LDS
-        const u16 *rv = (const u16 *)a.r.raw + (size_t)(c.row0 + min(lane, c.n - 1)) * ld + 2 * a.H * a.D8 + head * a.V8;
-        const int b0 = ((int)blockIdx.z - 1) * 4 * ML_VB + wave * ML_VB;
-        uint4 x[ML_VB][2];
+        // v: operand (block b, token step s) has column 16 b + n16 in lane n16, tokens 32 s + 8 q4 ..; a wave turns 64 columns of the 64 rows round in LDS
+        const int b0 = ((int)blockIdx.z - 1) * 4 * ML_VB + wave * ML_VB, col = 16 * b0 + 8 * (lane & 7);
+        if (b0 >= ml_blocks(a.V)) return;
+        const u16 *rv = (const u16 *)a.r.raw + (size_t)c.row0 * ld + 2 * a.H * a.D8 + head * a.V8 + col;
+        uint4 x[8];
 #pragma unroll
-        for (int j = 0; j < ML_VB; ++j)
+        for (int i = 0; i < 8; ++i) x[i] = col < a.V8 ? *(const uint4 *)(rv + (size_t)min(8 * i + (lane >> 3), c.n - 1) * ld) : make_uint4(0, 0, 0, 0);
+        u16 *t = s_t + wave * ML * LV;
 #pragma unroll
-            for (int h = 0; h < 2; ++h) x[j][h] = 16 * (b0 + j) + 8 * h < a.V8 ? *(const uint4 *)(rv + 16 * (b0 + j) + 8 * h) : make_uint4(0, 0, 0, 0);
-        u16 *t = s_v[wave];
+        for (int i = 0; i < 8; ++i) {
+            u32 *d = (u32 *)(t + (8 * i + (lane >> 3)) * LV + 8 * (lane & 7));
+            d[0] = x[i].x, d[1] = x[i].y, d[2] = x[i].z, d[3] = x[i].w;
+        }
+        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // (a wave reads what it wrote)
 #pragma unroll
         for (int j = 0; j < ML_VB; ++j) {
-            if (b0 + j >= ml_blocks(a.V)) break;
-#pragma unroll
-            for (int h = 0; h < 2; ++h) {
-                u32 *d = (u32 *)(t + lane * LV + 8 * h);
-                d[0] = x[j][h].x, d[1] = x[j][h].y, d[2] = x[j][h].z, d[3] = x[j][h].w;
-            }
-            asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // (a wave reads what it wrote)
+            if (b0 + j >= ml_blocks(a.V)) continue;
 #pragma unroll
             for (int s = 0; s < 2; ++s) {
                 u32 w[4];
 #pragma unroll
-                for (int i = 0; i < 4; ++i) w[i] = t[(32 * s + 8 * q4 + 2 * i) * LV + n16] | (u32)t[(32 * s + 8 * q4 + 2 * i + 1) * LV + n16] << 16;
+                for (int i = 0; i < 4; ++i) w[i] = t[(32 * s + 8 * q4 + 2 * i) * LV + 16 * j + n16] | (u32)t[(32 * s + 8 * q4 + 2 * i + 1) * LV + 16 * j + n16] << 16;
                 *(uint4 *)(ws + at.v + (size_t)(2 * (b0 + j) + s) * 1024 + lane * 16) = make_uint4(w[0], w[1], w[2], w[3]);
             }
-            asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
         }
         return;
     }
@@ -216,7 +216,8 @@ __global__ void __launch_bounds__(256) k_mlstm_prep(const MlstmArgs a) {
         }
         s_b[lane] = b, s_c[lane] = m, s_g[lane] = g.i;
         const float bl = __shfl(b, 63, 64), cl = __shfl(m, 63, 64);
-        o_s[lane] = b, o_s[ML + lane] = m, o_s[2 * ML + lane] = lane < c.n ? stack_exp<false>(bl - b + g.i - cl) : 0.0f;
+        const float w = lane < c.n ? stack_exp<false>(bl - b + g.i - cl) : 0.0f;
+        s_w[lane] = w, o_s[lane] = b, o_s[ML + lane] = m, o_s[2 * ML + lane] = w;
     }
     ml_f32x4 acc[4];
 #pragma unroll
@@ -228,46 +229,134 @@ __global__ void __launch_bounds__(256) k_mlstm_prep(const MlstmArgs a) {
         for (int t = 0; t < 4; ++t)
             if (t <= wave) acc[t] = ml_mfma(qv, piece(rk, 16 * t + n16, 32 * p + 8 * q4), acc[t]);
     }
-    // k^T: operand (pair p, half e, token step s) has channel 32 p + 8 (n16 / 4) + 4 e + n16 % 4 in lane n16, tokens 32 s + 8 q4 ..
-    for (int i = wave; i < 4 * np; i += 4) {
-        const int p = i >> 2, e = (i >> 1) & 1, s = i & 1, d = 32 * p + 8 * (n16 >> 2) + 4 * e + (n16 & 3);
-        u16 v[8];
-#pragma unroll
-        for (int k = 0; k < 8; ++k) v[k] = rk[(size_t)min(32 * s + 8 * q4 + k, c.n - 1) * ld + min(d, a.D8 - 1)];
-        uint4 w = make_uint4(v[0] | (u32)v[1] << 16, v[2] | (u32)v[3] << 16, v[4] | (u32)v[5] << 16, v[6] | (u32)v[7] << 16);
-        if (d >= a.D) w = make_uint4(0, 0, 0, 0);
-        *(uint4 *)(ws + at.k + (size_t)i * 1024 + lane * 16) = w;
-    }
     __syncthreads();
+    // k^T: operand (pair p, half e, token step s) has channel 32 p + 8 (n16 / 4) + 4 e + n16 % 4 in lane n16, tokens 32 s + 8 q4 ..
+    for (int i = wave; i < 2 * np; i += 4) {
+        const int d = 32 * (i >> 1) + 8 * (n16 >> 2) + 4 * (i & 1) + (n16 & 3);
+        u16 v[2][8];
+#pragma unroll
+        for (int s = 0; s < 2; ++s)
+#pragma unroll
+            for (int k = 0; k < 8; ++k) v[s][k] = rk[(size_t)min(32 * s + 8 * q4 + k, c.n - 1) * ld + min(d, a.D8 - 1)];
+        float sum = 0.0f;
+#pragma unroll
+        for (int s = 0; s < 2; ++s) {
+#pragma unroll
+            for (int k = 0; k < 8; ++k) sum = fmaf(BF16::to_f32(v[s][k]), s_w[32 * s + 8 * q4 + k], sum);
+            uint4 w = make_uint4(v[s][0] | (u32)v[s][1] << 16, v[s][2] | (u32)v[s][3] << 16, v[s][4] | (u32)v[s][5] << 16, v[s][6] | (u32)v[s][7] << 16);
+            if (d >= a.D) w = make_uint4(0, 0, 0, 0);
+            *(uint4 *)(ws + at.k + (size_t)(2 * i + s) * 1024 + lane * 16) = w;
+        }
+        sum = xor32_sum(xor16_sum(sum));
+        if (q4 == 0) ((float *)(ws + at.n))[d] = d < a.D ? sum : 0.0f;
+    }
     // rows 16 wave + 4 q4 + i, columns 16 t + n16
+    float rows[4] = {0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll
     for (int t = 0; t < 4; ++t)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
             const int row = 16 * wave + 4 * q4 + i, s = 16 * t + n16;
             float x = s <= row && row < c.n ? a.scale * acc[t][i] * stack_exp<false>(s_b[row] - s_b[s] + s_g[s] - s_c[row]) : 0.0f, y = 0.0f;
+            rows[i] += x;
             const u16 hi = BF16::from_f32(x);
             y = x - BF16::to_f32(hi);
-            s_p[0][row][s] = hi, s_p[1][row][s] = BF16::from_f32(y);
+            s_t[row * LP + s] = hi, s_t[(ML + row) * LP + s] = BF16::from_f32(y);
         }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) rows[i] = lanes16_sum(rows[i]);
+    if (n16 == 0) *(ml_f32x4 *)(o_s + 3 * ML + 16 * wave + 4 * q4) = (ml_f32x4){rows[0], rows[1], rows[2], rows[3]};
     // (a wave reads the rows it wrote)
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     char *o_p = ws + at.p + (size_t)wave * 4096;
 #pragma unroll
     for (int s = 0; s < 2; ++s)
 #pragma unroll
-        for (int k = 0; k < 2; ++k) *(uint4 *)(o_p + (s * 2 + k) * 1024 + lane * 16) = *(const uint4 *)&s_p[k][16 * wave + n16][32 * s + 8 * q4];
+        for (int k = 0; k < 2; ++k) *(uint4 *)(o_p + (s * 2 + k) * 1024 + lane * 16) = *(const uint4 *)&s_t[(ML * k + 16 * wave + n16) * LP + 32 * s + 8 * q4];
+}
+
+// n and the maximum in front of every chunk (a thread per channel), then the denominators of a chunk's rows
+__global__ void __launch_bounds__(MLSTM_CHUNK_MAX_DIM) k_mlstm_chain(const MlstmArgs a) {
+    const int head = blockIdx.x, d = threadIdx.x, np32 = 32 * ml_pairs(a.D);
+    const RowRun run = a.r.runs[blockIdx.y];
+    int chunk0 = 0;
+    for (int r = 0; r < (int)blockIdx.y; ++r) chunk0 += (a.r.runs[r].n_rows + ML - 1) / ML;
+    const int chunks = (run.n_rows + ML - 1) / ML;
+    const MlState st = ml_state(a, run, head);
+    const bool fresh = a.r.pos[run.row0] == 0;
+    const MlChunk at = ml_chunk(a.D, a.V);
+    const size_t step = at.bytes * a.H;
+    char *ws = (char *)a.r.ws + ((size_t)chunk0 * a.H + head) * at.bytes;
+    float n = !fresh && d < a.D ? st.n[d] : 0.0f, m = fresh ? 0.0f : st.m[ml_blocks(a.V)];
+    const int dd = min(d, np32 - 1);
+    constexpr int U = 16;  // chunks in flight
+    for (int c0 = 0; c0 < chunks; c0 += U) {
+        float k[U], b[U], c[U];
+#pragma unroll
+        for (int i = 0; i < U; ++i) {
+            const char *p = ws + (size_t)min(c0 + i, chunks - 1) * step;
+            k[i] = ((const float *)(p + at.n))[dd], b[i] = ((const float *)(p + at.s))[ML - 1], c[i] = ((const float *)(p + at.s))[2 * ML - 1];
+        }
+#pragma unroll
+        for (int i = 0; i < U; ++i) {
+            if (c0 + i >= chunks) continue;
+            float *p = (float *)(ws + (size_t)(c0 + i) * step + at.n);
+            if (d < np32) p[d] = n;
+            if (d == 0) p[np32] = m;
+            const float next = fmaxf(m + b[i], c[i]);
+            n = fmaf(stack_exp<false>(m + b[i] - next), n, stack_exp<false>(c[i] - next) * k[i]), m = next;
+        }
+    }
+    __syncthreads();  // (everyone has read the old maximum)
+    if (d < a.D) st.n[d] = n;
+    if (d == 0) st.m[ml_blocks(a.V)] = m;
+}
+// one workgroup per (chunk, head), a wave per row; NP: channel pairs per lane
+template <int NP>
+__global__ void __launch_bounds__(256) k_mlstm_den(const MlstmArgs a) {
+    const int head = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const RowChunk c = row_chunk(a.r.runs, a.r.n_runs, blockIdx.y, ML);
+    const MlChunk at = ml_chunk(a.D, a.V);
+    const char *ws = (const char *)a.r.ws + ((size_t)blockIdx.y * a.H + head) * at.bytes;
+    const float *n = (const float *)(ws + at.n), *s = (const float *)(ws + at.s);
+    const int last = 32 * ml_pairs(a.D);
+    const float m = n[last];
+    float2 nv[NP];
+#pragma unroll
+    for (int p = 0; p < NP; ++p) {
+        const int d = 2 * (lane + 64 * p);
+        nv[p] = d < last ? *(const float2 *)(n + d) : make_float2(0, 0);  // (zeros past the channels)
+    }
+    constexpr int U = 8;  // rows of a wave in flight
+    for (int t0 = wave * 16; t0 < wave * 16 + 16; t0 += U) {
+        u32 q[U][NP];
+#pragma unroll
+        for (int i = 0; i < U; ++i)
+#pragma unroll
+            for (int p = 0; p < NP; ++p)
+                q[i][p] = *(const u32 *)((const u16 *)a.r.raw + (size_t)(c.row0 + min(t0 + i, c.n - 1)) * a.r.ld + head * a.D8 + min(2 * (lane + 64 * p), a.D8 - 2));
+#pragma unroll
+        for (int i = 0; i < U; ++i) {
+            if (t0 + i >= c.n) continue;
+            float dot = 0.0f;
+#pragma unroll
+            for (int p = 0; p < NP; ++p) dot = fmaf(lo_f32<BF16>(q[i][p]), nv[p].x, fmaf(hi_f32<BF16>(q[i][p]), nv[p].y, dot));
+            dot = lanes_sum(dot);
+            const float b = s[t0 + i], cc = s[ML + t0 + i], mt = fmaxf(m + b, cc);
+            const float nq = fmaf(a.scale * stack_exp<false>(m + b - mt), dot, stack_exp<false>(cc - mt) * s[3 * ML + t0 + i]);
+            if (lane == 0) a.den[(size_t)(c.row0 + t0 + i) * a.H + head] = fmaxf(fabsf(nq), stack_exp<false>(-mt)) + a.den_eps;
+        }
+    }
 }
 
 // NPW: 32-channel pairs per wave (D <= 128 NPW).  A chunk's operands are loaded where the previous chunk's have just been used, out of the L2: a head's workgroups share
 // the reading of the chunk behind that from further away, a line per thread (into LDS that nobody reads).
 template <int NPW>
-__global__ void __launch_bounds__(256, NPW <= 2 ? 2 : 1) k_mlstm_scan(const MlstmArgs a) {
+__global__ void __launch_bounds__(256, 1) k_mlstm_scan(const MlstmArgs a) {
     __shared__ __attribute__((aligned(16))) ml_f32x4 s_o[2][4][4][64];
     __shared__ __attribute__((aligned(1024))) char s_warm[1024];
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), n16 = lane & 15, q4 = lane >> 4;
-    const int head = (int)blockIdx.x % a.H, cb = (int)blockIdx.x / a.H, blocks = ml_blocks(a.V), V4 = ml_up4(a.V), D = a.D, np = ml_pairs(D);  // (head fastest: a head's columns share an L2 where H is a multiple of 8)
-    const bool has_n = cb == blocks;  // this workgroup carries n
+    const int head = (int)blockIdx.x % a.H, cb = (int)blockIdx.x / a.H, V4 = ml_up4(a.V), D = a.D, np = ml_pairs(D);  // (head fastest: a head's columns share an L2 where H is a multiple of 8)
     const RowRun run = a.r.runs[blockIdx.y];
     int chunk0 = 0;
     for (int r = 0; r < (int)blockIdx.y; ++r) chunk0 += (a.r.runs[r].n_rows + ML - 1) / ML;
@@ -279,7 +368,6 @@ __global__ void __launch_bounds__(256, NPW <= 2 ? 2 : 1) k_mlstm_scan(const Mlst
     auto place = [&](int j, int e, int i) -> float * {
         const int d = 32 * (wave * NPW + j) + 8 * q4 + 4 * e + i;
         if (d >= D) return nullptr;
-        if (has_n) return n16 == 0 ? st.n + d : nullptr;
         return col < a.V ? st.S + (size_t)d * V4 + col : nullptr;
     };
 #pragma unroll
@@ -321,7 +409,7 @@ __global__ void __launch_bounds__(256, NPW <= 2 ? 2 : 1) k_mlstm_scan(const Mlst
         for (int s = 0; s < 2; ++s) {
 #pragma unroll
             for (int h = 0; h < 2; ++h) p[s][h] = *(const uint4 *)(ws + place_of.p + wave * 4096 + (s * 2 + h) * 1024);
-            v[s] = *(const uint4 *)(ws + place_of.v + (size_t)(2 * min(cb, blocks - 1) + s) * 1024);
+            v[s] = *(const uint4 *)(ws + place_of.v + (size_t)(2 * cb + s) * 1024);
 #pragma unroll
             for (int h = 0; h < 2; ++h) w[s][h] = *(const ml_f32x4 *)((const float *)(ws - lane * 16 + place_of.s) + 2 * ML + 32 * s + 8 * q4 + 4 * h);
         }
@@ -354,7 +442,7 @@ __global__ void __launch_bounds__(256, NPW <= 2 ? 2 : 1) k_mlstm_scan(const Mlst
 #pragma unroll
             for (int i = 0; i < 8; ++i) f[i] = S[j][i >> 2][i & 3];
 #pragma unroll
-            for (int i = 0; i < 4; ++i) hi[i] = ml_part(f[2 * i], f[2 * i + 1]), lo[i] = pack2<BF16>(f[2 * i], f[2 * i + 1]);
+            for (int i = 0; i < 4; ++i) hi[i] = ml_part(f[2 * i], f[2 * i + 1]), lo[i] = w4m_pack<BF16>(f[2 * i], f[2 * i + 1]);
             const uint4 h = make_uint4(hi[0], hi[1], hi[2], hi[3]), l = make_uint4(lo[0], lo[1], lo[2], lo[3]);
 #pragma unroll
             for (int t = 0; t < 4; ++t) acc[t] = ml_mfma(q[t][j], h, acc[t]);
@@ -369,16 +457,13 @@ __global__ void __launch_bounds__(256, NPW <= 2 ? 2 : 1) k_mlstm_scan(const Mlst
         float f[2][8];
 #pragma unroll
         for (int s = 0; s < 2; ++s) {
-            u32 x[4] = {v[s].x, v[s].y, v[s].z, v[s].w};
-#pragma unroll
-            for (int i = 0; i < 4; ++i) x[i] = has_n ? 0x3F803F80u : x[i];  // (n: v = 1)
+            const u32 x[4] = {v[s].x, v[s].y, v[s].z, v[s].w};
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 f[s][2 * i] = lo_f32<BF16>(x[i]) * (add * w[s][i >> 1][2 * (i & 1)]);
                 f[s][2 * i + 1] = hi_f32<BF16>(x[i]) * (add * w[s][i >> 1][2 * (i & 1) + 1]);
             }
-            const uint4 vv = make_uint4(x[0], x[1], x[2], x[3]);
-            own = ml_mfma(p[s][0], vv, own), own = ml_mfma(p[s][1], vv, own);
+            own = ml_mfma(p[s][0], v[s], own), own = ml_mfma(p[s][1], v[s], own);
         }
         load_pv(ch + 1);
         // the state behind the chunk: values times their key weights, in three parts
@@ -392,7 +477,7 @@ __global__ void __launch_bounds__(256, NPW <= 2 ? 2 : 1) k_mlstm_scan(const Mlst
             for (int h = 0; h < 3; ++h) {
                 u32 x[4];
 #pragma unroll
-                for (int i = 0; i < 4; ++i) x[i] = ml_part(f[s][2 * i], f[s][2 * i + 1]);
+                for (int i = 0; i < 4; ++i) x[i] = h < 2 ? ml_part(f[s][2 * i], f[s][2 * i + 1]) : w4m_pack<BF16>(f[s][2 * i], f[s][2 * i + 1]);
                 const uint4 part = make_uint4(x[0], x[1], x[2], x[3]);
 #pragma unroll
                 for (int j = 0; j < NPW; ++j)
@@ -406,20 +491,15 @@ __global__ void __launch_bounds__(256, NPW <= 2 ? 2 : 1) k_mlstm_scan(const Mlst
             if (wave * NPW + j >= np) S[j][0] = S[j][1] = zero;  // (channels that do not exist saw another pair's keys)
         asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");  // (LDS only: the next chunk's loads stay in flight)
         const ml_f32x4 all = (s_o[ch & 1][0][wave][lane] + s_o[ch & 1][1][wave][lane]) + (s_o[ch & 1][2][wave][lane] + s_o[ch & 1][3][wave][lane]);
-        float o[4], mt[4];
+        float o[4];
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-            mt[i] = fmaxf(m + cbv[i], ccv[i]);
-            o[i] = fmaf(a.scale * stack_exp<false>(m + cbv[i] - mt[i]), all[i], stack_exp<false>(ccv[i] - mt[i]) * own[i]);
+            const float mt = fmaxf(m + cbv[i], ccv[i]);
+            o[i] = fmaf(a.scale * stack_exp<false>(m + cbv[i] - mt), all[i], stack_exp<false>(ccv[i] - mt) * own[i]);
         }
         const int t0 = ML * ch + 16 * wave + 4 * q4;
         const size_t at = ((size_t)run.row0 + t0) * a.H + head;
-        if (has_n) {
-            if (n16 == 0)
-#pragma unroll
-                for (int i = 0; i < 4; ++i)
-                    if (t0 + i < run.n_rows) a.den[at + (size_t)i * a.H] = fmaxf(fabsf(o[i]), stack_exp<false>(-mt[i])) + a.den_eps;
-        } else if (col < a.V) {
+        if (col < a.V) {
             float *dst = a.o + at * a.V8 + col;
             const int row = a.H * a.V8;
             if (ML * (ch + 1) <= run.n_rows)
@@ -483,7 +563,14 @@ int mlstm_chunks_launch(const MlstmArgs &a, int chunks, hipStream_t st) {
     PIE_REQUIRE(a.r.ws && chunks > 0 && chunks <= 65535 && a.D <= MLSTM_CHUNK_MAX_DIM, PIE_E_ARG, "mLSTM: the chunk form needs its workspace, and keys of at most 512 channels");
     hipLaunchKernelGGL(k_mlstm_prep, dim3((unsigned)a.H, (unsigned)chunks, (unsigned)(1 + (ml_blocks(a.V) + 4 * ML_VB - 1) / (4 * ML_VB))), dim3(256), 0, st, a);
     PIE_LAUNCH_CHECK();
-    const dim3 grid((unsigned)(a.H * (ml_blocks(a.V) + 1)), (unsigned)a.r.n_runs);
+    hipLaunchKernelGGL(k_mlstm_chain, dim3((unsigned)a.H, (unsigned)a.r.n_runs), dim3((unsigned)((32 * ml_pairs(a.D) + 63) / 64 * 64)), 0, st, a);
+    PIE_LAUNCH_CHECK();
+    const dim3 dg((unsigned)a.H, (unsigned)chunks);
+    if (a.D <= 128) hipLaunchKernelGGL(k_mlstm_den<1>, dg, dim3(256), 0, st, a);
+    else if (a.D <= 256) hipLaunchKernelGGL(k_mlstm_den<2>, dg, dim3(256), 0, st, a);
+    else hipLaunchKernelGGL(k_mlstm_den<4>, dg, dim3(256), 0, st, a);
+    PIE_LAUNCH_CHECK();
+    const dim3 grid((unsigned)(a.H * ml_blocks(a.V)), (unsigned)a.r.n_runs);
     if (a.D <= 128) hipLaunchKernelGGL(k_mlstm_scan<1>, grid, dim3(256), 0, st, a);
     else if (a.D <= 256) hipLaunchKernelGGL(k_mlstm_scan<2>, grid, dim3(256), 0, st, a);
     else hipLaunchKernelGGL(k_mlstm_scan<4>, grid, dim3(256), 0, st, a);
