@@ -52,7 +52,7 @@ def causal_conv(h, w):
     taps, out = w.shape[1], h.copy()
     for back in range(taps):
         shifted = np.zeros_like(h)
-        shifted[back:] = h[:len(h) - back] if back else h
+        shifted[back:] = h[:max(len(h) - back, 0)]
         out = out + shifted * w[:, taps - 1 - back]
     return out
 
