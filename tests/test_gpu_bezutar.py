@@ -231,9 +231,8 @@ def test_bigrams_cross_every_cut(bigram):
     ca, cb, got = m.make_cache(), m.make_cache(), []
     for lo, hi in ((0, 1), (1, 2), (2, 4), (4, 30), (30, 31), (31, 60)):
         got.append(m.step_portions([(a[lo:hi], ca), (b[lo:hi], cb)], [list(range(hi - lo))] * 2).cpu().numpy())
-    at = [0]
     for part, (lo, hi) in zip(got, ((0, 1), (1, 2), (2, 4), (4, 30), (30, 31), (31, 60))):
-        assert bu.err(part[:hi - lo], wa[lo:hi]) < 5e-5 and bu.err(part[hi - lo:], wb[lo:hi]) < 5e-5, at
+        assert bu.err(part[:hi - lo], wa[lo:hi]) < 5e-5 and bu.err(part[hi - lo:], wb[lo:hi]) < 5e-5, lo
 
 
 @BOTH
