@@ -581,14 +581,30 @@ typedef struct {
     const void *bigram;        /* bf16 [buckets + 1][width], or NULL: row (previous token * mul_prev + token * mul_cur) mod buckets is added to the embedding,
                                 * at a sequence's first token row `buckets`; the previous token stands at the end of layer 0's state */
     long long mul_prev, mul_cur;
-    int buckets, reserved;
+    int buckets;
+    float logit_cap;           /* > 0: logits = logit_cap * tanh(logits / logit_cap) */
+    const void *side_embed;    /* bf16 [vocab][n_layers * side_dim], or NULL: every layer's part of a token's side vector (pie_stack_layer: w_side_gate) */
+    int side_dim, reserved;
 } pie_stack_config;
 
-enum { PIE_MIXER_LATENT = 1, PIE_MIXER_ATTENTION = 2, PIE_MIXER_DELTA = 3, PIE_MIXER_MLSTM = 4, PIE_MIXER_MINGRU = 5 };
-enum { PIE_FF_NONE = 0, PIE_FF_RELU2 = 1, PIE_FF_TABLE_MOE = 2, PIE_FF_ROUTED_MOE = 3, PIE_FF_XIELU = 4 };
+enum { PIE_MIXER_LATENT = 1, PIE_MIXER_ATTENTION = 2, PIE_MIXER_DELTA = 3, PIE_MIXER_MLSTM = 4, PIE_MIXER_MINGRU = 5, PIE_MIXER_GATED_DELTA = 6, PIE_MIXER_TIME_MIX = 7 };
+enum { PIE_FF_NONE = 0, PIE_FF_RELU2 = 1, PIE_FF_TABLE_MOE = 2, PIE_FF_ROUTED_MOE = 3, PIE_FF_XIELU = 4, PIE_FF_GEGLU = 5 };
 enum { PIE_ACT_SILU = 0, PIE_ACT_CLIPPED = 1 };
 
-/* One layer: x += post1(mixer(pre1(x))); x += post2(ff(pre2(x))).  With hyper-connections (hyper1, hyper2: fp32 [streams (in) + streams (out) + streams *
+/* Time mixing with a decaying matrix state per head (RWKV-6).  Every projection reads its own mix h + (h' - h) mu of the row h and its predecessor h' in the sequence (zeros in
+ * front of the first; the predecessor is part of the state): mu fp32 [5 (r, k, v, gate, decay)][width rounded up to 64].  w_r, w_k, w_v, w_gate packed [heads * dim8, width], w_low packed
+ * [rank8, width]; decay = exp(-exp(w_decay tanh(w_low .) + decay_bias)), w_decay bf16 [heads * dim][rank8] row-major, decay_bias fp32 [heads * dim]; o = (S + diag(bonus) k v^T)^T r, then
+ * S = diag(decay) S + k v^T; bonus fp32 [heads * dim]; every head over its root mean square (eps of the layer), times o_norm (fp32 [heads * dim]) and silu(gate), times out_scale. */
+typedef struct {
+    int heads, dim, rank;
+    float out_scale;
+    const void *w_r, *w_k, *w_v, *w_gate, *w_low, *w_decay;
+    const float *mu, *decay_bias, *bonus, *o_norm;
+} pie_stack_time_mix;
+
+/* One layer: x += post1(mixer(pre1(x))); x += post2(ff(pre2(x))).  norm_after: x = post1(residual_scale x + mixer(x)); x = post2(residual_scale x + ff(x)) instead (no pre norms).
+ * w_side_gate packed [side_dim, width] (NULL: none), w_side_proj packed [width, side_dim], side_norm: behind both sublayers, x += side_norm(w_side_proj (gelu(w_side_gate x) * e)), e the part
+ * of side_embed that belongs to the row's token and this layer.  gelu: z / 2 (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))).  With hyper-connections (hyper1, hyper2: fp32 [streams (in) + streams (out) + streams *
  * streams (mix, [from][to])]; RMS norms in front, none behind) instead: u = sum in[s] x_s, y = sublayer(pre(u)), x_t <- sum mix[s][t] x_s + out[t] y.
  * conv_taps > 0: the mixer reads h + conv(h), h = pre1(.), conv(h)_t = sum_j conv[j] h_(t - taps + 1 + j) per channel with zeros in front of the sequence; conv
  * fp32 [conv_taps][width rounded up to 64]; the last conv_taps - 1 inputs are part of the layer's state.  Below, dim8 / vdim8 / rank8 = dim / vdim / rank rounded up to 8; rows and columns past a
@@ -606,10 +622,18 @@ enum { PIE_ACT_SILU = 0, PIE_ACT_CLIPPED = 1 };
  * none), then the first rot_dims dimensions rotated in neighbouring pairs by position * rot_freq[i] (fp32 [rot_dims / 2]), cos and sin times rot_gain;
  * value_norm: every head's value over its root mean square; score = scale * q . k; sink: added to the softmax's denominator as sink * exp(0); out_gate:
  * every head's output times the sigmoid of its gate.  kv_from = j >= 0: no keys and values of its own (no k, v rows in w_in), layer j's cached ones are
- * read; else -1.  w_o packed [width, heads * vdim8], o_bias bf16 [width] (NULL: none).
+ * read; else -1.  w_o packed [width, heads * vdim8], o_bias bf16 [width] (NULL: none).  chunk > 0: position i sees the positions of its own chunk, i / chunk = j / chunk, instead of a
+ * window.  row_norm: the query and key norms run over all heads of a row at once (weights fp32 [heads * dim8], [kv_heads * dim8]), and the values are the keys in front of their norm (no v in
+ * w_in; vdim = dim; no rotation).  distance fp32 [heads][far + 1] (NULL: none): distance[h][min(i - j, far)] is added to the scaled score.  head_sink as above (then sink is 0).  out_scale:
+ * factor on the heads' outputs.  time_mix.heads > 0: time mixing beside the attention, on the same input; then w_o is packed [width, heads * vdim8 + time_mix.heads * time_mix.dim8].
+ * Time mix mixer: time_mix alone (heads, dim, w_in are not used).
  * Delta mixer (generalised delta rule on a dim x dim state per head):  w_in packed [5 heads * dim8 (r, k, v, gate, removal rate) + rank8 (decay, low rank),
  * width], in_bias as above; w_decay bf16 [heads * dim][rank8] row-major; decay_bias fp32 [heads * dim]; decay = exp(-decay_scale * sigmoid(w_decay tanh(.) +
  * decay_bias)); unit key k / sqrt(sum k^2 + unit_eps); o_norm fp32 [heads * dim]; w_o packed [width, heads * dim8].
+ * Gated delta mixer (one decay per head, a dim x vdim state):  w_in packed [kv_heads * dim8 (q) + kv_heads * dim8 (k) + heads * vdim8 (v) + heads * vdim8 (gate) + heads rounded up to 8 (step size) +
+ * the same (decay), width]; q, k, v each through a causal convolution over time per channel (mix_conv fp32 [mix_taps][channels of q, k, v], the last tap the current token's, zeros in front of the
+ * sequence) and silu; unit queries and keys x / sqrt(sum x^2 + unit_eps), queries times scale; b = sigmoid(.), g = exp(-decay_rate softplus(. + decay_bias)) (both fp32 [heads]); S <- g S; u = b (v - S^T k);
+ * S <- S + k u^T; o = S^T q; every head over its root mean square, times o_norm (fp32 [vdim], shared by the heads) and silu(gate); w_o packed [width, heads * vdim8].
  * mLSTM mixer (matrix memory with exponential gates):  w_in packed [heads * dim8 (q) + heads * dim8 (k) + heads * vdim8 (v) + heads * vdim8 (output gate) + heads
  * rounded up to 8 (input gate) + the same (forget gate), width]; the two gates plus gate_bias; q times scale; log gates i = c(.), f = log sigmoid(c(.)), c(z) = gate_cap
  * tanh(z / gate_cap); m_t = max(f + m_(t-1), i) from m = 0; S_t = exp(f + m_(t-1) - m_t) S_(t-1) + exp(i - m_t) k v^T, n_t likewise with k alone; o = S_t^T q /
@@ -618,6 +642,7 @@ enum { PIE_ACT_SILU = 0, PIE_ACT_CLIPPED = 1 };
  * minGRU mixer:  heads = 1, dim = its size; w_in packed [dim8 (update gate) + dim8 (candidate) + dim8 (output gate), width], in_bias as above; z = sigmoid(.), candidate
  * u + 1/2 where u >= 0, else sigmoid(u); S_t = (1 - z) S_(t-1) + z candidate; output S_t silu(output gate); w_o packed [width, dim8].
  * Dense feed-forwards: w_down act(w_up h), act RELU2: max(z, 0)^2; XIELU: act_alpha z^2 + z / 2 for z > 0, act_beta (exp(z) - 1 - z) + z / 2 else.
+ * GEGLU: w_up packed [2 * size, width] with rows (2 i, 2 i + 1) = (gate_i, up_i), up_bias bf16 [2 * size] in that order (NULL: none): w_down (gelu(gate) * up) + down_bias (bf16 [width], NULL: none).
  * Experts: w_gate_up experts x packed [2 * size, width] with rows (2 i, 2 i + 1) = (gate_i, up_i); w_down experts x packed [width, size].  act SILU:
  * silu(g) u; CLIPPED: g = min(gate, act_limit), u = clamp(up, +-act_limit), g sigmoid(act_alpha g) (u + 1).
  * TABLE_MOE: table int32 [vocab][top], every chosen expert weighs 1 / top.  ROUTED_MOE: w_router packed [experts, width], the `top` experts with the largest
@@ -650,13 +675,19 @@ typedef struct {
     const float *gate_bias;    /* mLSTM: fp32 [2][heads], input then forget gate */
     const void *w_uq;
     const float *head_sink;
+    const float *distance, *decay_rate, *mix_conv;
+    int chunk, far, row_norm, mix_taps, norm_after;
+    float out_scale, residual_scale;
+    const void *up_bias, *down_bias, *w_side_gate, *w_side_proj;
+    pie_stack_norm side_norm;
+    pie_stack_time_mix time_mix;
 } pie_stack_layer;
 
 int pie_stack_create(const pie_stack_config *cfg, pie_stack **out);
 int pie_stack_destroy(pie_stack *s);
 int pie_stack_set_layer(pie_stack *s, int i, const pie_stack_layer *layer);
 /* elements per cached token of layer i (its page is [64][that many] in the stack's dtype; 0: the layer caches no tokens), bytes of one page, and
- * fp32 numbers of recurrent state per sequence (0: none; the mixer's, then the convolution's last inputs, then -- layer 0 -- the embedding's previous token).  A latent page holds token after token; a page of keys and values is laid out in matrix-core
+ * fp32 numbers of recurrent state per sequence (0: none; the mixer's, then the convolution's last inputs, then -- layer 0 -- the embedding's previous token, then the time mixing's previous row).  A latent page holds token after token; a page of keys and values is laid out in matrix-core
  * operand order (csrc/page_attn.hip) and means something as a whole only. */
 int pie_stack_page_row(const pie_stack *s, int i);
 size_t pie_stack_state_floats(const pie_stack *s, int i);

@@ -84,19 +84,24 @@ def _fields(spec: str, types: dict) -> list:
     return out
 
 
-_CT = {"i": C.c_int, "f": C.c_float, "p": C.c_void_p, "z": C.c_size_t, "l": C.c_longlong, "n": pie_stack_norm}
+class pie_stack_time_mix(C.Structure):
+    _fields_ = _fields("i:heads dim rank f:out_scale p:w_r w_k w_v w_gate w_low w_decay mu decay_bias bonus o_norm", {"i": C.c_int, "f": C.c_float, "p": C.c_void_p})
+
+
+_CT = {"i": C.c_int, "f": C.c_float, "p": C.c_void_p, "z": C.c_size_t, "l": C.c_longlong, "n": pie_stack_norm, "t": pie_stack_time_mix}
 
 
 class pie_stack_config(C.Structure):
     _fields_ = _fields("i:dtype width vocab n_layers f:logit_scale embed_scale p:embed head n:final_norm i:streams max_positions p:positions bigram "
-                       "l:mul_prev mul_cur i:buckets reserved", _CT)
+                       "l:mul_prev mul_cur i:buckets f:logit_cap p:side_embed i:side_dim reserved", _CT)
 
 
 class pie_stack_layer(C.Structure):
     _fields_ = _fields("n:pre1 post1 pre2 post2 i:mixer heads dim vdim rank window f:scale eps p:w_in w_uk w_uv w_o w_kv c_norm "
                        "i:kv_heads kv_from rot_dims value_norm out_gate f:rot_gain sink decay_scale unit_eps p:rot_freq q_norm k_norm decay_bias o_norm "
                        "in_bias o_bias w_decay i:ff ff_size p:w_up w_down i:experts top shared_size act f:act_alpha act_limit p:table w_router w_router_rows correction "
-                       "w_gate_up w_expert_down s_gate_up s_down shared_gate hyper1 hyper2 conv i:conv_taps q_rank rot_dim f:gate_cap act_beta p:gate_bias w_uq head_sink", _CT)
+                       "w_gate_up w_expert_down s_gate_up s_down shared_gate hyper1 hyper2 conv i:conv_taps q_rank rot_dim f:gate_cap act_beta p:gate_bias w_uq head_sink "
+                       "distance decay_rate mix_conv i:chunk far row_norm mix_taps norm_after f:out_scale residual_scale p:up_bias down_bias w_side_gate w_side_proj n:side_norm t:time_mix", _CT)
 
 
 class pie_stack_batch(C.Structure):
@@ -105,8 +110,8 @@ class pie_stack_batch(C.Structure):
 
 
 PIE_NORM_NONE, PIE_NORM_DYN_TANH, PIE_NORM_RMS = 0, 1, 2
-PIE_MIXER_LATENT, PIE_MIXER_ATTENTION, PIE_MIXER_DELTA, PIE_MIXER_MLSTM, PIE_MIXER_MINGRU = 1, 2, 3, 4, 5
-PIE_FF_NONE, PIE_FF_RELU2, PIE_FF_TABLE_MOE, PIE_FF_ROUTED_MOE, PIE_FF_XIELU = 0, 1, 2, 3, 4
+PIE_MIXER_LATENT, PIE_MIXER_ATTENTION, PIE_MIXER_DELTA, PIE_MIXER_MLSTM, PIE_MIXER_MINGRU, PIE_MIXER_GATED_DELTA, PIE_MIXER_TIME_MIX = 1, 2, 3, 4, 5, 6, 7
+PIE_FF_NONE, PIE_FF_RELU2, PIE_FF_TABLE_MOE, PIE_FF_ROUTED_MOE, PIE_FF_XIELU, PIE_FF_GEGLU = 0, 1, 2, 3, 4, 5
 PIE_ACT_SILU, PIE_ACT_CLIPPED = 0, 1
 
 

@@ -20,7 +20,7 @@ CSRC = PKG / "csrc"
 LIB_DIR = PKG / "lib"
 LIB = LIB_DIR / "libpie_hip.so"
 BASE_LIB = LIB_DIR / "libpie_base.so"
-BASE_SOURCES = ["base.hip", "w16_gemm.hip", "w16_grouped.hip", "rows_gemm.hip", "latent_attn.hip", "window_attn.hip", "page_attn.hip", "delta_rule.hip", "mlstm.hip", "mingru.hip", "head_out.hip", "row_update.hip", "stream_update.hip", "layer_stack.hip", "page_pool.cpp"]
+BASE_SOURCES = ["base.hip", "w16_gemm.hip", "w16_grouped.hip", "rows_gemm.hip", "latent_attn.hip", "window_attn.hip", "page_attn.hip", "delta_rule.hip", "gated_delta.hip", "time_mix.hip", "mlstm.hip", "mingru.hip", "head_out.hip", "row_update.hip", "stream_update.hip", "layer_stack.hip", "page_pool.cpp"]
 SOURCES = ["w4_gemv.hip", "ops.hip", "decoder.hip", "prefill.hip", "vision.hip", "w4m_gemm.hip", "tp_comm.hip", "sampler.hip", "paged_i8.hip"]
 # packed-fp32-ops off: hipcc otherwise forms v_pk_{add,mul,fma}_f32 from ordinary float code, and some of their forms are not reliable here
 FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-ffp-contract=off", "-fno-fast-math",

@@ -12,22 +12,12 @@
 //   o_t = S^T (W_t r_t) + sum_{i<=t} A'_ti v_i - sum_{i<=t} B'_ti p_i,     A', B' likewise with r_t and W_t
 //   S  <- W_16 S + sum_i (W_16 / W_i) (k_i v_i^T - a_i u_i p_i^T)
 // Everything but S and p is known beforehand: one launch (all chunks of all heads in parallel) takes the channel vectors, A, B, A', B' and T = (I + B)^-1 and
-// leaves T U, R, K, -A and T A, A', -B' in matrix operand order; a second walks the chunks, one workgroup per head and 16 value columns, whose four waves
-// split the key channels of S (which stays in accumulators and is its own B operand); a third takes the heads' norm and gate.  W_16 is
+// leaves T U, R, K, -A and T A, A', -B' in matrix operand order; a second walks the chunks (chunk_scan.hpp, SCAN_DELTA); a third takes the heads' norm and gate.  W_16 is
 // above exp(-16 decay_scale): the quotients are formed as W_t times 1 / W_i, which fp32 holds up to DELTA_MAX_DECAY.
-#include <algorithm>
-
-#include "stack_types.hpp"
-
-typedef __attribute__((ext_vector_type(4))) float dr_f32x4;
-typedef __attribute__((ext_vector_type(8))) __bf16 dr_bf16x8;
+#include "chunk_scan.hpp"
+#include "low_rank.hpp"
 
 namespace {
-
-constexpr int DC = 16;  // tokens of a chunk
-constexpr size_t DELTA_SEGMENT_BYTES = 96u << 20;
-
-__device__ __forceinline__ void lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }  // (loads and stores stay in flight)
 
 // CP: power of two >= D; NT threads; AHEAD: few workgroups, where latency counts and registers do not
 template <class E, int CP, int NT, bool AHEAD>
@@ -150,25 +140,6 @@ __global__ void __launch_bounds__(NT, AHEAD ? 1 : 4) k_delta_step(const DeltaArg
 }
 
 // ---------------------------------------------------------------- chunk form
-__host__ __device__ __forceinline__ int dr_blocks(int D) { return (D + 15) / 16; }
-// per (chunk, head): T U, R, K, -A [blocks][64 lanes][4] each; T A, A', -B' [64][4]; W_16 [16 blocks]
-__host__ __device__ __forceinline__ size_t dr_chunk_floats(int D) { return (size_t)dr_blocks(D) * (4 * 256 + 16) + 3 * 256; }
-
-__device__ __forceinline__ dr_f32x4 dr_mfma(float a, float b, const dr_f32x4 &c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
-
-struct DeltaChunk {
-    int row0, n;  // rows [row0, row0 + n)
-};
-__device__ __forceinline__ DeltaChunk dr_chunk(const DeltaArgs &a, int i) {
-    int r = 0;
-    for (;;) {
-        const int n = (a.runs[r].n_rows + DC - 1) / DC;
-        if (i < n || r + 1 >= a.n_runs) break;
-        i -= n, ++r;
-    }
-    return {a.runs[r].row0 + DC * i, min(DC, a.runs[r].n_rows - DC * i)};
-}
-
 // One workgroup per (chunk, head).  A wave owns four tokens; its lanes own channel pairs.
 // NB: 16-channel blocks per wave in the products (D <= 64 NB).  Dynamic LDS: see delta_prep_lds().
 template <class E, int NB>
@@ -182,21 +153,9 @@ __global__ void __launch_bounds__(256) k_delta_prep(const DeltaArgs a) {
     // (the low-rank input of the decay lies where the channel vectors come later)
     const int D = a.D, nblk = dr_blocks(D), lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), n16 = lane & 15, q = lane >> 4;
     const int head = blockIdx.x, HD8 = a.H * a.D8;  // (head fastest: workgroups that run together read whole rows)
-    const DeltaChunk c = dr_chunk(a, a.chunk_lo + (int)blockIdx.y);
+    const ScanChunk c = scan_chunk(a.runs, a.n_runs, a.chunk_lo + (int)blockIdx.y);
     if (c.n <= 0) return;
-    const int R32 = (a.R8 + 31) & ~31, LR = R32 + 8;
-    u16 *s_hi = (u16 *)s_u, *s_lo = s_hi + DC * LR;
-    float *s_low = s_u;
-    struct Pair {
-        float x, y;
-    };
-    auto pair_at = [&](const T *p) -> Pair {
-        if constexpr (F32) return {((const float2 *)p)->x, ((const float2 *)p)->y};
-        else {
-            const u32 w = *(const u32 *)p;
-            return {lo_f32<BF16>(w), hi_f32<BF16>(w)};
-        }
-    };
+    typedef ElemPair Pair;
     auto bias_at = [&](int at) -> Pair {
         if (!a.bias) return {0.0f, 0.0f};
         const u32 w = *(const u32 *)(a.bias + at);
@@ -204,14 +163,9 @@ __global__ void __launch_bounds__(256) k_delta_prep(const DeltaArgs a) {
     };
     // All loads without branches around them: they leave together, and what lies outside is dropped afterwards.
     const T *raw = (const T *)a.raw + (size_t)c.row0 * a.ld;
-    constexpr int LN = 4;  // pairs of the low-rank input per thread that travel ahead (ranks up to 128): sixteen lanes per token
-    const int tr = threadIdx.x >> 4, lr = 2 * (threadIdx.x & 15);
-    Pair low[LN], lowb[LN];
-#pragma unroll
-    for (int j = 0; j < LN; ++j) {
-        const int at = 5 * HD8 + min(lr + 32 * j, a.R8 - 2);
-        low[j] = pair_at(raw + (size_t)min(tr, c.n - 1) * a.ld + at), lowb[j] = bias_at(at);
-    }
+    const LowRankArgs low = {raw + 5 * HD8, a.ld, c.n, a.rank, a.R8, a.bias ? a.bias + 5 * HD8 : nullptr, a.w_decay + (size_t)head * D * a.R8, a.decay_bias + head * D, D};
+    LowRank<E, NB> lr;
+    lr.load(low);
     Pair xr[NP][TP], xk[NP][TP], xa[NP][TP], bx[NP][3];
 #pragma unroll
     for (int p = 0; p < NP; ++p) {
@@ -219,71 +173,14 @@ __global__ void __launch_bounds__(256) k_delta_prep(const DeltaArgs a) {
 #pragma unroll
         for (int j = 0; j < TP; ++j) {
             const T *x = raw + (size_t)min(TP * wave + j, c.n - 1) * a.ld;
-            xr[p][j] = pair_at(x + d), xk[p][j] = pair_at(x + HD8 + d), xa[p][j] = pair_at(x + 4 * HD8 + d);
+            xr[p][j] = load_pair<E>(x + d), xk[p][j] = load_pair<E>(x + HD8 + d), xa[p][j] = load_pair<E>(x + 4 * HD8 + d);
         }
         bx[p][0] = bias_at(d), bx[p][1] = bias_at(HD8 + d), bx[p][2] = bias_at(4 * HD8 + d);
     }
-    // the decay's weights (the first WS steps)
-    constexpr int WS = 4;
-    uint4 wd[F32 ? 1 : NB][WS];
-    float db[NB];
-    auto decay_weights = [&](int j, int s) {
-        const int d = 16 * (wave * NB + j) + n16, at = 32 * s + 8 * q;
-        const uint4 w = *(const uint4 *)(a.w_decay + (size_t)(head * D + min(d, D - 1)) * a.R8 + min(at, a.R8 - 8));
-        return d < D && at < a.R8 ? w : make_uint4(0, 0, 0, 0);
-    };
-    if constexpr (!F32)
-#pragma unroll
-        for (int j = 0; j < NB; ++j) {
-#pragma unroll
-            for (int s = 0; s < WS; ++s) wd[j][s] = decay_weights(j, s);
-            db[j] = a.decay_bias[head * D + min(16 * (wave * NB + j) + n16, D - 1)];
-        }
-    auto put_low = [&](int j, const Pair &v, const Pair &b) {
-        auto f = [&](int i, float z) { return tr < c.n && i < a.rank ? F32 ? tanhf(z) : fast_tanh(z) : 0.0f; };
-        const float x = f(j, v.x + b.x), y = f(j + 1, v.y + b.y);
-        if constexpr (F32) s_low[tr * LR + j] = x, s_low[tr * LR + j + 1] = y;
-        else {
-            const u32 hi = pack2<BF16>(x, y);
-            *(u32 *)(s_hi + tr * LR + j) = hi, *(u32 *)(s_lo + tr * LR + j) = pack2<BF16>(x - lo_f32<BF16>(hi), y - hi_f32<BF16>(hi));
-        }
-    };
-#pragma unroll
-    for (int j = 0; j < LN; ++j)
-        if (32 * j < R32) put_low(lr + 32 * j, low[j], lowb[j]);
-    for (int j = lr + 32 * LN; j < R32; j += 32) {
-        const int at = 5 * HD8 + min(j, a.R8 - 2);
-        put_low(j, pair_at(raw + (size_t)min(tr, c.n - 1) * a.ld + at), bias_at(at));
-    }
+    lr.load_weights(low, wave, lane);
+    lr.put(low, s_u);
     lds_barrier();
-    auto log_decay = [&](int t, int d, float z) { s_l[t * LD + d] = t < c.n && d < D ? -a.decay_scale * stack_sigmoid<F32>(z) : 0.0f; };
-    if constexpr (F32) {
-        for (int i = threadIdx.x; i < DC * 16 * nblk; i += 256) {
-            const int t = i / (16 * nblk), d = i % (16 * nblk);
-            float z = 0.0f;
-            if (d < D)
-                for (int j = 0; j < a.rank; ++j) z = fmaf(s_low[t * LR + j], BF16::to_f32(a.w_decay[(size_t)(head * D + d) * a.R8 + j]), z);
-            log_decay(t, d, z + a.decay_bias[head * D + min(d, D - 1)]);
-        }
-    } else {
-#pragma unroll
-        for (int j = 0; j < NB; ++j) {
-            const int b = wave * NB + j, d = 16 * b + n16;
-            if (b >= nblk) break;
-            dr_f32x4 z = {0.0f, 0.0f, 0.0f, 0.0f};
-            auto product = [&](int s, const uint4 &w) {
-                const uint4 hi = *(const uint4 *)(s_hi + n16 * LR + 32 * s + 8 * q), lo = *(const uint4 *)(s_lo + n16 * LR + 32 * s + 8 * q);
-                z = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(dr_bf16x8, hi), __builtin_bit_cast(dr_bf16x8, w), z, 0, 0, 0);
-                z = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(dr_bf16x8, lo), __builtin_bit_cast(dr_bf16x8, w), z, 0, 0, 0);
-            };
-#pragma unroll
-            for (int s = 0; s < WS; ++s)
-                if (32 * s < R32) product(s, wd[j][s]);
-            for (int s = WS; 32 * s < R32; ++s) product(s, decay_weights(j, s));
-#pragma unroll
-            for (int i = 0; i < 4; ++i) log_decay(4 * q + i, d, z[i] + db[j]);
-        }
-    }
+    lr.product(low, s_u, wave, lane, [&](int t, int d, float z) { s_l[t * LD + d] = t < c.n && d < D ? -a.decay_scale * stack_sigmoid<F32>(z) : 0.0f; });
     lds_barrier();  // the low-rank input has been read
     {
         float unit[TP];
@@ -342,22 +239,12 @@ __global__ void __launch_bounds__(256) k_delta_prep(const DeltaArgs a) {
             for (int i = 0; i < 4; ++i) s_m[(wave * DC + 4 * q + i) * LM + n16] = acc[i];
     }
     lds_barrier();
-    float *out = a.ws + ((size_t)blockIdx.y * a.H + head) * dr_chunk_floats(D);
+    float *out = a.ws + ((size_t)blockIdx.y * a.H + head) * scan_chunk_floats(SCAN_DELTA, D);
     float *o_r = out + nblk * 256, *o_k = o_r + nblk * 256, *o_a = o_k + nblk * 256, *o_m = o_a + nblk * 256;
     float *s_t = s_m + 4 * DC * LM;
     if (wave == 0) {
-        float tc[DC];  // column n16 of (I + B)^-1: forward substitution, column by column of B (stored transposed: rows are read whole)
-#pragma unroll
-        for (int t = 0; t < DC; ++t) tc[t] = t == n16 ? 1.0f : 0.0f;
-#pragma unroll
-        for (int i = 0; i < DC - 1; ++i)
-#pragma unroll
-            for (int t4 = i / 4; t4 < DC / 4; ++t4) {
-                const dr_f32x4 col = *(const dr_f32x4 *)(s_m + (DC + i) * LM + 4 * t4);
-#pragma unroll
-                for (int k = 0; k < 4; ++k)
-                    if (4 * t4 + k > i) tc[4 * t4 + k] = fmaf(-col[k], tc[i], tc[4 * t4 + k]);
-            }
+        float tc[DC];
+        scan_inverse<LM>(s_m + DC * LM, n16, tc);
         if (q == 0)
 #pragma unroll
             for (int t = 0; t < DC; ++t) s_t[t * LM + n16] = tc[t];
@@ -393,167 +280,6 @@ __global__ void __launch_bounds__(256) k_delta_prep(const DeltaArgs a) {
     }
 }
 
-// A chunk's operands are further away than a chunk takes, so they travel through LDS by DMA, RING - 1 chunks ahead; every wave fetches, waits for and reads
-// only its own.
-template <class E, int NB>
-struct ScanLds {
-    static constexpr int DW = 16 * sizeof(typename E::type) / 4, VI = 16 * DW / 64;  // dwords of a token's 16 values; DMA instructions for the chunk's
-    static constexpr int OPS = 4 * NB + 2 + VI;                                      // DMA instructions per wave and chunk
-    static constexpr int WAVE = (4 * NB + 2) * 1024 + VI * 256, SLOT = 4 * WAVE;
-    static constexpr int PB = NB <= 3 ? 2 : 1;  // buffers of the exchanges between the waves
-    static constexpr int RING = 5 * SLOT <= 128 * 1024 ? 5 : 3 * SLOT <= 136 * 1024 ? 3 : 2;
-};
-template <class E, int NB>
-__global__ void __launch_bounds__(256, 1) k_delta_scan(const DeltaArgs a) {
-    typedef typename E::type T;
-    typedef ScanLds<E, NB> L;
-    __shared__ __attribute__((aligned(1024))) char s_ring[L::RING * L::SLOT];
-    __shared__ dr_f32x4 s_p[L::PB][4][64], s_o[L::PB][4][64];
-    const int D = a.D, nblk = dr_blocks(D), lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), n16 = lane & 15, q = lane >> 4;
-    const int head = (int)blockIdx.x % a.H, cb = (int)blockIdx.x / a.H, col = 16 * cb + n16;  // (head fastest: the column blocks of a head share an L2 where H is a multiple of 8)
-    const RowRun run = a.runs[blockIdx.y];
-    int chunk0 = 0;
-    for (int r = 0; r < (int)blockIdx.y; ++r) chunk0 += (a.runs[r].n_rows + DC - 1) / DC;
-    const int c_lo = max(a.chunk_lo - chunk0, 0), c_hi = min(a.chunk_hi - chunk0, (run.n_rows + DC - 1) / DC);  // this launch's chunks of the run
-    if (c_lo >= c_hi) return;
-    const size_t slot = min((unsigned)a.slots[min(a.row_seq[run.row0], a.n_seqs - 1)], (unsigned)a.n_slots - 1u);
-    float *state = a.state + slot * a.slot_floats + (size_t)head * D * D;
-    const bool fresh = c_lo == 0 && a.pos[run.row0] == 0;
-    dr_f32x4 S[NB];  // S[16 b + 4 q + i][col]
-#pragma unroll
-    for (int j = 0; j < NB; ++j)
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int d = 16 * (wave * NB + j) + 4 * q + i;
-            S[j][i] = !fresh && d < D && col < D ? state[(size_t)d * D + col] : 0.0f;
-        }
-    const size_t per = dr_chunk_floats(D);
-    const float *ws = a.ws + ((ptrdiff_t)(chunk0 - a.chunk_lo) * a.H + head) * (ptrdiff_t)per;  // chunk c of the run at c * H * per
-    const char *vp = (const char *)((const T *)a.raw + (size_t)run.row0 * a.ld + 2 * a.H * a.D8 + head * a.D8 + 16 * cb);
-    const float vbias = a.bias ? BF16::to_f32(a.bias[2 * a.H * a.D8 + head * a.D8 + min(col, D - 1)]) : 0.0f;
-    const unsigned lds0 = (unsigned)(size_t)(__attribute__((address_space(3))) void *)s_ring + (unsigned)(wave * L::WAVE);
-    auto scalar = [&](const void *p) {
-        const unsigned long long v = (unsigned long long)(uintptr_t)p;
-        return (unsigned long long)(unsigned)__builtin_amdgcn_readfirstlane((int)(unsigned)v) | ((unsigned long long)(unsigned)__builtin_amdgcn_readfirstlane((int)(unsigned)(v >> 32)) << 32);
-    };
-    auto fetch = [&](int cc, int at) {  // chunk cc (behind the end: the last one again, the waits count instructions) into ring slot `at`
-        const int c = min(cc, c_hi - 1);
-        const unsigned dst0 = lds0 + (unsigned)(at * L::SLOT);
-        const unsigned long long base = scalar(ws + (size_t)c * a.H * per);
-        auto piece = [&](unsigned byte, unsigned dst) {
-            unsigned keep;
-            asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %3\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, %2\n\ts_mov_b32 m0, %0"
-                         : "=&s"(keep)
-                         : "v"(byte + (unsigned)lane * 16u), "s"(base), "s"(dst)
-                         : "memory");
-        };
-#pragma unroll
-        for (int j = 0; j < NB; ++j) {
-            const int b = min(wave * NB + j, nblk - 1);  // (blocks past the end meet channels that stay zero)
-#pragma unroll
-            for (int k = 0; k < 4; ++k) piece((unsigned)(k * nblk + b) * 1024u, dst0 + (unsigned)(4 * j + k) * 1024u);
-        }
-        piece((unsigned)nblk * 4096u + (unsigned)min(wave, 2) * 1024u, dst0 + 4096u * NB);
-        piece((unsigned)nblk * 4096u + 3072u, dst0 + 4096u * NB + 1024u);  // W_16 of all channels (and what lies behind it)
-        const unsigned long long vbase = scalar(vp + (size_t)(DC * c) * a.ld * sizeof(T));
-#pragma unroll
-        for (int k = 0; k < L::VI; ++k) {
-            const int t = min((64 / L::DW) * k + lane / L::DW, run.n_rows - 1 - DC * c);
-            const unsigned off = (unsigned)(t * a.ld) * (unsigned)sizeof(T) + (unsigned)(lane % L::DW) * 4u;
-            unsigned keep;
-            asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %3\n\ts_nop 0\n\tglobal_load_lds_dword %1, %2\n\ts_mov_b32 m0, %0"
-                         : "=&s"(keep)
-                         : "v"(off), "s"(vbase), "s"(dst0 + 4096u * NB + 2048u + 256u * k)
-                         : "memory");
-        }
-    };
-    const dr_f32x4 zero = {0.0f, 0.0f, 0.0f, 0.0f};
-    auto store_o = [&](int c) {  // chunk c's outputs: one per thread
-        const float *p = (const float *)s_o[c % L::PB] + threadIdx.x;
-        const float o = (p[0] + p[256]) + (p[512] + p[768]);
-        const int l = threadIdx.x >> 2, t = DC * c + 4 * (l >> 4) + (threadIdx.x & 3), d = 16 * cb + (l & 15);
-        if (t < run.n_rows && d < D) a.o[((size_t)(run.row0 + t) * a.H + head) * a.D8 + d] = o;
-    };
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // (the state's loads: the waits below count DMAs)
-#pragma unroll
-    for (int i = 0; i < L::RING - 1; ++i) fetch(c_lo + i, i);
-    int at = 0;
-    for (int c = c_lo; c < c_hi; ++c) {
-        asm volatile("s_waitcnt vmcnt(%0)" ::"n"((L::RING - 2) * L::OPS) : "memory");
-        fetch(c + L::RING - 1, at ? at - 1 : L::RING - 1);  // into the previous chunk's slot
-        const char *mine = s_ring + at * L::SLOT + wave * L::WAVE;
-        at = at + 1 < L::RING ? at + 1 : 0;
-        auto operand = [&](int piece) { return *(const dr_f32x4 *)(mine + piece * 1024 + lane * 16); };
-        dr_f32x4 u[NB], r[NB], k[NB], m[NB], w[NB], v, x = operand(4 * NB);
-#pragma unroll
-        for (int j = 0; j < NB; ++j) u[j] = operand(4 * j);
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int t = 4 * q + i;
-            const float e = E::load((const T *)(mine + (4 * NB + 2) * 1024) + t * 16 + n16) + vbias;
-            v[i] = DC * c + t < run.n_rows && col < D ? e : 0.0f;
-        }
-#pragma unroll
-        for (int j = 0; j < NB; ++j) r[j] = operand(4 * j + 1), k[j] = operand(4 * j + 2), w[j] = *(const dr_f32x4 *)(mine + (4 * NB + 1) * 1024 + (16 * min(wave * NB + j, nblk - 1) + 4 * q) * 4);
-        dr_f32x4 P = zero, O = zero;
-#pragma unroll
-        for (int j = 0; j < NB; ++j)
-#pragma unroll
-            for (int i = 0; i < 4; ++i) P = dr_mfma(u[j][i], S[j][i], P);
-        if (wave == 0)
-#pragma unroll
-            for (int i = 0; i < 4; ++i) P = dr_mfma(x[i], v[i], P);
-        s_p[c % L::PB][wave][lane] = P;
-#pragma unroll
-        for (int j = 0; j < NB; ++j) m[j] = operand(4 * j + 3);
-#pragma unroll
-        for (int j = 0; j < NB; ++j)
-#pragma unroll
-            for (int i = 0; i < 4; ++i) O = dr_mfma(r[j][i], S[j][i], O);
-        if (wave == 1)
-#pragma unroll
-            for (int i = 0; i < 4; ++i) O = dr_mfma(x[i], v[i], O);
-#pragma unroll
-        for (int j = 0; j < NB; ++j) S[j] *= w[j];
-#pragma unroll
-        for (int i = 0; i < 4; ++i)
-#pragma unroll
-            for (int j = 0; j < NB; ++j) S[j] = dr_mfma(k[j][i], v[i], S[j]);
-        // the four waves' shares of P meet (LDS only: the DMAs stay in flight)
-        asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
-        P = (s_p[c % L::PB][0][lane] + s_p[c % L::PB][1][lane]) + (s_p[c % L::PB][2][lane] + s_p[c % L::PB][3][lane]);
-        if (c > c_lo) store_o(c - 1);
-#pragma unroll
-        for (int i = 0; i < 4; ++i)
-#pragma unroll
-            for (int j = 0; j < NB; ++j) S[j] = dr_mfma(m[j][i], P[i], S[j]);
-        if (wave == 2)
-#pragma unroll
-            for (int i = 0; i < 4; ++i) O = dr_mfma(x[i], P[i], O);
-#pragma unroll
-        for (int j = 0; j < NB; ++j)
-            if (wave * NB + j >= nblk) S[j] = zero;  // (a block that does not exist saw another's operands)
-        if constexpr (L::PB == 1) asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");  // everyone has read P and the previous outputs
-        s_o[c % L::PB][wave][lane] = O;
-    }
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // the look-ahead DMAs: LDS is handed on when the workgroup ends
-    __syncthreads();
-    store_o(c_hi - 1);
-#pragma unroll
-    for (int j = 0; j < NB; ++j)
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            const int d = 16 * (wave * NB + j) + 4 * q + i;
-            if (d < D && col < D) state[(size_t)d * D + col] = S[j][i];
-        }
-}
-
-// chunks whose operands are made and used at a time
-int delta_segment(int H, int D) {
-    const size_t bytes = H * dr_chunk_floats(D) * 4;
-    return (int)std::max((size_t)16, DELTA_SEGMENT_BYTES / bytes);
-}
-
 size_t delta_prep_lds(int NB, int R8) {
     const int R32 = (R8 + 31) & ~31;
     const size_t vec = (size_t)DC * (64 * NB + 4) * 4, low = (size_t)DC * (R32 + 8) * 4;  // (fp32, or bf16 halves)
@@ -570,16 +296,16 @@ int delta_chunks_nb(const DeltaArgs &a, int chunks, int row0, int rows, hipStrea
         raised = true;
     }
     DeltaArgs seg = a;
-    const int step = delta_segment(a.H, a.D);
-    for (int c = 0; c < chunks; c += step) {  // a segment's operands are read back before they leave the last-level cache
-        seg.chunk_lo = c, seg.chunk_hi = std::min(chunks, c + step);
-        hipLaunchKernelGGL((k_delta_prep<E, NB>), dim3((unsigned)a.H, (unsigned)(seg.chunk_hi - c)), dim3(256), lds, st, seg);
-        PIE_LAUNCH_CHECK();
-        hipLaunchKernelGGL((k_delta_scan<E, NB>), dim3((unsigned)(a.H * dr_blocks(a.D)), (unsigned)a.n_runs), dim3(256), 0, st, seg);
-        PIE_LAUNCH_CHECK();
-    }
+    const int v0 = 2 * a.H * a.D8;
+    const ScanArgs scan = {(const typename E::type *)a.raw + v0, a.bias ? a.bias + v0 : nullptr, a.ld, a.H, a.D, a.D, a.D8, a.pos, a.row_seq, a.slots, a.n_seqs, a.n_slots, a.runs, a.n_runs, a.state,
+                           a.slot_floats, a.ws, a.o, 0, 0};
+    const int rc = scan_chunks<E, NB, SCAN_DELTA>(scan, chunks, st, [&](int lo, int hi) {
+        seg.chunk_lo = lo, seg.chunk_hi = hi;
+        hipLaunchKernelGGL((k_delta_prep<E, NB>), dim3((unsigned)a.H, (unsigned)(hi - lo)), dim3(256), lds, st, seg);
+    });
+    if (rc) return rc;
     const int g0 = 3 * a.H * a.D8;
-    const HeadOutArgs h = {a.o, nullptr, (const typename E::type *)a.raw + g0, a.bias ? a.bias + g0 : nullptr, a.ld, a.H, a.D, a.D8, a.o_norm, a.eps, a.out, a.ld_out};
+    const HeadOutArgs h = {a.o, nullptr, (const typename E::type *)a.raw + g0, a.bias ? a.bias + g0 : nullptr, a.ld, a.H, a.D, a.D8, a.o_norm, a.eps, a.out, a.ld_out, false, false, 1.0f};
     return head_out_launch(sizeof(typename E::type) == 4 ? PIE_F32 : PIE_BF16, h, row0, rows, st);
 }
 template <class E>
@@ -610,8 +336,8 @@ int delta_step_go(const DeltaArgs &a, hipStream_t st) {
 }  // namespace
 
 int delta_chunks(int n_rows) { return (n_rows + DC - 1) / DC; }
-size_t delta_ws_floats(int chunks, int H, int D) { return (size_t)std::min(chunks, delta_segment(H, D)) * H * dr_chunk_floats(D); }
-int delta_launches(int chunks, int H, int D) { return 2 * ((chunks + delta_segment(H, D) - 1) / delta_segment(H, D)) + 1; }
+size_t delta_ws_floats(int chunks, int H, int D) { return scan_ws_floats(SCAN_DELTA, chunks, H, D); }
+int delta_launches(int chunks, int H, int D) { return scan_launches(SCAN_DELTA, chunks, H, D) + 1; }
 
 static int delta_check(const DeltaArgs &a) {
     PIE_REQUIRE(a.D > 0 && a.D <= DELTA_MAX_DIM && a.rank > 0 && a.rank <= DELTA_MAX_RANK && a.H > 0 && a.H <= 65535, PIE_E_SHAPE,

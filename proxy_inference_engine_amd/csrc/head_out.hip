@@ -1,5 +1,5 @@
 // head_out.hip -- what stands between a recurrence and its output projection: every head's output (over a denominator of its own, where there is one) over its
-// root mean square, times a weight and the sigmoid of its gate.  One wave per row and HB heads; lanes own channel pairs, NP each.
+// root mean square, times a weight and the sigmoid (or silu) of its gate.  One wave per row and HB heads; lanes own channel pairs, NP each.
 #include "stack_types.hpp"
 
 namespace {
@@ -32,7 +32,8 @@ __global__ void __launch_bounds__(256) k_head_out(const HeadOutArgs a, int row0)
                 const u32 v = *(const u32 *)(a.gate_bias + at);
                 g[k][p].x += lo_f32<BF16>(v), g[k][p].y += hi_f32<BF16>(v);
             }
-            w[k][p] = make_float2(a.w[head * D + min(d, D - 1)], a.w[head * D + min(d + 1, D - 1)]);
+            const float *wh = a.w + (a.shared_w ? 0 : head * D);
+            w[k][p] = make_float2(wh[min(d, D - 1)], wh[min(d + 1, D - 1)]);
         }
     }
     const float inv_d = 1.0f / (float)D;
@@ -54,7 +55,8 @@ __global__ void __launch_bounds__(256) k_head_out(const HeadOutArgs a, int row0)
         for (int p = 0; p < NP; ++p) {
             const int d = 2 * (lane + 64 * p);
             if (d >= D) break;
-            const float x = o[k][p].x * inv * w[k][p].x * stack_sigmoid<F32>(g[k][p].x), y = o[k][p].y * inv * w[k][p].y * stack_sigmoid<F32>(g[k][p].y);  // (past an odd head's end: zero)
+            float x = o[k][p].x * inv * w[k][p].x * stack_sigmoid<F32>(g[k][p].x), y = o[k][p].y * inv * w[k][p].y * stack_sigmoid<F32>(g[k][p].y);  // (past an odd head's end: zero)
+            x *= a.silu ? g[k][p].x * a.scale : a.scale, y *= a.silu ? g[k][p].y * a.scale : a.scale;
             if constexpr (F32) *(float2 *)(out + d) = make_float2(x, y);
             else *(u32 *)(out + d) = pack2<BF16>(x, y);
         }

@@ -7,11 +7,15 @@
 //                         With a query latent: [query latent | latent | rotated key | gate] Linear; norms, key rotation, append; queries out of their latent, rotated
 //   attention             [q | k | v | gate] Linear; norms, rotation and page writes; attention over keys and values (page_attn.hip)
 //   delta rule            [r | k | v | gate | rate | decay] Linear; recurrence (delta_rule.hip)
+//   gated delta rule      [q | k | v | gate | step | decay] Linear; short convolution and recurrence (gated_delta.hip)
+//   time mixing           the row and its predecessor mixed five ways, beside the update in front; Linears of the mixes; recurrence (time_mix.hip).  It runs alone or
+//                         beside an attention over the same row: then one list of Linears makes both inputs (few rows), and one output projection reads both outputs
 //   mLSTM                 [q | k | v | gate | i | f] Linear; recurrence (mlstm.hip); head norm and gate (head_out.hip)
 //   minGRU                [z | candidate | gate] Linear; recurrence (mingru.hip)
-// and an output projection.  Feed-forwards: dense up (relu^2 or xIELU), down; or experts: gate|up and down over the active experts (and a shared one).
+// and an output projection.  Feed-forwards: dense up (relu^2, xIELU, or a gelu gate and up), down; or experts: gate|up and down over the active experts (and a shared one).
 // Norms: element-wise ones ride in the epilogue of the kernel that produces their input (x += post(y), h = next(x)); a norm over the whole row is applied,
 // with the same additions, by one launch behind the sublayer (row_update.hip), which also takes the experts' weighted sum.
+// A layer may norm the sum instead (x = post(alpha x + y)), and may add, behind its sublayers, a vector of the row's token that the row gates (side input: gate Linear, projection, update).
 // Hyper-connections keep several residual streams: one launch behind every sublayer mixes them, takes the next sublayer's input out of them, and norms (and, for a mixer,
 // convolves) it (stream_update.hip); the first one starts the streams from the embedding.
 // A pass of more rows than the weight-streaming Linear is for (BIG_ROWS; bf16) multiplies through the tiled GEMMs instead (w16_gemm.hpp, grouped by expert
@@ -30,7 +34,7 @@
 size_t w16l_workspace_bytes(int M, int N, int K);
 int w16l_gemm_launch(int dtype, const void *w16m, const void *x, int ldx, int M, int N, int K, void *y, void *workspace, hipStream_t st, const void *bias,
                      void *swiglu_act, bool *fused, int ldy);
-int w16l_act_launch(const void *w16m, const void *x, int ldx, int M, int N, int K, void *y, int ldy, int act, float alpha, float beta, hipStream_t st);
+int w16l_act_launch(const void *w16m, const void *x, int ldx, int M, int N, int K, void *y, int ldy, int act, float alpha, float beta, const void *bias, hipStream_t st);
 int w16l_grouped_launch(const void *w16m, size_t w_stride, const void *x, int ldx, size_t x_rows, const int *list, const void *tiles, int tm, int block, int tile_rows, int N, int K,
                         void *y, int ldy, int act, float act_alpha, float act_limit, hipStream_t st);
 
@@ -97,25 +101,37 @@ __device__ __forceinline__ void store4(typename E::type *p, float4 y) {
     else *(float4 *)p = y;
 }
 template <class E>
-__global__ void __launch_bounds__(256) k_stack_embed(const int *ids, const u16 *table, int vocab, int W, float scale, bool plain, PointNorm next, float *x, int ldx,
-                                                     typename E::type *h, int ldh) {  // plain: h = x
+__global__ void __launch_bounds__(256) k_stack_embed(const int *ids, const u16 *table, int vocab, int W, float scale, const u16 *positions, int max_positions, const int *pos, bool plain, PointNorm next,
+                                                     float *x, int ldx, typename E::type *h, int ldh) {  // plain: h = x; positions: nullable
     const size_t m = blockIdx.y;
     const int n = (blockIdx.x * 256 + threadIdx.x) * 4;
     if (n >= W) return;
-    const u16 *src = table + (size_t)min(max(ids[m], 0), vocab - 1) * W + n;
+    const u16 *src = table + (size_t)min(max(ids[m], 0), vocab - 1) * W + n, *at = positions ? positions + (size_t)min(max(pos[m], 0), max_positions - 1) * W + n : nullptr;
     if (n + 4 <= W && !(W & 3)) {
         const uint2 t = *(const uint2 *)src;
-        const float4 v = make_float4(lo_f32<BF16>(t.x) * scale, hi_f32<BF16>(t.x) * scale, lo_f32<BF16>(t.y) * scale, hi_f32<BF16>(t.y) * scale);
+        float4 v = make_float4(lo_f32<BF16>(t.x) * scale, hi_f32<BF16>(t.x) * scale, lo_f32<BF16>(t.y) * scale, hi_f32<BF16>(t.y) * scale);
+        if (at) {
+            const uint2 p = *(const uint2 *)at;
+            v.x += lo_f32<BF16>(p.x), v.y += hi_f32<BF16>(p.x), v.z += lo_f32<BF16>(p.y), v.w += hi_f32<BF16>(p.y);
+        }
         const float4 y = plain ? v : point_norm4(next, n, v);
         *(float4 *)(x + m * ldx + n) = v;
         store4<E>(h + m * ldh + n, y);
         return;
     }
     for (int i = 0; i < min(4, W - n); ++i) {
-        const float v = BF16::to_f32(src[i]) * scale;
+        const float v = BF16::to_f32(src[i]) * scale + (at ? BF16::to_f32(at[i]) : 0.0f);
         x[m * ldx + n + i] = v;
         h[m * ldh + n + i] = E::pack(plain ? v : point_norm(next, n + i, v));
     }
+}
+
+// y = gelu(y) * the row's token's side vector (bf16, many rows)
+__global__ void __launch_bounds__(256) k_side_gate(u16 *y, int ldy, TokenVectors side, int M, int N) {
+    const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x, m = i / N, n = i % N;
+    if (m >= (size_t)M) return;
+    u16 *p = y + m * ldy + n;
+    *p = BF16::from_f32(gelu_tanh<false>(BF16::to_f32(*p)) * BF16::to_f32(token_vector(side, m)[n]));
 }
 
 // y = sum over the token's slots of its experts' weighted outputs (+ sigmoid(gate . input) * shared output); x += post(y); h = next(x)
@@ -315,7 +331,7 @@ struct pie_stack {
     std::vector<char> have;
     // workspace, by rows of a pass
     Buf<float> x, c_raw, part, part_s, attn_ws, gemm_ws, y32, logits_e, rec_ws, rec_o, rec_den;
-    Buf<char> h, hc, q, qu, cq, ql, oc, o, act, act_e, act_s, y, ctx, kv;
+    Buf<char> h, hc, q, qu, cq, ql, oc, o, act, act_e, act_s, y, ctx, kv, mixes, mixed, side;
     Buf<RowStat> stats;
     Buf<int> route_ints;
     Buf<RouteLayer> route_dev;
@@ -342,7 +358,9 @@ PointNorm norm_of(const pie_stack_norm &n) { return {n.w, n.b, n.param}; }
 StackNorm row_norm_of(const pie_stack_norm &n) { return {n.w, n.b, n.param, n.kind}; }
 bool is_moe(const pie_stack_layer &L) { return L.ff == PIE_FF_TABLE_MOE || L.ff == PIE_FF_ROUTED_MOE; }
 KvGeometry geometry(const pie_stack_layer &L) { return kv_geometry(L.heads, L.kv_heads, L.dim, L.vdim); }
-bool is_dense(const pie_stack_layer &L) { return L.ff == PIE_FF_RELU2 || L.ff == PIE_FF_XIELU; }
+bool is_dense(const pie_stack_layer &L) { return L.ff == PIE_FF_RELU2 || L.ff == PIE_FF_XIELU || L.ff == PIE_FF_GEGLU; }
+bool has_time_mix(const pie_stack_layer &L) { return L.time_mix.heads > 0; }
+int gated_channels(const pie_stack_layer &L);
 bool own_cache(const pie_stack_layer &L) { return (L.mixer == PIE_MIXER_LATENT && (!L.q_rank || L.kv_from < 0)) || (L.mixer == PIE_MIXER_ATTENTION && L.kv_from < 0); }
 // columns of the mixer's input projection, and what its output projection reads
 int in_columns(const pie_stack_layer &L) {
@@ -354,16 +372,25 @@ int in_columns(const pie_stack_layer &L) {
         case PIE_MIXER_DELTA: return 5 * L.heads * up8(L.dim) + up8(L.rank);
         case PIE_MIXER_MLSTM: return 2 * L.heads * (up8(L.dim) + up8(L.vdim)) + 2 * up8(L.heads);
         case PIE_MIXER_MINGRU: return 3 * up8(L.dim);
-        default: return L.heads * up8(L.dim) + (own_cache(L) ? L.kv_heads * (up8(L.dim) + up8(L.vdim)) : 0) + gate;
+        case PIE_MIXER_GATED_DELTA: return gated_channels(L) + L.heads * up8(L.vdim) + 2 * up8(L.heads);
+        case PIE_MIXER_TIME_MIX: return 0;
+        default: return L.heads * up8(L.dim) + (own_cache(L) ? L.kv_heads * (up8(L.dim) + (L.row_norm ? 0 : up8(L.vdim))) : 0) + gate;
     }
 }
-int out_columns(const pie_stack_layer &L) { return L.heads * up8(L.mixer == PIE_MIXER_DELTA || L.mixer == PIE_MIXER_MINGRU ? L.dim : L.vdim); }
+int time_mix_columns(const pie_stack_layer &L) { return has_time_mix(L) ? L.time_mix.heads * up8(L.time_mix.dim) : 0; }  // of each of its projections, and of its output
+int out_columns(const pie_stack_layer &L) {
+    if (L.mixer == PIE_MIXER_TIME_MIX) return time_mix_columns(L);
+    return L.heads * up8(L.mixer == PIE_MIXER_DELTA || L.mixer == PIE_MIXER_MINGRU ? L.dim : L.vdim) + time_mix_columns(L);
+}
+int gated_channels(const pie_stack_layer &L) { return gated_delta_channels(L.heads, L.kv_heads, up8(L.dim), up8(L.vdim)); }
 int up4(int n) { return (n + 3) & ~3; }
 int latent_row(const pie_stack_layer &L) { return up8(L.rank) + up8(L.rot_dim); }  // numbers of a cached latent row
 
-// A layer's recurrent state: the mixer's, the last inputs of the convolution in front of it, and (layer 0) the embedding's previous token
+// A layer's recurrent state: the mixer's (a gated delta rule's with its convolution's last inputs at `ring`), the last inputs of the convolution in front of it, (layer 0) the embedding's
+// previous token, and the previous row that time mixing reads
 struct StateLayout {
     size_t conv, prev, total;  // where the second and the third begin
+    size_t ring, row;
 };
 StateLayout state_layout(const pie_stack *s, int i) {
     const pie_stack_layer &L = s->layers[i];
@@ -371,10 +398,16 @@ StateLayout state_layout(const pie_stack *s, int i) {
     if (L.mixer == PIE_MIXER_DELTA) mixer = (size_t)L.heads * L.dim * L.dim;
     else if (L.mixer == PIE_MIXER_MLSTM) mixer = mlstm_state_floats(L.heads, L.dim, L.vdim);
     else if (L.mixer == PIE_MIXER_MINGRU) mixer = L.dim;
-    const size_t conv = L.conv_taps > 1 ? (size_t)(L.conv_taps - 1) * up4(s->cfg.width) : 0, prev = i == 0 && s->cfg.bigram ? 4 : 0;
-    if (!conv && !prev && (L.mixer == PIE_MIXER_DELTA || !mixer)) return {mixer, mixer, mixer};
+    else if (has_time_mix(L)) mixer = (size_t)L.time_mix.heads * L.time_mix.dim * L.time_mix.dim;
+    size_t ring = 0;
+    if (L.mixer == PIE_MIXER_GATED_DELTA) {
+        ring = ((size_t)L.heads * L.dim * L.vdim + 3) / 4 * 4;
+        mixer = ring + (L.mix_taps > 1 ? (size_t)L.mix_taps * gated_channels(L) : 0);
+    }
+    const size_t row = has_time_mix(L) ? up4(s->cfg.width) : 0, conv = L.conv_taps > 1 ? (size_t)(L.conv_taps - 1) * up4(s->cfg.width) : 0, prev = i == 0 && s->cfg.bigram ? 4 : 0;
+    if (!conv && !prev && (L.mixer == PIE_MIXER_DELTA || !mixer)) return {mixer, mixer, mixer, 0, 0};
     mixer = (mixer + 3) / 4 * 4;
-    return {mixer, mixer + conv, mixer + conv + prev};
+    return {mixer, mixer + conv, mixer + conv + prev + row, ring, mixer + conv + prev};
 }
 
 // How a pass is laid out: rows of the leading short runs, and what the long runs behind them see.
@@ -411,20 +444,21 @@ ChunkPart chunk_part(const pie_stack *s, const pie_stack_batch &b, const pie_sta
     while (p.runs < b.n_runs && (!chunks || b.runs_host[4 * p.runs + 1] < CHUNK_RUN)) p.rows += b.runs_host[4 * p.runs++ + 1];
     for (int i = p.runs; i < b.n_runs; ++i) {
         const int n = b.runs_host[4 * i + 1];
-        p.chunks += L.mixer == PIE_MIXER_DELTA ? delta_chunks(n) : L.mixer == PIE_MIXER_MLSTM ? mlstm_chunks(n) : mingru_chunks(n);
+        p.chunks += L.mixer == PIE_MIXER_MLSTM ? mlstm_chunks(n) : L.mixer == PIE_MIXER_MINGRU ? mingru_chunks(n) : delta_chunks(n);
     }
     return p;
 }
 
 int stack_reserve(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipStream_t st) {
     const size_t M = (size_t)b.n_rows, E = esize(s), W64 = up64(s->cfg.width), WA = act_stride(s->cfg.width);
-    size_t q = 0, c = 0, ql = 0, o = 0, act = 0, act_e = 0, act_s = 0, part = 0, part_s = 0, ints = 0, ctx = 0, kv = 0, ws = 0, le = 0, rw = 0, ro = 0, rd = 0, hc = 0, qu = 0, cq = 0;
+    size_t mx = 0, md = 0, sd = 0, q = 0, c = 0, ql = 0, o = 0, act = 0, act_e = 0, act_s = 0, part = 0, part_s = 0, ints = 0, ctx = 0, kv = 0, ws = 0, le = 0, rw = 0, ro = 0, rd = 0, hc = 0, qu = 0, cq = 0;
     const size_t streams = std::max(s->cfg.streams, 1);
     auto gemm = [&](int N, int K) { ws = std::max(ws, w16l_workspace_bytes((int)M, N, K) / 4); };
     for (const pie_stack_layer &L : s->layers) {
         const int NI = in_columns(L), KO = out_columns(L);
         q = std::max(q, (size_t)NI), o = std::max(o, (size_t)act_stride(KO));
-        if (plan.big) gemm(NI, s->cfg.width), gemm(s->cfg.width, KO);
+        if (plan.big && NI) gemm(NI, s->cfg.width);
+        if (plan.big) gemm(s->cfg.width, KO);
         if (L.mixer == PIE_MIXER_LATENT) {
             c = std::max(c, (size_t)up8(L.rank)), ql = std::max(ql, (size_t)L.heads * up8(L.rank));
             if (L.q_rank) {
@@ -439,6 +473,21 @@ int stack_reserve(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
             }
         }
         if (L.conv_taps > 0 && b.n_runs < b.n_rows) hc = WA;
+        if (L.mixer == PIE_MIXER_GATED_DELTA) {
+            const int chunks = chunk_part(s, b, L).chunks;
+            md = std::max(md, (size_t)gated_channels(L)), ro = std::max(ro, (size_t)L.heads * up8(L.vdim));
+            if (chunks) rw = std::max(rw, gated_delta_ws_floats(chunks, L.heads, L.dim));
+        }
+        if (has_time_mix(L)) {
+            const int chunks = chunk_part(s, b, L).chunks, NT = time_mix_columns(L), R8 = up8(L.time_mix.rank);
+            mx = TIME_MIXES * WA, md = std::max(md, (size_t)4 * NT + R8), ro = std::max(ro, (size_t)NT);
+            if (chunks) rw = std::max(rw, time_mix_ws_floats(chunks, L.time_mix.heads, L.time_mix.dim));
+            if (plan.big) gemm(NT, s->cfg.width), gemm(R8, s->cfg.width);
+        }
+        if (L.w_side_gate) {
+            sd = act_stride(s->cfg.side_dim);
+            if (plan.big) gemm(up8(s->cfg.side_dim), s->cfg.width), gemm(s->cfg.width, s->cfg.side_dim);
+        }
         if (L.mixer == PIE_MIXER_MLSTM) ro = std::max(ro, (size_t)L.heads * up8(L.vdim)), rd = std::max(rd, (size_t)L.heads);
         if (L.mixer == PIE_MIXER_DELTA || L.mixer == PIE_MIXER_MLSTM || L.mixer == PIE_MIXER_MINGRU) {
             const int chunks = chunk_part(s, b, L).chunks;
@@ -466,7 +515,7 @@ int stack_reserve(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
         (rc = s->o.need(M * o * E, &moved)) || (rc = s->act.need(M * act * E, &moved)) || (rc = s->act_e.need(M * act_e * E, &moved)) ||
         (rc = s->act_s.need(M * act_s * E, &moved)) || (rc = s->stats.need((size_t)b.n_want * ST_TILES, &moved)) || (rc = s->y.need(plan.big ? M * W64 * E : 0, &moved)) ||
         (rc = s->y32.need(plan.big ? 0 : M * W64, &moved)) || (rc = s->logits_e.need(M * le, &moved)) || (rc = s->rec_ws.need(rw, &moved)) || (rc = s->rec_o.need(M * ro, &moved)) ||
-        (rc = s->rec_den.need(M * rd, &moved)) || (rc = s->hc.need(M * hc * E, &moved)) || (rc = s->qu.need(M * qu * E, &moved)) || (rc = s->cq.need(M * cq * E, &moved)) || (rc = s->ctx.need(ctx * E, &moved)) ||
+        (rc = s->rec_den.need(M * rd, &moved)) || (rc = s->hc.need(M * hc * E, &moved)) || (rc = s->mixes.need(M * mx * E, &moved)) || (rc = s->mixed.need(M * md * E, &moved)) || (rc = s->side.need(M * sd * E, &moved)) || (rc = s->qu.need(M * qu * E, &moved)) || (rc = s->cq.need(M * cq * E, &moved)) || (rc = s->ctx.need(ctx * E, &moved)) ||
         (rc = s->kv.need(kv * E, &moved)) || (rc = s->gemm_ws.need(ws, &moved)))
         return rc;
     int n_moe = 0;
@@ -511,6 +560,7 @@ int plan_splits(const pie_stack_batch &b, const pie_stack_layer &L, int n_tiles)
     if (n_tiles <= 0) return 1;
     long ctx = (long)b.table_width * PAGE_TOKENS;
     if (L.window > 0 && L.window + 64 < ctx) ctx = L.window + 64;
+    if (L.chunk > 0 && L.chunk + 64 < ctx) ctx = L.chunk + 64;
     long s = 256 / n_tiles;
     s = std::min(s, ctx / 64);
     s = std::min(s, 64L);
@@ -536,12 +586,22 @@ size_t attn_ws(const pie_stack *s, const pie_stack_batch &b, const Plan &plan, c
     return L.mixer == PIE_MIXER_ATTENTION ? page_attn_ws_floats(p.M, geometry(L), splits) : latent_attn_ws_floats(p.M, L.heads, L.rank, splits);
 }
 
-// what a sublayer's input is made of: the norm in front of it, with hyper-connections the streams' shares (nullptr: their sum), and the layer whose convolution follows (or -1)
+// what a sublayer's input is made of: the norm in front of it, with hyper-connections the streams' shares (nullptr: their sum), the layer whose convolution follows (or -1), and the layer
+// whose time mixing reads it (or -1)
 struct Into {
     const pie_stack_norm *norm;
     const float *in;
-    int conv;
+    int conv, mix;
 };
+// what a sublayer's output goes through on its way into the residual: x += norm(y + bias), or (after) x = norm(scale x + y + bias)
+struct OutOf {
+    const pie_stack_norm &norm;
+    const float *hyper;  // hyper-connections: the sublayer's, instead
+    const u16 *bias;
+    bool after;
+    float scale;
+};
+OutOf out_of(const pie_stack_layer &L, const pie_stack_norm &norm, const float *hyper, const void *bias) { return {norm, hyper, (const u16 *)bias, L.norm_after != 0, L.residual_scale}; }
 
 struct Pass {
     pie_stack *s;
@@ -593,55 +653,70 @@ struct Pass {
     }
     // x += post(y); h = next(x) over y = s->y (bf16; many rows) or s->y32
     // route (few rows): the layer whose experts the rows choose on their way
-    void update(const pie_stack_norm &post, const Into &into, const u16 *bias = nullptr, int route = -1) {
+    TokenMixArgs mix_args(int li) const {
+        TokenMixArgs t = {};
+        const StateLayout at = state_layout(s, li);
+        t.mu = s->layers[li].time_mix.mu, t.ldmu = up64(s->cfg.width), t.state = b.states[li] + at.row, t.slot_floats = at.total;
+        t.pos = b.pos, t.row_seq = b.row_seq, t.slots = b.slots, t.n_seqs = b.n_seqs, t.n_slots = (int)b.n_slots, t.runs = (const RowRun *)b.runs, t.n_runs = b.n_runs;
+        t.out = s->mixes.p, t.ldo = act_stride(s->cfg.width);
+        return t;
+    }
+    // the mixes that layer li's time mixing reads, of the residual as it stands
+    void token_mix(int li) {
+        if (!rc) rc = token_mix_launch(s->cfg.dtype, mix_args(li), s->x.p, up64(s->cfg.width), b.n_rows, s->cfg.width, st), ++launches;
+    }
+    void update(const OutOf &out, const Into &into, int route = -1) {
         if (rc) return;
-        const pie_stack_norm &next = *into.norm;
+        const pie_stack_norm &next = *into.norm, &post = out.norm;
         const int W = s->cfg.width, W64 = up64(W), WA = act_stride(W);
-        if (plan.big && pointwise(post) && pointwise(next) && !bias) {
+        const bool single = b.n_runs == b.n_rows;
+        if (plan.big && pointwise(post) && pointwise(next) && !out.bias && !out.after && into.mix < 0) {
             hipLaunchKernelGGL(k_point_residual, dim3((unsigned)((W + 1023) / 1024), (unsigned)b.n_rows), dim3(256), 0, st, (const u16 *)s->y.p, W, norm_of(post), norm_of(next), s->x.p, W64,
                                (u16 *)s->h.p, WA, W);
             if (hipGetLastError() != hipSuccess) rc = pie::fail(PIE_E_HIP, "residual launch failed");
         } else {
             RowUpdateArgs a = {};
-            a.y = plan.big ? (const void *)s->y.p : s->y32.p, a.y32 = !plan.big, a.ldy = plan.big ? W : W64, a.bias = bias;
+            a.y = plan.big ? (const void *)s->y.p : s->y32.p, a.y32 = !plan.big, a.ldy = plan.big ? W : W64, a.bias = out.bias, a.after = out.after, a.alpha = out.scale;
+            if (into.mix >= 0 && single) a.mix = mix_args(into.mix);
             a.post = row_norm_of(post), a.next = row_norm_of(next), a.x = s->x.p, a.ldx = W64, a.h = s->h.p, a.ldh = WA, a.M = b.n_rows, a.W = W;
             if (route >= 0) a.route = s->route_dev.p + s->route_at[route], a.experts = s->layers[route].experts, a.router = (const u16 *)s->layers[route].w_router_rows, a.arrived = s->arrived.p;
             rc = row_update_launch(s->cfg.dtype, a, st);
         }
         ++launches;
+        if (into.mix >= 0 && !single) token_mix(into.mix);
     }
-    // a sublayer's last product [W, K], its norm, the residual sum and the next sublayer's norm; hyper (or null): its connections
-    void output(const void *w, const void *x, int ldx, int K, const pie_stack_norm &post, const Into &next, const float *hyper, const u16 *bias = nullptr,
-                int route = -1) {
+    // a sublayer's last product [W, K], its norm, the residual sum and the next sublayer's norm
+    void output(const void *w, const void *x, int ldx, int K, const OutOf &out, const Into &next, int route = -1) {
         const int W = s->cfg.width, W64 = up64(W), WA = act_stride(W), M = b.n_rows;
         if (plan.big) {
             gemm(w, x, ldx, M, W, K, s->y.p, W);
-            return hyper ? streams(hyper, next) : update(post, next, bias);
+            return out.hyper ? streams(out.hyper, next) : update(out, next);
         }
         RowsArgs o = {};
         o.m = {(const char *)w, W, K, x, ldx, s->y32.p, W64};
         o.M = M;
-        if (!hyper && pointwise(post) && pointwise(*next.norm) && !bias && route < 0) {
-            o.epi = ROWS_RESIDUAL, o.res = s->x.p, o.ld_res = W64, o.post = norm_of(post), o.next = norm_of(*next.norm), o.h = s->h.p, o.ldh = WA;
+        if (!out.hyper && pointwise(out.norm) && pointwise(*next.norm) && !out.bias && !out.after && route < 0 && next.mix < 0) {
+            o.epi = ROWS_RESIDUAL, o.res = s->x.p, o.ld_res = W64, o.post = norm_of(out.norm), o.next = norm_of(*next.norm), o.h = s->h.p, o.ldh = WA;
             return linear(o);
         }
         o.epi = ROWS_SCALE_F32, o.scale = 1.0f;
         linear(o);
-        if (hyper) streams(hyper, next);
-        else update(post, next, bias, route);
+        if (out.hyper) streams(out.hyper, next);
+        else update(out, next, route);
     }
     void linear(const RowsArgs &a, int batches = 1) {
         if (!rc) rc = rows_gemm_launch(s->cfg.dtype, a, batches, st), ++launches;
     }
 };
 
-// y = h . W^T in the stack's dtype
-void project(Pass &p, const void *w, int N, void *y) {
+// y = x . W^T in the stack's dtype (x nullptr: h)
+void project(Pass &p, const void *w, int N, void *y, const void *x = nullptr) {
     pie_stack *s = p.s;
     const int W = s->cfg.width, WA = act_stride(W);
-    if (p.plan.big) return p.gemm(w, s->h.p, WA, p.b.n_rows, N, W, y, N);
+    if (!x) x = s->h.p;
+    if (p.plan.big) return p.gemm(w, x, WA, p.b.n_rows, N, W, y, N);
     RowsArgs a = {};
-    a.m = {(const char *)w, N, W, s->h.p, WA, y, N};
+    a.m = {(const char *)w, N, W, x, WA, y, N};
     a.M = p.b.n_rows, a.epi = ROWS_STORE;
     p.linear(a);
 }
@@ -693,7 +768,7 @@ void latent_attend(Pass &p, int li, const pie_stack_layer &L, const LatentQuerie
         for (int i = p.plan.short_runs; i < b.n_runs; ++i) tiles += (b.runs_host[4 * i + 1] + 127) / 128;
         if (!p.rc) p.rc = window_attn_launch(w, tiles, p.st), p.launches += 2;
     }
-    p.output(L.w_o, s->o.p, LO, KO, L.post1, next, L.hyper1, nullptr, route);
+    p.output(L.w_o, s->o.p, LO, KO, out_of(L, L.post1, L.hyper1, nullptr), next, route);
 }
 
 // queries straight from the layer's input
@@ -757,24 +832,25 @@ void latent_query_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &n
     latent_attend(p, li, L, {s->qu.p, q_rot, NQ, finish}, riders, next, route);
 }
 
-void attention_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next, int route) {
+// the attention of a layer whose projections are in s->q; its heads' outputs go to the front of s->o
+void attend(Pass &p, int li, const pie_stack_layer &L, int LO) {
     pie_stack *s = p.s;
     const pie_stack_batch &b = p.b;
-    const int NI = in_columns(L), KO = out_columns(L), LO = act_stride(KO), dt = s->cfg.dtype;
+    const int NI = in_columns(L), dt = s->cfg.dtype;
     const bool own = L.kv_from < 0;
     const KvGeometry geo = geometry(L);
     void *slab = b.slabs[own ? li : L.kv_from];
     const PageTable pages = {b.table, b.table_width, (int)b.n_pages, b.n_seqs};
-    project(p, L.w_in, NI, s->q.p);
     if (p.rc) return;
     KvPrepArgs k = {};
-    k.raw = s->q.p, k.ld = NI, k.M = b.n_rows, k.bias = (const u16 *)L.in_bias, k.geo = geo, k.own = own, k.value_norm = L.value_norm != 0;
+    k.raw = s->q.p, k.ld = NI, k.M = b.n_rows, k.bias = (const u16 *)L.in_bias, k.geo = geo, k.own = own, k.value_norm = L.value_norm != 0, k.row_norm = L.row_norm != 0;
     k.q_norm = L.q_norm, k.k_norm = L.k_norm, k.eps = L.eps, k.freq = L.rot_freq, k.rot_dims = L.rot_dims, k.rot_gain = L.rot_gain;
     k.pos = b.pos, k.row_seq = b.row_seq, k.pages = pages, k.slab = slab;
     p.rc = kv_prep_launch(dt, k, p.st), ++p.launches;
     PageAttnArgs a = {};
     a.q = s->q.p, a.ldq = NI, a.slab = slab, a.pages = pages, a.geo = geo, a.pos = b.pos, a.row_seq = b.row_seq, a.runs = (const RowRun *)b.runs;
-    a.window = L.window, a.scale = L.scale, a.sink = L.sink, a.out = s->o.p, a.ld_out = LO, a.ws = s->attn_ws.p;
+    a.window = L.window, a.chunk = L.chunk, a.distance = L.distance, a.far = L.far, a.head_sink = L.head_sink, a.out_scale = L.out_scale;
+    a.scale = L.scale, a.sink = L.sink, a.out = s->o.p, a.ld_out = LO, a.ws = s->attn_ws.p;
     if (L.out_gate) {
         const int at = NI - up8(L.heads);
         a.gate = (const char *)s->q.p + at * esize(s), a.ldg = NI, a.gate_bias = L.in_bias ? (const u16 *)L.in_bias + at : nullptr;
@@ -787,7 +863,105 @@ void attention_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next
         for (int i = sp.runs; i < b.n_runs; ++i) a.n_tiles += page_attn_long_tiles(b.runs_host[4 * i + 1], geo);
         p.rc = page_attn_long_launch(a, p.st), ++p.launches;
     }
-    p.output(L.w_o, s->o.p, LO, KO, L.post1, next, L.hyper1, (const u16 *)L.o_bias, route);
+}
+
+void attention_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next, int route) {
+    const int KO = out_columns(L), LO = act_stride(KO);
+    project(p, L.w_in, in_columns(L), p.s->q.p);
+    attend(p, li, L, LO);
+    p.output(L.w_o, p.s->o.p, LO, KO, out_of(L, L.post1, L.hyper1, L.o_bias), next, route);
+}
+
+// time mixing, alone or beside an attention over the same rows; the mixes of the rows with their predecessors are in s->mixes
+void time_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next, int route) {
+    pie_stack *s = p.s;
+    const pie_stack_batch &b = p.b;
+    const pie_stack_time_mix &t = L.time_mix;
+    const bool beside = L.mixer == PIE_MIXER_ATTENTION;
+    const int W = s->cfg.width, WA = act_stride(W), M = b.n_rows, N = time_mix_columns(L), R8 = up8(t.rank), KO = out_columns(L), LO = act_stride(KO), dt = s->cfg.dtype;
+    const size_t E = esize(s), part = (size_t)M * N * E, mix = (size_t)M * WA * E;
+    char *at[TIME_MIXES];  // r, k, v, gate, low-rank input of the decay
+    for (int i = 0; i < TIME_MIXES; ++i) at[i] = s->mixed.p + i * part;
+    const void *w[TIME_MIXES] = {t.w_r, t.w_k, t.w_v, t.w_gate, t.w_low};
+    if (p.plan.big) {
+        if (beside) project(p, L.w_in, in_columns(L), s->q.p);
+        for (int i = 0; i < TIME_MIXES; ++i) project(p, w[i], i < 4 ? N : R8, at[i], s->mixes.p + i * mix);
+    } else {
+        RowsArgs a = {};
+        a.M = M, a.epi = ROWS_STORE;
+        if (beside) a.mats[a.n_mats++] = {(const char *)L.w_in, in_columns(L), W, s->h.p, WA, s->q.p, in_columns(L)};
+        for (int i = 0; i < TIME_MIXES; ++i) a.mats[a.n_mats++] = {(const char *)w[i], i < 4 ? N : R8, W, s->mixes.p + i * mix, WA, at[i], i < 4 ? N : R8};
+        p.linear(a, a.n_mats);
+    }
+    if (beside) attend(p, li, L, LO);
+    if (p.rc) return;
+    TimeMixArgs m = {};
+    m.r = at[0], m.k = at[1], m.v = at[2], m.gate = at[3], m.low = at[4], m.ld = N, m.ld_low = R8, m.M = M, m.H = t.heads, m.D = t.dim, m.D8 = up8(t.dim), m.rank = t.rank, m.R8 = R8;
+    m.w_decay = (const u16 *)t.w_decay, m.decay_bias = t.decay_bias, m.bonus = t.bonus, m.o_norm = t.o_norm, m.eps = L.eps, m.out_scale = t.out_scale;
+    m.pos = b.pos, m.row_seq = b.row_seq, m.slots = b.slots, m.n_seqs = b.n_seqs, m.n_slots = (int)b.n_slots, m.runs = (const RowRun *)b.runs;
+    m.state = b.states[li], m.slot_floats = state_layout(s, li).total, m.ws = s->rec_ws.p, m.o = s->rec_o.p, m.out = s->o.p + (size_t)(KO - N) * E, m.ld_out = LO;
+    const ChunkPart cp = chunk_part(s, b, L);
+    m.n_runs = cp.runs;
+    if (cp.runs) p.rc = time_mix_step_launch(dt, m, p.st), ++p.launches;
+    if (!p.rc && cp.chunks) {
+        m.runs += cp.runs, m.n_runs = b.n_runs - cp.runs;
+        p.rc = time_mix_chunks_launch(dt, m, cp.chunks, cp.rows, M - cp.rows, p.st), p.launches += time_mix_chunk_launches(cp.chunks, t.heads, t.dim);
+    }
+    p.output(L.w_o, s->o.p, LO, KO, out_of(L, L.post1, L.hyper1, L.o_bias), next, route);
+}
+
+void gated_delta_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next, int route) {
+    pie_stack *s = p.s;
+    const pie_stack_batch &b = p.b;
+    const int NI = in_columns(L), KO = out_columns(L), LO = act_stride(KO), dt = s->cfg.dtype;
+    project(p, L.w_in, NI, s->q.p);
+    if (p.rc) return;
+    const StateLayout at = state_layout(s, li);
+    GatedDeltaArgs d = {};
+    d.raw = s->q.p, d.ld = NI, d.M = b.n_rows, d.H = L.heads, d.G = L.kv_heads, d.D = L.dim, d.D8 = up8(L.dim), d.V = L.vdim, d.V8 = up8(L.vdim), d.H8 = up8(L.heads);
+    d.conv = L.mix_conv, d.taps = L.mix_taps, d.ldw = gated_channels(L), d.decay_rate = L.decay_rate, d.decay_bias = L.decay_bias, d.o_norm = L.o_norm;
+    d.scale = L.scale, d.unit_eps = L.unit_eps, d.eps = L.eps, d.pos = b.pos, d.row_seq = b.row_seq, d.slots = b.slots, d.n_seqs = b.n_seqs, d.n_slots = (int)b.n_slots;
+    d.runs = (const RowRun *)b.runs, d.n_runs = b.n_runs, d.state = b.states[li], d.slot_floats = at.total, d.ring = at.ring, d.ws = s->rec_ws.p, d.o = s->rec_o.p, d.out = s->o.p, d.ld_out = LO;
+    if (b.n_runs < b.n_rows) {
+        d.mixed = s->mixed.p;
+        int tiles = 0;
+        for (int i = 0; i < b.n_runs; ++i) tiles += conv_tiles(b.runs_host[4 * i + 1]);
+        p.rc = gated_delta_conv_launch(dt, d, tiles, p.st), ++p.launches;
+    }
+    const ChunkPart cp = chunk_part(s, b, L);
+    d.n_runs = cp.runs;
+    if (!p.rc && cp.runs) p.rc = gated_delta_step_launch(dt, d, 0, cp.rows, p.st), p.launches += L.vdim > 256 ? 2 : 1;
+    if (!p.rc && cp.chunks) {
+        d.runs += cp.runs, d.n_runs = b.n_runs - cp.runs;
+        p.rc = gated_delta_chunks_launch(dt, d, cp.chunks, cp.rows, b.n_rows - cp.rows, p.st), p.launches += gated_delta_chunk_launches(cp.chunks, L.heads, L.dim);
+    }
+    p.output(L.w_o, s->o.p, LO, KO, out_of(L, L.post1, L.hyper1, nullptr), next, route);
+}
+
+// x += side_norm(w_side_proj (gelu(w_side_gate x) * the token's vector for this layer)); h (= x on the way in) = next(x)
+void side_input(Pass &p, int li, const pie_stack_layer &L, const Into &next) {
+    pie_stack *s = p.s;
+    const int M = p.b.n_rows, W = s->cfg.width, WA = act_stride(W), D = s->cfg.side_dim, DA = act_stride(D);
+    const TokenVectors side = {(const u16 *)s->cfg.side_embed, (size_t)s->cfg.n_layers * D, (size_t)li * D, p.b.ids, s->cfg.vocab};
+    int ld = DA;
+    if (p.plan.big) {
+        const int D8 = up8(D);
+        ld = up64(D);
+        if (D8 == ld) p.gemm(L.w_side_gate, s->h.p, WA, M, D8, W, s->side.p, ld);
+        else if (!p.rc) {  // (rows longer than the product: its plan must not split K)
+            p.rc = w16l_act_launch(L.w_side_gate, s->h.p, WA, M, D, W, s->side.p, ld, MFMA_ACT_NONE, 0.0f, 0.0f, nullptr, p.st), ++p.launches;
+        }
+        if (p.rc) return;
+        hipLaunchKernelGGL(k_side_gate, dim3((unsigned)(((size_t)M * D + 255) / 256)), dim3(256), 0, p.st, (u16 *)s->side.p, ld, side, M, D);
+        if (hipGetLastError() != hipSuccess) p.rc = pie::fail(PIE_E_HIP, "side input launch failed");
+        ++p.launches;
+    } else {
+        RowsArgs a = {};
+        a.m = {(const char *)L.w_side_gate, D, W, s->h.p, WA, s->side.p, ld};
+        a.M = M, a.epi = ROWS_GELU_SIDE, a.side = side;
+        p.linear(a);
+    }
+    p.output(L.w_side_proj, s->side.p, ld, D, {L.side_norm, nullptr, nullptr, false, 1.0f}, next);
 }
 
 void delta_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next, int route) {
@@ -808,7 +982,7 @@ void delta_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next, in
         d.runs += dp.runs, d.n_runs = b.n_runs - dp.runs;
         p.rc = delta_chunks_launch(s->cfg.dtype, d, dp.chunks, dp.rows, b.n_rows - dp.rows, p.st), p.launches += delta_launches(dp.chunks, L.heads, L.dim);
     }
-    p.output(L.w_o, s->o.p, LO, KO, L.post1, next, L.hyper1, nullptr, route);
+    p.output(L.w_o, s->o.p, LO, KO, out_of(L, L.post1, L.hyper1, nullptr), next, route);
 }
 
 RecurrentArgs recurrent_args(const Pass &p, int li, int ld) {
@@ -830,9 +1004,9 @@ void mlstm_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next, in
         m.r.runs += cp.runs, m.r.n_runs = b.n_runs - cp.runs;
         p.rc = mlstm_chunks_launch(m, cp.chunks, p.st), p.launches += 4;
     }
-    const HeadOutArgs h = {s->rec_o.p, s->rec_den.p, (const char *)s->q.p + (size_t)H * (2 * D8 + V8) * esize(s), nullptr, NI, H, L.vdim, V8, L.o_norm, L.eps, s->o.p, LO};
+    const HeadOutArgs h = {s->rec_o.p, s->rec_den.p, (const char *)s->q.p + (size_t)H * (2 * D8 + V8) * esize(s), nullptr, NI, H, L.vdim, V8, L.o_norm, L.eps, s->o.p, LO, false, false, 1.0f};
     if (!p.rc) p.rc = head_out_launch(dt, h, 0, b.n_rows, p.st), ++p.launches;
-    p.output(L.w_o, s->o.p, LO, KO, L.post1, next, L.hyper1, nullptr, route);
+    p.output(L.w_o, s->o.p, LO, KO, out_of(L, L.post1, L.hyper1, nullptr), next, route);
 }
 
 void mingru_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next, int route) {
@@ -849,7 +1023,7 @@ void mingru_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next, i
         m.r.runs += cp.runs, m.r.n_runs = b.n_runs - cp.runs;
         p.rc = mingru_chunks_launch(dt, m, cp.chunks, p.st), p.launches += 3;
     }
-    p.output(L.w_o, s->o.p, LO, KO, L.post1, next, L.hyper1, nullptr, route);
+    p.output(L.w_o, s->o.p, LO, KO, out_of(L, L.post1, L.hyper1, nullptr), next, route);
 }
 
 void feed_forward(Pass &p, int li, const pie_stack_layer &L, const Into &into, bool routed) {  // routed: the experts have been chosen already
@@ -857,16 +1031,17 @@ void feed_forward(Pass &p, int li, const pie_stack_layer &L, const Into &into, b
     const int M = p.b.n_rows, W = s->cfg.width, W64 = up64(W), WA = act_stride(W), F = L.ff_size, FA = act_stride(F), dt = s->cfg.dtype;
     const pie_stack_norm &next = *into.norm;
     if (is_dense(L)) {
-        const bool relu = L.ff == PIE_FF_RELU2;
+        const bool relu = L.ff == PIE_FF_RELU2, gated = L.ff == PIE_FF_GEGLU;
         if (p.plan.big) {
-            if (!p.rc) p.rc = w16l_act_launch(L.w_up, s->h.p, WA, M, F, W, s->act.p, FA, relu ? MFMA_ACT_RELU2 : MFMA_ACT_XIELU, L.act_alpha, L.act_beta, p.st), ++p.launches;
+            const int act = gated ? MFMA_ACT_GELU : relu ? MFMA_ACT_RELU2 : MFMA_ACT_XIELU;
+            if (!p.rc) p.rc = w16l_act_launch(L.w_up, s->h.p, WA, M, gated ? 2 * F : F, W, s->act.p, FA, act, L.act_alpha, L.act_beta, gated ? L.up_bias : nullptr, p.st), ++p.launches;
         } else {
             RowsArgs u = {};
-            u.m = {(const char *)L.w_up, F, W, s->h.p, WA, s->act.p, FA};
-            u.M = M, u.epi = relu ? ROWS_RELU2 : ROWS_XIELU, u.act_alpha = L.act_alpha, u.act_limit = L.act_beta;
+            u.m = {(const char *)L.w_up, gated ? 2 * F : F, W, s->h.p, WA, s->act.p, FA};
+            u.M = M, u.epi = gated ? ROWS_GELU_MUL : relu ? ROWS_RELU2 : ROWS_XIELU, u.bias = gated ? (const u16 *)L.up_bias : nullptr, u.act_alpha = L.act_alpha, u.act_limit = L.act_beta;
             p.linear(u);
         }
-        return p.output(L.w_down, s->act.p, FA, F, L.post2, into, L.hyper2);
+        return p.output(L.w_down, s->act.p, FA, F, out_of(L, L.post2, L.hyper2, L.down_bias), into);
     }
     const RouteLayer &r = s->route[li];
     const int S = L.shared_size, SA = act_stride(S);
@@ -942,17 +1117,19 @@ int stack_enqueue(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
     // what sublayer 1 of layer i (n: the final norm) takes in, and sublayer 2
     const int S = s->cfg.streams;
     auto mixer_in = [&](int i) -> Into {
-        if (i >= n) return {&s->cfg.final_norm, nullptr, -1};
-        return {&s->layers[i].pre1, s->layers[i].hyper1, s->layers[i].conv_taps > 0 ? i : -1};
+        if (i >= n) return {&s->cfg.final_norm, nullptr, -1, -1};
+        return {&s->layers[i].pre1, s->layers[i].hyper1, s->layers[i].conv_taps > 0 ? i : -1, has_time_mix(s->layers[i]) ? i : -1};
     };
+    const pie_stack_norm plain = {nullptr, nullptr, 0.0f, PIE_NORM_NONE};
+    const u16 *positions = (const u16 *)s->cfg.positions;
     const pie_stack_norm &first = *mixer_in(0).norm;
     const dim3 ge((unsigned)((W + 1023) / 1024), (unsigned)M);
     if (S) p.streams(nullptr, mixer_in(0));
     else if (dt == PIE_F32)
-        hipLaunchKernelGGL(k_stack_embed<ElemF32>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, s->cfg.embed_scale, !pointwise(first), norm_of(first), s->x.p, W64,
+        hipLaunchKernelGGL(k_stack_embed<ElemF32>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, s->cfg.embed_scale, positions, s->cfg.max_positions, b.pos, !pointwise(first), norm_of(first), s->x.p, W64,
                            (float *)s->h.p, WA);
     else
-        hipLaunchKernelGGL(k_stack_embed<ElemBF16>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, s->cfg.embed_scale, !pointwise(first), norm_of(first), s->x.p, W64,
+        hipLaunchKernelGGL(k_stack_embed<ElemBF16>, ge, dim3(256), 0, st, b.ids, (const u16 *)s->cfg.embed, V, W, s->cfg.embed_scale, positions, s->cfg.max_positions, b.pos, !pointwise(first), norm_of(first), s->x.p, W64,
                            (u16 *)s->h.p, WA);
     PIE_LAUNCH_CHECK();
     p.launches += !S;
@@ -961,20 +1138,25 @@ int stack_enqueue(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
         a.next = row_norm_of(first), a.x = s->x.p, a.ldx = W64, a.h = s->h.p, a.ldh = WA, a.M = M, a.W = W;
         p.rc = row_update_launch(dt, a, st), ++p.launches;
     }
+    if (n && has_time_mix(s->layers[0])) p.token_mix(0);
     for (int i = 0; i < n && !p.rc; ++i) {
         const pie_stack_layer &L = s->layers[i];
-        const Into after = mixer_in(i + 1), next = L.ff == PIE_FF_NONE ? after : Into{&L.pre2, L.hyper2, -1};
+        const bool side = L.w_side_gate != nullptr;
+        const Into last = mixer_in(i + 1), after = side ? Into{&plain, nullptr, -1, -1} : last, next = L.ff == PIE_FF_NONE ? after : Into{&L.pre2, L.hyper2, -1, -1};
         // some rows: the launch that makes the router's input also chooses the experts (for very few rows, spreading the router over the chip takes less time)
         const bool routed = L.ff == PIE_FF_ROUTED_MOE && !plan.big && L.w_router_rows && M >= ROUTE_MIN_ROWS && M <= ROUTE_FEW_ROWS && (long)L.experts * W <= ROUTE_FEW_WEIGHTS && W <= 8192;
         const int route = routed ? i : -1;
         switch (L.mixer) {
             case PIE_MIXER_LATENT: L.q_rank ? latent_query_mixer(p, i, L, next, route) : latent_mixer(p, i, L, next, route); break;
-            case PIE_MIXER_ATTENTION: attention_mixer(p, i, L, next, route); break;
+            case PIE_MIXER_ATTENTION: has_time_mix(L) ? time_mixer(p, i, L, next, route) : attention_mixer(p, i, L, next, route); break;
+            case PIE_MIXER_TIME_MIX: time_mixer(p, i, L, next, route); break;
+            case PIE_MIXER_GATED_DELTA: gated_delta_mixer(p, i, L, next, route); break;
             case PIE_MIXER_DELTA: delta_mixer(p, i, L, next, route); break;
             case PIE_MIXER_MLSTM: mlstm_mixer(p, i, L, next, route); break;
             default: mingru_mixer(p, i, L, next, route); break;
         }
         if (L.ff != PIE_FF_NONE && !p.rc) feed_forward(p, i, L, after, routed);
+        if (side && !p.rc) side_input(p, i, L, last);
         if (b.tap && !p.rc && S) p.rc = stream_sum_launch(s->x.p, W64, S, b.tap + (size_t)i * M * W, M, W, st);
         else if (b.tap && !p.rc)
             PIE_HIP_TRY(hipMemcpy2DAsync(b.tap + (size_t)i * M * W, (size_t)W * 4, s->x.p, (size_t)W64 * 4, (size_t)W * 4, (size_t)M, hipMemcpyDeviceToDevice, st));
@@ -982,7 +1164,7 @@ int stack_enqueue(pie_stack *s, const pie_stack_batch &b, const Plan &plan, hipS
     if (b.n_want > 0) {
         RowsArgs a = {};
         a.m = {(const char *)s->cfg.head, V, W, s->h.p, WA, b.logits, V};
-        a.M = b.n_want, a.epi = ROWS_SCALE_F32, a.scale = s->cfg.logit_scale, a.rows = b.want;
+        a.M = b.n_want, a.epi = s->cfg.logit_cap > 0.0f ? ROWS_SOFTCAP : ROWS_SCALE_F32, a.scale = s->cfg.logit_scale, a.act_limit = s->cfg.logit_cap, a.rows = b.want;
         p.linear(a);
         if (!p.rc && b.next) {
             hipLaunchKernelGGL(k_f32_stats, dim3(ST_TILES, (unsigned)b.n_want), dim3(256), 0, st, b.logits, V, s->stats.p);
@@ -1001,7 +1183,16 @@ bool norm_ok(const pie_stack_norm &n) {
     return n.kind == PIE_NORM_NONE || (n.kind == PIE_NORM_DYN_TANH && n.w && n.b) || (n.kind == PIE_NORM_RMS && n.w);
 }
 int mixer_ok(const pie_stack *s, int i, const pie_stack_layer &L) {
-    PIE_REQUIRE(L.heads > 0 && L.dim > 0 && L.w_in && L.w_o && norm_ok(L.pre1) && norm_ok(L.post1), PIE_E_ARG, "pie_stack_set_layer: missing mixer weights or sizes");
+    PIE_REQUIRE((L.mixer == PIE_MIXER_TIME_MIX || (L.heads > 0 && L.dim > 0 && L.w_in)) && L.w_o && norm_ok(L.pre1) && norm_ok(L.post1), PIE_E_ARG, "pie_stack_set_layer: missing mixer weights or sizes");
+    if (has_time_mix(L)) {
+        const pie_stack_time_mix &t = L.time_mix;
+        PIE_REQUIRE(L.mixer == PIE_MIXER_ATTENTION || L.mixer == PIE_MIXER_TIME_MIX, PIE_E_ARG, "pie_stack_set_layer: time mixing runs alone or beside an attention");
+        PIE_REQUIRE(t.dim > 0 && t.dim <= TIME_MIX_MAX_DIM && t.rank > 0 && t.rank <= TIME_MIX_MAX_RANK, PIE_E_SHAPE, "pie_stack_set_layer: bad sizes (time mixing: dim at most 256, rank at most 1024)");
+        PIE_REQUIRE(t.w_r && t.w_k && t.w_v && t.w_gate && t.w_low && t.w_decay && t.mu && t.decay_bias && t.bonus && t.o_norm, PIE_E_ARG, "pie_stack_set_layer: missing time mixing weights");
+        PIE_REQUIRE(!s->cfg.streams && L.pre1.kind == PIE_NORM_NONE, PIE_E_ARG, "pie_stack_set_layer: time mixing reads the residual itself");
+    }
+    if (L.norm_after) PIE_REQUIRE(!s->cfg.streams && L.pre1.kind == PIE_NORM_NONE && L.pre2.kind == PIE_NORM_NONE && !is_moe(L), PIE_E_ARG, "pie_stack_set_layer: norms behind the sum go with plain sublayer inputs and dense feed-forwards");
+    if (L.w_side_gate) PIE_REQUIRE(s->cfg.side_embed && s->cfg.side_dim > 0 && !s->cfg.streams && L.w_side_proj && norm_ok(L.side_norm), PIE_E_ARG, "pie_stack_set_layer: a side input needs its table, projection and norm");
     if (L.mixer == PIE_MIXER_LATENT) {
         PIE_REQUIRE(L.vdim > 0 && L.rank > 0 && L.q_rank >= 0 && L.rot_dim >= 0 && latent_row(L) <= 2048, PIE_E_SHAPE, "pie_stack_set_layer: bad mixer sizes (kv_rank + rot_dim at most 2048)");
         PIE_REQUIRE(L.w_uk && L.w_uv && (L.c_norm || !own_cache(L)), PIE_E_ARG, "pie_stack_set_layer: missing mixer weights");
@@ -1014,7 +1205,17 @@ int mixer_ok(const pie_stack *s, int i, const pie_stack_layer &L) {
             PIE_REQUIRE(F.mixer == PIE_MIXER_LATENT && own_cache(F) && F.rank == L.rank && F.rot_dim == L.rot_dim, PIE_E_SHAPE,
                         "pie_stack_set_layer: kv_from names a latent layer with a cache of its own, of the same sizes");
         }
+    } else if (L.mixer == PIE_MIXER_TIME_MIX) {
+        PIE_REQUIRE(has_time_mix(L), PIE_E_SHAPE, "pie_stack_set_layer: time mixing without heads");
+    } else if (L.mixer == PIE_MIXER_GATED_DELTA) {
+        PIE_REQUIRE(L.kv_heads > 0 && L.heads % L.kv_heads == 0 && L.dim <= GATED_MAX_DIM && L.vdim > 0 && L.vdim <= HEAD_OUT_MAX_DIM, PIE_E_SHAPE,
+                    "pie_stack_set_layer: bad mixer sizes (gated delta rule: dim at most 256, vdim at most 2048, heads a multiple of kv_heads)");
+        PIE_REQUIRE(L.mix_taps > 0 && L.mix_taps <= CONV_MAX_TAPS && L.mix_conv, PIE_E_SHAPE, "pie_stack_set_layer: a convolution of 1 .. 16 taps, with its weights");
+        PIE_REQUIRE(L.decay_rate && L.decay_bias && L.o_norm, PIE_E_ARG, "pie_stack_set_layer: missing mixer weights");
     } else if (L.mixer == PIE_MIXER_ATTENTION) {
+        PIE_REQUIRE(L.chunk >= 0 && (!L.chunk || L.window <= 0) && (!L.distance || L.far >= 0) && (!L.head_sink || L.sink == 0.0f), PIE_E_ARG, "pie_stack_set_layer: a window or chunks, and one kind of sink");
+        PIE_REQUIRE(!L.row_norm || (L.dim == L.vdim && !L.rot_dims && !L.value_norm && L.q_norm && L.k_norm && L.kv_from < 0), PIE_E_SHAPE,
+                    "pie_stack_set_layer: norms over all heads go with values that are the layer's own keys, without rotation");
         PIE_REQUIRE(L.vdim > 0 && L.kv_heads > 0 && L.heads % L.kv_heads == 0 && L.dim <= PAGE_ATTN_ROWS_DIM && L.vdim <= PAGE_ATTN_ROWS_DIM, PIE_E_SHAPE,
                     "pie_stack_set_layer: bad mixer sizes (heads of at most 1024 numbers, a multiple of kv_heads)");
         PIE_REQUIRE(L.rot_dims >= 0 && L.rot_dims <= L.dim && L.rot_dims % 2 == 0 && (L.rot_dims == 0 || L.rot_freq), PIE_E_SHAPE, "pie_stack_set_layer: bad rotation");
@@ -1052,8 +1253,9 @@ int pie_stack_create(const pie_stack_config *cfg, pie_stack **out) {
     PIE_REQUIRE(cfg->width > 0 && cfg->vocab > 0 && cfg->n_layers >= 0, PIE_E_SHAPE, "pie_stack_create: bad sizes");
     PIE_REQUIRE(cfg->embed && cfg->head && norm_ok(cfg->final_norm), PIE_E_ARG, "pie_stack_create: missing weights");
     PIE_REQUIRE(cfg->streams >= 0 && cfg->streams <= STREAMS_MAX && (cfg->streams == 0 || cfg->width <= ROW_UPDATE_MAX_WIDTH), PIE_E_SHAPE, "pie_stack_create: at most 16 streams, of at most 32768 numbers");
-    PIE_REQUIRE((!cfg->positions && !cfg->bigram) || (cfg->streams > 0 && (!cfg->positions || cfg->max_positions > 0) && (!cfg->bigram || (cfg->buckets > 0 && cfg->n_layers > 0))), PIE_E_ARG,
-                "pie_stack_create: position and bigram vectors go with streams, and need their sizes");
+    PIE_REQUIRE((!cfg->positions || cfg->max_positions > 0) && (!cfg->bigram || (cfg->streams > 0 && cfg->buckets > 0 && cfg->n_layers > 0)), PIE_E_ARG,
+                "pie_stack_create: position and bigram vectors need their sizes, and bigrams go with streams");
+    PIE_REQUIRE(cfg->logit_cap >= 0.0f && (!cfg->side_embed || cfg->side_dim > 0), PIE_E_ARG, "pie_stack_create: bad logit cap or side vectors");
     pie_stack *s = new (std::nothrow) pie_stack();
     PIE_REQUIRE(s, PIE_E_HIP, "pie_stack_create: out of host memory");
     s->cfg = *cfg;

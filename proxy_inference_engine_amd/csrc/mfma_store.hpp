@@ -34,7 +34,8 @@ __device__ __forceinline__ u32 w4m_pack<F16>(float lo, float hi) {
 // the accumulators it does not fit the registers), MFMA_ACT_CLIPPED (columns paired as for SWIGLU: g sigmoid(alpha g) (u + 1) with g = min(gate, limit),
 // u = clamp(up, +-limit) of the rounded pair).
 // MFMA_ACT_XIELU: of the rounded value, like RELU2 on the way out of LDS (act_alpha, act_limit: its two factors).
-enum { MFMA_ACT_NONE = 0, MFMA_ACT_SWIGLU = 1, MFMA_ACT_RELU2 = 2, MFMA_ACT_CLIPPED = 3, MFMA_ACT_XIELU = 4 };
+// MFMA_ACT_GELU: columns paired as for SWIGLU: gelu_tanh(gate) up of the accumulators, with the bias, before any rounding.
+enum { MFMA_ACT_NONE = 0, MFMA_ACT_SWIGLU = 1, MFMA_ACT_RELU2 = 2, MFMA_ACT_CLIPPED = 3, MFMA_ACT_XIELU = 4, MFMA_ACT_GELU = 5 };
 template <class T>
 __device__ __forceinline__ u32 mfma_relu2(u32 w) {
     const float a = fmaxf(lo_f32<T>(w), 0.0f), b = fmaxf(hi_f32<T>(w), 0.0f);
@@ -47,7 +48,7 @@ __device__ __forceinline__ u32 mfma_xielu(u32 w, float up, float down) {
 template <class T, int MB, int SW, int ACT>
 __device__ __forceinline__ void mfma_tile_store(const f32x16_t (&acc)[SW][MB], char *ot, int lane, int nt0, int m0, int rows, int N, int ldy, u16 *y,
                                                 const u16 *bias, bool skip_stores = false, float act_alpha = 0.0f, float act_limit = 0.0f) {
-    constexpr bool SWIGLU = ACT == MFMA_ACT_SWIGLU || ACT == MFMA_ACT_CLIPPED;  // two columns make one
+    constexpr bool SWIGLU = ACT == MFMA_ACT_SWIGLU || ACT == MFMA_ACT_CLIPPED || ACT == MFMA_ACT_GELU;  // two columns make one
     constexpr int MT = 32 * MB;
     constexpr int OB = (SWIGLU ? 32 : 64) * SW;  // output bytes per row of the wave's tile
     constexpr int SL = OB / 8, RPB = 256 / OB;    // 8-byte slots per row; rows per 256-byte bank row
@@ -60,6 +61,16 @@ __device__ __forceinline__ void mfma_tile_store(const f32x16_t (&acc)[SW][MB], c
 #pragma unroll
             for (int q = 0; q < 4; ++q) {
                 const int col = 32 * (nt0 + s) + 4 * kh + 8 * q;
+                if constexpr (ACT == MFMA_ACT_GELU) {  // (N is a multiple of 8: whole quads)
+                    float b[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+                    if (bias && col < N) {
+                        const uint2 w = *reinterpret_cast<const uint2 *>(bias + col);
+                        b[0] = lo_f32<T>(w.x), b[1] = hi_f32<T>(w.x), b[2] = lo_f32<T>(w.y), b[3] = hi_f32<T>(w.y);
+                    }
+                    const float o0 = gelu_tanh<false>(acc[s][mi][4 * q] + b[0]) * (acc[s][mi][4 * q + 1] + b[1]), o1 = gelu_tanh<false>(acc[s][mi][4 * q + 2] + b[2]) * (acc[s][mi][4 * q + 3] + b[3]);
+                    *reinterpret_cast<u32 *>(ot + (32 * mi + n) * OB + (((4 * s + q) ^ sv) << 3) + 4 * kh) = w4m_pack<T>(o0, o1);
+                    continue;
+                }
                 u32 p01 = w4m_pack<T>(acc[s][mi][4 * q], acc[s][mi][4 * q + 1]), p23 = w4m_pack<T>(acc[s][mi][4 * q + 2], acc[s][mi][4 * q + 3]);  // the Linear's rounding
                 if (bias && col < N) {
                     uint2 bw;

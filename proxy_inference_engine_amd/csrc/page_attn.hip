@@ -1,5 +1,6 @@
 // page_attn.hip -- softmax attention with grouped heads over paged keys and values (PIE_MIXER_ATTENTION): query / key norm, rotation, value norm, the page
-// writes, and the attention itself with its denominator sink and per-head output gate.
+// writes, and the attention itself with its denominator sink and per-head output gate.  What a query sees ends at a window or at the start of its chunk of positions; a score may
+// have a learned number added that depends on the head and the key's distance.
 //
 // Keys and values lie in the pages in matrix-core operand order (KvGeometry), so an operand load is one contiguous KiB per wave, straight from memory to
 // the registers that are the operand, or linearly through LDS: no swizzle, no transpose.
@@ -103,7 +104,94 @@ __global__ void __launch_bounds__(256) k_kv_prep(const KvPrepArgs a) {
     }
 }
 
+// One workgroup per row: the norms run over all heads of the row at once, and values are the keys in front of their norm.
+template <class E>
+__global__ void __launch_bounds__(256) k_kv_prep_row(const KvPrepArgs a) {
+    typedef typename E::type T;
+    __shared__ float s_red[2][4];
+    const KvGeometry &geo = a.geo;
+    const int m = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, nq = geo.H * geo.D8, n = nq + (a.own ? geo.G * geo.D8 : 0);
+    T *x = (T *)a.raw + (size_t)m * a.ld;
+    struct Eight {
+        float v[8];
+    };
+    auto eight = [&](int i) {  // with the bias (heads are padded to a multiple of 8 with zeros)
+        Eight e;
+        if constexpr (sizeof(T) == 2) {
+            const uint4 w = *(const uint4 *)(x + i);
+            const u32 u[4] = {w.x, w.y, w.z, w.w};
+#pragma unroll
+            for (int k = 0; k < 4; ++k) e.v[2 * k] = lo_f32<BF16>(u[k]), e.v[2 * k + 1] = hi_f32<BF16>(u[k]);
+        } else {
+#pragma unroll
+            for (int k = 0; k < 8; ++k) e.v[k] = x[i + k];
+        }
+        if (a.bias) {
+            const uint4 w = *(const uint4 *)(a.bias + i);
+            const u32 u[4] = {w.x, w.y, w.z, w.w};
+#pragma unroll
+            for (int k = 0; k < 4; ++k) e.v[2 * k] += lo_f32<BF16>(u[k]), e.v[2 * k + 1] += hi_f32<BF16>(u[k]);
+        }
+        return e;
+    };
+    auto put = [&](T *p, const float (&v)[8]) {
+        if constexpr (sizeof(T) == 2) *(uint4 *)p = make_uint4(pack2<BF16>(v[0], v[1]), pack2<BF16>(v[2], v[3]), pack2<BF16>(v[4], v[5]), pack2<BF16>(v[6], v[7]));
+        else
+#pragma unroll
+            for (int k = 0; k < 8; ++k) p[k] = v[k];
+    };
+    constexpr int KEEP = 4;  // pieces of eight numbers per thread that stay in registers
+    Eight kept[KEEP];
+    float ss[2] = {0.0f, 0.0f};
+#pragma unroll
+    for (int j = 0; j < KEEP; ++j) {
+        const int i = 8 * (threadIdx.x + 256 * j);
+        if (i >= n) break;
+        kept[j] = eight(i);
+    }
+    auto add = [&](int i, const Eight &e) {
+        float s = 0.0f;
+#pragma unroll
+        for (int k = 0; k < 8; ++k) s = fmaf(e.v[k], e.v[k], s);
+        if (i < nq) ss[0] += s;
+        else ss[1] += s;
+    };
+    auto each = [&](auto &&f) {
+#pragma unroll
+        for (int j = 0; j < KEEP; ++j) {
+            const int i = 8 * (threadIdx.x + 256 * j);
+            if (i < n) f(i, kept[j]);
+        }
+        for (int i = 8 * (threadIdx.x + 256 * KEEP); i < n; i += 8 * 256) f(i, eight(i));
+    };
+    each(add);
+    ss[0] = lanes_sum(ss[0]), ss[1] = lanes_sum(ss[1]);
+    if (lane == 0) s_red[0][wave] = ss[0], s_red[1][wave] = ss[1];
+    const int t = a.pos[m], tl = t & (PAGE_TOKENS - 1);
+    T *page = (T *)a.slab + (size_t)page_of(a.pages, a.row_seq[m], t) * geo.page_elems();
+    __syncthreads();
+    float inv[2];
+#pragma unroll
+    for (int k = 0; k < 2; ++k) inv[k] = 1.0f / sqrtf(((s_red[k][0] + s_red[k][1]) + (s_red[k][2] + s_red[k][3])) / (float)((k ? geo.G : geo.H) * geo.dim) + a.eps);
+    each([&](int i, const Eight &e) {
+        const bool is_q = i < nq;
+        const float *w = is_q ? a.q_norm + i : a.k_norm + i - nq;
+        const float4 w0 = *(const float4 *)w, w1 = *(const float4 *)(w + 4);
+        const float f = inv[!is_q];
+        const float v[8] = {e.v[0] * f * w0.x, e.v[1] * f * w0.y, e.v[2] * f * w0.z, e.v[3] * f * w0.w, e.v[4] * f * w1.x, e.v[5] * f * w1.y, e.v[6] * f * w1.z, e.v[7] * f * w1.w};
+        if (is_q) return put(x + i, v);
+        const int g = (i - nq) / geo.D8, d = (i - nq) % geo.D8;
+        T *head = page + g * geo.head_elems();
+        put(head + geo.key(tl, d), v);
+#pragma unroll
+        for (int k = 0; k < 8; ++k)
+            if (d + k < geo.vdim) head[geo.value(tl, d + k)] = E::pack(e.v[k]);
+    });
+}
+
 // ---------------------------------------------------------------- common pieces
+// the first position that a query at t sees
+__device__ __forceinline__ int pg_first_key(const PageAttnArgs &a, int t) { return a.chunk > 0 ? t - t % a.chunk : a.window > 0 ? max(0, t - a.window + 1) : 0; }
 struct PgTile {
     RowRun run;
     int g, gs, p0, live;  // key/value head, heads per group, first pair, live pairs
@@ -138,22 +226,63 @@ __device__ __forceinline__ float pg_gate(const PageAttnArgs &a, bool is32, int r
     return 1.0f / (1.0f + expf(-z));
 }
 
+// What a head's sums are multiplied by at the end, when its weights are relative to the exponent m (base 2) and sum to l
+__device__ __forceinline__ float pg_factor(const PageAttnArgs &a, bool is32, int row, int head, float m, float l) {
+    const float gate = pg_gate(a, is32, row, head) * a.out_scale;
+    if (a.head_sink) {
+        const float s = a.head_sink[head] * PG_LOG2E, mm = fmaxf(m, s), f = __builtin_amdgcn_exp2f(m - mm);
+        return gate * f / (l * f + __builtin_amdgcn_exp2f(s - mm));
+    }
+    return gate / (l + (a.sink > 0.0f ? a.sink * __builtin_amdgcn_exp2f(-m) : 0.0f));
+}
+
+// The numbers added to the scores by distance (PageAttnArgs::distance): the heads of one group, in LDS where they fit
+constexpr int PG_TABLE = 3072;
+enum { PG_PLAIN = 0, PG_NEAR_LDS = 1, PG_NEAR_GLOBAL = 2 };
+struct PgDistance {
+    const float *near;  // the pair's head: [far + 1]
+    int far;
+    float last;         // near[far], times log2 e
+};
+template <int DIST>
+__device__ __forceinline__ PgDistance pg_distance(const PageAttnArgs &a, const PgTile &tile, int head, float *lds) {
+    if constexpr (DIST == PG_PLAIN) return {nullptr, 0, 0.0f};
+    const int n = a.far + 1;
+    const float *rows = a.distance + (size_t)tile.g * tile.gs * n;
+    if constexpr (DIST == PG_NEAR_LDS) {
+        for (int i = threadIdx.x; i < tile.gs * n; i += 256) lds[i] = rows[i];
+        __syncthreads();
+        rows = lds;
+    }
+    const float *near = rows + (size_t)(head - tile.g * tile.gs) * n;
+    return {near, a.far, near[a.far] * PG_LOG2E};
+}
+
 // one 32-key block's scores -> weights: masks, moves the running maximum, splits the weights into bf16 halves
-template <int DT>
-__device__ __forceinline__ void pg_softmax(const f32x16_t &s, bool masked, int t0, int h, int t_q, int t_min, float sl2, float &m_run, float &l_run, f32x16_t (&o)[DT], u32 (&hi)[8],
-                                           u32 (&lo)[8]) {
+// near (DIST): keys of the block are nearer than the last row of the distance table
+template <int DT, int DIST>
+__device__ __forceinline__ void pg_softmax(const f32x16_t &s, bool masked, bool near, const PgDistance &dist, int t0, int h, int t_q, int t_min, float sl2, float &m_run, float &l_run,
+                                           f32x16_t (&o)[DT], u32 (&hi)[8], u32 (&lo)[8]) {
     float sc[16], mloc = PG_NEG;
+    if constexpr (DIST == PG_PLAIN) {
+#pragma unroll
+        for (int i = 0; i < 16; ++i) sc[i] = s[i] * sl2;
+    } else if (near) {
+#pragma unroll
+        for (int i = 0; i < 16; ++i) sc[i] = fmaf(s[i], sl2, dist.near[min(max(t_q - (t0 + (i & 3) + 8 * (i >> 2) + 4 * h), 0), dist.far)] * PG_LOG2E);
+    } else {
+#pragma unroll
+        for (int i = 0; i < 16; ++i) sc[i] = fmaf(s[i], sl2, dist.last);
+    }
     if (masked) {
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
             const int t = t0 + (i & 3) + 8 * (i >> 2) + 4 * h;
-            sc[i] = t <= t_q && t >= t_min ? s[i] * sl2 : PG_NEG;
-            mloc = fmaxf(mloc, sc[i]);
+            sc[i] = t <= t_q && t >= t_min ? sc[i] : PG_NEG;
         }
-    } else {
-#pragma unroll
-        for (int i = 0; i < 16; ++i) sc[i] = s[i] * sl2, mloc = fmaxf(mloc, sc[i]);
     }
+#pragma unroll
+    for (int i = 0; i < 16; ++i) mloc = fmaxf(mloc, sc[i]);
     mloc = xor32_max(mloc);
     // the running maximum moves only when a score exceeds it by 2^8: weights of up to 256 are as exact as weights of up to 1, and rescaling is rare
     if (__builtin_amdgcn_ballot_w64(mloc > m_run + 8.0f)) {
@@ -177,7 +306,7 @@ __device__ __forceinline__ void pg_softmax(const f32x16_t &s, bool masked, int t
 
 // ---------------------------------------------------------------- short form
 // KS, DT: upper bounds of D16 / 16 and V32 / 32
-template <int KS, int DT>
+template <int KS, int DT, int DIST>
 __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_page_attn(const PageAttnArgs a) {
     __shared__ __attribute__((aligned(16))) float s_o[4][DT * 4][64][4];
     __shared__ float s_m[4][32], s_l[4][32];
@@ -185,12 +314,13 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_page_attn(const PageAt
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), c = lane & 31, h = lane >> 5;
     const PgTile tile = pg_tile<32>(a, blockIdx.x);
     if (tile.live <= 0) return;  // (a grid larger than the runs need)
-    const int t_hi = a.pos[tile.row(tile.live - 1)], t_lo = a.window > 0 ? max(0, a.pos[tile.row(0)] - a.window + 1) : 0;
+    const int t_hi = a.pos[tile.row(tile.live - 1)], q_lo = a.pos[tile.row(0)], t_lo = pg_first_key(a, q_lo);
     const int first = t_lo / 32, nb = t_hi / 32 - first + 1, per = (nb + a.splits - 1) / a.splits;
     const int b_begin = first + (int)blockIdx.y * per, b_end = min(first + nb, b_begin + per);
 
     const int p = min(c, tile.live - 1), row = tile.row(p), head = tile.head(p);
-    const int t_q = a.pos[row], t_min = a.window > 0 ? t_q - a.window + 1 : 0;
+    const int t_q = a.pos[row], t_min = pg_first_key(a, t_q);
+    const PgDistance dist = pg_distance<DIST>(a, tile, head, (float *)s_o);  // (the sums come there when nobody looks up distances any more)
     uint4 qf[KS];
 #pragma unroll
     for (int s = 0; s < KS; ++s)
@@ -242,7 +372,7 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_page_attn(const PageAt
             if (16 * s < geo.D16) s0 = MfmaT<BF16>::run(kf[s], qf[s], s0);
         load_k(nx, pn);  // on its way during the softmax and the second product
         u32 hi[8], lo[8];
-        pg_softmax<DT>(s0, true, b * 32, h, t_q, t_min, sl2, m_run, l_run, o, hi, lo);
+        pg_softmax<DT, DIST>(s0, true, q_lo - (b * 32 + 31) < dist.far, dist, b * 32, h, t_q, t_min, sl2, m_run, l_run, o, hi, lo);
 #pragma unroll
         for (int d = 0; d < DT; ++d)
             if (32 * d < geo.V32)
@@ -272,7 +402,7 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_page_attn(const PageAt
     if (c >= tile.live) return;
     const size_t pr = (size_t)row * geo.H + head, MH = (size_t)a.M * geo.H;
     float factor = 1.0f;
-    if (a.splits == 1) factor = pg_gate(a, false, row, head) / (l + (a.sink > 0.0f ? a.sink * __builtin_amdgcn_exp2f(-mx) : 0.0f));
+    if (a.splits == 1) factor = pg_factor(a, false, row, head, mx, l);
 #pragma unroll
     for (int j = 0; j < DT; ++j) {
         const int q = wave * DT + j, d0 = 32 * (q >> 2) + 8 * (q & 3) + 4 * h;  // registers 4 k .. + 3 of block d <-> dims 32 d + 8 k + 4 h + {0 .. 3}
@@ -296,9 +426,8 @@ __global__ void __launch_bounds__(64) k_page_combine(const PageAttnArgs a) {
     const int row = (int)(pr / geo.H), head = (int)(pr % geo.H), lane = threadIdx.x;
     const float2 ml = lane < a.splits ? *(const float2 *)(a.ws + (size_t)a.splits * MH * geo.V32 + (lane * MH + pr) * 2) : make_float2(PG_NEG, 0.0f);
     const float mx = wave_max(ml.y > 0.0f ? ml.x : PG_NEG), f = ml.y > 0.0f ? __builtin_amdgcn_exp2f(ml.x - mx) : 0.0f;
-    const float total = wave_sum(ml.y * f) + (a.sink > 0.0f ? a.sink * __builtin_amdgcn_exp2f(-mx) : 0.0f);
     __shared__ float s_f[64];
-    s_f[lane] = f * (pg_gate(a, false, row, head) / total);
+    s_f[lane] = f * pg_factor(a, false, row, head, mx, wave_sum(ml.y * f));
     __syncthreads();
     const LatentMerge m = {a.ws, a.splits, a.M, geo.H, geo.V32};
     for (int d = lane * 4; d < geo.V8; d += 256) {
@@ -308,23 +437,25 @@ __global__ void __launch_bounds__(64) k_page_combine(const PageAttnArgs a) {
 }
 
 // ---------------------------------------------------------------- long form
-template <int KS, int DT>
+template <int KS, int DT, int DIST>
 __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_page_attn_long(const PageAttnArgs a) {
     constexpr int BUF = PAGE_TOKENS * (16 * KS + 32 * DT) * 2;
     __shared__ __attribute__((aligned(1024))) char s_kv[2 * BUF];
+    __shared__ float s_near[DIST == PG_NEAR_LDS ? PG_TABLE : 1];
     const KvGeometry &geo = a.geo;
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), c = lane & 31, h = lane >> 5;
     const PgTile tile = pg_tile<128>(a, (int)gridDim.x / geo.G * geo.G - geo.G - (int)blockIdx.x / geo.G * geo.G + (int)blockIdx.x % geo.G);  // later rows (more keys) first
     if (tile.live <= 0) return;
-    const int t_last = tile.run.pos0 + (tile.p0 + tile.live - 1) / tile.gs, t_lo = a.window > 0 ? max(0, tile.run.pos0 + tile.p0 / tile.gs - a.window + 1) : 0;
+    const int t_last = tile.run.pos0 + (tile.p0 + tile.live - 1) / tile.gs, t_lo = pg_first_key(a, tile.run.pos0 + tile.p0 / tile.gs);
     const int g0 = t_lo / PAGE_TOKENS, g1 = t_last / PAGE_TOKENS;
 
     const int w0 = 32 * wave;
     const bool busy = w0 < tile.live;
     const int p = min(w0 + c, tile.live - 1), row = tile.row(p), head = tile.head(p);
-    const int t_q = tile.run.pos0 + row - tile.run.row0, t_min = a.window > 0 ? t_q - a.window + 1 : 0;
+    const int t_q = tile.run.pos0 + row - tile.run.row0, t_min = pg_first_key(a, t_q);
+    const PgDistance dist = pg_distance<DIST>(a, tile, head, s_near);
     const int q_lo = tile.run.pos0 + (tile.p0 + min(w0, tile.live - 1)) / tile.gs, q_hi = tile.run.pos0 + (tile.p0 + min(w0 + 31, tile.live - 1)) / tile.gs;  // the wave's positions
-    const int k_lo = a.window > 0 ? q_lo - a.window + 1 : 0, k_full = a.window > 0 ? q_hi - a.window + 1 : 0;
+    const int k_lo = pg_first_key(a, q_lo), k_full = pg_first_key(a, q_hi);
     uint4 qf[KS];
 #pragma unroll
     for (int s = 0; s < KS; ++s)
@@ -373,7 +504,7 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_page_attn_long(const P
             for (int s = 0; s < KS; ++s)
                 if (16 * s < geo.D16) s0 = MfmaT<BF16>::run(*(const uint4 *)(kb + s * 1024), qf[s], s0);
             u32 hi[8], lo[8];
-            pg_softmax<DT>(s0, !(t0 + 31 <= q_lo && t0 >= k_full), t0, h, t_q, t_min, sl2, m_run, l_run, o, hi, lo);
+            pg_softmax<DT, DIST>(s0, !(t0 + 31 <= q_lo && t0 >= k_full), q_lo - (t0 + 31) < dist.far, dist, t0, h, t_q, t_min, sl2, m_run, l_run, o, hi, lo);
 #pragma unroll
             for (int d = 0; d < DT; ++d)
                 if (32 * d < geo.V32)
@@ -387,7 +518,7 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_page_attn_long(const P
     }
     const float l = xor32_sum(l_run);
     if (w0 + c >= tile.live) return;
-    const float factor = pg_gate(a, false, row, head) / (l + (a.sink > 0.0f ? a.sink * __builtin_amdgcn_exp2f(-m_run) : 0.0f));
+    const float factor = pg_factor(a, false, row, head, m_run, l);
     u16 *dst = (u16 *)a.out + (size_t)row * a.ld_out + head * geo.V8;
 #pragma unroll
     for (int d = 0; d < DT; ++d)
@@ -409,7 +540,8 @@ __global__ void __launch_bounds__(256) k_page_attn_rows(const PageAttnArgs a) {
     for (int d = threadIdx.x; d < geo.dim; d += 256) s_q[d] = E::load((const T *)a.q + (size_t)row * a.ldq + head * geo.D8 + d);
     for (int d = lane; d < geo.vdim; d += 64) s_o[wave][d] = 0.0f;
     __syncthreads();
-    const int t_q = a.pos[row], t_lo = a.window > 0 ? max(0, t_q - a.window + 1) : 0, seq = a.row_seq[row];
+    const int t_q = a.pos[row], t_lo = pg_first_key(a, t_q), seq = a.row_seq[row];
+    const float *near = a.distance ? a.distance + (size_t)head * (a.far + 1) : nullptr;
     float m = PG_NEG, l = 0.0f;
     for (int t = t_lo + wave; t <= t_q; t += 4) {
         const T *kv = (const T *)a.slab + (size_t)page_of(a.pages, seq, t) * geo.page_elems() + g * geo.head_elems();
@@ -417,21 +549,24 @@ __global__ void __launch_bounds__(256) k_page_attn_rows(const PageAttnArgs a) {
         float s = 0.0f;
         for (int d = lane; d < geo.dim; d += 64) s = fmaf(s_q[d], E::load(kv + geo.key(tl, d)), s);
         s = wave_sum(s) * a.scale;
+        if (near) s += near[min(t_q - t, a.far)];
         const float m2 = fmaxf(m, s), f = expf(m - m2), w = expf(s - m2);
         l = l * f + w, m = m2;
         for (int d = lane; d < geo.vdim; d += 64) s_o[wave][d] = fmaf(w, E::load(kv + geo.value(tl, d)), s_o[wave][d] * f);
     }
     if (lane == 0) s_m[wave] = m, s_l[wave] = l;
     __syncthreads();
-    const float mx = fmaxf(fmaxf(s_m[0], s_m[1]), fmaxf(s_m[2], s_m[3]));
-    float f[4], sum = a.sink > 0.0f ? a.sink * expf(-mx) : 0.0f;
+    float mx = fmaxf(fmaxf(s_m[0], s_m[1]), fmaxf(s_m[2], s_m[3]));
+    if (a.head_sink) mx = fmaxf(mx, a.head_sink[head]);
+    float f[4], sum = a.head_sink ? expf(a.head_sink[head] - mx) : a.sink > 0.0f ? a.sink * expf(-mx) : 0.0f;
 #pragma unroll
     for (int w = 0; w < 4; ++w) f[w] = s_l[w] > 0.0f ? expf(s_m[w] - mx) : 0.0f, sum += s_l[w] * f[w];
-    const float factor = pg_gate(a, sizeof(T) == 4, row, head) / sum;
+    const float factor = pg_gate(a, sizeof(T) == 4, row, head) * a.out_scale / sum;
     for (int d = threadIdx.x; d < geo.vdim; d += 256)
         ((T *)a.out)[(size_t)row * a.ld_out + head * geo.V8 + d] = E::pack((s_o[0][d] * f[0] + s_o[1][d] * f[1] + s_o[2][d] * f[2] + s_o[3][d] * f[3]) * factor);
 }
 
+bool pg_lds_table(const PageAttnArgs &a) { return a.distance && (long)(a.geo.H / a.geo.G) * (a.far + 1) <= PG_TABLE; }
 int pg_class(const KvGeometry &g) {  // 32-wide classes of the instantiations
     const int n = ((g.D16 + 31) / 32 * 32 > g.V32 ? (g.D16 + 31) / 32 : g.V32 / 32);
     return n <= 4 ? n : n <= 6 ? 6 : 8;
@@ -446,6 +581,14 @@ bool page_attn_mfma(int dtype, const KvGeometry &g) { return dtype == PIE_BF16 &
 
 int kv_prep_launch(int dtype, const KvPrepArgs &a, hipStream_t st) {
     if (a.M <= 0) return PIE_OK;
+    if (a.row_norm) {
+        PIE_REQUIRE(a.q_norm && (a.k_norm || !a.own) && a.geo.dim == a.geo.vdim && a.rot_dims == 0 && !a.value_norm && a.ld % 8 == 0, PIE_E_SHAPE,
+                    "paged attention: norms over all heads go with values that are the keys, without rotation");
+        if (dtype == PIE_F32) hipLaunchKernelGGL(k_kv_prep_row<ElemF32>, dim3((unsigned)a.M), dim3(256), 0, st, a);
+        else hipLaunchKernelGGL(k_kv_prep_row<ElemBF16>, dim3((unsigned)a.M), dim3(256), 0, st, a);
+        PIE_LAUNCH_CHECK();
+        return PIE_OK;
+    }
     const int wide = a.geo.dim > a.geo.vdim ? a.geo.dim : a.geo.vdim;
     const int hb = a.M < 64 || wide > 256 ? 1 : wide > 128 ? 4 : 8;  // few rows: a wave per head
     auto units = [&](int n) { return (n + hb - 1) / hb; };
@@ -465,12 +608,12 @@ int kv_prep_launch(int dtype, const KvPrepArgs &a, hipStream_t st) {
 
 #define PG_CLASSES(GO) \
     switch (pg_class(a.geo)) { \
-        case 1: GO(2, 1); break; \
-        case 2: GO(4, 2); break; \
-        case 3: GO(6, 3); break; \
-        case 4: GO(8, 4); break; \
-        case 6: GO(12, 6); break; \
-        default: GO(16, 8); break; \
+        case 1: { GO(2, 1); } break; \
+        case 2: { GO(4, 2); } break; \
+        case 3: { GO(6, 3); } break; \
+        case 4: { GO(8, 4); } break; \
+        case 6: { GO(12, 6); } break; \
+        default: { GO(16, 8); } break; \
     }
 
 int page_attn_launch(int dtype, const PageAttnArgs &a, hipStream_t st) {
@@ -488,7 +631,11 @@ int page_attn_launch(int dtype, const PageAttnArgs &a, hipStream_t st) {
     PIE_REQUIRE(a.splits >= 1 && a.splits <= 64 && (a.splits == 1 || a.ws), PIE_E_ARG, "paged attention: 1 .. 64 key splits, which need their workspace");
     PIE_REQUIRE(a.ldq % 8 == 0 && a.ld_out % 4 == 0, PIE_E_ALIGN, "paged attention: row strides");
     const dim3 grid((unsigned)a.n_tiles, (unsigned)a.splits);
-#define PG_GO(K_, D_) hipLaunchKernelGGL((k_page_attn<K_, D_>), grid, dim3(256), 0, st, a)
+    const bool lds_table = pg_lds_table(a);
+#define PG_GO(K_, D_) \
+    if (!a.distance) hipLaunchKernelGGL((k_page_attn<K_, D_, PG_PLAIN>), grid, dim3(256), 0, st, a); \
+    else if (lds_table) hipLaunchKernelGGL((k_page_attn<K_, D_, PG_NEAR_LDS>), grid, dim3(256), 0, st, a); \
+    else hipLaunchKernelGGL((k_page_attn<K_, D_, PG_NEAR_GLOBAL>), grid, dim3(256), 0, st, a)
     PG_CLASSES(PG_GO)
 #undef PG_GO
     PIE_LAUNCH_CHECK();
@@ -503,7 +650,11 @@ int page_attn_long_launch(const PageAttnArgs &a, hipStream_t st) {
     if (a.n_tiles <= 0) return PIE_OK;
     PIE_REQUIRE(page_attn_mfma(PIE_BF16, a.geo) && a.ldq % 8 == 0 && a.ld_out % 4 == 0, PIE_E_SHAPE, "paged attention: the long form takes heads of up to 256 numbers");
     const dim3 grid((unsigned)a.n_tiles);
-#define PG_GO(K_, D_) hipLaunchKernelGGL((k_page_attn_long<K_, D_>), grid, dim3(256), 0, st, a)
+    const bool lds_table = pg_lds_table(a);
+#define PG_GO(K_, D_) \
+    if (!a.distance) hipLaunchKernelGGL((k_page_attn_long<K_, D_, PG_PLAIN>), grid, dim3(256), 0, st, a); \
+    else if (lds_table) hipLaunchKernelGGL((k_page_attn_long<K_, D_, PG_NEAR_LDS>), grid, dim3(256), 0, st, a); \
+    else hipLaunchKernelGGL((k_page_attn_long<K_, D_, PG_NEAR_GLOBAL>), grid, dim3(256), 0, st, a)
     PG_CLASSES(PG_GO)
 #undef PG_GO
     PIE_LAUNCH_CHECK();

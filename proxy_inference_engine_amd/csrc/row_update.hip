@@ -1,7 +1,10 @@
-// row_update.hip -- what stands between two sublayers when a norm needs the whole row: x += post(y); h = next(x).
+// row_update.hip -- what stands between two sublayers when a norm needs the whole row: x += post(y), or x = post(alpha x + y); h = next(x).
 //
 // One workgroup per row.  y is a sublayer's output (plus a bias), or the weighted sum of a row's experts; the row stays in registers from the first read to
 // the last store, so the norms' sums cost one exchange through LDS each and x, y and h pass through memory once.
+//
+// In front of a mixer that reads every token mixed with its predecessor, the mixes are made of the new x: by the same workgroup where every run is one row (the predecessor is
+// the sequence's state), by a launch behind it (k_token_mix) where runs are longer.
 //
 // Few rows in front of a mixture: the workgroup goes on with its row's router logits (the row is in LDS, a wave per expert), chooses the experts, and the
 // last workgroup to arrive makes the row lists -- the router, the choice and the lists are no launches of their own.
@@ -76,6 +79,47 @@ __device__ __forceinline__ void row_route(const RowUpdateArgs &a, const float (&
     route_lists(L, a.M, s_cnt, [&](int i) { return __hip_atomic_load(L.chosen + i, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT); }, 0, 0, 0);
 }
 
+// the mixes of one quad of row m's columns; before: the predecessor's
+template <class E>
+__device__ __forceinline__ void token_mix4(const TokenMixArgs &a, size_t m, size_t M, int n, int W, const float (&x)[4], const float (&before)[4]) {
+    typedef typename E::type T;
+#pragma unroll
+    for (int s = 0; s < TIME_MIXES; ++s) {
+        const float4 mu = *(const float4 *)(a.mu + (size_t)s * a.ldmu + n);  // (padded)
+        const float y[4] = {fmaf(before[0] - x[0], mu.x, x[0]), fmaf(before[1] - x[1], mu.y, x[1]), fmaf(before[2] - x[2], mu.z, x[2]), fmaf(before[3] - x[3], mu.w, x[3])};
+        T *out = (T *)a.out + (s * M + m) * a.ldo + n;
+        if (n + 4 <= W) {
+            if constexpr (sizeof(T) == 2) *(uint2 *)out = make_uint2(pack2<BF16>(y[0], y[1]), pack2<BF16>(y[2], y[3]));
+            else *(float4 *)out = make_float4(y[0], y[1], y[2], y[3]);
+        } else
+            for (int i = 0; i < W - n; ++i) out[i] = E::pack(y[i]);
+    }
+}
+__device__ __forceinline__ float *token_mix_state(const TokenMixArgs &a, int m) {
+    return a.state + min((unsigned)a.slots[min(a.row_seq[m], a.n_seqs - 1)], (unsigned)a.n_slots - 1u) * a.slot_floats;
+}
+
+// A thread takes four columns of a row.  The workgroup of a run's first row reads what the state holds and then writes the run's last row there.
+template <class E>
+__global__ void __launch_bounds__(256) k_token_mix(const TokenMixArgs a, const float *x, int ldx, int W) {
+    const int n = (blockIdx.x * 256 + threadIdx.x) * 4, m = blockIdx.y;
+    if (n >= W) return;
+    const bool first = m == 0 || a.row_seq[m - 1] != a.row_seq[m];
+    const float4 v = *(const float4 *)(x + (size_t)m * ldx + n);
+    float4 p = make_float4(0, 0, 0, 0);
+    if (!first) p = *(const float4 *)(x + (size_t)(m - 1) * ldx + n);
+    else {
+        float *held = token_mix_state(a, m) + n;
+        if (a.pos[m] > 0) p = *(const float4 *)held;
+        int last = m;
+        for (int r = 0; r < a.n_runs; ++r)
+            if (a.runs[r].row0 == m) last = m + a.runs[r].n_rows - 1;
+        *(float4 *)held = *(const float4 *)(x + (size_t)last * ldx + n);
+    }
+    const float xv[4] = {v.x, v.y, v.z, v.w}, pv[4] = {p.x, p.y, p.z, p.w};
+    token_mix4<E>(a, m, gridDim.y, n, W, xv, pv);
+}
+
 template <class E, int THREADS, int NQ, bool ROUTE = false>
 __global__ void __launch_bounds__(THREADS) k_row_update(const RowUpdateArgs a) {
     typedef typename E::type T;
@@ -134,6 +178,12 @@ __global__ void __launch_bounds__(THREADS) k_row_update(const RowUpdateArgs a) {
 #pragma unroll
             for (int i = 0; i < 4; ++i)
                 if (n0 + 4 * THREADS * q + i >= a.W) y[q][i] = xv[q][i] = 0.0f;
+        if (a.after) {
+#pragma unroll
+            for (int q = 0; q < NQ; ++q)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) y[q][i] = fmaf(a.alpha, xv[q][i], y[q][i]), xv[q][i] = 0.0f;
+        }
         norm_row<THREADS, NQ>(a.post, a.W, y, red[0]);
 #pragma unroll
         for (int q = 0; q < NQ; ++q) {
@@ -150,6 +200,19 @@ __global__ void __launch_bounds__(THREADS) k_row_update(const RowUpdateArgs a) {
 #pragma unroll
             for (int i = 0; i < 4; ++i)
                 if (n0 + 4 * THREADS * q + i >= a.W) xv[q][i] = 0.0f;
+    }
+    if (a.mix.mu) {
+        float *held = token_mix_state(a.mix, (int)m);
+        const bool fresh = a.mix.pos[m] == 0;
+#pragma unroll
+        for (int q = 0; q < NQ; ++q) {
+            const int n = n0 + 4 * THREADS * q;
+            if (n >= a.W) break;
+            const float4 p = fresh ? make_float4(0, 0, 0, 0) : *(const float4 *)(held + n);
+            const float pv[4] = {p.x, p.y, p.z, p.w};
+            token_mix4<E>(a.mix, m, gridDim.x, n, a.W, xv[q], pv);
+            *(float4 *)(held + n) = make_float4(xv[q][0], xv[q][1], xv[q][2], xv[q][3]);
+        }
     }
     norm_row<THREADS, NQ>(a.next, a.W, xv, red[1]);
     T *h = (T *)a.h + m * a.ldh;
@@ -199,6 +262,17 @@ int row_update_launch(int dtype, const RowUpdateArgs &a, hipStream_t st) {
     PIE_REQUIRE(!a.route || (a.router && a.arrived && a.experts > 0 && ((size_t)a.W + 8 + 3 * a.experts) * 4 <= 64 * 1024 - 1024 && a.W <= 16384), PIE_E_SHAPE, "row update: too wide to route beside");
     if (dtype == PIE_F32) row_go<ElemF32>(a, st);
     else row_go<ElemBF16>(a, st);
+    PIE_LAUNCH_CHECK();
+    return PIE_OK;
+}
+
+int token_mix_launch(int dtype, const TokenMixArgs &a, const float *x, int ldx, int M, int W, hipStream_t st) {
+    if (M <= 0) return PIE_OK;
+    PIE_REQUIRE(a.mu && a.state && a.out && a.slots && a.runs && a.n_runs > 0, PIE_E_ARG, "token mixes: missing operand");
+    PIE_REQUIRE(W > 0 && M <= 65535 && ldx % 4 == 0 && a.ldo % 4 == 0 && a.ldmu % 4 == 0 && a.ldmu >= ((W + 3) & ~3) && a.slot_floats % 4 == 0, PIE_E_ALIGN, "token mixes: row strides must be multiples of 4");
+    const dim3 grid((unsigned)((W + 1023) / 1024), (unsigned)M);
+    if (dtype == PIE_F32) hipLaunchKernelGGL(k_token_mix<ElemF32>, grid, dim3(256), 0, st, a, x, ldx, W);
+    else hipLaunchKernelGGL(k_token_mix<ElemBF16>, grid, dim3(256), 0, st, a, x, ldx, W);
     PIE_LAUNCH_CHECK();
     return PIE_OK;
 }

@@ -6,8 +6,10 @@
 // v_mfma_f32_16x16x32_bf16; the B operand is the matching 16 B of up to 16 rows of x, read through L2.  One row of x uses one of the 16 columns,
 // which costs nothing: the matrix cores are idle either way.  The K-split partial sums meet in LDS.
 //
-// The same kernel runs batched over heads (per-head up- / down-projections), grouped over the active experts of a mixture (row lists), and for
+// The same kernel runs batched over heads (per-head up- / down-projections), over a list of unlike matrices, grouped over the active experts of a mixture (row lists), and for
 // any M (blockIdx.z walks 16 * NT rows at a time).
+#include <algorithm>
+
 #include "stack_types.hpp"
 
 size_t w16m_size(int N, int K);
@@ -31,6 +33,11 @@ __device__ __forceinline__ bool rows_select(const RowsArgs &a, RowsWork &k) {
     k.w = a.m.w, k.x = a.m.x, k.y = a.m.y, k.N = a.m.N, k.K = a.m.K, k.ldx = a.m.ldx, k.ldy = a.m.ldy;
     k.count = a.M, k.row0 = 0, k.rows = a.rows, k.xoff = k.yoff = 0;
     const int b = blockIdx.y;
+    if (a.n_mats) {
+        const RowsMat &m = a.mats[b];
+        k.w = m.w, k.x = m.x, k.y = m.y, k.N = m.N, k.K = m.K, k.ldx = m.ldx, k.ldy = m.ldy;
+        return true;
+    }
     if (a.shared.w && b == (int)gridDim.y - 1) {
         k.w = a.shared.w, k.x = a.shared.x, k.y = a.shared.y, k.N = a.shared.N, k.K = a.shared.K, k.ldx = a.shared.ldx, k.ldy = a.shared.ldy;
         return true;
@@ -47,7 +54,7 @@ __device__ __forceinline__ bool rows_select(const RowsArgs &a, RowsWork &k) {
     return true;
 }
 
-// One finished value (m: result row inside the group, n: feature); pair: the value of feature n + 1 (ROWS_SILU_MUL, ROWS_CLIP_MUL)
+// One finished value (m: result row inside the group, n: feature); pair: the value of feature n + 1 (ROWS_SILU_MUL, ROWS_CLIP_MUL, ROWS_GELU_MUL)
 template <class E>
 __device__ __forceinline__ void rows_finish(const RowsArgs &a, const RowsWork &k, int m, int n, float v, float pair) {
     typedef typename E::type T;
@@ -67,6 +74,14 @@ __device__ __forceinline__ void rows_finish(const RowsArgs &a, const RowsWork &k
         case ROWS_CLIP_MUL:
             if (!(n & 1)) ((T *)k.y)[row * k.ldy + (n >> 1)] = E::pack(clipped_glu(v, pair, a.act_alpha, a.act_limit));
             break;
+        case ROWS_GELU_MUL:
+            if (!(n & 1)) {
+                if (a.bias) v += BF16::to_f32(a.bias[n]), pair += BF16::to_f32(a.bias[n + 1]);
+                ((T *)k.y)[row * k.ldy + (n >> 1)] = E::pack(gelu_tanh<sizeof(T) == 4>(v) * pair);
+            }
+            break;
+        case ROWS_GELU_SIDE: ((T *)k.y)[row * k.ldy + n] = E::pack(gelu_tanh<sizeof(T) == 4>(v) * BF16::to_f32(token_vector(a.side, row)[n])); break;
+        case ROWS_SOFTCAP: ((float *)k.y)[row * k.ldy + n] = a.act_limit * stack_tanh<sizeof(T) == 4>(v * a.scale / a.act_limit); break;
         case ROWS_SPLIT:
             if (n < a.split) ((T *)k.y)[row * k.ldy + n] = E::pack(v);
             else a.y2[row * a.ldy2 + n - a.split] = v;
@@ -200,7 +215,7 @@ __global__ void __launch_bounds__(512) k_rows_w16m(const RowsArgs a) {
 #pragma unroll
         for (int t = 0; t < NT; ++t) *(mf_f32x4 *)(s_red + (((wave * NN + n) * NT + t) * 16 + c) * ST + 4 * kq) = acc[n][t];
     __syncthreads();
-    const bool paired = a.epi == ROWS_SILU_MUL || a.epi == ROWS_CLIP_MUL;
+    const bool paired = a.epi == ROWS_SILU_MUL || a.epi == ROWS_CLIP_MUL || a.epi == ROWS_GELU_MUL;
     for (int id = threadIdx.x; id < NW * NN * NT * 256; id += 512) {
         const int nl = id & 15, ml = (id >> 4) % (16 * NT), wn2 = id / (256 * NT), w = wn2 / NN, nn = wn2 % NN;
         const int n = ((int)blockIdx.x * NW * NN + wn2) * 16 + nl, m = i0 + ml;
@@ -295,9 +310,16 @@ size_t rows_weight_bytes(int dtype, int N, int K) {
 
 int rows_gemm_launch(int dtype, const RowsArgs &a, int batches, hipStream_t st) {
     if (a.M <= 0 || batches <= 0) return PIE_OK;
-    PIE_REQUIRE(a.m.N > 0 && a.m.K > 0, PIE_E_SHAPE, "row-wise Linear: empty matrix");
+    PIE_REQUIRE(a.n_mats || (a.m.N > 0 && a.m.K > 0), PIE_E_SHAPE, "row-wise Linear: empty matrix");
     PIE_REQUIRE(batches < 65535 && (!rows_riders(a) || !(a.shared.w || a.active)), PIE_E_SHAPE, "row-wise Linear: too many batches");
-    const int n_max = a.shared.w && a.shared.N > a.m.N ? a.shared.N : a.m.N, k_max = a.shared.w && a.shared.K > a.m.K ? a.shared.K : a.m.K;
+    PIE_REQUIRE(a.n_mats == 0 || (a.n_mats == batches && a.n_mats <= ROWS_LIST && !rows_riders(a) && !a.shared.w && !a.active && !a.rows && a.merge.splits <= 0 && !a.x_norm), PIE_E_ARG,
+                "row-wise Linear: a list of matrices is a launch of its own");
+    int n_max = a.shared.w && a.shared.N > a.m.N ? a.shared.N : a.m.N, k_max = a.shared.w && a.shared.K > a.m.K ? a.shared.K : a.m.K;
+    for (int i = 0; i < a.n_mats; ++i) {
+        const RowsMat &m = a.mats[i];
+        PIE_REQUIRE(m.N > 0 && m.K > 0 && m.ldx % 8 == 0 && pie_aligned(m.x, 16) && pie_aligned(m.w, 16), PIE_E_ALIGN, "row-wise Linear: 16-byte alignment required");
+        n_max = i ? std::max(n_max, m.N) : m.N, k_max = i ? std::max(k_max, m.K) : m.K;
+    }
     PIE_REQUIRE(!a.x_norm || (dtype == PIE_BF16 && a.M <= 16 && batches == 1 && !a.active && !a.shared.w && !a.rows && a.merge.splits <= 0), PIE_E_SHAPE, "row-wise Linear: too many rows to norm on the way in");
     if (dtype == PIE_F32) {
         const dim3 grid((unsigned)((n_max + 15) / 16), (unsigned)(batches + rows_riders(a)), (unsigned)((a.M + 15) / 16));

@@ -1,6 +1,6 @@
 // stack_types.hpp -- what the kernels of the layer-stack models share: the element types, the norms that ride in epilogues, and the operand
-// descriptions of the row-wise Linear (rows_gemm.hip), the attentions (latent_attn.hip, window_attn.hip, page_attn.hip), the recurrences (delta_rule.hip, mlstm.hip,
-// mingru.hip) and what stands between sublayers (row_update.hip, stream_update.hip).
+// descriptions of the row-wise Linear (rows_gemm.hip), the attentions (latent_attn.hip, window_attn.hip, page_attn.hip), the recurrences (delta_rule.hip, gated_delta.hip,
+// time_mix.hip, mlstm.hip, mingru.hip) and what stands between sublayers (row_update.hip, stream_update.hip).
 //
 // Every activation row has a stride that is a multiple of 8 elements (act_stride(), or packed); a Linear reads 64 ceil(K / 64) elements of it.  The columns past K meet zero
 // weights, so they only have to be finite: the owner zero-fills its buffers once and keeps 64 elements of slack behind each.
@@ -23,6 +23,19 @@ struct ElemF32 {
     static __device__ __forceinline__ float load(const float *p) { return *p; }
     static __device__ __forceinline__ float pack(float v) { return v; }
 };
+
+// two neighbouring numbers
+struct ElemPair {
+    float x, y;
+};
+template <class E>
+__device__ __forceinline__ ElemPair load_pair(const typename E::type *p) {
+    if constexpr (sizeof(typename E::type) == 4) return {((const float2 *)p)->x, ((const float2 *)p)->y};
+    else {
+        const u32 w = *(const u32 *)p;
+        return {lo_f32<BF16>(w), hi_f32<BF16>(w)};
+    }
+}
 
 // A norm without statistics, applied element by element in fp32: w * tanh(alpha x) + b (Dynamic Tanh).  Because it needs no reduction over the row,
 // the kernel that produces an element can apply both the norm behind its own sublayer and the norm in front of the next one.
@@ -57,6 +70,20 @@ template <bool F32>
 __device__ __forceinline__ float stack_sigmoid(float x) {
     return F32 ? 1.0f / (1.0f + expf(-x)) : __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(x * -STACK_LOG2E));
 }
+
+template <bool F32>
+__device__ __forceinline__ float stack_silu(float x) { return x * stack_sigmoid<F32>(x); }
+template <bool F32>
+__device__ __forceinline__ float stack_tanh(float x) { return F32 ? tanhf(x) : fast_tanh(x); }
+// z / 2 (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3)))
+template <bool F32>
+__device__ __forceinline__ float gelu_tanh(float z) {
+    constexpr float c = 0.79788456080286535588f;
+    return 0.5f * z * (1.0f + stack_tanh<F32>(c * z * fmaf(0.044715f * z, z, 1.0f)));
+}
+// log(1 + e^z)
+template <bool F32>
+__device__ __forceinline__ float stack_softplus(float z) { return fmaxf(z, 0.0f) + log1pf(F32 ? expf(-fabsf(z)) : __builtin_amdgcn_exp2f(-fabsf(z) * STACK_LOG2E)); }
 
 // sin and cos of an angle: the library's in fp32 stacks; else reduced to one turn in two steps, then the trigonometric unit (absolute error about 1e-6)
 template <bool F32>
@@ -262,6 +289,9 @@ enum RowsEpi {
     ROWS_RESIDUAL = 5,   // x[m][n] += post(v);  h[m][n] = T(next(x[m][n]))
     ROWS_CLIP_MUL = 6,   // rows (2 i, 2 i + 1) = (gate_i, up_i): y[m][i] = T(clipped_glu(gate, up))
     ROWS_XIELU = 7,      // y[m][n] = T(xielu(v))
+    ROWS_GELU_MUL = 8,   // rows (2 i, 2 i + 1) = (gate_i, up_i), plus the bias: y[m][i] = T(gelu_tanh(gate) * up)
+    ROWS_GELU_SIDE = 9,  // y[m][n] = T(gelu_tanh(v) * the row's token's side vector[n])
+    ROWS_SOFTCAP = 10,   // y[m][n] = act_limit tanh(v * scale / act_limit), fp32 (capped logits)
 };
 // g sigmoid(alpha g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit)
 __device__ __forceinline__ float clipped_glu(float gate, float up, float alpha, float limit) {
@@ -277,6 +307,15 @@ struct RowsMat {      // one weight matrix with its operand and result
     void *y;
     int ldy;
 };
+// a vector per token id
+struct TokenVectors {
+    const u16 *table;  // bf16 [vocab][ld], the vector at `at`
+    size_t ld, at;
+    const int *ids;    // [M]
+    int vocab;
+};
+__device__ __forceinline__ const u16 *token_vector(const TokenVectors &t, size_t m) { return t.table + (size_t)min(max(t.ids[m], 0), t.vocab - 1) * t.ld + t.at; }
+constexpr int ROWS_LIST = 6;
 struct RowsArgs {
     RowsMat m;
     int M;                 // rows of x (grouped: an upper bound for one expert's rows)
@@ -288,9 +327,13 @@ struct RowsArgs {
     bool gather;           // grouped: x row = list[position] (else x row = position); y row = position always
     RowsMat shared;        // blockIdx.y == batches - 1 when shared.w: all M rows, this matrix (the expert every token takes)
     const int *rows;       // ungrouped, nullable: x row of result row i
+    RowsMat mats[ROWS_LIST];  // n_mats > 0: blockIdx.y picks one of these instead of m, each with its own sizes and operands
+    int n_mats;
+    const u16 *bias;       // ROWS_GELU_MUL: bf16 [N], nullable
+    TokenVectors side;     // ROWS_GELU_SIDE
     int epi;
     float scale;
-    float act_alpha, act_limit;  // ROWS_CLIP_MUL; ROWS_XIELU: its two factors
+    float act_alpha, act_limit;  // ROWS_CLIP_MUL, ROWS_SOFTCAP; ROWS_XIELU: its two factors
     int split;
     float *y2;
     int ldy2;
@@ -402,6 +445,7 @@ struct KvPrepArgs {
     KvGeometry geo;
     bool own, value_norm;   // own: the layer has keys and values of its own
     const float *q_norm, *k_norm;
+    bool row_norm;          // the norms run over all heads of a row at once, weights [heads][D8], and values are the keys in front of their norm (no v in raw); no rotation
     float eps;
     const float *freq;
     int rot_dims;
@@ -423,7 +467,12 @@ struct PageAttnArgs {
     int n_runs, n_tiles, M;
     bool single;            // every run is one row
     int window;             // keys j with 0 <= i - j < window; <= 0: no limit
-    float scale, sink;      // sink: what the softmax's denominator has besides the keys, as the weight of one more score of 0
+    int chunk;              // > 0: keys of the query's own chunk (i / chunk = j / chunk) instead
+    const float *distance;  // fp32 [H][far + 1], nullable: added to the scaled score of a key min(i - j, far) tokens back
+    int far;
+    const float *head_sink; // fp32 [H], nullable: one more score in the denominator (then sink is 0)
+    float out_scale;        // factor on every head's output
+    float scale, sink;      // score = scale q . k (+ distance); sink: what the softmax's denominator has besides the keys, as the weight of one more score of 0
     const void *gate;       // [M][ldg] T logits per head, nullable: every head's output times their sigmoid
     const u16 *gate_bias;   // bf16 [H], nullable
     int ldg;
@@ -467,7 +516,61 @@ int delta_chunks(int n_rows);
 size_t delta_ws_floats(int chunks, int H, int D);
 int delta_launches(int chunks, int H, int D);
 
-// every head's output over its root mean square, times w and the sigmoid of its gate (head_out.hip)
+// causal convolutions over time: taps at most, rows of a run per tile (conv_tiles())
+constexpr int CONV_MAX_TAPS = 16, CONV_ROWS = 16;
+
+// ---------------------------------------------------------------- gated delta rule (gated_delta.hip)
+constexpr int GATED_MAX_DIM = 256;
+struct GatedDeltaArgs {
+    const void *raw;        // [M][ld] T: q, k [G][D8] each, v, gate [H][V8] each, step size, decay [H8] each
+    int ld, M, H, G, D, D8, V, V8, H8;
+    const float *conv;      // fp32 [taps][ldw] over the channels of q, k, v; the last tap reads the token itself
+    int taps, ldw;
+    const float *decay_rate, *decay_bias, *o_norm;  // fp32 [H], [H], [V]
+    float scale, unit_eps, eps;
+    const int *pos, *row_seq, *slots;
+    int n_seqs, n_slots;
+    const RowRun *runs;
+    int n_runs;
+    float *state;           // [n_slots][slot_floats]: [H][D][V], then (at ring) [taps][channels] the last inputs of the convolution, position p at p mod taps
+    size_t slot_floats, ring;
+    void *mixed;            // [M][channels] T: convolved and activated q, k, v; nullptr (step form, every run one row): taken on the way
+    float *ws, *o;          // chunk form: gated_delta_ws_floats(); outputs [M][H][V8] in front of norm and gate (also heads of more than 256 columns)
+    void *out;              // [M][ld_out] T, head h at h * V8
+    int ld_out;
+};
+__host__ __device__ static inline int gated_delta_channels(int H, int G, int D8, int V8) { return 2 * G * D8 + H * V8; }
+int gated_delta_conv_launch(int dtype, const GatedDeltaArgs &a, int tiles, hipStream_t st);  // all runs; tiles: sum of conv_tiles()
+int gated_delta_step_launch(int dtype, const GatedDeltaArgs &a, int row0, int rows, hipStream_t st);
+int gated_delta_chunks_launch(int dtype, const GatedDeltaArgs &a, int chunks, int row0, int rows, hipStream_t st);
+size_t gated_delta_ws_floats(int chunks, int H, int D);
+int gated_delta_chunk_launches(int chunks, int H, int D);
+
+// ---------------------------------------------------------------- time mixing with a decaying matrix state (time_mix.hip)
+constexpr int TIME_MIX_MAX_DIM = 256, TIME_MIX_MAX_RANK = 1024, TIME_MIXES = 5;
+struct TimeMixArgs {
+    const void *r, *k, *v, *gate;  // [M][ld] T each, head h at h * D8
+    const void *low;               // [M][ld_low] T: the decay's low-rank input
+    int ld, ld_low, M, H, D, D8, rank, R8;
+    const u16 *w_decay;            // bf16 [H * D][R8]
+    const float *decay_bias, *bonus, *o_norm;  // fp32 [H * D] each
+    float eps, out_scale;
+    const int *pos, *row_seq, *slots;
+    int n_seqs, n_slots;
+    const RowRun *runs;
+    int n_runs;
+    float *state;                  // [n_slots][slot_floats], of which [H][D][D] (key channel, value column)
+    size_t slot_floats;
+    float *ws, *o;                 // chunk form
+    void *out;                     // [M][ld_out] T, head h at h * D8
+    int ld_out;
+};
+int time_mix_step_launch(int dtype, const TimeMixArgs &a, hipStream_t st);
+int time_mix_chunks_launch(int dtype, const TimeMixArgs &a, int chunks, int row0, int rows, hipStream_t st);
+size_t time_mix_ws_floats(int chunks, int H, int D);
+int time_mix_chunk_launches(int chunks, int H, int D);
+
+// every head's output over its root mean square, times w and the sigmoid (or silu) of its gate (head_out.hip)
 struct HeadOutArgs {
     const float *o;         // [M][H][D8]
     const float *den;       // [M][H], what o is divided by first; nullable
@@ -478,6 +581,8 @@ struct HeadOutArgs {
     float eps;
     void *out;              // [M][ld_out] T, head h at h * D8
     int ld_out;
+    bool shared_w, silu;    // w is [D], the same for all heads; gates are z sigmoid(z)
+    float scale;
 };
 constexpr int HEAD_OUT_MAX_DIM = 2048;
 int head_out_launch(int dtype, const HeadOutArgs &a, int row0, int rows, hipStream_t st);
@@ -546,6 +651,19 @@ struct StackNorm {
     int kind;
 };
 constexpr int ROW_UPDATE_MAX_WIDTH = 32768;
+// mixes of every row with its predecessor in the sequence: out[s][m] = x_m + (x_(m-1) - x_m) mu[s], s < TIME_MIXES; the state carries the last row
+struct TokenMixArgs {
+    const float *mu;        // fp32 [TIME_MIXES][ldmu]; nullptr: none
+    int ldmu;
+    float *state;           // [n_slots][slot_floats], of which [W rounded up to 4]
+    size_t slot_floats;
+    const int *pos, *row_seq, *slots;
+    int n_seqs, n_slots;
+    const RowRun *runs;
+    int n_runs;
+    void *out;              // [TIME_MIXES][M][ldo] T
+    int ldo;
+};
 struct RowUpdateArgs {
     const void *y;          // [M][ldy] (nullptr: x stays as it is, h = next(x)); experts: [M * top][ldy] by position
     bool y32;               // y is fp32 (else bf16)
@@ -555,6 +673,8 @@ struct RowUpdateArgs {
     const float *weight;    // nullable: 1 / top each
     int top;
     StackNorm post, next;
+    bool after;             // the norm runs over the sum: x = post(alpha x + y)
+    float alpha;
     float *x;               // [M][ldx]
     int ldx;
     void *h;                // [M][ldh] T
@@ -564,12 +684,14 @@ struct RowUpdateArgs {
     int experts;
     const u16 *router;      // bf16 [experts][W rounded up to 8], zeros past W
     int *arrived;           // one int, zero before and after
+    TokenMixArgs mix;       // of the new x; only where every run is one row
 };
 int row_update_launch(int dtype, const RowUpdateArgs &a, hipStream_t st);
+int token_mix_launch(int dtype, const TokenMixArgs &a, const float *x, int ldx, int M, int W, hipStream_t st);  // any runs
 
 // ---------------------------------------------------------------- residual streams (stream_update.hip)
 // x_t <- sum_s mix[s][t] x_s + out[t] y;  h = next(sum_s in[s] x_s), and the causal convolution over time in front of a mixer: h + conv(h)
-constexpr int STREAMS_MAX = 16, CONV_MAX_TAPS = 16;
+constexpr int STREAMS_MAX = 16;
 struct StackEmbed {
     const int *ids;         // nullptr: the streams are in memory already
     const u16 *table, *bigram, *positions;  // bf16 [vocab][W]; [buckets + 1][W], [max_positions][W], nullable

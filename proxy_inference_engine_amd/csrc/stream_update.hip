@@ -172,8 +172,6 @@ __global__ void __launch_bounds__(THREADS) k_stream_update(const StreamUpdateArg
 }
 
 // ---------------------------------------------------------------- the convolution over longer runs
-constexpr int CONV_ROWS = 16;
-
 // TAPS: taps at most.  A thread owns four columns and walks CONV_ROWS rows of one run with the last inputs in registers; the run's first tile carries the state.
 template <class E, int TAPS>
 __global__ void __launch_bounds__(256) k_conv(const ConvArgs a, const typename E::type *hc, typename E::type *h, int ldh, int W) {

@@ -91,7 +91,7 @@ struct W16Args {
 // expert's tiles start at a block -- with all its column tiles, row tile fastest: a block's tiles stream the same weight tiles through one L2 at the same time.
 template <class T, int MB, int SW, int ACT, bool GRP = false>
 __global__ void __launch_bounds__(256) k_w16l_gemm(const W16Args a) {
-    constexpr bool SWIGLU = ACT == MFMA_ACT_SWIGLU || ACT == MFMA_ACT_CLIPPED;
+    constexpr bool SWIGLU = ACT == MFMA_ACT_SWIGLU || ACT == MFMA_ACT_CLIPPED || ACT == MFMA_ACT_GELU;
     constexpr int MT = 32 * MB, XJ = MB;  // rows per tile; DMA instructions per wave and tile (MT / 8 row groups over 4 waves)
     constexpr int WL = 4 * SW;            // weight loads per wave and step
     constexpr int XB = 4, CHUNK = MT * 128;  // x buffers (tile v lives in buffer v % 4); bytes each

@@ -18,18 +18,22 @@ static int w16_fill(W16Args &a, const void *w16m, const void *x, int ldx, int N,
     return PIE_OK;
 }
 
-// y = T(act(x . W^T)), bf16; act: MFMA_ACT_RELU2 or MFMA_ACT_XIELU (alpha, beta: its factors)
-int w16l_act_launch(const void *w16m, const void *x, int ldx, int M, int N, int K, void *y, int ldy, int act, float alpha, float beta, hipStream_t st) {
+// y = T(act(x . W^T)), bf16; act: MFMA_ACT_NONE, MFMA_ACT_RELU2, MFMA_ACT_XIELU (alpha, beta: its factors) or MFMA_ACT_GELU of the interleaved matrix, N / 2 wide (bias bf16 [N], nullable)
+int w16l_act_launch(const void *w16m, const void *x, int ldx, int M, int N, int K, void *y, int ldy, int act, float alpha, float beta, const void *bias, hipStream_t st) {
     W16Args a = {};
     if (int rc = w16_fill(a, w16m, x, ldx, N, K, y, ldy)) return rc;
     PIE_REQUIRE((size_t)256 * ldx * 2 < (1ull << 32), PIE_E_SHAPE, "16-bit GEMM: row stride too long");
-    PIE_REQUIRE(act == MFMA_ACT_RELU2 || act == MFMA_ACT_XIELU, PIE_E_ARG, "16-bit GEMM: unknown activation");
+    PIE_REQUIRE(act == MFMA_ACT_NONE || act == MFMA_ACT_RELU2 || act == MFMA_ACT_XIELU || (act == MFMA_ACT_GELU && N % 8 == 0), PIE_E_ARG, "16-bit GEMM: unknown activation");
+    PIE_REQUIRE(!bias || (act == MFMA_ACT_GELU && pie_aligned(bias, 8)), PIE_E_ARG, "16-bit GEMM: a bias goes with the paired gelu");
+    a.bias = (const u16 *)bias;
     int mb = 8;  // the largest row tile that still gives the chip a round of workgroups
     while (mb > 2 && (M <= 16 * mb || a.tn * ((M + 32 * mb - 1) / (32 * mb)) < 200)) mb >>= 1;
     a.M = M, a.tm = (M + 32 * mb - 1) / (32 * mb), a.bm = a.bm < a.tm ? a.bm : a.tm, a.act_alpha = alpha, a.act_limit = beta;
     const dim3 grid((unsigned)(8 * ((a.tn + 7) / 8) * a.tm));
 #define ACT_GO(MB_) \
     if (act == MFMA_ACT_RELU2) hipLaunchKernelGGL((k_w16l_gemm<BF16, MB_, 2, MFMA_ACT_RELU2>), grid, dim3(256), 0, st, a); \
+    else if (act == MFMA_ACT_GELU) hipLaunchKernelGGL((k_w16l_gemm<BF16, MB_, 2, MFMA_ACT_GELU>), grid, dim3(256), 0, st, a); \
+    else if (act == MFMA_ACT_NONE) hipLaunchKernelGGL((k_w16l_gemm<BF16, MB_, 2, MFMA_ACT_NONE>), grid, dim3(256), 0, st, a); \
     else hipLaunchKernelGGL((k_w16l_gemm<BF16, MB_, 2, MFMA_ACT_XIELU>), grid, dim3(256), 0, st, a)
     if (mb == 2) { ACT_GO(2); }
     else if (mb == 4) { ACT_GO(4); }

@@ -119,7 +119,7 @@ class Model(LayerStackModel):
             rows.append(pad(get(p + "g", H, W), up8(H), W))
             bias.append(torch.zeros(up8(H), 1, dtype=torch.bfloat16, device=rows[0].device))
             out = {"mixer": _ffi.PIE_MIXER_ATTENTION, "heads": H, "dim": D, "vdim": V, "kv_heads": G, "kv_from": -1 if own else m.kv_from, "scale": m.scale,
-                   "value_norm": 1, "out_gate": 1, "sink": SINK, "w_in": pack(torch.cat(rows)), "in_bias": torch.cat(bias)[:, 0].to(torch.bfloat16).contiguous(),
+                   "value_norm": 1, "out_gate": 1, "out_scale": 1.0, "sink": SINK, "w_in": pack(torch.cat(rows)), "in_bias": torch.cat(bias)[:, 0].to(torch.bfloat16).contiguous(),
                    "q_norm": flat(p + "q.norm", D), "w_o": pack(pad_head_columns(get(p + "o", W, H * V), H, V)),
                    "o_bias": get(p + "o.b", W).to(torch.bfloat16).contiguous()}
             if own:

@@ -1,6 +1,6 @@
 """Models whose layers are listed one by one, run by the native layer stack (csrc/layer_stack.hip) over paged caches and recurrent state.
 
-A design's module (models/taduzen, models/kodupel, models/bezutar) reads its config.json and packs its checkpoint into `pie_stack_layer` descriptions; this class is what every such
+A design's module (models/taduzen, models/kodupel, models/bezutar, models/lagelorn) reads its config.json and packs its checkpoint into `pie_stack_layer` descriptions; this class is what every such
 model shares with the engines: the cache protocol (make_cache, enable_paged_kv), the calling convention (`model(inputs, cache=)`), the greedy fast
 path (`step`) and the multi-sequence passes (`step_batch`, `prefill_batch`, `step_mixed`, `step_portions`).  Every one of them is the same pass:
 rows of any sequences, each with its own position, in one batch."""
@@ -30,12 +30,14 @@ class Norm(NamedTuple):
 
 class Embedding(NamedTuple):
     """What the residual starts from besides the token's vector.  streams > 0: equal copies of it (hyper-connections); positions: bf16 [rows, width] by position -- no sequence
-    grows beyond them; bigram: bf16 [buckets + 1, width] by (previous token * mul_prev + token * mul_cur) mod buckets, the last row at a sequence's first token."""
+    grows beyond them; bigram: bf16 [buckets + 1, width] by (previous token * mul_prev + token * mul_cur) mod buckets, the last row at a sequence's first token.  side: bf16 [vocab, layers *
+    side size]: not part of the residual's start, but of what every layer adds to it."""
     streams: int = 0
     positions: torch.Tensor | None = None
     bigram: torch.Tensor | None = None
     mul_prev: int = 0
     mul_cur: int = 0
+    side: torch.Tensor | None = None
 
 
 def up8(n: int) -> int:
@@ -95,9 +97,9 @@ def pack_linear(w: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
 
 class LayerStackModel:
     def __init__(self, args, dtype: torch.dtype, width: int, vocab: int, logit_scale: float, layers: list[dict], embed: torch.Tensor, head: torch.Tensor,
-                 final_norm: Norm, embed_scale: float = 1.0, embedding: Embedding = Embedding()):
-        """layers: per layer the fields of pie_stack_layer -- tensors for its pointers, Norms for its norms, numbers for the rest
-        (absent fields are zero).  embed: bf16 [vocab, width]; head: packed."""
+                 final_norm: Norm, embed_scale: float = 1.0, embedding: Embedding = Embedding(), logit_cap: float = 0.0):
+        """layers: per layer the fields of pie_stack_layer -- tensors for its pointers, Norms for its norms, dicts for structures inside it, numbers for
+        the rest (absent fields are zero).  embed: bf16 [vocab, width]; head: packed."""
         self.args, self.dtype, self.width, self.vocab_size = args, dtype, width, vocab
         self.device = embed.device
         self.layers = layers
@@ -106,13 +108,12 @@ class LayerStackModel:
         lib = _ffi.base()
         cfg = _ffi.pie_stack_config(_ffi.stack_dtype_code(dtype), width, vocab, len(layers), logit_scale, embed_scale, embed.data_ptr(), head.data_ptr(), self._norm(final_norm), embedding.streams, self.max_positions or 0,
                                     *(None if t is None else t.data_ptr() for t in (embedding.positions, embedding.bigram)), embedding.mul_prev, embedding.mul_cur,
-                                    0 if embedding.bigram is None else embedding.bigram.shape[0] - 1)
+                                    0 if embedding.bigram is None else embedding.bigram.shape[0] - 1, logit_cap, *((None, 0) if embedding.side is None else (embedding.side.data_ptr(), embedding.side.shape[1] // len(layers))))
         self._stack = C.c_void_p()
         _ffi.check(lib.pie_stack_create(C.byref(cfg), C.byref(self._stack)))
         for i, fields in enumerate(layers):
             lay = _ffi.pie_stack_layer()
-            for name, v in fields.items():
-                setattr(lay, name, self._norm(v) if isinstance(v, Norm) else v.data_ptr() if isinstance(v, torch.Tensor) else v)
+            self._fill(lay, fields)
             _ffi.check(lib.pie_stack_set_layer(self._stack, i, C.byref(lay)))
         self.row_elems = [lib.pie_stack_page_row(self._stack, i) for i in range(len(layers))]
         self.state_floats = [int(lib.pie_stack_state_floats(self._stack, i)) for i in range(len(layers))]
@@ -124,6 +125,14 @@ class LayerStackModel:
         self._page_blocks = 16
         self._bufs: dict = {}      # per decode batch size: the persistent buffers a captured step points at
         torch.cuda.synchronize(self.device)
+
+    @classmethod
+    def _fill(cls, struct, fields: dict) -> None:
+        for name, v in fields.items():
+            if isinstance(v, dict):
+                cls._fill(getattr(struct, name), v)
+            else:
+                setattr(struct, name, cls._norm(v) if isinstance(v, Norm) else v.data_ptr() if isinstance(v, torch.Tensor) else v)
 
     @staticmethod
     def _norm(n: Norm):

@@ -16,11 +16,11 @@ from typing import Any
 import torch
 
 from .. import _ffi, hip_ops
-from . import bezutar, kodupel, taduzen
+from . import bezutar, kodupel, lagelorn, taduzen
 from .llama import Model, ModelArgs
 
 _ARCH_ALIASES = {"llama": "llama", "mistral": "llama"}  # models/utils.py:139-155 (the Llama-shaped subset)
-_ARCHITECTURES = {"Taduzen": taduzen, "Kodupel": kodupel, "Bezutar": bezutar}  # config["architecture"]: designs whose config.json lists the layers one by one
+_ARCHITECTURES = {"Taduzen": taduzen, "Kodupel": kodupel, "Bezutar": bezutar, "Lagelorn": lagelorn}  # config["architecture"]: designs whose config.json lists the layers one by one
 
 
 @dataclass
