@@ -66,7 +66,7 @@ def parse():
                     "IPC-mapped peer memory (default) or RCCL (ncclAllReduce on the launch stream): the comparator for the first run on a real node")
     ap.add_argument("--knob", action="append", default=[], metavar="NAME=VALUE", help="developer: one of the library's test / tuning switches (_ffi.KNOBS) for this run")
     ap.add_argument("--bits", type=int, choices=[2, 4, 6, 8], default=4, help="8 / 6 / 2: MLX int8 / int6 / int2 g=64 weights (W8S / W6S / W2S units; a different workload than the metric's)")
-    ap.add_argument("--design", choices=["taduzen", "kodupel", "bezutar"], help="instead of the metric's workload: prefill and decode throughput of a layer-stack design at sizes that resemble a "
+    ap.add_argument("--design", choices=["taduzen", "kodupel", "bezutar", "lagelorn"], help="instead of the metric's workload: prefill and decode throughput of a layer-stack design at sizes that resemble a "
                     "real model's layers, each beside the dense bf16 Llama of equal size (one JSON line; not the BASELINE.json metric)")
     ap.add_argument("--design-only", default="", help="--design: run only the cases whose name contains this (e.g. dense4096/new/decode1)")
     ap.add_argument("--dense", action="store_true", help="BASELINE.json configs[2]: unquantised bf16 weights (a different workload than the metric's)")
@@ -171,11 +171,21 @@ DESIGN_SIZES = {
     # width, heads, ranks and feed-forward width
     "bezutar": {
         "wide4096": {"width": 4096, "streams": 4, "heads": 32, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "q_rank": 1536, "mlstm": {"heads": 8, "dim": 256, "vdim": 512},
-                     "gru": 4096, "ff": 14336, "near": {"width": 4096, "mixer": {"heads": 32, "dim": 128, "vdim": 128, "kv_rank": 512, "window": None}, "mlp": {"ff": 14336}},
+                     "gru": 4096, "ff": 14336, "near": ("taduzen", {"width": 4096, "mixer": {"heads": 32, "dim": 128, "vdim": 128, "kv_rank": 512, "window": None}, "mlp": {"ff": 14336}}),
                      "like": {"hidden_size": 4096, "intermediate_size": 14336, "num_attention_heads": 32, "num_key_value_heads": 8}},
         "slim2048": {"width": 2048, "streams": 2, "heads": 16, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "q_rank": 768, "mlstm": {"heads": 8, "dim": 128, "vdim": 256},
-                     "gru": 2048, "ff": 8192, "near": {"width": 2048, "mixer": {"heads": 16, "dim": 128, "vdim": 128, "kv_rank": 512, "window": None}, "mlp": {"ff": 8192}},
+                     "gru": 2048, "ff": 8192, "near": ("taduzen", {"width": 2048, "mixer": {"heads": 16, "dim": 128, "vdim": 128, "kv_rank": 512, "window": None}, "mlp": {"ff": 8192}}),
                      "like": {"hidden_size": 2048, "intermediate_size": 8192, "num_attention_heads": 16, "num_key_value_heads": 4}},
+    },
+    # layers: gated delta rule, attention beside time mixing, twice, each with a feed-forward; `near`: the Kodupel (attention and generalised delta rule, mixtures) of equal width, heads and
+    # active feed-forward width
+    "lagelorn": {
+        "wide4096": {"width": 4096, "heads": 32, "kv_heads": 8, "dim": 128, "chunk": 4096, "delta": {"heads": 32, "kv_heads": 16, "dim": 128, "vdim": 128, "conv": 4}, "time_mix": 32, "rank": 128,
+                     "side": 256, "ff": 14336, "near": ("kodupel", "wide4096"),
+                     "like": {"hidden_size": 4096, "intermediate_size": 14336, "num_attention_heads": 32, "num_key_value_heads": 8}},
+        "slim2048": {"width": 2048, "heads": 16, "kv_heads": 4, "dim": 128, "chunk": 4096, "delta": {"heads": 16, "kv_heads": 16, "dim": 128, "vdim": 256, "conv": 4}, "time_mix": 16, "rank": 64,
+                     "side": 128, "ff": 8448, "near": ("kodupel", "fine2048"),
+                     "like": {"hidden_size": 2048, "intermediate_size": 8448, "num_attention_heads": 16, "num_key_value_heads": 4}},
     },
 }
 DESIGN_VOCAB = 32768
@@ -295,12 +305,51 @@ def bezutar_checkpoint(size, n_layers, vocab):
     return cfg, w
 
 
+def lagelorn_checkpoint(size, n_layers, vocab):
+    """(config, device weights) of a random Lagelorn model of one of its DESIGN_SIZES."""
+    W, H, G, D, R, S, F, d, HR = (size[k] for k in ("width", "heads", "kv_heads", "dim", "rank", "side", "ff", "delta", "time_mix"))
+    left = {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5, "bias_max": 128, "mask": {"size": size["chunk"]}}
+    kinds = [("delta", d), ("parallel", {"left": left, "right": {"heads": HR, "dim": D}, "left_scale": 0.7, "right_scale": 0.7})]
+    layers = [{"type": kinds[i % 2][0], "mixer": kinds[i % 2][1], "mlp": {"kind": "dense", "ff": F}} for i in range(n_layers)]
+    cfg = {"architecture": "Lagelorn", "vocab": vocab, "width": W, "max_positions": 8192, "token_side": {"dim": S}, "norm": {"eps": 1e-6}, "postln_alpha": 2.0, "logit_softcap": 30.0, "layers": layers}
+    gen = torch.Generator(device="cuda").manual_seed(0)
+    w = {}
+
+    def put(name, *shape, std=None, mean=0.0):
+        w[name] = (torch.randn(shape, generator=gen, device="cuda") * (shape[-1] ** -0.5 if std is None else std) + mean).to(torch.bfloat16)
+    put("embed", vocab, W, std=1.0), put("pos", 8192, W, std=0.2), put("side.embed", vocab, n_layers * S, std=1.0)
+    for i, lay in enumerate(layers):
+        p = f"l{i}."
+        put(p + "norm1", W, std=0.02, mean=1.0), put(p + "norm2", W, std=0.02, mean=1.0), put(p + "side.gate", S, W), put(p + "side.proj", W, S), put(p + "side.norm", W, std=0.02, mean=0.2)
+        if lay["type"] == "delta":
+            for n, c in (("q", d["kv_heads"] * d["dim"]), ("k", d["kv_heads"] * d["dim"]), ("v", d["heads"] * d["vdim"])):
+                put(p + f"mix.{n}", c, W), put(p + f"mix.{n}.conv", c, d["conv"], std=0.5)
+            put(p + "mix.g", d["heads"] * d["vdim"], W), put(p + "mix.a", d["heads"], W), put(p + "mix.b", d["heads"], W), put(p + "mix.A_log", d["heads"], std=0.5)
+            put(p + "mix.dt_bias", d["heads"], std=1.0, mean=-3.0), put(p + "mix.norm", d["vdim"], std=0.02, mean=1.0), put(p + "mix.o", W, d["heads"] * d["vdim"])
+        else:
+            q = p + "mix.left."
+            put(q + "q", H * D, W), put(q + "q.b", H * D, std=0.02), put(q + "k", G * D, W), put(q + "k.b", G * D, std=0.02), put(q + "q.norm", H * D, std=0.02, mean=1.0)
+            put(q + "k.norm", G * D, std=0.02, mean=1.0), put(q + "rel", 32, H, std=0.5), put(q + "sink", H, std=1.0), put(q + "o", W, H * D)
+            q = p + "mix.right."
+            for n in "rkvgw":
+                put(q + "mu." + n, W, std=0.2, mean=0.5)
+            for n in "rkvg":
+                put(q + n, HR * D, W)
+            put(q + "w1", R, W), put(q + "w2", HR * D, R), put(q + "w0", HR * D, std=1.0, mean=-3.0), put(q + "u", HR, D, std=0.3), put(q + "norm", HR * D, std=0.02, mean=1.0), put(q + "o", W, HR * D)
+        for n in ("gate", "up"):
+            put(p + f"mlp.{n}", F, W), put(p + f"mlp.{n}.b", F, std=0.02)
+        put(p + "mlp.down", W, F), put(p + "mlp.down.b", W, std=0.02)
+    put("final.norm", W, std=0.02, mean=1.0)
+    put("head", vocab, W)
+    return cfg, w
+
+
 def design_bench(args):
     """--design: throughput of a layer-stack design beside the dense bf16 Llama of equal size (and, where one is close, another design), DESIGN_LAYERS layers each."""
     from proxy_inference_engine_amd.models.llama import Model as Llama, ModelArgs as LlamaArgs
-    from proxy_inference_engine_amd.models import bezutar, kodupel, taduzen
+    from proxy_inference_engine_amd.models import bezutar, kodupel, lagelorn, taduzen
     from proxy_inference_engine_amd.models.utils import synthetic_checkpoint
-    design, checkpoint = {"taduzen": (taduzen, taduzen_checkpoint), "kodupel": (kodupel, kodupel_checkpoint), "bezutar": (bezutar, bezutar_checkpoint)}[args.design]
+    designs = {"taduzen": (taduzen, taduzen_checkpoint), "kodupel": (kodupel, kodupel_checkpoint), "bezutar": (bezutar, bezutar_checkpoint), "lagelorn": (lagelorn, lagelorn_checkpoint)}
     rows = []
     rng = np.random.default_rng(0)
 
@@ -315,15 +364,15 @@ def design_bench(args):
         return 1e3 * (time.perf_counter() - t0) / n
 
     for name, size in DESIGN_SIZES[args.design].items():
-        for which in ("new", *(("taduzen",) if "near" in size else ()), "llama"):
+        near = size.get("near")  # another design, and its size (or the name of one)
+        for which in ("new", *((near[0],) if near else ()), "llama"):
             if not any(args.design_only in f"{name}/{which}/{c}" for c in ("decode1", "decode8", "decode32", "prefill512", "prefill4096")):
                 continue
-            if which == "new":
-                cfg, w = checkpoint(size, DESIGN_LAYERS, DESIGN_VOCAB)
+            if which != "llama":
+                design, checkpoint = designs[args.design if which == "new" else which]
+                sized = size if which == "new" else DESIGN_SIZES[which][near[1]] if isinstance(near[1], str) else near[1]
+                cfg, w = checkpoint(sized, DESIGN_LAYERS, DESIGN_VOCAB)
                 model = design.Model(design.ModelArgs(**cfg), w)
-            elif which == "taduzen":
-                cfg, w = taduzen_checkpoint(size["near"], DESIGN_LAYERS, DESIGN_VOCAB)
-                model = taduzen.Model(taduzen.ModelArgs(**cfg), w)
             else:
                 cfg = dict(size["like"], model_type="llama", num_hidden_layers=DESIGN_LAYERS, vocab_size=DESIGN_VOCAB, rms_norm_eps=1e-6, tie_word_embeddings=False,
                            quantization=None)

@@ -91,69 +91,126 @@ __global__ void __launch_bounds__(256) k_gated_conv(const GatedDeltaArgs a, int 
 }
 
 // ---------------------------------------------------------------- step form
+// A token's inputs leave first, the state behind them: the convolution, the lengths and the exchanges of the first token run while the state is still on its way.
 // CV: value columns of a workgroup; RPT: key channels per thread (RPT * NT / CV >= D)
 template <class E, int CV, int NT, int RPT>
-__global__ void __launch_bounds__(NT) k_gated_step(const GatedDeltaArgs a) {
+__global__ void __launch_bounds__(NT, 4) k_gated_step(const GatedDeltaArgs a) {
     typedef typename E::type T;
     constexpr bool F32 = sizeof(T) == 4;
-    constexpr int SL = NT / CV, RP = RPT * SL;
-    static_assert(NT % CV == 0 && CV % 64 == 0, "slices");
+    constexpr int SL = NT / CV, RP = RPT * SL, NI = (2 * RP + 2 * CV + NT - 1) / NT, AHEAD = 3;  // AHEAD: older inputs of the convolution that travel with the token's own
+    static_assert(NT % CV == 0 && CV % 64 == 0 && RP % 64 == 0, "slices");
     __shared__ __attribute__((aligned(16))) float s_q[RP], s_k[RP], s_v[CV], s_g[CV], s_p[SL][CV], s_o[SL][CV], s_ss[CV / 64];
-    const int head = blockIdx.y, D = a.D, V = a.V, lane = threadIdx.x & 63, group = head / (a.H / a.G), c0 = CV * blockIdx.z;
+    const int head = blockIdx.y, D = a.D, V = a.V, lane = threadIdx.x & 63, w0 = __builtin_amdgcn_readfirstlane((int)threadIdx.x), group = head / (a.H / a.G), c0 = CV * blockIdx.z;
     const RowRun run = a.runs[blockIdx.x];
-    const int c = threadIdx.x % CV, col = c0 + c, slice = threadIdx.x / CV, d0 = slice * RPT, C = gated_delta_channels(a.H, a.G, a.D8, a.V8), taps = a.taps;
+    const int c = threadIdx.x % CV, col = c0 + c, slice = w0 / CV, d0 = slice * RPT, C = gated_delta_channels(a.H, a.G, a.D8, a.V8), taps = a.taps;
     float *slot = gated_state(a, run.row0), *state = slot + (size_t)head * D * V, *ring = slot + a.ring;
-    float S[RPT];
-    const int pos0 = a.pos[run.row0];
+    const int pos0 = a.pos[run.row0], at = pos0 % taps;
+    const bool convolve = !a.mixed;
+
+    // what the wave's lanes fetch: q, k, v, gate (what lies past a head: its last number, dropped afterwards)
+    struct Place {
+        int kind, i, ch;  // 0 .. 3, 4: nothing; index in LDS; column of raw
+        bool live;
+    };
+    auto place = [&](int n) -> Place {
+        const int first = w0 + n * NT, kind = first < RP ? 0 : first < 2 * RP ? 1 : first < 2 * RP + CV ? 2 : first < 2 * RP + 2 * CV ? 3 : 4;
+        const int i = first + lane - (kind == 0 ? 0 : kind == 1 ? RP : kind == 2 ? 2 * RP : 2 * RP + CV), d = i + (kind >= 2 ? c0 : 0), size = kind >= 2 ? V : D;
+        const int base = kind == 0 ? group * a.D8 : kind == 1 ? (a.G + group) * a.D8 : 2 * a.G * a.D8 + (kind == 3 ? a.H + head : head) * a.V8;
+        return {kind, i, base + min(d, size - 1), d < size};
+    };
+    float now[NI], w[NI][AHEAD + 1], old[NI][AHEAD], raw_b, raw_a;
+    auto fetch = [&](size_t m) {
+        const T *x = (const T *)a.raw + m * a.ld;
 #pragma unroll
-    for (int i = 0; i < RPT; ++i) S[i] = pos0 > 0 && col < V && d0 + i < D ? state[(size_t)(d0 + i) * V + col] : 0.0f;
-    const float o_norm = a.o_norm[min(col, V - 1)];
+        for (int n = 0; n < NI; ++n) {
+            const Place p = place(n);
+            if (p.kind == 4) continue;
+            now[n] = E::load(p.kind == 3 || convolve ? x + p.ch : (const T *)a.mixed + m * C + p.ch);
+            if (p.kind == 3 || !convolve) continue;
+            w[n][AHEAD] = a.conv[(size_t)(taps - 1) * a.ldw + p.ch];
+            if (taps > 1)
+#pragma unroll
+                for (int k = 0; k < AHEAD; ++k) {
+                    const int back = min(k + 1, taps - 1);
+                    w[n][k] = a.conv[(size_t)(taps - 1 - back) * a.ldw + p.ch], old[n][k] = ring[(size_t)(at < back ? at + taps - back : at - back) * C + p.ch];
+                }
+        }
+        const T *p = x + C + a.H * a.V8 + head;
+        raw_b = E::load(p), raw_a = E::load(p + a.H8);
+    };
+    auto place_inputs = [&] {
+#pragma unroll
+        for (int n = 0; n < NI; ++n) {
+            const Place p = place(n);
+            if (p.kind == 4) continue;
+            float v = now[n];
+            if (p.kind == 3) v = stack_silu<F32>(v);
+            else if (convolve) {
+                v *= w[n][AHEAD];
+#pragma unroll
+                for (int k = 0; k < AHEAD; ++k)
+                    if (k + 1 < taps && pos0 > k) v = fmaf(w[n][k], old[n][k], v);
+                for (int back = AHEAD + 1; back < taps; ++back)
+                    if (pos0 >= back) v = fmaf(a.conv[(size_t)(taps - 1 - back) * a.ldw + p.ch], ring[(size_t)(at < back ? at + taps - back : at - back) * C + p.ch], v);
+                if (taps > 1 && p.live && (p.kind == 2 || (head % (a.H / a.G) == 0 && blockIdx.z == 0))) ring[(size_t)at * C + p.ch] = now[n];
+                v = stack_silu<F32>(v);
+                if constexpr (!F32) v = round_T<BF16>(v);  // (as the launch that convolves runs leaves it)
+            }
+            (p.kind == 0 ? s_q : p.kind == 1 ? s_k : p.kind == 2 ? s_v : s_g)[p.i] = p.live ? v : 0.0f;
+        }
+    };
+    fetch(run.row0);
+    const float rate = a.decay_rate[head], bias = a.decay_bias[head], o_norm = a.o_norm[min(col, V - 1)];
+    __builtin_amdgcn_sched_barrier(0);
+    float S[RPT];
+    const unsigned row4 = 4u * (unsigned)V;
+    unsigned at0 = 4u * (unsigned)min(col, V - 1) + (unsigned)min(d0, D - 1) * row4;  // bytes: a head's state is at most 2 MiB
+    {
+        unsigned off = at0;
+#pragma unroll
+        for (int i = 0; i < RPT; ++i) S[i] = *(const float *)((const char *)state + off), off += d0 + i + 1 < D ? row4 : 0u;
+    }  // (rows past D meet keys and queries of zero)
+    __builtin_amdgcn_sched_barrier(0);
 
     for (int j = 0; j < run.n_rows; ++j) {
         const size_t m = run.row0 + j;
-        const T *x = (const T *)a.raw + m * a.ld;
-        const GatedStep step = gated_step<E>(a, m, head);
-        for (int i = threadIdx.x; i < 2 * RP + 2 * CV; i += NT) {  // q, k, v, gate; what lies past a head: nothing
-            const bool is_q = i < RP, is_k = !is_q && i < 2 * RP, is_g = i >= 2 * RP + CV;
-            const int d = is_q ? i : is_k ? i - RP : c0 + (is_g ? i - 2 * RP - CV : i - 2 * RP), size = is_q || is_k ? D : V;
-            const int ch = is_q ? group * a.D8 + d : is_k ? (a.G + group) * a.D8 + d : 2 * a.G * a.D8 + head * a.V8 + d;
-            float v = 0.0f;
-            if (d < size) {
-                if (is_g) v = stack_silu<F32>(E::load(x + a.H * a.V8 + ch));
-                else if (a.mixed) v = E::load((const T *)a.mixed + m * C + ch);
-                else {
-                    const float now = E::load(x + ch);
-                    v = now * a.conv[(size_t)(taps - 1) * a.ldw + ch];
-                    for (int k = 1; k < taps; ++k)
-                        if (pos0 >= k) v = fmaf(a.conv[(size_t)(taps - 1 - k) * a.ldw + ch], ring[(size_t)((pos0 - k) % taps) * C + ch], v);
-                    if (taps > 1 && (!(is_q || is_k) || (head % (a.H / a.G) == 0 && blockIdx.z == 0))) ring[(size_t)(pos0 % taps) * C + ch] = now;
-                    v = stack_silu<F32>(v);
-                    if constexpr (!F32) v = round_T<BF16>(v);  // (as the launch that convolves runs leaves it)
-                }
-            }
-            float *dst = is_q ? s_q + i : is_k ? s_k + i - RP : is_g ? s_g + i - 2 * RP - CV : s_v + i - 2 * RP;
-            *dst = v;
-        }
+        place_inputs();
+        const float g = stack_exp<F32>(-rate * stack_softplus<F32>(raw_a + bias)), b = stack_sigmoid<F32>(raw_b);
         lds_barrier();
         float qq = 0.0f, kk = 0.0f;  // every wave: the lengths
         for (int d = lane; d < RP; d += 64) qq = fmaf(s_q[d], s_q[d], qq), kk = fmaf(s_k[d], s_k[d], kk);
-        const float uq = a.scale / sqrtf(lanes_sum(qq) + a.unit_eps), uk = 1.0f / sqrtf(lanes_sum(kk) + a.unit_eps), g = stack_exp<F32>(step.log_g);
+        const float uq = a.scale / sqrtf(lanes_sum(qq) + a.unit_eps), uk = 1.0f / sqrtf(lanes_sum(kk) + a.unit_eps);
+        if (j == 0 && pos0 == 0)
+#pragma unroll
+            for (int i = 0; i < RPT; ++i) S[i] = 0.0f;
         float p = 0.0f;
 #pragma unroll
-        for (int i = 0; i < RPT; ++i) p = fmaf(s_k[d0 + i], S[i], p);
+        for (int i = 0; i < RPT; ++i) {
+            p = fmaf(s_k[d0 + i], S[i], p);
+            if (i % 8 == 7) __builtin_amdgcn_sched_barrier(0);  // (else all the vectors' numbers are in registers at once)
+        }
         s_p[slice][c] = p;
         lds_barrier();
         p = 0.0f;
 #pragma unroll
         for (int i = 0; i < SL; ++i) p += s_p[i][c];
-        const float u = step.b * (s_v[c] - g * (p * uk)) * uk;
+        const float u = b * (s_v[c] - g * (p * uk)) * uk;
         float o = 0.0f;
 #pragma unroll
         for (int i = 0; i < RPT; ++i) {
             S[i] = fmaf(s_k[d0 + i], u, g * S[i]);
             o = fmaf(s_q[d0 + i], S[i], o);
+            if (i % 8 == 7) __builtin_amdgcn_sched_barrier(0);
         }
         s_o[slice][c] = o * uq;
+        if (j + 1 < run.n_rows) fetch(m + 1);
+        else if (col < V)  // the state leaves while the output is finished
+        {
+            asm volatile("" : "+v"(at0));  // (the addresses are made again: kept since the loads, they would take a register each)
+#pragma unroll
+            for (int i = 0; i < RPT; ++i, at0 += row4)
+                if (d0 + i < D) *(float *)((char *)state + at0) = S[i];
+        }
         lds_barrier();
         if (gridDim.z > 1) {  // norm and gate need the other workgroups' columns too
             if (threadIdx.x < CV && col < V) {
@@ -168,6 +225,7 @@ __global__ void __launch_bounds__(NT) k_gated_step(const GatedDeltaArgs a) {
             o = 0.0f;
 #pragma unroll
             for (int i = 0; i < SL; ++i) o += s_o[i][c];
+            o = col < V ? o : 0.0f;
             const float sum = lanes_sum(o * o);
             if (lane == 0) s_ss[threadIdx.x >> 6] = sum;
         }
@@ -180,10 +238,6 @@ __global__ void __launch_bounds__(NT) k_gated_step(const GatedDeltaArgs a) {
         }
         lds_barrier();  // the vectors are written again
     }
-    if (col < V)
-#pragma unroll
-        for (int i = 0; i < RPT; ++i)
-            if (d0 + i < D) state[(size_t)(d0 + i) * V + col] = S[i];
 }
 
 // ---------------------------------------------------------------- chunk form: the operands
@@ -331,10 +385,11 @@ int gated_step_go(const GatedDeltaArgs &a, hipStream_t st) {
     const dim3 grid((unsigned)a.n_runs, (unsigned)a.H, (unsigned)((a.V + cv - 1) / cv));
 #define GS_GO(CV_, NT_, R_) hipLaunchKernelGGL((k_gated_step<E, CV_, NT_, R_>), grid, dim3(NT_), 0, st, a)
 #define GS_D(CV_, NT_) \
-    if (a.D <= 64) GS_GO(CV_, NT_, 64 * CV_ / NT_); \
-    else if (a.D <= 128) GS_GO(CV_, NT_, 128 * CV_ / NT_); \
-    else GS_GO(CV_, NT_, 256 * CV_ / NT_)
+    if (a.D <= 64) { GS_GO(CV_, NT_, 64 * CV_ / NT_); } \
+    else if (a.D <= 128) { GS_GO(CV_, NT_, 128 * CV_ / NT_); } \
+    else { GS_GO(CV_, NT_, 256 * CV_ / NT_); }
     if (cv == 64) { GS_D(64, 512); }
+    else if (cv == 128 && a.D <= 128 && (long)a.n_runs * a.H > 256) { GS_D(128, 512); }
     else if (cv == 128) { GS_D(128, 1024); }
     else { GS_D(256, 1024); }
 #undef GS_D

@@ -902,7 +902,7 @@ void time_mixer(Pass &p, int li, const pie_stack_layer &L, const Into &next, int
     m.state = b.states[li], m.slot_floats = state_layout(s, li).total, m.ws = s->rec_ws.p, m.o = s->rec_o.p, m.out = s->o.p + (size_t)(KO - N) * E, m.ld_out = LO;
     const ChunkPart cp = chunk_part(s, b, L);
     m.n_runs = cp.runs;
-    if (cp.runs) p.rc = time_mix_step_launch(dt, m, p.st), ++p.launches;
+    if (cp.runs) p.rc = time_mix_step_launch(dt, m, 0, cp.rows, p.st), p.launches += t.dim > 128 ? 2 : 1;
     if (!p.rc && cp.chunks) {
         m.runs += cp.runs, m.n_runs = b.n_runs - cp.runs;
         p.rc = time_mix_chunks_launch(dt, m, cp.chunks, cp.rows, M - cp.rows, p.st), p.launches += time_mix_chunk_launches(cp.chunks, t.heads, t.dim);

@@ -244,17 +244,21 @@ struct PgDistance {
     int far;
     float last;         // near[far], times log2 e
 };
+// group g's rows on their way into LDS: before anything else, a barrier in front of pg_distance()
 template <int DIST>
-__device__ __forceinline__ PgDistance pg_distance(const PageAttnArgs &a, const PgTile &tile, int head, float *lds) {
+__device__ __forceinline__ void pg_distance_load(const PageAttnArgs &a, int g, float *lds) {
+    if constexpr (DIST == PG_NEAR_LDS) {
+        const int n = a.geo.H / a.geo.G * (a.far + 1);
+        const float *rows = a.distance + (size_t)g * n;
+        for (int i = threadIdx.x; i < n; i += 256) lds[i] = rows[i];
+    }
+}
+template <int DIST>
+__device__ __forceinline__ PgDistance pg_distance(const PageAttnArgs &a, const PgTile &tile, int head, const float *lds) {
     if constexpr (DIST == PG_PLAIN) return {nullptr, 0, 0.0f};
     const int n = a.far + 1;
-    const float *rows = a.distance + (size_t)tile.g * tile.gs * n;
-    if constexpr (DIST == PG_NEAR_LDS) {
-        for (int i = threadIdx.x; i < tile.gs * n; i += 256) lds[i] = rows[i];
-        __syncthreads();
-        rows = lds;
-    }
-    const float *near = rows + (size_t)(head - tile.g * tile.gs) * n;
+    if constexpr (DIST == PG_NEAR_LDS) __syncthreads();
+    const float *near = DIST == PG_NEAR_LDS ? lds + (head - tile.g * tile.gs) * n : a.distance + (size_t)head * n;
     return {near, a.far, near[a.far] * PG_LOG2E};
 }
 
@@ -305,12 +309,14 @@ __device__ __forceinline__ void pg_softmax(const f32x16_t &s, bool masked, bool 
 }
 
 // ---------------------------------------------------------------- short form
-// KS, DT: upper bounds of D16 / 16 and V32 / 32
-template <int KS, int DT, int DIST>
+// KS, DT: upper bounds of D16 / 16 and V32 / 32 (FULL: heads are exactly that wide, and no load hangs on a branch)
+template <int KS, int DT, int DIST, bool FULL>
 __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_page_attn(const PageAttnArgs a) {
     __shared__ __attribute__((aligned(16))) float s_o[4][DT * 4][64][4];
     __shared__ float s_m[4][32], s_l[4][32];
     const KvGeometry &geo = a.geo;
+    const int D8 = FULL ? 16 * KS : geo.D8, D16 = FULL ? 16 * KS : geo.D16, V8 = FULL ? 32 * DT : geo.V8, V32 = FULL ? 32 * DT : geo.V32;
+    pg_distance_load<DIST>(a, (int)blockIdx.x % geo.G, (float *)s_o);  // (the sums come there when nobody looks up distances any more)
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), c = lane & 31, h = lane >> 5;
     const PgTile tile = pg_tile<32>(a, blockIdx.x);
     if (tile.live <= 0) return;  // (a grid larger than the runs need)
@@ -320,11 +326,10 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_page_attn(const PageAt
 
     const int p = min(c, tile.live - 1), row = tile.row(p), head = tile.head(p);
     const int t_q = a.pos[row], t_min = pg_first_key(a, t_q);
-    const PgDistance dist = pg_distance<DIST>(a, tile, head, (float *)s_o);  // (the sums come there when nobody looks up distances any more)
     uint4 qf[KS];
 #pragma unroll
     for (int s = 0; s < KS; ++s)
-        qf[s] = 16 * s + 8 * h < geo.D8 ? *(const uint4 *)((const u16 *)a.q + (size_t)row * a.ldq + head * geo.D8 + 16 * s + 8 * h) : make_uint4(0, 0, 0, 0);
+        qf[s] = FULL || 16 * s + 8 * h < D8 ? *(const uint4 *)((const u16 *)a.q + (size_t)row * a.ldq + head * D8 + 16 * s + 8 * h) : make_uint4(0, 0, 0, 0);
 
     const u16 *slab = (const u16 *)a.slab + tile.g * geo.head_elems() + lane * 8;
     const size_t page_elems = geo.page_elems();
@@ -339,14 +344,14 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_page_attn(const PageAt
     auto load_k = [&](int b, const u16 *pp) {
 #pragma unroll
         for (int s = 0; s < KS; ++s)
-            if (16 * s < geo.D16) kf[s] = *(const uint4 *)(pp + (b & 1) * 32 * geo.D16 + s * 512);
+            if (FULL || 16 * s < D16) kf[s] = *(const uint4 *)(pp + (b & 1) * 32 * D16 + s * 512);
     };
     auto load_v = [&](int b, const u16 *pp) {
 #pragma unroll
         for (int d = 0; d < DT; ++d)
-            if (32 * d < geo.V32)
+            if (FULL || 32 * d < V32)
 #pragma unroll
-                for (int s = 0; s < 2; ++s) vf[d][s] = *(const uint4 *)(pp + PAGE_TOKENS * geo.D16 + (b & 1) * 32 * geo.V32 + d * 1024 + s * 512);
+                for (int s = 0; s < 2; ++s) vf[d][s] = *(const uint4 *)(pp + PAGE_TOKENS * D16 + (b & 1) * 32 * V32 + d * 1024 + s * 512);
     };
 
     f32x16_t o[DT];
@@ -361,6 +366,7 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_page_attn(const PageAt
         load_k(b_begin + wave, pp);
         load_v(b_begin + wave, pp);
     }
+    const PgDistance dist = pg_distance<DIST>(a, tile, head, (const float *)s_o);
     for (int b = b_begin + wave; b < b_end; b += 4) {
         const int nx = min(b + 4, b_end - 1);
         const u16 *pn = block(nx);
@@ -369,13 +375,13 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_page_attn(const PageAt
         for (int i = 0; i < 16; ++i) s0[i] = 0.0f;
 #pragma unroll
         for (int s = 0; s < KS; ++s)
-            if (16 * s < geo.D16) s0 = MfmaT<BF16>::run(kf[s], qf[s], s0);
+            if (FULL || 16 * s < D16) s0 = MfmaT<BF16>::run(kf[s], qf[s], s0);
         load_k(nx, pn);  // on its way during the softmax and the second product
         u32 hi[8], lo[8];
         pg_softmax<DT, DIST>(s0, true, q_lo - (b * 32 + 31) < dist.far, dist, b * 32, h, t_q, t_min, sl2, m_run, l_run, o, hi, lo);
 #pragma unroll
         for (int d = 0; d < DT; ++d)
-            if (32 * d < geo.V32)
+            if (FULL || 32 * d < V32)
 #pragma unroll
                 for (int s = 0; s < 2; ++s) {
                     o[d] = MfmaT<BF16>::run(vf[d][s], make_uint4(hi[4 * s], hi[4 * s + 1], hi[4 * s + 2], hi[4 * s + 3]), o[d]);
@@ -406,15 +412,15 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_page_attn(const PageAt
 #pragma unroll
     for (int j = 0; j < DT; ++j) {
         const int q = wave * DT + j, d0 = 32 * (q >> 2) + 8 * (q & 3) + 4 * h;  // registers 4 k .. + 3 of block d <-> dims 32 d + 8 k + 4 h + {0 .. 3}
-        if (d0 >= geo.V8) continue;
+        if (d0 >= V8) continue;
         const pg_f32x4 v = (*(const pg_f32x4 *)s_o[0][q][lane] + *(const pg_f32x4 *)s_o[1][q][lane]) + (*(const pg_f32x4 *)s_o[2][q][lane] + *(const pg_f32x4 *)s_o[3][q][lane]);
         if (a.splits == 1)
-            *(uint2 *)((u16 *)a.out + (size_t)row * a.ld_out + head * geo.V8 + d0) = make_uint2(w4m_pack<BF16>(v[0] * factor, v[1] * factor), w4m_pack<BF16>(v[2] * factor, v[3] * factor));
+            *(uint2 *)((u16 *)a.out + (size_t)row * a.ld_out + head * V8 + d0) = make_uint2(w4m_pack<BF16>(v[0] * factor, v[1] * factor), w4m_pack<BF16>(v[2] * factor, v[3] * factor));
         else
-            *(pg_f32x4 *)(a.ws + ((size_t)blockIdx.y * MH + pr) * geo.V32 + d0) = v;
+            *(pg_f32x4 *)(a.ws + ((size_t)blockIdx.y * MH + pr) * V32 + d0) = v;
     }
     if (a.splits > 1 && wave == 0 && h == 0) {
-        float *ml = a.ws + (size_t)a.splits * MH * geo.V32 + ((size_t)blockIdx.y * MH + pr) * 2;
+        float *ml = a.ws + (size_t)a.splits * MH * V32 + ((size_t)blockIdx.y * MH + pr) * 2;
         ml[0] = mx, ml[1] = l;
     }
 }
@@ -437,12 +443,14 @@ __global__ void __launch_bounds__(64) k_page_combine(const PageAttnArgs a) {
 }
 
 // ---------------------------------------------------------------- long form
-template <int KS, int DT, int DIST>
+template <int KS, int DT, int DIST, bool FULL>
 __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_page_attn_long(const PageAttnArgs a) {
     constexpr int BUF = PAGE_TOKENS * (16 * KS + 32 * DT) * 2;
     __shared__ __attribute__((aligned(1024))) char s_kv[2 * BUF];
     __shared__ float s_near[DIST == PG_NEAR_LDS ? PG_TABLE : 1];
     const KvGeometry &geo = a.geo;
+    const int D8 = FULL ? 16 * KS : geo.D8, D16 = FULL ? 16 * KS : geo.D16, V8 = FULL ? 32 * DT : geo.V8, V32 = FULL ? 32 * DT : geo.V32;
+    pg_distance_load<DIST>(a, (int)blockIdx.x % geo.G, s_near);
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), c = lane & 31, h = lane >> 5;
     const PgTile tile = pg_tile<128>(a, (int)gridDim.x / geo.G * geo.G - geo.G - (int)blockIdx.x / geo.G * geo.G + (int)blockIdx.x % geo.G);  // later rows (more keys) first
     if (tile.live <= 0) return;
@@ -459,10 +467,10 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_page_attn_long(const P
     uint4 qf[KS];
 #pragma unroll
     for (int s = 0; s < KS; ++s)
-        qf[s] = 16 * s + 8 * h < geo.D8 ? *(const uint4 *)((const u16 *)a.q + (size_t)row * a.ldq + head * geo.D8 + 16 * s + 8 * h) : make_uint4(0, 0, 0, 0);
+        qf[s] = FULL || 16 * s + 8 * h < D8 ? *(const uint4 *)((const u16 *)a.q + (size_t)row * a.ldq + head * D8 + 16 * s + 8 * h) : make_uint4(0, 0, 0, 0);
 
     const unsigned lds0 = (unsigned)(size_t)(__attribute__((address_space(3))) void *)s_kv;
-    const int units = (geo.D16 + geo.V32) / 8;  // KiB of a head's page
+    const int units = (D16 + V32) / 8;  // KiB of a head's page
     int pg_first = g0, pg = page_of(a.pages, tile.run.seq, (pg_first + lane) * PAGE_TOKENS);
     auto fetch = [&](int g, int buf) {
         int i = g - pg_first;
@@ -496,18 +504,18 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_page_attn_long(const P
         for (int half = 0; half < 2; ++half) {
             const int t0 = g * PAGE_TOKENS + 32 * half;
             if (!busy || t0 > q_hi || t0 + 31 < k_lo) continue;
-            const char *kb = buf + half * 64 * geo.D16 + lane * 16, *vb = buf + 2 * PAGE_TOKENS * geo.D16 + half * 64 * geo.V32 + lane * 16;
+            const char *kb = buf + half * 64 * D16 + lane * 16, *vb = buf + 2 * PAGE_TOKENS * D16 + half * 64 * V32 + lane * 16;
             f32x16_t s0;
 #pragma unroll
             for (int i = 0; i < 16; ++i) s0[i] = 0.0f;
 #pragma unroll
             for (int s = 0; s < KS; ++s)
-                if (16 * s < geo.D16) s0 = MfmaT<BF16>::run(*(const uint4 *)(kb + s * 1024), qf[s], s0);
+                if (FULL || 16 * s < D16) s0 = MfmaT<BF16>::run(*(const uint4 *)(kb + s * 1024), qf[s], s0);
             u32 hi[8], lo[8];
             pg_softmax<DT, DIST>(s0, !(t0 + 31 <= q_lo && t0 >= k_full), q_lo - (t0 + 31) < dist.far, dist, t0, h, t_q, t_min, sl2, m_run, l_run, o, hi, lo);
 #pragma unroll
             for (int d = 0; d < DT; ++d)
-                if (32 * d < geo.V32)
+                if (FULL || 32 * d < V32)
 #pragma unroll
                     for (int s = 0; s < 2; ++s) {
                         const uint4 v = *(const uint4 *)(vb + d * 2048 + s * 1024);
@@ -519,13 +527,13 @@ __global__ void __launch_bounds__(256, DT <= 4 ? 2 : 1) k_page_attn_long(const P
     const float l = xor32_sum(l_run);
     if (w0 + c >= tile.live) return;
     const float factor = pg_factor(a, false, row, head, m_run, l);
-    u16 *dst = (u16 *)a.out + (size_t)row * a.ld_out + head * geo.V8;
+    u16 *dst = (u16 *)a.out + (size_t)row * a.ld_out + head * V8;
 #pragma unroll
     for (int d = 0; d < DT; ++d)
 #pragma unroll
         for (int k = 0; k < 4; ++k) {
             const int d0 = 32 * d + 8 * k + 4 * h;
-            if (d0 < geo.V8)
+            if (d0 < V8)
                 *(uint2 *)(dst + d0) = make_uint2(w4m_pack<BF16>(o[d][4 * k] * factor, o[d][4 * k + 1] * factor), w4m_pack<BF16>(o[d][4 * k + 2] * factor, o[d][4 * k + 3] * factor));
         }
 }
@@ -632,12 +640,16 @@ int page_attn_launch(int dtype, const PageAttnArgs &a, hipStream_t st) {
     PIE_REQUIRE(a.ldq % 8 == 0 && a.ld_out % 4 == 0, PIE_E_ALIGN, "paged attention: row strides");
     const dim3 grid((unsigned)a.n_tiles, (unsigned)a.splits);
     const bool lds_table = pg_lds_table(a);
+#define PG_DIST(K_, D_, F_) \
+    if (!a.distance) hipLaunchKernelGGL((k_page_attn<K_, D_, PG_PLAIN, F_>), grid, dim3(256), 0, st, a); \
+    else if (lds_table) hipLaunchKernelGGL((k_page_attn<K_, D_, PG_NEAR_LDS, F_>), grid, dim3(256), 0, st, a); \
+    else hipLaunchKernelGGL((k_page_attn<K_, D_, PG_NEAR_GLOBAL, false>), grid, dim3(256), 0, st, a)
 #define PG_GO(K_, D_) \
-    if (!a.distance) hipLaunchKernelGGL((k_page_attn<K_, D_, PG_PLAIN>), grid, dim3(256), 0, st, a); \
-    else if (lds_table) hipLaunchKernelGGL((k_page_attn<K_, D_, PG_NEAR_LDS>), grid, dim3(256), 0, st, a); \
-    else hipLaunchKernelGGL((k_page_attn<K_, D_, PG_NEAR_GLOBAL>), grid, dim3(256), 0, st, a)
+    if (a.geo.D8 == 16 * K_ && a.geo.V8 == 32 * D_) { PG_DIST(K_, D_, true); } \
+    else { PG_DIST(K_, D_, false); }
     PG_CLASSES(PG_GO)
 #undef PG_GO
+#undef PG_DIST
     PIE_LAUNCH_CHECK();
     if (a.splits > 1) {
         hipLaunchKernelGGL(k_page_combine, dim3((unsigned)(a.M * a.geo.H)), dim3(64), 0, st, a);
@@ -651,12 +663,16 @@ int page_attn_long_launch(const PageAttnArgs &a, hipStream_t st) {
     PIE_REQUIRE(page_attn_mfma(PIE_BF16, a.geo) && a.ldq % 8 == 0 && a.ld_out % 4 == 0, PIE_E_SHAPE, "paged attention: the long form takes heads of up to 256 numbers");
     const dim3 grid((unsigned)a.n_tiles);
     const bool lds_table = pg_lds_table(a);
+#define PG_DIST(K_, D_, F_) \
+    if (!a.distance) hipLaunchKernelGGL((k_page_attn_long<K_, D_, PG_PLAIN, F_>), grid, dim3(256), 0, st, a); \
+    else if (lds_table) hipLaunchKernelGGL((k_page_attn_long<K_, D_, PG_NEAR_LDS, F_>), grid, dim3(256), 0, st, a); \
+    else hipLaunchKernelGGL((k_page_attn_long<K_, D_, PG_NEAR_GLOBAL, false>), grid, dim3(256), 0, st, a)
 #define PG_GO(K_, D_) \
-    if (!a.distance) hipLaunchKernelGGL((k_page_attn_long<K_, D_, PG_PLAIN>), grid, dim3(256), 0, st, a); \
-    else if (lds_table) hipLaunchKernelGGL((k_page_attn_long<K_, D_, PG_NEAR_LDS>), grid, dim3(256), 0, st, a); \
-    else hipLaunchKernelGGL((k_page_attn_long<K_, D_, PG_NEAR_GLOBAL>), grid, dim3(256), 0, st, a)
+    if (a.geo.D8 == 16 * K_ && a.geo.V8 == 32 * D_) { PG_DIST(K_, D_, true); } \
+    else { PG_DIST(K_, D_, false); }
     PG_CLASSES(PG_GO)
 #undef PG_GO
+#undef PG_DIST
     PIE_LAUNCH_CHECK();
     return PIE_OK;
 }

@@ -330,8 +330,11 @@ int rows_gemm_launch(int dtype, const RowsArgs &a, int batches, hipStream_t st) 
     PIE_REQUIRE(a.merge.splits <= 64 && (a.merge.splits <= 0 || (a.merge.M == a.M && a.M <= MERGE_ROWS && a.merge.ldr <= MERGE_LDR && a.merge.ldr % 8 == 0 && !a.active && !a.rows)), PIE_E_SHAPE,
                 "row-wise Linear: too many rows or columns to merge key splits on the way in");
     PIE_REQUIRE(a.m.ldx % 8 == 0 && a.x_batch % 8 == 0 && pie_aligned(a.m.x, 16) && pie_aligned(a.m.w, 16), PIE_E_ALIGN, "row-wise Linear: 16-byte alignment required");
-    if (a.M <= 16 || a.active) return rows_go<1, 1>(a, n_max, k_max, batches, st);
-    const bool wide = batches == 1 && n_max >= 32 * 140;  // two feature blocks per wave where half as many workgroups still fill most of the chip
+    int n_all = batches == 1 ? n_max : 0;
+    for (int i = 0; i < a.n_mats; ++i) n_all += a.mats[i].N;
+    const bool narrow = (long)batches * n_max <= 16 * 64 && !a.merge.splits;  // so few workgroups that they should not all read all rows
+    if (a.M <= 16 || a.active || narrow) return rows_go<1, 1>(a, n_max, k_max, batches, st);
+    const bool wide = n_all >= 32 * 140;  // two feature blocks per wave where half as many workgroups still fill most of the chip
     if (a.M <= 32) return wide ? rows_go<2, 2>(a, n_max, k_max, batches, st) : rows_go<2, 1>(a, n_max, k_max, batches, st);
     return wide ? rows_go<4, 2>(a, n_max, k_max, batches, st) : rows_go<4, 1>(a, n_max, k_max, batches, st);
 }

@@ -565,7 +565,7 @@ struct TimeMixArgs {
     void *out;                     // [M][ld_out] T, head h at h * D8
     int ld_out;
 };
-int time_mix_step_launch(int dtype, const TimeMixArgs &a, hipStream_t st);
+int time_mix_step_launch(int dtype, const TimeMixArgs &a, int row0, int rows, hipStream_t st);
 int time_mix_chunks_launch(int dtype, const TimeMixArgs &a, int chunks, int row0, int rows, hipStream_t st);
 size_t time_mix_ws_floats(int chunks, int H, int D);
 int time_mix_chunk_launches(int chunks, int H, int D);

@@ -3,7 +3,8 @@
 // with the decay w = exp(-exp(w2 tanh(.) + b)) per head and key channel, and a bonus u for the current token.  What it reads are projections of the token mixed with its
 // predecessor (row_update.hip); every head's output over its root mean square, times a weight and the silu of its gate, goes to the output projection.
 //
-// Step form (decoded tokens, short runs): one workgroup per (run, head), the state in registers, a thread RPT key channels of one value column; decay, norm and gate on the way.
+// Step form (decoded tokens, short runs): one workgroup per (run, head), the state in registers, a thread RPT key channels of one value column; decay, norm and gate on the way
+// (heads of more than 128 channels: two workgroups, and head_out.hip behind them).
 //
 // Chunk form (longer runs), 16 tokens at a time.  With L_t the sum of the log decays inside the chunk up to t (per channel) and S the state in front of it,
 //   o_t = S^T (e^{L_(t-1)} r_t) + sum_{i<=t} Y_ti v_i,   Y_ti = sum_d r_td k_id e^{L_(t-1) - L_i} for i < t,  sum_d r_td k_td u_d for i = t
@@ -21,24 +22,42 @@ __device__ __forceinline__ float *time_mix_state(const TimeMixArgs &a, const Row
 }
 
 // ---------------------------------------------------------------- step form
-// CV: value columns, a power of two >= D; RPT: key channels per thread
+// A token's inputs leave first, the state behind them: the decay and the exchanges of the first token run while the state is still on its way.
+// CV: value columns of a workgroup; RPT: key channels per thread (RPT * NT / CV >= D)
 template <class E, int CV, int NT, int RPT>
-__global__ void __launch_bounds__(NT) k_time_mix_step(const TimeMixArgs a) {
+__global__ void __launch_bounds__(NT, 4) k_time_mix_step(const TimeMixArgs a) {
     typedef typename E::type T;
     constexpr bool F32 = sizeof(T) == 4;
-    constexpr int SL = NT / CV, CPT = (CV + NT / 8 - 1) / (NT / 8), WS = 2;
-    static_assert(NT % CV == 0 && CV % 64 == 0 && RPT * SL == CV, "slices");
-    __shared__ __attribute__((aligned(16))) float s_r[CV], s_k[CV], s_v[CV], s_g[CV], s_w[CV], s_u[CV], s_low[TIME_MIX_MAX_RANK], s_o[SL][CV], s_ss[CV / 64];
-    const int head = blockIdx.y, D = a.D, lane = threadIdx.x & 63;
+    constexpr int SL = NT / CV, RP = RPT * SL, NI = (2 * RP + 2 * CV + NT - 1) / NT, CPT = (RP + NT / 8 - 1) / (NT / 8), WS = 2;  // WS: pieces of the decay's weights that travel with the token
+    static_assert(NT % CV == 0 && CV % 64 == 0 && RP % 64 == 0, "slices");
+    __shared__ __attribute__((aligned(16))) float s_r[RP], s_k[RP], s_w[RP], s_u[RP], s_v[CV], s_g[CV], s_low[TIME_MIX_MAX_RANK], s_o[SL][CV], s_ss[CV / 64];
+    const int head = blockIdx.y, D = a.D, lane = threadIdx.x & 63, w0 = __builtin_amdgcn_readfirstlane((int)threadIdx.x), c0 = CV * blockIdx.z;
     const RowRun run = a.runs[blockIdx.x];
-    const int c = threadIdx.x % CV, slice = threadIdx.x / CV, d0 = slice * RPT, dc = min(c, D - 1);
+    const int c = threadIdx.x % CV, col = c0 + c, slice = w0 / CV, d0 = slice * RPT;
     float *state = time_mix_state(a, run, head);
     const bool fresh = a.pos[run.row0] == 0;
-    float S[RPT];
+
+    // what the wave's lanes fetch: r, k, v, gate (what lies past a head: its last number, dropped afterwards)
+    struct Place {
+        int kind, i, d;  // 0 .. 3, 4: nothing; index in LDS; channel
+        bool live;
+    };
+    auto place = [&](int n) -> Place {
+        const int first = w0 + n * NT, kind = first < RP ? 0 : first < 2 * RP ? 1 : first < 2 * RP + CV ? 2 : first < 2 * RP + 2 * CV ? 3 : 4;
+        const int i = first + lane - (kind == 0 ? 0 : kind == 1 ? RP : kind == 2 ? 2 * RP : 2 * RP + CV), d = i + (kind >= 2 ? c0 : 0);
+        return {kind, i, min(d, D - 1), d < D};
+    };
+    float now[NI], low;
+    auto fetch = [&](size_t m) {
 #pragma unroll
-    for (int i = 0; i < RPT; ++i) S[i] = !fresh && c < D && d0 + i < D ? state[(size_t)(d0 + i) * D + c] : 0.0f;
-    // what all tokens share leaves together with the state: the decay's weights (eight lanes per channel, the first WS pieces), the bonus and the head's norm
-    uint4 wd[CPT][WS];
+        for (int n = 0; n < NI; ++n) {
+            const Place p = place(n);
+            if (p.kind < 4) now[n] = E::load((const T *)(p.kind == 0 ? a.r : p.kind == 1 ? a.k : p.kind == 2 ? a.v : a.gate) + m * a.ld + head * a.D8 + p.d);
+        }
+        low = E::load((const T *)a.low + m * a.ld_low + min((int)threadIdx.x, a.R8 - 1));
+    };
+    fetch(run.row0);
+    uint4 wd[CPT][WS];  // eight lanes per channel
     float db[CPT];
     auto weights = [&](int d, int i) { return *(const uint4 *)(a.w_decay + (size_t)(head * D + min(d, D - 1)) * a.R8 + min(i, a.R8 - 8)); };
 #pragma unroll
@@ -48,20 +67,29 @@ __global__ void __launch_bounds__(NT) k_time_mix_step(const TimeMixArgs a) {
         for (int s = 0; s < WS; ++s) wd[k][s] = weights(d, (threadIdx.x & 7) * 8 + 64 * s);
         db[k] = a.decay_bias[head * D + min(d, D - 1)];
     }
-    const float o_norm = a.o_norm[head * D + dc];
-    if (threadIdx.x < CV) s_u[c] = c < D ? a.bonus[head * D + dc] : 0.0f;
+    const float o_norm = a.o_norm[head * D + min(col, D - 1)];
+    if (threadIdx.x < RP) s_u[threadIdx.x] = (int)threadIdx.x < D ? a.bonus[head * D + threadIdx.x] : 0.0f;
+    __builtin_amdgcn_sched_barrier(0);
+    float S[RPT];
+    const unsigned row4 = 4u * (unsigned)D;
+    unsigned at0 = 4u * (unsigned)min(col, D - 1) + (unsigned)min(d0, D - 1) * row4;  // bytes: a head's state is at most 2 MiB
+    {
+        unsigned off = at0;
+#pragma unroll
+        for (int i = 0; i < RPT; ++i) S[i] = *(const float *)((const char *)state + off), off += d0 + i + 1 < D ? row4 : 0u;
+    }  // (rows past D meet r and k of zero)
+    __builtin_amdgcn_sched_barrier(0);
 
     for (int j = 0; j < run.n_rows; ++j) {
-        const size_t m = run.row0 + j, at = m * a.ld + head * a.D8;
-        for (int i = threadIdx.x; i < 4 * CV; i += NT) {  // r, k, v, gate; channels past D: nothing
-            const int what = i / CV, d = i % CV;
-            float v = 0.0f;
-            if (d < D) v = E::load((const T *)(what == 0 ? a.r : what == 1 ? a.k : what == 2 ? a.v : a.gate) + at + d);
-            if (what == 3) v = stack_silu<F32>(v);
-            float *dst = what == 0 ? s_r : what == 1 ? s_k : what == 2 ? s_v : s_g;
-            dst[d] = v;
+        const size_t m = run.row0 + j;
+#pragma unroll
+        for (int n = 0; n < NI; ++n) {
+            const Place p = place(n);
+            if (p.kind < 4) (p.kind == 0 ? s_r : p.kind == 1 ? s_k : p.kind == 2 ? s_v : s_g)[p.i] = !p.live ? 0.0f : p.kind == 3 ? stack_silu<F32>(now[n]) : now[n];
         }
-        for (int i = threadIdx.x; i < a.R8; i += NT) s_low[i] = i < a.rank ? stack_tanh<F32>(E::load((const T *)a.low + m * a.ld_low + i)) : 0.0f;
+        if ((int)threadIdx.x < a.R8) s_low[threadIdx.x] = (int)threadIdx.x < a.rank ? stack_tanh<F32>(low) : 0.0f;
+#pragma unroll 1
+        for (int i = threadIdx.x + NT; i < a.R8; i += NT) s_low[i] = i < a.rank ? stack_tanh<F32>(E::load((const T *)a.low + m * a.ld_low + i)) : 0.0f;
         lds_barrier();
         auto part = [&](float z, int i, const uint4 &w) {
             const float4 l0 = *(const float4 *)(s_low + i), l1 = *(const float4 *)(s_low + i + 4);
@@ -75,38 +103,63 @@ __global__ void __launch_bounds__(NT) k_time_mix_step(const TimeMixArgs a) {
 #pragma unroll
             for (int s = 0; s < WS; ++s)
                 if ((int)(threadIdx.x & 7) * 8 + 64 * s < a.R8) z = part(z, (threadIdx.x & 7) * 8 + 64 * s, wd[k][s]);
+#pragma unroll 1
             for (int i = (threadIdx.x & 7) * 8 + 64 * WS; i < a.R8; i += 64) z = part(z, i, weights(d, i));
             z = lanes8_sum(z);
-            if ((threadIdx.x & 7) == 0 && d < CV) s_w[d] = d < D ? stack_exp<F32>(-stack_exp<F32>(z + db[k])) : 1.0f;
+            if ((threadIdx.x & 7) == 0 && d < RP) s_w[d] = d < D ? stack_exp<F32>(-stack_exp<F32>(z + db[k])) : 1.0f;
         }
-        const float v = s_v[c];
-        float o = 0.0f, bonus = 0.0f;
+        if (j == 0 && fresh)
 #pragma unroll
-        for (int i = 0; i < RPT; ++i) o = fmaf(s_r[d0 + i], S[i], o), bonus = fmaf(s_r[d0 + i] * s_u[d0 + i], s_k[d0 + i], bonus);
-        s_o[slice][c] = fmaf(bonus, v, o);
+            for (int i = 0; i < RPT; ++i) S[i] = 0.0f;
+        const float v = s_v[c];
+        float o = 0.0f;
+#pragma unroll
+        for (int i = 0; i < RPT; ++i) {
+            o = fmaf(s_r[d0 + i], S[i], o);
+            if (i % 8 == 7) __builtin_amdgcn_sched_barrier(0);  // (else all the vectors' numbers are in registers at once)
+        }
+        s_o[slice][c] = o;
+        float bonus = 0.0f;  // of the current token: the waves that finish the outputs
+        if (threadIdx.x < CV) {
+            for (int d = lane; d < RP; d += 64) bonus = fmaf(s_r[d] * s_u[d], s_k[d], bonus);
+            bonus = lanes_sum(bonus);
+        }
         lds_barrier();
 #pragma unroll
-        for (int i = 0; i < RPT; ++i) S[i] = fmaf(s_k[d0 + i], v, s_w[d0 + i] * S[i]);
+        for (int i = 0; i < RPT; ++i) {
+            S[i] = fmaf(s_k[d0 + i], v, s_w[d0 + i] * S[i]);
+            if (i % 8 == 7) __builtin_amdgcn_sched_barrier(0);
+        }
+        if (j + 1 < run.n_rows) fetch(m + 1);
+        else if (col < D)  // the state leaves while the output is finished
+        {
+            asm volatile("" : "+v"(at0));  // (the addresses are made again: kept since the loads, they would take a register each)
+#pragma unroll
+            for (int i = 0; i < RPT; ++i, at0 += row4)
+                if (d0 + i < D) *(float *)((char *)state + at0) = S[i];
+        }
         if (threadIdx.x < CV) {  // whole waves
-            o = 0.0f;
+            o = bonus * v;
 #pragma unroll
             for (int i = 0; i < SL; ++i) o += s_o[i][c];
-            const float sum = lanes_sum(o * o);
-            if (lane == 0) s_ss[threadIdx.x >> 6] = sum;
+            o = col < D ? o : 0.0f;
+            if (gridDim.z > 1) {  // norm and gate need the other workgroups' columns too
+                if (col < D) a.o[(m * a.H + head) * a.D8 + col] = o;
+            } else {
+                const float sum = lanes_sum(o * o);
+                if (lane == 0) s_ss[threadIdx.x >> 6] = sum;
+            }
         }
         lds_barrier();
-        if (threadIdx.x < CV && c < D) {
+        if (gridDim.z > 1) continue;
+        if (threadIdx.x < CV && col < D) {
             float sum = s_ss[0];
 #pragma unroll
             for (int i = 1; i < CV / 64; ++i) sum += s_ss[i];
-            ((T *)a.out)[m * a.ld_out + head * a.D8 + c] = E::pack(o * (1.0f / sqrtf(sum / (float)D + a.eps)) * o_norm * s_g[c] * a.out_scale);
+            ((T *)a.out)[m * a.ld_out + head * a.D8 + col] = E::pack(o * (1.0f / sqrtf(sum / (float)D + a.eps)) * o_norm * s_g[c] * a.out_scale);
         }
         lds_barrier();  // the channel vectors are written again
     }
-    if (c < D)
-#pragma unroll
-        for (int i = 0; i < RPT; ++i)
-            if (d0 + i < D) state[(size_t)(d0 + i) * D + c] = S[i];
 }
 
 // ---------------------------------------------------------------- chunk form: the operands
@@ -253,10 +306,12 @@ int time_mix_chunks_go(const TimeMixArgs &a, int chunks, hipStream_t st) {
 
 template <class E>
 int time_mix_step_go(const TimeMixArgs &a, hipStream_t st) {
-    const dim3 grid((unsigned)a.n_runs, (unsigned)a.H);
+    const dim3 grid((unsigned)a.n_runs, (unsigned)a.H, a.D <= 128 ? 1 : 2);
+    const bool many = (long)a.n_runs * a.H > 256;
     if (a.D <= 64) hipLaunchKernelGGL((k_time_mix_step<E, 64, 512, 8>), grid, dim3(512), 0, st, a);
+    else if (a.D <= 128 && many) hipLaunchKernelGGL((k_time_mix_step<E, 128, 512, 32>), grid, dim3(512), 0, st, a);
     else if (a.D <= 128) hipLaunchKernelGGL((k_time_mix_step<E, 128, 1024, 16>), grid, dim3(1024), 0, st, a);
-    else hipLaunchKernelGGL((k_time_mix_step<E, 256, 1024, 64>), grid, dim3(1024), 0, st, a);
+    else hipLaunchKernelGGL((k_time_mix_step<E, 128, 1024, 32>), grid, dim3(1024), 0, st, a);
     PIE_LAUNCH_CHECK();
     return PIE_OK;
 }
@@ -273,10 +328,17 @@ int time_mix_check(const TimeMixArgs &a) {
 size_t time_mix_ws_floats(int chunks, int H, int D) { return scan_ws_floats(SCAN_LINEAR, chunks, H, D); }
 int time_mix_chunk_launches(int chunks, int H, int D) { return scan_launches(SCAN_LINEAR, chunks, H, D) + 1; }
 
-int time_mix_step_launch(int dtype, const TimeMixArgs &a, hipStream_t st) {
+static int time_mix_head_out(int dtype, const TimeMixArgs &a, int row0, int rows, hipStream_t st) {
+    const HeadOutArgs h = {a.o, nullptr, a.gate, nullptr, a.ld, a.H, a.D, a.D8, a.o_norm, a.eps, a.out, a.ld_out, false, true, a.out_scale};
+    return head_out_launch(dtype, h, row0, rows, st);
+}
+
+int time_mix_step_launch(int dtype, const TimeMixArgs &a, int row0, int rows, hipStream_t st) {
     if (a.n_runs <= 0) return PIE_OK;
     if (const int rc = time_mix_check(a)) return rc;
-    return dtype == PIE_F32 ? time_mix_step_go<ElemF32>(a, st) : time_mix_step_go<ElemBF16>(a, st);
+    PIE_REQUIRE(a.D <= 128 || a.o, PIE_E_ARG, "time mixing: wide heads need their output buffer");
+    if (const int rc = dtype == PIE_F32 ? time_mix_step_go<ElemF32>(a, st) : time_mix_step_go<ElemBF16>(a, st)) return rc;
+    return a.D > 128 ? time_mix_head_out(dtype, a, row0, rows, st) : PIE_OK;
 }
 
 int time_mix_chunks_launch(int dtype, const TimeMixArgs &a, int chunks, int row0, int rows, hipStream_t st) {
@@ -284,6 +346,5 @@ int time_mix_chunks_launch(int dtype, const TimeMixArgs &a, int chunks, int row0
     if (const int rc = time_mix_check(a)) return rc;
     PIE_REQUIRE(a.ws && a.o && chunks > 0 && a.n_runs <= 65535, PIE_E_ARG, "time mixing: the chunk form needs its workspace");
     if (const int rc = dtype == PIE_F32 ? time_mix_chunks_go<ElemF32>(a, chunks, st) : time_mix_chunks_go<ElemBF16>(a, chunks, st)) return rc;
-    const HeadOutArgs h = {a.o, nullptr, a.gate, nullptr, a.ld, a.H, a.D, a.D8, a.o_norm, a.eps, a.out, a.ld_out, false, true, a.out_scale};
-    return head_out_launch(dtype, h, row0, rows, st);
+    return time_mix_head_out(dtype, a, row0, rows, st);
 }

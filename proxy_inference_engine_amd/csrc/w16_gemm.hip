@@ -159,7 +159,8 @@ int w16l_gemm_launch(int dtype, const void *w16m, const void *x, int ldx, int M,
 #ifdef W16L_PROF
     a.prof = g_w16_prof;
 #endif
-    const dim3 grid((unsigned)(8 * ((a.tn + 7) / 8) * a.tm), (unsigned)plan.S);
+    a.narrow = a.tn < 8 && a.tm >= 8;
+    const dim3 grid((unsigned)(a.narrow ? 8 * ((a.tm + 7) / 8) * a.tn : 8 * ((a.tn + 7) / 8) * a.tm), (unsigned)plan.S);
 #define W16_GO(TT, MB_, SW_, SG_) hipLaunchKernelGGL((k_w16l_gemm<TT, MB_, SW_, SG_>), grid, dim3(256), 0, st, a)
 #define W16_SW(TT, MB_) \
     if (sg) W16_GO(TT, MB_, 2, true); \

@@ -75,6 +75,7 @@ struct W16Args {
     const int4 *tiles;  // [tm] {expert, row0, rows, 0}; rows = 0: nothing to do
     const int *list;
     size_t w_stride;    // bytes between the experts' matrices
+    bool narrow;    // fewer column tiles than XCDs: these take row tiles instead, each with all columns
     int bm, bc;     // the XCD-local traversal's block: bm row tiles x bc column tiles (bm * bc ~ the 32 workgroups an XCD runs at once)
 #ifdef W16L_PROF
     unsigned long long *prof;  // per workgroup {s_memtime, s_memrealtime} at entry and exit (tools/w16_bench prof)
@@ -87,6 +88,7 @@ struct W16Args {
 // one column tile, then of the column tile 8 further -- they stream the SAME weight tiles at the same time, so each XCD's L2 fetches a
 // weight tile once per pass (16-bit weights are 4x the int4 kernel's bytes: re-read per row tile they would be 3.7 GB of HBM traffic for
 // gate|up at 4096 rows); grid.y = K splits.
+// narrow (fewer than 8 column tiles, at least 8 row tiles): an XCD takes every eighth row tile with all column tiles.
 // GRP: many matrices of one shape, each with its own rows (a mixture's experts).  An XCD takes every eighth block of bm row tiles -- an
 // expert's tiles start at a block -- with all its column tiles, row tile fastest: a block's tiles stream the same weight tiles through one L2 at the same time.
 template <class T, int MB, int SW, int ACT, bool GRP = false>
@@ -115,6 +117,12 @@ __global__ void __launch_bounds__(256) k_w16l_gemm(const W16Args a) {
         m0 = __builtin_amdgcn_readfirstlane(tile.y), rows = __builtin_amdgcn_readfirstlane(tile.z);
         if (rows <= 0) return;
         weights += (size_t)__builtin_amdgcn_readfirstlane(tile.x) * a.w_stride;
+    } else if (a.narrow) {
+        const int mt = (sq / a.tn) * 8 + xcd;
+        ncol = sq % a.tn;
+        if (mt >= a.tm) return;
+        m0 = mt * MT;
+        rows = a.M - m0 < MT ? a.M - m0 : MT;
     } else {
         const int cl = (a.tn + 7) >> 3;                       // local columns (the grid holds tm * cl workgroups per XCD)
         const int cb = sq / (a.tm * a.bc), r1 = sq - cb * a.tm * a.bc;

@@ -29,7 +29,8 @@ int w16l_act_launch(const void *w16m, const void *x, int ldx, int M, int N, int 
     int mb = 8;  // the largest row tile that still gives the chip a round of workgroups
     while (mb > 2 && (M <= 16 * mb || a.tn * ((M + 32 * mb - 1) / (32 * mb)) < 200)) mb >>= 1;
     a.M = M, a.tm = (M + 32 * mb - 1) / (32 * mb), a.bm = a.bm < a.tm ? a.bm : a.tm, a.act_alpha = alpha, a.act_limit = beta;
-    const dim3 grid((unsigned)(8 * ((a.tn + 7) / 8) * a.tm));
+    a.narrow = a.tn < 8 && a.tm >= 8;
+    const dim3 grid((unsigned)(a.narrow ? 8 * ((a.tm + 7) / 8) * a.tn : 8 * ((a.tn + 7) / 8) * a.tm));
 #define ACT_GO(MB_) \
     if (act == MFMA_ACT_RELU2) hipLaunchKernelGGL((k_w16l_gemm<BF16, MB_, 2, MFMA_ACT_RELU2>), grid, dim3(256), 0, st, a); \
     else if (act == MFMA_ACT_GELU) hipLaunchKernelGGL((k_w16l_gemm<BF16, MB_, 2, MFMA_ACT_GELU>), grid, dim3(256), 0, st, a); \

@@ -426,6 +426,24 @@ def test_batches_of_decoded_tokens(batch, dtype):
         assert lu.err(got, np.stack([want[-k] for _, want in todo])) < TOL[dtype]
 
 
+@BOTH
+@pytest.mark.parametrize("size", [(128, 128), (96, 256), (40, 100)], ids=str)
+def test_many_states_at_once(size, dtype):
+    """More (sequence, head) pairs than compute units, decoded and in short portions: wide heads take other workgroup shapes then."""
+    D, V = size
+    cfg = lu.config([(lu.delta(8, 4, D, V, 4), None), (lu.parallel(lu.left(2, 1, 8), lu.right(8, D)), None)], width=64, vocab=60)
+    w = lu.weights(cfg, seed=20)
+    m, wn = build(cfg, w, dtype, pages=50, slots=42), lu.as_numpy(w)
+    todo = [lu.sequence(cfg, wn, 12 + i % 9, seed=i) for i in range(42)]
+    caches = [m.make_cache() for _ in todo]
+    m.step_portions([(t[:-6], c) for (t, _), c in zip(todo, caches)], [[]] * 42)
+    got = m.step_portions([(t[-6:-3], c) for (t, _), c in zip(todo, caches)], [[0, 1, 2]] * 42).cpu().numpy()
+    assert lu.err(got, np.concatenate([want[-6:-3] for _, want in todo])) < TOL[dtype]
+    for k in range(3, 0, -1):
+        got = m.step_batch(torch.tensor([t[-k] for t, _ in todo]), caches)[2].cpu().numpy()
+        assert lu.err(got, np.stack([want[-k] for _, want in todo])) < TOL[dtype], k
+
+
 def test_logits_do_not_depend_on_the_batch():
     """The same request alone and among 20 others: equal to rounding, far below what bf16 itself costs."""
     cfg = lu.CONFIGS["mixed"]
