@@ -591,8 +591,8 @@ enum { PIE_MIXER_LATENT = 1, PIE_MIXER_ATTENTION = 2, PIE_MIXER_DELTA = 3, PIE_M
 enum { PIE_FF_NONE = 0, PIE_FF_RELU2 = 1, PIE_FF_TABLE_MOE = 2, PIE_FF_ROUTED_MOE = 3, PIE_FF_XIELU = 4, PIE_FF_GEGLU = 5 };
 enum { PIE_ACT_SILU = 0, PIE_ACT_CLIPPED = 1 };
 
-/* Time mixing with a decaying matrix state per head (RWKV-6).  Every projection reads its own mix h + (h' - h) mu of the row h and its predecessor h' in the sequence (zeros in
- * front of the first; the predecessor is part of the state): mu fp32 [5 (r, k, v, gate, decay)][width rounded up to 64].  w_r, w_k, w_v, w_gate packed [heads * dim8, width], w_low packed
+/* Time mixing with a decaying matrix state per head (RWKV-6).  The operands of the five projections are x_t + (x_(t-1) - x_t) mu, with a mu for each (x_(-1) = 0; the last
+ * row is kept in the state): mu fp32 [5 (r, k, v, gate, decay)][width rounded up to 64].  w_r, w_k, w_v, w_gate packed [heads * dim8, width], w_low packed
  * [rank8, width]; decay = exp(-exp(w_decay tanh(w_low .) + decay_bias)), w_decay bf16 [heads * dim][rank8] row-major, decay_bias fp32 [heads * dim]; o = (S + diag(bonus) k v^T)^T r, then
  * S = diag(decay) S + k v^T; bonus fp32 [heads * dim]; every head over its root mean square (eps of the layer), times o_norm (fp32 [heads * dim]) and silu(gate), times out_scale. */
 typedef struct {
