@@ -116,6 +116,26 @@ def test_every_time_mixing_size_class(size, dtype):
 
 
 @BOTH
+def test_time_mixing_alone(dtype, monkeypatch):
+    """The stack's mixer without an attention beside it: a layer whose description has the one half only."""
+    from proxy_inference_engine_amd import _ffi
+    from proxy_inference_engine_amd.models.layer_stack import LayerStackModel, pack_linear, pad_head_columns
+    cfg = lu.config([(lu.parallel(lu.left(2, 1, 8), lu.right(3, 20)), lu.dense()), (lu.parallel(lu.left(2, 1, 8), lu.right(3, 20)), None)], width=76)
+    w = lu.weights(cfg, seed=8)
+    for i in range(2):
+        w[f"l{i}.mix.left.o"].zero_()
+    real = LayerStackModel.__init__
+    keep = ("post1", "post2", "eps", "norm_after", "residual_scale", "w_side_gate", "w_side_proj", "side_norm", "time_mix", "ff", "ff_size", "w_up", "up_bias", "w_down", "down_bias")
+
+    def half(self, args, dtype, width, vocab, scale, layers, *rest, **kw):
+        alone = [{k: v for k, v in lay.items() if k in keep} | {"mixer": _ffi.PIE_MIXER_TIME_MIX, "kv_from": -1, "w_o": pack_linear(pad_head_columns(w[f"l{i}.mix.right.o"].cuda(), 3, 20), dtype)}
+                 for i, lay in enumerate(layers)]
+        real(self, args, dtype, width, vocab, scale, alone, *rest, **kw)
+    monkeypatch.setattr(LayerStackModel, "__init__", half)
+    both_ways(cfg, w, dtype, 150, [3, 19, 36, 116, 132, 133, 134])
+
+
+@BOTH
 @pytest.mark.parametrize("n", [2, 3, 7, 8, 15, 16, 17, 31, 33, 63, 64, 65, 79])
 def test_recurrent_runs_of_every_length(n, dtype):
     """Runs that end inside, at and just behind a chunk, twice in a row; the row in front of a portion is the last one of the portion before."""
